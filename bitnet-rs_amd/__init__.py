@@ -90,6 +90,32 @@ def _optr(t):
     return None if t is None else _ptr(t)
 
 
+def _addr(t):
+    """Device address of a torch tensor for a struct field (None: null)."""
+    return None if t is None else (t if isinstance(t, int) else t.data_ptr())
+
+
+ACT_NONE, ACT_SILU, ACT_SIGMOID, ACT_RELU2 = 0, 1, 2, 3
+IN_PLAIN, IN_NORM, IN_RESIDUAL_NORM = 0, 1, 2
+LINEAR_BLOCK = 128
+
+
+class VectorInput(C.Structure):
+    _fields_ = [("x", _vp), ("kind", C.c_int32), ("eps", C.c_float), ("weight_offset", C.c_float), ("weight", _vp), ("y", _vp), ("post_weight", _vp),
+                ("scale", _vp), ("gate", _vp), ("x_out", _vp), ("n", C.c_int32), ("mean_n", C.c_int32)]
+
+
+class LatentRows(C.Structure):
+    _fields_ = [("z", _vp), ("ldz", _sz), ("q_rank", C.c_int32), ("kv_rank", C.c_int32), ("rot_dim", C.c_int32), ("q_weight", _vp), ("kv_weight", _vp),
+                ("eps", C.c_float), ("cq", _vp), ("ldcq", _sz), ("ccache", _vp), ("rcache", _vp), ("ldc", _sz), ("ldr", _sz), ("rope_cos", _vp),
+                ("rope_sin", _vp), ("pos", _vp)]
+
+
+class LatentAttention(C.Structure):
+    _fields_ = [("heads", _sz), ("dimp", _sz), ("qd", _sz), ("vdimp", _sz), ("kv_rank", _sz), ("rot_dim", _sz), ("scale", C.c_float), ("sink", _vp),
+                ("ccache", _vp), ("rcache", _vp), ("ldc", _sz), ("ldr", _sz), ("capacity", _sz), ("rope_cos", _vp), ("rope_sin", _vp)]
+
+
 class HipLib:
     """ctypes view of libbitnet_hip.so.  One method per exported symbol."""
 
@@ -527,6 +553,65 @@ class HipLib:
     def argmax_dev(self, v, n: int, scratch, n_wg: int, token, stream: int = 0) -> None:
         self._check(self.c.bitnet_hip_argmax_dev(_ptr(v), n, _ptr(scratch), n_wg, _ptr(token), _vp(stream)))
 
+    # -- bf16-weight operators and sequence mixers (include/bitnet_hip.h section 5) -----------------------------
+    def embed_bf16_dev(self, table, ld: int, tokens, out, n: int, width: int, vocab: int, offset=None, stream: int = 0) -> None:
+        self._call("embed_bf16_dev", _ptr(table), _sz(ld), _ptr(tokens), _optr(offset), _sz(n), _sz(width), _sz(vocab), _ptr(out), _vp(stream))
+
+    def residual_norm_rows_dev(self, x, m: int, width: int, eps: float, weight_offset: float, y=None, ldy: int = 0, post_weight=None, scale=None,
+                               next_weight=None, h=None, ldh: int = 0, h_f32: bool = True, stream: int = 0) -> None:
+        self._call("residual_norm_rows_dev", _ptr(x), _optr(y), _sz(ldy), _optr(post_weight), _optr(scale), _optr(next_weight), C.c_float(weight_offset),
+                   C.c_float(eps), _sz(m), _sz(width), _optr(h), _sz(ldh), C.c_int(h_f32), _vp(stream))
+
+    def gated_norm_rows_dev(self, o, ldo: int, weight, gate, ldg: int, eps: float, gate_f32: bool, m: int, n: int, mean_n: int, h, ldh: int, h_f32: bool,
+                            stream: int = 0) -> None:
+        self._call("gated_norm_rows_dev", _ptr(o), _sz(ldo), _ptr(weight), _ptr(gate), _sz(ldg), C.c_float(eps), C.c_int(gate_f32), _sz(m), _sz(n),
+                   _sz(mean_n), _ptr(h), _sz(ldh), C.c_int(h_f32), _vp(stream))
+
+    def dense_matmul_dev(self, a, lda: int, a_f32: bool, w, ldw: int, m: int, n: int, k: int, c, ldc: int, c_f32: bool, bias=None, act0: int = 0,
+                         act1: int = 0, act_split: int = 0, batch: int = 1, a_batch: int = 0, w_batch: int = 0, c_batch: int = 0, stream: int = 0) -> None:
+        self._call("dense_matmul_dev", _ptr(a), _sz(lda), C.c_int(a_f32), _ptr(w), _sz(ldw), _optr(bias), _sz(m), _sz(n), _sz(k), C.c_int(act0),
+                   C.c_int(act1), _sz(act_split), _ptr(c), _sz(ldc), C.c_int(c_f32), _sz(batch), _sz(a_batch), _sz(w_batch), _sz(c_batch), _vp(stream))
+
+    def dense_gemv_dev(self, x, w, rows: int, cols: int, ld: int, y, kind: int = 0, eps: float = 0.0, weight_offset: float = 0.0, weight=None, res=None,
+                       post_weight=None, scale=None, gate=None, x_out=None, n: int = 0, mean_n: int = 0, bias=None, act0: int = 0, act1: int = 0,
+                       act_split: int = 0, batch: int = 1, w_batch: int = 0, x_batch: int = 0, y_batch: int = 0, latent=None, latent_f32: bool = False,
+                       stream: int = 0) -> None:
+        vi = VectorInput(_addr(x), kind, eps, weight_offset, _addr(weight), _addr(res), _addr(post_weight), _addr(scale), _addr(gate), _addr(x_out), n, mean_n)
+        self._call("dense_gemv_dev", C.byref(vi), _ptr(w), _sz(rows), _sz(cols), _sz(ld), _optr(bias), C.c_int(act0), C.c_int(act1), _sz(act_split), _ptr(y),
+                   _sz(batch), _sz(w_batch), _sz(x_batch), _sz(y_batch), C.byref(latent) if latent is not None else None, C.c_int(latent_f32), _vp(stream))
+
+    def latent_rows_dev(self, rows, m: int, f32: bool, stream: int = 0) -> None:
+        self._call("latent_rows_dev", C.byref(rows), _sz(m), C.c_int(f32), _vp(stream))
+
+    def latent_scratch_bytes(self, heads: int, ldc: int, nq: int) -> int:
+        self.c.bitnet_hip_latent_scratch_bytes.restype = _sz
+        return int(self.c.bitnet_hip_latent_scratch_bytes(_sz(heads), _sz(ldc), _sz(nq)))
+
+    def latent_decode_dev(self, attn, q, qabs, pos, q0: int, nq: int, f32: bool, scratch, stream: int = 0) -> None:
+        self._call("latent_decode_dev", C.byref(attn), _ptr(q), _ptr(qabs), _ptr(pos), _sz(q0), _sz(nq), C.c_int(f32), _ptr(scratch), _vp(stream))
+
+    def latent_merge_dev(self, attn, uv, pos, q0: int, nq: int, scratch, out, ldo: int, out_bf16: bool, stream: int = 0) -> None:
+        self._call("latent_merge_dev", C.byref(attn), _ptr(uv), _ptr(pos), _sz(q0), _sz(nq), _ptr(scratch), _ptr(out), _sz(ldo), C.c_int(out_bf16), _vp(stream))
+
+    def latent_prefill_dev(self, attn, q, k, vt, ldvt: int, n_ctx: int, nq: int, out, ldo: int, stream: int = 0) -> None:
+        self._call("latent_prefill_dev", C.byref(attn), _ptr(q), _ptr(k), _ptr(vt), _sz(ldvt), _sz(n_ctx), _sz(nq), _ptr(out), _sz(ldo), _vp(stream))
+
+    def linear_recurrent_dev(self, qkv, ld: int, n: int, heads: int, dimp: int, vdimp: int, decay_pow, state, out, ldo: int, stream: int = 0) -> None:
+        self._call("linear_recurrent_dev", _ptr(qkv), _sz(ld), _sz(n), _sz(heads), _sz(dimp), _sz(vdimp), _ptr(decay_pow), _ptr(state), _ptr(out), _sz(ldo),
+                   _vp(stream))
+
+    def linear_workspace_bytes(self, n: int, heads: int, dimp: int, vdimp: int) -> int:
+        self.c.bitnet_hip_linear_workspace_bytes.restype = _sz
+        return int(self.c.bitnet_hip_linear_workspace_bytes(_sz(n), _sz(heads), _sz(dimp), _sz(vdimp)))
+
+    def linear_chunked_dev(self, qkv, ld: int, n: int, heads: int, dimp: int, vdimp: int, decay_pow, state, out, ldo: int, workspace, workspace_bytes: int,
+                           stream: int = 0) -> None:
+        self._call("linear_chunked_dev", _ptr(qkv), _sz(ld), _sz(n), _sz(heads), _sz(dimp), _sz(vdimp), _ptr(decay_pow), _ptr(state), _ptr(out), _sz(ldo),
+                   _ptr(workspace), _sz(workspace_bytes), _vp(stream))
+
+    def _call(self, name: str, *args) -> None:
+        self._check(getattr(self.c, "bitnet_hip_" + name)(*args))
+
     def hbm_read_ceiling(self, nbytes: int = 2 << 30, iters: int = 10, stream: int = 0):
         """Measured read-only stream ceiling of the device: (best, mean) GB/s."""
         best, mean = C.c_double(0.0), C.c_double(0.0)
@@ -678,50 +763,50 @@ class GgufFile:
         return bool(self.c.bitnet_host_gguf_loader_is_qk256(sh, len(shape), available))
 
 
-class HostDecoder:
-    """ctypes view of the C++ Decoder (mirror of the reference's Rust-side
-    TransformerModel / KVCache / greedy loop).  No arithmetic here."""
+def _host_lib(path: str = HOST_LIB_PATH):
+    if not os.path.exists(path):
+        raise FileNotFoundError(f"{path} not found: build it with __graft_entry__.build() -- there is no fallback path")
+    load()  # the kernel library must be loadable first
+    L = C.CDLL(path)
+    i32p, fp = C.POINTER(C.c_int32), C.POINTER(C.c_float)
+    L.bitnet_host_open_model.restype = C.c_void_p
+    L.bitnet_host_open_model.argtypes = [C.c_char_p, C.c_int, C.c_int]
+    L.bitnet_host_open_error.restype = C.c_char_p
+    L.bitnet_host_registered.restype = C.c_char_p
+    L.bitnet_host_destroy.argtypes = [C.c_void_p]
+    L.bitnet_host_error.restype = C.c_char_p
+    L.bitnet_host_error.argtypes = [C.c_void_p]
+    L.bitnet_host_vocab.argtypes = [C.c_void_p]
+    L.bitnet_host_width.argtypes = [C.c_void_p]
+    L.bitnet_host_reset.argtypes = [C.c_void_p]
+    L.bitnet_host_feed.argtypes = [C.c_void_p, i32p, C.c_int]
+    L.bitnet_host_run.argtypes = [C.c_void_p, C.c_int, C.c_int, C.c_int, fp]
+    L.bitnet_host_prefill.argtypes = [C.c_void_p, C.c_int, C.c_int, C.c_int, fp]
+    L.bitnet_host_forward.argtypes = [C.c_void_p, i32p, C.c_int, i32p, C.c_int, fp]
+    L.bitnet_host_prepare_graphs.argtypes = [C.c_void_p, C.c_int]
+    L.bitnet_host_position.argtypes = [C.c_void_p]
+    L.bitnet_host_history.argtypes = [C.c_void_p, i32p, C.c_int]
+    L.bitnet_host_last_logits.argtypes = [C.c_void_p, _f32p]
+    L.bitnet_host_last_hidden.argtypes = [C.c_void_p, _f32p]
+    L.bitnet_host_weight_bytes.argtypes = [C.c_void_p]
+    L.bitnet_host_weight_bytes.restype = C.c_uint64
+    return L
 
-    def __init__(self, cfg, path: str = HOST_LIB_PATH):
-        if not os.path.exists(path):
-            raise FileNotFoundError(f"{path} not found: build it with __graft_entry__.build() -- there is no fallback path")
-        load()  # the kernel library must be loadable first
-        self.c = C.CDLL(path)
-        L = self.c
-        L.bitnet_host_create.restype = C.c_void_p
-        L.bitnet_host_create.argtypes = [C.POINTER(HostConfig)]
-        L.bitnet_host_destroy.argtypes = [C.c_void_p]
-        L.bitnet_host_error.restype = C.c_char_p
-        L.bitnet_host_error.argtypes = [C.c_void_p]
-        L.bitnet_host_set_layer_qk256.argtypes = [C.c_void_p, C.c_int, _f32p, _f32p] + [_u8p] * 7
-        L.bitnet_host_set_layer_i2s.argtypes = [C.c_void_p, C.c_int, _f32p, _f32p, C.POINTER(_u8p), C.POINTER(_f32p), _sz]
-        L.bitnet_host_set_globals.argtypes = [C.c_void_p, C.POINTER(C.c_uint16), _f32p]
-        L.bitnet_host_reset.argtypes = [C.c_void_p]
-        L.bitnet_host_feed.argtypes = [C.c_void_p, C.POINTER(C.c_int32), C.c_int]
-        L.bitnet_host_run.argtypes = [C.c_void_p, C.c_int, C.c_int, C.c_int, C.POINTER(C.c_float)]
-        L.bitnet_host_run_reference.argtypes = [C.c_void_p, C.c_int, C.c_int]
-        L.bitnet_host_prepare_graphs.argtypes = [C.c_void_p, C.c_int]
-        L.bitnet_host_set_act_mode.argtypes = [C.c_void_p, C.c_int]
-        L.bitnet_host_act_mode.argtypes = [C.c_void_p]
-        L.bitnet_host_position.argtypes = [C.c_void_p]
-        L.bitnet_host_last_prefill_path.argtypes = [C.c_void_p]
-        L.bitnet_host_saturation_fallbacks.argtypes = [C.c_void_p]
-        L.bitnet_host_history.argtypes = [C.c_void_p, C.POINTER(C.c_int32), C.c_int]
-        L.bitnet_host_last_logits.argtypes = [C.c_void_p, _f32p]
-        L.bitnet_host_last_hidden.argtypes = [C.c_void_p, _f32p]
-        L.bitnet_host_probe_gateup.argtypes = [C.c_void_p, C.c_int, C.POINTER(C.c_float), C.POINTER(C.c_double)]
-        L.bitnet_host_probe_kernel.argtypes = [C.c_void_p, C.c_int, C.c_int, C.POINTER(C.c_float), C.POINTER(C.c_double)]
-        L.bitnet_host_weight_bytes.argtypes = [C.c_void_p]
-        L.bitnet_host_weight_bytes.restype = C.c_uint64
-        self.cfg = cfg
-        hc = HostConfig(**{k: (float(v) if k in ("eps", "rope_theta") else int(v)) for k, v in cfg.asdict().items()})
-        self.h = L.bitnet_host_create(C.byref(hc))
-        if not self.h:
-            raise BitNetHipError(ERR_GPU, "bitnet_host_create failed (allocation)")
-        err = self.error()
-        if err:
-            self.close()  # a dead decoder (rejected configuration, failed allocation) is destroyed before the error is raised
-            raise BitNetHipError(ERR_GPU, err)
+
+def registered_models() -> list[str]:
+    """Architecture names (config.json) and file suffixes the host library serves."""
+    load()
+    L = C.CDLL(HOST_LIB_PATH)
+    L.bitnet_host_registered.restype = C.c_char_p
+    return L.bitnet_host_registered().decode().split(",")
+
+
+class HostSequence:
+    """One model with its live sequence: what every design shares (host/sequence.hpp).  No arithmetic here."""
+
+    c = None
+    h = None
+    vocab = width = 0
 
     def error(self) -> str:
         e = self.c.bitnet_host_error(self.h)
@@ -735,6 +820,120 @@ class HostDecoder:
         if self.h:
             self.c.bitnet_host_destroy(self.h)
             self.h = None
+
+    def reset(self) -> None:
+        self._check(self.c.bitnet_host_reset(self.h))
+
+    def feed(self, tokens) -> None:
+        t = _np(tokens, np.int32)
+        self._check(self.c.bitnet_host_feed(self.h, t.ctypes.data_as(C.POINTER(C.c_int32)), t.size))
+
+    def run(self, n: int, with_logits: bool = True, use_graph: bool = True) -> float:
+        ms = C.c_float(0)
+        self._check(self.c.bitnet_host_run(self.h, n, int(with_logits), int(use_graph), C.byref(ms)))
+        return ms.value
+
+    def prefill(self, n: int, with_logits: bool = True, digits: int = 4) -> float:
+        ms = C.c_float(0)
+        self._check(self.c.bitnet_host_prefill(self.h, n, int(with_logits), digits, C.byref(ms)))
+        return ms.value
+
+    def forward(self, tokens, want=()) -> np.ndarray:
+        """The next tokens of the sequence, forced; logits [len(want), vocab] of the places `want` among them."""
+        t, w = _np(tokens, np.int32), _np(list(want), np.int32)
+        out = np.zeros((w.size, self.vocab), np.float32)
+        self._check(self.c.bitnet_host_forward(self.h, t.ctypes.data_as(C.POINTER(C.c_int32)), t.size, w.ctypes.data_as(C.POINTER(C.c_int32)), w.size,
+                                               out.ctypes.data_as(_f32p)))
+        return out
+
+    def generate(self, prompt, n: int, use_graph: bool = True) -> np.ndarray:
+        """Greedy continuation of `prompt` on a fresh sequence: the prompt in one portion, then n - 1 steps."""
+        self.reset()
+        p = _np(prompt, np.int32)
+        self.feed(p)
+        self.prefill(p.size, with_logits=True, digits=2)
+        if n > 1:
+            self.run(n - 1, with_logits=True, use_graph=use_graph)
+        return self.history(p.size + n)[p.size:]
+
+    def prepare_graphs(self, with_logits: bool = True) -> None:
+        """capture + instantiate the step graph of every form a sequence can reach, ahead of time (nothing executes)"""
+        self._check(self.c.bitnet_host_prepare_graphs(self.h, int(with_logits)))
+
+    def position(self) -> int:
+        return int(self.c.bitnet_host_position(self.h))
+
+    def history(self, n: int) -> np.ndarray:
+        out = np.zeros(n, np.int32)
+        self._check(self.c.bitnet_host_history(self.h, out.ctypes.data_as(C.POINTER(C.c_int32)), n))
+        return out
+
+    def last_logits(self) -> np.ndarray:
+        out = np.zeros(self.vocab, np.float32)
+        self._check(self.c.bitnet_host_last_logits(self.h, out.ctypes.data_as(_f32p)))
+        return out
+
+    def last_hidden(self) -> np.ndarray:
+        out = np.zeros(self.width, np.float32)
+        self._check(self.c.bitnet_host_last_hidden(self.h, out.ctypes.data_as(_f32p)))
+        return out
+
+    def weight_bytes(self) -> int:
+        return int(self.c.bitnet_host_weight_bytes(self.h))
+
+
+class HostModel(HostSequence):
+    """A model opened by path: the class config.json (or the file's suffix) names."""
+
+    def __init__(self, path: str, dtype: str = "bfloat16", max_pos: int = 4096, lib_path: str = HOST_LIB_PATH):
+        if dtype not in ("bfloat16", "float32"):
+            raise ValueError(f"dtype {dtype}")
+        self.c = _host_lib(lib_path)
+        self.h = self.c.bitnet_host_open_model(path.encode(), int(dtype == "float32"), max_pos)
+        if not self.h:
+            raise BitNetHipError(ERR_INVALID_ARGUMENT, self.c.bitnet_host_open_error().decode(errors="replace"))
+        self.vocab, self.width = int(self.c.bitnet_host_vocab(self.h)), int(self.c.bitnet_host_width(self.h))
+
+    def stack_probe(self, kind: int, n: int, reps: int):
+        """(microseconds, bytes, flops) of one launch of a kernel group of the stack (bench.py)."""
+        us, b, f = C.c_float(0), C.c_double(0), C.c_double(0)
+        self.c.bitnet_host_stack_probe.argtypes = [C.c_void_p, C.c_int, C.c_int, C.c_int, C.POINTER(C.c_float), C.POINTER(C.c_double), C.POINTER(C.c_double)]
+        self._check(self.c.bitnet_host_stack_probe(self.h, kind, n, reps, C.byref(us), C.byref(b), C.byref(f)))
+        return us.value, b.value, f.value
+
+
+def open_model(path: str, dtype: str = "bfloat16", max_pos: int = 4096) -> HostModel:
+    return HostModel(path, dtype, max_pos)
+
+
+class HostDecoder(HostSequence):
+    """ctypes view of the C++ Decoder (mirror of the reference's Rust-side
+    TransformerModel / KVCache / greedy loop).  No arithmetic here."""
+
+    def __init__(self, cfg, path: str = HOST_LIB_PATH):
+        L = self.c = _host_lib(path)
+        L.bitnet_host_create.restype = C.c_void_p
+        L.bitnet_host_create.argtypes = [C.POINTER(HostConfig)]
+        L.bitnet_host_set_layer_qk256.argtypes = [C.c_void_p, C.c_int, _f32p, _f32p] + [_u8p] * 7
+        L.bitnet_host_set_layer_i2s.argtypes = [C.c_void_p, C.c_int, _f32p, _f32p, C.POINTER(_u8p), C.POINTER(_f32p), _sz]
+        L.bitnet_host_set_globals.argtypes = [C.c_void_p, C.POINTER(C.c_uint16), _f32p]
+        L.bitnet_host_run_reference.argtypes = [C.c_void_p, C.c_int, C.c_int]
+        L.bitnet_host_set_act_mode.argtypes = [C.c_void_p, C.c_int]
+        L.bitnet_host_act_mode.argtypes = [C.c_void_p]
+        L.bitnet_host_last_prefill_path.argtypes = [C.c_void_p]
+        L.bitnet_host_saturation_fallbacks.argtypes = [C.c_void_p]
+        L.bitnet_host_probe_gateup.argtypes = [C.c_void_p, C.c_int, C.POINTER(C.c_float), C.POINTER(C.c_double)]
+        L.bitnet_host_probe_kernel.argtypes = [C.c_void_p, C.c_int, C.c_int, C.POINTER(C.c_float), C.POINTER(C.c_double)]
+        self.cfg = cfg
+        self.vocab, self.width = int(cfg.vocab), int(cfg.hidden)
+        hc = HostConfig(**{k: (float(v) if k in ("eps", "rope_theta") else int(v)) for k, v in cfg.asdict().items()})
+        self.h = L.bitnet_host_create(C.byref(hc))
+        if not self.h:
+            raise BitNetHipError(ERR_GPU, "bitnet_host_create failed (allocation)")
+        err = self.error()
+        if err:
+            self.close()  # a dead decoder (rejected configuration, failed allocation) is destroyed before the error is raised
+            raise BitNetHipError(ERR_GPU, err)
 
     def load_gguf(self, gguf: "GgufFile") -> None:
         self.c.bitnet_host_load_gguf.argtypes = [C.c_void_p, C.c_void_p]
@@ -757,18 +956,6 @@ class HostDecoder:
         e, f = _np(g["embed_f16"], np.uint16), _np(g["final_norm"], np.float32)
         self._check(self.c.bitnet_host_set_globals(self.h, e.ctypes.data_as(C.POINTER(C.c_uint16)), f.ctypes.data_as(_f32p)))
 
-    def reset(self) -> None:
-        self._check(self.c.bitnet_host_reset(self.h))
-
-    def feed(self, tokens) -> None:
-        t = _np(tokens, np.int32)
-        self._check(self.c.bitnet_host_feed(self.h, t.ctypes.data_as(C.POINTER(C.c_int32)), t.size))
-
-    def run(self, n: int, with_logits: bool = True, use_graph: bool = True) -> float:
-        ms = C.c_float(0)
-        self._check(self.c.bitnet_host_run(self.h, n, int(with_logits), int(use_graph), C.byref(ms)))
-        return ms.value
-
     def set_kv_f16(self, on: bool) -> None:
         """Opt-in f16 KV cache (fresh sequence only)."""
         self.c.bitnet_host_set_kv_f16.argtypes = [C.c_void_p, C.c_int]
@@ -786,10 +973,6 @@ class HostDecoder:
         self.c.bitnet_host_trace_step.argtypes = [C.c_void_p, C.c_char_p, C.c_int]
         os.makedirs(directory, exist_ok=True)
         self._check(self.c.bitnet_host_trace_step(self.h, directory.encode(), int(with_logits)))
-
-    def prepare_graphs(self, with_logits: bool = True) -> None:
-        """capture + instantiate the step graph of every attention form a sequence can reach, ahead of time (nothing executes)"""
-        self._check(self.c.bitnet_host_prepare_graphs(self.h, int(with_logits)))
 
     def run_reference(self, n: int, with_logits: bool = True) -> None:
         """n UNFUSED steps on the bit-exact reference-order kernels (the checker of the fast step; slow)."""
@@ -835,12 +1018,6 @@ class HostDecoder:
         self._check(self.c.bitnet_host_phase_times(self.h, out))
         return {"matmul_us": round(out[0], 1), "attention_us": round(out[1], 1), "gather_wait_us": round(out[2], 1), "gather_us": round(out[3], 1)}
 
-    def prefill(self, n: int, with_logits: bool = True, digits: int = 4) -> float:
-        self.c.bitnet_host_prefill.argtypes = [C.c_void_p, C.c_int, C.c_int, C.c_int, C.POINTER(C.c_float)]
-        ms = C.c_float(0)
-        self._check(self.c.bitnet_host_prefill(self.h, n, int(with_logits), digits, C.byref(ms)))
-        return ms.value
-
     def last_prefill_path(self) -> int:
         """What the last prefill() ran: 0 digit planes (+ f16 hand-over / hybrid o / down), 1 the f16 chain, 2 the QB32 chain."""
         return int(self.c.bitnet_host_last_prefill_path(self.h))
@@ -848,24 +1025,6 @@ class HostDecoder:
     def saturation_fallbacks(self) -> int:
         """Prompts this decoder repeated on the row-scaled forms because an f16 hand-over value was clamped (bitnet_hip_f16_saturations)."""
         return int(self.c.bitnet_host_saturation_fallbacks(self.h))
-
-    def position(self) -> int:
-        return int(self.c.bitnet_host_position(self.h))
-
-    def history(self, n: int) -> np.ndarray:
-        out = np.zeros(n, np.int32)
-        self._check(self.c.bitnet_host_history(self.h, out.ctypes.data_as(C.POINTER(C.c_int32)), n))
-        return out
-
-    def last_logits(self) -> np.ndarray:
-        out = np.zeros(self.cfg.vocab, np.float32)
-        self._check(self.c.bitnet_host_last_logits(self.h, out.ctypes.data_as(_f32p)))
-        return out
-
-    def last_hidden(self) -> np.ndarray:
-        out = np.zeros(self.cfg.hidden, np.float32)
-        self._check(self.c.bitnet_host_last_hidden(self.h, out.ctypes.data_as(_f32p)))
-        return out
 
     def probe_gateup(self, reps: int):
         us, b = C.c_float(0), C.c_double(0)
@@ -876,6 +1035,3 @@ class HostDecoder:
         us, b = C.c_float(0), C.c_double(0)
         self._check(self.c.bitnet_host_probe_kernel(self.h, kind, reps, C.byref(us), C.byref(b)))
         return us.value, b.value
-
-    def weight_bytes(self) -> int:
-        return int(self.c.bitnet_host_weight_bytes(self.h))

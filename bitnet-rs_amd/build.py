@@ -1,6 +1,7 @@
 """Builds libbitnet_hip.so (gfx950 code objects only) in-tree with hipcc.
 
     python bitnet-rs_amd/build.py [--force]
+    python bitnet-rs_amd/build.py --program trace_run    (only what that program needs; prints its path)
 
 hipcc cross-compiles without a GPU.  The .so stays next to this file so it travels
 with the source snapshot to the GPU box (it is git-ignored, not gpurun-ignored).
@@ -28,6 +29,8 @@ COMMON_FLAGS = [
     "-fPIC",
     "-Wall",
     "-Wno-unused-result",
+    # packed-FP32 instructions are left out: some of their forms have given wrong results on this hardware
+    "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops",
     f"-I{INCLUDE}",
     f"-I{CSRC}",
 ]
@@ -125,7 +128,51 @@ def _build(force: bool, verbose: bool, OBJ_DIR: str, LIB_PATH: str, extra_all: l
         subprocess.check_call(cmd)
     if not extra_all:
         _build_host(force, verbose, LIB_PATH)
+        for name in PROGRAMS:
+            build_program(name)
     return LIB_PATH
+
+
+# Programs linked from the same objects as the libraries: the kernels and host files of the models they serve, and no others.
+STACK_CSRC = ["abi_core.hip", "abi_dense.hip", "kernels_decode.hip", "kernels_dense.hip", "kernels_latent.hip", "kernels_linear.hip"]
+STACK_HOST = ["sequence.cpp", "registry.cpp", "safetensors.cpp", "stack_model.cpp", "lasapel.cpp"]
+PROGRAMS = {"trace_run": (STACK_CSRC, STACK_HOST + ["trace_run.cpp"])}
+HOST_FLAGS = ["-O2", "-std=c++17", "-fPIC", "-Wall", "-Wno-unused-result", "-Wno-int-in-bool-context", "-D__HIP_PLATFORM_AMD__"]
+
+
+def build_program(name: str, force: bool = False) -> str:
+    import fcntl
+
+    csrc, host = PROGRAMS[name]
+    os.makedirs(OBJ_DIR, exist_ok=True)
+    target = os.path.join(OBJ_DIR, name)
+    with open(os.path.join(OBJ_DIR, ".lock"), "w") as lock:
+        fcntl.flock(lock, fcntl.LOCK_EX)
+        headers = [os.path.join(d, f) for d in (CSRC, INCLUDE, HOST_DIR) for f in os.listdir(d) if f.endswith((".hpp", ".h"))]
+        headers.append(os.path.abspath(__file__))
+        objs, procs = [], []
+        for src in csrc + host:
+            obj = os.path.join(OBJ_DIR, src.rsplit(".", 1)[0] + ".o")
+            objs.append(obj)
+            spath = os.path.join(CSRC if src in csrc else HOST_DIR, src)
+            if force or _stale(obj, [spath] + headers):
+                part = obj + ".part"
+                cmd = [HIPCC, *COMMON_FLAGS, *EXTRA.get(src, [])] if src in csrc else ["g++", *HOST_FLAGS, f"-I{INCLUDE}", f"-I{HOST_DIR}", "-I/opt/rocm/include"]
+                procs.append((src, obj, part, subprocess.Popen([*cmd, "-c", spath, "-o", part], stdout=subprocess.PIPE, stderr=subprocess.STDOUT, text=True)))
+        failed = False
+        for src, obj, part, p in procs:
+            out, _ = p.communicate()
+            if p.returncode != 0:
+                failed = True
+                sys.stderr.write(f"--- compiling {src} failed ---\n{out}\n")
+            else:
+                os.replace(part, obj)
+        if failed:
+            raise RuntimeError("compilation failed")
+        if force or procs or _stale(target, objs):
+            subprocess.check_call([HIPCC, f"--offload-arch={ARCH}", *objs, "-o", target + ".part", "-Wl,-rpath,/opt/rocm/lib"])
+            os.replace(target + ".part", target)
+    return target
 
 
 HOST_DIR = os.path.join(HERE, "host")
@@ -135,12 +182,13 @@ HOST_LIB_PATH = os.path.join(HERE, "libbitnet_host.so")
 def _build_host(force: bool, verbose: bool, kernel_lib: str) -> str:
     """The C++ host layer above the C ABI (decode loop, graph capture).  Plain host C++:
     it only includes include/bitnet_hip.h and the HIP runtime API."""
-    srcs = [os.path.join(HOST_DIR, f) for f in sorted(os.listdir(HOST_DIR)) if f.endswith(".cpp")]
+    mains = {f"{name}.cpp" for name in PROGRAMS}
+    srcs = [os.path.join(HOST_DIR, f) for f in sorted(os.listdir(HOST_DIR)) if f.endswith(".cpp") and f not in mains]
     deps = srcs + [os.path.join(HOST_DIR, f) for f in os.listdir(HOST_DIR) if f.endswith(".hpp")]
     deps += [os.path.join(INCLUDE, f) for f in os.listdir(INCLUDE)] + [kernel_lib]
     if force or _stale(HOST_LIB_PATH, deps):
         cmd = [
-            "g++", "-O2", "-std=c++17", "-fPIC", "-shared", "-Wall", "-Wno-unused-result", "-Wno-int-in-bool-context", "-D__HIP_PLATFORM_AMD__",
+            "g++", *HOST_FLAGS, "-shared",
             f"-I{INCLUDE}", f"-I{HOST_DIR}", "-I/opt/rocm/include", *srcs, "-o", HOST_LIB_PATH,
             f"-L{HERE}", "-lbitnet_hip", "-L/opt/rocm/lib", "-lamdhip64", "-Wl,-rpath,$ORIGIN", "-Wl,-rpath,/opt/rocm/lib",
         ]
@@ -151,4 +199,7 @@ def _build_host(force: bool, verbose: bool, kernel_lib: str) -> str:
 
 
 if __name__ == "__main__":
+    if "--program" in sys.argv:
+        print(build_program(sys.argv[sys.argv.index("--program") + 1], force="--force" in sys.argv))
+        sys.exit(0)
     print(build(force="--force" in sys.argv, verbose=True, diag="--diag" in sys.argv))

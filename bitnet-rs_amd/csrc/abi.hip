@@ -16,8 +16,6 @@
 
 namespace bitnet_hip {
 
-thread_local std::string g_last_error;
-
 namespace {
 
 // The provider trait is Send + Sync (K/lib.rs:39) and a KernelManager is shared through an Arc per layer
@@ -25,8 +23,6 @@ namespace {
 // other one, weights_free included.  Handles therefore map to REFERENCE-COUNTED matrices: a call holds its own
 // reference for its whole duration, weights_free only drops the table's, and the device memory goes with the last one.
 std::mutex g_mu;
-bool g_inited = false;
-int g_device = 0;
 std::atomic<int> g_kernel{BITNET_HIP_KERNEL_AUTO};  // default kernel of the calls that do not name one
 uint64_t g_next_handle = 1;
 using WeightsRef = std::shared_ptr<Weights>;
@@ -50,13 +46,12 @@ WeightsRef lookup(bitnet_hip_weights_t h) {
     return it == g_weights.end() ? WeightsRef() : it->second;
 }
 
-int ensure_init() {
-    {
-        std::lock_guard<std::mutex> lk(g_mu);
-        if (g_inited) return BITNET_HIP_OK;
-    }
-    return bitnet_hip_init(-1);
-}
+// bitnet_hip_cleanup drops the table; matrices still used by a running call go with that call's reference
+[[maybe_unused]] const bool g_cleanup_registered = (at_cleanup([] {
+                                                        std::lock_guard<std::mutex> lk(g_mu);
+                                                        g_weights.clear();
+                                                    }),
+                                                    true);
 
 int register_weights(Weights *w, bitnet_hip_weights_t *out) {
     WeightsRef ref(w, free_weights);
@@ -79,20 +74,6 @@ struct DevBuf {
         return static_cast<T *>(p);
     }
 };
-
-// Sizes are computed as products of caller-supplied dimensions: refuse anything whose products could
-// wrap size_t or exceed the kernels' 32-bit row/column indices before multiplying.
-bool dims_sane(size_t a, size_t b, size_t c = 1) {
-    const size_t lim = size_t(1) << 31;
-    if (a >= lim || b >= lim || c >= lim) return false;
-    unsigned long long ab = 0, abc = 0;
-    if (__builtin_mul_overflow((unsigned long long)a, (unsigned long long)b, &ab)) return false;
-    if (__builtin_mul_overflow(ab, (unsigned long long)c, &abc)) return false;
-    return abc < (1ull << 44);
-}
-#define BH_CHECK_DIMS(...)                                                                               \
-    if (!dims_sane(__VA_ARGS__))                                                                         \
-    return set_error(BITNET_HIP_ERR_INVALID_ARGUMENT, "dimensions too large for this library (%s)", #__VA_ARGS__)
 
 int run_gemv(Weights &w, const float *x_dev, float *y_dev, size_t m, const GemvFusion &fu, hipStream_t stream, int kernel = -1) {
     if (kernel < 0) kernel = g_kernel.load(std::memory_order_relaxed);
@@ -156,88 +137,7 @@ int run_gemv(Weights &w, const float *x_dev, float *y_dev, size_t m, const GemvF
 
 using namespace bitnet_hip;
 
-#define BH_GUARD_BEGIN try {
-#define BH_GUARD_END                                                                     \
-    }                                                                                    \
-    catch (const std::exception &e) {                                                    \
-        return set_error(BITNET_HIP_ERR_EXECUTION, "%s", e.what());                      \
-    }                                                                                    \
-    catch (...) {                                                                        \
-        return set_error(BITNET_HIP_ERR_EXECUTION, "unknown C++ exception");             \
-    }
-
 extern "C" {
-
-int bitnet_hip_init(int device) {
-    BH_GUARD_BEGIN
-    int count = 0;
-    hipError_t e = hipGetDeviceCount(&count);
-    if (e != hipSuccess || count <= 0)
-        return set_error(BITNET_HIP_ERR_GPU, "no HIP device available (hipGetDeviceCount: %s)",
-                         hipGetErrorString(e));
-    if (device < 0) {
-        if (hipGetDevice(&device) != hipSuccess) device = 0;
-    }
-    if (device >= count)
-        return set_error(BITNET_HIP_ERR_INVALID_ARGUMENT, "device %d out of range (%d visible)", device,
-                         count);
-    BH_HIP_TRY(hipSetDevice(device));
-    hipDeviceProp_t prop;
-    BH_HIP_TRY(hipGetDeviceProperties(&prop, device));
-    if (strncmp(prop.gcnArchName, "gfx950", 6) != 0)
-        return set_error(BITNET_HIP_ERR_UNSUPPORTED,
-                         "device %d is %s; this library carries gfx950 (MI355X) code objects only",
-                         device, prop.gcnArchName);
-    std::lock_guard<std::mutex> lk(g_mu);
-    g_device = device;
-    g_inited = true;
-    g_last_error.clear();
-    return BITNET_HIP_OK;
-    BH_GUARD_END
-}
-
-void bitnet_hip_cleanup(void) {
-    try {
-        std::lock_guard<std::mutex> lk(g_mu);
-        g_weights.clear();  // matrices still used by a running call go with that call's reference
-        g_inited = false;
-        g_last_error.clear();
-    } catch (...) {
-    }
-}
-
-int bitnet_hip_is_available(void) {
-    int count = 0;
-    return hipGetDeviceCount(&count) == hipSuccess && count > 0 ? 1 : 0;
-}
-
-int bitnet_hip_device_count(void) {
-    int count = 0;
-    return hipGetDeviceCount(&count) == hipSuccess ? count : 0;
-}
-
-const char *bitnet_hip_get_last_error(void) {
-    return g_last_error.empty() ? nullptr : g_last_error.c_str();
-}
-
-int bitnet_hip_get_device_info(int device, bitnet_hip_device_info *out) {
-    BH_GUARD_BEGIN
-    if (!out) return set_error(BITNET_HIP_ERR_INVALID_ARGUMENT, "Null pointer passed to get_device_info");
-    hipDeviceProp_t prop;
-    BH_HIP_TRY(hipGetDeviceProperties(&prop, device));
-    memset(out, 0, sizeof(*out));
-    out->device_id = device;
-    strncpy(out->name, prop.name, sizeof(out->name) - 1);
-    strncpy(out->gcn_arch, prop.gcnArchName, sizeof(out->gcn_arch) - 1);
-    out->total_memory = prop.totalGlobalMem;
-    out->compute_unit_count = prop.multiProcessorCount;
-    out->max_wavefront_size = prop.warpSize;
-    out->max_shared_memory_per_workgroup = prop.sharedMemPerBlock;
-    out->supports_fp16 = 1;
-    out->supports_bf16 = 1;
-    return BITNET_HIP_OK;
-    BH_GUARD_END
-}
 
 int bitnet_hip_set_kernel(int kernel) {
     if (kernel < BITNET_HIP_KERNEL_AUTO || kernel > BITNET_HIP_KERNEL_MFMA_TILED)
@@ -882,14 +782,6 @@ int bitnet_hip_rmsnorm(const float *input, size_t in_len, const float *gamma, si
     BH_GUARD_END
 }
 
-int bitnet_hip_advance_pos_dev(int32_t *pos_dev, void *stream) {
-    BH_GUARD_BEGIN
-    if (!pos_dev) return set_error(BITNET_HIP_ERR_INVALID_ARGUMENT, "Null pointer passed to advance_pos_dev");
-    BH_HIP_TRY(launch_advance_pos(pos_dev, (hipStream_t)stream));
-    return BITNET_HIP_OK;
-    BH_GUARD_END
-}
-
 int bitnet_hip_add_dev(const float *a_dev, const float *b_dev, float *out_dev, size_t n, void *stream) {
     BH_GUARD_BEGIN
     if (!a_dev || !b_dev || !out_dev) return set_error(BITNET_HIP_ERR_INVALID_ARGUMENT, "Null pointer passed to add_dev");
@@ -1309,17 +1201,6 @@ int bitnet_hip_logits_f16_dev(const void *table, const float *x, const float *ga
     BH_HIP_TRY(launch_logits_f16(table, x, gamma, eps, (int)hidden, (int)vocab, logits, bv, bi, (int)n_wg, (hipStream_t)stream));
     if (token_dev || pos_dev)
         BH_HIP_TRY(launch_argmax_final(bv, bi, (int)n_wg, token_dev, pos_dev, history_dev, n_forced_dev, (hipStream_t)stream));
-    return BITNET_HIP_OK;
-    BH_GUARD_END
-}
-
-int bitnet_hip_argmax_dev(const float *v, size_t n, void *scratch, size_t n_wg, int32_t *token_dev, void *stream) {
-    BH_GUARD_BEGIN
-    if (!v || !scratch || !token_dev) return set_error(BITNET_HIP_ERR_INVALID_ARGUMENT, "Null pointer passed to argmax_dev");
-    if (n == 0 || n_wg == 0) return set_error(BITNET_HIP_ERR_INVALID_ARGUMENT, "argmax: empty input");
-    float *bv = static_cast<float *>(scratch);
-    int *bi = reinterpret_cast<int *>(bv + n_wg);
-    BH_HIP_TRY(launch_argmax(v, (int)n, bv, bi, (int)n_wg, token_dev, (hipStream_t)stream));
     return BITNET_HIP_OK;
     BH_GUARD_END
 }

@@ -40,6 +40,35 @@ inline int set_error(int code, const char *fmt, ...) {
                                            #expr);                                             \
     } while (0)
 
+// abi_core.hip: initialises the library for the calling thread's device on first use; cleanup work of another file
+int ensure_init();
+extern int g_device;
+void at_cleanup(void (*fn)());
+
+// Sizes are computed as products of caller-supplied dimensions: refuse anything whose products could
+// wrap size_t or exceed the kernels' 32-bit row/column indices before multiplying.
+inline bool dims_sane(size_t a, size_t b, size_t c = 1) {
+    const size_t lim = size_t(1) << 31;
+    if (a >= lim || b >= lim || c >= lim) return false;
+    unsigned long long ab = 0, abc = 0;
+    if (__builtin_mul_overflow((unsigned long long)a, (unsigned long long)b, &ab)) return false;
+    if (__builtin_mul_overflow(ab, (unsigned long long)c, &abc)) return false;
+    return abc < (1ull << 44);
+}
+#define BH_CHECK_DIMS(...)                                                                               \
+    if (!dims_sane(__VA_ARGS__))                                                                         \
+    return set_error(BITNET_HIP_ERR_INVALID_ARGUMENT, "dimensions too large for this library (%s)", #__VA_ARGS__)
+
+#define BH_GUARD_BEGIN try {
+#define BH_GUARD_END                                                                     \
+    }                                                                                    \
+    catch (const std::exception &e) {                                                    \
+        return set_error(BITNET_HIP_ERR_EXECUTION, "%s", e.what());                      \
+    }                                                                                    \
+    catch (...) {                                                                        \
+        return set_error(BITNET_HIP_ERR_EXECUTION, "unknown C++ exception");             \
+    }
+
 inline size_t div_ceil(size_t a, size_t b) { return (a + b - 1) / b; }
 
 // Code -> value maps used by the reference (SURVEY.md 8a "code-map summary"),

@@ -210,7 +210,7 @@ __global__ __launch_bounds__(256 * NH) void k_attn_partial(const float *__restri
     __syncthreads();
     BH_ASTAMP(2);  // q, the new key / value are in LDS (the seven RoPE operands have arrived)
     // ---- scores: lane = position, wave = 32-dim slice; all 32 loads of a thread in flight ---
-    // Two partial sums per head (even / odd dims) so that each v_pk_fma_f32 takes an adjacent (q[d], q[d+1]) pair
+    // Two partial sums per head (even / odd dims) so that each fma takes an adjacent (q[d], q[d+1]) pair
     // from one LDS read and an adjacent (k[d], k[d+1]) register pair: no operand shuffling.
     if (KV16) {
         if (last) {  // the new token's key comes from LDS, rounded as the cache will hold it

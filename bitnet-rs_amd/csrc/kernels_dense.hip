@@ -1,0 +1,630 @@
+// kernels_dense.hip -- operators on bf16 weight matrices (gfx950): embedding rows, residual + norm rows, the many-row matmul
+// and the matrix-vector product of the decode step with its input transform folded in.
+//
+// Precision: residual stream, norms and accumulation are f32 everywhere.  The matmul multiplies bf16 activations on the matrix
+// cores, or -- a_f32 -- f32 activations with f32 multiply-adds; the matrix-vector product always multiplies f32 activations.
+#include <algorithm>
+
+#include "dense.hpp"
+
+namespace bitnet_hip {
+
+// ---- embedding rows ---------------------------------------------------------------------------------------------------
+__global__ void k_embed_bf16(const uint16_t *__restrict__ table, size_t ld, const int *__restrict__ tokens, const int *__restrict__ offset,
+                             int width, int vocab, float *__restrict__ out) {
+    int tok = tokens[(offset ? *offset : 0) + blockIdx.x];
+    tok = tok < 0 ? 0 : (tok >= vocab ? vocab - 1 : tok);
+    for (int i = threadIdx.x; i < width; i += blockDim.x) out[(size_t)blockIdx.x * width + i] = bf2f(table[(size_t)tok * ld + i]);
+}
+
+hipError_t launch_embed_bf16(const uint16_t *table, size_t ld, const int *tokens, const int *offset, int n, int width, int vocab, float *out,
+                             hipStream_t s) {
+    hipLaunchKernelGGL(k_embed_bf16, dim3(n), dim3(256), 0, s, table, ld, tokens, offset, width, vocab, out);
+    return hipGetLastError();
+}
+
+__global__ void k_gather_rows(const float *__restrict__ x, const int *__restrict__ rows, int width, float *__restrict__ out) {
+    const float *src = x + (size_t)rows[blockIdx.x] * width;
+    for (int i = threadIdx.x; i < width; i += blockDim.x) out[(size_t)blockIdx.x * width + i] = src[i];
+}
+
+hipError_t launch_gather_rows(const float *x, const int *rows, int n, int width, float *out, hipStream_t s) {
+    hipLaunchKernelGGL(k_gather_rows, dim3(n), dim3(256), 0, s, x, rows, width, out);
+    return hipGetLastError();
+}
+
+// ---- residual + norm rows ---------------------------------------------------------------------------------------------
+// x += scale * norm(y; post_w); h = norm(x; next_w).  One workgroup per row; rows of up to 4096 columns stay in registers.
+constexpr int kRowRegs = 16;
+
+template <class TH>
+__global__ __launch_bounds__(256) void k_residual_norm_rows(float *__restrict__ x, const float *__restrict__ y, size_t ldy, const float *__restrict__ post_w,
+                                                            const float *__restrict__ scale, const float *__restrict__ next_w, float offset, float eps,
+                                                            int width, TH *__restrict__ h, size_t ldh) {
+    __shared__ float slot[4];
+    const int tid = threadIdx.x;
+    float *xr = x + (size_t)blockIdx.x * width;
+    const float *yr = y ? y + (size_t)blockIdx.x * ldy : nullptr;
+    const bool regs = width <= 256 * kRowRegs;
+    float xv[kRowRegs];
+    if (yr) {
+        float ss = 0.f, yv[kRowRegs];
+        if (regs) {
+#pragma unroll
+            for (int j = 0; j < kRowRegs; ++j) {
+                const int i = tid + 256 * j;
+                yv[j] = i < width ? yr[i] : 0.f;
+                xv[j] = i < width ? xr[i] : 0.f;
+                ss += yv[j] * yv[j];
+            }
+        } else {
+            for (int i = tid; i < width; i += 256) ss += yr[i] * yr[i];
+        }
+        const float inv = 1.0f / sqrtf(group_sum<4>(ss, slot) / (float)width + eps);
+        if (regs) {
+#pragma unroll
+            for (int j = 0; j < kRowRegs; ++j) {
+                const int i = tid + 256 * j;
+                if (i < width) {
+                    xv[j] += (scale ? scale[i] : 1.0f) * (yv[j] * inv * (offset + post_w[i]));
+                    xr[i] = xv[j];
+                }
+            }
+        } else {
+            for (int i = tid; i < width; i += 256) xr[i] += (scale ? scale[i] : 1.0f) * (yr[i] * inv * (offset + post_w[i]));
+        }
+    } else if (regs) {
+#pragma unroll
+        for (int j = 0; j < kRowRegs; ++j) xv[j] = tid + 256 * j < width ? xr[tid + 256 * j] : 0.f;
+    }
+    if (!h) return;
+    float ss = 0.f;
+    if (regs) {
+#pragma unroll
+        for (int j = 0; j < kRowRegs; ++j) ss += xv[j] * xv[j];
+    } else {
+        for (int i = tid; i < width; i += 256) ss += xr[i] * xr[i];
+    }
+    const float inv = 1.0f / sqrtf(group_sum<4>(ss, slot) / (float)width + eps);
+    TH *hr = h + (size_t)blockIdx.x * ldh;
+    if (regs) {
+#pragma unroll
+        for (int j = 0; j < kRowRegs; ++j) {
+            const int i = tid + 256 * j;
+            if (i < width) st_act(hr, i, xv[j] * inv * (offset + next_w[i]));
+        }
+    } else {
+        for (int i = tid; i < width; i += 256) st_act(hr, i, xr[i] * inv * (offset + next_w[i]));
+    }
+    for (int i = width + tid; i < (int)ldh; i += 256) st_act(hr, i, 0.f);
+}
+
+hipError_t launch_residual_norm_rows(float *x, const float *y, size_t ldy, const float *post_w, const float *scale, const float *next_w,
+                                     float offset, float eps, int m, int width, void *h, size_t ldh, int h_f32, hipStream_t s) {
+    if (h_f32)
+        hipLaunchKernelGGL(k_residual_norm_rows<float>, dim3(m), dim3(256), 0, s, x, y, ldy, post_w, scale, next_w, offset, eps, width, (float *)h, ldh);
+    else
+        hipLaunchKernelGGL(k_residual_norm_rows<uint16_t>, dim3(m), dim3(256), 0, s, x, y, ldy, post_w, scale, next_w, offset, eps, width, (uint16_t *)h, ldh);
+    return hipGetLastError();
+}
+
+// h = norm(o; w) * gate (gate: already through its sigmoid); the mean runs over mean_n elements, padding columns of o are zero
+template <class TG, class TH>
+__global__ __launch_bounds__(256) void k_gated_norm_rows(const float *__restrict__ o, size_t ldo, const float *__restrict__ w, const TG *__restrict__ gate,
+                                                         size_t ldg, float eps, int n, int mean_n, TH *__restrict__ h, size_t ldh) {
+    __shared__ float slot[4];
+    const int tid = threadIdx.x;
+    const float *orow = o + (size_t)blockIdx.x * ldo;
+    const TG *grow = gate + (size_t)blockIdx.x * ldg;
+    TH *hr = h + (size_t)blockIdx.x * ldh;
+    float ss = 0.f;
+    for (int i = tid; i < n; i += 256) ss += orow[i] * orow[i];
+    const float inv = 1.0f / sqrtf(group_sum<4>(ss, slot) / (float)mean_n + eps);
+    for (int i = tid; i < n; i += 256) st_act(hr, i, orow[i] * inv * w[i] * ld_act(grow, i));
+    for (int i = n + tid; i < (int)ldh; i += 256) st_act(hr, i, 0.f);
+}
+
+hipError_t launch_gated_norm_rows(const float *o, size_t ldo, const float *w, const void *gate, size_t ldg, int gate_f32, float eps, int m, int n,
+                                  int mean_n, void *h, size_t ldh, int h_f32, hipStream_t s) {
+    auto go = [&](auto *fn, auto *g, auto *out) { hipLaunchKernelGGL(fn, dim3(m), dim3(256), 0, s, o, ldo, w, g, ldg, eps, n, mean_n, out, ldh); };
+    if (gate_f32 && h_f32)
+        go(k_gated_norm_rows<float, float>, (const float *)gate, (float *)h);
+    else if (gate_f32)
+        go(k_gated_norm_rows<float, uint16_t>, (const float *)gate, (uint16_t *)h);
+    else if (!h_f32)
+        go(k_gated_norm_rows<uint16_t, uint16_t>, (const uint16_t *)gate, (uint16_t *)h);
+    else
+        return hipErrorInvalidValue;
+    return hipGetLastError();
+}
+
+// ---- latent rows ------------------------------------------------------------------------------------------------------
+template <class T>
+__device__ void latent_row(const LatentRows &p, int row, float *slot) {
+    const int tid = threadIdx.x;
+    const float *z = p.z + (size_t)row * p.ldz;
+    if (p.cq) {
+        float ss = 0.f;
+        for (int i = tid; i < p.q_rank; i += 256) ss += z[i] * z[i];
+        const float inv = 1.0f / sqrtf(group_sum<4>(ss, slot) / (float)p.q_rank + p.eps);
+        T *o = (T *)p.cq + (size_t)row * p.ldcq;
+        for (int i = tid; i < p.ldcq; i += 256) st_act(o, i, i < p.q_rank ? z[i] * inv * p.q_weight[i] : 0.f);
+    }
+    if (p.kv_rank == 0) return;
+    const int pos = *p.pos + row;
+    const float *zc = z + p.q_rank, *zr = zc + p.kv_rank;
+    float ss = 0.f;
+    for (int i = tid; i < p.kv_rank; i += 256) ss += zc[i] * zc[i];
+    const float inv = 1.0f / sqrtf(group_sum<4>(ss, slot) / (float)p.kv_rank + p.eps);
+    T *c = (T *)p.ccache + (size_t)pos * p.ldc;
+    for (int i = tid; i < p.kv_rank; i += 256) st_act(c, i, zc[i] * inv * p.kv_weight[i]);
+    const int half = p.rot_dim / 2;
+    T *r = (T *)p.rcache + (size_t)pos * p.ldr;
+    for (int i = tid; i < half; i += 256) {
+        const float cs = p.rope_cos[(size_t)pos * half + i], sn = p.rope_sin[(size_t)pos * half + i];
+        const float u = zr[i], v = zr[i + half];
+        st_act(r, i, u * cs - v * sn);
+        st_act(r, i + half, v * cs + u * sn);
+    }
+}
+
+template <class T>
+__global__ __launch_bounds__(256) void k_latent_rows(LatentRows p) {
+    __shared__ float slot[4];
+    latent_row<T>(p, blockIdx.x, slot);
+}
+
+hipError_t launch_latent_rows(const LatentRows &a, hipStream_t s) {
+    if (a.f32)
+        hipLaunchKernelGGL(k_latent_rows<float>, dim3(a.m), dim3(256), 0, s, a);
+    else
+        hipLaunchKernelGGL(k_latent_rows<uint16_t>, dim3(a.m), dim3(256), 0, s, a);
+    return hipGetLastError();
+}
+
+// ---- matrix-vector product --------------------------------------------------------------------------------------------
+// One launch per product of the decode step.  Every workgroup forms the whole input vector (L2-resident, a few KiB) in LDS --
+// norm, residual + norm, or gated norm -- then its waves take rows: LPR lanes per row, 16 bytes of weights per lane and chunk,
+// R rows x U chunks in flight.  The first block of weights is requested ahead of the input transform.
+struct GemvK {
+    GemvArgs a;
+    LatentRows lat;
+    int kp;        // columns rounded up to whole LPR * 8 * U steps: length of the LDS vector
+    int groups;    // row groups (R * 64 / LPR rows each) of one batch member
+    int lat_wg;    // workgroup index that writes the latent row, or -1
+};
+
+__device__ void form_input(const VecIn &in, const float *x, int cols, int kp, float *xs, float *slot, bool writer) {
+    const int tid = threadIdx.x;
+    const int n = in.n;
+    if (in.kind == BITNET_HIP_IN_PLAIN) {
+        for (int i = tid; i < kp; i += 256) xs[i] = i < cols ? x[i] : 0.f;
+        __syncthreads();
+        return;
+    }
+    constexpr int NR = 4;  // float4 registers: vectors of up to 4096 elements
+    if ((n & 3) == 0 && n <= 1024 * NR) {
+        f32x4 xv[NR];
+        const int n4 = n >> 2;
+#pragma unroll
+        for (int j = 0; j < NR; ++j) {
+            const int i = tid + 256 * j;
+            xv[j] = i < n4 ? reinterpret_cast<const f32x4 *>(x)[i] : f32x4{0.f, 0.f, 0.f, 0.f};
+        }
+        if (in.kind == BITNET_HIP_IN_RESIDUAL_NORM && in.y) {
+            f32x4 yv[NR], pw[NR], sc[NR];
+            float ss = 0.f;
+#pragma unroll
+            for (int j = 0; j < NR; ++j) {
+                const int i = tid + 256 * j;
+                const bool ok = i < n4;
+                yv[j] = ok ? reinterpret_cast<const f32x4 *>(in.y)[i] : f32x4{0.f, 0.f, 0.f, 0.f};
+                pw[j] = ok ? reinterpret_cast<const f32x4 *>(in.post_weight)[i] : f32x4{0.f, 0.f, 0.f, 0.f};
+                sc[j] = ok && in.scale ? reinterpret_cast<const f32x4 *>(in.scale)[i] : f32x4{1.f, 1.f, 1.f, 1.f};
+            }
+#pragma unroll
+            for (int j = 0; j < NR; ++j) ss += yv[j].x * yv[j].x + yv[j].y * yv[j].y + yv[j].z * yv[j].z + yv[j].w * yv[j].w;
+            const float inv = 1.0f / sqrtf(group_sum<4>(ss, slot) / (float)in.mean_n + in.eps);
+#pragma unroll
+            for (int j = 0; j < NR; ++j) {
+                const int i = tid + 256 * j;
+                if (i >= n4) continue;
+                xv[j] += sc[j] * (yv[j] * inv * (in.offset + pw[j]));
+                if (writer) reinterpret_cast<f32x4 *>(in.x_out)[i] = xv[j];
+            }
+        }
+        f32x4 wv[NR], gv[NR];
+        float ss = 0.f;
+#pragma unroll
+        for (int j = 0; j < NR; ++j) {
+            const int i = tid + 256 * j;
+            wv[j] = i < n4 ? reinterpret_cast<const f32x4 *>(in.weight)[i] : f32x4{0.f, 0.f, 0.f, 0.f};
+            gv[j] = in.gate && i < n4 ? reinterpret_cast<const f32x4 *>(in.gate)[i] : f32x4{1.f, 1.f, 1.f, 1.f};
+            ss += xv[j].x * xv[j].x + xv[j].y * xv[j].y + xv[j].z * xv[j].z + xv[j].w * xv[j].w;
+        }
+        const float inv = 1.0f / sqrtf(group_sum<4>(ss, slot) / (float)in.mean_n + in.eps);
+#pragma unroll
+        for (int j = 0; j < NR; ++j) {
+            const int i = tid + 256 * j;
+            if (i < n4) reinterpret_cast<f32x4 *>(xs)[i] = xv[j] * inv * (in.offset + wv[j]) * gv[j];
+        }
+    } else {
+        float ss = 0.f;
+        if (in.kind == BITNET_HIP_IN_RESIDUAL_NORM && in.y) {
+            for (int i = tid; i < n; i += 256) ss += in.y[i] * in.y[i];
+            const float inv = 1.0f / sqrtf(group_sum<4>(ss, slot) / (float)in.mean_n + in.eps);
+            ss = 0.f;
+            for (int i = tid; i < n; i += 256) {
+                const float v = x[i] + (in.scale ? in.scale[i] : 1.0f) * (in.y[i] * inv * (in.offset + in.post_weight[i]));
+                xs[i] = v;
+                if (writer) in.x_out[i] = v;
+                ss += v * v;
+            }
+        } else {
+            for (int i = tid; i < n; i += 256) {
+                xs[i] = x[i];
+                ss += x[i] * x[i];
+            }
+        }
+        const float inv = 1.0f / sqrtf(group_sum<4>(ss, slot) / (float)in.mean_n + in.eps);
+        for (int i = tid; i < n; i += 256) xs[i] = xs[i] * inv * (in.offset + in.weight[i]) * (in.gate ? in.gate[i] : 1.0f);
+    }
+    for (int i = n + tid; i < kp; i += 256) xs[i] = 0.f;
+    __syncthreads();
+}
+
+template <int LPR, int R, int U>
+__global__ __launch_bounds__(256) void k_dense_gemv(GemvK p) {
+    extern __shared__ __attribute__((aligned(16))) float xs[];
+    __shared__ float slot[4];
+    __shared__ float wbv[4];
+    __shared__ int wbi[4];
+    const GemvArgs &a = p.a;
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    if ((int)blockIdx.x == p.lat_wg) {  // (the whole workgroup)
+        if (p.lat.f32)
+            latent_row<float>(p.lat, 0, slot);
+        else
+            latent_row<uint16_t>(p.lat, 0, slot);
+        return;
+    }
+    const int n_wg = p.lat_wg >= 0 ? p.lat_wg : (int)gridDim.x;
+    const int b = blockIdx.y;
+    const int sub = lane / LPR, l = lane % LPR;
+    constexpr int G = 64 / LPR;
+    const uint16_t *wb = a.w + (size_t)b * a.w_batch;
+    const int step = LPR * 8 * U;
+    const int last_col = a.cols - 8;
+    int g = blockIdx.x * 4 + wave;
+    u32x4 w[R][U];
+    auto fetch = [&](int grp, int k0) {
+        const int row0 = (grp * G + sub) * R;
+#pragma unroll
+        for (int r = 0; r < R; ++r) {
+            const int row = row0 + r < a.rows ? row0 + r : a.rows - 1;
+            const uint16_t *wr = wb + (size_t)row * a.ld;
+#pragma unroll
+            for (int u = 0; u < U; ++u) {
+                const int col = k0 + (u * LPR + l) * 8;
+                w[r][u] = __builtin_nontemporal_load(reinterpret_cast<const u32x4 *>(wr + (col < last_col ? col : last_col)));
+            }
+        }
+    };
+    if (g < p.groups) fetch(g, 0);
+    form_input(a.in, a.in.x + (size_t)b * a.x_batch, a.cols, p.kp, xs, slot, blockIdx.x == 0 && b == 0 && a.in.x_out);
+    float bv = -INFINITY;
+    int bi = 0x7fffffff;
+    for (; g < p.groups; g += n_wg * 4) {
+        float acc[R];
+#pragma unroll
+        for (int r = 0; r < R; ++r) acc[r] = 0.f;
+        for (int k0 = 0; k0 < p.kp; k0 += step) {
+            u32x4 c[R][U];
+#pragma unroll
+            for (int r = 0; r < R; ++r)
+#pragma unroll
+                for (int u = 0; u < U; ++u) c[r][u] = w[r][u];
+            if (k0 + step < p.kp)
+                fetch(g, k0 + step);
+            else if (g + n_wg * 4 < p.groups)
+                fetch(g + n_wg * 4, 0);
+#pragma unroll
+            for (int u = 0; u < U; ++u) {
+                const f32x4 x0 = *reinterpret_cast<const f32x4 *>(xs + k0 + (u * LPR + l) * 8);
+                const f32x4 x1 = *reinterpret_cast<const f32x4 *>(xs + k0 + (u * LPR + l) * 8 + 4);
+#pragma unroll
+                for (int r = 0; r < R; ++r) {
+                    const u32x4 v = c[r][u];
+                    acc[r] = fmaf(x0.x, __builtin_bit_cast(float, v.x << 16), acc[r]);
+                    acc[r] = fmaf(x0.y, __builtin_bit_cast(float, v.x & 0xffff0000u), acc[r]);
+                    acc[r] = fmaf(x0.z, __builtin_bit_cast(float, v.y << 16), acc[r]);
+                    acc[r] = fmaf(x0.w, __builtin_bit_cast(float, v.y & 0xffff0000u), acc[r]);
+                    acc[r] = fmaf(x1.x, __builtin_bit_cast(float, v.z << 16), acc[r]);
+                    acc[r] = fmaf(x1.y, __builtin_bit_cast(float, v.z & 0xffff0000u), acc[r]);
+                    acc[r] = fmaf(x1.z, __builtin_bit_cast(float, v.w << 16), acc[r]);
+                    acc[r] = fmaf(x1.w, __builtin_bit_cast(float, v.w & 0xffff0000u), acc[r]);
+                }
+            }
+        }
+        const int row0 = (g * G + sub) * R;
+#pragma unroll
+        for (int r = 0; r < R; ++r) {
+            acc[r] = LPR == 8 ? acc[r] + dpp<0x141>(acc[r]) : row_sum(acc[r]);  // (8 lanes: row_half_mirror first)
+            if (LPR == 8) {
+                acc[r] += dpp<0xb1>(acc[r]);  // quad_perm [1,0,3,2]
+                acc[r] += dpp<0x4e>(acc[r]);  // quad_perm [2,3,0,1]
+            }
+            if (LPR == 64) acc[r] = rows_sum(acc[r]);
+        }
+        if (l == 0) {
+#pragma unroll
+            for (int r = 0; r < R; ++r) {
+                const int row = row0 + r;
+                if (row >= a.rows) continue;
+                float v = acc[r];
+                if (a.bias) v += a.bias[row];
+                v = activate(v, row < a.act_split ? a.act0 : a.act1);
+                a.y[(size_t)b * a.y_batch + row] = v;
+                if (a.best_val) {
+                    const float t = v != v ? -INFINITY : v;
+                    if (t > bv || (t == bv && row < bi)) {
+                        bv = t;
+                        bi = row;
+                    }
+                }
+            }
+        }
+    }
+    if (a.best_val) {
+        // one candidate per row group of lanes, then per wave
+#pragma unroll
+        for (int off = 32; off >= LPR; off >>= 1) {
+            const float ov = __shfl_xor(bv, off, 64);
+            const int oi = __shfl_xor(bi, off, 64);
+            if (ov > bv || (ov == bv && oi < bi)) {
+                bv = ov;
+                bi = oi;
+            }
+        }
+        if (lane == 0) {
+            wbv[wave] = bv;
+            wbi[wave] = bi;
+        }
+        __syncthreads();
+        if (tid == 0) {
+            for (int i = 1; i < 4; ++i)
+                if (wbv[i] > bv || (wbv[i] == bv && wbi[i] < bi)) {
+                    bv = wbv[i];
+                    bi = wbi[i];
+                }
+            a.best_val[blockIdx.x] = bv;
+            a.best_idx[blockIdx.x] = bi;
+        }
+    }
+}
+
+template <int LPR, int R>
+static void gemv_pick_u(int u, const GemvK &k, dim3 grid, hipStream_t s) {
+    const size_t lds = (size_t)k.kp * 4;
+    void (*fn)(GemvK) = u == 1 ? k_dense_gemv<LPR, R, 1> : u == 2 ? k_dense_gemv<LPR, R, 2> : u == 3 ? k_dense_gemv<LPR, R, 3>
+                      : u == 4 ? k_dense_gemv<LPR, R, 4> : k_dense_gemv<LPR, R, 5>;
+    if (lds > 65536) (void)hipFuncSetAttribute(reinterpret_cast<const void *>(fn), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+    hipLaunchKernelGGL(fn, grid, dim3(256), lds, s, k);
+}
+
+hipError_t launch_dense_gemv(const GemvArgs &a, int *n_wg_out, hipStream_t s) {
+    GemvK k;
+    k.a = a;
+    k.a.latent = nullptr;
+    if (a.act_split == 0) k.a.act_split = a.rows;
+    if (k.a.in.mean_n == 0) k.a.in.mean_n = a.in.n;
+    const int lpr = a.cols <= 64 ? 8 : a.cols <= 256 ? 16 : 64;
+    const int chunks = (a.cols + lpr * 8 - 1) / (lpr * 8);
+    int u = chunks < 5 ? chunks : 5;
+    if (chunks > 5)
+        for (int c = 4; c >= 3; --c)
+            if ((chunks + c - 1) / c * c < (chunks + u - 1) / u * u) u = c;
+    const int step = lpr * 8 * u;
+    k.kp = (a.cols + step - 1) / step * step;
+    if ((size_t)k.kp * 4 > 150 * 1024) return hipErrorInvalidValue;
+    // rows per lane group: enough workgroups to reach every CU twice, then more rows in flight per wave
+    const int per = 64 / lpr;
+    auto wgs = [&](int r) { return ((long)a.rows + 4l * per * r - 1) / (4l * per * r) * a.batch; };
+    int r = 1;
+    if (wgs(4) >= 1024) r = 4;
+    else if (wgs(2) >= 512) r = 2;
+    k.groups = (a.rows + per * r - 1) / (per * r);
+    int n_wg = (k.groups + 3) / 4;
+    const int cap = 1024;  // four workgroups per CU
+    if (a.batch == 1 && n_wg > cap) {
+        const int rounds = (n_wg + cap - 1) / cap;
+        n_wg = (n_wg + rounds - 1) / rounds;
+    }
+    if (n_wg_out) *n_wg_out = n_wg;
+    k.lat_wg = a.latent ? n_wg : -1;
+    if (a.latent) k.lat = *a.latent;
+    const dim3 grid(n_wg + (a.latent ? 1 : 0), a.batch);
+    if (lpr == 8)
+        r == 4 ? gemv_pick_u<8, 4>(u, k, grid, s) : r == 2 ? gemv_pick_u<8, 2>(u, k, grid, s) : gemv_pick_u<8, 1>(u, k, grid, s);
+    else if (lpr == 16)
+        r == 4 ? gemv_pick_u<16, 4>(u, k, grid, s) : r == 2 ? gemv_pick_u<16, 2>(u, k, grid, s) : gemv_pick_u<16, 1>(u, k, grid, s);
+    else
+        r == 4 ? gemv_pick_u<64, 4>(u, k, grid, s) : r == 2 ? gemv_pick_u<64, 2>(u, k, grid, s) : gemv_pick_u<64, 1>(u, k, grid, s);
+    return hipGetLastError();
+}
+
+// ---- many-row matmul --------------------------------------------------------------------------------------------------
+// C[m][n] = act(A[m][k] . W[n][k]^T + bias).  128 x 128 workgroup tile, four waves of 64 x 64, K steps of 64 columns staged in
+// LDS by LDS-DMA, two buffers.  LDS image of a row: eight 16-byte units, unit q stored at q ^ (row & 7).  The MFMA's A operand
+// is the weight tile (rows = output columns n), its B operand the activation tile, so a lane holds four consecutive n of one row.
+constexpr int kTileM = 128, kTileN = 128, kTileK = 64;
+
+__device__ __forceinline__ void dma1k(const void *lane_ptr, unsigned lds_dst) {
+    unsigned keep;
+    asm volatile("s_mov_b32 %0, m0\n\ts_mov_b32 m0, %2\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %1, off\n\ts_mov_b32 m0, %0"
+                 : "=&s"(keep)
+                 : "v"(lane_ptr), "s"(lds_dst)
+                 : "memory");
+}
+
+template <bool CF32>
+__global__ __launch_bounds__(256, 2) void k_dense_gemm(GemmArgsD p, int tiles_n, int tiles_m, int swizzle) {
+    extern __shared__ __attribute__((aligned(1024))) uint8_t lds[];
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
+    // workgroup -> tile: consecutive workgroups land on the eight XCDs in turn; give each XCD a contiguous run of tiles that
+    // walks the row tiles of one weight tile first
+    int id = blockIdx.x;
+    const int total = tiles_n * tiles_m;
+    if (swizzle) id = (id & 7) * (total >> 3) + (id >> 3);
+    // groups of eight row tiles share the weight tiles they walk
+    const int gm = 8;
+    const int group = id / (gm * tiles_n), first = group * gm, size = tiles_m - first < gm ? tiles_m - first : gm;
+    const int tm = first + (id % (gm * tiles_n)) % size, tn = (id % (gm * tiles_n)) / size;
+    const int m0 = tm * kTileM, n0 = tn * kTileN;
+    const uint16_t *A = (const uint16_t *)p.a + (size_t)blockIdx.y * p.a_batch;
+    const uint16_t *W = p.w + (size_t)blockIdx.y * p.w_batch;
+    // LDS-DMA: one instruction stages eight rows of 64 columns (1 KiB); wave w stages rows [32 w, 32 w + 32) of both tiles
+    const int drow = lane >> 3, dunit = (lane & 7) ^ drow;
+    const uint16_t *ga[4], *gw[4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        const int r = wave * 32 + i * 8 + drow;
+        const int ar = m0 + r < p.m ? m0 + r : p.m - 1, wr = n0 + r < p.n ? n0 + r : p.n - 1;
+        ga[i] = A + (size_t)ar * p.lda + dunit * 8;
+        gw[i] = W + (size_t)wr * p.ldw + dunit * 8;
+    }
+    const unsigned base = (unsigned)(uintptr_t)(__attribute__((address_space(3))) uint8_t *)lds;
+    auto stage = [&](int k0, int buf) {
+        const unsigned dst = base + buf * 32768 + wave * 4096;
+#pragma unroll
+        for (int i = 0; i < 4; ++i) {
+            dma1k(ga[i] + k0, dst + i * 1024);
+            dma1k(gw[i] + k0, dst + 16384 + i * 1024);
+        }
+    };
+    const int wn = (wave & 1) * 64, wm = (wave >> 1) * 64;
+    const int r16 = lane & 15, g = lane >> 4;
+    f32x4 acc[4][4];
+#pragma unroll
+    for (int i = 0; i < 4; ++i)
+#pragma unroll
+        for (int j = 0; j < 4; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+    const int steps = p.k / kTileK;
+    stage(0, 0);
+    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    __syncthreads();
+    for (int t = 0; t < steps; ++t) {
+        if (t + 1 < steps) stage((t + 1) * kTileK, (t + 1) & 1);
+        const uint8_t *la = lds + (t & 1) * 32768, *lw = la + 16384;
+#pragma unroll
+        for (int kk = 0; kk < 2; ++kk) {
+            bf16x8 fa[4], fw[4];
+            const int q = ((kk * 4 + g) ^ (r16 & 7)) * 16;
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                fw[i] = *reinterpret_cast<const bf16x8 *>(lw + (wn + i * 16 + r16) * 128 + q);
+                fa[i] = *reinterpret_cast<const bf16x8 *>(la + (wm + i * 16 + r16) * 128 + q);
+            }
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+#pragma unroll
+                for (int j = 0; j < 4; ++j) acc[i][j] = mfma_bf16(fw[i], fa[j], acc[i][j]);
+        }
+        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // the next tile has landed
+        __syncthreads();
+    }
+    const bool vec = (p.ldc & 3) == 0;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        const int n = n0 + wn + i * 16 + g * 4;
+        if (n >= p.n) continue;
+        float bias[4];
+#pragma unroll
+        for (int e = 0; e < 4; ++e) bias[e] = p.bias && n + e < p.n ? p.bias[n + e] : 0.f;
+#pragma unroll
+        for (int j = 0; j < 4; ++j) {
+            const int m = m0 + wm + j * 16 + r16;
+            if (m >= p.m) continue;
+            float v[4];
+#pragma unroll
+            for (int e = 0; e < 4; ++e) v[e] = activate(acc[i][j][e] + bias[e], n + e < p.act_split ? p.act0 : p.act1);
+            const size_t o = (size_t)blockIdx.y * p.c_batch + (size_t)m * p.ldc + n;
+            if (vec && n + 3 < p.n) {
+                if (CF32)
+                    *reinterpret_cast<f32x4 *>((float *)p.c + o) = f32x4{v[0], v[1], v[2], v[3]};
+                else
+                    *reinterpret_cast<bf16x4 *>((uint16_t *)p.c + o) = bf16x4{(__bf16)v[0], (__bf16)v[1], (__bf16)v[2], (__bf16)v[3]};
+            } else {
+                for (int e = 0; e < 4 && n + e < p.n; ++e) {
+                    if (CF32)
+                        ((float *)p.c)[o + e] = v[e];
+                    else
+                        ((uint16_t *)p.c)[o + e] = f2bf(v[e]);
+                }
+            }
+        }
+    }
+}
+
+// f32 activations: f32 multiply-adds on a 64 x 64 tile, 4 x 4 per thread
+__global__ __launch_bounds__(256) void k_dense_gemm_f32(GemmArgsD p) {
+    __shared__ float sa[16][68], sw[16][68];
+    const int tid = threadIdx.x, tx = tid & 15, ty = tid >> 4;
+    const int m0 = blockIdx.y * 64, n0 = blockIdx.x * 64;
+    const float *A = (const float *)p.a + (size_t)blockIdx.z * p.a_batch;
+    const uint16_t *W = p.w + (size_t)blockIdx.z * p.w_batch;
+    float acc[4][4] = {};
+    const int lr = tid >> 2, lk = (tid & 3) * 4;
+    const int ar = m0 + lr < p.m ? m0 + lr : p.m - 1, wr = n0 + lr < p.n ? n0 + lr : p.n - 1;
+    for (int k0 = 0; k0 < p.k; k0 += 16) {
+        const f32x4 av = *reinterpret_cast<const f32x4 *>(A + (size_t)ar * p.lda + k0 + lk);
+        const u32x2 wv = *reinterpret_cast<const u32x2 *>(W + (size_t)wr * p.ldw + k0 + lk);
+        __syncthreads();
+        sa[lk][lr] = av.x, sa[lk + 1][lr] = av.y, sa[lk + 2][lr] = av.z, sa[lk + 3][lr] = av.w;
+        sw[lk][lr] = bf2f(wv.x & 0xffffu), sw[lk + 1][lr] = bf2f(wv.x >> 16), sw[lk + 2][lr] = bf2f(wv.y & 0xffffu), sw[lk + 3][lr] = bf2f(wv.y >> 16);
+        __syncthreads();
+#pragma unroll
+        for (int k = 0; k < 16; ++k) {
+            float x[4], w[4];
+#pragma unroll
+            for (int i = 0; i < 4; ++i) x[i] = sa[k][ty * 4 + i], w[i] = sw[k][tx * 4 + i];
+#pragma unroll
+            for (int i = 0; i < 4; ++i)
+#pragma unroll
+                for (int j = 0; j < 4; ++j) acc[i][j] = fmaf(x[i], w[j], acc[i][j]);
+        }
+    }
+    for (int i = 0; i < 4; ++i) {
+        const int m = m0 + ty * 4 + i;
+        if (m >= p.m) break;
+        for (int j = 0; j < 4; ++j) {
+            const int n = n0 + tx * 4 + j;
+            if (n >= p.n) break;
+            const float v = activate(acc[i][j] + (p.bias ? p.bias[n] : 0.f), n < p.act_split ? p.act0 : p.act1);
+            const size_t o = (size_t)blockIdx.z * p.c_batch + (size_t)m * p.ldc + n;
+            if (p.c_f32)
+                ((float *)p.c)[o] = v;
+            else
+                ((uint16_t *)p.c)[o] = f2bf(v);
+        }
+    }
+}
+
+hipError_t launch_dense_gemm(const GemmArgsD &args, hipStream_t s) {
+    GemmArgsD a = args;
+    if (a.m <= 0 || a.n <= 0) return hipSuccess;
+    if (a.act_split == 0) a.act_split = a.n;
+    if (a.a_f32) {
+        hipLaunchKernelGGL(k_dense_gemm_f32, dim3((a.n + 63) / 64, (a.m + 63) / 64, a.batch), dim3(256), 0, s, a);
+        return hipGetLastError();
+    }
+    const int tn = (a.n + kTileN - 1) / kTileN, tm = (a.m + kTileM - 1) / kTileM;
+    const int swz = (tn * tm) % 8 == 0 ? 1 : 0;
+    if (a.c_f32)
+        hipLaunchKernelGGL(k_dense_gemm<true>, dim3(tn * tm, a.batch), dim3(256), 65536, s, a, tn, tm, swz);
+    else
+        hipLaunchKernelGGL(k_dense_gemm<false>, dim3(tn * tm, a.batch), dim3(256), 65536, s, a, tn, tm, swz);
+    return hipGetLastError();
+}
+
+}  // namespace bitnet_hip

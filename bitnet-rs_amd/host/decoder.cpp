@@ -17,42 +17,6 @@
 
 namespace bitnet_host {
 
-namespace {
-struct Event {  // RAII: an error return between create and destroy must not leak the event
-    hipEvent_t e = nullptr;
-    ~Event() {
-        if (e) hipEventDestroy(e);
-    }
-};
-}  // namespace
-
-#define HCHK(expr)                                                                     \
-    do {                                                                               \
-        hipError_t _e = (expr);                                                        \
-        if (_e != hipSuccess) {                                                        \
-            char _b[256];                                                              \
-            snprintf(_b, sizeof(_b), "HIP error %s at %s:%d (%s)", hipGetErrorName(_e), __FILE__, __LINE__, #expr); \
-            err_ = _b;                                                                 \
-            return BITNET_HIP_ERR_GPU;                                                 \
-        }                                                                              \
-    } while (0)
-#define BCHK(expr)                       \
-    do {                                 \
-        int _rc = (expr);                \
-        if (_rc != 0) return fail(#expr); \
-    } while (0)
-
-int Decoder::fail_arg(const char *what) {
-    err_ = what;
-    return BITNET_HIP_ERR_INVALID_ARGUMENT;
-}
-
-int Decoder::fail(const char *what) {
-    const char *e = bitnet_hip_get_last_error();
-    err_ = std::string(what) + ": " + (e ? e : "error");
-    return BITNET_HIP_ERR_EXECUTION;
-}
-
 template <class T>
 static hipError_t dalloc(T **p, size_t n) {
     return hipMalloc(reinterpret_cast<void **>(p), n * sizeof(T) ? n * sizeof(T) : 1);
@@ -76,7 +40,6 @@ static std::string config_problem(const Config &c) {
 Decoder::Decoder(const Config &cfg) : c_(cfg), layers_(cfg.n_layers > 0 && cfg.n_layers <= 4096 ? (size_t)cfg.n_layers : 0) {
     // A rejected configuration or a failed allocation leaves a DEAD object: error() says why, every other entry point
     // returns an error without touching a member (c_ used to keep the rejected n_layers while layers_ was empty).
-    dead_ = true;
     err_ = config_problem(cfg);
     if (!err_.empty()) {
         layers_.clear();
@@ -87,17 +50,7 @@ Decoder::Decoder(const Config &cfg) : c_(cfg), layers_(cfg.n_layers > 0 && cfg.n
     if (const char *e = getenv("BITNET_HOST_KV16")) kv_f16_ = atoi(e) != 0;  // opt-in f16 KV cache (long contexts)
     if (const char *e = getenv("BITNET_HOST_ACT")) act_mode_ = atoi(e) != 0 ? 1 : 0;  // 0: exact f32 activations between the kernels
     if (const char *e = getenv("BITNET_HOST_PREFILL_CHAIN")) prefill_chain_ = atoi(e) != 0 ? 1 : 0;  // the prompt forward's f16 activation chain
-    if (bitnet_hip_init(-1) != 0) {
-        const char *e = bitnet_hip_get_last_error();
-        err_ = e ? e : "bitnet_hip_init failed";
-        return;
-    }
-    hipStream_t s;
-    if (hipStreamCreateWithFlags(&s, hipStreamNonBlocking) != hipSuccess) {
-        err_ = "hipStreamCreate failed";
-        return;
-    }
-    stream_ = s;
+    if (init_sequence(c_.vocab, c_.hidden, c_.max_pos) != 0) return;
     const size_t H = c_.hidden, D = c_.head_dim, half = D / 2;
     {
         // bitnet_hip_gemv_attn_merge_dev's shape limits (include/bitnet_hip.h)
@@ -122,15 +75,12 @@ Decoder::Decoder(const Config &cfg) : c_(cfg), layers_(cfg.n_layers > 0 && cfg.n
     }
     ok &= dalloc(&ref_n_, H > (size_t)c_.ffn ? H : (size_t)c_.ffn) == hipSuccess && dalloc(&ref_gu_, 2 * (size_t)c_.ffn) == hipSuccess &&
           dalloc(&ref_t_, H) == hipSuccess;
-    ok &= dalloc(&logits_, (size_t)c_.vocab) == hipSuccess;
     ok &= hipMalloc(&scratch_, 8 * (size_t)logits_wgs_) == hipSuccess;
     {
         const size_t sb = bitnet_hip_attention_scratch_bytes((size_t)c_.n_kv_heads, (size_t)c_.max_pos);
         // zero-filled: the merging o-projection reads records of chunks past the context (and gives them zero weight)
         ok = ok && hipMalloc((void **)&attn_scratch_, sb) == hipSuccess && hipMemset(attn_scratch_, 0, sb) == hipSuccess;
     }
-    ok &= dalloc(&pos_, 1) == hipSuccess && dalloc(&n_forced_, 1) == hipSuccess && dalloc(&token_, 1) == hipSuccess;
-    ok &= dalloc(&history_, (size_t)c_.max_pos + 2) == hipSuccess;
     ok &= dalloc(&rope_sin_, (size_t)c_.max_pos * half) == hipSuccess;
     ok &= dalloc(&rope_cos_, (size_t)c_.max_pos * half) == hipSuccess;
     for (auto &L : layers_) {
@@ -172,8 +122,7 @@ Decoder::~Decoder() {
             if (p) hipFree(p);
     }
     for (void *p : {(void *)embed_, (void *)final_norm_, (void *)rope_sin_, (void *)rope_cos_, (void *)x_, (void *)x2_,
-                    (void *)qkv_, (void *)att_, (void *)h_, (void *)ref_n_, (void *)ref_gu_, (void *)ref_t_, qa_x_, qa_x2_, qa_att_, qa_h_, (void *)st_x_, (void *)st_x2_, (void *)logits_, scratch_, (void *)attn_scratch_, (void *)pos_, (void *)n_forced_,
-                    (void *)history_, (void *)token_})
+                    (void *)qkv_, (void *)att_, (void *)h_, (void *)ref_n_, (void *)ref_gu_, (void *)ref_t_, qa_x_, qa_x2_, qa_att_, qa_h_, (void *)st_x_, (void *)st_x2_, scratch_, (void *)attn_scratch_})
         if (p) hipFree(p);
     for (void *p : {(void *)pf_x_, (void *)pf_qkv_, (void *)pf_att_, (void *)pf_h_, pf_gemm_ws_, pf_attn_ws_, sp_kv_send_, sp_kv_all_,
                     (void *)sp_block_pos_, (void *)sp_tokens_, pf_xh_, pf_atth_, pf_hh_, (void *)pf_stats_, pf_qb_})
@@ -183,7 +132,6 @@ Decoder::~Decoder() {
     if (sp_ev_pack_) hipEventDestroy((hipEvent_t)sp_ev_pack_);
     if (sp_ev_gather_) hipEventDestroy((hipEvent_t)sp_ev_gather_);
     if (comm_stream_) hipStreamDestroy((hipStream_t)comm_stream_);
-    if (stream_) hipStreamDestroy((hipStream_t)stream_);
 }
 
 // A layer that already holds weights gives them back first, and every captured step graph goes (the graphs
@@ -197,14 +145,6 @@ void Decoder::release_layer(Layer &L) {
         *h = 0;
     }
     drop_graphs();
-}
-
-void Decoder::drop_graphs() {
-    for (int i = 0; i < kGraphs; ++i) {
-        if (graph_exec_[i]) hipGraphExecDestroy((hipGraphExec_t)graph_exec_[i]);
-        if (graph_[i]) hipGraphDestroy((hipGraph_t)graph_[i]);
-        graph_exec_[i] = graph_[i] = nullptr;
-    }
 }
 
 // the four fused handles of a layer from its seven uploaded projections; frees the seven on every path
@@ -334,48 +274,6 @@ int Decoder::set_globals(const uint16_t *embed_f16, const float *final_norm) {
     HCHK(hipMemcpy(embed_, embed_f16, n, hipMemcpyHostToDevice));
     HCHK(hipMemcpy(final_norm_, final_norm, (size_t)c_.hidden * 4, hipMemcpyHostToDevice));
     return 0;
-}
-
-int Decoder::reset() {
-    host_forced_ = 0;
-    HCHK(hipMemset(pos_, 0, 4));
-    HCHK(hipMemset(n_forced_, 0, 4));
-    HCHK(hipMemset(history_, 0, ((size_t)c_.max_pos + 2) * 4));
-    return 0;
-}
-
-int Decoder::feed(const int32_t *tokens, int n) {
-    const int p = position();
-    if (p < 0) return BITNET_HIP_ERR_GPU;
-    const int base = p > host_forced_ ? p : host_forced_;
-    if (n < 0 || (n > 0 && !tokens)) {
-        err_ = "feed: null tokens";
-        return BITNET_HIP_ERR_INVALID_ARGUMENT;
-    }
-    for (int i = 0; i < n; ++i)
-        if (tokens[i] < 0 || tokens[i] >= c_.vocab) {  // TransformerModel::embed's index_select fails on it (T:1390-1426)
-            char b[96];
-            snprintf(b, sizeof(b), "token id %d out of range [0, %d)", tokens[i], c_.vocab);
-            err_ = b;
-            return BITNET_HIP_ERR_INVALID_ARGUMENT;
-        }
-    if (base + n > c_.max_pos) {
-        err_ = "KV cache overflow";  // T:1190-1194
-        return BITNET_HIP_ERR_INVALID_ARGUMENT;
-    }
-    HCHK(hipMemcpy(history_ + base, tokens, (size_t)n * 4, hipMemcpyHostToDevice));
-    host_forced_ = base + n;
-    HCHK(hipMemcpy(n_forced_, &host_forced_, 4, hipMemcpyHostToDevice));
-    return 0;
-}
-
-int Decoder::position() {
-    int p = -1;
-    if (hipMemcpy(&p, pos_, 4, hipMemcpyDeviceToHost) != hipSuccess) {
-        err_ = "position readback failed";
-        return -1;
-    }
-    return p;
 }
 
 // The decode attention in the form and cache type this decoder runs: form 0 two kernels (64-position records), 1 records only
@@ -632,88 +530,14 @@ int Decoder::form_at(int pos) const {
     return 0;
 }
 
-int Decoder::prepare_graphs(bool with_logits) {
-    if (!embed_) {
-        err_ = "model globals not set";
-        return BITNET_HIP_ERR_INVALID_ARGUMENT;
-    }
-    unsigned forms = 0;
-    for (int pos = 0; pos + 1 < c_.max_pos; ++pos) forms |= 1u << form_at(pos);
-    for (int f = 0; f < kGraphs / 2; ++f)
-        if (forms & (1u << f))
-            if (int rc = ensure_graph(with_logits, f)) return rc;
-    return 0;
-}
-
-int Decoder::ensure_graph(bool with_logits, int form) {
-    const int gi = 2 * form + (with_logits ? 1 : 0);
-    if (graph_exec_[gi]) return 0;
-    hipStream_t s = (hipStream_t)stream_;
-    hipGraph_t g = nullptr;
-    HCHK(hipStreamBeginCapture(s, hipStreamCaptureModeGlobal));
-    const int rc = step_launches(with_logits, form);
-    const hipError_t e = hipStreamEndCapture(s, &g);
-    if (rc != 0) {
-        if (g) hipGraphDestroy(g);
-        return rc;
-    }
-    HCHK(e);
-    hipGraphExec_t ex = nullptr;
-    HCHK(hipGraphInstantiate(&ex, g, nullptr, nullptr, 0));
-    graph_[gi] = g;
-    graph_exec_[gi] = ex;
-    return 0;
-}
-
 int Decoder::run(int n, bool with_logits, bool use_graph, float *elapsed_ms) {
-    if (!embed_) {
-        err_ = "model globals not set";
-        return BITNET_HIP_ERR_INVALID_ARGUMENT;
-    }
-    const int p = position();
-    if (p < 0) return BITNET_HIP_ERR_GPU;
-    if (p + n > c_.max_pos - 1) {
-        err_ = "KV cache overflow";  // T:1190-1194
-        return BITNET_HIP_ERR_INVALID_ARGUMENT;
-    }
-    if (!with_logits && p + n > host_forced_) {
-        // a step without logits samples nothing: the NEXT position's token must already be in the history
-        err_ = "run(with_logits = false) past the fed tokens: nothing would choose the next token";
-        return BITNET_HIP_ERR_INVALID_ARGUMENT;
-    }
-    if (!trace_dir_.empty()) {  // BITNET_TRACE_DIR: every step eagerly, with read-backs (slow by design)
-        for (int i = 0; i < n; ++i) {
-            const int rc = trace_step(trace_dir_.c_str(), with_logits);
-            if (rc) return rc;
-        }
-        if (elapsed_ms) *elapsed_ms = 0.f;
-        return 0;
-    }
-    hipStream_t s = (hipStream_t)stream_;
-    if (use_graph) {
-        for (int i = 0; i < n; ++i) {  // every form this run needs (at most three captures)
-            int rc = ensure_graph(with_logits, form_at(p + i));
-            if (rc) return rc;
-        }
-    }
-    Event ev0, ev1;
-    HCHK(hipEventCreate(&ev0.e));
-    HCHK(hipEventCreate(&ev1.e));
-    hipEvent_t e0 = ev0.e, e1 = ev1.e;
-    HCHK(hipEventRecord(e0, s));
+    if (trace_dir_.empty()) return Sequence::run(n, with_logits, use_graph, elapsed_ms);
+    if (int rc = check_run(n, with_logits)) return rc;
     for (int i = 0; i < n; ++i) {
-        if (use_graph) {
-            HCHK(hipGraphLaunch((hipGraphExec_t)graph_exec_[2 * form_at(p + i) + (with_logits ? 1 : 0)], s));
-        } else {
-            int rc = step_launches(with_logits, form_at(p + i));
-            if (rc) return rc;
-        }
+        const int rc = trace_step(trace_dir_.c_str(), with_logits);
+        if (rc) return rc;
     }
-    HCHK(hipEventRecord(e1, s));
-    HCHK(hipStreamSynchronize(s));
-    float ms = 0.f;
-    HCHK(hipEventElapsedTime(&ms, e0, e1));
-    if (elapsed_ms) *elapsed_ms = ms;
+    if (elapsed_ms) *elapsed_ms = 0.f;
     return 0;
 }
 
@@ -1280,18 +1104,6 @@ void Decoder::global_objects(void *ptrs[7]) const {
     ptrs[0] = embed_, ptrs[1] = final_norm_, ptrs[2] = rope_sin_, ptrs[3] = rope_cos_, ptrs[4] = history_, ptrs[5] = pos_, ptrs[6] = stream_;
 }
 
-int Decoder::history(int32_t *out, int n) {
-    if (!out || n < 0 || n > c_.max_pos + 2) {
-        err_ = "history: n out of range";
-        return BITNET_HIP_ERR_INVALID_ARGUMENT;
-    }
-    HCHK(hipMemcpy(out, history_, (size_t)n * 4, hipMemcpyDeviceToHost));
-    return 0;
-}
-int Decoder::last_logits(float *out) {
-    HCHK(hipMemcpy(out, logits_, (size_t)c_.vocab * 4, hipMemcpyDeviceToHost));
-    return 0;
-}
 int Decoder::last_hidden(float *out) {
     HCHK(hipMemcpy(out, x_, (size_t)c_.hidden * 4, hipMemcpyDeviceToHost));
     return 0;
@@ -1402,9 +1214,9 @@ int Decoder::probe_gateup(int reps, float *us_per_launch, double *bytes_per_laun
 using bitnet_host::Decoder;
 
 namespace {
-// a null handle or a dead decoder (rejected configuration, failed allocation): nothing but error() / destroy may be called
+// a null handle, a dead decoder (rejected configuration, failed allocation) or a model of another design: nothing here may be called
 inline Decoder *live(void *d) {
-    Decoder *p = static_cast<Decoder *>(d);
+    Decoder *p = d ? dynamic_cast<Decoder *>(static_cast<bitnet_host::Sequence *>(d)) : nullptr;
     return p && !p->dead() ? p : nullptr;
 }
 }  // namespace
@@ -1428,13 +1240,11 @@ void *bitnet_host_create(const bitnet_host_config *cfg) {
     // Nothing is thrown across the C boundary: a configuration the kernels cannot take comes back as a decoder
     // whose error() says why (every later call on it fails), allocation failures as nullptr.
     try {
-        return new Decoder(c);
+        return static_cast<bitnet_host::Sequence *>(new Decoder(c));
     } catch (...) {
         return nullptr;
     }
 }
-void bitnet_host_destroy(void *d) { delete static_cast<Decoder *>(d); }
-const char *bitnet_host_error(void *d) { return d ? static_cast<Decoder *>(d)->error().c_str() : "null decoder"; }
 int bitnet_host_set_layer_qk256(void *d, int layer, const float *attn_norm, const float *ffn_norm, const uint8_t *q,
                                 const uint8_t *k, const uint8_t *v, const uint8_t *o, const uint8_t *gate,
                                 const uint8_t *up, const uint8_t *down) {
@@ -1459,21 +1269,10 @@ int bitnet_host_set_globals(void *d, const uint16_t *embed_f16, const float *fin
     LIVE(BITNET_HIP_ERR_INVALID_ARGUMENT);
     return D->set_globals(embed_f16, final_norm);
 }
-int bitnet_host_reset(void *d) { LIVE(BITNET_HIP_ERR_INVALID_ARGUMENT); return D->reset(); }
-int bitnet_host_feed(void *d, const int32_t *tokens, int n) { LIVE(BITNET_HIP_ERR_INVALID_ARGUMENT); return D->feed(tokens, n); }
 int bitnet_host_set_kv_f16(void *d, int on) { LIVE(BITNET_HIP_ERR_INVALID_ARGUMENT); return D->set_kv_f16(on != 0); }
 int bitnet_host_set_act_mode(void *d, int mode) { LIVE(BITNET_HIP_ERR_INVALID_ARGUMENT); return D->set_act_mode(mode); }
 int bitnet_host_act_mode(void *d) { LIVE(0); return D->qact_path() ? 1 : 0; }
-int bitnet_host_prepare_graphs(void *d, int with_logits) { LIVE(BITNET_HIP_ERR_INVALID_ARGUMENT); return D->prepare_graphs(with_logits != 0); }
 int bitnet_host_run_reference(void *d, int n, int with_logits) { LIVE(BITNET_HIP_ERR_INVALID_ARGUMENT); return D->run_reference(n, with_logits != 0); }
-int bitnet_host_run(void *d, int n, int with_logits, int use_graph, float *elapsed_ms) {
-    LIVE(BITNET_HIP_ERR_INVALID_ARGUMENT);
-    return D->run(n, with_logits != 0, use_graph != 0, elapsed_ms);
-}
-int bitnet_host_prefill(void *d, int n, int with_logits, int digits, float *elapsed_ms) {
-    LIVE(BITNET_HIP_ERR_INVALID_ARGUMENT);
-    return D->prefill(n, with_logits != 0, digits, elapsed_ms);
-}
 int bitnet_host_prefill_sharded(void *d, int n, int rank, int world, bitnet_host_allgather_fn gather, void *gather_ctx, int with_logits,
                                 int digits, int wire_f16, float *elapsed_ms) {
     LIVE(BITNET_HIP_ERR_INVALID_ARGUMENT);
@@ -1513,12 +1312,8 @@ void bitnet_host_global_objects(void *d, void **ptrs7) {
     for (int i = 0; i < 7; ++i) ptrs7[i] = nullptr;
     if (Decoder *D = live(d)) D->global_objects(ptrs7);
 }
-int bitnet_host_position(void *d) { LIVE(-1); return D->position(); }
 int bitnet_host_last_prefill_path(void *d) { LIVE(-1); return D->last_prefill_path(); }
 int bitnet_host_saturation_fallbacks(void *d) { LIVE(-1); return D->saturation_fallbacks(); }
-int bitnet_host_history(void *d, int32_t *out, int n) { LIVE(BITNET_HIP_ERR_INVALID_ARGUMENT); return D->history(out, n); }
-int bitnet_host_last_logits(void *d, float *out) { LIVE(BITNET_HIP_ERR_INVALID_ARGUMENT); return D->last_logits(out); }
-int bitnet_host_last_hidden(void *d, float *out) { LIVE(BITNET_HIP_ERR_INVALID_ARGUMENT); return D->last_hidden(out); }
 int bitnet_host_blake3_hex(const void *data, size_t len, char *out65) {
     if (!out65 || (!data && len)) return -1;
     const std::string h = bitnet_host::Blake3::hex(data, len);
@@ -1534,5 +1329,4 @@ int bitnet_host_probe_kernel(void *d, int kind, int reps, float *us_per_launch, 
     LIVE(BITNET_HIP_ERR_INVALID_ARGUMENT);
     return D->probe_kernel(kind, reps, us_per_launch, bytes_per_launch);
 }
-uint64_t bitnet_host_weight_bytes(void *d) { LIVE(0); return D->weight_bytes(); }
 }

@@ -17,6 +17,7 @@
 #include <vector>
 
 #include "bitnet_hip.h"
+#include "sequence.hpp"
 
 extern "C" {
 // The collective of the token-parallel prefill as the host supplies it: gather `bytes_per_rank` bytes from every rank into
@@ -59,17 +60,12 @@ struct ProjSpec {
     int8_t code_map[4] = {-2, -1, 0, 1};
 };
 
-class Decoder {
+class Decoder : public Sequence {
   public:
     explicit Decoder(const Config &cfg);
-    ~Decoder();
-    Decoder(const Decoder &) = delete;
-    Decoder &operator=(const Decoder &) = delete;
+    ~Decoder() override;
 
     const Config &config() const { return c_; }
-    const std::string &error() const { return err_; }
-    bool dead() const { return dead_; }  // construction failed: only error() and the destructor may be used
-    void set_error(const std::string &e) { err_ = e; }
 
     // weights (uploaded once; fused q|k|v and interleaved gate/up handles are built here)
     int set_layer_qk256(int layer, const LayerWeightsQk256 &w);
@@ -78,14 +74,8 @@ class Decoder {
     int set_layer_specs(int layer, const float *attn_norm, const float *ffn_norm, const ProjSpec p[7]);
     int set_globals(const uint16_t *embed_f16, const float *final_norm);
 
-    // KVCache::clear (T:1251-1255) + token history
-    int reset();
-    // Put `n` forced tokens at positions [pos, pos+n) of the history (the prompt).
-    int feed(const int32_t *tokens, int n);
-    // Run `n` single-token steps (T:1482-1504 body each).  with_logits=false skips the
-    // logits GEMV for prompt positions nobody samples from.  Uses the captured graph
-    // when use_graph, else eager launches.  Synchronises the stream before returning.
-    int run(int n, bool with_logits, bool use_graph, float *elapsed_ms);
+    // Every step eagerly, with read-backs, when BITNET_TRACE_DIR is set (slow by design); else the shared loop.
+    int run(int n, bool with_logits, bool use_graph, float *elapsed_ms) override;
     // The same n steps UNFUSED, in the reference's op order, every projection on the reference-order (bit-exact)
     // kernel: the checker bench.py and the tests hold the fast step against at the full model size.  Eager, slow.
     int run_reference(int n, bool with_logits);
@@ -102,7 +92,7 @@ class Decoder {
     // T:1557-1597): tiled matmuls + causal attention, KV cache filled for positions 0..n-1.
     // with_logits samples the token after the prompt exactly as run() does for the last
     // prompt position.  digits: fixed-point digits per activation in the matmuls (2..4).
-    int prefill(int n, bool with_logits, int digits, float *elapsed_ms);
+    int prefill(int n, bool with_logits, int digits, float *elapsed_ms) override;
     // Token-parallel prefill of ONE long prompt over `world` GPUs, one process per GPU:
     // this rank runs the first n fed tokens' zigzag chunks rank and 2 world - 1 - rank through every layer (weights are
     // replicated: all seven projections are collective-free); per layer ONE all-gather of the raw k|v rows through
@@ -133,10 +123,7 @@ class Decoder {
     // history, pos, stream}.
     void layer_objects(int layer, uint64_t handles[4], void *ptrs[4]) const;
     void global_objects(void *ptrs[7]) const;
-    int position();                                  // tokens consumed so far
-    int history(int32_t *out, int n);                // first n tokens of the sequence
-    int last_logits(float *out);                     // [vocab], of the last step run with logits
-    int last_hidden(float *out);                     // residual stream after the last block (pre final norm)
+    int last_hidden(float *out) override;
     // Activation trace of ONE decode step in the reference's format (crates/bitnet-trace/src/lib.rs:46-168: one JSON file per
     // tensor -- name, shape, dtype, blake3 of the raw f32 bytes, rms, num_elements, seq, layer, stage -- in `dir`): the step
     // runs eagerly, every intermediate is materialised as f32 and read back after its kernel.  Stages: embeddings; per
@@ -149,30 +136,20 @@ class Decoder {
     int probe_gateup(int reps, float *us_per_launch, double *bytes_per_launch);
     // Same for any kernel of the step: kind 0 q|k|v, 1 attention, 2 o_proj, 3 gate|up, 4 down, 5 logits.
     int probe_kernel(int kind, int reps, float *us_per_launch, double *bytes_per_launch);
-    size_t weight_bytes() const { return weight_bytes_; }  // algorithmic bytes of all I2_S matrices
-    void *stream() const { return stream_; }
+    size_t weight_bytes() const override { return weight_bytes_; }  // algorithmic bytes of all I2_S matrices
 
   private:
-    int fail(const char *what);
-    int fail_arg(const char *what);
-    bool dead_ = false;
     // attention form of a step: 0 = two kernels, 64-position chunks; 1 = one kernel + merging o-projection (short
     // contexts); 2 = two kernels, 128-position chunks (more chunks than CUs)
     struct Tracer;
     int step_launches(bool with_logits, int form, Tracer *tr = nullptr);
     int step_launches_reference(bool with_logits);
-    int ensure_graph(bool with_logits, int form);
-  public:
-    // Captures and instantiates the step graph of every attention form a sequence can reach (by position: form_at) ahead of
-    // time, so that no run() pays for a capture in the middle of a generation.  Nothing executes.
-    int prepare_graphs(bool with_logits);
-  private:
-    int form_at(int pos) const;
+    bool ready() const override { return embed_ != nullptr; }
+    int step(bool with_logits, int form) override { return step_launches(with_logits, form); }
+    int form_at(int pos) const override;
     bool merge_ok_ = false;  // the o-projection can merge the attention chunk records itself (short contexts)
 
     Config c_;
-    std::string err_;
-    void *stream_ = nullptr;
     struct Layer {
         float *attn_norm = nullptr, *ffn_norm = nullptr;
         bitnet_hip_weights_t qkv = 0, o = 0, gateup = 0, down = 0;
@@ -181,13 +158,12 @@ class Decoder {
     };
     int attn_launch(Layer &L, int form, float *out, void *qout);
     void release_layer(Layer &L);  // frees the layer's handles, subtracts their bytes, drops the captured graphs
-    void drop_graphs();
     int adopt_projections(Layer &L, bitnet_hip_weights_t h[7]);
     std::vector<Layer> layers_;
     void *embed_ = nullptr;
     float *final_norm_ = nullptr;
     float *rope_sin_ = nullptr, *rope_cos_ = nullptr;
-    float *x_ = nullptr, *x2_ = nullptr, *qkv_ = nullptr, *att_ = nullptr, *h_ = nullptr, *logits_ = nullptr;
+    float *x_ = nullptr, *x2_ = nullptr, *qkv_ = nullptr, *att_ = nullptr, *h_ = nullptr;
     void *qa_x_ = nullptr, *qa_x2_ = nullptr, *qa_att_ = nullptr, *qa_h_ = nullptr;  // QAct records of x, x2, attention output, silu(gate)*up
     double *st_x_ = nullptr, *st_x2_ = nullptr;                                       // LayerNorm statistics pairs of x, x2
     int act_mode_ = 1;
@@ -196,8 +172,6 @@ class Decoder {
     float *ref_n_ = nullptr, *ref_gu_ = nullptr, *ref_t_ = nullptr;  // unfused reference step: normalised row, gate|up tiles, projection out
     void *scratch_ = nullptr;
     float *attn_scratch_ = nullptr;
-    int32_t *pos_ = nullptr, *n_forced_ = nullptr, *history_ = nullptr, *token_ = nullptr;
-    int host_forced_ = 0;
     // sharded prefill buffers (grown on demand)
     int sp_cap_ = 0, sp_ctx_ = 0;
     void *sp_kv_send_ = nullptr, *sp_kv_all_ = nullptr;
@@ -227,38 +201,29 @@ class Decoder {
     int prefill_chain_ = -1;  // BITNET_HOST_PREFILL_CHAIN: -1 automatic (the block-scaled format, whose matmul runs on f16 activations anyway), 0 off, 1 on
     size_t pf_gemm_ws_bytes_ = 0, pf_attn_ws_bytes_ = 0;
     size_t weight_bytes_ = 0;
-    static constexpr int kGraphs = 6;
-    void *graph_exec_[kGraphs] = {};  // [2 * form + with_logits], forms 0..2 (form_at)
-    void *graph_[kGraphs] = {};
     int logits_wgs_ = 512;  // two workgroups per CU: whole rounds on the 256 CUs (768 / 1280 workgroups are 15-20 % slower)
 };
 
 }  // namespace bitnet_host
 
-// C shim for the Python tests / bench (ctypes).  Not part of the kernel boundary.
+// C shim for the Python tests / bench (ctypes).  Not part of the kernel boundary.  The entries every model shares (destroy, error,
+// reset, feed, run, prefill, forward, position, ...) are in registry.hpp; the handles are the same.
 extern "C" {
 typedef struct bitnet_host_config {
     int32_t hidden, n_layers, n_heads, n_kv_heads, head_dim, ffn, vocab, max_pos;
     float eps, rope_theta;
 } bitnet_host_config;
 void *bitnet_host_create(const bitnet_host_config *cfg);
-void bitnet_host_destroy(void *d);
-const char *bitnet_host_error(void *d);
 int bitnet_host_set_layer_qk256(void *d, int layer, const float *attn_norm, const float *ffn_norm,
                                 const uint8_t *q, const uint8_t *k, const uint8_t *v, const uint8_t *o,
                                 const uint8_t *gate, const uint8_t *up, const uint8_t *down);
 int bitnet_host_set_layer_i2s(void *d, int layer, const float *attn_norm, const float *ffn_norm,
                               const uint8_t *const *w7, const float *const *scales7, size_t block_size);
 int bitnet_host_set_globals(void *d, const uint16_t *embed_f16, const float *final_norm);
-int bitnet_host_reset(void *d);
-int bitnet_host_feed(void *d, const int32_t *tokens, int n);
-int bitnet_host_run(void *d, int n, int with_logits, int use_graph, float *elapsed_ms);
 int bitnet_host_run_reference(void *d, int n, int with_logits);
-int bitnet_host_prepare_graphs(void *d, int with_logits);
 int bitnet_host_set_act_mode(void *d, int mode);
 int bitnet_host_set_kv_f16(void *d, int on);
 int bitnet_host_act_mode(void *d);
-int bitnet_host_prefill(void *d, int n, int with_logits, int digits, float *elapsed_ms);
 int bitnet_host_finish_prefill(void *d, int n, const float *last_row, int with_logits);
 // per-phase medians of the NEXT bitnet_host_prefill_sharded calls (off by default: 8 event records per layer); out[4] = projections,
 // attention, exposed all-gather wait, all-gather on its own stream -- microseconds per layer, medians over the layers of the last call
@@ -271,13 +236,8 @@ int bitnet_host_prefill_sharded(void *d, int n, int rank, int world, bitnet_host
 int bitnet_host_rccl_allgather(void *nccl_comm, const void *send_dev, void *recv_dev, size_t bytes_per_rank, void *stream);
 void bitnet_host_layer_objects(void *d, int layer, uint64_t *handles4, void **ptrs4);
 void bitnet_host_global_objects(void *d, void **ptrs7);
-int bitnet_host_position(void *d);
-int bitnet_host_history(void *d, int32_t *out, int n);
-int bitnet_host_last_logits(void *d, float *out);
-int bitnet_host_last_hidden(void *d, float *out);
 int bitnet_host_trace_step(void *d, const char *dir, int with_logits);
 int bitnet_host_blake3_hex(const void *data, size_t len, char *out65);  // the trace records' hash (host/blake3.hpp), 64 hex digits + NUL
 int bitnet_host_probe_gateup(void *d, int reps, float *us_per_launch, double *bytes_per_launch);
 int bitnet_host_probe_kernel(void *d, int kind, int reps, float *us_per_launch, double *bytes_per_launch);
-uint64_t bitnet_host_weight_bytes(void *d);
 }

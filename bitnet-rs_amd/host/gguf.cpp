@@ -11,8 +11,10 @@
 #include <cstdlib>
 #include <cstring>
 #include <limits>
+#include <memory>
 
 #include "decoder.hpp"
+#include "registry.hpp"
 
 namespace bitnet_host {
 
@@ -699,6 +701,27 @@ int load_gguf_into(Decoder &dec, const GgufFile &g) {
     return dec.set_globals(table.data(), finv.data());
 }
 
+// A .gguf file by path: the decoder its metadata describes, filled.  f32: exact f32 activations between the kernels.
+static Sequence *open_gguf(const std::string &path, const OpenOptions &opt, std::string &err) {
+    std::unique_ptr<GgufFile> g(GgufFile::open(path.c_str(), &err));
+    GgufConfig gc;
+    if (!g || g->config(&gc, &err) != 0) return nullptr;
+    Config c;
+    c.vocab = (int)gc.vocab, c.hidden = (int)gc.hidden, c.n_layers = (int)gc.n_layers;
+    c.n_heads = (int)gc.n_heads, c.n_kv_heads = (int)(gc.n_kv_heads ? gc.n_kv_heads : gc.n_heads);
+    c.head_dim = gc.n_heads ? (int)(gc.hidden / gc.n_heads) : 0;
+    c.ffn = (int)gc.ffn, c.max_pos = opt.max_pos;
+    if (gc.has_rope_theta) c.rope_theta = gc.rope_theta;
+    if (gc.has_eps) c.eps = gc.eps;
+    std::unique_ptr<Decoder> d(new Decoder(c));
+    if (d->dead() || (opt.f32 && d->set_act_mode(0) != 0) || load_gguf_into(*d, *g) != 0) {
+        err = d->error();
+        return nullptr;
+    }
+    return d.release();
+}
+static const RegisterFileFormat kGgufFormat(".gguf", open_gguf);
+
 }  // namespace bitnet_host
 
 // ---- C shim ---------------------------------------------------------------------------------------
@@ -778,7 +801,8 @@ int bitnet_host_gguf_check_projection(void *gp, int64_t idx, uint64_t rows, uint
     return 0;
 }
 int bitnet_host_load_gguf(void *decoder, void *g) {
-    if (!decoder || !g || static_cast<Decoder *>(decoder)->dead()) return BITNET_HIP_ERR_INVALID_ARGUMENT;
-    return load_gguf_into(*static_cast<Decoder *>(decoder), *static_cast<GgufFile *>(g));
+    Decoder *dec = decoder ? dynamic_cast<Decoder *>(static_cast<Sequence *>(decoder)) : nullptr;
+    if (!dec || !g || dec->dead()) return BITNET_HIP_ERR_INVALID_ARGUMENT;
+    return load_gguf_into(*dec, *static_cast<GgufFile *>(g));
 }
 }

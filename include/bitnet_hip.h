@@ -559,6 +559,118 @@ int bitnet_hip_argmax_dev(const float *v_dev, size_t n, void *scratch_dev, size_
  * best pass in GB/s (1e9 B/s) to *best_gbs and the mean to *mean_gbs.  Allocates and frees its buffer. */
 int bitnet_hip_hbm_read_ceiling(size_t bytes, int iters, double *best_gbs, double *mean_gbs, void *stream);
 
+/* ------------------------------------------------------------------------- */
+/* 5. bf16-weight operators and sequence mixers (designs outside the reference: */
+/*    no reference interface corresponds to them)                              */
+/* ------------------------------------------------------------------------- */
+
+/* Weights: bf16 row-major [rows][ld], ld a multiple of 64, columns past the matrix zero.  Activation matrices have leading
+ * dimensions that are multiples of 64; what lies past their columns must be finite.  f32 flags: the activations / caches named
+ * are f32 and every product is an f32 multiply-add (no reduced-precision matrix mode); otherwise they are bf16 on the matrix
+ * cores with f32 accumulation.  Norms, scores, softmax weights, the residual stream and recurrent states are f32 in both. */
+#define BITNET_HIP_ACT_NONE 0
+#define BITNET_HIP_ACT_SILU 1
+#define BITNET_HIP_ACT_SIGMOID 2
+#define BITNET_HIP_ACT_RELU2 3 /* square of relu */
+
+/* out[i][width] = table[tokens[*offset + i]] as f32 (offset NULL = 0) */
+int bitnet_hip_embed_bf16_dev(const uint16_t *table_dev, size_t ld, const int32_t *tokens_dev, const int32_t *offset_dev, size_t n,
+                              size_t width, size_t vocab, float *out_dev, void *stream);
+/* x[i] += scale * norm(y[i]; post_weight) (y NULL: skipped), then h[i] = norm(x[i]; next_weight) (h NULL: skipped), padding columns of h
+ * zero; norm(v; w) = v / sqrt(mean(v^2) + eps) * (weight_offset + w). */
+int bitnet_hip_residual_norm_rows_dev(float *x_dev, const float *y_dev, size_t ldy, const float *post_weight_dev, const float *scale_dev,
+                                      const float *next_weight_dev, float weight_offset, float eps, size_t m, size_t width, void *h_dev,
+                                      size_t ldh, int h_f32, void *stream);
+/* h[i] = norm(o[i]; weight) * gate[i] over n columns; the mean divides by mean_n (padded heads hold zeros). */
+int bitnet_hip_gated_norm_rows_dev(const float *o_dev, size_t ldo, const float *weight_dev, const void *gate_dev, size_t ldg, float eps,
+                                   int gate_f32, size_t m, size_t n, size_t mean_n, void *h_dev, size_t ldh, int h_f32,
+                                   void *stream);
+/* out[i] = x[rows[i]] */
+int bitnet_hip_gather_rows_dev(const float *x_dev, const int32_t *rows_dev, size_t n, size_t width, float *out_dev, void *stream);
+/* C[m][n] = act(A[m][k] . W[n][k]^T + bias), k a multiple of 64 (<= lda, ldw); columns below act_split take act0, the others act1
+ * (act_split 0: all act0).  batch > 1: that many products, the operands *_batch elements apart. */
+int bitnet_hip_dense_matmul_dev(const void *a_dev, size_t lda, int a_f32, const uint16_t *w_dev, size_t ldw, const float *bias_dev,
+                                size_t m, size_t n, size_t k, int act0, int act1, size_t act_split, void *c_dev, size_t ldc, int c_f32,
+                                size_t batch, size_t a_batch, size_t w_batch, size_t c_batch, void *stream);
+
+/* How a matrix-vector product forms its input (every workgroup does so: no launch of its own). */
+#define BITNET_HIP_IN_PLAIN 0
+#define BITNET_HIP_IN_NORM 1          /* norm(x; weight) [* gate] */
+#define BITNET_HIP_IN_RESIDUAL_NORM 2 /* x' = x + scale * norm(y; post_weight) -> x_out (not x itself); norm(x'; weight) */
+typedef struct bitnet_hip_vector_input {
+    const float *x;
+    int32_t kind;
+    float eps, weight_offset;
+    const float *weight, *y, *post_weight, *scale, *gate; /* y NULL: nothing is added; scale, gate NULL: 1 */
+    float *x_out;                                         /* NULL: not stored */
+    int32_t n, mean_n;                                    /* elements, and what the mean divides by (0 = n) */
+} bitnet_hip_vector_input;
+/* The latent rows of a down-projection output z [m][ldz] = [q_rank | kv_rank | rot_dim]: cq[i] = norm(first q_rank; q_weight) (cq NULL:
+ * skipped), and at position p = *pos + i of the caches the latent norm(next kv_rank; kv_weight) and the last rot_dim rotated by the
+ * tables' row p (element j with element j + rot_dim / 2).  kv_rank 0: z has no key part.  Plain weights.  f32: cq and the caches. */
+typedef struct bitnet_hip_latent_rows {
+    const float *z;
+    size_t ldz;
+    int32_t q_rank, kv_rank, rot_dim;
+    const float *q_weight, *kv_weight;
+    float eps;
+    void *cq;
+    size_t ldcq;
+    void *ccache, *rcache; /* [capacity][ldc], [capacity][ldr]; ldc % 64 == 0, ldr % 32 == 0, zero-filled once */
+    size_t ldc, ldr;
+    const float *rope_cos, *rope_sin; /* [capacity][rot_dim / 2] */
+    const int32_t *pos;
+} bitnet_hip_latent_rows;
+int bitnet_hip_latent_rows_dev(const bitnet_hip_latent_rows *rows, size_t m, int f32, void *stream);
+/* y[rows] = act(W . input + bias), f32 throughout; cols a multiple of 8, <= ld, <= 38400.  batch > 1: member b uses W + b w_batch,
+ * x + b x_batch, y + b y_batch (PLAIN input only).  latent (nullable): one more workgroup writes that latent row (m = 1). */
+int bitnet_hip_dense_gemv_dev(const bitnet_hip_vector_input *input, const uint16_t *w_dev, size_t rows, size_t cols, size_t ld,
+                              const float *bias_dev, int act0, int act1, size_t act_split, float *y_dev, size_t batch, size_t w_batch,
+                              size_t x_batch, size_t y_batch, const bitnet_hip_latent_rows *latent, int latent_f32, void *stream);
+/* the same product as bitnet_hip_logits_f16_dev's tail: logits, greedy token, history and position (scratch >= 8 KiB; the token's and
+ * the position's pointers as there) */
+int bitnet_hip_dense_logits_dev(const bitnet_hip_vector_input *input, const uint16_t *w_dev, size_t vocab, size_t cols, size_t ld,
+                                float *logits_dev, void *scratch_dev, int32_t *token_dev, int32_t *pos_dev, int32_t *history_dev,
+                                const int32_t *n_forced_dev, void *stream);
+
+/* Attention over the latent cache.  Head h's query [qd = dimp + ldr]: dimp unrotated (zero-padded to a multiple of 32), then the part to
+ * rotate (rot_dim of ldr).  score = (unrotated . W_uk c + rotated . r) * scale; the softmax's denominator also holds exp(sink[h]). */
+typedef struct bitnet_hip_latent_attention {
+    size_t heads, dimp, qd, vdimp, kv_rank, rot_dim; /* vdimp % 16 == 0 */
+    float scale;
+    const float *sink; /* [heads] */
+    const void *ccache, *rcache;
+    size_t ldc, ldr, capacity;
+    const float *rope_cos, *rope_sin;
+} bitnet_hip_latent_attention;
+size_t bitnet_hip_latent_scratch_bytes(size_t heads, size_t ldc, size_t nq);
+/* nq queries at positions *pos + q0 + i, each over the keys up to its own.  q f32 [nq][heads * qd] (rotated part raw), qabs f32
+ * [nq][heads * ldc] = W_uk^T q.  Leaves records in scratch; latent_merge turns them into out [nq][ldo] = W_uv (weighted sum of c)
+ * (uv: bf16 [heads * vdimp][ldc]), f32 or bf16. */
+int bitnet_hip_latent_decode_dev(const bitnet_hip_latent_attention *attn, const float *q_dev, const float *qabs_dev, const int32_t *pos_dev,
+                                 size_t q0, size_t nq, int f32, float *scratch_dev, void *stream);
+int bitnet_hip_latent_merge_dev(const bitnet_hip_latent_attention *attn, const uint16_t *uv_dev, const int32_t *pos_dev, size_t q0,
+                                size_t nq, const float *scratch_dev, void *out_dev, size_t ldo, int out_bf16, void *stream);
+/* A portion of a prompt, bf16: the LAST nq of n_ctx positions attend.  q bf16 [nq][heads * qd], k bf16 [n_ctx][heads * dimp] = W_uk c,
+ * vt bf16 [heads * vdimp][ldvt] = (W_uv c)^T with columns up to the next multiple of 64 finite; out bf16 [nq][ldo].
+ * qd <= 256 and vdimp <= 256 (bitnet_hip_latent_prefill_supported). */
+int bitnet_hip_latent_prefill_supported(size_t qd, size_t vdimp);
+int bitnet_hip_latent_prefill_dev(const bitnet_hip_latent_attention *attn, const uint16_t *q_dev, const uint16_t *k_dev,
+                                  const uint16_t *vt_dev, size_t ldvt, size_t n_ctx, size_t nq, uint16_t *out_dev, size_t ldo, void *stream);
+
+/* Linear attention with a constant decay d per head: S_t = d S_(t-1) + k_t v_t^T, o_t = S_t^T q_t.  qkv [n][ld] =
+ * [heads * dimp | heads * dimp | heads * vdimp]; state f32 [heads][vdimp][dimp], in and out; out f32 [n][ldo];
+ * decay_pow f32 [heads][BITNET_HIP_LINEAR_BLOCK + 1] = d^i.  recurrent: qkv f32, token by token.  chunked: qkv bf16, matrix cores
+ * (dimp, vdimp multiples of 32, <= 256: bitnet_hip_linear_chunked_supported). */
+#define BITNET_HIP_LINEAR_BLOCK 128
+int bitnet_hip_linear_recurrent_dev(const float *qkv_dev, size_t ld, size_t n, size_t heads, size_t dimp, size_t vdimp,
+                                    const float *decay_pow_dev, float *state_dev, float *out_dev, size_t ldo, void *stream);
+size_t bitnet_hip_linear_workspace_bytes(size_t n, size_t heads, size_t dimp, size_t vdimp);
+int bitnet_hip_linear_chunked_supported(size_t dimp, size_t vdimp);
+int bitnet_hip_linear_chunked_dev(const uint16_t *qkv_dev, size_t ld, size_t n, size_t heads, size_t dimp, size_t vdimp,
+                                  const float *decay_pow_dev, float *state_dev, float *out_dev, size_t ldo, void *workspace_dev,
+                                  size_t workspace_bytes, void *stream);
+
 #ifdef __cplusplus
 }
 #endif

@@ -1,0 +1,146 @@
+"""Plain restatement of the mixer-stack designs (TEST INFRASTRUCTURE, float64 numpy): one function per mechanism,
+whole sequences only, no cache, no state carried between calls.  It shares no code with the product path (which has no
+Python arithmetic at all) and is written for clarity: a token at a time where that is the plainest form.
+
+    logits, layers = forward(config, tensors, tokens)
+
+config is the parsed config.json, tensors maps names to arrays.
+"""
+from __future__ import annotations
+
+import math
+
+import numpy as np
+
+F = np.float64
+
+
+# ---- norms -----------------------------------------------------------------------------------------------------------
+def rms_divide(x, eps):
+    return x / np.sqrt(np.mean(x * x, axis=-1, keepdims=True) + eps)
+
+
+def norm_plain(x, w, eps):
+    return rms_divide(x, eps) * w
+
+
+def norm_around_zero(x, w, eps):
+    return rms_divide(x, eps) * (1.0 + w)
+
+
+# ---- activations -----------------------------------------------------------------------------------------------------
+def silu(z):
+    return z / (1.0 + np.exp(-z))
+
+
+def sigmoid(z):
+    return 1.0 / (1.0 + np.exp(-z))
+
+
+def relu_squared(z):
+    return np.maximum(z, 0.0) ** 2
+
+
+# ---- rotary positions ------------------------------------------------------------------------------------------------
+def rotary_frequencies(rot):
+    """(frequency per pair, factor on cos and sin)"""
+    dims, base = rot["dims"], float(rot["base"])
+    f = np.array([base ** (-2.0 * i / dims) for i in range(dims // 2)], F)
+    s = rot.get("scaling")
+    if not s:
+        return f, 1.0
+
+    def dim_of(turns):
+        return dims * math.log(s["original"] / (2.0 * math.pi * turns)) / (2.0 * math.log(base))
+
+    lo, hi = max(math.floor(dim_of(s["fast"])), 0), min(math.ceil(dim_of(s["slow"])), dims - 1)
+    for i in range(dims // 2):
+        ramp = min(max((i - lo) / max(hi - lo, 0.001), 0.0), 1.0)
+        f[i] = f[i] / s["factor"] * ramp + f[i] * (1.0 - ramp)
+    return f, 0.1 * math.log(s["factor"]) + 1.0
+
+
+def rotate(v, positions, rot):
+    """v [tokens, ..., dims]: element i turns with element i + dims / 2"""
+    f, mult = rotary_frequencies(rot)
+    half = rot["dims"] // 2
+    out = np.array(v, F)
+    for t, p in enumerate(positions):
+        a = p * f
+        c, s = np.cos(a) * mult, np.sin(a) * mult
+        u, w = v[t][..., :half], v[t][..., half:2 * half]
+        out[t][..., :half] = u * c - w * s
+        out[t][..., half:2 * half] = w * c + u * s
+    return out
+
+
+# ---- mixers ----------------------------------------------------------------------------------------------------------
+def latent_of(h, t, p, m, eps):
+    """the pair a layer with its own down-projection leaves behind: (normed latent, rotated shared key part)"""
+    z = h @ t[p + "dkv"].T
+    c = norm_plain(z[:, :m["kv_rank"]], t[p + "dkv.norm"], eps)
+    return c, rotate(z[:, m["kv_rank"]:], range(len(h)), m["rot"])
+
+
+def latent_attention(h, t, p, m, eps, shared=None):
+    n, H, D, R, V = len(h), m["heads"], m["dim"], m["rot_dim"], m["vdim"]
+    c, kr = latent_of(h, t, p, m, eps) if shared is None else shared
+    q = norm_plain(h @ t[p + "dq"].T, t[p + "dq.norm"], eps) @ t[p + "uq"].T
+    q = q.reshape(n, H, D + R)
+    qr = rotate(q[:, :, D:], range(n), m["rot"])
+    k = (c @ t[p + "uk"].T).reshape(n, H, D)
+    v = (c @ t[p + "uv"].T).reshape(n, H, V)
+    out = np.zeros((n, H, V), F)
+    for a in range(H):
+        s = (q[:, a, :D] @ k[:, a].T + qr[:, a] @ kr.T) * m["scale"]
+        s[np.triu_indices(n, 1)] = -np.inf
+        top = np.maximum(s.max(axis=1), t[p + "sink"][a])
+        e = np.exp(s - top[:, None])
+        den = e.sum(axis=1) + np.exp(t[p + "sink"][a] - top)
+        out[:, a] = (e / den[:, None]) @ v[:, a]
+    return out.reshape(n, H * V) @ t[p + "o"].T, (c, kr)
+
+
+def lightning(h, t, p, m, eps):
+    n, H, D, V = len(h), m["heads"], m["dim"], m["vdim"]
+    q = silu(h @ t[p + "q"].T).reshape(n, H, D)
+    k = silu(h @ t[p + "k"].T).reshape(n, H, D)
+    v = silu(h @ t[p + "v"].T).reshape(n, H, V)
+    o = np.zeros((n, H, V), F)
+    for a in range(H):
+        S = np.zeros((D, V), F)
+        for i in range(n):
+            S = m["decay"][a] * S + np.outer(k[i, a], v[i, a])
+            o[i, a] = S.T @ q[i, a]
+    y = norm_plain(o.reshape(n, H * V), t[p + "norm"], eps) * sigmoid(h @ t[p + "g"].T)
+    return y @ t[p + "o"].T
+
+
+# ---- feed-forward ----------------------------------------------------------------------------------------------------
+def dense_mlp(h, t, p):
+    z = relu_squared(h @ t[p + "up"].T + t[p + "up.b"])
+    return z @ t[p + "down"].T + t[p + "down.b"]
+
+
+# ---- the stack -------------------------------------------------------------------------------------------------------
+def forward(config, tensors, tokens):
+    """(logits [n, vocab], residual stream after every layer [layers, n, width])"""
+    t = {k: np.asarray(v, F) for k, v in tensors.items()}
+    eps = config["norm"]["eps"]
+    x = t["embed"][np.asarray(tokens)]
+    after, latents = [], {}
+    for i, layer in enumerate(config["layers"]):
+        p, m = f"l{i}.", layer["mixer"]
+        h = norm_around_zero(x, t[p + "norm1"], eps)
+        if layer["type"] == "latent_attention":
+            y, latents[i] = latent_attention(h, t, p + "mix.", m, eps, latents[m["kv_from"]] if "kv_from" in m else None)
+        elif layer["type"] == "lightning":
+            y = lightning(h, t, p + "mix.", m, eps)
+        else:
+            raise ValueError(layer["type"])
+        x = x + norm_around_zero(y, t[p + "norm1b"], eps) * t[p + "ls1"]
+        if layer.get("mlp"):
+            y = dense_mlp(norm_around_zero(x, t[p + "norm2"], eps), t, p + "mlp.")
+            x = x + norm_around_zero(y, t[p + "norm2b"], eps) * t[p + "ls2"]
+        after.append(x)
+    return norm_around_zero(x, t["final.norm"], eps) @ t["head"].T, np.stack(after)

@@ -1,0 +1,159 @@
+"""Helpers of the mixer-stack tests: bf16 arrays, a safetensors writer, small random models (names, shapes and configurations of
+the designs the host library registers) and device buffers."""
+import json
+import os
+import struct
+
+import numpy as np
+
+
+def bf16_bits(a) -> np.ndarray:
+    """float32 -> bf16 bit patterns, round to nearest even"""
+    u = np.ascontiguousarray(a, np.float32).view(np.uint32)
+    return ((u + 0x7FFF + ((u >> 16) & 1)) >> 16).astype(np.uint16)
+
+
+def bf16_value(bits) -> np.ndarray:
+    return (np.asarray(bits, np.uint16).astype(np.uint32) << 16).view(np.float32)
+
+
+def rounded(a) -> np.ndarray:
+    return bf16_value(bf16_bits(a))
+
+
+def up_to(v: int, a: int) -> int:
+    return -(-v // a) * a
+
+
+def padded(a, ld: int) -> np.ndarray:
+    """last axis zero-padded to ld"""
+    a = np.asarray(a)
+    out = np.zeros(a.shape[:-1] + (ld,), a.dtype)
+    out[..., :a.shape[-1]] = a
+    return out
+
+
+def save_model(folder: str, config: dict, tensors: dict) -> str:
+    """config.json + model.safetensors (tensors: float arrays, stored as bf16)"""
+    os.makedirs(folder, exist_ok=True)
+    with open(os.path.join(folder, "config.json"), "w") as f:
+        json.dump(config, f)
+    head, at, parts = {}, 0, []
+    for name, t in tensors.items():
+        raw = bf16_bits(t).tobytes()
+        head[name] = {"dtype": "BF16", "shape": list(np.shape(t)), "data_offsets": [at, at + len(raw)]}
+        at += len(raw)
+        parts.append(raw)
+    h = json.dumps(head).encode()
+    with open(os.path.join(folder, "model.safetensors"), "wb") as f:
+        f.write(struct.pack("<Q", len(h)) + h + b"".join(parts))
+    return folder
+
+
+def latent_layer(heads=3, dim=24, rot_dim=16, vdim=40, q_rank=56, kv_rank=72, scale=0.17, base=10000.0, scaling=None, kv_from=None, ff=None) -> dict:
+    rot = {"base": base, "dims": rot_dim}
+    if scaling:
+        rot["scaling"] = scaling
+    m = {"heads": heads, "dim": dim, "rot_dim": rot_dim, "vdim": vdim, "q_rank": q_rank, "kv_rank": kv_rank, "scale": scale, "rot": rot}
+    if kv_from is not None:
+        m["kv_from"] = kv_from
+    return {"type": "latent_attention", "mixer": m, "mlp": {"kind": "dense", "ff": ff} if ff else None}
+
+
+def lightning_layer(heads=2, dim=40, vdim=24, decay=None, ff=None) -> dict:
+    decay = decay if decay is not None else [float(np.exp(-2.0 ** -(1 + 3 * h))) for h in range(heads)]
+    return {"type": "lightning", "mixer": {"heads": heads, "dim": dim, "vdim": vdim, "decay": decay}, "mlp": {"kind": "dense", "ff": ff} if ff else None}
+
+
+def lasapel(layers, width=112, vocab=150, eps=1e-5) -> dict:
+    return {"architecture": "Lasapel", "vocab": vocab, "width": width, "norm": {"eps": eps}, "layers": layers}
+
+
+def random_tensors(config: dict, seed: int) -> dict:
+    """bf16-representable weights; every norm, scale, bias and sink away from its neutral value"""
+    g = np.random.default_rng(seed)
+    W, V = config["width"], config["vocab"]
+    t = {}
+
+    def mat(name, rows, cols, gain=1.0):
+        t[name] = rounded(g.standard_normal((rows, cols)) * gain / np.sqrt(cols))
+
+    def around(name, n, centre, spread):
+        t[name] = rounded(centre + spread * g.standard_normal(n))
+
+    t["embed"] = rounded(g.standard_normal((V, W)))
+    for i, layer in enumerate(config["layers"]):
+        p, m = f"l{i}.", layer["mixer"]
+        H = m["heads"]
+        for name in ("norm1", "norm1b") + (("norm2", "norm2b") if layer["mlp"] else ()):
+            around(p + name, W, 0.0, 0.3)
+        around(p + "ls1", W, 0.7, 0.2)
+        q = p + "mix."
+        if layer["type"] == "latent_attention":
+            mat(q + "dq", m["q_rank"], W)
+            around(q + "dq.norm", m["q_rank"], 1.0, 0.3)
+            mat(q + "uq", H * (m["dim"] + m["rot_dim"]), m["q_rank"], 1.5)
+            if "kv_from" not in m:
+                mat(q + "dkv", m["kv_rank"] + m["rot_dim"], W)
+                around(q + "dkv.norm", m["kv_rank"], 1.0, 0.3)
+            mat(q + "uk", H * m["dim"], m["kv_rank"], 1.5)
+            mat(q + "uv", H * m["vdim"], m["kv_rank"])
+            around(q + "sink", H, 0.5, 1.0)
+            mat(q + "o", W, H * m["vdim"])
+        else:
+            for k, n in (("q", m["dim"]), ("k", m["dim"]), ("v", m["vdim"]), ("g", m["vdim"])):
+                mat(q + k, H * n, W)
+            around(q + "norm", H * m["vdim"], 1.0, 0.3)
+            mat(q + "o", W, H * m["vdim"])
+        if layer["mlp"]:
+            around(p + "ls2", W, 0.7, 0.2)
+            F = layer["mlp"]["ff"]
+            mat(p + "mlp.up", F, W)
+            around(p + "mlp.up.b", F, 0.1, 0.2)
+            mat(p + "mlp.down", W, F)
+            around(p + "mlp.down.b", W, 0.0, 0.2)
+    around("final.norm", W, 0.0, 0.3)
+    mat("head", V, W)
+    return t
+
+
+# ---- device buffers ----------------------------------------------------------------------------------------------------
+def dev(a, dtype=None):
+    import torch
+
+    t = torch.from_numpy(np.ascontiguousarray(a))
+    return (t if dtype is None else t.to(dtype)).cuda()
+
+
+def dev_f32(a):
+    return dev(np.asarray(a, np.float32))
+
+
+def dev_bf16(a):
+    """bf16 bit patterns on the device (as int16)"""
+    return dev(bf16_bits(a).view(np.int16))
+
+
+def zeros_f32(*shape):
+    import torch
+
+    return torch.zeros(shape, dtype=torch.float32, device="cuda")
+
+
+def zeros_bf16(*shape):
+    import torch
+
+    return torch.zeros(shape, dtype=torch.int16, device="cuda")
+
+
+def host(t) -> np.ndarray:
+    import torch
+
+    torch.cuda.synchronize()
+    a = t.cpu().numpy()
+    return bf16_value(a.view(np.uint16)) if a.dtype == np.int16 else a
+
+
+def rms_error(got, want) -> float:
+    got, want = np.asarray(got, np.float64), np.asarray(want, np.float64)
+    return float(np.sqrt(np.mean((got - want) ** 2)) / max(np.sqrt(np.mean(want ** 2)), 1e-30))

@@ -39,7 +39,7 @@ GEMMF16_QB = "_ZN10bitnet_hip11k_gemm_f16aILi0ELi4ELi2ELi5EEEvNS_8GemmArgsEj"  #
 
 def _compile(src, tmp):
     out = os.path.join(tmp, src.replace(".hip", ".s"))
-    cmd = [HIPCC, "--offload-arch=gfx950", "-O3", "-std=c++17", f"-I{ROOT}/include", f"-I{CSRC}", "-S", "--cuda-device-only",
+    cmd = [HIPCC, "--offload-arch=gfx950", "-O3", "-std=c++17", "-Xclang", "-target-feature", "-Xclang", "-packed-fp32-ops", f"-I{ROOT}/include", f"-I{CSRC}", "-S", "--cuda-device-only",
            "-Rpass-analysis=kernel-resource-usage", os.path.join(CSRC, src), "-o", out]
     p = subprocess.run(cmd, capture_output=True, text=True, timeout=900)
     assert p.returncode == 0, p.stderr[-2000:]
