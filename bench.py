@@ -620,12 +620,60 @@ def bench_sharded_prefill(args, pkg, synth, dist_, r, hip, cfg, dec):
     dist_.finalize(r)
 
 
+def timed_model(model, prompt, steps: int, warmup: int, digits: int = 2) -> dict:
+    """Prompt portion (second of two passes) and `steps` greedy single-token steps behind it, of any model of the library."""
+    n = len(prompt)
+    for _ in range(2):
+        model.reset()
+        model.feed(prompt)
+        prefill_ms = model.prefill(n, with_logits=True, digits=digits)
+    model.prepare_graphs(True)
+    model.run(warmup)
+    ms = model.run(steps)
+    return {"prompt": n, "prefill_ms": round(prefill_ms, 3), "prefill_tok_s": round(n / prefill_ms * 1e3, 1), "decode_keys": [n + warmup + 1, n + warmup + steps],
+            "decode_ms_per_token": round(ms / steps, 4), "decode_tok_s": round(steps / ms * 1e3, 1)}
+
+
+def bench_stack(args, pkg, synth):
+    """--workload lasapel: prompt and decode throughput of the Lasapel design at sizes that resemble a real model's layers, beside the
+    library's BitNet model (QK256) with the same width, feed-forward, heads, vocabulary and number of layers."""
+    import tempfile
+
+    rows = []
+    max_pos = 4096 + 64 + args.steps + args.warmup
+    for size in args.sizes.split(","):
+        s = synth.STACK_SIZES[size]
+        row = {"size": size, "layers": args.layers or 8, **{k: s[k] for k in ("width", "ff", "heads", "vocab")}}
+        with tempfile.TemporaryDirectory() as tmp:
+            model = pkg.open_model(synth.write_lasapel(tmp, synth.lasapel_config(size, row["layers"])), "bfloat16", max_pos)
+            row["lasapel"] = [timed_model(model, synth.prompt(n, s["vocab"], 1), args.steps, args.warmup) for n in (128, 4096)]
+            row["lasapel_weight_bytes"] = model.weight_bytes()
+            model.close()
+        if not args.no_also:
+            cfg = synth.ModelConfig(hidden=s["width"], n_layers=row["layers"], n_heads=s["heads"], n_kv_heads=s["n_kv"], ffn=s["ff"], vocab=s["vocab"], max_pos=max_pos)
+            dec = pkg.HostDecoder(cfg)
+            layer = synth.make_layer(cfg, 0, fmt="qk256")
+            for l in range(cfg.n_layers):
+                dec.set_layer_qk256(l, layer)
+            dec.set_globals(synth.make_globals(cfg))
+            row["bitnet_qk256"] = [timed_model(dec, synth.prompt(n, s["vocab"], 1), args.steps, args.warmup) for n in (128, 4096)]
+            row["bitnet_weight_bytes"] = dec.weight_bytes() + 2 * cfg.vocab * cfg.hidden
+            dec.close()
+        rows.append(row)
+        print(f"{size} done", file=sys.stderr, flush=True)
+    first = rows[0]["lasapel"][0]
+    return {"metric": "Lasapel decode tokens/s (128-token prompt)", "value": first["decode_tok_s"], "unit": "tokens/s", "n_gpus": 1, "steps": args.steps,
+            "warmup": args.warmup, "ms_per_step": first["decode_ms_per_token"], "higher_is_better": True, "scaling": "weak", "vs_baseline": None, "dtype": "bf16",
+            "data": "synthetic", "config": {"model": f"Lasapel {rows[0]['size']}", "layers": rows[0]["layers"], "sizes": args.sizes}, "sizes": rows}
+
+
 def main():
     ap = argparse.ArgumentParser()
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=None, help="timed steps (default 256; 512 for --workload c4: BASELINE configs[3] = 4k-token prefill + 512 decode)")
     ap.add_argument("--warmup", type=int, default=16)
-    ap.add_argument("--workload", default="c2", choices=["c2", "c3", "c4", "c5", "stream"])
+    ap.add_argument("--workload", default="c2", choices=["c2", "c3", "c4", "c5", "stream", "lasapel"])
+    ap.add_argument("--sizes", default="2b,1b,5b", help="lasapel workload: which of the model sizes (synth.STACK_SIZES)")
     ap.add_argument("--stream-layers", type=int, default=64, help="i2s_stream: gate|up matrices laid end to end (64 = 708 MB BitNet32-F16 / 566 MB QK256)")
     ap.add_argument("--stream-launches", type=int, default=None, help="stream workload only: a fixed number of launches and no timing (profiler counter passes)")
     ap.add_argument("--stream-format", default="i2s", choices=["i2s", "qk256"])
@@ -684,6 +732,12 @@ def main():
     hip = pkg.load()
     hip.init(local_rank)
 
+    if args.workload == "lasapel":
+        line = bench_stack(args, pkg, synth)
+        if rank == 0:
+            print(json.dumps(line), flush=True)
+        dist_.finalize(r)
+        return
     global PROMPT_LEN
     PROMPT_LEN = args.prompt or {"c4": 4096, "c5": 8192}.get(args.workload, 128)
     if args.workload == "stream":  # the streaming-rate probe alone (tools/profile_round.sh runs its counter passes through this)

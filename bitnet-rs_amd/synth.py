@@ -13,6 +13,10 @@ from __future__ import annotations
 
 from dataclasses import dataclass, asdict
 
+import json
+import os
+import struct
+
 import numpy as np
 
 BITNET_2B_4T = dict(hidden=2560, n_layers=30, n_heads=20, n_kv_heads=5, head_dim=128, ffn=6912, vocab=128256, max_pos=4096, eps=1e-5, rope_theta=10000.0)
@@ -103,3 +107,73 @@ def prompt(n: int, vocab: int, bos: int = 128000) -> np.ndarray:
     ids = (1000 + 37 * np.arange(n)) % vocab
     ids[0] = bos % vocab
     return ids.astype(np.int32)
+
+
+# ---- random models of the mixer-stack designs, at sizes that resemble a real model's layers -------------------------
+STACK_SIZES = {  # width, ff, heads, kv heads of the BitNet model of equal size, q_rank, vocab
+    "1b": dict(width=1536, ff=4096, heads=12, n_kv=3, q_rank=768, vocab=32768),
+    "2b": dict(width=2560, ff=6912, heads=20, n_kv=5, q_rank=1536, vocab=128256),
+    "5b": dict(width=4096, ff=8192, heads=32, n_kv=8, q_rank=1536, vocab=32768),
+}
+
+
+def lasapel_config(size: str, n_layers: int) -> dict:
+    """latent attention (heads of 128 + 64 rotated / 128, latent 512) and linear attention (heads of 128 / 128) in turn, every layer
+    with a feed-forward; the fifth layer reads the first one's cache."""
+    s = STACK_SIZES[size]
+    layers = []
+    for i in range(n_layers):
+        if i % 2 == 0:
+            m = {"heads": s["heads"], "dim": 128, "rot_dim": 64, "vdim": 128, "q_rank": s["q_rank"], "kv_rank": 512, "scale": 0.0722,
+                 "rot": {"base": 500000.0, "dims": 64, "scaling": {"factor": 8.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}
+            if i == 4:
+                m["kv_from"] = 0
+            layers.append({"type": "latent_attention", "mixer": m, "mlp": {"kind": "dense", "ff": s["ff"]}})
+        else:
+            decay = [float(np.exp(-(2.0 ** (-8.0 * (h + 1) / s["heads"])))) for h in range(s["heads"])]
+            layers.append({"type": "lightning", "mixer": {"heads": s["heads"], "dim": 128, "vdim": 128, "decay": decay}, "mlp": {"kind": "dense", "ff": s["ff"]}})
+    return {"architecture": "Lasapel", "vocab": s["vocab"], "width": s["width"], "norm": {"eps": 1e-6}, "layers": layers}
+
+
+def write_lasapel(folder: str, config: dict, seed: int = 42) -> str:
+    """config.json + model.safetensors with random bf16 weights (slices of one random block, scaled per tensor)."""
+    block = _stream(seed, 7).standard_normal(1 << 22, dtype=np.float32)
+    shapes = {"embed": (config["vocab"], config["width"]), "head": (config["vocab"], config["width"]), "final.norm": (config["width"],)}
+    W = config["width"]
+    for i, layer in enumerate(config["layers"]):
+        p, m = f"l{i}.", layer["mixer"]
+        q, H = p + "mix.", m["heads"]
+        shapes.update({p + n: (W,) for n in ("norm1", "norm1b", "norm2", "norm2b", "ls1", "ls2")})
+        if layer["type"] == "latent_attention":
+            shapes.update({q + "dq": (m["q_rank"], W), q + "dq.norm": (m["q_rank"],), q + "uq": (H * (m["dim"] + m["rot_dim"]), m["q_rank"]),
+                           q + "uk": (H * m["dim"], m["kv_rank"]), q + "uv": (H * m["vdim"], m["kv_rank"]), q + "sink": (H,), q + "o": (W, H * m["vdim"])})
+            if "kv_from" not in m:
+                shapes.update({q + "dkv": (m["kv_rank"] + m["rot_dim"], W), q + "dkv.norm": (m["kv_rank"],)})
+        else:
+            shapes.update({q + n: (H * d, W) for n, d in (("q", m["dim"]), ("k", m["dim"]), ("v", m["vdim"]), ("g", m["vdim"]))})
+            shapes.update({q + "norm": (H * m["vdim"],), q + "o": (W, H * m["vdim"])})
+        f = layer["mlp"]["ff"]
+        shapes.update({p + "mlp.up": (f, W), p + "mlp.up.b": (f,), p + "mlp.down": (W, f), p + "mlp.down.b": (W,)})
+    os.makedirs(folder, exist_ok=True)
+    with open(os.path.join(folder, "config.json"), "w") as fh:
+        json.dump(config, fh)
+    head, at = {}, 0
+    for name, shape in shapes.items():
+        n = 2 * int(np.prod(shape))
+        head[name] = {"dtype": "BF16", "shape": list(shape), "data_offsets": [at, at + n]}
+        at += n
+    h = json.dumps(head).encode()
+    with open(os.path.join(folder, "model.safetensors"), "wb") as fh:
+        fh.write(struct.pack("<Q", len(h)) + h)
+        for k, (name, shape) in enumerate(shapes.items()):
+            n = int(np.prod(shape))
+            if len(shape) == 2:
+                gain, centre = (1.0 if name == "embed" else 1.0 / np.sqrt(shape[1])), 0.0
+            else:
+                gain, centre = 0.1, (1.0 if name.endswith("q.norm") or name.endswith("v.norm") or name.endswith("mix.norm") else 0.5 if ".ls" in name else 0.0)
+            bits = ((block * np.float32(gain) + np.float32(centre)).view(np.uint32) >> 16).astype(np.uint16)
+            start = (k * 9973) % block.size
+            bits = np.roll(bits, -start)
+            for a in range(0, n, block.size):
+                fh.write(bits[: min(block.size, n - a)].tobytes())
+    return folder

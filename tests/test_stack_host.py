@@ -1,0 +1,164 @@
+"""Host side of the mixer-stack models without a GPU: registry, configuration and tensor checks, and known values of the plain
+restatement the GPU tests compare with."""
+import copy
+import math
+import os
+import struct
+
+import numpy as np
+import pytest
+
+from oracle import stack_oracle as so
+from tests import stack_util as u
+
+
+@pytest.fixture(scope="module")
+def built(pkg):
+    pkg.build()
+    return pkg
+
+
+BASE = u.lasapel([u.latent_layer(ff=24), u.lightning_layer()], width=40, vocab=20)
+
+
+def test_registry_names(built):
+    names = built.registered_models()
+    assert "Lasapel" in names and ".gguf" in names
+
+
+def broken(change):
+    c = copy.deepcopy(BASE)
+    change(c)
+    return c
+
+
+@pytest.mark.parametrize("change,message", [
+    (lambda c: c.pop("width"), "width: missing"),
+    (lambda c: c.update(width=0), "width: not an integer"),
+    (lambda c: c.update(layers=[]), "layers: missing"),
+    (lambda c: c["norm"].pop("eps"), "norm.eps: missing"),
+    (lambda c: c["layers"][0].update(type="other"), r"layers\[0\].type: unknown mixer"),
+    (lambda c: c["layers"][0]["mixer"].pop("kv_rank"), r"layers\[0\].mixer.kv_rank: missing"),
+    (lambda c: c["layers"][0]["mixer"]["rot"].pop("base"), r"layers\[0\].mixer.rot.base: missing"),
+    (lambda c: c["layers"][0]["mlp"].update(kind="sparse"), r"layers\[0\].mlp.kind: unknown"),
+    (lambda c: c["layers"][1]["mixer"].update(decay=["a"]), r"layers\[1\].mixer.decay: not an array of numbers"),
+    (lambda c: c.update(architecture="Nothing"), "'Nothing' is not registered"),
+])
+def test_bad_configurations_say_why(built, tmp_path, change, message):
+    path = u.save_model(str(tmp_path), broken(change), u.random_tensors(BASE, 1))
+    with pytest.raises(built.BitNetHipError, match=message):
+        built.open_model(path)
+
+
+def test_bad_files_say_why(built, tmp_path):
+    with pytest.raises(built.BitNetHipError, match="neither a known file format"):
+        built.open_model(str(tmp_path / "nothing"))
+    path = u.save_model(str(tmp_path / "m"), BASE, u.random_tensors(BASE, 1))
+    with open(os.path.join(path, "config.json"), "w") as f:
+        f.write('{"architecture": ')
+    with pytest.raises(built.BitNetHipError, match="JSON"):
+        built.open_model(path)
+    path = u.save_model(str(tmp_path / "n"), BASE, u.random_tensors(BASE, 1))
+    st = os.path.join(path, "model.safetensors")
+    data = open(st, "rb").read()
+    for raw, message in ((data[:4], "cannot be read"), (struct.pack("<Q", 1 << 40) + data[8:], "header longer"), (data[:-2], "bad byte range")):
+        open(st, "wb").write(raw)
+        with pytest.raises(built.BitNetHipError, match=message):
+            built.open_model(path)
+
+
+def test_no_gpu_is_an_error(built, tmp_path):
+    import torch
+
+    if torch.cuda.is_available():
+        pytest.skip("GPU present")
+    with pytest.raises(built.BitNetHipError, match="no HIP device"):
+        built.open_model(u.save_model(str(tmp_path), BASE, u.random_tensors(BASE, 1)))
+
+
+def test_entry_points_check_shapes_before_any_launch(built):
+    hip = built.load()
+    bad = [
+        (lambda: hip.dense_matmul_dev(8, 96, False, 8, 96, 4, 4, 96, 8, 4, True), "multiple of 64"),
+        (lambda: hip.dense_matmul_dev(8, 64, False, 8, 64, 4, 8, 64, 8, 4, True), "dense_matmul"),
+        (lambda: hip.dense_gemv_dev(8, 8, 4, 12, 64, 8), "bad shape"),
+        (lambda: hip.dense_gemv_dev(8, 8, 4, 64, 64, 8, kind=built.IN_RESIDUAL_NORM, weight=8, res=8, post_weight=8, x_out=8, n=64), "buffer of its own"),
+        (lambda: hip.linear_recurrent_dev(8, 96, 1, 1, 32, 24, 8, 8, 8, 32), "bad shape"),
+        (lambda: hip.linear_chunked_dev(8, 96, 1, 1, 32, 32, 8, 8, 8, 32, 8, 16), "workspace"),
+        (lambda: hip.latent_decode_dev(built.LatentAttention(1, 20, 52, 16, 64, 16, 1.0, 8, 8, 8, 64, 32, 64, 8, 8), 8, 8, 8, 0, 1, True, 8), "bad shape"),
+    ]
+    for call, message in bad:
+        with pytest.raises(built.BitNetHipError, match=message):
+            call()
+
+
+# ---- the oracle itself -------------------------------------------------------------------------------------------------
+def test_oracle_rotation_and_yarn():
+    f, mult = so.rotary_frequencies({"dims": 8, "base": 10000.0})
+    assert mult == 1.0 and np.allclose(f, [1, 0.1, 0.01, 0.001])
+    x = np.arange(8.0)[None]
+    y = so.rotate(x, [3], {"dims": 8, "base": 10000.0})[0]
+    assert np.isclose(y[1], 1 * math.cos(0.3) - 5 * math.sin(0.3)) and np.isclose(y[5], 5 * math.cos(0.3) + 1 * math.sin(0.3))
+    s = {"factor": 4.0, "original": 64, "fast": 8.0, "slow": 1.0}
+    f2, mult = so.rotary_frequencies({"dims": 16, "base": 100.0, "scaling": s})
+    f1, _ = so.rotary_frequencies({"dims": 16, "base": 100.0})
+    assert np.isclose(mult, 0.1 * math.log(4) + 1)
+    # lo = floor(16 ln(64 / 16 pi) / (2 ln 100)) = 0, hi = ceil(16 ln(64 / 2 pi) / (2 ln 100)) = 5
+    for i in range(8):
+        ramp = min(i / 5, 1.0)
+        assert np.isclose(f2[i], f1[i] * (1 - ramp) + f1[i] / 4 * ramp)
+
+
+def test_oracle_linear_attention_by_powers():
+    """the recurrence against the sum over all earlier tokens with explicit powers of the decay"""
+    g = np.random.default_rng(0)
+    m, W, n = {"heads": 2, "dim": 3, "vdim": 4, "decay": [0.7, 1.0]}, 6, 5
+    t = {k: g.standard_normal((2 * (3 if k in "qk" else 4), W)) for k in "qkvg"}
+    t.update(o=np.eye(8), norm=np.ones(8))
+    h = g.standard_normal((n, W))
+    got = so.lightning(h, t, "", m, 1e-6)
+    q, k, v = (so.silu(h @ t[x].T).reshape(n, 2, -1) for x in "qkv")
+    o = np.zeros((n, 2, 4))
+    for i in range(n):
+        for j in range(i + 1):
+            for a in range(2):
+                o[i, a] += m["decay"][a] ** (i - j) * (q[i, a] @ k[j, a]) * v[j, a]
+    assert np.allclose(got, so.norm_plain(o.reshape(n, 8), 1.0, 1e-6) * so.sigmoid(h @ t["g"].T))
+
+
+def test_oracle_sink_takes_a_share():
+    """one token: the weight of its only key is exp(s) / (exp(s) + exp(sink))"""
+    config = u.lasapel([u.latent_layer(heads=1, dim=4, rot_dim=2, vdim=4, q_rank=4, kv_rank=4)], width=8, vocab=5)
+    t = {k: np.asarray(v, np.float64) for k, v in u.random_tensors(config, 3).items()}
+    h, m, p = np.random.default_rng(1).standard_normal((1, 8)), config["layers"][0]["mixer"], "l0.mix."
+    t[p + "o"] = np.eye(8, 4)
+    outs = {}
+    for sink in (-50.0, 0.3):
+        t[p + "sink"] = np.array([sink])
+        outs[sink], (c, kr) = so.latent_attention(h, t, p, m, 1e-6)
+    q = so.norm_plain(h @ t[p + "dq"].T, t[p + "dq.norm"], 1e-6) @ t[p + "uq"].T
+    s = (q[0, :4] @ (t[p + "uk"] @ c[0]) + q[0, 4:] @ kr[0]) * m["scale"]
+    assert np.allclose(outs[0.3], outs[-50.0] * np.exp(s) / (np.exp(s) + np.exp(0.3)))
+
+
+def test_trace_runner_refuses_bad_use(built):
+    import subprocess
+
+    build = built._load_build_module()
+    prog = build.build_program("trace_run")
+    for args in ([], ["--model", "x", "--dtype", "float16", "--out", "y", "--max-tokens", "5"], ["--nonsense", "1"]):
+        p = subprocess.run([prog, *args], capture_output=True, text=True, stdin=subprocess.DEVNULL, timeout=60)
+        assert p.returncode == 1 and "trace_run" in p.stderr
+
+
+def test_command_line_arguments(built, capsys):
+    import importlib
+
+    cli = importlib.import_module("bitnet-rs_amd.cli")
+    a = cli.parse(["--model", "m", "--tokens", "3,1,4", "--new", "5"])
+    assert a.tokens == [3, 1, 4] and a.max_pos == 10 and a.dtype == "bfloat16"
+    for bad in (["--model", "m", "--tokens", "x"], ["--model", "m", "--tokens", "1", "--new", "0"], ["--tokens", "1"]):
+        with pytest.raises(SystemExit):
+            cli.parse(bad)
+    assert cli.main(["--model", "/nothing", "--tokens", "1"]) == 1
+    assert "neither a known file format" in capsys.readouterr().err

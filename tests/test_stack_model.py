@@ -1,0 +1,285 @@
+"""Whole mixer-stack models through the framework's own entry points (open by path, prompt portions, captured single-token steps,
+greedy generation), against oracle/stack_oracle.py on small random models."""
+import numpy as np
+import pytest
+
+from oracle import stack_oracle as so
+from tests import stack_util as u
+
+pytestmark = pytest.mark.gpu
+
+YARN = {"factor": 6.0, "original": 48, "fast": 8.0, "slow": 1.0}
+# small models that differ in everything a configuration can say; none of the sizes is a multiple the kernels would like
+MODELS = {
+    "latent_only": u.lasapel([u.latent_layer(ff=70)], width=96, vocab=130),
+    "latent_without_ff": u.lasapel([u.latent_layer(heads=1, dim=8, rot_dim=2, vdim=8, q_rank=8, kv_rank=8, base=50.0)], width=40, vocab=33, eps=1e-3),
+    "lightning_only": u.lasapel([u.lightning_layer()], width=72, vocab=90),
+    "lightning_with_ff": u.lasapel([u.lightning_layer(heads=3, dim=24, vdim=72, decay=[1.0, 0.5, 0.0], ff=88)], width=136, vocab=101),
+    "mixed": u.lasapel([u.lightning_layer(heads=5, dim=16, vdim=16, ff=48), u.latent_layer(heads=5, scaling=YARN, ff=200), u.lightning_layer(),
+                        u.latent_layer(heads=2, dim=48, vdim=24, q_rank=24, kv_from=1, scaling=YARN), u.latent_layer(kv_rank=24, scale=0.3, ff=64)],
+                       width=152, vocab=190),
+    "wide_heads": u.lasapel([u.latent_layer(heads=2, dim=100, rot_dim=60, vdim=140, q_rank=120, kv_rank=200, scaling=dict(YARN, factor=1.5, slow=2.0), ff=33),
+                             u.lightning_layer(heads=1, dim=200, vdim=136)], width=200, vocab=64),
+    "huge_heads": u.lasapel([u.latent_layer(heads=1, dim=230, rot_dim=40, vdim=270, q_rank=40, kv_rank=600), u.lightning_layer(heads=1, dim=290, vdim=48)],
+                            width=88, vocab=70),
+    "many_heads": u.lasapel([u.latent_layer(heads=19, dim=16, rot_dim=8, vdim=16, q_rank=40, kv_rank=136, ff=16)], width=64, vocab=500),
+}
+LIMIT = {"float32": 2e-5, "bfloat16": 6e-2}
+
+
+class Case:
+    def __init__(self, pkg, root, name):
+        self.config = MODELS[name]
+        self.tensors = u.random_tensors(self.config, sum(map(ord, name)))
+        self.path = u.save_model(str(root / name), self.config, self.tensors)
+        self.pkg, self.models, self.truth = pkg, {}, {}
+
+    def model(self, dtype, max_pos=400):
+        if dtype not in self.models:
+            self.models[dtype] = self.pkg.open_model(self.path, dtype, max_pos)
+        m = self.models[dtype]
+        m.reset()
+        return m
+
+    def oracle(self, tokens):
+        key = bytes(np.asarray(tokens, np.int32))
+        if key not in self.truth:
+            self.truth[key] = so.forward(self.config, self.tensors, tokens)
+        return self.truth[key]
+
+
+@pytest.fixture(scope="module")
+def cases(pkg, hip, tmp_path_factory):
+    root, made = tmp_path_factory.mktemp("stack"), {}
+
+    def get(name):
+        if name not in made:
+            made[name] = Case(pkg, root, name)
+        return made[name]
+
+    yield get
+    for c in made.values():
+        for m in c.models.values():
+            m.close()
+
+
+def tokens_of(config, n, seed=0):
+    return np.random.default_rng([n, seed]).integers(0, config["vocab"], n).astype(np.int32)
+
+
+def error(got, want) -> float:
+    """per position: rms of the difference (means taken off) over the rms of all logits; the worst"""
+    d = np.asarray(got, np.float64) - want
+    d -= d.mean(axis=1, keepdims=True)
+    w = want - want.mean(axis=1, keepdims=True)
+    return float(np.sqrt((d ** 2).mean(axis=1)).max() / np.sqrt((w ** 2).mean()))
+
+
+def in_portions(m, tokens, sizes):
+    out, at, i = [], 0, 0
+    while at < len(tokens):
+        n = min(sizes[i % len(sizes)], len(tokens) - at)
+        out.append(m.forward(tokens[at:at + n], range(n)))
+        at, i = at + n, i + 1
+    return np.concatenate(out)
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("name", list(MODELS))
+def test_prompt_and_decoding(cases, name, dtype):
+    """the whole prompt at once, and token by token through the cache: every position"""
+    c = cases(name)
+    t = tokens_of(c.config, 75)
+    want = c.oracle(t)[0]
+    assert error(c.model(dtype).forward(t, range(len(t))), want) < LIMIT[dtype]
+    assert error(in_portions(c.model(dtype), t, [1]), want) < LIMIT[dtype]
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("sizes", [[2], [3, 1, 2], [64, 1], [63, 2, 65], [127, 2, 1, 130], [129], [40, 100, 2, 1, 1]])
+def test_portions(cases, dtype, sizes):
+    c = cases("mixed")
+    t = tokens_of(c.config, 290)
+    want = c.oracle(t)[0]
+    assert error(in_portions(c.model(dtype), t, sizes), want) < LIMIT[dtype]
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_first_tokens(cases, dtype):
+    """sequences of one, two and three tokens: the sink weighs most there, states are empty"""
+    c = cases("mixed")
+    for n in (1, 2, 3):
+        t = tokens_of(c.config, n, 5)
+        want = c.oracle(t)[0]
+        assert error(c.model(dtype).forward(t, range(n)), want) < LIMIT[dtype]
+        assert error(in_portions(c.model(dtype), t, [1]), want) < LIMIT[dtype]
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_residual_stream_after_each_layer(cases, pkg, tmp_path, dtype):
+    """the model cut after each of its layers: the stream ahead of the final norm, from the prompt and from a step"""
+    c = cases("mixed")
+    t = tokens_of(c.config, 21)
+    after = c.oracle(t)[1]
+    for k in range(1, len(c.config["layers"]) + 1):
+        config = dict(c.config, layers=c.config["layers"][:k])
+        m = pkg.open_model(u.save_model(str(tmp_path / str(k)), config, c.tensors), dtype, 64)
+        m.feed(t)
+        m.prefill(20, with_logits=False)
+        assert u.rms_error(m.last_hidden(), after[k - 1, 19]) < LIMIT[dtype]
+        m.run(1)
+        assert u.rms_error(m.last_hidden(), after[k - 1, 20]) < LIMIT[dtype]
+        m.close()
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_long_decoding(cases, dtype):
+    """300 steps behind a short prompt: several cache tiles, states carried all the way"""
+    c = cases("mixed")
+    t = tokens_of(c.config, 310, 3)
+    want = c.oracle(t)[0]
+    m = c.model(dtype)
+    got = [m.forward(t[:10], range(10))] + [m.forward(t[i:i + 1], [0]) for i in range(10, 310)]
+    assert error(np.concatenate(got), want) < LIMIT[dtype]
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_requests_follow_one_another(cases, dtype):
+    """a slot used again: nothing of the longer sequence before shows in the next one, and a repeat is bit for bit the same"""
+    c = cases("mixed")
+    long, short = tokens_of(c.config, 200, 1), tokens_of(c.config, 30, 2)
+    m = c.model(dtype)
+    first = m.forward(short, range(30))
+    for before in (long, long[:65]):
+        m.reset()
+        m.forward(before, [])
+        m.forward(before[:1], [0])
+        m.reset()
+        assert np.array_equal(m.forward(short, range(30)), first)
+    assert error(first, c.oracle(short)[0]) < LIMIT[dtype]
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_graph_replays_match_eager_steps(cases, dtype):
+    c = cases("mixed")
+    t = tokens_of(c.config, 40, 4)
+    out = []
+    for use_graph in (True, False):
+        m = c.model(dtype)
+        m.feed(t)
+        m.prefill(20, with_logits=False)
+        rows = []
+        for _ in range(20):
+            m.run(1, use_graph=use_graph)
+            rows.append(m.last_logits())
+        out.append(np.stack(rows))
+    assert np.array_equal(out[0], out[1])
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("name", ["mixed", "lightning_only", "many_heads"])
+def test_greedy_generation(cases, name, dtype):
+    """generate(): each token is the argmax of the oracle's logits over what was generated so far (or as good as it)"""
+    c = cases(name)
+    p = tokens_of(c.config, 12, 6)
+    m = c.model(dtype)
+    new = m.generate(p, 16)
+    want = c.oracle(np.concatenate([p, new]))[0]
+    spread = np.sqrt(((want - want.mean(axis=1, keepdims=True)) ** 2).mean())
+    for i, tok in enumerate(new):
+        row = want[len(p) - 1 + i]
+        assert row.max() - row[tok] <= 2 * LIMIT[dtype] * spread, (i, tok)
+    assert np.array_equal(m.generate(p, 16, use_graph=False), new)
+    if dtype == "float32":
+        assert sum(want[len(p) - 1 + i].argmax() == tok for i, tok in enumerate(new)) >= 15
+
+
+def one_key_model(cases_root, pkg, far):
+    """One latent layer in which the query of a marked token scores one other marked token far above all others: the value it
+    carries must come through however far back it lies."""
+    W, V = 32, 40
+    layer = u.latent_layer(heads=1, dim=8, rot_dim=2, vdim=8, q_rank=8, kv_rank=8, scale=1.0, base=1e6)
+    config = u.lasapel([layer], width=W, vocab=V, eps=1e-6)
+    t = u.random_tensors(config, 11)
+    t["embed"] = u.rounded(np.random.default_rng(8).standard_normal((V, W)) * 0.05)
+    t["embed"][:, 0] = 1.0   # every token
+    t["embed"][1, 1] = 6.0   # the token looked for
+    t["embed"][2, 2] = 6.0   # the token that looks
+    for k in ("dq", "dkv", "uq", "uk"):
+        t["l0.mix." + k] *= 0.02
+    t["l0.mix.dq"][0, 2] = t["l0.mix.dkv"][0, 1] = 1.0
+    t["l0.mix.dq"][1, 0] = t["l0.mix.dkv"][1, 0] = 0.5
+    t["l0.mix.dq.norm"][:], t["l0.mix.dkv.norm"][:] = 1.0, 1.0
+    t["l0.norm1"][:] = 0.0
+    t["l0.mix.uq"][0, 0], t["l0.mix.uk"][0, 0] = 3.0, 3.0
+    t = {k: u.rounded(v) for k, v in t.items()}
+    return config, t, u.save_model(str(cases_root / f"far{far}"), config, t)
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("far", [0, 1, 62, 63, 64, 127, 128, 300, 398])
+def test_one_far_key(pkg, hip, tmp_path, dtype, far):
+    """with and without the looked-for token: the last position's logits differ as the oracle's do, in a prompt and decoded"""
+    config, t, path = one_key_model(tmp_path, pkg, far)
+    n = 400
+    base = np.random.default_rng(far).integers(3, 40, n).astype(np.int32)
+    base[-1] = 2
+    marked = base.copy()
+    marked[far] = 1
+    m = pkg.open_model(path, dtype, n + 8)
+    for tokens in (base, marked):
+        want = so.forward(config, t, tokens)[0][-1:]
+        m.reset()
+        assert error(m.forward(tokens, [n - 1]), want) < LIMIT[dtype]
+        m.reset()
+        m.forward(tokens[:-1], [])
+        assert error(m.forward(tokens[-1:], [0]), want) < LIMIT[dtype]
+    a, b = so.forward(config, t, base)[0][-1], so.forward(config, t, marked)[0][-1]
+    assert u.rms_error(a - a.mean(), b - b.mean()) > 0.2  # the key shows
+    m.close()
+
+
+def test_errors_leave_a_usable_model(cases, pkg):
+    c = cases("lightning_only")
+    m = c.model("bfloat16")
+    with pytest.raises(pkg.BitNetHipError, match="out of range"):
+        m.forward([c.config["vocab"]], [0])
+    with pytest.raises(pkg.BitNetHipError, match="wanted place"):
+        m.forward([1, 2], [2])
+    with pytest.raises(pkg.BitNetHipError, match="overflow"):
+        m.forward(np.zeros(401, np.int32), [])
+    m.reset()
+    t = tokens_of(c.config, 9)
+    assert error(m.forward(t, range(9)), c.oracle(t)[0]) < LIMIT["bfloat16"]
+
+
+def test_command_line_generates(cases, capsys):
+    import importlib
+
+    cli = importlib.import_module("bitnet-rs_amd.cli")
+    c = cases("mixed")
+    p = tokens_of(c.config, 9, 7)
+    assert cli.main(["--model", c.path, "--tokens", ",".join(map(str, p)), "--new", "6"]) == 0
+    assert capsys.readouterr().out.strip() == ",".join(map(str, c.model("bfloat16").generate(p, 6)))
+
+
+def test_trace_runner_matches_the_library(cases, pkg, tmp_path):
+    """the program's logits are those of the same portions through the library, bit for bit"""
+    import json
+    import subprocess
+
+    c = cases("mixed")
+    prog = pkg._load_build_module().build_program("trace_run")
+    a, b = tokens_of(c.config, 20, 8), tokens_of(c.config, 7, 9)
+    steps = [("a", a[:12], [0, 11], []), ("a", a[12:13], [], []), ("a", a[13:], [6, 1], ["a"]), ("b", b, [6], ["b"])]
+    text = "".join(json.dumps({"step": i, "entries": [{"id": n, "tokens": t.tolist(), "want": w}], "end": e}) + "\n" for i, (n, t, w, e) in enumerate(steps))
+    p = subprocess.run([prog, "--model", c.path, "--dtype", "float32", "--out", str(tmp_path), "--max-tokens", "64"], input=text, capture_output=True, text=True, timeout=60)
+    assert p.returncode == 0 and p.stdout.split("\n")[:4] == [f"done {i}" for i in range(4)], p.stderr
+    m = c.model("float32")
+    for i, (name, t, w, _) in enumerate(steps):
+        if name == "b":
+            m.reset()
+        want = m.forward(t, w)
+        if w:
+            assert np.array_equal(np.fromfile(str(tmp_path / f"{i}.f32"), np.float32).reshape(want.shape), want)
+    assert not (tmp_path / "1.f32").exists()
