@@ -673,7 +673,7 @@ def main():
     ap.add_argument("--steps", type=int, default=None, help="timed steps (default 256; 512 for --workload c4: BASELINE configs[3] = 4k-token prefill + 512 decode)")
     ap.add_argument("--warmup", type=int, default=16)
     ap.add_argument("--workload", default="c2", choices=["c2", "c3", "c4", "c5", "stream", "lasapel"])
-    ap.add_argument("--sizes", default="2b,1b,5b", help="lasapel workload: which of the model sizes (synth.STACK_SIZES)")
+    ap.add_argument("--sizes", default="2b,1b,3b", help="lasapel workload: which of the model sizes (synth.STACK_SIZES)")
     ap.add_argument("--stream-layers", type=int, default=64, help="i2s_stream: gate|up matrices laid end to end (64 = 708 MB BitNet32-F16 / 566 MB QK256)")
     ap.add_argument("--stream-launches", type=int, default=None, help="stream workload only: a fixed number of launches and no timing (profiler counter passes)")
     ap.add_argument("--stream-format", default="i2s", choices=["i2s", "qk256"])

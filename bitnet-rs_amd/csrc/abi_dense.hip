@@ -211,7 +211,7 @@ int bitnet_hip_latent_prefill_dev(const bitnet_hip_latent_attention *attn, const
     LatentAttn a;
     if (int rc = to_attn(attn, a)) return rc;
     BH_REQUIRE(q && k && vt && out && nq > 0 && nq <= n_ctx && n_ctx <= attn->capacity && ldvt % 8 == 0 && ldvt >= (n_ctx + 63) / 64 * 64 &&
-                   ldo >= attn->heads * attn->vdimp && ldo % 4 == 0,
+                   ldo >= attn->heads * attn->vdimp && ldo % 4 == 0 && attn->vdimp % 32 == 0,
                "latent_prefill: bad arguments");
     if (!latent_prefill_supported(a.qd, a.vdimp)) return set_error(BITNET_HIP_ERR_UNSUPPORTED, "latent_prefill: head of %d / %d columns", a.qd, a.vdimp);
     a.qb = q, a.k = k, a.vt = vt, a.ldvt = ldvt, a.n_ctx = (int)n_ctx, a.nq = (int)nq, a.out = out, a.ldo = ldo;

@@ -454,10 +454,12 @@ hipError_t launch_dense_gemv(const GemvArgs &a, int *n_wg_out, hipStream_t s) {
 }
 
 // ---- many-row matmul --------------------------------------------------------------------------------------------------
-// C[m][n] = act(A[m][k] . W[n][k]^T + bias).  128 x 128 workgroup tile, four waves of 64 x 64, K steps of 64 columns staged in
-// LDS by LDS-DMA, two buffers.  LDS image of a row: eight 16-byte units, unit q stored at q ^ (row & 7).  The MFMA's A operand
-// is the weight tile (rows = output columns n), its B operand the activation tile, so a lane holds four consecutive n of one row.
-constexpr int kTileM = 128, kTileN = 128, kTileK = 64;
+// C[m][n] = act(A[m][k] . W[n][k]^T + bias).  T x T workgroup tile, four waves of T/2 x T/2, K steps of 64 columns staged in LDS by
+// LDS-DMA, ST buffers (ST - 1 steps ahead): 128 x 128 with two buffers where the launch fills the chip, 64 x 64 with four where it
+// does not and a step would wait for memory.  LDS image of a row: eight 16-byte units, unit q stored at q ^ ((row >> 1) & 7): the
+// sixteen rows of a ds_read_b128 then cover all 64 banks once.  The MFMA's A operand is the weight tile (rows = output columns n),
+// its B operand the activation tile, so a lane holds four consecutive n of one row.
+constexpr int kTileK = 64;
 
 __device__ __forceinline__ void dma1k(const void *lane_ptr, unsigned lds_dst) {
     unsigned keep;
@@ -467,82 +469,88 @@ __device__ __forceinline__ void dma1k(const void *lane_ptr, unsigned lds_dst) {
                  : "memory");
 }
 
-template <bool CF32>
+template <int T, int ST, bool CF32>
 __global__ __launch_bounds__(256, 2) void k_dense_gemm(GemmArgsD p, int tiles_n, int tiles_m, int swizzle) {
     extern __shared__ __attribute__((aligned(1024))) uint8_t lds[];
+    constexpr int ND = T / 32;          // DMA instructions per wave, operand and step (eight rows each)
+    constexpr int F = T / 32;           // 16-row fragments per wave and operand
+    constexpr unsigned HALF = T * 128, BUF = 2 * HALF;
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
-    // workgroup -> tile: consecutive workgroups land on the eight XCDs in turn; give each XCD a contiguous run of tiles that
-    // walks the row tiles of one weight tile first
+    // workgroup -> tile: consecutive workgroups land on the eight XCDs in turn; give each XCD a contiguous run of tiles, and walk
+    // the tiles in groups of eight row tiles so that what runs together shares both operands in the XCD's L2
     int id = blockIdx.x;
     const int total = tiles_n * tiles_m;
     if (swizzle) id = (id & 7) * (total >> 3) + (id >> 3);
-    // groups of eight row tiles share the weight tiles they walk
     const int gm = 8;
     const int group = id / (gm * tiles_n), first = group * gm, size = tiles_m - first < gm ? tiles_m - first : gm;
     const int tm = first + (id % (gm * tiles_n)) % size, tn = (id % (gm * tiles_n)) / size;
-    const int m0 = tm * kTileM, n0 = tn * kTileN;
+    const int m0 = tm * T, n0 = tn * T;
     const uint16_t *A = (const uint16_t *)p.a + (size_t)blockIdx.y * p.a_batch;
     const uint16_t *W = p.w + (size_t)blockIdx.y * p.w_batch;
-    // LDS-DMA: one instruction stages eight rows of 64 columns (1 KiB); wave w stages rows [32 w, 32 w + 32) of both tiles
-    const int drow = lane >> 3, dunit = (lane & 7) ^ drow;
-    const uint16_t *ga[4], *gw[4];
+    const int drow = lane >> 3;
+    const uint16_t *ga[ND], *gw[ND];
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
-        const int r = wave * 32 + i * 8 + drow;
+    for (int i = 0; i < ND; ++i) {
+        const int r = wave * (T / 4) + i * 8 + drow, unit = (lane & 7) ^ ((r >> 1) & 7);
         const int ar = m0 + r < p.m ? m0 + r : p.m - 1, wr = n0 + r < p.n ? n0 + r : p.n - 1;
-        ga[i] = A + (size_t)ar * p.lda + dunit * 8;
-        gw[i] = W + (size_t)wr * p.ldw + dunit * 8;
+        ga[i] = A + (size_t)ar * p.lda + unit * 8;
+        gw[i] = W + (size_t)wr * p.ldw + unit * 8;
     }
     const unsigned base = (unsigned)(uintptr_t)(__attribute__((address_space(3))) uint8_t *)lds;
-    auto stage = [&](int k0, int buf) {
-        const unsigned dst = base + buf * 32768 + wave * 4096;
+    auto stage = [&](int t) {
+        const unsigned dst = base + (t % ST) * BUF + wave * (T / 4) * 128;
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-            dma1k(ga[i] + k0, dst + i * 1024);
-            dma1k(gw[i] + k0, dst + 16384 + i * 1024);
+        for (int i = 0; i < ND; ++i) {
+            dma1k(ga[i] + t * kTileK, dst + i * 1024);
+            dma1k(gw[i] + t * kTileK, dst + HALF + i * 1024);
         }
     };
-    const int wn = (wave & 1) * 64, wm = (wave >> 1) * 64;
-    const int r16 = lane & 15, g = lane >> 4;
-    f32x4 acc[4][4];
+    const int wn = (wave & 1) * (T / 2), wm = (wave >> 1) * (T / 2);
+    const int r16 = lane & 15, g = lane >> 4, sw = (r16 >> 1) & 7;
+    f32x4 acc[F][F];
 #pragma unroll
-    for (int i = 0; i < 4; ++i)
+    for (int i = 0; i < F; ++i)
 #pragma unroll
-        for (int j = 0; j < 4; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+        for (int j = 0; j < F; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
     const int steps = p.k / kTileK;
-    stage(0, 0);
-    asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-    __syncthreads();
+#pragma unroll
+    for (int t = 0; t < ST - 1; ++t)
+        if (t < steps) stage(t);
     for (int t = 0; t < steps; ++t) {
-        if (t + 1 < steps) stage((t + 1) * kTileK, (t + 1) & 1);
-        const uint8_t *la = lds + (t & 1) * 32768, *lw = la + 16384;
+        // step t's tile has landed once at most the ST - 2 later ones are outstanding (loads return in order); the barrier also says
+        // that every wave has left the buffer the next request overwrites
+        if (ST > 2 && t + ST - 2 < steps)
+            asm volatile("s_waitcnt vmcnt(%0)" ::"n"((ST - 2) * 2 * ND) : "memory");
+        else
+            asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+        __syncthreads();
+        if (t + ST - 1 < steps) stage(t + ST - 1);
+        const uint8_t *la = lds + (t % ST) * BUF, *lw = la + HALF;
 #pragma unroll
         for (int kk = 0; kk < 2; ++kk) {
-            bf16x8 fa[4], fw[4];
-            const int q = ((kk * 4 + g) ^ (r16 & 7)) * 16;
+            bf16x8 fa[F], fw[F];
+            const int q = ((kk * 4 + g) ^ sw) * 16;
 #pragma unroll
-            for (int i = 0; i < 4; ++i) {
+            for (int i = 0; i < F; ++i) {
                 fw[i] = *reinterpret_cast<const bf16x8 *>(lw + (wn + i * 16 + r16) * 128 + q);
                 fa[i] = *reinterpret_cast<const bf16x8 *>(la + (wm + i * 16 + r16) * 128 + q);
             }
 #pragma unroll
-            for (int i = 0; i < 4; ++i)
+            for (int i = 0; i < F; ++i)
 #pragma unroll
-                for (int j = 0; j < 4; ++j) acc[i][j] = mfma_bf16(fw[i], fa[j], acc[i][j]);
+                for (int j = 0; j < F; ++j) acc[i][j] = mfma_bf16(fw[i], fa[j], acc[i][j]);
         }
-        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");  // the next tile has landed
-        __syncthreads();
     }
     const bool vec = (p.ldc & 3) == 0;
 #pragma unroll
-    for (int i = 0; i < 4; ++i) {
+    for (int i = 0; i < F; ++i) {
         const int n = n0 + wn + i * 16 + g * 4;
         if (n >= p.n) continue;
         float bias[4];
 #pragma unroll
         for (int e = 0; e < 4; ++e) bias[e] = p.bias && n + e < p.n ? p.bias[n + e] : 0.f;
 #pragma unroll
-        for (int j = 0; j < 4; ++j) {
+        for (int j = 0; j < F; ++j) {
             const int m = m0 + wm + j * 16 + r16;
             if (m >= p.m) continue;
             float v[4];
@@ -564,6 +572,13 @@ __global__ __launch_bounds__(256, 2) void k_dense_gemm(GemmArgsD p, int tiles_n,
             }
         }
     }
+}
+
+template <int T, int ST>
+static void gemm_go(const GemmArgsD &a, hipStream_t s) {
+    const int tn = (a.n + T - 1) / T, tm = (a.m + T - 1) / T, swz = (tn * tm) % 8 == 0 ? 1 : 0;
+    auto fn = a.c_f32 ? k_dense_gemm<T, ST, true> : k_dense_gemm<T, ST, false>;
+    hipLaunchKernelGGL(fn, dim3(tn * tm, a.batch), dim3(256), ST * T * 256, s, a, tn, tm, swz);
 }
 
 // f32 activations: f32 multiply-adds on a 64 x 64 tile, 4 x 4 per thread
@@ -618,12 +633,10 @@ hipError_t launch_dense_gemm(const GemmArgsD &args, hipStream_t s) {
         hipLaunchKernelGGL(k_dense_gemm_f32, dim3((a.n + 63) / 64, (a.m + 63) / 64, a.batch), dim3(256), 0, s, a);
         return hipGetLastError();
     }
-    const int tn = (a.n + kTileN - 1) / kTileN, tm = (a.m + kTileM - 1) / kTileM;
-    const int swz = (tn * tm) % 8 == 0 ? 1 : 0;
-    if (a.c_f32)
-        hipLaunchKernelGGL(k_dense_gemm<true>, dim3(tn * tm, a.batch), dim3(256), 65536, s, a, tn, tm, swz);
+    if ((long)((a.n + 127) / 128) * ((a.m + 127) / 128) * a.batch >= 256)
+        gemm_go<128, 2>(a, s);
     else
-        hipLaunchKernelGGL(k_dense_gemm<false>, dim3(tn * tm, a.batch), dim3(256), 65536, s, a, tn, tm, swz);
+        gemm_go<64, 4>(a, s);
     return hipGetLastError();
 }
 

@@ -19,11 +19,12 @@ __device__ __forceinline__ void split_range(int n_keys, int &per, int &used) {
     used = (tiles + per - 1) / per;
 }
 
-// element i of the rotated part of query head (raw part at q)
-__device__ __forceinline__ float rotated(const float *q, const float *cs, const float *sn, int half, int i) {
-    if (i < half) return q[i] * cs[i] - q[i + half] * sn[i];
-    if (i < 2 * half) return q[i] * cs[i - half] + q[i - half] * sn[i - half];
-    return 0.f;
+// element i of the rotated part of a query head (raw part at q); elements past 2 * half are zero
+template <class T>
+__device__ __forceinline__ float rotated(const T *q, const float *cs, const float *sn, int half, int i) {
+    const int n = 2 * half, a = min(i, n - 1), b = a < half ? a + half : a - half, c = a < half ? a : a - half;
+    const float x = ld_act(q, a), y = ld_act(q, b), s = sn[c], live = i < n ? 1.0f : 0.0f;  // (a product, not a branch around the loads)
+    return (x * cs[c] + (a < half ? -y : y) * s) * live;
 }
 
 size_t latent_scratch_floats(int heads, int ldc, int nq) { return (size_t)nq * heads * kLatentSplits * (kLatentRecHead + ldc); }
@@ -132,27 +133,29 @@ __global__ __launch_bounds__(256) void k_latent_decode(LatentAttn p) {
     };
     fetch(k0);
     {
-        // the query rows: latent part, then the rotated part
-        const int half = p.rot_dim / 2;
+        // the query rows, sixteen threads each: latent part, then the rotated part
+        const int half = p.rot_dim / 2, row = tid >> 4, c4 = (tid & 15) * 4, h = min(h0 + row, p.heads - 1);
+        const float *qa = p.qabs + ((size_t)qi * p.heads + h) * p.ldc + c4;
+        const float *qr = p.q + ((size_t)qi * p.heads + h) * p.qd + p.dimp;
         const float *cs = p.rope_cos + (size_t)pos * half, *sn = p.rope_sin + (size_t)pos * half;
-        const int pairs = kt / 2;
-        for (int idx = tid; idx < 16 * pairs; idx += 256) {
-            const int row = idx / pairs, i = (idx - row * pairs) * 2, h = h0 + row;
-            float v0 = 0.f, v1 = 0.f;
-            if (h < p.heads) {
-                if (i < p.ldc) {
-                    const float *qa = p.qabs + ((size_t)qi * p.heads + h) * p.ldc;
-                    v0 = qa[i], v1 = qa[i + 1];
-                } else {
-                    const float *qr = p.q + ((size_t)qi * p.heads + h) * p.qd + p.dimp;
-                    v0 = rotated(qr, cs, sn, half, i - p.ldc), v1 = rotated(qr, cs, sn, half, i + 1 - p.ldc);
-                }
-            }
+        const int n64 = p.ldc >> 6;
+        f32x4 v[kDecNT];
+#pragma unroll
+        for (int t = 0; t < kDecNT; ++t)
+            if (t < n64) v[t] = *reinterpret_cast<const f32x4 *>(qa + t * 64);
+        auto put = [&](int i, float a, float b) {
             uint32_t hi, lo;
-            split2(v0, v1, hi, lo);
+            split2(a, b, hi, lo);
             *reinterpret_cast<uint32_t *>(qh + row * qs + i * 2) = hi;
             *reinterpret_cast<uint32_t *>(ql + row * qs + i * 2) = lo;
-        }
+        };
+        for (int i = (tid & 15) * 2; i < p.ldr; i += 32) put(p.ldc + i, rotated(qr, cs, sn, half, i), rotated(qr, cs, sn, half, i + 1));
+#pragma unroll
+        for (int t = 0; t < kDecNT; ++t)
+            if (t < n64) {
+                put(t * 64 + c4, v[t].x, v[t].y);
+                put(t * 64 + c4 + 2, v[t].z, v[t].w);
+            }
     }
     __syncthreads();
     f32x4 o[kDecNT];
@@ -342,7 +345,7 @@ hipError_t launch_latent_merge(const LatentMerge &a, hipStream_t s) {
 template <int NK, int NV, int QT>
 __global__ __launch_bounds__(256, NV > 8 ? 1 : 2) void k_latent_prefill(LatentAttn p, int n_qb) {
     extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
-    constexpr int KS = NK * 64 + 16, VS = kLatentTile * 2 + 16, NVL = (NV + 1) / 2;
+    constexpr int KS = NK * 64 + 16, VS = kLatentTile * 2 + 16, NVL = NV / 2;
     uint8_t *lk = lds, *lv = lds + kLatentTile * KS;
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r16 = lane & 15, g = lane >> 4;
     // consecutive workgroups go to the eight XCDs in turn: a head's blocks stay on one of them, longest blocks first
@@ -363,20 +366,11 @@ __global__ __launch_bounds__(256, NV > 8 ? 1 : 2) void k_latent_prefill(LatentAt
 #pragma unroll
         for (int kk = 0; kk < NK; ++kk) {
             const int d = kk * 32 + g * 8;
-            if (d < p.dimp) {
+            if (kk * 32 < p.dimp) {
                 qf[t][kk] = *reinterpret_cast<const bf16x8 *>(q + d);
             } else {
-                const uint16_t *qr = q + p.dimp;
 #pragma unroll
-                for (int e = 0; e < 8; ++e) {
-                    const int i = d + e - p.dimp;
-                    float v = 0.f;
-                    if (i < half)
-                        v = bf2f(qr[i]) * cs[i] - bf2f(qr[i + half]) * sn[i];
-                    else if (i < 2 * half)
-                        v = bf2f(qr[i]) * cs[i - half] + bf2f(qr[i - half]) * sn[i - half];
-                    qf[t][kk][e] = (__bf16)v;
-                }
+                for (int e = 0; e < 8; ++e) qf[t][kk][e] = (__bf16)rotated(q + p.dimp, cs, sn, half, d + e - p.dimp);
             }
         }
     }
@@ -394,35 +388,36 @@ __global__ __launch_bounds__(256, NV > 8 ? 1 : 2) void k_latent_prefill(LatentAt
     const uint16_t *V = (const uint16_t *)p.vt + (size_t)h * p.vdimp * p.ldvt;
     const size_t ldk = (size_t)p.heads * p.dimp;
     u32x4 kreg[NK], vreg[NVL];
+    // four threads per key: 64 bytes of every 32-column step, latent keys first, then the shared rotated part (both multiples of 32
+    // columns: one address form per step); eight threads per row of V^T
+    const unsigned koff = (unsigned)((tid >> 2) * ldk * 2 + (tid & 3) * 16), roff = (unsigned)((tid >> 2) * p.ldr * 2 + (tid & 3) * 16);
+    const unsigned voff = (unsigned)((tid >> 3) * p.ldvt * 2 + (tid & 7) * 16);
     auto fetch = [&](int key0) {
+        const char *kb = (const char *)(K + (size_t)key0 * ldk), *rb = (const char *)(R + (size_t)key0 * p.ldr), *vb = (const char *)(V + key0);
 #pragma unroll
         for (int j = 0; j < NK; ++j) {
-            const int idx = tid + 256 * j, row = idx / (NK * 4), d = (idx % (NK * 4)) * 8;
-            const int key = min(key0 + row, p.n_ctx - 1);
-            kreg[j] = d < p.dimp ? *reinterpret_cast<const u32x4 *>(K + key * ldk + d)
-                    : d < p.dimp + p.ldr ? *reinterpret_cast<const u32x4 *>(R + (size_t)key * p.ldr + d - p.dimp) : u32x4{0u, 0u, 0u, 0u};
+            if (j * 32 < p.dimp)
+                kreg[j] = *reinterpret_cast<const u32x4 *>(kb + j * 64 + koff);
+            else if (j * 32 < p.qd)
+                kreg[j] = *reinterpret_cast<const u32x4 *>(rb + (j * 64 - p.dimp * 2) + roff);
         }
 #pragma unroll
-        for (int j = 0; j < NVL; ++j) {
-            const int idx = tid + 256 * j, row = idx >> 3;
-            vreg[j] = row < p.vdimp ? *reinterpret_cast<const u32x4 *>(V + (size_t)row * p.ldvt + key0 + (idx & 7) * 8) : u32x4{0u, 0u, 0u, 0u};
-        }
+        for (int j = 0; j < NVL; ++j)
+            if (j * 32 < p.vdimp) vreg[j] = *reinterpret_cast<const u32x4 *>(vb + (size_t)j * 64 * p.ldvt + voff);
     };
+#pragma unroll
+    for (int j = 0; j < NK; ++j) kreg[j] = u32x4{0u, 0u, 0u, 0u};
+#pragma unroll
+    for (int j = 0; j < NVL; ++j) vreg[j] = u32x4{0u, 0u, 0u, 0u};
     const int n_tiles = (min(p.n_ctx, pos0 + q0 + 64 * QT) + kLatentTile - 1) / kLatentTile;
     fetch(0);
     for (int kt0 = 0; kt0 < n_tiles; ++kt0) {
         const int key0 = kt0 * kLatentTile;
         __syncthreads();
 #pragma unroll
-        for (int j = 0; j < NK; ++j) {
-            const int idx = tid + 256 * j, row = idx / (NK * 4), c = idx % (NK * 4);
-            *reinterpret_cast<u32x4 *>(lk + row * KS + c * 16) = kreg[j];
-        }
+        for (int j = 0; j < NK; ++j) *reinterpret_cast<u32x4 *>(lk + (tid >> 2) * KS + j * 64 + (tid & 3) * 16) = kreg[j];
 #pragma unroll
-        for (int j = 0; j < NVL; ++j) {
-            const int idx = tid + 256 * j;
-            if (NV % 2 == 0 || (idx >> 3) < NV * 16) *reinterpret_cast<u32x4 *>(lv + (idx >> 3) * VS + (idx & 7) * 16) = vreg[j];
-        }
+        for (int j = 0; j < NVL; ++j) *reinterpret_cast<u32x4 *>(lv + ((tid >> 3) + 32 * j) * VS + (tid & 7) * 16) = vreg[j];
         __syncthreads();
         if (kt0 + 1 < n_tiles) fetch(key0 + kLatentTile);
         if (key0 > pos0 + qw + 16 * QT - 1) continue;  // every key of the tile lies ahead of this wave's queries
@@ -519,7 +514,7 @@ static hipError_t prefill_go(const LatentAttn &a, hipStream_t s) {
 
 hipError_t launch_latent_prefill(const LatentAttn &a, hipStream_t s) {
     const int nk = a.qd / 32, nv = a.vdimp / 16;
-    if (a.qd % 32 || a.vdimp % 16 || !latent_prefill_supported(a.qd, a.vdimp)) return hipErrorInvalidValue;
+    if (a.qd % 32 || a.dimp % 32 || a.vdimp % 32 || !latent_prefill_supported(a.qd, a.vdimp)) return hipErrorInvalidValue;
     if (nv > 8) return prefill_go<8, 16, 1>(a, s);
     if (nk <= 2) return nv <= 2 ? prefill_go<2, 2, 2>(a, s) : nv <= 4 ? prefill_go<2, 4, 2>(a, s) : prefill_go<2, 8, 2>(a, s);
     if (nk <= 4) return nv <= 4 ? prefill_go<4, 4, 2>(a, s) : prefill_go<4, 8, 2>(a, s);

@@ -84,6 +84,13 @@ struct LinearWs {
 
 constexpr int kTS = kLinBlock * 2 + 16;  // bytes per row of a transposed [column][token] tile
 
+// 16 bytes of row t at column c, or zero where either lies outside: the address is clamped, so loads stay unconditional
+__device__ __forceinline__ u32x4 load_or_zero(const uint16_t *m, size_t ld, int t, int n, int c, int cols) {
+    const u32x4 v = *reinterpret_cast<const u32x4 *>(m + (size_t)min(t, n - 1) * ld + min(c, cols - 8));
+    const bool ok = t < n && c < cols;
+    return u32x4{ok ? v.x : 0u, ok ? v.y : 0u, ok ? v.z : 0u, ok ? v.w : 0u};
+}
+
 // two tokens' eight columns -> eight (token, token + 1) dwords
 __device__ __forceinline__ void pair_columns(u32x4 a, u32x4 b, uint32_t out[8]) {
 #pragma unroll
@@ -103,17 +110,21 @@ __global__ __launch_bounds__(256) void k_linear_sums(LinearAttn p, LinearWs w) {
     const int t0 = blk * kLinBlock, len = min(kLinBlock, p.n - t0);
     const float *pw = p.decay_pow + (size_t)h * (kLinBlock + 1);
     const uint16_t *K = (const uint16_t *)p.qkv + (size_t)(p.heads + h) * p.dimp, *V = (const uint16_t *)p.qkv + 2 * (size_t)p.heads * p.dimp + (size_t)h * p.vdimp;
-    const u32x4 zero = {0u, 0u, 0u, 0u};
+    K += (size_t)t0 * p.ld, V += (size_t)t0 * p.ld;
+    u32x4 kv[2][4];
 #pragma unroll
     for (int j = 0; j < 2; ++j) {
         const int idx = tid + 256 * j, c = (idx & 7) * 8, t = (idx >> 3) * 2;
-        const size_t r0 = (size_t)(t0 + t) * p.ld, r1 = r0 + p.ld;
-        const bool a = t < len, b = t + 1 < len;
-        const u32x4 va = a && v0 + c < p.vdimp ? *reinterpret_cast<const u32x4 *>(V + r0 + v0 + c) : zero;
-        const u32x4 vb = b && v0 + c < p.vdimp ? *reinterpret_cast<const u32x4 *>(V + r1 + v0 + c) : zero;
-        const u32x4 ka = a && k0 + c < p.dimp ? *reinterpret_cast<const u32x4 *>(K + r0 + k0 + c) : zero;
-        const u32x4 kb = b && k0 + c < p.dimp ? *reinterpret_cast<const u32x4 *>(K + r1 + k0 + c) : zero;
-        const float pa = a ? pw[len - 1 - t] : 0.f, pb = b ? pw[len - 2 - t] : 0.f;
+        kv[j][0] = load_or_zero(V, p.ld, t, len, v0 + c, p.vdimp);
+        kv[j][1] = load_or_zero(V, p.ld, t + 1, len, v0 + c, p.vdimp);
+        kv[j][2] = load_or_zero(K, p.ld, t, len, k0 + c, p.dimp);
+        kv[j][3] = load_or_zero(K, p.ld, t + 1, len, k0 + c, p.dimp);
+    }
+#pragma unroll
+    for (int j = 0; j < 2; ++j) {
+        const int idx = tid + 256 * j, c = (idx & 7) * 8, t = (idx >> 3) * 2;
+        const u32x4 va = kv[j][0], vb = kv[j][1], ka = kv[j][2], kb = kv[j][3];
+        const float pa = pw[max(len - 1 - t, 0)], pb = pw[max(len - 2 - t, 0)];  // (tokens past the end are zero)
         uint32_t o[8];
         pair_columns(va, vb, o);
 #pragma unroll
@@ -186,39 +197,39 @@ __global__ __launch_bounds__(512) void k_linear_out(LinearAttn p, LinearWs w) {
     const int blk = blockIdx.x, h = blockIdx.y, t0 = blk * kLinBlock, len = min(kLinBlock, p.n - t0);
     const uint16_t *Q = (const uint16_t *)p.qkv + (size_t)h * p.dimp, *K = Q + (size_t)p.heads * p.dimp;
     const uint16_t *V = (const uint16_t *)p.qkv + 2 * (size_t)p.heads * p.dimp + (size_t)h * p.vdimp;
-    const u32x4 zero = {0u, 0u, 0u, 0u};
+    Q += (size_t)t0 * p.ld, K += (size_t)t0 * p.ld, V += (size_t)t0 * p.ld;
     if (tid <= kLinBlock) pw[tid] = p.decay_pow[(size_t)h * (kLinBlock + 1) + tid];
-    for (int idx = tid; idx < kLinBlock * NK * 4; idx += 512) {
-        const int t = idx / (NK * 4), c = (idx % (NK * 4)) * 8;
-        *reinterpret_cast<u32x4 *>(lk + t * KS + c * 2) = t < len && c < p.dimp ? *reinterpret_cast<const u32x4 *>(K + (size_t)(t0 + t) * p.ld + c) : zero;
-    }
-    for (int idx = tid; idx < kLinBlock / 2 * NV * 2; idx += 512) {
-        const int t = (idx / (NV * 2)) * 2, c = (idx % (NV * 2)) * 8;
-        const u32x4 a = t < len && c < p.vdimp ? *reinterpret_cast<const u32x4 *>(V + (size_t)(t0 + t) * p.ld + c) : zero;
-        const u32x4 b = t + 1 < len && c < p.vdimp ? *reinterpret_cast<const u32x4 *>(V + (size_t)(t0 + t + 1) * p.ld + c) : zero;
-        uint32_t o[8];
-        pair_columns(a, b, o);
-#pragma unroll
-        for (int e = 0; e < 8; ++e) *reinterpret_cast<uint32_t *>(lv + (c + e) * kTS + t * 2) = o[e];
-    }
     const int i = wave * 16 + r16;  // this lane's query within the block
     bf16x8 q[NK];
 #pragma unroll
-    for (int kk = 0; kk < NK; ++kk) {
-        const int c = kk * 32 + g * 8;
-        q[kk] = __builtin_bit_cast(bf16x8, i < len && c < p.dimp ? *reinterpret_cast<const u32x4 *>(Q + (size_t)(t0 + i) * p.ld + c) : zero);
+    for (int kk = 0; kk < NK; ++kk) q[kk] = __builtin_bit_cast(bf16x8, load_or_zero(Q, p.ld, i, len, kk * 32 + g * 8, p.dimp));
+    {
+        u32x4 kr[NK], vr[NV / 4][2];
+#pragma unroll
+        for (int j = 0; j < NK; ++j) kr[j] = load_or_zero(K, p.ld, tid >> 2, len, j * 32 + (tid & 3) * 8, p.dimp);  // four threads per token
+#pragma unroll
+        for (int j = 0; j < NV / 4; ++j)  // eight threads per pair of tokens
+#pragma unroll
+            for (int e = 0; e < 2; ++e) vr[j][e] = load_or_zero(V, p.ld, (tid >> 3) * 2 + e, len, j * 64 + (tid & 7) * 8, p.vdimp);
+#pragma unroll
+        for (int j = 0; j < NK; ++j) *reinterpret_cast<u32x4 *>(lk + (tid >> 2) * KS + j * 64 + (tid & 3) * 16) = kr[j];
+#pragma unroll
+        for (int j = 0; j < NV / 4; ++j) {
+            uint32_t o[8];
+            pair_columns(vr[j][0], vr[j][1], o);
+#pragma unroll
+            for (int e = 0; e < 8; ++e) *reinterpret_cast<uint32_t *>(lv + (j * 64 + (tid & 7) * 8 + e) * kTS + (tid >> 3) * 4) = o[e];
+        }
     }
     f32x4 o[NV];
     const size_t sb = ((size_t)h * w.nb + blk) * p.vdimp * p.dimp;
 #pragma unroll
     for (int v = 0; v < NV; ++v) {
         o[v] = f32x4{0.f, 0.f, 0.f, 0.f};
-        if (v * 16 >= p.vdimp) continue;
 #pragma unroll
         for (int kk = 0; kk < NK; ++kk) {
-            const int c = kk * 32 + g * 8;
-            if (kk * 32 >= p.dimp) continue;
-            const size_t at = sb + (size_t)(v * 16 + r16) * p.dimp + c;
+            // (rows past vdimp are never stored, columns past dimp meet a zero query: clamped addresses, no branches around the loads)
+            const size_t at = sb + (size_t)min(v * 16 + r16, p.vdimp - 1) * p.dimp + min(kk * 32 + g * 8, p.dimp - 8);
             o[v] = mfma_bf16(*reinterpret_cast<const bf16x8 *>(w.hi + at), q[kk], o[v]);
             o[v] = mfma_bf16(*reinterpret_cast<const bf16x8 *>(w.lo + at), q[kk], o[v]);
         }

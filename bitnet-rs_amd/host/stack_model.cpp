@@ -55,7 +55,7 @@ StackModel::StackModel(const StackSpec &spec, bool f32, int max_pos) : spec_(spe
                     return;
                 }
             }
-            L.dimp = (int)up_to(m.dim, 32), L.rotp = (int)up_to(std::max(m.rot_dim, 1), 32), L.vdimp = (int)up_to(m.vdim, 16), L.ldc = (int)up_to(m.kv_rank, 64);
+            L.dimp = (int)up_to(m.dim, 32), L.rotp = (int)up_to(std::max(m.rot_dim, 1), 32), L.vdimp = (int)up_to(m.vdim, 32), L.ldc = (int)up_to(m.kv_rank, 64);
             if (L.ldc > 1024) {
                 err_ = "stack: kv_rank above 1024";
                 return;

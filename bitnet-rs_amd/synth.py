@@ -113,7 +113,7 @@ def prompt(n: int, vocab: int, bos: int = 128000) -> np.ndarray:
 STACK_SIZES = {  # width, ff, heads, kv heads of the BitNet model of equal size, q_rank, vocab
     "1b": dict(width=1536, ff=4096, heads=12, n_kv=3, q_rank=768, vocab=32768),
     "2b": dict(width=2560, ff=6912, heads=20, n_kv=5, q_rank=1536, vocab=128256),
-    "5b": dict(width=4096, ff=8192, heads=32, n_kv=8, q_rank=1536, vocab=32768),
+    "3b": dict(width=3072, ff=8192, heads=24, n_kv=6, q_rank=1536, vocab=32768),
 }
 
 

@@ -651,9 +651,9 @@ int bitnet_hip_latent_decode_dev(const bitnet_hip_latent_attention *attn, const 
                                  size_t q0, size_t nq, int f32, float *scratch_dev, void *stream);
 int bitnet_hip_latent_merge_dev(const bitnet_hip_latent_attention *attn, const uint16_t *uv_dev, const int32_t *pos_dev, size_t q0,
                                 size_t nq, const float *scratch_dev, void *out_dev, size_t ldo, int out_bf16, void *stream);
-/* A portion of a prompt, bf16: the LAST nq of n_ctx positions attend.  q bf16 [nq][heads * qd], k bf16 [n_ctx][heads * dimp] = W_uk c,
- * vt bf16 [heads * vdimp][ldvt] = (W_uv c)^T with columns up to the next multiple of 64 finite; out bf16 [nq][ldo].
- * qd <= 256 and vdimp <= 256 (bitnet_hip_latent_prefill_supported). */
+/* A portion of a prompt, bf16: the LAST nq of n_ctx positions attend.  q bf16 [nq][heads * qd], k bf16 [n_ctx][heads * dimp] = W_uk c
+ * (rows up to the next multiple of 64 readable), vt bf16 [heads * vdimp][ldvt] = (W_uv c)^T (columns up to the next multiple of 64
+ * finite); out bf16 [nq][ldo].  vdimp % 32 == 0, qd <= 256 and vdimp <= 256 (bitnet_hip_latent_prefill_supported). */
 int bitnet_hip_latent_prefill_supported(size_t qd, size_t vdimp);
 int bitnet_hip_latent_prefill_dev(const bitnet_hip_latent_attention *attn, const uint16_t *q_dev, const uint16_t *k_dev,
                                   const uint16_t *vt_dev, size_t ldvt, size_t n_ctx, size_t nq, uint16_t *out_dev, size_t ldo, void *stream);

@@ -118,7 +118,7 @@ class Latent:
         g = rng(L, nq, heads, dim, seed)
         self.L, self.nq, self.heads, self.f32 = L, nq, heads, f32
         store = (lambda a: a.astype(np.float32)) if f32 else u.rounded
-        self.dimp, self.rotp, self.vdimp, self.ldc, self.cap = u.up_to(dim, 32), u.up_to(rot, 32), u.up_to(vdim, 16), u.up_to(rank, 64), u.up_to(L, 64)
+        self.dimp, self.rotp, self.vdimp, self.ldc, self.cap = u.up_to(dim, 32), u.up_to(rot, 32), u.up_to(vdim, 32), u.up_to(rank, 64), u.up_to(L, 64)
         self.qd = self.dimp + self.rotp
         q = store(g.standard_normal((nq, heads, dim + rot)))
         c, kr = store(g.standard_normal((L, rank))), store(g.standard_normal((L, rot)))
@@ -175,7 +175,7 @@ class Latent:
         return u.host(out)
 
     def prefill(self, hip):
-        k = np.einsum("lc,hdc->lhd", self.c_host[:self.L], self.uk_host)
+        k = np.einsum("lc,hdc->lhd", self.c_host, self.uk_host)
         vt = np.einsum("lc,hvc->hvl", self.c_host, self.uv_host)
         out = u.zeros_bf16(self.nq, self.heads, self.vdimp)
         hip.latent_prefill_dev(self.attn, u.dev_bf16(self.q), u.dev_bf16(k), u.dev_bf16(vt), self.cap, self.L, self.nq, out, self.heads * self.vdimp)
