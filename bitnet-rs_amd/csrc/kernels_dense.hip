@@ -198,7 +198,22 @@ __device__ void form_input(const VecIn &in, const float *x, int cols, int kp, fl
     const int tid = threadIdx.x;
     const int n = in.n;
     if (in.kind == BITNET_HIP_IN_PLAIN) {
-        for (int i = tid; i < kp; i += 256) xs[i] = i < cols ? x[i] : 0.f;
+        if ((cols & 3) == 0 && ((uintptr_t)x & 15) == 0) {
+            constexpr int NV = 8;  // sixteen-byte loads in flight per thread
+            const int c4 = cols >> 2, k4 = kp >> 2;
+            for (int i0 = tid; i0 < k4; i0 += 256 * NV) {
+                f32x4 v[NV];
+#pragma unroll
+                for (int j = 0; j < NV; ++j) v[j] = reinterpret_cast<const f32x4 *>(x)[min(i0 + 256 * j, c4 - 1)];
+#pragma unroll
+                for (int j = 0; j < NV; ++j) {
+                    const int i = i0 + 256 * j;
+                    if (i < k4) reinterpret_cast<f32x4 *>(xs)[i] = i < c4 ? v[j] : f32x4{0.f, 0.f, 0.f, 0.f};
+                }
+            }
+        } else {
+            for (int i = tid; i < kp; i += 256) xs[i] = i < cols ? x[i] : 0.f;
+        }
         __syncthreads();
         return;
     }
@@ -209,7 +224,8 @@ __device__ void form_input(const VecIn &in, const float *x, int cols, int kp, fl
 #pragma unroll
         for (int j = 0; j < NR; ++j) {
             const int i = tid + 256 * j;
-            xv[j] = i < n4 ? reinterpret_cast<const f32x4 *>(x)[i] : f32x4{0.f, 0.f, 0.f, 0.f};
+            const f32x4 v = reinterpret_cast<const f32x4 *>(x)[min(i, n4 - 1)];
+            xv[j] = v * (i < n4 ? 1.0f : 0.0f);
         }
         if (in.kind == BITNET_HIP_IN_RESIDUAL_NORM && in.y) {
             f32x4 yv[NR], pw[NR], sc[NR];
@@ -217,10 +233,17 @@ __device__ void form_input(const VecIn &in, const float *x, int cols, int kp, fl
 #pragma unroll
             for (int j = 0; j < NR; ++j) {
                 const int i = tid + 256 * j;
-                const bool ok = i < n4;
-                yv[j] = ok ? reinterpret_cast<const f32x4 *>(in.y)[i] : f32x4{0.f, 0.f, 0.f, 0.f};
-                pw[j] = ok ? reinterpret_cast<const f32x4 *>(in.post_weight)[i] : f32x4{0.f, 0.f, 0.f, 0.f};
-                sc[j] = ok && in.scale ? reinterpret_cast<const f32x4 *>(in.scale)[i] : f32x4{1.f, 1.f, 1.f, 1.f};
+                const int c = min(i, n4 - 1);
+                const f32x4 v = reinterpret_cast<const f32x4 *>(in.y)[c];
+                yv[j] = v * (i < n4 ? 1.0f : 0.0f);
+                pw[j] = reinterpret_cast<const f32x4 *>(in.post_weight)[c];
+            }
+            if (in.scale) {
+#pragma unroll
+                for (int j = 0; j < NR; ++j) sc[j] = reinterpret_cast<const f32x4 *>(in.scale)[min(tid + 256 * j, n4 - 1)];
+            } else {
+#pragma unroll
+                for (int j = 0; j < NR; ++j) sc[j] = f32x4{1.f, 1.f, 1.f, 1.f};
             }
 #pragma unroll
             for (int j = 0; j < NR; ++j) ss += yv[j].x * yv[j].x + yv[j].y * yv[j].y + yv[j].z * yv[j].z + yv[j].w * yv[j].w;
@@ -238,9 +261,15 @@ __device__ void form_input(const VecIn &in, const float *x, int cols, int kp, fl
 #pragma unroll
         for (int j = 0; j < NR; ++j) {
             const int i = tid + 256 * j;
-            wv[j] = i < n4 ? reinterpret_cast<const f32x4 *>(in.weight)[i] : f32x4{0.f, 0.f, 0.f, 0.f};
-            gv[j] = in.gate && i < n4 ? reinterpret_cast<const f32x4 *>(in.gate)[i] : f32x4{1.f, 1.f, 1.f, 1.f};
+            wv[j] = reinterpret_cast<const f32x4 *>(in.weight)[min(i, n4 - 1)];
             ss += xv[j].x * xv[j].x + xv[j].y * xv[j].y + xv[j].z * xv[j].z + xv[j].w * xv[j].w;
+        }
+        if (in.gate) {
+#pragma unroll
+            for (int j = 0; j < NR; ++j) gv[j] = reinterpret_cast<const f32x4 *>(in.gate)[min(tid + 256 * j, n4 - 1)];
+        } else {
+#pragma unroll
+            for (int j = 0; j < NR; ++j) gv[j] = f32x4{1.f, 1.f, 1.f, 1.f};
         }
         const float inv = 1.0f / sqrtf(group_sum<4>(ss, slot) / (float)in.mean_n + in.eps);
 #pragma unroll
@@ -454,27 +483,29 @@ hipError_t launch_dense_gemv(const GemvArgs &a, int *n_wg_out, hipStream_t s) {
 }
 
 // ---- many-row matmul --------------------------------------------------------------------------------------------------
-// C[m][n] = act(A[m][k] . W[n][k]^T + bias).  T x T workgroup tile, four waves of T/2 x T/2, K steps of 64 columns staged in LDS by
-// LDS-DMA, ST buffers (ST - 1 steps ahead): 128 x 128 with two buffers where the launch fills the chip, 64 x 64 with four where it
-// does not and a step would wait for memory.  LDS image of a row: eight 16-byte units, unit q stored at q ^ ((row >> 1) & 7): the
-// sixteen rows of a ds_read_b128 then cover all 64 banks once.  The MFMA's A operand is the weight tile (rows = output columns n),
-// its B operand the activation tile, so a lane holds four consecutive n of one row.
+// C[m][n] = act(A[m][k] . W[n][k]^T + bias).  Workgroup tile TN x TM in WN x WM waves, K steps of 64 columns staged in LDS by LDS-DMA,
+// ST buffers.  256 x 256 in eight waves of 128 x 64 where the launch has the tiles for it (half the bytes per
+// product of 128 x 128, and a fragment read from LDS feeds four to eight MFMAs), 128 x 128, and 64 x 64 with four buffers for launches
+// that do not fill the chip and would wait for memory at every step.  LDS image of a row: eight 16-byte units, unit q stored at
+// q ^ ((row >> 1) & 7): the sixteen rows of a ds_read_b128 cover all 64 banks once.  The MFMA's A operand is the weight tile (rows =
+// output columns n), its B operand the activation tile, so a lane holds four consecutive n of one row.
 constexpr int kTileK = 64;
 
-__device__ __forceinline__ void dma1k(const void *lane_ptr, unsigned lds_dst) {
+// 64 lanes x 16 bytes from (scalar base + lane offset) to LDS bytes [lds_dst, lds_dst + 1024); invisible to hipcc's vmcnt bookkeeping
+__device__ __forceinline__ void dma1k(unsigned lane_off, const void *sbase, unsigned lds_dst) {
     unsigned keep;
-    asm volatile("s_mov_b32 %0, m0\n\ts_mov_b32 m0, %2\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %1, off\n\ts_mov_b32 m0, %0"
+    asm volatile("s_mov_b32 %0, m0\n\ts_mov_b32 m0, %3\n\ts_nop 0\n\tglobal_load_lds_dwordx4 %1, %2\n\ts_mov_b32 m0, %0"
                  : "=&s"(keep)
-                 : "v"(lane_ptr), "s"(lds_dst)
+                 : "v"(lane_off), "s"(sbase), "s"(lds_dst)
                  : "memory");
 }
 
-template <int T, int ST, bool CF32>
-__global__ __launch_bounds__(256, 2) void k_dense_gemm(GemmArgsD p, int tiles_n, int tiles_m, int swizzle) {
+template <int TN, int TM, int WN, int WM, int ST, bool CF32>
+__global__ __launch_bounds__(64 * WN * WM, 2) void k_dense_gemm(GemmArgsD p, int tiles_n, int tiles_m, int swizzle) {
     extern __shared__ __attribute__((aligned(1024))) uint8_t lds[];
-    constexpr int ND = T / 32;          // DMA instructions per wave, operand and step (eight rows each)
-    constexpr int F = T / 32;           // 16-row fragments per wave and operand
-    constexpr unsigned HALF = T * 128, BUF = 2 * HALF;
+    constexpr int NW = WN * WM, DN = TN / NW / 8, DM = TM / NW / 8;  // DMA instructions per wave and step (eight rows each)
+    constexpr int FN = TN / WN / 16, FM = TM / WM / 16;              // 16-row fragments per wave
+    constexpr unsigned ABUF = TM * 128, BUF = ABUF + TN * 128;
     const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6);
     // workgroup -> tile: consecutive workgroups land on the eight XCDs in turn; give each XCD a contiguous run of tiles, and walk
     // the tiles in groups of eight row tiles so that what runs together shares both operands in the XCD's L2
@@ -484,73 +515,93 @@ __global__ __launch_bounds__(256, 2) void k_dense_gemm(GemmArgsD p, int tiles_n,
     const int gm = 8;
     const int group = id / (gm * tiles_n), first = group * gm, size = tiles_m - first < gm ? tiles_m - first : gm;
     const int tm = first + (id % (gm * tiles_n)) % size, tn = (id % (gm * tiles_n)) / size;
-    const int m0 = tm * T, n0 = tn * T;
+    const int m0 = tm * TM, n0 = tn * TN;
     const uint16_t *A = (const uint16_t *)p.a + (size_t)blockIdx.y * p.a_batch;
     const uint16_t *W = p.w + (size_t)blockIdx.y * p.w_batch;
     const int drow = lane >> 3;
-    const uint16_t *ga[ND], *gw[ND];
+    // (lane offsets from the tile's first row: a tile spans less than 4 GiB)
+    const uint16_t *A0 = A + (size_t)m0 * p.lda, *W0 = W + (size_t)n0 * p.ldw;
+    unsigned oa[DM], ow[DN];
 #pragma unroll
-    for (int i = 0; i < ND; ++i) {
-        const int r = wave * (T / 4) + i * 8 + drow, unit = (lane & 7) ^ ((r >> 1) & 7);
-        const int ar = m0 + r < p.m ? m0 + r : p.m - 1, wr = n0 + r < p.n ? n0 + r : p.n - 1;
-        ga[i] = A + (size_t)ar * p.lda + unit * 8;
-        gw[i] = W + (size_t)wr * p.ldw + unit * 8;
+    for (int i = 0; i < DM; ++i) {
+        const int r = wave * (TM / NW) + i * 8 + drow, unit = (lane & 7) ^ ((r >> 1) & 7);
+        oa[i] = (unsigned)(min(r, p.m - 1 - m0) * p.lda + unit * 8) * 2;
+    }
+#pragma unroll
+    for (int i = 0; i < DN; ++i) {
+        const int r = wave * (TN / NW) + i * 8 + drow, unit = (lane & 7) ^ ((r >> 1) & 7);
+        ow[i] = (unsigned)(min(r, p.n - 1 - n0) * p.ldw + unit * 8) * 2;
     }
     const unsigned base = (unsigned)(uintptr_t)(__attribute__((address_space(3))) uint8_t *)lds;
     auto stage = [&](int t) {
-        const unsigned dst = base + (t % ST) * BUF + wave * (T / 4) * 128;
+        const unsigned dst = base + (t % ST) * BUF;
 #pragma unroll
-        for (int i = 0; i < ND; ++i) {
-            dma1k(ga[i] + t * kTileK, dst + i * 1024);
-            dma1k(gw[i] + t * kTileK, dst + HALF + i * 1024);
+        for (int i = 0; i < DM; ++i) dma1k(oa[i], A0 + t * kTileK, dst + wave * (TM / NW) * 128 + i * 1024);
+#pragma unroll
+        for (int i = 0; i < DN; ++i) dma1k(ow[i], W0 + t * kTileK, dst + ABUF + wave * (TN / NW) * 128 + i * 1024);
+    };
+    const int wn = (wave % WN) * (TN / WN), wm = (wave / WN) * (TM / WM);
+    const int r16 = lane & 15, g = lane >> 4, sw = (r16 >> 1) & 7;
+    f32x4 acc[FN][FM];
+#pragma unroll
+    for (int i = 0; i < FN; ++i)
+#pragma unroll
+        for (int j = 0; j < FM; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+    const int steps = p.k / kTileK;
+    // Fragments are read half a step (32 columns) ahead of the MFMAs that use them, reads and MFMAs interleaved: the middle of a step
+    // waits for the next tile, and the barrier there also says that every wave has left the tile whose buffer is requested next.
+    bf16x8 fa[2][FM], fw[2][FN];
+    auto read = [&](int t, int kk) {
+        const uint8_t *la = lds + (t % ST) * BUF, *lw = la + ABUF;
+        const int q = ((kk * 4 + g) ^ sw) * 16;
+#pragma unroll
+        for (int j = 0; j < FM; ++j) fa[kk][j] = *reinterpret_cast<const bf16x8 *>(la + (wm + j * 16 + r16) * 128 + q);
+#pragma unroll
+        for (int i = 0; i < FN; ++i) fw[kk][i] = *reinterpret_cast<const bf16x8 *>(lw + (wn + i * 16 + r16) * 128 + q);
+    };
+    auto multiply = [&](int kk) {
+#pragma unroll
+        for (int i = 0; i < FN; ++i)
+#pragma unroll
+            for (int j = 0; j < FM; ++j) acc[i][j] = mfma_bf16(fw[kk][i], fa[kk][j], acc[i][j]);
+#pragma unroll
+        for (int i = 0; i < (FN + FM) / 2; ++i) {
+            __builtin_amdgcn_sched_group_barrier(0x100, 2, 0);                         // two LDS reads
+            __builtin_amdgcn_sched_group_barrier(0x008, 2 * FN * FM / (FN + FM), 0);  // their share of the MFMAs
         }
     };
-    const int wn = (wave & 1) * (T / 2), wm = (wave >> 1) * (T / 2);
-    const int r16 = lane & 15, g = lane >> 4, sw = (r16 >> 1) & 7;
-    f32x4 acc[F][F];
 #pragma unroll
-    for (int i = 0; i < F; ++i)
-#pragma unroll
-        for (int j = 0; j < F; ++j) acc[i][j] = f32x4{0.f, 0.f, 0.f, 0.f};
-    const int steps = p.k / kTileK;
-#pragma unroll
-    for (int t = 0; t < ST - 1; ++t)
+    for (int t = 0; t < ST; ++t)
         if (t < steps) stage(t);
+    // (loads return in order: a tile is there once at most the later ones are outstanding)
+    if (steps >= ST)
+        asm volatile("s_waitcnt vmcnt(%0)" ::"n"((ST - 1) * (DM + DN)) : "memory");
+    else
+        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+    __syncthreads();
+    read(0, 0);
     for (int t = 0; t < steps; ++t) {
-        // step t's tile has landed once at most the ST - 2 later ones are outstanding (loads return in order); the barrier also says
-        // that every wave has left the buffer the next request overwrites
-        if (ST > 2 && t + ST - 2 < steps)
-            asm volatile("s_waitcnt vmcnt(%0)" ::"n"((ST - 2) * 2 * ND) : "memory");
+        read(t, 1);
+        multiply(0);
+        if (t + ST - 1 < steps)
+            asm volatile("s_waitcnt vmcnt(%0) lgkmcnt(0)" ::"n"((ST - 2) * (DM + DN)) : "memory");
         else
-            asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+            asm volatile("s_waitcnt vmcnt(0) lgkmcnt(0)" ::: "memory");
         __syncthreads();
-        if (t + ST - 1 < steps) stage(t + ST - 1);
-        const uint8_t *la = lds + (t % ST) * BUF, *lw = la + HALF;
-#pragma unroll
-        for (int kk = 0; kk < 2; ++kk) {
-            bf16x8 fa[F], fw[F];
-            const int q = ((kk * 4 + g) ^ sw) * 16;
-#pragma unroll
-            for (int i = 0; i < F; ++i) {
-                fw[i] = *reinterpret_cast<const bf16x8 *>(lw + (wn + i * 16 + r16) * 128 + q);
-                fa[i] = *reinterpret_cast<const bf16x8 *>(la + (wm + i * 16 + r16) * 128 + q);
-            }
-#pragma unroll
-            for (int i = 0; i < F; ++i)
-#pragma unroll
-                for (int j = 0; j < F; ++j) acc[i][j] = mfma_bf16(fw[i], fa[j], acc[i][j]);
-        }
+        if (t + ST < steps) stage(t + ST);
+        read(t + 1, 0);  // (behind the last step: bytes nobody uses)
+        multiply(1);
     }
     const bool vec = (p.ldc & 3) == 0;
 #pragma unroll
-    for (int i = 0; i < F; ++i) {
+    for (int i = 0; i < FN; ++i) {
         const int n = n0 + wn + i * 16 + g * 4;
         if (n >= p.n) continue;
         float bias[4];
 #pragma unroll
         for (int e = 0; e < 4; ++e) bias[e] = p.bias && n + e < p.n ? p.bias[n + e] : 0.f;
 #pragma unroll
-        for (int j = 0; j < F; ++j) {
+        for (int j = 0; j < FM; ++j) {
             const int m = m0 + wm + j * 16 + r16;
             if (m >= p.m) continue;
             float v[4];
@@ -574,11 +625,17 @@ __global__ __launch_bounds__(256, 2) void k_dense_gemm(GemmArgsD p, int tiles_n,
     }
 }
 
-template <int T, int ST>
-static void gemm_go(const GemmArgsD &a, hipStream_t s) {
+template <int T, int WN, int WM, int ST>
+static hipError_t gemm_go(const GemmArgsD &a, hipStream_t s) {
     const int tn = (a.n + T - 1) / T, tm = (a.m + T - 1) / T, swz = (tn * tm) % 8 == 0 ? 1 : 0;
-    auto fn = a.c_f32 ? k_dense_gemm<T, ST, true> : k_dense_gemm<T, ST, false>;
-    hipLaunchKernelGGL(fn, dim3(tn * tm, a.batch), dim3(256), ST * T * 256, s, a, tn, tm, swz);
+    constexpr size_t lds = (size_t)ST * T * 256;
+    auto fn = a.c_f32 ? k_dense_gemm<T, T, WN, WM, ST, true> : k_dense_gemm<T, T, WN, WM, ST, false>;
+    if (lds > 65536) {
+        const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(fn), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+        if (e != hipSuccess) return e;
+    }
+    hipLaunchKernelGGL(fn, dim3(tn * tm, a.batch), dim3(64 * WN * WM), lds, s, a, tn, tm, swz);
+    return hipGetLastError();
 }
 
 // f32 activations: f32 multiply-adds on a 64 x 64 tile, 4 x 4 per thread
@@ -633,11 +690,14 @@ hipError_t launch_dense_gemm(const GemmArgsD &args, hipStream_t s) {
         hipLaunchKernelGGL(k_dense_gemm_f32, dim3((a.n + 63) / 64, (a.m + 63) / 64, a.batch), dim3(256), 0, s, a);
         return hipGetLastError();
     }
-    if ((long)((a.n + 127) / 128) * ((a.m + 127) / 128) * a.batch >= 256)
-        gemm_go<128, 2>(a, s);
-    else
-        gemm_go<64, 4>(a, s);
-    return hipGetLastError();
+    auto tiles = [&](int t) { return (long)((a.n + t - 1) / t) * ((a.m + t - 1) / t) * a.batch; };
+    if (a.k <= 1024 && tiles(64) >= 1024) return gemm_go<64, 2, 2, 2>(a, s);  // few steps: what counts is how many workgroups overlap their ends
+    if (tiles(128) >= 200) {
+        // measured per K step: 2.05 us for a round of 256 large tiles (one per CU), 1.15 us for a round of 512 of the others (two per CU)
+        const double large = 2.05 * ((tiles(256) + 255) / 256), small = 1.15 * ((tiles(128) + 511) / 512);
+        return large <= small ? gemm_go<256, 2, 4, 2>(a, s) : gemm_go<128, 2, 2, 2>(a, s);
+    }
+    return gemm_go<64, 2, 2, 4>(a, s);
 }
 
 }  // namespace bitnet_hip

@@ -27,6 +27,13 @@ __device__ __forceinline__ float rotated(const T *q, const float *cs, const floa
     return (x * cs[c] + (a < half ? -y : y) * s) * live;
 }
 
+// (no canonicalising v_max of an MFMA result ahead of it; no NaNs here)
+__device__ __forceinline__ float max3(float a, float b, float c) {
+    float r;
+    asm("v_max3_f32 %0, %1, %2, %3" : "=v"(r) : "v"(a), "v"(b), "v"(c));
+    return r;
+}
+
 size_t latent_scratch_floats(int heads, int ldc, int nq) { return (size_t)nq * heads * kLatentSplits * (kLatentRecHead + ldc); }
 
 // ---- decode, any size -------------------------------------------------------------------------------------------------
@@ -108,6 +115,8 @@ constexpr int kDecKK = 20;  // most 32-column steps of ldc + ldr
 constexpr int kDecNT = 9;   // most 16-column tiles of ldc per wave
 constexpr int kCtStride = kLatentTile * 2 + 16;
 
+// NCK, NRK: 32-column steps of the latent and of the rotated part when known at compile time (no branches between the loads), else 0
+template <int NCK, int NRK>
 __global__ __launch_bounds__(256) void k_latent_decode(LatentAttn p) {
     extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
     __shared__ float smax[4][16], ssum[4][16];
@@ -118,30 +127,31 @@ __global__ __launch_bounds__(256) void k_latent_decode(LatentAttn p) {
     split_range(n_keys, per, used);
     if ((int)blockIdx.x >= used) return;
     const int k0 = blockIdx.x * per * kLatentTile, k1 = min(k0 + per * kLatentTile, n_keys);
-    const int kt = p.ldc + p.ldr, nkk = kt / 32, nck = p.ldc / 32, ntiles = p.ldc / 16;
+    constexpr int MKK = NCK ? NCK + NRK : kDecKK, MNT = NCK ? NCK / 2 : kDecNT;
+    const int nck = NCK ? NCK : p.ldc / 32, nkk = NCK ? NCK + NRK : nck + p.ldr / 32, kt = nkk * 32, ntiles = nck * 2, ldc = nck * 32;
     const int qs = kt * 2 + 16;  // bytes per query row
-    uint8_t *ct = lds, *qh = ct + (size_t)p.ldc * kCtStride, *ql = qh + 16 * qs, *ph = ql + 16 * qs, *pl = ph + 16 * kCtStride;
+    uint8_t *ct = lds, *qh = ct + (size_t)ldc * kCtStride, *ql = qh + 16 * qs, *ph = ql + 16 * qs, *pl = ph + 16 * kCtStride;
     const uint16_t *C = (const uint16_t *)p.ccache, *R = (const uint16_t *)p.rcache;
-    u32x4 b[kDecKK];
+    u32x4 b[MKK];
     auto fetch = [&](int key0) {
         const int key = key0 + wave * 16 + r16;  // below the capacity, a multiple of 64
 #pragma unroll
-        for (int kk = 0; kk < kDecKK; ++kk)
+        for (int kk = 0; kk < MKK; ++kk)
             if (kk < nkk)
-                b[kk] = kk < nck ? *reinterpret_cast<const u32x4 *>(C + (size_t)key * p.ldc + kk * 32 + g * 8)
+                b[kk] = kk < nck ? *reinterpret_cast<const u32x4 *>(C + (size_t)key * ldc + kk * 32 + g * 8)
                                  : *reinterpret_cast<const u32x4 *>(R + (size_t)key * p.ldr + (kk - nck) * 32 + g * 8);
     };
     fetch(k0);
     {
         // the query rows, sixteen threads each: latent part, then the rotated part
         const int half = p.rot_dim / 2, row = tid >> 4, c4 = (tid & 15) * 4, h = min(h0 + row, p.heads - 1);
-        const float *qa = p.qabs + ((size_t)qi * p.heads + h) * p.ldc + c4;
+        const float *qa = p.qabs + ((size_t)qi * p.heads + h) * ldc + c4;
         const float *qr = p.q + ((size_t)qi * p.heads + h) * p.qd + p.dimp;
         const float *cs = p.rope_cos + (size_t)pos * half, *sn = p.rope_sin + (size_t)pos * half;
-        const int n64 = p.ldc >> 6;
-        f32x4 v[kDecNT];
+        const int n64 = nck >> 1;
+        f32x4 v[MNT];
 #pragma unroll
-        for (int t = 0; t < kDecNT; ++t)
+        for (int t = 0; t < MNT; ++t)
             if (t < n64) v[t] = *reinterpret_cast<const f32x4 *>(qa + t * 64);
         auto put = [&](int i, float a, float b) {
             uint32_t hi, lo;
@@ -149,30 +159,32 @@ __global__ __launch_bounds__(256) void k_latent_decode(LatentAttn p) {
             *reinterpret_cast<uint32_t *>(qh + row * qs + i * 2) = hi;
             *reinterpret_cast<uint32_t *>(ql + row * qs + i * 2) = lo;
         };
-        for (int i = (tid & 15) * 2; i < p.ldr; i += 32) put(p.ldc + i, rotated(qr, cs, sn, half, i), rotated(qr, cs, sn, half, i + 1));
+        for (int i = (tid & 15) * 2; i < p.ldr; i += 32) put(ldc + i, rotated(qr, cs, sn, half, i), rotated(qr, cs, sn, half, i + 1));
 #pragma unroll
-        for (int t = 0; t < kDecNT; ++t)
+        for (int t = 0; t < MNT; ++t)
             if (t < n64) {
                 put(t * 64 + c4, v[t].x, v[t].y);
                 put(t * 64 + c4 + 2, v[t].z, v[t].w);
             }
     }
     __syncthreads();
-    f32x4 o[kDecNT];
+    f32x4 o[MNT];
 #pragma unroll
-    for (int t = 0; t < kDecNT; ++t) o[t] = f32x4{0.f, 0.f, 0.f, 0.f};
+    for (int t = 0; t < MNT; ++t) o[t] = f32x4{0.f, 0.f, 0.f, 0.f};
     float m[4], l[4];
 #pragma unroll
     for (int i = 0; i < 4; ++i) m[i] = -INFINITY, l[i] = 0.f;
     const bool even = (lane & 1) == 0;
     for (int key0 = k0; key0 < k1; key0 += kLatentTile) {
-        f32x4 s = f32x4{0.f, 0.f, 0.f, 0.f};
+        f32x4 s4[4];  // independent chains: high / low half of the query, even / odd step
 #pragma unroll
-        for (int kk = 0; kk < kDecKK; ++kk) {
+        for (int i = 0; i < 4; ++i) s4[i] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int kk = 0; kk < MKK; ++kk) {
             if (kk >= nkk) continue;
             const bf16x8 bv = __builtin_bit_cast(bf16x8, b[kk]);
-            s = mfma_bf16(*reinterpret_cast<const bf16x8 *>(qh + r16 * qs + kk * 64 + g * 16), bv, s);
-            s = mfma_bf16(*reinterpret_cast<const bf16x8 *>(ql + r16 * qs + kk * 64 + g * 16), bv, s);
+            s4[kk & 1] = mfma_bf16(*reinterpret_cast<const bf16x8 *>(qh + r16 * qs + kk * 64 + g * 16), bv, s4[kk & 1]);
+            s4[2 + (kk & 1)] = mfma_bf16(*reinterpret_cast<const bf16x8 *>(ql + r16 * qs + kk * 64 + g * 16), bv, s4[2 + (kk & 1)]);
             if (kk < nck) {
                 const uint32_t x0 = even ? b[kk].z : b[kk].x, x1 = even ? b[kk].w : b[kk].y;
                 const uint32_t a0 = even ? b[kk].x : b[kk].z, a1 = even ? b[kk].y : b[kk].w;
@@ -187,6 +199,7 @@ __global__ __launch_bounds__(256) void k_latent_decode(LatentAttn p) {
             }
         }
         if (key0 + kLatentTile < k1) fetch(key0 + kLatentTile);
+        f32x4 s = (s4[0] + s4[1]) + (s4[2] + s4[3]);
         const bool live = key0 + wave * 16 + r16 < k1;
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
@@ -217,7 +230,7 @@ __global__ __launch_bounds__(256) void k_latent_decode(LatentAttn p) {
             pa[ks][1] = *reinterpret_cast<const bf16x8 *>(pl + r16 * kCtStride + ks * 64 + g * 16);
         }
 #pragma unroll
-        for (int t = 0; t < kDecNT; ++t) {
+        for (int t = 0; t < MNT; ++t) {
             const int tile = t * 4 + wave;
             if (tile >= ntiles) continue;
             o[t] *= f32x4{al[0], al[1], al[2], al[3]};
@@ -238,9 +251,9 @@ __global__ __launch_bounds__(256) void k_latent_decode(LatentAttn p) {
     for (int i = 0; i < 4; ++i) {
         const int row = g * 4 + i, h = h0 + row;
         if (h >= p.heads) continue;
-        float *rec = p.scratch + (((size_t)qi * p.heads + h) * kLatentSplits + blockIdx.x) * (kLatentRecHead + p.ldc);
+        float *rec = p.scratch + (((size_t)qi * p.heads + h) * kLatentSplits + blockIdx.x) * (kLatentRecHead + ldc);
 #pragma unroll
-        for (int t = 0; t < kDecNT; ++t)
+        for (int t = 0; t < MNT; ++t)
             if (t * 4 + wave < ntiles) rec[kLatentRecHead + (t * 4 + wave) * 16 + r16] = o[t][i];
         if (wave == 0 && r16 == 0) rec[0] = m[i], rec[1] = (ssum[0][row] + ssum[1][row]) + (ssum[2][row] + ssum[3][row]);
     }
@@ -268,11 +281,12 @@ hipError_t launch_latent_decode(const LatentAttn &a, hipStream_t s) {
     const int kt = a.ldc + a.ldr;
     if (kt > 32 * kDecKK || a.ldc > 64 * kDecNT || a.ldc % 64 || a.ldr % 32) return decode_any<uint16_t>(a, dim3(splits, a.heads, a.nq), s);
     const size_t lds = (size_t)a.ldc * kCtStride + (size_t)32 * (kt * 2 + 16) + (size_t)32 * kCtStride;
+    auto fn = a.ldc == 512 && a.ldr == 64 ? k_latent_decode<16, 2> : k_latent_decode<0, 0>;
     if (lds > 65536) {
-        const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(k_latent_decode), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+        const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(fn), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
         if (e != hipSuccess) return e;
     }
-    hipLaunchKernelGGL(k_latent_decode, dim3(splits, (a.heads + 15) / 16, a.nq), dim3(256), lds, s, a);
+    hipLaunchKernelGGL(fn, dim3(splits, (a.heads + 15) / 16, a.nq), dim3(256), lds, s, a);
     return hipGetLastError();
 }
 
@@ -343,15 +357,17 @@ hipError_t launch_latent_merge(const LatentMerge &a, hipStream_t s) {
 // One workgroup: one head, 64 QT queries, four waves of 16 QT; key tiles of 64 staged through registers into LDS one step ahead.
 // NK: 32-column steps of a key (dimp + ldr), NV: 16-row tiles of V^T.
 template <int NK, int NV, int QT>
-__global__ __launch_bounds__(256, NV > 8 ? 1 : 2) void k_latent_prefill(LatentAttn p, int n_qb) {
+__global__ __launch_bounds__(256, NV > 8 ? 1 : QT == 1 ? 3 : 2) void k_latent_prefill(LatentAttn p, int n_qb) {
     extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
     constexpr int KS = NK * 64 + 16, VS = kLatentTile * 2 + 16, NVL = NV / 2;
     uint8_t *lk = lds, *lv = lds + kLatentTile * KS;
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r16 = lane & 15, g = lane >> 4;
-    // consecutive workgroups go to the eight XCDs in turn: a head's blocks stay on one of them, longest blocks first
-    const int x = blockIdx.x & 7, rest = blockIdx.x >> 3;
-    const int h = x + 8 * (rest / n_qb), qb = n_qb - 1 - rest % n_qb;
-    if (h >= p.heads) return;
+    // Consecutive workgroups go to the eight XCDs in turn.  Longest blocks first; an XCD keeps heads / 8 heads of its own (their keys
+    // and values stay in its L2), the heads left over move from XCD to XCD with the block so that all eight carry the same work.
+    const int x = blockIdx.x & 7, rest = blockIdx.x >> 3, own = p.heads >> 3, left = p.heads & 7, per = own + (left ? 1 : 0);
+    const int level = rest / per, slot = rest - level * per, r = (x + 8 * left - (level % 8) * left) & 7;
+    if (slot == own && r >= left) return;
+    const int h = slot < own ? x * own + slot : 8 * own + r, qb = n_qb - 1 - level;
     const int q0 = qb * 64 * QT, pos0 = p.n_ctx - p.nq;
     const int qw = q0 + wave * 16 * QT;  // this wave's first query
     const int half = p.rot_dim / 2;
@@ -361,6 +377,7 @@ __global__ __launch_bounds__(256, NV > 8 ? 1 : 2) void k_latent_prefill(LatentAt
     for (int t = 0; t < QT; ++t) {
         const int qi = min(qw + t * 16 + r16, p.nq - 1);
         qpos[t] = pos0 + qw + t * 16 + r16;
+        const float sign = p.scale < 0.f ? -1.0f : 1.0f;
         const uint16_t *q = (const uint16_t *)p.qb + (size_t)qi * p.heads * p.qd + (size_t)h * p.qd;
         const float *cs = p.rope_cos + (size_t)(pos0 + qi) * half, *sn = p.rope_sin + (size_t)(pos0 + qi) * half;
 #pragma unroll
@@ -368,13 +385,18 @@ __global__ __launch_bounds__(256, NV > 8 ? 1 : 2) void k_latent_prefill(LatentAt
             const int d = kk * 32 + g * 8;
             if (kk * 32 < p.dimp) {
                 qf[t][kk] = *reinterpret_cast<const bf16x8 *>(q + d);
+                if (p.scale < 0.f)
+#pragma unroll
+                    for (int e = 0; e < 8; ++e) qf[t][kk][e] = -qf[t][kk][e];
             } else {
 #pragma unroll
-                for (int e = 0; e < 8; ++e) qf[t][kk][e] = (__bf16)rotated(q + p.dimp, cs, sn, half, d + e - p.dimp);
+                for (int e = 0; e < 8; ++e) qf[t][kk][e] = (__bf16)(sign * rotated(q + p.dimp, cs, sn, half, d + e - p.dimp));
             }
         }
     }
-    const float c2 = p.scale * 1.44269504088896f, sink2 = p.sink[h] * 1.44269504088896f;
+    // scores stay unscaled up to the exponential (their maximum is then the maximum of the scaled ones: a negative scale's sign goes
+    // into the query)
+    const float c2 = fabsf(p.scale) * 1.44269504088896f, sink2 = p.sink[h] * 1.44269504088896f;
     f32x4 o[NV][QT];
     float m[QT], l[QT];
 #pragma unroll
@@ -433,30 +455,50 @@ __global__ __launch_bounds__(256, NV > 8 ? 1 : 2) void k_latent_prefill(LatentAt
                 for (int t = 0; t < QT; ++t) s[kt][t] = mfma_bf16(a, qf[t][kk], s[kt][t]);
             }
         }
-        const bool diag = key0 + kLatentTile - 1 > pos0 + qw;
-        bf16x8 ph[2][QT], pl[2][QT];
+        if (key0 + kLatentTile - 1 > pos0 + qw)  // the diagonal
+#pragma unroll
+            for (int t = 0; t < QT; ++t)
+#pragma unroll
+                for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) s[kt][t][i] = key0 + kt * 16 + g * 4 + i > qpos[t] ? -INFINITY : s[kt][t][i];
+        float mn[QT];
+        bool grows = false;
 #pragma unroll
         for (int t = 0; t < QT; ++t) {
-            float mx = -INFINITY;
+            // (hipcc does not count the wait states between an MFMA's result and inline asm that reads it)
+            asm volatile("s_nop 11" : "+v"(s[0][t]), "+v"(s[1][t]), "+v"(s[2][t]), "+v"(s[3][t]));
+            float mx = max3(s[0][t][0], s[0][t][1], s[0][t][2]);
+            mx = max3(mx, s[0][t][3], s[1][t][0]);
+            mx = max3(mx, s[1][t][1], s[1][t][2]);
+            mx = max3(mx, s[1][t][3], s[2][t][0]);
+            mx = max3(mx, s[2][t][1], s[2][t][2]);
+            mx = max3(mx, s[2][t][3], s[3][t][0]);
+            mx = max3(mx, s[3][t][1], s[3][t][2]);
+            mx = rows_max(max3(mx, s[3][t][3], -INFINITY));
+            mn[t] = fmaxf(m[t], mx * c2);
+            grows = grows || mn[t] > m[t];
+        }
+        if (__any(grows)) {
 #pragma unroll
-            for (int kt = 0; kt < 4; ++kt)
+            for (int t = 0; t < QT; ++t) {
+                const float al = __builtin_amdgcn_exp2f(m[t] - mn[t]);
+                m[t] = mn[t];
+                l[t] *= al;
 #pragma unroll
-                for (int i = 0; i < 4; ++i) {
-                    float v = s[kt][t][i] * c2;
-                    if (diag && key0 + kt * 16 + g * 4 + i > qpos[t]) v = -INFINITY;
-                    s[kt][t][i] = v;
-                    mx = fmaxf(mx, v);
-                }
-            const float mn = fmaxf(m[t], rows_max(mx)), al = __builtin_amdgcn_exp2f(m[t] - mn);
-            m[t] = mn;
-            l[t] *= al;
+                for (int v = 0; v < NV; ++v) o[v][t] *= al;
+            }
+        }
+        bf16x8 ph[2][QT], pl[2][QT];
 #pragma unroll
-            for (int ks = 0; ks < 2; ++ks) {
+        for (int ks = 0; ks < 2; ++ks)
+#pragma unroll
+            for (int t = 0; t < QT; ++t) {
                 u32x4 hi, lo;
 #pragma unroll
                 for (int j = 0; j < 4; ++j) {
                     const int kt = 2 * ks + (j >> 1), i = (j & 1) * 2;
-                    const float a = __builtin_amdgcn_exp2f(s[kt][t][i] - mn), b = __builtin_amdgcn_exp2f(s[kt][t][i + 1] - mn);
+                    const float a = __builtin_amdgcn_exp2f(fmaf(s[kt][t][i], c2, -m[t])), b = __builtin_amdgcn_exp2f(fmaf(s[kt][t][i + 1], c2, -m[t]));
                     l[t] += a + b;
                     uint32_t uh, ul;
                     split2(a, b, uh, ul);
@@ -466,9 +508,6 @@ __global__ __launch_bounds__(256, NV > 8 ? 1 : 2) void k_latent_prefill(LatentAt
                 ph[ks][t] = __builtin_bit_cast(bf16x8, hi);
                 pl[ks][t] = __builtin_bit_cast(bf16x8, lo);
             }
-#pragma unroll
-            for (int v = 0; v < NV; ++v) o[v][t] *= al;
-        }
 #pragma unroll
         for (int v = 0; v < NV; ++v)
 #pragma unroll
