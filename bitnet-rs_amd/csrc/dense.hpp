@@ -121,7 +121,7 @@ struct LinearAttn {
 
 constexpr int kLinBlock = 128;     // tokens per block of the chunked linear attention
 constexpr int kLatentTile = 64;    // keys per step of the decode attention
-constexpr int kLatentSplits = 64;  // most records per (query, head)
+constexpr int kLatentSplits = 128;  // most records per (query, head)
 constexpr int kLatentRecHead = 4;  // floats ahead of a record's vector: running maximum, sum, unused
 
 hipError_t launch_embed_bf16(const uint16_t *table, size_t ld, const int *tokens, const int *offset, int n, int width, int vocab, float *out,

@@ -295,6 +295,7 @@ hipError_t launch_latent_decode(const LatentAttn &a, hipStream_t s) {
 template <class TO>
 __global__ __launch_bounds__(512) void k_latent_merge(LatentMerge p) {
     extern __shared__ __attribute__((aligned(16))) float o[];  // [ldc], then four partial vectors
+    static_assert(kLatentSplits == 128, "two records per lane of a wave");
     __shared__ float ws[kLatentSplits], sden;
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const int h = blockIdx.x, qi = blockIdx.z;
@@ -304,11 +305,23 @@ __global__ __launch_bounds__(512) void k_latent_merge(LatentMerge p) {
     const float *rec = p.scratch + ((size_t)qi * p.heads + h) * kLatentSplits * stride;
     if (wave == 0) {
         const float sink = p.sink[h];
-        const float mv = lane < used ? rec[lane * stride] : -INFINITY, lv = lane < used ? rec[lane * stride + 1] : 0.f;
-        const float M = fmaxf(sink, rows_max(row_max(mv)));
-        const float w = lane < used ? expf(mv - M) : 0.f;
-        ws[lane] = w;
-        const float den = wave_sum(w * lv) + expf(sink - M);
+        float mv[2], lv[2], M = sink;
+#pragma unroll
+        for (int e = 0; e < 2; ++e) {
+            const int r = lane + 64 * e;
+            mv[e] = r < used ? rec[r * stride] : -INFINITY;
+            lv[e] = r < used ? rec[r * stride + 1] : 0.f;
+            M = fmaxf(M, mv[e]);
+        }
+        M = rows_max(row_max(M));
+        float den = 0.f;
+#pragma unroll
+        for (int e = 0; e < 2; ++e) {
+            const float w = lane + 64 * e < used ? expf(mv[e] - M) : 0.f;
+            ws[lane + 64 * e] = w;
+            den += w * lv[e];
+        }
+        den = wave_sum(den) + expf(sink - M);
         if (lane == 0) sden = den;
     }
     __syncthreads();

@@ -82,7 +82,14 @@ struct LinearWs {
     int nb;
 };
 
-constexpr int kTS = kLinBlock * 2 + 16;  // bytes per row of a transposed [column][token] tile
+// A transposed [column][token] tile in LDS: 256 bytes per column, its sixteen 16-byte units (eight tokens each) permuted per column so
+// that both the pair-wise writes (eight column groups at once) and the fragment reads (sixteen columns at once) cover all 64 banks.
+static_assert(kLinBlock == 128, "the tile's permutation is made for 128 tokens");
+constexpr int kTileBytes = kLinBlock * 2;
+__device__ __forceinline__ int tile_at(int col, int token) {
+    const int c = col >> 3, f = (2 * ((col ^ c) & 7)) ^ (c & 1);
+    return col * kTileBytes + ((((token >> 3) ^ f) & 15) << 4) + (token & 7) * 2;
+}
 
 // 16 bytes of row t at column c, or zero where either lies outside: the address is clamped, so loads stay unconditional
 __device__ __forceinline__ u32x4 load_or_zero(const uint16_t *m, size_t ld, int t, int n, int c, int cols) {
@@ -103,7 +110,7 @@ __device__ __forceinline__ void pair_columns(u32x4 a, u32x4 b, uint32_t out[8]) 
 // sums[block] = sum over the block's tokens t of d^(last - t) v_t k_t^T, one 64 x 64 piece per workgroup
 __global__ __launch_bounds__(256) void k_linear_sums(LinearAttn p, LinearWs w) {
     extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
-    uint8_t *lv = lds, *kh = lds + 64 * kTS, *kl = kh + 64 * kTS;
+    uint8_t *lv = lds, *kh = lds + 64 * kTileBytes, *kl = kh + 64 * kTileBytes;
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r16 = lane & 15, g = lane >> 4;
     const int blk = blockIdx.x, h = blockIdx.y, nk = (p.dimp + 63) / 64;
     const int k0 = (blockIdx.z % nk) * 64, v0 = (blockIdx.z / nk) * 64;
@@ -128,14 +135,14 @@ __global__ __launch_bounds__(256) void k_linear_sums(LinearAttn p, LinearWs w) {
         uint32_t o[8];
         pair_columns(va, vb, o);
 #pragma unroll
-        for (int e = 0; e < 8; ++e) *reinterpret_cast<uint32_t *>(lv + (c + e) * kTS + t * 2) = o[e];
+        for (int e = 0; e < 8; ++e) *reinterpret_cast<uint32_t *>(lv + tile_at(c + e, t)) = o[e];
 #pragma unroll
         for (int e = 0; e < 8; ++e) {
             const uint32_t xa = (e & 1) ? ka[e >> 1] & 0xffff0000u : ka[e >> 1] << 16, xb = (e & 1) ? kb[e >> 1] & 0xffff0000u : kb[e >> 1] << 16;
             uint32_t hi, lo;
             split2(__builtin_bit_cast(float, xa) * pa, __builtin_bit_cast(float, xb) * pb, hi, lo);
-            *reinterpret_cast<uint32_t *>(kh + (c + e) * kTS + t * 2) = hi;
-            *reinterpret_cast<uint32_t *>(kl + (c + e) * kTS + t * 2) = lo;
+            *reinterpret_cast<uint32_t *>(kh + tile_at(c + e, t)) = hi;
+            *reinterpret_cast<uint32_t *>(kl + tile_at(c + e, t)) = lo;
         }
     }
     __syncthreads();
@@ -144,11 +151,11 @@ __global__ __launch_bounds__(256) void k_linear_sums(LinearAttn p, LinearWs w) {
     for (int i = 0; i < 4; ++i) acc[i] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
     for (int ks = 0; ks < kLinBlock / 32; ++ks) {
-        const bf16x8 a = *reinterpret_cast<const bf16x8 *>(lv + (wave * 16 + r16) * kTS + ks * 64 + g * 16);
+        const bf16x8 a = *reinterpret_cast<const bf16x8 *>(lv + tile_at(wave * 16 + r16, ks * 32 + g * 8));
 #pragma unroll
         for (int i = 0; i < 4; ++i) {
-            acc[i] = mfma_bf16(a, *reinterpret_cast<const bf16x8 *>(kh + (i * 16 + r16) * kTS + ks * 64 + g * 16), acc[i]);
-            acc[i] = mfma_bf16(a, *reinterpret_cast<const bf16x8 *>(kl + (i * 16 + r16) * kTS + ks * 64 + g * 16), acc[i]);
+            acc[i] = mfma_bf16(a, *reinterpret_cast<const bf16x8 *>(kh + tile_at(i * 16 + r16, ks * 32 + g * 8)), acc[i]);
+            acc[i] = mfma_bf16(a, *reinterpret_cast<const bf16x8 *>(kl + tile_at(i * 16 + r16, ks * 32 + g * 8)), acc[i]);
         }
     }
     float *dst = w.sums + ((size_t)h * w.nb + blk) * p.vdimp * p.dimp;
@@ -186,12 +193,12 @@ __global__ __launch_bounds__(256) void k_linear_scan(LinearAttn p, LinearWs w) {
     p.state[(size_t)h * size + e] = s;
 }
 
-// o = d^(i + 1) S q_i + sum over j <= i of d^(i - j) (k_j . q_i) v_j; eight waves of 16 queries
+// o = d^(i + 1) S q_i + sum over j <= i of d^(i - j) (k_j . q_i) v_j; four waves of 32 queries
 template <int NK, int NV>
-__global__ __launch_bounds__(512) void k_linear_out(LinearAttn p, LinearWs w) {
+__global__ __launch_bounds__(256, NV > 8 ? 1 : 2) void k_linear_out(LinearAttn p, LinearWs w) {
     extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
     __shared__ float pw[kLinBlock + 1];
-    constexpr int KS = NK * 64 + 16;
+    constexpr int KS = NK * 64 + 16, QT = 2;
     uint8_t *lk = lds, *lv = lds + kLinBlock * KS;
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r16 = lane & 15, g = lane >> 4;
     const int blk = blockIdx.x, h = blockIdx.y, t0 = blk * kLinBlock, len = min(kLinBlock, p.n - t0);
@@ -199,82 +206,113 @@ __global__ __launch_bounds__(512) void k_linear_out(LinearAttn p, LinearWs w) {
     const uint16_t *V = (const uint16_t *)p.qkv + 2 * (size_t)p.heads * p.dimp + (size_t)h * p.vdimp;
     Q += (size_t)t0 * p.ld, K += (size_t)t0 * p.ld, V += (size_t)t0 * p.ld;
     if (tid <= kLinBlock) pw[tid] = p.decay_pow[(size_t)h * (kLinBlock + 1) + tid];
-    const int i = wave * 16 + r16;  // this lane's query within the block
-    bf16x8 q[NK];
+    bf16x8 q[QT][NK];
+    int qi[QT];  // this lane's queries within the block
 #pragma unroll
-    for (int kk = 0; kk < NK; ++kk) q[kk] = __builtin_bit_cast(bf16x8, load_or_zero(Q, p.ld, i, len, kk * 32 + g * 8, p.dimp));
-    {
+    for (int t = 0; t < QT; ++t) {
+        qi[t] = wave * 32 + t * 16 + r16;
+#pragma unroll
+        for (int kk = 0; kk < NK; ++kk) q[t][kk] = __builtin_bit_cast(bf16x8, load_or_zero(Q, p.ld, qi[t], len, kk * 32 + g * 8, p.dimp));
+    }
+#pragma unroll
+    for (int half = 0; half < 2; ++half) {
         u32x4 kr[NK], vr[NV / 4][2];
+        const int tk = half * 64 + (tid >> 2), tv = half * 64 + (tid >> 3) * 2;
 #pragma unroll
-        for (int j = 0; j < NK; ++j) kr[j] = load_or_zero(K, p.ld, tid >> 2, len, j * 32 + (tid & 3) * 8, p.dimp);  // four threads per token
+        for (int j = 0; j < NK; ++j) kr[j] = load_or_zero(K, p.ld, tk, len, j * 32 + (tid & 3) * 8, p.dimp);  // four threads per token
 #pragma unroll
         for (int j = 0; j < NV / 4; ++j)  // eight threads per pair of tokens
 #pragma unroll
-            for (int e = 0; e < 2; ++e) vr[j][e] = load_or_zero(V, p.ld, (tid >> 3) * 2 + e, len, j * 64 + (tid & 7) * 8, p.vdimp);
+            for (int e = 0; e < 2; ++e) vr[j][e] = load_or_zero(V, p.ld, tv + e, len, j * 64 + (tid & 7) * 8, p.vdimp);
 #pragma unroll
-        for (int j = 0; j < NK; ++j) *reinterpret_cast<u32x4 *>(lk + (tid >> 2) * KS + j * 64 + (tid & 3) * 16) = kr[j];
+        for (int j = 0; j < NK; ++j) *reinterpret_cast<u32x4 *>(lk + tk * KS + j * 64 + (tid & 3) * 16) = kr[j];
 #pragma unroll
         for (int j = 0; j < NV / 4; ++j) {
             uint32_t o[8];
             pair_columns(vr[j][0], vr[j][1], o);
 #pragma unroll
-            for (int e = 0; e < 8; ++e) *reinterpret_cast<uint32_t *>(lv + (j * 64 + (tid & 7) * 8 + e) * kTS + (tid >> 3) * 4) = o[e];
+            for (int e = 0; e < 8; ++e) *reinterpret_cast<uint32_t *>(lv + tile_at(j * 64 + (tid & 7) * 8 + e, tv)) = o[e];
         }
     }
-    f32x4 o[NV];
+    f32x4 o[NV][QT];
     const size_t sb = ((size_t)h * w.nb + blk) * p.vdimp * p.dimp;
 #pragma unroll
     for (int v = 0; v < NV; ++v) {
-        o[v] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int t = 0; t < QT; ++t) o[v][t] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int kk = 0; kk < NK; ++kk) {
             // (rows past vdimp are never stored, columns past dimp meet a zero query: clamped addresses, no branches around the loads)
             const size_t at = sb + (size_t)min(v * 16 + r16, p.vdimp - 1) * p.dimp + min(kk * 32 + g * 8, p.dimp - 8);
-            o[v] = mfma_bf16(*reinterpret_cast<const bf16x8 *>(w.hi + at), q[kk], o[v]);
-            o[v] = mfma_bf16(*reinterpret_cast<const bf16x8 *>(w.lo + at), q[kk], o[v]);
+            const bf16x8 hi = *reinterpret_cast<const bf16x8 *>(w.hi + at), lo = *reinterpret_cast<const bf16x8 *>(w.lo + at);
+#pragma unroll
+            for (int t = 0; t < QT; ++t) {
+                o[v][t] = mfma_bf16(hi, q[t][kk], o[v][t]);
+                o[v][t] = mfma_bf16(lo, q[t][kk], o[v][t]);
+            }
         }
     }
     __syncthreads();
-    const float di = pw[i + 1];
 #pragma unroll
-    for (int v = 0; v < NV; ++v) o[v] *= di;
-    if (wave * 16 < len)
-        for (int kt = 0; kt <= wave; kt += 2) {
-            f32x4 s[2];
+    for (int t = 0; t < QT; ++t) {
+        const float di = pw[qi[t] + 1];
 #pragma unroll
-            for (int j = 0; j < 2; ++j) {
-                s[j] = f32x4{0.f, 0.f, 0.f, 0.f};
+        for (int v = 0; v < NV; ++v) o[v][t] *= di;
+    }
+    for (int kt = 0; kt <= 2 * wave + 1 && kt * 16 < len; kt += 2) {
+        f32x4 s[2][QT];
 #pragma unroll
-                for (int kk = 0; kk < NK; ++kk) s[j] = mfma_bf16(*reinterpret_cast<const bf16x8 *>(lk + ((kt + j) * 16 + r16) * KS + kk * 64 + g * 16), q[kk], s[j]);
+        for (int j = 0; j < 2; ++j) {
+#pragma unroll
+            for (int t = 0; t < QT; ++t) s[j][t] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int kk = 0; kk < NK; ++kk) {
+                const bf16x8 a = *reinterpret_cast<const bf16x8 *>(lk + ((kt + j) * 16 + r16) * KS + kk * 64 + g * 16);
+#pragma unroll
+                for (int t = 0; t < QT; ++t) s[j][t] = mfma_bf16(a, q[t][kk], s[j][t]);
+            }
+        }
+        bf16x8 ph[QT], pl[QT];
+#pragma unroll
+        for (int t = 0; t < QT; ++t) {
+            u32x4 hi, lo;
+#pragma unroll
+            for (int j = 0; j < 2; ++j)
 #pragma unroll
                 for (int e = 0; e < 4; ++e) {
-                    const int back = i - ((kt + j) * 16 + g * 4 + e);
-                    s[j][e] = back >= 0 ? s[j][e] * pw[back] : 0.f;
+                    const int back = qi[t] - ((kt + j) * 16 + g * 4 + e);
+                    s[j][t][e] = back >= 0 ? s[j][t][e] * pw[max(back, 0)] : 0.f;
                 }
-            }
-            u32x4 hi, lo;
 #pragma unroll
             for (int j = 0; j < 4; ++j) {
                 uint32_t uh, ul;
-                split2(s[j >> 1][(j & 1) * 2], s[j >> 1][(j & 1) * 2 + 1], uh, ul);
+                split2(s[j >> 1][t][(j & 1) * 2], s[j >> 1][t][(j & 1) * 2 + 1], uh, ul);
                 hi[j] = uh;
                 lo[j] = ul;
             }
-            const bf16x8 ph = __builtin_bit_cast(bf16x8, hi), pl = __builtin_bit_cast(bf16x8, lo);
+            ph[t] = __builtin_bit_cast(bf16x8, hi);
+            pl[t] = __builtin_bit_cast(bf16x8, lo);
+        }
 #pragma unroll
-            for (int v = 0; v < NV; ++v) {
-                const uint8_t *row = lv + (v * 16 + r16) * kTS + kt * 32 + g * 8;
-                const u32x2 a0 = *reinterpret_cast<const u32x2 *>(row), a1 = *reinterpret_cast<const u32x2 *>(row + 32);
-                const bf16x8 a = __builtin_bit_cast(bf16x8, u32x4{a0.x, a0.y, a1.x, a1.y});
-                o[v] = mfma_bf16(a, ph, o[v]);
-                o[v] = mfma_bf16(a, pl, o[v]);
+        for (int v = 0; v < NV; ++v) {
+            const u32x2 a0 = *reinterpret_cast<const u32x2 *>(lv + tile_at(v * 16 + r16, kt * 16 + g * 4));
+            const u32x2 a1 = *reinterpret_cast<const u32x2 *>(lv + tile_at(v * 16 + r16, kt * 16 + 16 + g * 4));
+            const bf16x8 a = __builtin_bit_cast(bf16x8, u32x4{a0.x, a0.y, a1.x, a1.y});
+#pragma unroll
+            for (int t = 0; t < QT; ++t) {
+                o[v][t] = mfma_bf16(a, ph[t], o[v][t]);
+                o[v][t] = mfma_bf16(a, pl[t], o[v][t]);
             }
         }
-    if (i >= len) return;
-    float *dst = p.out + (size_t)(t0 + i) * p.ldo + (size_t)h * p.vdimp + g * 4;
+    }
 #pragma unroll
-    for (int v = 0; v < NV; ++v)
-        if (v * 16 < p.vdimp) *reinterpret_cast<f32x4 *>(dst + v * 16) = o[v];
+    for (int t = 0; t < QT; ++t) {
+        if (qi[t] >= len) continue;
+        float *dst = p.out + (size_t)(t0 + qi[t]) * p.ldo + (size_t)h * p.vdimp + g * 4;
+#pragma unroll
+        for (int v = 0; v < NV; ++v)
+            if (v * 16 < p.vdimp) *reinterpret_cast<f32x4 *>(dst + v * 16) = o[v][t];
+    }
 }
 
 static int n_blocks(int n) { return (n + kLinBlock - 1) / kLinBlock; }
@@ -283,12 +321,12 @@ bool linear_chunked_supported(int dimp, int vdimp) { return dimp % 32 == 0 && vd
 
 template <int NK, int NV>
 static hipError_t out_go(const LinearAttn &a, const LinearWs &w, hipStream_t s) {
-    const size_t lds = (size_t)kLinBlock * (NK * 64 + 16) + (size_t)NV * 16 * kTS;
+    const size_t lds = (size_t)kLinBlock * (NK * 64 + 16) + (size_t)NV * 16 * kTileBytes;
     if (lds > 65536) {
         const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(k_linear_out<NK, NV>), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
         if (e != hipSuccess) return e;
     }
-    hipLaunchKernelGGL((k_linear_out<NK, NV>), dim3(w.nb, a.heads), dim3(512), lds, s, a, w);
+    hipLaunchKernelGGL((k_linear_out<NK, NV>), dim3(w.nb, a.heads), dim3(256), lds, s, a, w);
     return hipGetLastError();
 }
 
@@ -301,7 +339,7 @@ hipError_t launch_linear_chunked(const LinearAttn &a, hipStream_t s) {
     w.hi = (uint16_t *)(w.sums + cells);
     w.lo = w.hi + cells;
     const int pieces = ((a.dimp + 63) / 64) * ((a.vdimp + 63) / 64);
-    hipLaunchKernelGGL(k_linear_sums, dim3(w.nb, a.heads, pieces), dim3(256), 3 * 64 * kTS, s, a, w);
+    hipLaunchKernelGGL(k_linear_sums, dim3(w.nb, a.heads, pieces), dim3(256), 3 * 64 * kTileBytes, s, a, w);
     hipLaunchKernelGGL(k_linear_scan, dim3((a.dimp * a.vdimp + 255) / 256, a.heads), dim3(256), 0, s, a, w);
     const int nk = a.dimp / 32, nv = a.vdimp / 16;
     if (nk <= 2) return nv <= 4 ? out_go<2, 4>(a, w, s) : nv <= 8 ? out_go<2, 8>(a, w, s) : out_go<2, 16>(a, w, s);

@@ -199,7 +199,7 @@ def test_latent_decode(hip, pkg, shape, L, f32):
 
 @pytest.mark.parametrize("f32", [True, False])
 def test_latent_decode_long_and_several_queries(hip, pkg, f32):
-    t = Latent(pkg, 4500, 3, 5, 32, 32, 32, 64, f32)  # more tiles than records
+    t = Latent(pkg, 8500, 2, 5, 32, 32, 32, 64, f32)  # more tiles than records
     t.check(t.decode(hip), 1e-5 if f32 else 1e-4)
     t = Latent(pkg, 130, 70, *SHAPES[1], f32)
     t.check(t.decode(hip), 1e-5 if f32 else 1e-4)
