@@ -894,13 +894,6 @@ class HostModel(HostSequence):
             raise BitNetHipError(ERR_INVALID_ARGUMENT, self.c.bitnet_host_open_error().decode(errors="replace"))
         self.vocab, self.width = int(self.c.bitnet_host_vocab(self.h)), int(self.c.bitnet_host_width(self.h))
 
-    def stack_probe(self, kind: int, n: int, reps: int):
-        """(microseconds, bytes, flops) of one launch of a kernel group of the stack (bench.py)."""
-        us, b, f = C.c_float(0), C.c_double(0), C.c_double(0)
-        self.c.bitnet_host_stack_probe.argtypes = [C.c_void_p, C.c_int, C.c_int, C.c_int, C.POINTER(C.c_float), C.POINTER(C.c_double), C.POINTER(C.c_double)]
-        self._check(self.c.bitnet_host_stack_probe(self.h, kind, n, reps, C.byref(us), C.byref(b), C.byref(f)))
-        return us.value, b.value, f.value
-
 
 def open_model(path: str, dtype: str = "bfloat16", max_pos: int = 4096) -> HostModel:
     return HostModel(path, dtype, max_pos)

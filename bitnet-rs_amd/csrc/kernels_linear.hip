@@ -91,11 +91,13 @@ __device__ __forceinline__ int tile_at(int col, int token) {
     return col * kTileBytes + ((((token >> 3) ^ f) & 15) << 4) + (token & 7) * 2;
 }
 
-// 16 bytes of row t at column c, or zero where either lies outside: the address is clamped, so loads stay unconditional
-__device__ __forceinline__ u32x4 load_or_zero(const uint16_t *m, size_t ld, int t, int n, int c, int cols) {
-    const u32x4 v = *reinterpret_cast<const u32x4 *>(m + (size_t)min(t, n - 1) * ld + min(c, cols - 8));
-    const bool ok = t < n && c < cols;
-    return u32x4{ok ? v.x : 0u, ok ? v.y : 0u, ok ? v.z : 0u, ok ? v.w : 0u};
+// 16 bytes of row t at column c with both clamped into the matrix (loads stay unconditional), and their clearing outside of it
+__device__ __forceinline__ u32x4 load_at(const uint16_t *m, size_t ld, int t, int n, int c, int cols) {
+    return *reinterpret_cast<const u32x4 *>(m + (size_t)min(t, n - 1) * ld + min(c, cols - 8));
+}
+__device__ __forceinline__ u32x4 zero_outside(u32x4 v, int t, int n, int c, int cols) {
+    const uint32_t keep = t < n && c < cols ? 0xffffffffu : 0u;
+    return u32x4{v.x & keep, v.y & keep, v.z & keep, v.w & keep};
 }
 
 // two tokens' eight columns -> eight (token, token + 1) dwords
@@ -122,14 +124,19 @@ __global__ __launch_bounds__(256) void k_linear_sums(LinearAttn p, LinearWs w) {
 #pragma unroll
     for (int j = 0; j < 2; ++j) {
         const int idx = tid + 256 * j, c = (idx & 7) * 8, t = (idx >> 3) * 2;
-        kv[j][0] = load_or_zero(V, p.ld, t, len, v0 + c, p.vdimp);
-        kv[j][1] = load_or_zero(V, p.ld, t + 1, len, v0 + c, p.vdimp);
-        kv[j][2] = load_or_zero(K, p.ld, t, len, k0 + c, p.dimp);
-        kv[j][3] = load_or_zero(K, p.ld, t + 1, len, k0 + c, p.dimp);
+        kv[j][0] = load_at(V, p.ld, t, len, v0 + c, p.vdimp);
+        kv[j][1] = load_at(V, p.ld, t + 1, len, v0 + c, p.vdimp);
+        kv[j][2] = load_at(K, p.ld, t, len, k0 + c, p.dimp);
+        kv[j][3] = load_at(K, p.ld, t + 1, len, k0 + c, p.dimp);
     }
+    __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
     for (int j = 0; j < 2; ++j) {
         const int idx = tid + 256 * j, c = (idx & 7) * 8, t = (idx >> 3) * 2;
+        kv[j][0] = zero_outside(kv[j][0], t, len, v0 + c, p.vdimp);
+        kv[j][1] = zero_outside(kv[j][1], t + 1, len, v0 + c, p.vdimp);
+        kv[j][2] = zero_outside(kv[j][2], t, len, k0 + c, p.dimp);
+        kv[j][3] = zero_outside(kv[j][3], t + 1, len, k0 + c, p.dimp);
         const u32x4 va = kv[j][0], vb = kv[j][1], ka = kv[j][2], kb = kv[j][3];
         const float pa = pw[max(len - 1 - t, 0)], pb = pw[max(len - 2 - t, 0)];  // (tokens past the end are zero)
         uint32_t o[8];
@@ -197,7 +204,7 @@ __global__ __launch_bounds__(256) void k_linear_scan(LinearAttn p, LinearWs w) {
 template <int NK, int NV>
 __global__ __launch_bounds__(256, NV > 8 ? 1 : 2) void k_linear_out(LinearAttn p, LinearWs w) {
     extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
-    __shared__ float pw[kLinBlock + 1];
+    __shared__ float pw[2 * kLinBlock + 1];  // [kLinBlock + i] = decay^i, zero for i < 0
     constexpr int KS = NK * 64 + 16, QT = 2;
     uint8_t *lk = lds, *lv = lds + kLinBlock * KS;
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r16 = lane & 15, g = lane >> 4;
@@ -205,25 +212,33 @@ __global__ __launch_bounds__(256, NV > 8 ? 1 : 2) void k_linear_out(LinearAttn p
     const uint16_t *Q = (const uint16_t *)p.qkv + (size_t)h * p.dimp, *K = Q + (size_t)p.heads * p.dimp;
     const uint16_t *V = (const uint16_t *)p.qkv + 2 * (size_t)p.heads * p.dimp + (size_t)h * p.vdimp;
     Q += (size_t)t0 * p.ld, K += (size_t)t0 * p.ld, V += (size_t)t0 * p.ld;
-    if (tid <= kLinBlock) pw[tid] = p.decay_pow[(size_t)h * (kLinBlock + 1) + tid];
+    if (tid <= kLinBlock) pw[kLinBlock + tid] = p.decay_pow[(size_t)h * (kLinBlock + 1) + tid];
+    if (tid < kLinBlock) pw[tid] = 0.f;
     bf16x8 q[QT][NK];
     int qi[QT];  // this lane's queries within the block
 #pragma unroll
     for (int t = 0; t < QT; ++t) {
         qi[t] = wave * 32 + t * 16 + r16;
 #pragma unroll
-        for (int kk = 0; kk < NK; ++kk) q[t][kk] = __builtin_bit_cast(bf16x8, load_or_zero(Q, p.ld, qi[t], len, kk * 32 + g * 8, p.dimp));
+        for (int kk = 0; kk < NK; ++kk) q[t][kk] = __builtin_bit_cast(bf16x8, load_at(Q, p.ld, qi[t], len, kk * 32 + g * 8, p.dimp));
     }
 #pragma unroll
     for (int half = 0; half < 2; ++half) {
         u32x4 kr[NK], vr[NV / 4][2];
         const int tk = half * 64 + (tid >> 2), tv = half * 64 + (tid >> 3) * 2;
 #pragma unroll
-        for (int j = 0; j < NK; ++j) kr[j] = load_or_zero(K, p.ld, tk, len, j * 32 + (tid & 3) * 8, p.dimp);  // four threads per token
+        for (int j = 0; j < NK; ++j) kr[j] = load_at(K, p.ld, tk, len, j * 32 + (tid & 3) * 8, p.dimp);  // four threads per token
 #pragma unroll
         for (int j = 0; j < NV / 4; ++j)  // eight threads per pair of tokens
 #pragma unroll
-            for (int e = 0; e < 2; ++e) vr[j][e] = load_or_zero(V, p.ld, tv + e, len, j * 64 + (tid & 7) * 8, p.vdimp);
+            for (int e = 0; e < 2; ++e) vr[j][e] = load_at(V, p.ld, tv + e, len, j * 64 + (tid & 7) * 8, p.vdimp);
+        __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+        for (int j = 0; j < NK; ++j) kr[j] = zero_outside(kr[j], tk, len, j * 32 + (tid & 3) * 8, p.dimp);
+#pragma unroll
+        for (int j = 0; j < NV / 4; ++j)
+#pragma unroll
+            for (int e = 0; e < 2; ++e) vr[j][e] = zero_outside(vr[j][e], tv + e, len, j * 64 + (tid & 7) * 8, p.vdimp);
 #pragma unroll
         for (int j = 0; j < NK; ++j) *reinterpret_cast<u32x4 *>(lk + tk * KS + j * 64 + (tid & 3) * 16) = kr[j];
 #pragma unroll
@@ -234,28 +249,45 @@ __global__ __launch_bounds__(256, NV > 8 ? 1 : 2) void k_linear_out(LinearAttn p
             for (int e = 0; e < 8; ++e) *reinterpret_cast<uint32_t *>(lv + tile_at(j * 64 + (tid & 7) * 8 + e, tv)) = o[e];
         }
     }
+    // The state part: a value tile's operands are requested one tile ahead (the scheduling barriers keep hipcc from moving the
+    // requests down to their uses, where each would wait for memory on its own).
+#pragma unroll
+    for (int t = 0; t < QT; ++t)
+#pragma unroll
+        for (int kk = 0; kk < NK; ++kk)
+            q[t][kk] = __builtin_bit_cast(bf16x8, zero_outside(__builtin_bit_cast(u32x4, q[t][kk]), qi[t], len, kk * 32 + g * 8, p.dimp));
     f32x4 o[NV][QT];
     const size_t sb = ((size_t)h * w.nb + blk) * p.vdimp * p.dimp;
-#pragma unroll
-    for (int v = 0; v < NV; ++v) {
-#pragma unroll
-        for (int t = 0; t < QT; ++t) o[v][t] = f32x4{0.f, 0.f, 0.f, 0.f};
+    bf16x8 hi[2][NK], lo[2][NK];
+    auto request = [&](int v) {
 #pragma unroll
         for (int kk = 0; kk < NK; ++kk) {
             // (rows past vdimp are never stored, columns past dimp meet a zero query: clamped addresses, no branches around the loads)
             const size_t at = sb + (size_t)min(v * 16 + r16, p.vdimp - 1) * p.dimp + min(kk * 32 + g * 8, p.dimp - 8);
-            const bf16x8 hi = *reinterpret_cast<const bf16x8 *>(w.hi + at), lo = *reinterpret_cast<const bf16x8 *>(w.lo + at);
+            hi[v & 1][kk] = *reinterpret_cast<const bf16x8 *>(w.hi + at);
+            lo[v & 1][kk] = *reinterpret_cast<const bf16x8 *>(w.lo + at);
+        }
+    };
+    request(0);
+#pragma unroll
+    for (int v = 0; v < NV; ++v) {
+        if (v + 1 < NV) request(v + 1);
+        __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+        for (int t = 0; t < QT; ++t) o[v][t] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int kk = 0; kk < NK; ++kk)
 #pragma unroll
             for (int t = 0; t < QT; ++t) {
-                o[v][t] = mfma_bf16(hi, q[t][kk], o[v][t]);
-                o[v][t] = mfma_bf16(lo, q[t][kk], o[v][t]);
+                o[v][t] = mfma_bf16(hi[v & 1][kk], q[t][kk], o[v][t]);
+                o[v][t] = mfma_bf16(lo[v & 1][kk], q[t][kk], o[v][t]);
             }
-        }
+        __builtin_amdgcn_sched_barrier(0);
     }
     __syncthreads();
 #pragma unroll
     for (int t = 0; t < QT; ++t) {
-        const float di = pw[qi[t] + 1];
+        const float di = pw[kLinBlock + qi[t] + 1];
 #pragma unroll
         for (int v = 0; v < NV; ++v) o[v][t] *= di;
     }
@@ -279,10 +311,7 @@ __global__ __launch_bounds__(256, NV > 8 ? 1 : 2) void k_linear_out(LinearAttn p
 #pragma unroll
             for (int j = 0; j < 2; ++j)
 #pragma unroll
-                for (int e = 0; e < 4; ++e) {
-                    const int back = qi[t] - ((kt + j) * 16 + g * 4 + e);
-                    s[j][t][e] = back >= 0 ? s[j][t][e] * pw[max(back, 0)] : 0.f;
-                }
+                for (int e = 0; e < 4; ++e) s[j][t][e] *= pw[kLinBlock + qi[t] - ((kt + j) * 16 + g * 4 + e)];
 #pragma unroll
             for (int j = 0; j < 4; ++j) {
                 uint32_t uh, ul;

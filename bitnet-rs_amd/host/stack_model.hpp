@@ -74,8 +74,6 @@ class StackModel : public Sequence {
     int forward(const int32_t *tokens, int n, const int32_t *want, int n_want, float *logits) override;
     int last_hidden(float *out) override;
     size_t weight_bytes() const override { return weight_bytes_; }
-    // mean time of one launch of a kernel group over `reps` passes of the whole stack (bench.py): see kProbe* in the source
-    int probe(int kind, int n, int reps, float *us_per_launch, double *bytes, double *flops);
 
   protected:
     bool ready() const override { return head_ != nullptr && layers_set_ == spec_.layers.size(); }
@@ -165,8 +163,3 @@ class StackModel : public Sequence {
 };
 
 }  // namespace bitnet_host
-
-extern "C" {
-// kind 0.. of StackModel::probe; n = rows (1: the single-token step's kernels)
-int bitnet_host_stack_probe(void *d, int kind, int n, int reps, float *us_per_launch, double *bytes, double *flops);
-}
