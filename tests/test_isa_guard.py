@@ -6,7 +6,7 @@ vmcnt wait of its own inside the tile loop.  hipcc
 requests, so a stray load added to the loop -- by an edit or by a new compiler's scheduling -- would turn `vmcnt(4)` into a
 race on the tiles without failing to build.  This test compiles the two prefill sources to ISA and asserts, for the
 instantiations bench.py runs:
-  * zero scratch, and the register ceilings that give two waves per SIMD (<= 256; the validated counts are 226 / 230 / 189);
+  * zero scratch, and the register ceilings that give two waves per SIMD (<= 256; the validated counts are 226 / 238 / 184);
   * in the attention tile loop: every global load / LDS-DMA and every `vmcnt` wait sits inside an inline-asm block
     (;;#ASMSTART .. ;;#ASMEND), none is compiler-emitted, no stores, no scratch traffic, and the per-iteration DMA count is
     the 8 pieces the `vmcnt(4)` arithmetic assumes (4 K pieces + 4 V^T pieces per wave and tile);
@@ -103,7 +103,7 @@ VMEM = re.compile(r"^(global_|buffer_|flat_|scratch_)")
 def test_resources_of_the_benchmarked_instantiations(isa):
     _, ua = isa["kernels_prefill_attn.hip"]
     _, ug = isa["kernels_gemm.hip"]
-    for name, usage, ceiling in ((ATTN, ua, 230), (GEMM64, ug, 232), (GEMM32, ug, 168), (GEMMF16, ug, 200), (GEMMF16_R5, ug, 224), (GEMMF16_R5_QK, ug, 208),
+    for name, usage, ceiling in ((ATTN, ua, 230), (GEMM64, ug, 240), (GEMM32, ug, 168), (GEMMF16, ug, 200), (GEMMF16_R5, ug, 224), (GEMMF16_R5_QK, ug, 208),
                                  (GEMMFP6, ug, 244), (GEMMFP6_X, ug, 232), (GEMMFP6_QB, ug, 254), (GEMMF16_QB, ug, 254)):
         u = usage[name]
         assert u["ScratchSize"] == 0, (name, u)
