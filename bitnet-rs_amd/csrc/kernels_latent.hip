@@ -122,11 +122,6 @@ __global__ __launch_bounds__(256) void k_latent_decode(LatentAttn p) {
     __shared__ float smax[4][16], ssum[4][16];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r16 = lane & 15, g = lane >> 4;
     const int h0 = blockIdx.y * 16, qi = blockIdx.z;
-    const int pos = *p.pos + p.q0 + qi, n_keys = pos + 1;
-    int per, used;
-    split_range(n_keys, per, used);
-    if ((int)blockIdx.x >= used) return;
-    const int k0 = blockIdx.x * per * kLatentTile, k1 = min(k0 + per * kLatentTile, n_keys);
     constexpr int MKK = NCK ? NCK + NRK : kDecKK, MNT = NCK ? NCK / 2 : kDecNT;
     const int nck = NCK ? NCK : p.ldc / 32, nkk = NCK ? NCK + NRK : nck + p.ldr / 32, kt = nkk * 32, ntiles = nck * 2, ldc = nck * 32;
     const int qs = kt * 2 + 16;  // bytes per query row
@@ -141,7 +136,14 @@ __global__ __launch_bounds__(256) void k_latent_decode(LatentAttn p) {
                 b[kk] = kk < nck ? *reinterpret_cast<const u32x4 *>(C + (size_t)key * ldc + kk * 32 + g * 8)
                                  : *reinterpret_cast<const u32x4 *>(R + (size_t)key * p.ldr + (kk - nck) * 32 + g * 8);
     };
-    fetch(k0);
+    // up to kLatentSplits tiles a record is one tile: requested before the position is known (any tile below the capacity may be read)
+    fetch(blockIdx.x * kLatentTile);
+    const int pos = *p.pos + p.q0 + qi, n_keys = pos + 1;
+    int per, used;
+    split_range(n_keys, per, used);
+    if ((int)blockIdx.x >= used) return;
+    const int k0 = blockIdx.x * per * kLatentTile, k1 = min(k0 + per * kLatentTile, n_keys);
+    if (per > 1) fetch(k0);
     {
         // the query rows, sixteen threads each: latent part, then the rotated part
         const int half = p.rot_dim / 2, row = tid >> 4, c4 = (tid & 15) * 4, h = min(h0 + row, p.heads - 1);
@@ -329,7 +331,7 @@ __global__ __launch_bounds__(512) void k_latent_merge(LatentMerge p) {
     const int grp = tid >> 7, t = tid & 127;
     for (int i = t * 4; i < p.ldc; i += 512) {
         f32x4 a = f32x4{0.f, 0.f, 0.f, 0.f};
-#pragma unroll 8
+#pragma unroll 16
         for (int r = grp; r < used; r += 4) a += ws[r] * *reinterpret_cast<const f32x4 *>(rec + r * stride + kLatentRecHead + i);
         *reinterpret_cast<f32x4 *>(part + grp * p.ldc + i) = a;
     }
