@@ -39,7 +39,7 @@ def main(argv=None) -> int:
         sys.path.insert(0, ROOT)
     pkg = importlib.import_module("bitnet-rs_amd")
     if not os.path.exists(pkg.LIB_PATH) or not os.path.exists(pkg.HOST_LIB_PATH):
-        pkg.build()
+        pkg._load_build_module().build()
     try:
         model = pkg.open_model(a.model, a.dtype, a.max_pos)
         print(",".join(str(t) for t in model.generate(a.tokens, a.new)))

@@ -107,34 +107,38 @@ __global__ __launch_bounds__(256) void k_latent_decode_any(LatentAttn p) {
 }
 
 // ---- decode, matrix cores ---------------------------------------------------------------------------------------------
-// One workgroup per (record, 16 heads, query), 64 keys per step.  Scores: wave w takes keys [16 w, 16 w + 16), the latent rows
-// going from memory straight into the MFMA's B operand (a lane: one key, eight columns); the f32 query is a (high, low) pair.
-// The same registers leave the tile transposed in LDS (key pairs from two neighbouring lanes), and the waves share the columns
-// of O += P C.
+// One workgroup per (record, 16 heads, query), 64 keys per step, eight waves.  Scores: wave w takes keys [16 (w & 3), + 16) and one half
+// of the columns, the rows going from memory straight into the MFMA's B operand (a lane: one key, eight columns); the f32 query is a
+// (high, low) pair.  The same registers leave the tile transposed in LDS (key pairs from two neighbouring lanes), and the waves share
+// the columns of O += P C.
 constexpr int kDecKK = 20;  // most 32-column steps of ldc + ldr
-constexpr int kDecNT = 9;   // most 16-column tiles of ldc per wave
+constexpr int kDecNT = 5;   // most 16-column tiles of ldc per wave
 constexpr int kCtStride = kLatentTile * 2 + 16;
 
 // NCK, NRK: 32-column steps of the latent and of the rotated part when known at compile time (no branches between the loads), else 0
 template <int NCK, int NRK>
-__global__ __launch_bounds__(256) void k_latent_decode(LatentAttn p) {
+__global__ __launch_bounds__(512) void k_latent_decode(LatentAttn p) {
     extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
     __shared__ float smax[4][16], ssum[4][16];
+    __shared__ f32x4 spart[4][64];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r16 = lane & 15, g = lane >> 4;
+    const int kg = wave & 3, half_cols = wave >> 2;
     const int h0 = blockIdx.y * 16, qi = blockIdx.z;
-    constexpr int MKK = NCK ? NCK + NRK : kDecKK, MNT = NCK ? NCK / 2 : kDecNT;
+    constexpr int MKK = NCK ? (NCK + NRK + 1) / 2 : kDecKK / 2, MNT = NCK ? NCK / 4 : kDecNT;
     const int nck = NCK ? NCK : p.ldc / 32, nkk = NCK ? NCK + NRK : nck + p.ldr / 32, kt = nkk * 32, ntiles = nck * 2, ldc = nck * 32;
+    const int kk0 = half_cols * ((nkk + 1) / 2), kn = half_cols ? nkk / 2 : (nkk + 1) / 2;  // this wave's steps
     const int qs = kt * 2 + 16;  // bytes per query row
     uint8_t *ct = lds, *qh = ct + (size_t)ldc * kCtStride, *ql = qh + 16 * qs, *ph = ql + 16 * qs, *pl = ph + 16 * kCtStride;
     const uint16_t *C = (const uint16_t *)p.ccache, *R = (const uint16_t *)p.rcache;
     u32x4 b[MKK];
     auto fetch = [&](int key0) {
-        const int key = key0 + wave * 16 + r16;  // below the capacity, a multiple of 64
+        const int key = key0 + kg * 16 + r16;  // below the capacity, a multiple of 64
 #pragma unroll
-        for (int kk = 0; kk < MKK; ++kk)
-            if (kk < nkk)
-                b[kk] = kk < nck ? *reinterpret_cast<const u32x4 *>(C + (size_t)key * ldc + kk * 32 + g * 8)
-                                 : *reinterpret_cast<const u32x4 *>(R + (size_t)key * p.ldr + (kk - nck) * 32 + g * 8);
+        for (int i = 0; i < MKK; ++i) {
+            const int kk = min(kk0 + i, nkk - 1);
+            const uint16_t *src = kk < nck ? C + (size_t)key * ldc + kk * 32 : R + (size_t)key * p.ldr + (kk - nck) * 32;
+            b[i] = *reinterpret_cast<const u32x4 *>(src + g * 8);
+        }
     };
     // up to kLatentSplits tiles a record is one tile: requested before the position is known (any tile below the capacity may be read)
     fetch(blockIdx.x * kLatentTile);
@@ -145,28 +149,27 @@ __global__ __launch_bounds__(256) void k_latent_decode(LatentAttn p) {
     const int k0 = blockIdx.x * per * kLatentTile, k1 = min(k0 + per * kLatentTile, n_keys);
     if (per > 1) fetch(k0);
     {
-        // the query rows, sixteen threads each: latent part, then the rotated part
-        const int half = p.rot_dim / 2, row = tid >> 4, c4 = (tid & 15) * 4, h = min(h0 + row, p.heads - 1);
-        const float *qa = p.qabs + ((size_t)qi * p.heads + h) * ldc + c4;
+        // the query rows, 32 threads each: latent part, then the rotated part
+        const int half = p.rot_dim / 2, row = tid >> 5, c4 = (tid & 31) * 4, h = min(h0 + row, p.heads - 1);
+        const float *qa = p.qabs + ((size_t)qi * p.heads + h) * ldc;
         const float *qr = p.q + ((size_t)qi * p.heads + h) * p.qd + p.dimp;
         const float *cs = p.rope_cos + (size_t)pos * half, *sn = p.rope_sin + (size_t)pos * half;
-        const int n64 = nck >> 1;
-        f32x4 v[MNT];
+        constexpr int NQ = NCK ? (NCK + 3) / 4 : kDecNT;  // 128 columns at a time
+        f32x4 v[NQ];
 #pragma unroll
-        for (int t = 0; t < MNT; ++t)
-            if (t < n64) v[t] = *reinterpret_cast<const f32x4 *>(qa + t * 64);
-        auto put = [&](int i, float a, float b) {
+        for (int t = 0; t < NQ; ++t) v[t] = *reinterpret_cast<const f32x4 *>(qa + min(t * 128 + c4, ldc - 4));
+        auto put = [&](int i, float x, float y) {
             uint32_t hi, lo;
-            split2(a, b, hi, lo);
+            split2(x, y, hi, lo);
             *reinterpret_cast<uint32_t *>(qh + row * qs + i * 2) = hi;
             *reinterpret_cast<uint32_t *>(ql + row * qs + i * 2) = lo;
         };
-        for (int i = (tid & 15) * 2; i < p.ldr; i += 32) put(ldc + i, rotated(qr, cs, sn, half, i), rotated(qr, cs, sn, half, i + 1));
+        for (int i = (tid & 31) * 2; i < p.ldr; i += 64) put(ldc + i, rotated(qr, cs, sn, half, i), rotated(qr, cs, sn, half, i + 1));
 #pragma unroll
-        for (int t = 0; t < MNT; ++t)
-            if (t < n64) {
-                put(t * 64 + c4, v[t].x, v[t].y);
-                put(t * 64 + c4 + 2, v[t].z, v[t].w);
+        for (int t = 0; t < NQ; ++t)
+            if (t * 128 + c4 < ldc) {
+                put(t * 128 + c4, v[t].x, v[t].y);
+                put(t * 128 + c4 + 2, v[t].z, v[t].w);
             }
     }
     __syncthreads();
@@ -182,18 +185,19 @@ __global__ __launch_bounds__(256) void k_latent_decode(LatentAttn p) {
 #pragma unroll
         for (int i = 0; i < 4; ++i) s4[i] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int kk = 0; kk < MKK; ++kk) {
-            if (kk >= nkk) continue;
-            const bf16x8 bv = __builtin_bit_cast(bf16x8, b[kk]);
-            s4[kk & 1] = mfma_bf16(*reinterpret_cast<const bf16x8 *>(qh + r16 * qs + kk * 64 + g * 16), bv, s4[kk & 1]);
-            s4[2 + (kk & 1)] = mfma_bf16(*reinterpret_cast<const bf16x8 *>(ql + r16 * qs + kk * 64 + g * 16), bv, s4[2 + (kk & 1)]);
+        for (int i = 0; i < MKK; ++i) {
+            if (i >= kn) continue;
+            const int kk = kk0 + i;
+            const bf16x8 bv = __builtin_bit_cast(bf16x8, b[i]);
+            s4[i & 1] = mfma_bf16(*reinterpret_cast<const bf16x8 *>(qh + r16 * qs + kk * 64 + g * 16), bv, s4[i & 1]);
+            s4[2 + (i & 1)] = mfma_bf16(*reinterpret_cast<const bf16x8 *>(ql + r16 * qs + kk * 64 + g * 16), bv, s4[2 + (i & 1)]);
             if (kk < nck) {
-                const uint32_t x0 = even ? b[kk].z : b[kk].x, x1 = even ? b[kk].w : b[kk].y;
-                const uint32_t a0 = even ? b[kk].x : b[kk].z, a1 = even ? b[kk].y : b[kk].w;
+                const uint32_t x0 = even ? b[i].z : b[i].x, x1 = even ? b[i].w : b[i].y;
+                const uint32_t a0 = even ? b[i].x : b[i].z, a1 = even ? b[i].y : b[i].w;
                 const uint32_t r0 = (uint32_t)__builtin_amdgcn_update_dpp(0, (int)x0, 0xb1, 0xf, 0xf, true);
                 const uint32_t r1 = (uint32_t)__builtin_amdgcn_update_dpp(0, (int)x1, 0xb1, 0xf, 0xf, true);
                 const uint32_t f0 = even ? a0 : r0, s0 = even ? r0 : a0, f1 = even ? a1 : r1, s1 = even ? r1 : a1;
-                uint8_t *dst = ct + (size_t)(kk * 32 + g * 8 + (even ? 0 : 4)) * kCtStride + (wave * 16 + (r16 & ~1)) * 2;
+                uint8_t *dst = ct + (size_t)(kk * 32 + g * 8 + (even ? 0 : 4)) * kCtStride + (kg * 16 + (r16 & ~1)) * 2;
                 *reinterpret_cast<uint32_t *>(dst) = __builtin_amdgcn_perm(s0, f0, 0x05040100u);
                 *reinterpret_cast<uint32_t *>(dst + kCtStride) = __builtin_amdgcn_perm(s0, f0, 0x07060302u);
                 *reinterpret_cast<uint32_t *>(dst + 2 * kCtStride) = __builtin_amdgcn_perm(s1, f1, 0x05040100u);
@@ -202,12 +206,17 @@ __global__ __launch_bounds__(256) void k_latent_decode(LatentAttn p) {
         }
         if (key0 + kLatentTile < k1) fetch(key0 + kLatentTile);
         f32x4 s = (s4[0] + s4[1]) + (s4[2] + s4[3]);
-        const bool live = key0 + wave * 16 + r16 < k1;
+        if (half_cols) spart[kg][lane] = s;
+        __syncthreads();
+        if (!half_cols) {
+            s += spart[kg][lane];
+            const bool live = key0 + kg * 16 + r16 < k1;
 #pragma unroll
-        for (int i = 0; i < 4; ++i) {
-            s[i] = live ? s[i] * p.scale : -INFINITY;
-            const float mx = row_max(s[i]);
-            if (r16 == 0) smax[wave][g * 4 + i] = mx;
+            for (int i = 0; i < 4; ++i) {
+                s[i] = live ? s[i] * p.scale : -INFINITY;
+                const float mx = row_max(s[i]);
+                if (r16 == 0) smax[kg][g * 4 + i] = mx;
+            }
         }
         __syncthreads();
         float al[4];
@@ -217,13 +226,18 @@ __global__ __launch_bounds__(256) void k_latent_decode(LatentAttn p) {
             const float mn = fmaxf(m[i], fmaxf(fmaxf(smax[0][row], smax[1][row]), fmaxf(smax[2][row], smax[3][row])));
             al[i] = expf(m[i] - mn);
             m[i] = mn;
-            const float w = expf(s[i] - mn);
-            l[i] = l[i] * al[i] + row_sum(w);
-            uint32_t hi, lo;
-            split2(w, 0.f, hi, lo);
-            *reinterpret_cast<uint16_t *>(ph + row * kCtStride + (wave * 16 + r16) * 2) = (uint16_t)hi;
-            *reinterpret_cast<uint16_t *>(pl + row * kCtStride + (wave * 16 + r16) * 2) = (uint16_t)lo;
         }
+        if (!half_cols)
+#pragma unroll
+            for (int i = 0; i < 4; ++i) {
+                const int row = g * 4 + i;
+                const float w = expf(s[i] - m[i]);
+                l[i] = l[i] * al[i] + row_sum(w);
+                uint32_t hi, lo;
+                split2(w, 0.f, hi, lo);
+                *reinterpret_cast<uint16_t *>(ph + row * kCtStride + (kg * 16 + r16) * 2) = (uint16_t)hi;
+                *reinterpret_cast<uint16_t *>(pl + row * kCtStride + (kg * 16 + r16) * 2) = (uint16_t)lo;
+            }
         __syncthreads();
         bf16x8 pa[2][2];
 #pragma unroll
@@ -233,7 +247,7 @@ __global__ __launch_bounds__(256) void k_latent_decode(LatentAttn p) {
         }
 #pragma unroll
         for (int t = 0; t < MNT; ++t) {
-            const int tile = t * 4 + wave;
+            const int tile = t * 8 + wave;
             if (tile >= ntiles) continue;
             o[t] *= f32x4{al[0], al[1], al[2], al[3]};
 #pragma unroll
@@ -245,9 +259,9 @@ __global__ __launch_bounds__(256) void k_latent_decode(LatentAttn p) {
         }
         __syncthreads();
     }
-    if (r16 == 0)
+    if (!half_cols && r16 == 0)
 #pragma unroll
-        for (int i = 0; i < 4; ++i) ssum[wave][g * 4 + i] = l[i];
+        for (int i = 0; i < 4; ++i) ssum[kg][g * 4 + i] = l[i];
     __syncthreads();
 #pragma unroll
     for (int i = 0; i < 4; ++i) {
@@ -256,7 +270,7 @@ __global__ __launch_bounds__(256) void k_latent_decode(LatentAttn p) {
         float *rec = p.scratch + (((size_t)qi * p.heads + h) * kLatentSplits + blockIdx.x) * (kLatentRecHead + ldc);
 #pragma unroll
         for (int t = 0; t < MNT; ++t)
-            if (t * 4 + wave < ntiles) rec[kLatentRecHead + (t * 4 + wave) * 16 + r16] = o[t][i];
+            if (t * 8 + wave < ntiles) rec[kLatentRecHead + (t * 8 + wave) * 16 + r16] = o[t][i];
         if (wave == 0 && r16 == 0) rec[0] = m[i], rec[1] = (ssum[0][row] + ssum[1][row]) + (ssum[2][row] + ssum[3][row]);
     }
 }
@@ -281,14 +295,14 @@ hipError_t launch_latent_decode(const LatentAttn &a, hipStream_t s) {
     const int splits = min(kLatentSplits, (a.capacity + kLatentTile - 1) / kLatentTile);
     if (a.f32) return decode_any<float>(a, dim3(splits, a.heads, a.nq), s);
     const int kt = a.ldc + a.ldr;
-    if (kt > 32 * kDecKK || a.ldc > 64 * kDecNT || a.ldc % 64 || a.ldr % 32) return decode_any<uint16_t>(a, dim3(splits, a.heads, a.nq), s);
+    if (kt > 32 * kDecKK || a.ldc > 128 * kDecNT || a.ldc % 64 || a.ldr % 32) return decode_any<uint16_t>(a, dim3(splits, a.heads, a.nq), s);
     const size_t lds = (size_t)a.ldc * kCtStride + (size_t)32 * (kt * 2 + 16) + (size_t)32 * kCtStride;
     auto fn = a.ldc == 512 && a.ldr == 64 ? k_latent_decode<16, 2> : k_latent_decode<0, 0>;
     if (lds > 65536) {
         const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(fn), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
         if (e != hipSuccess) return e;
     }
-    hipLaunchKernelGGL(fn, dim3(splits, (a.heads + 15) / 16, a.nq), dim3(256), lds, s, a);
+    hipLaunchKernelGGL(fn, dim3(splits, (a.heads + 15) / 16, a.nq), dim3(512), lds, s, a);
     return hipGetLastError();
 }
 

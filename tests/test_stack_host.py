@@ -14,7 +14,7 @@ from tests import stack_util as u
 
 @pytest.fixture(scope="module")
 def built(pkg):
-    pkg.build()
+    pkg._load_build_module().build()
     return pkg
 
 
