@@ -487,8 +487,11 @@ hipError_t launch_dense_gemv(const GemvArgs &a, int *n_wg_out, hipStream_t s) {
 // ST buffers.  256 x 256 in eight waves of 128 x 64 where the launch has the tiles for it (half the bytes per
 // product of 128 x 128, and a fragment read from LDS feeds four to eight MFMAs), 128 x 128, and 64 x 64 with four buffers for launches
 // that do not fill the chip and would wait for memory at every step.  LDS image of a row: eight 16-byte units, unit q stored at
-// q ^ ((row >> 1) & 7): the sixteen rows of a ds_read_b128 cover all 64 banks once.  The MFMA's A operand is the weight tile (rows =
-// output columns n), its B operand the activation tile, so a lane holds four consecutive n of one row.
+// q ^ ((row >> 1) & 7) (activations) or q ^ weight_key(row) (weights): the sixteen rows of a ds_read_b128 cover all 64 banks once.  The
+// MFMA's A operand is the weight tile (rows = output columns n), its B operand the activation tile; for bf16
+// outputs row r of weight fragment i is column 4 FN (r / 4) + 4 i + r % 4 of the wave's tile, so that a lane ends up with 4 FN consecutive
+// columns of one output row (stores of 32-byte pieces cost more than the arithmetic of a short product); f32 outputs keep 16 i + r, four
+// lanes of 16 bytes side by side.
 constexpr int kTileK = 64;
 
 // 64 lanes x 16 bytes from (scalar base + lane offset) to LDS bytes [lds_dst, lds_dst + 1024); invisible to hipcc's vmcnt bookkeeping
@@ -498,6 +501,11 @@ __device__ __forceinline__ void dma1k(unsigned lane_off, const void *sbase, unsi
                  : "=&s"(keep)
                  : "v"(lane_off), "s"(sbase), "s"(lds_dst)
                  : "memory");
+}
+
+template <int FN, bool CF32>
+__device__ __forceinline__ int weight_key(int row) {
+    return CF32 ? (row >> 1) & 7 : ((row / (4 * FN)) & 3) * 2 + ((row >> 1) & 1);
 }
 
 template <int TN, int TM, int WN, int WM, int ST, bool CF32>
@@ -519,18 +527,19 @@ __global__ __launch_bounds__(64 * WN * WM, 2) void k_dense_gemm(GemmArgsD p, int
     const uint16_t *A = (const uint16_t *)p.a + (size_t)blockIdx.y * p.a_batch;
     const uint16_t *W = p.w + (size_t)blockIdx.y * p.w_batch;
     const int drow = lane >> 3;
-    // (lane offsets from the tile's first row: a tile spans less than 4 GiB)
+    // (lane offsets from the tile's first row: a tile spans less than 4 GiB; rows past the end read the tile's own rows over again)
+    const unsigned rows_m = min(TM, p.m - m0), rows_n = min(TN, p.n - n0);
     const uint16_t *A0 = A + (size_t)m0 * p.lda, *W0 = W + (size_t)n0 * p.ldw;
     unsigned oa[DM], ow[DN];
 #pragma unroll
     for (int i = 0; i < DM; ++i) {
         const int r = wave * (TM / NW) + i * 8 + drow, unit = (lane & 7) ^ ((r >> 1) & 7);
-        oa[i] = (unsigned)(min(r, p.m - 1 - m0) * p.lda + unit * 8) * 2;
+        oa[i] = (unsigned)((unsigned)r % rows_m * p.lda + unit * 8) * 2;
     }
 #pragma unroll
     for (int i = 0; i < DN; ++i) {
-        const int r = wave * (TN / NW) + i * 8 + drow, unit = (lane & 7) ^ ((r >> 1) & 7);
-        ow[i] = (unsigned)(min(r, p.n - 1 - n0) * p.ldw + unit * 8) * 2;
+        const int r = wave * (TN / NW) + i * 8 + drow, unit = (lane & 7) ^ weight_key<FN, CF32>(r);
+        ow[i] = (unsigned)((unsigned)r % rows_n * p.ldw + unit * 8) * 2;
     }
     const unsigned base = (unsigned)(uintptr_t)(__attribute__((address_space(3))) uint8_t *)lds;
     auto stage = [&](int t) {
@@ -542,6 +551,8 @@ __global__ __launch_bounds__(64 * WN * WM, 2) void k_dense_gemm(GemmArgsD p, int
     };
     const int wn = (wave % WN) * (TN / WN), wm = (wave / WN) * (TM / WM);
     const int r16 = lane & 15, g = lane >> 4, sw = (r16 >> 1) & 7;
+    constexpr int FS = CF32 ? 16 : 4;  // columns between fragments; neither step changes a row's key: one for all fragments
+    const int wr = CF32 ? wn + r16 : wn + (r16 >> 2) * 4 * FN + (r16 & 3);
     f32x4 acc[FN][FM];
 #pragma unroll
     for (int i = 0; i < FN; ++i)
@@ -553,11 +564,11 @@ __global__ __launch_bounds__(64 * WN * WM, 2) void k_dense_gemm(GemmArgsD p, int
     bf16x8 fa[2][FM], fw[2][FN];
     auto read = [&](int t, int kk) {
         const uint8_t *la = lds + (t % ST) * BUF, *lw = la + ABUF;
-        const int q = ((kk * 4 + g) ^ sw) * 16;
+        const int q = ((kk * 4 + g) ^ sw) * 16, qw = ((kk * 4 + g) ^ weight_key<FN, CF32>(wr)) * 16;
 #pragma unroll
         for (int j = 0; j < FM; ++j) fa[kk][j] = *reinterpret_cast<const bf16x8 *>(la + (wm + j * 16 + r16) * 128 + q);
 #pragma unroll
-        for (int i = 0; i < FN; ++i) fw[kk][i] = *reinterpret_cast<const bf16x8 *>(lw + (wn + i * 16 + r16) * 128 + q);
+        for (int i = 0; i < FN; ++i) fw[kk][i] = *reinterpret_cast<const bf16x8 *>(lw + (wr + i * FS) * 128 + qw);
     };
     auto multiply = [&](int kk) {
 #pragma unroll
@@ -592,33 +603,64 @@ __global__ __launch_bounds__(64 * WN * WM, 2) void k_dense_gemm(GemmArgsD p, int
         read(t + 1, 0);  // (behind the last step: bytes nobody uses)
         multiply(1);
     }
-    const bool vec = (p.ldc & 3) == 0;
+    // this lane's columns: nl + i * FS + e
+    const int nl = n0 + wn + g * (CF32 ? 4 : 4 * FN), nlast = nl + (FN - 1) * FS + 3;
+    const bool vec = (p.ldc & 7) == 0 && (p.c_batch & 7) == 0 && ((uintptr_t)p.c & 15) == 0;
+    // the activation: one for the whole wave unless the split runs through its columns
+    const int mine = nlast < p.act_split ? p.act0 : nl >= p.act_split ? p.act1 : -1, act0 = __builtin_amdgcn_readfirstlane(mine);
+    const int act = __all(mine == act0) ? act0 : -1;
 #pragma unroll
-    for (int i = 0; i < FN; ++i) {
-        const int n = n0 + wn + i * 16 + g * 4;
-        if (n >= p.n) continue;
-        float bias[4];
+    for (int j = 0; j < FM; ++j) {
+        const int m = m0 + wm + j * 16 + r16;
+        if (m >= p.m) continue;
+        const size_t o = (size_t)blockIdx.y * p.c_batch + (size_t)m * p.ldc + nl;
+        if (p.bias)
 #pragma unroll
-        for (int e = 0; e < 4; ++e) bias[e] = p.bias && n + e < p.n ? p.bias[n + e] : 0.f;
+            for (int i = 0; i < FN; ++i)
 #pragma unroll
-        for (int j = 0; j < FM; ++j) {
-            const int m = m0 + wm + j * 16 + r16;
-            if (m >= p.m) continue;
-            float v[4];
+                for (int e = 0; e < 4; ++e) acc[i][j][e] += p.bias[min(nl + i * FS + e, p.n - 1)];
+        auto apply = [&](auto f) {
 #pragma unroll
-            for (int e = 0; e < 4; ++e) v[e] = activate(acc[i][j][e] + bias[e], n + e < p.act_split ? p.act0 : p.act1);
-            const size_t o = (size_t)blockIdx.y * p.c_batch + (size_t)m * p.ldc + n;
-            if (vec && n + 3 < p.n) {
-                if (CF32)
-                    *reinterpret_cast<f32x4 *>((float *)p.c + o) = f32x4{v[0], v[1], v[2], v[3]};
-                else
-                    *reinterpret_cast<bf16x4 *>((uint16_t *)p.c + o) = bf16x4{(__bf16)v[0], (__bf16)v[1], (__bf16)v[2], (__bf16)v[3]};
-            } else {
-                for (int e = 0; e < 4 && n + e < p.n; ++e) {
-                    if (CF32)
-                        ((float *)p.c)[o + e] = v[e];
-                    else
-                        ((uint16_t *)p.c)[o + e] = f2bf(v[e]);
+            for (int i = 0; i < FN; ++i)
+#pragma unroll
+                for (int e = 0; e < 4; ++e) acc[i][j][e] = f(acc[i][j][e], nl + i * FS + e);
+        };
+        if (act < 0)
+            apply([&](float v, int n) {
+                const int f = n < p.act_split ? p.act0 : p.act1;
+                const float sg = __builtin_amdgcn_rcpf(1.0f + __expf(-v)), r = fmaxf(v, 0.0f);
+                return f == BITNET_HIP_ACT_SILU ? v * sg : f == BITNET_HIP_ACT_SIGMOID ? sg : f == BITNET_HIP_ACT_RELU2 ? r * r : v;
+            });
+        else if (act == BITNET_HIP_ACT_SILU)
+            apply([](float v, int) { return v * __builtin_amdgcn_rcpf(1.0f + __expf(-v)); });
+        else if (act == BITNET_HIP_ACT_SIGMOID)
+            apply([](float v, int) { return __builtin_amdgcn_rcpf(1.0f + __expf(-v)); });
+        else if (act == BITNET_HIP_ACT_RELU2)
+            apply([](float v, int) { return activate(v, BITNET_HIP_ACT_RELU2); });
+        if (CF32) {
+#pragma unroll
+            for (int i = 0; i < FN; ++i) {
+                float *dst = (float *)p.c + o + i * FS;
+                if (vec && nl + i * FS + 3 < p.n) {
+                    *reinterpret_cast<f32x4 *>(dst) = acc[i][j];
+                } else {
+#pragma unroll
+                    for (int e = 0; e < 4; ++e)
+                        if (nl + i * FS + e < p.n) dst[e] = acc[i][j][e];
+                }
+            }
+        } else {
+#pragma unroll
+            for (int i = 0; i < FN; i += 2) {
+                uint16_t *dst = (uint16_t *)p.c + o + i * FS;
+                if (vec && nl + i * FS + 7 < p.n) {
+                    *reinterpret_cast<bf16x8 *>(dst) =
+                        bf16x8{(__bf16)acc[i][j][0],     (__bf16)acc[i][j][1],     (__bf16)acc[i][j][2],     (__bf16)acc[i][j][3],
+                               (__bf16)acc[i + 1][j][0], (__bf16)acc[i + 1][j][1], (__bf16)acc[i + 1][j][2], (__bf16)acc[i + 1][j][3]};
+                } else {
+#pragma unroll
+                    for (int e = 0; e < 8; ++e)
+                        if (nl + i * FS + e < p.n) dst[e] = f2bf(acc[i + (e >> 2)][j][e & 3]);
                 }
             }
         }
@@ -693,8 +735,9 @@ hipError_t launch_dense_gemm(const GemmArgsD &args, hipStream_t s) {
     auto tiles = [&](int t) { return (long)((a.n + t - 1) / t) * ((a.m + t - 1) / t) * a.batch; };
     if (a.k <= 1024 && tiles(64) >= 1024) return gemm_go<64, 2, 2, 2>(a, s);  // few steps: what counts is how many workgroups overlap their ends
     if (tiles(128) >= 200) {
-        // measured per K step: 2.05 us for a round of 256 large tiles (one per CU), 1.15 us for a round of 512 of the others (two per CU)
-        const double large = 2.05 * ((tiles(256) + 255) / 256), small = 1.15 * ((tiles(128) + 511) / 512);
+        // measured per K step: 2.05 us for a round of 256 large tiles (one per CU), 1.15 us for a round of 512 of the others (two per CU);
+        // a column tile of the large kind that sticks out over the last column costs a third more
+        const double large = (a.n % 256 ? 2.7 : 2.05) * ((tiles(256) + 255) / 256), small = 1.15 * ((tiles(128) + 511) / 512);
         return large <= small ? gemm_go<256, 2, 4, 2>(a, s) : gemm_go<128, 2, 2, 2>(a, s);
     }
     return gemm_go<64, 2, 2, 4>(a, s);
