@@ -464,7 +464,7 @@ hipError_t launch_dense_gemv(const GemvArgs &a, int *n_wg_out, hipStream_t s) {
     else if (wgs(2) >= 512) r = 2;
     k.groups = (a.rows + per * r - 1) / (per * r);
     int n_wg = (k.groups + 3) / 4;
-    const int cap = 1024;  // four workgroups per CU
+    const int cap = 768;  // three workgroups per CU: each forms the whole input again (measured: 512 and 1024 are slower)
     if (a.batch == 1 && n_wg > cap) {
         const int rounds = (n_wg + cap - 1) / cap;
         n_wg = (n_wg + rounds - 1) / rounds;
