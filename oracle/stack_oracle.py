@@ -28,6 +28,11 @@ def norm_around_zero(x, w, eps):
     return rms_divide(x, eps) * (1.0 + w)
 
 
+def layer_norm(x, w, b, eps):
+    d = x - np.mean(x, axis=-1, keepdims=True)
+    return d / np.sqrt(np.mean(d * d, axis=-1, keepdims=True) + eps) * w + b
+
+
 # ---- activations -----------------------------------------------------------------------------------------------------
 def silu(z):
     return z / (1.0 + np.exp(-z))
@@ -39,6 +44,10 @@ def sigmoid(z):
 
 def relu_squared(z):
     return np.maximum(z, 0.0) ** 2
+
+
+def softplus(z):
+    return np.maximum(z, 0.0) + np.log1p(np.exp(-np.abs(z)))
 
 
 # ---- rotary positions ------------------------------------------------------------------------------------------------
@@ -116,16 +125,129 @@ def lightning(h, t, p, m, eps):
     return y @ t[p + "o"].T
 
 
+def query_temperature(p, m):
+    s = m["q_temp"]
+    return 1.0 + s["coef"] * math.log(math.floor((p + 1) / s["every"]) + 1.0)
+
+
+def differential_attention(h, t, p, m, eps):
+    """two softmax maps per head over the same values; the second, weighted, is taken from the first"""
+    n, H, G, D, V = len(h), m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+    q = norm_plain((h @ t[p + "q"].T).reshape(n, H, 2, D), t[p + "q.norm"], eps)
+    k = norm_plain((h @ t[p + "k"].T).reshape(n, G, 2, D), t[p + "k.norm"], eps)
+    v = (h @ t[p + "v"].T).reshape(n, G, V)
+    lam = math.exp(t[p + "lq1"] @ t[p + "lk1"]) - math.exp(t[p + "lq2"] @ t[p + "lk2"]) + m["diff"]
+    temp = np.array([query_temperature(i, m) for i in range(n)])
+    out = np.zeros((n, H, V), F)
+    for a in range(H):
+        g = a // (H // G)
+        maps = []
+        for j in range(2):
+            s = (q[:, a, j] * temp[:, None]) @ k[:, g, j].T * m["scale"]
+            s[np.triu_indices(n, 1)] = -np.inf
+            e = np.exp(s - s.max(axis=1, keepdims=True))
+            maps.append(e / e.sum(axis=1, keepdims=True) @ v[:, g])
+        out[:, a] = rms_divide(maps[0] - lam * maps[1], eps) * (1.0 - m["diff"])
+    return out.reshape(n, H * V) @ t[p + "o"].T
+
+
+def short_convolution(x, w):
+    """x [tokens, channels], w [channels, taps]: the last tap meets the current token, zeros stand ahead of the first"""
+    taps = w.shape[1]
+    out = np.zeros_like(x)
+    for i in range(len(x)):
+        for j in range(taps):
+            if i - (taps - 1 - j) >= 0:
+                out[i] += w[:, j] * x[i - (taps - 1 - j)]
+    return out
+
+
+def unit(x):
+    return x / np.sqrt(np.sum(x * x, axis=-1, keepdims=True) + 1e-6)
+
+
+def gated_delta(h, t, p, m, eps):
+    n, H, G, D, V = len(h), m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+    q, k, v = (silu(short_convolution(h @ t[p + x].T, t[p + x + ".conv"])) for x in "qkv")
+    q, k, v = unit(q.reshape(n, G, D)) * D ** -0.5, unit(k.reshape(n, G, D)), v.reshape(n, H, V)
+    beta = sigmoid(h @ t[p + "b"].T)
+    decay = np.exp(-np.exp(t[p + "A_log"]) * softplus(h @ t[p + "a"].T + t[p + "dt_bias"]))
+    o = np.zeros((n, H, V), F)
+    for a in range(H):
+        g = a // (H // G)
+        S = np.zeros((D, V), F)
+        for i in range(n):
+            S = decay[i, a] * S
+            S = S + np.outer(k[i, g], beta[i, a] * (v[i, a] - S.T @ k[i, g]))
+            o[i, a] = S.T @ q[i, g]
+    y = norm_plain(o, t[p + "norm"], eps).reshape(n, H * V) * silu(h @ t[p + "g"].T)
+    return y @ t[p + "o"].T
+
+
 # ---- feed-forward ----------------------------------------------------------------------------------------------------
 def dense_mlp(h, t, p):
     z = relu_squared(h @ t[p + "up"].T + t[p + "up.b"])
     return z @ t[p + "down"].T + t[p + "down.b"]
 
 
+def expert(h, t, p):
+    return relu_squared(h @ t[p + "up"].T) @ t[p + "down"].T
+
+
+def route(h, router, top, scale):
+    """per token: the chosen experts (largest score first) and their weights"""
+    z = h @ router.T
+    s = np.exp(z - z.max(axis=1, keepdims=True))
+    s /= s.sum(axis=1, keepdims=True)
+    ids = np.argsort(-s, axis=1, kind="stable")[:, :top]
+    w = np.take_along_axis(s, ids, 1)
+    return ids, w / (w.sum(axis=1, keepdims=True) + 1e-20) * scale
+
+
+def expert_mlp(h, t, p, f):
+    r = f["router"]
+    ids, w = route(h, t[p + "router"], r["top"], r["scale"])
+    out = expert(h, t, p + "shared.") if f.get("shared") else np.zeros_like(h)
+    for i in range(len(h)):
+        for e, x in zip(ids[i], w[i]):
+            out[i] += x * expert(h[i:i + 1], t, p + f"e{e}.")[0]
+    return out
+
+
 # ---- the stack -------------------------------------------------------------------------------------------------------
 def forward(config, tensors, tokens):
-    """(logits [n, vocab], residual stream after every layer [layers, n, width])"""
+    """(logits [n, vocab], residual stream after every layer run [runs, n, width])"""
     t = {k: np.asarray(v, F) for k, v in tensors.items()}
+    return {"Lasapel": forward_lasapel, "Mimolix": forward_mimolix}[config["architecture"]](config, t, tokens)
+
+
+def layer_runs(config):
+    """(layer, first of a pass) in the order they run"""
+    n, loop = len(config["layers"]), config.get("loop")
+    if not loop:
+        return [(i, False) for i in range(n)]
+    body = [(i, i == loop["start"]) for i in range(loop["start"], loop["stop"])]
+    return [(i, False) for i in range(loop["start"])] + body * loop["times"] + [(i, False) for i in range(loop["stop"], n)]
+
+
+def forward_mimolix(config, t, tokens):
+    eps, mult = config["norm"]["eps"], config["residual_mult"]
+    x0 = t["embed"][np.asarray(tokens)] * config["embedding"]["scale"]
+    x, after = x0, []
+    for i, enters in layer_runs(config):
+        p, layer = f"l{i}.", config["layers"][i]
+        if enters:
+            x = np.concatenate([x, x0], axis=1) @ t["loop.in"].T
+        h = layer_norm(x, t[p + "norm1"], t[p + "norm1.b"], eps)
+        y = {"attention": differential_attention, "delta": gated_delta}[layer["type"]](h, t, p + "mix.", layer["mixer"], eps)
+        if layer.get("mlp"):
+            y = y + expert_mlp(h, t, p + "mlp.", layer["mlp"])
+        x = x + mult * y
+        after.append(x)
+    return layer_norm(x, t["final.norm"], t["final.norm.b"], eps) @ t["head"].T, np.stack(after)
+
+
+def forward_lasapel(config, t, tokens):
     eps = config["norm"]["eps"]
     x = t["embed"][np.asarray(tokens)]
     after, latents = [], {}
