@@ -96,13 +96,36 @@ def _addr(t):
 
 
 ACT_NONE, ACT_SILU, ACT_SIGMOID, ACT_RELU2 = 0, 1, 2, 3
-IN_PLAIN, IN_NORM, IN_RESIDUAL_NORM = 0, 1, 2
+IN_PLAIN, IN_NORM, IN_RESIDUAL_NORM, IN_CONCAT = 0, 1, 2, 3
 LINEAR_BLOCK = 128
 
 
 class VectorInput(C.Structure):
     _fields_ = [("x", _vp), ("kind", C.c_int32), ("eps", C.c_float), ("weight_offset", C.c_float), ("weight", _vp), ("y", _vp), ("post_weight", _vp),
-                ("scale", _vp), ("gate", _vp), ("x_out", _vp), ("n", C.c_int32), ("mean_n", C.c_int32)]
+                ("scale", _vp), ("gate", _vp), ("x_out", _vp), ("n", C.c_int32), ("mean_n", C.c_int32),
+                ("mult", C.c_float), ("center", C.c_int32), ("bias", _vp), ("x2", _vp), ("h_out", _vp)]
+
+
+class SumRows(C.Structure):
+    _fields_ = [("x", _vp), ("m", _sz), ("width", _sz), ("y", _vp), ("ldy", _sz), ("mult", C.c_float), ("expert_rows", _vp), ("ld_expert", _sz), ("top", _sz),
+                ("slots", _vp), ("slot_weights", _vp), ("weight", _vp), ("bias", _vp), ("x2", _vp), ("weight_offset", C.c_float), ("eps", C.c_float),
+                ("center", C.c_int32), ("h_f32", C.c_int32), ("h", _vp), ("ldh", _sz)]
+
+
+class Gqa(C.Structure):
+    _fields_ = [(n, _sz) for n in ("heads", "kv_heads", "maps", "dim", "dimp", "vdim", "vdimp", "capacity")] + [
+        ("eps", C.c_float), ("lam", C.c_float), ("out_scale", C.c_float), ("q_weight", _vp), ("k_weight", _vp), ("q_factor", _vp), ("kcache", _vp), ("vcache", _vp)]
+
+
+class Delta(C.Structure):
+    _fields_ = [(n, _sz) for n in ("heads", "kv_heads", "dim", "dimp", "vdim", "vdimp", "taps")] + [
+        ("conv", _vp), ("decay_rate", _vp), ("dt_bias", _vp), ("norm", _vp), ("q_scale", C.c_float), ("unit_eps", C.c_float), ("eps", C.c_float), ("state", _vp),
+        ("ring", _vp)]
+
+
+class ExpertsPlan(C.Structure):
+    _fields_ = [(n, _vp) for n in ("counts", "offsets", "n_tiles", "tiles", "ids", "slots", "tokens", "weights")] + [
+        (n, _sz) for n in ("m", "experts", "top", "tile", "max_tiles")]
 
 
 class LatentRows(C.Structure):
@@ -554,8 +577,76 @@ class HipLib:
         self._check(self.c.bitnet_hip_argmax_dev(_ptr(v), n, _ptr(scratch), n_wg, _ptr(token), _vp(stream)))
 
     # -- bf16-weight operators and sequence mixers (include/bitnet_hip.h section 5) -----------------------------
-    def embed_bf16_dev(self, table, ld: int, tokens, out, n: int, width: int, vocab: int, offset=None, stream: int = 0) -> None:
-        self._call("embed_bf16_dev", _ptr(table), _sz(ld), _ptr(tokens), _optr(offset), _sz(n), _sz(width), _sz(vocab), _ptr(out), _vp(stream))
+    def embed_bf16_dev(self, table, ld: int, tokens, out, n: int, width: int, vocab: int, offset=None, scale: float = 1.0, stream: int = 0) -> None:
+        self._call("embed_bf16_dev", _ptr(table), _sz(ld), _ptr(tokens), _optr(offset), _sz(n), _sz(width), _sz(vocab), C.c_float(scale), _ptr(out), _vp(stream))
+
+    def sum_norm_rows_dev(self, rows: "SumRows", stream: int = 0) -> None:
+        self._call("sum_norm_rows_dev", C.byref(rows), _vp(stream))
+
+    def gqa_scratch_bytes(self, heads: int, maps: int, vdimp: int, nq: int) -> int:
+        self.c.bitnet_hip_gqa_scratch_bytes.restype = _sz
+        return int(self.c.bitnet_hip_gqa_scratch_bytes(_sz(heads), _sz(maps), _sz(vdimp), _sz(nq)))
+
+    def gqa_rows_dev(self, a: "Gqa", rows, ld: int, rows_f32: bool, cache_f32: bool, pos, n: int, stream: int = 0) -> None:
+        self._call("gqa_rows_dev", C.byref(a), _ptr(rows), _sz(ld), C.c_int(rows_f32), C.c_int(cache_f32), _ptr(pos), _sz(n), _vp(stream))
+
+    def gqa_step_dev(self, a: "Gqa", row, pos, scratch, stream: int = 0) -> None:
+        self._call("gqa_step_dev", C.byref(a), _ptr(row), _ptr(pos), _ptr(scratch), _vp(stream))
+
+    def gqa_any_dev(self, a: "Gqa", q, ldq: int, q_f32: bool, cache_f32: bool, pos, q0: int, nq: int, scratch, stream: int = 0) -> None:
+        self._call("gqa_any_dev", C.byref(a), _ptr(q), _sz(ldq), C.c_int(q_f32), C.c_int(cache_f32), _ptr(pos), _sz(q0), _sz(nq), _ptr(scratch), _vp(stream))
+
+    def gqa_merge_dev(self, a: "Gqa", pos, q0: int, nq: int, scratch, out, ldo: int, out_bf16: bool, stream: int = 0) -> None:
+        self._call("gqa_merge_dev", C.byref(a), _ptr(pos), _sz(q0), _sz(nq), _ptr(scratch), _ptr(out), _sz(ldo), C.c_int(out_bf16), _vp(stream))
+
+    def gqa_prefill_dev(self, a: "Gqa", q, ldq: int, n_ctx: int, nq: int, out, ldo: int, stream: int = 0) -> None:
+        self._call("gqa_prefill_dev", C.byref(a), _ptr(q), _sz(ldq), _sz(n_ctx), _sz(nq), _ptr(out), _sz(ldo), _vp(stream))
+
+    def delta_step_dev(self, d: "Delta", row, ba, pos, out, stream: int = 0) -> None:
+        self._call("delta_step_dev", C.byref(d), _ptr(row), _ptr(ba), _ptr(pos), _ptr(out), _vp(stream))
+
+    def delta_rows_dev(self, d: "Delta", rows, ld: int, rows_f32: bool, ba, ldba: int, pos, n: int, qk, v, gates, stream: int = 0) -> None:
+        self._call("delta_rows_dev", C.byref(d), _ptr(rows), _sz(ld), C.c_int(rows_f32), _ptr(ba), _sz(ldba), _ptr(pos), _sz(n), _ptr(qk), _ptr(v), _ptr(gates),
+                   _vp(stream))
+
+    def delta_keep_dev(self, d: "Delta", rows, ld: int, rows_f32: bool, pos, n: int, stream: int = 0) -> None:
+        self._call("delta_keep_dev", C.byref(d), _ptr(rows), _sz(ld), C.c_int(rows_f32), _ptr(pos), _sz(n), _vp(stream))
+
+    def delta_recurrent_dev(self, d: "Delta", qk, v, gates, rows, ld: int, rows_f32: bool, n: int, out, ldo: int, stream: int = 0) -> None:
+        self._call("delta_recurrent_dev", C.byref(d), _ptr(qk), _ptr(v), _ptr(gates), _ptr(rows), _sz(ld), C.c_int(rows_f32), _sz(n), _ptr(out), _sz(ldo), _vp(stream))
+
+    def delta_workspace_bytes(self, n: int, heads: int, dimp: int, vdimp: int) -> int:
+        self.c.bitnet_hip_delta_workspace_bytes.restype = _sz
+        return int(self.c.bitnet_hip_delta_workspace_bytes(_sz(n), _sz(heads), _sz(dimp), _sz(vdimp)))
+
+    def delta_chunked_dev(self, d: "Delta", qk, v, gates, rows, ld: int, n: int, out, ldo: int, workspace, nbytes: int, stream: int = 0) -> None:
+        self._call("delta_chunked_dev", C.byref(d), _ptr(qk), _ptr(v), _ptr(gates), _ptr(rows), _sz(ld), _sz(n), _ptr(out), _sz(ldo), _ptr(workspace), _sz(nbytes),
+                   _vp(stream))
+
+    def experts_plan_bytes(self, m: int, experts: int, top: int) -> int:
+        self.c.bitnet_hip_experts_plan_bytes.restype = _sz
+        return int(self.c.bitnet_hip_experts_plan_bytes(_sz(m), _sz(experts), _sz(top)))
+
+    def experts_plan_make(self, workspace, nbytes: int, m: int, experts: int, top: int, tile: int) -> "ExpertsPlan":
+        p = ExpertsPlan()
+        self._call("experts_plan_make", _ptr(workspace), _sz(nbytes), _sz(m), _sz(experts), _sz(top), _sz(tile), C.byref(p))
+        return p
+
+    def experts_route_dev(self, logits, ldz: int, scale: float, plan: "ExpertsPlan", stream: int = 0) -> None:
+        self._call("experts_route_dev", _ptr(logits), _sz(ldz), C.c_float(scale), C.byref(plan), _vp(stream))
+
+    def experts_matmul_dev(self, plan: "ExpertsPlan", gather: bool, a, lda: int, a_f32: bool, w, n: int, k: int, ldw: int, act: int, c, ldc: int, c_f32: bool,
+                           stream: int = 0) -> None:
+        self._call("experts_matmul_dev", C.byref(plan), C.c_int(gather), _ptr(a), _sz(lda), C.c_int(a_f32), _ptr(w), _sz(n), _sz(k), _sz(ldw), C.c_int(act), _ptr(c),
+                   _sz(ldc), C.c_int(c_f32), _vp(stream))
+
+    def experts_up_dev(self, logits, experts: int, top: int, scale: float, x, w, rows: int, cols: int, ld: int, act: int, y, ldy: int, ids, stream: int = 0) -> None:
+        self._call("experts_up_dev", _ptr(logits), _sz(experts), _sz(top), C.c_float(scale), _ptr(x), _ptr(w), _sz(rows), _sz(cols), _sz(ld), C.c_int(act), _ptr(y),
+                   _sz(ldy), _ptr(ids), _vp(stream))
+
+    def experts_out_dev(self, x0, w0, cols0: int, ld0: int, bias, x1, ldx1: int, w1, cols1: int, ld1: int, ids, top: int, rows: int, y, stream: int = 0) -> None:
+        self._call("experts_out_dev", _ptr(x0), _ptr(w0), _sz(cols0), _sz(ld0), _optr(bias), _ptr(x1), _sz(ldx1), _ptr(w1), _sz(cols1), _sz(ld1), _ptr(ids), _sz(top),
+                   _sz(rows), _ptr(y), _vp(stream))
 
     def residual_norm_rows_dev(self, x, m: int, width: int, eps: float, weight_offset: float, y=None, ldy: int = 0, post_weight=None, scale=None,
                                next_weight=None, h=None, ldh: int = 0, h_f32: bool = True, stream: int = 0) -> None:
@@ -575,8 +666,9 @@ class HipLib:
     def dense_gemv_dev(self, x, w, rows: int, cols: int, ld: int, y, kind: int = 0, eps: float = 0.0, weight_offset: float = 0.0, weight=None, res=None,
                        post_weight=None, scale=None, gate=None, x_out=None, n: int = 0, mean_n: int = 0, bias=None, act0: int = 0, act1: int = 0,
                        act_split: int = 0, batch: int = 1, w_batch: int = 0, x_batch: int = 0, y_batch: int = 0, latent=None, latent_f32: bool = False,
-                       stream: int = 0) -> None:
-        vi = VectorInput(_addr(x), kind, eps, weight_offset, _addr(weight), _addr(res), _addr(post_weight), _addr(scale), _addr(gate), _addr(x_out), n, mean_n)
+                       mult: float = 1.0, center: bool = False, norm_bias=None, x2=None, h_out=None, stream: int = 0) -> None:
+        vi = VectorInput(_addr(x), kind, eps, weight_offset, _addr(weight), _addr(res), _addr(post_weight), _addr(scale), _addr(gate), _addr(x_out), n, mean_n, mult, int(center),
+                         _addr(norm_bias), _addr(x2), _addr(h_out))
         self._call("dense_gemv_dev", C.byref(vi), _ptr(w), _sz(rows), _sz(cols), _sz(ld), _optr(bias), C.c_int(act0), C.c_int(act1), _sz(act_split), _ptr(y),
                    _sz(batch), _sz(w_batch), _sz(x_batch), _sz(y_batch), C.byref(latent) if latent is not None else None, C.c_int(latent_f32), _vp(stream))
 

@@ -1,4 +1,4 @@
-// abi_dense.hip -- section 5 of include/bitnet_hip.h: bf16-weight operators and sequence mixers.  Shapes are checked here against
+// abi_dense.hip -- section 5 of include/bitnet_hip.h, first part: bf16-weight operators, latent and linear attention.  Shapes are checked here against
 // what the kernels assume; the kernels live in kernels_dense.hip, kernels_latent.hip and kernels_linear.hip.
 #include "dense.hpp"
 
@@ -32,14 +32,19 @@ int to_latent_rows(const bitnet_hip_latent_rows *r, size_t m, int f32, LatentRow
 
 int to_vec_in(const bitnet_hip_vector_input *in, size_t cols, VecIn &o) {
     BH_REQUIRE(in && in->x, "vector input: null pointer");
-    BH_REQUIRE(in->kind >= BITNET_HIP_IN_PLAIN && in->kind <= BITNET_HIP_IN_RESIDUAL_NORM, "vector input: unknown kind %d", in->kind);
+    BH_REQUIRE(in->kind >= BITNET_HIP_IN_PLAIN && in->kind <= BITNET_HIP_IN_CONCAT, "vector input: unknown kind %d", in->kind);
     if (in->kind != BITNET_HIP_IN_PLAIN) {
-        BH_REQUIRE(in->weight && in->n > 0 && (size_t)in->n <= cols && in->mean_n >= 0, "vector input: bad norm");
-        if (in->kind == BITNET_HIP_IN_RESIDUAL_NORM && in->y)
-            BH_REQUIRE(in->post_weight && in->x_out != in->x && in->x_out != in->y, "vector input: the residual needs a norm and a buffer of its own");
+        if (in->kind == BITNET_HIP_IN_CONCAT)
+            BH_REQUIRE(in->x2 && in->n > 0 && 2 * (size_t)in->n <= cols, "vector input: bad second half");
+        else
+            BH_REQUIRE(in->weight && in->n > 0 && (size_t)in->n <= cols && in->mean_n >= 0, "vector input: bad norm");
+        if (in->kind >= BITNET_HIP_IN_RESIDUAL_NORM && in->y)
+            BH_REQUIRE((in->post_weight || in->mult != 0.f) && (!in->x_out || (in->x_out != in->x && in->x_out != in->y)),
+                       "vector input: the residual needs a norm or a factor, and a buffer of its own");
     }
     o.x = in->x, o.kind = in->kind, o.eps = in->eps, o.offset = in->weight_offset, o.weight = in->weight, o.y = in->y, o.post_weight = in->post_weight;
     o.scale = in->scale, o.gate = in->gate, o.x_out = in->y ? in->x_out : nullptr, o.n = in->n, o.mean_n = in->mean_n ? in->mean_n : in->n;
+    o.mult = in->mult, o.center = in->center, o.bias = in->bias, o.x2 = in->x2, o.h_out = in->h_out;
     return 0;
 }
 
@@ -58,12 +63,12 @@ int to_attn(const bitnet_hip_latent_attention *a, LatentAttn &o) {
 extern "C" {
 
 int bitnet_hip_embed_bf16_dev(const uint16_t *table, size_t ld, const int32_t *tokens, const int32_t *offset, size_t n, size_t width, size_t vocab,
-                              float *out, void *stream) {
+                              float scale, float *out, void *stream) {
     BH_GUARD_BEGIN
     BH_REQUIRE(table && tokens && out, "Null pointer passed to embed_bf16_dev");
     BH_REQUIRE(n > 0 && width > 0 && vocab > 0 && ld >= width, "embed_bf16: bad shape");
     BH_CHECK_DIMS(n, width);
-    BH_HIP_TRY(launch_embed_bf16(table, ld, tokens, offset, (int)n, (int)width, (int)vocab, out, (hipStream_t)stream));
+    BH_HIP_TRY(launch_embed_bf16(table, ld, tokens, offset, (int)n, (int)width, (int)vocab, scale, out, (hipStream_t)stream));
     return BITNET_HIP_OK;
     BH_GUARD_END
 }

@@ -1,5 +1,5 @@
-// dense.hpp -- device helpers and launcher declarations of the bf16-weight operators (kernels_dense.hip) and the sequence
-// mixers (kernels_latent.hip, kernels_linear.hip).
+// dense.hpp -- device helpers and launcher declarations of the bf16-weight operators (kernels_dense.hip, kernels_experts.hip) and the
+// sequence mixers (kernels_latent.hip, kernels_linear.hip, kernels_gqa.hip, kernels_delta.hip).
 //
 // Storage: weights bf16 row-major [rows][ld], ld a multiple of 64, columns past the matrix zero.  Activation matrices likewise
 // have ld a multiple of 64; what lies past their columns must be FINITE (a weight's zero column cancels it).
@@ -27,6 +27,10 @@ struct VecIn {
     float *x_out = nullptr;
     const float *gate = nullptr;
     int n = 0, mean_n = 0;        // elements; what the mean divides by (padded heads hold zeros: fewer than n)
+    float mult = 1.f;             // without post_weight: x + mult * y
+    int center = 0;               // layer norm, with bias
+    const float *bias = nullptr, *x2 = nullptr;
+    float *h_out = nullptr;       // the vector formed
 };
 
 struct GemvArgs {
@@ -55,6 +59,42 @@ struct GemmArgsD {
     int a_f32 = 0, c_f32 = 0;
     int batch = 1;
     size_t a_batch = 0, w_batch = 0, c_batch = 0;
+    // grouped form: the row tiles come from a list, (matrix, first row, rows) each; matrix i lies at w + i w_batch
+    const int4 *tiles = nullptr;
+    const int *n_tiles = nullptr;  // on the device
+    int max_tiles = 0, tile = 0;
+    const int *gather = nullptr;   // activation row of each row (nullptr: the row itself)
+};
+
+typedef bitnet_hip_sum_rows SumRows;
+typedef bitnet_hip_gqa Gqa;
+typedef bitnet_hip_delta Delta;
+typedef bitnet_hip_experts_plan ExpertsPlan;
+
+struct GqaStep {
+    const float *row = nullptr;    // raw projections of the token
+    const int *pos = nullptr;
+    float *scratch = nullptr;
+};
+
+struct ExpertsUp {
+    const float *logits = nullptr;
+    int experts = 0, top = 0;
+    float scale = 1.f;
+    const float *x = nullptr;
+    const uint16_t *w = nullptr;
+    int rows = 0, cols = 0, ld = 0, act = 0;
+    float *y = nullptr;
+    int ldy = 0;
+    int *ids = nullptr;
+};
+
+struct ExpertsOut {
+    const float *x0 = nullptr, *x1 = nullptr, *bias = nullptr;
+    const uint16_t *w0 = nullptr, *w1 = nullptr;
+    int cols0 = 0, ld0 = 0, cols1 = 0, ld1 = 0, ldx1 = 0, top = 0, rows = 0;
+    const int *ids = nullptr;
+    float *y = nullptr;
 };
 
 // rows of a down-projection output z -> normed query latent, normed key latent and rotated key part
@@ -124,8 +164,16 @@ constexpr int kLatentTile = 64;    // keys per step of the decode attention
 constexpr int kLatentSplits = 128;  // most records per (query, head)
 constexpr int kLatentRecHead = 4;  // floats ahead of a record's vector: running maximum, sum, unused
 
-hipError_t launch_embed_bf16(const uint16_t *table, size_t ld, const int *tokens, const int *offset, int n, int width, int vocab, float *out,
+constexpr int kGqaTile = 128;      // keys per workgroup and step of the decode attention
+constexpr int kGqaSplits = 128;    // most records per (query, head, map)
+constexpr int kGqaRecHead = 4;     // floats ahead of a record's vector: running maximum (of base-2 scores), sum, unused
+constexpr int kDeltaChunk = 64;    // tokens per chunk of the delta rule
+constexpr int kDeltaSegment = 2048;  // tokens per pass over the workspace
+constexpr int kMaxExperts = 1024, kMaxTop = 32;
+
+hipError_t launch_embed_bf16(const uint16_t *table, size_t ld, const int *tokens, const int *offset, int n, int width, int vocab, float scale, float *out,
                              hipStream_t s);
+hipError_t launch_sum_norm_rows(const SumRows &a, hipStream_t s);
 hipError_t launch_residual_norm_rows(float *x, const float *y, size_t ldy, const float *post_w, const float *scale, const float *next_w,
                                      float offset, float eps, int m, int width, void *h, size_t ldh, int h_f32, hipStream_t s);
 hipError_t launch_gated_norm_rows(const float *o, size_t ldo, const float *w, const void *gate, size_t ldg, int gate_f32, float eps, int m, int n,
@@ -143,6 +191,27 @@ size_t linear_workspace_bytes(int n, int heads, int dimp, int vdimp);
 bool linear_chunked_supported(int dimp, int vdimp);
 hipError_t launch_linear_recurrent(const LinearAttn &a, hipStream_t s);
 hipError_t launch_linear_chunked(const LinearAttn &a, hipStream_t s);
+size_t gqa_scratch_floats(size_t heads, size_t maps, size_t vdimp, size_t nq);
+bool gqa_supported(int dimp, int vdimp);
+hipError_t launch_gqa_rows(const Gqa &g, void *rows, size_t ld, int rows_f32, int cache_f32, const int *pos, int n, hipStream_t s);
+hipError_t launch_gqa_step(const Gqa &g, const GqaStep &a, hipStream_t s);
+hipError_t launch_gqa_any(const Gqa &g, const void *q, size_t ldq, int q_f32, int cache_f32, const int *pos, int q0, int nq, float *scratch, hipStream_t s);
+hipError_t launch_gqa_merge(const Gqa &g, const int *pos, int q0, int nq, const float *scratch, void *out, size_t ldo, int out_bf16, hipStream_t s);
+hipError_t launch_gqa_prefill(const Gqa &g, const uint16_t *q, size_t ldq, int n_ctx, int nq, uint16_t *out, size_t ldo, hipStream_t s);
+bool delta_supported(int dimp, int vdimp);
+bool delta_chunked_supported(int dimp, int vdimp);
+size_t delta_workspace_bytes(size_t n, size_t heads, size_t dimp, size_t vdimp);
+hipError_t launch_delta_step(const Delta &d, const float *row, const float *ba, const int *pos, float *out, hipStream_t s);
+hipError_t launch_delta_rows(const Delta &d, const void *rows, size_t ld, int rows_f32, const float *ba, size_t ldba, const int *pos, int n, float *qk,
+                             void *v, float *gates, hipStream_t s);
+hipError_t launch_delta_keep(const Delta &d, const void *rows, size_t ld, int rows_f32, const int *pos, int n, hipStream_t s);
+hipError_t launch_delta_recurrent(const Delta &d, const float *qk, const void *v, const float *gates, const void *rows, size_t ld, int rows_f32, int n,
+                                  void *out, size_t ldo, hipStream_t s);
+hipError_t launch_delta_chunked(const Delta &d, const float *qk, const uint16_t *v, const float *gates, const uint16_t *rows, size_t ld, int n,
+                                uint16_t *out, size_t ldo, void *workspace, hipStream_t s);
+hipError_t launch_experts_route(const float *logits, size_t ldz, float scale, const ExpertsPlan &p, hipStream_t s);
+hipError_t launch_experts_up(const ExpertsUp &a, hipStream_t s);
+hipError_t launch_experts_out(const ExpertsOut &a, hipStream_t s);
 
 // ---- device helpers --------------------------------------------------------------------------------------------------
 
@@ -227,6 +296,26 @@ __device__ __forceinline__ void split2(float a, float b, uint32_t &hi, uint32_t 
     lo = __builtin_amdgcn_perm(__builtin_bit_cast(uint32_t, lb), __builtin_bit_cast(uint32_t, la), 0x07060302u);
 }
 
+// eight floats as (high, low) fragments of the matrix cores
+struct SplitFrag {
+    bf16x8 hi, lo;
+};
+__device__ __forceinline__ SplitFrag split8(f32x4 a, f32x4 b) {
+    u32x4 h, l;
+    uint32_t x, y;
+    split2(a.x, a.y, x, y), h.x = x, l.x = y;
+    split2(a.z, a.w, x, y), h.y = x, l.y = y;
+    split2(b.x, b.y, x, y), h.z = x, l.z = y;
+    split2(b.z, b.w, x, y), h.w = x, l.w = y;
+    return {__builtin_bit_cast(bf16x8, h), __builtin_bit_cast(bf16x8, l)};
+}
+
 __device__ __forceinline__ f32x4 mfma_bf16(bf16x8 a, bf16x8 b, f32x4 c) { return __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, 0, 0, 0); }
+// a product of two split operands (the low x low term is below the last bit kept)
+__device__ __forceinline__ f32x4 mfma_split(const SplitFrag &a, const SplitFrag &b, f32x4 c) {
+    c = mfma_bf16(a.hi, b.hi, c);
+    c = mfma_bf16(a.hi, b.lo, c);
+    return mfma_bf16(a.lo, b.hi, c);
+}
 
 }  // namespace bitnet_hip

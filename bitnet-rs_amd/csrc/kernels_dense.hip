@@ -11,15 +11,15 @@ namespace bitnet_hip {
 
 // ---- embedding rows ---------------------------------------------------------------------------------------------------
 __global__ void k_embed_bf16(const uint16_t *__restrict__ table, size_t ld, const int *__restrict__ tokens, const int *__restrict__ offset,
-                             int width, int vocab, float *__restrict__ out) {
+                             int width, int vocab, float scale, float *__restrict__ out) {
     int tok = tokens[(offset ? *offset : 0) + blockIdx.x];
     tok = tok < 0 ? 0 : (tok >= vocab ? vocab - 1 : tok);
-    for (int i = threadIdx.x; i < width; i += blockDim.x) out[(size_t)blockIdx.x * width + i] = bf2f(table[(size_t)tok * ld + i]);
+    for (int i = threadIdx.x; i < width; i += blockDim.x) out[(size_t)blockIdx.x * width + i] = scale * bf2f(table[(size_t)tok * ld + i]);
 }
 
-hipError_t launch_embed_bf16(const uint16_t *table, size_t ld, const int *tokens, const int *offset, int n, int width, int vocab, float *out,
+hipError_t launch_embed_bf16(const uint16_t *table, size_t ld, const int *tokens, const int *offset, int n, int width, int vocab, float scale, float *out,
                              hipStream_t s) {
-    hipLaunchKernelGGL(k_embed_bf16, dim3(n), dim3(256), 0, s, table, ld, tokens, offset, width, vocab, out);
+    hipLaunchKernelGGL(k_embed_bf16, dim3(n), dim3(256), 0, s, table, ld, tokens, offset, width, vocab, scale, out);
     return hipGetLastError();
 }
 
@@ -105,6 +105,134 @@ hipError_t launch_residual_norm_rows(float *x, const float *y, size_t ldy, const
         hipLaunchKernelGGL(k_residual_norm_rows<float>, dim3(m), dim3(256), 0, s, x, y, ldy, post_w, scale, next_w, offset, eps, width, (float *)h, ldh);
     else
         hipLaunchKernelGGL(k_residual_norm_rows<uint16_t>, dim3(m), dim3(256), 0, s, x, y, ldy, post_w, scale, next_w, offset, eps, width, (uint16_t *)h, ldh);
+    return hipGetLastError();
+}
+
+// Rows of a block whose sublayers add up: x += mult * (y + the chosen experts' rows); h = norm(x) or [x; x2].  Four columns at a time, rows of up to
+// 4096 columns in registers.
+__device__ __forceinline__ f32x4 ld4(const float *p, size_t i) { return *reinterpret_cast<const f32x4 *>(p + i); }
+__device__ __forceinline__ f32x4 ld4(const uint16_t *p, size_t i) {
+    const u32x2 v = *reinterpret_cast<const u32x2 *>(p + i);
+    return f32x4{bf2f(v.x & 0xffffu), bf2f(v.x >> 16), bf2f(v.y & 0xffffu), bf2f(v.y >> 16)};
+}
+__device__ __forceinline__ void st4(float *p, size_t i, f32x4 v) { *reinterpret_cast<f32x4 *>(p + i) = v; }
+__device__ __forceinline__ void st4(uint16_t *p, size_t i, f32x4 v) {
+    *reinterpret_cast<bf16x4 *>(p + i) = bf16x4{(__bf16)v.x, (__bf16)v.y, (__bf16)v.z, (__bf16)v.w};
+}
+constexpr int kSumRegs = 4;
+
+template <class T, bool VEC>
+__global__ __launch_bounds__(256) void k_sum_norm_rows(SumRows p) {
+    __shared__ float slot[4];
+    const int tid = threadIdx.x, width = (int)p.width;
+    float *x = p.x + (size_t)blockIdx.x * width;
+    const float *y = p.y ? p.y + (size_t)blockIdx.x * p.ldy : nullptr;
+    T *h = p.h ? (T *)p.h + (size_t)blockIdx.x * p.ldh : nullptr;
+    const T *er = (const T *)p.expert_rows;
+    const int *slots = p.slots + (size_t)blockIdx.x * p.top;
+    const float *sw = p.slot_weights + (size_t)blockIdx.x * p.top;
+    const float *x2 = p.x2 ? p.x2 + (size_t)blockIdx.x * width : nullptr;
+    if (VEC) {
+        f32x4 v[kSumRegs];
+        const int n4 = width >> 2;
+#pragma unroll
+        for (int j = 0; j < kSumRegs; ++j) {
+            const int i = tid + 256 * j;
+            v[j] = f32x4{0.f, 0.f, 0.f, 0.f};
+            if (i < n4) v[j] = ld4(x, 4 * i);
+        }
+        if (y) {
+            f32x4 a[kSumRegs];
+#pragma unroll
+            for (int j = 0; j < kSumRegs; ++j) {
+                const int i = tid + 256 * j;
+                if (i < n4) a[j] = ld4(y, 4 * i);
+            }
+            for (int k = 0; k < (int)p.top; ++k) {
+                const T *row = er + (size_t)slots[k] * p.ld_expert;
+                const float w = sw[k];
+#pragma unroll
+                for (int j = 0; j < kSumRegs; ++j) {
+                    const int i = tid + 256 * j;
+                    if (i < n4) a[j] += w * ld4(row, 4 * i);
+                }
+            }
+#pragma unroll
+            for (int j = 0; j < kSumRegs; ++j) {
+                const int i = tid + 256 * j;
+                if (i < n4) {
+                    v[j] += p.mult * a[j];
+                    st4(x, 4 * i, v[j]);
+                }
+            }
+        }
+        if (!h) return;
+        if (x2) {
+#pragma unroll
+            for (int j = 0; j < kSumRegs; ++j) {
+                const int i = tid + 256 * j;
+                if (i < n4) {
+                    st4(h, 4 * i, v[j]);
+                    st4(h, width + 4 * i, ld4(x2, 4 * i));
+                }
+            }
+        } else {
+            float mean = 0.f, ss = 0.f;
+            if (p.center) {
+                float t = 0.f;
+#pragma unroll
+                for (int j = 0; j < kSumRegs; ++j) t += (v[j].x + v[j].y) + (v[j].z + v[j].w);
+                mean = group_sum<4>(t, slot) / (float)width;
+            }
+#pragma unroll
+            for (int j = 0; j < kSumRegs; ++j) {
+                if (tid + 256 * j < n4) v[j] -= mean;
+                ss += (v[j].x * v[j].x + v[j].y * v[j].y) + (v[j].z * v[j].z + v[j].w * v[j].w);
+            }
+            const float inv = 1.0f / sqrtf(group_sum<4>(ss, slot) / (float)width + p.eps);
+#pragma unroll
+            for (int j = 0; j < kSumRegs; ++j) {
+                const int i = tid + 256 * j;
+                if (i < n4) {
+                    f32x4 r = v[j] * inv * (p.weight_offset + ld4(p.weight, 4 * i));
+                    if (p.bias) r += ld4(p.bias, 4 * i);
+                    st4(h, 4 * i, r);
+                }
+            }
+        }
+    } else {  // (a thread comes back to its own columns only)
+        if (y)
+            for (int i = tid; i < width; i += 256) {
+                float a = y[i];
+                for (int k = 0; k < (int)p.top; ++k) a += sw[k] * ld_act(er + (size_t)slots[k] * p.ld_expert, i);
+                x[i] += p.mult * a;
+            }
+        if (!h) return;
+        if (x2) {
+            for (int i = tid; i < width; i += 256) {
+                st_act(h, i, x[i]);
+                st_act(h, width + i, x2[i]);
+            }
+        } else {
+            float mean = 0.f, ss = 0.f;
+            if (p.center) {
+                float t = 0.f;
+                for (int i = tid; i < width; i += 256) t += x[i];
+                mean = group_sum<4>(t, slot) / (float)width;
+            }
+            for (int i = tid; i < width; i += 256) ss += (x[i] - mean) * (x[i] - mean);
+            const float inv = 1.0f / sqrtf(group_sum<4>(ss, slot) / (float)width + p.eps);
+            for (int i = tid; i < width; i += 256) st_act(h, i, (x[i] - mean) * inv * (p.weight_offset + p.weight[i]) + (p.bias ? p.bias[i] : 0.f));
+        }
+    }
+    for (int i = (x2 ? 2 : 1) * width + tid; i < (int)p.ldh; i += 256) st_act(h, i, 0.f);
+}
+
+hipError_t launch_sum_norm_rows(const SumRows &a, hipStream_t s) {
+    // (four columns at a time: every row of every operand starts on its own alignment)
+    const bool vec = a.width % 4 == 0 && a.width <= 1024 * kSumRegs && a.ldy % 4 == 0 && a.ld_expert % 4 == 0 && a.ldh % 4 == 0;
+    auto fn = a.h_f32 ? (vec ? k_sum_norm_rows<float, true> : k_sum_norm_rows<float, false>) : (vec ? k_sum_norm_rows<uint16_t, true> : k_sum_norm_rows<uint16_t, false>);
+    hipLaunchKernelGGL(fn, dim3(a.m), dim3(256), 0, s, a);
     return hipGetLastError();
 }
 
@@ -227,7 +355,18 @@ __device__ void form_input(const VecIn &in, const float *x, int cols, int kp, fl
             const f32x4 v = reinterpret_cast<const f32x4 *>(x)[min(i, n4 - 1)];
             xv[j] = v * (i < n4 ? 1.0f : 0.0f);
         }
-        if (in.kind == BITNET_HIP_IN_RESIDUAL_NORM && in.y) {
+        if (in.kind >= BITNET_HIP_IN_RESIDUAL_NORM && in.y && !in.post_weight) {
+            f32x4 yv[NR];
+#pragma unroll
+            for (int j = 0; j < NR; ++j) yv[j] = reinterpret_cast<const f32x4 *>(in.y)[min(tid + 256 * j, n4 - 1)];
+#pragma unroll
+            for (int j = 0; j < NR; ++j) {
+                const int i = tid + 256 * j;
+                if (i >= n4) continue;
+                xv[j] += in.mult * yv[j];
+                if (writer && in.x_out) reinterpret_cast<f32x4 *>(in.x_out)[i] = xv[j];
+            }
+        } else if (in.kind >= BITNET_HIP_IN_RESIDUAL_NORM && in.y) {
             f32x4 yv[NR], pw[NR], sc[NR];
             float ss = 0.f;
 #pragma unroll
@@ -253,8 +392,32 @@ __device__ void form_input(const VecIn &in, const float *x, int cols, int kp, fl
                 const int i = tid + 256 * j;
                 if (i >= n4) continue;
                 xv[j] += sc[j] * (yv[j] * inv * (in.offset + pw[j]));
-                if (writer) reinterpret_cast<f32x4 *>(in.x_out)[i] = xv[j];
+                if (writer && in.x_out) reinterpret_cast<f32x4 *>(in.x_out)[i] = xv[j];
             }
+        }
+        if (in.kind == BITNET_HIP_IN_CONCAT) {
+#pragma unroll
+            for (int j = 0; j < NR; ++j) {
+                const int i = tid + 256 * j;
+                if (i >= n4) continue;
+                reinterpret_cast<f32x4 *>(xs)[i] = xv[j];
+                reinterpret_cast<f32x4 *>(xs)[n4 + i] = reinterpret_cast<const f32x4 *>(in.x2)[i];
+            }
+            for (int i = 2 * n + tid; i < kp; i += 256) xs[i] = 0.f;
+            __syncthreads();
+            return;
+        }
+        f32x4 bv[NR];
+        if (in.center) {
+            float t = 0.f;
+#pragma unroll
+            for (int j = 0; j < NR; ++j) {
+                t += (xv[j].x + xv[j].y) + (xv[j].z + xv[j].w);
+                bv[j] = in.bias ? reinterpret_cast<const f32x4 *>(in.bias)[min(tid + 256 * j, n4 - 1)] : f32x4{0.f, 0.f, 0.f, 0.f};
+            }
+            const float mean = group_sum<4>(t, slot) / (float)in.mean_n;
+#pragma unroll
+            for (int j = 0; j < NR; ++j) xv[j] -= tid + 256 * j < n4 ? mean : 0.f;
         }
         f32x4 wv[NR], gv[NR];
         float ss = 0.f;
@@ -275,18 +438,29 @@ __device__ void form_input(const VecIn &in, const float *x, int cols, int kp, fl
 #pragma unroll
         for (int j = 0; j < NR; ++j) {
             const int i = tid + 256 * j;
-            if (i < n4) reinterpret_cast<f32x4 *>(xs)[i] = xv[j] * inv * (in.offset + wv[j]) * gv[j];
+            if (i >= n4) continue;
+            f32x4 r = xv[j] * inv * (in.offset + wv[j]) * gv[j];
+            if (in.center) r += bv[j];
+            reinterpret_cast<f32x4 *>(xs)[i] = r;
+            if (writer && in.h_out) reinterpret_cast<f32x4 *>(in.h_out)[i] = r;
         }
     } else {
         float ss = 0.f;
-        if (in.kind == BITNET_HIP_IN_RESIDUAL_NORM && in.y) {
+        if (in.kind >= BITNET_HIP_IN_RESIDUAL_NORM && in.y && !in.post_weight) {
+            for (int i = tid; i < n; i += 256) {
+                const float v = x[i] + in.mult * in.y[i];
+                xs[i] = v;
+                if (writer && in.x_out) in.x_out[i] = v;
+                ss += v * v;
+            }
+        } else if (in.kind >= BITNET_HIP_IN_RESIDUAL_NORM && in.y) {
             for (int i = tid; i < n; i += 256) ss += in.y[i] * in.y[i];
             const float inv = 1.0f / sqrtf(group_sum<4>(ss, slot) / (float)in.mean_n + in.eps);
             ss = 0.f;
             for (int i = tid; i < n; i += 256) {
                 const float v = x[i] + (in.scale ? in.scale[i] : 1.0f) * (in.y[i] * inv * (in.offset + in.post_weight[i]));
                 xs[i] = v;
-                if (writer) in.x_out[i] = v;
+                if (writer && in.x_out) in.x_out[i] = v;
                 ss += v * v;
             }
         } else {
@@ -295,8 +469,27 @@ __device__ void form_input(const VecIn &in, const float *x, int cols, int kp, fl
                 ss += x[i] * x[i];
             }
         }
+        if (in.kind == BITNET_HIP_IN_CONCAT) {
+            for (int i = tid; i < n; i += 256) xs[n + i] = in.x2[i];
+            for (int i = 2 * n + tid; i < kp; i += 256) xs[i] = 0.f;
+            __syncthreads();
+            return;
+        }
+        if (in.center) {  // (a thread comes back to its own elements only)
+            float t = 0.f;
+            for (int i = tid; i < n; i += 256) t += xs[i];
+            const float mean = group_sum<4>(t, slot) / (float)in.mean_n;
+            ss = 0.f;
+            for (int i = tid; i < n; i += 256) {
+                xs[i] -= mean;
+                ss += xs[i] * xs[i];
+            }
+        }
         const float inv = 1.0f / sqrtf(group_sum<4>(ss, slot) / (float)in.mean_n + in.eps);
-        for (int i = tid; i < n; i += 256) xs[i] = xs[i] * inv * (in.offset + in.weight[i]) * (in.gate ? in.gate[i] : 1.0f);
+        for (int i = tid; i < n; i += 256) {
+            xs[i] = xs[i] * inv * (in.offset + in.weight[i]) * (in.gate ? in.gate[i] : 1.0f) + (in.center && in.bias ? in.bias[i] : 0.f);
+            if (writer && in.h_out) in.h_out[i] = xs[i];
+        }
     }
     for (int i = n + tid; i < kp; i += 256) xs[i] = 0.f;
     __syncthreads();
@@ -340,7 +533,7 @@ __global__ __launch_bounds__(256) void k_dense_gemv(GemvK p) {
         }
     };
     if (g < p.groups) fetch(g, 0);
-    form_input(a.in, a.in.x + (size_t)b * a.x_batch, a.cols, p.kp, xs, slot, blockIdx.x == 0 && b == 0 && a.in.x_out);
+    form_input(a.in, a.in.x + (size_t)b * a.x_batch, a.cols, p.kp, xs, slot, blockIdx.x == 0 && b == 0);
     float bv = -INFINITY;
     int bi = 0x7fffffff;
     for (; g < p.groups; g += n_wg * 4) {
@@ -508,7 +701,8 @@ __device__ __forceinline__ int weight_key(int row) {
     return CF32 ? (row >> 1) & 7 : ((row / (4 * FN)) & 3) * 2 + ((row >> 1) & 1);
 }
 
-template <int TN, int TM, int WN, int WM, int ST, bool CF32>
+// GROUPED: the row tiles come from a device list, (matrix, first row, rows) each; a matrix's tiles follow one another.
+template <int TN, int TM, int WN, int WM, int ST, bool CF32, bool GROUPED = false>
 __global__ __launch_bounds__(64 * WN * WM, 2) void k_dense_gemm(GemmArgsD p, int tiles_n, int tiles_m, int swizzle) {
     extern __shared__ __attribute__((aligned(1024))) uint8_t lds[];
     constexpr int NW = WN * WM, DN = TN / NW / 8, DM = TM / NW / 8;  // DMA instructions per wave and step (eight rows each)
@@ -518,23 +712,36 @@ __global__ __launch_bounds__(64 * WN * WM, 2) void k_dense_gemm(GemmArgsD p, int
     // workgroup -> tile: consecutive workgroups land on the eight XCDs in turn; give each XCD a contiguous run of tiles, and walk
     // the tiles in groups of eight row tiles so that what runs together shares both operands in the XCD's L2
     int id = blockIdx.x;
-    const int total = tiles_n * tiles_m;
-    if (swizzle) id = (id & 7) * (total >> 3) + (id >> 3);
-    const int gm = 8;
-    const int group = id / (gm * tiles_n), first = group * gm, size = tiles_m - first < gm ? tiles_m - first : gm;
-    const int tm = first + (id % (gm * tiles_n)) % size, tn = (id % (gm * tiles_n)) / size;
-    const int m0 = tm * TM, n0 = tn * TN;
+    int m0, n0, m_end;
     const uint16_t *A = (const uint16_t *)p.a + (size_t)blockIdx.y * p.a_batch;
     const uint16_t *W = p.w + (size_t)blockIdx.y * p.w_batch;
+    if (GROUPED) {
+        const int total = *p.n_tiles * tiles_n, per = (total + 7) >> 3;
+        if ((id >> 3) >= per) return;
+        id = (id & 7) * per + (id >> 3);
+        if (id >= total) return;
+        const int4 tile = p.tiles[id / tiles_n];
+        m0 = tile.y, m_end = tile.y + tile.z, n0 = id % tiles_n * TN;
+        W += (size_t)tile.x * p.w_batch;
+    } else {
+        const int total = tiles_n * tiles_m;
+        if (swizzle) id = (id & 7) * (total >> 3) + (id >> 3);
+        const int gm = 8;
+        const int group = id / (gm * tiles_n), first = group * gm, size = tiles_m - first < gm ? tiles_m - first : gm;
+        const int tm = first + (id % (gm * tiles_n)) % size, tn = (id % (gm * tiles_n)) / size;
+        m0 = tm * TM, n0 = tn * TN, m_end = p.m;
+    }
     const int drow = lane >> 3;
     // (lane offsets from the tile's first row: a tile spans less than 4 GiB; rows past the end read the tile's own rows over again)
-    const unsigned rows_m = min(TM, p.m - m0), rows_n = min(TN, p.n - n0);
-    const uint16_t *A0 = A + (size_t)m0 * p.lda, *W0 = W + (size_t)n0 * p.ldw;
+    const unsigned rows_m = min(TM, m_end - m0), rows_n = min(TN, p.n - n0);
+    const bool gathered = GROUPED && p.gather;
+    const uint16_t *A0 = gathered ? A : A + (size_t)m0 * p.lda, *W0 = W + (size_t)n0 * p.ldw;
     unsigned oa[DM], ow[DN];
 #pragma unroll
     for (int i = 0; i < DM; ++i) {
         const int r = wave * (TM / NW) + i * 8 + drow, unit = (lane & 7) ^ ((r >> 1) & 7);
-        oa[i] = (unsigned)((unsigned)r % rows_m * p.lda + unit * 8) * 2;
+        const unsigned row = gathered ? (unsigned)p.gather[m0 + (unsigned)r % rows_m] : (unsigned)r % rows_m;
+        oa[i] = (unsigned)(row * p.lda + unit * 8) * 2;
     }
 #pragma unroll
     for (int i = 0; i < DN; ++i) {
@@ -612,7 +819,7 @@ __global__ __launch_bounds__(64 * WN * WM, 2) void k_dense_gemm(GemmArgsD p, int
 #pragma unroll
     for (int j = 0; j < FM; ++j) {
         const int m = m0 + wm + j * 16 + r16;
-        if (m >= p.m) continue;
+        if (m >= m_end) continue;
         const size_t o = (size_t)blockIdx.y * p.c_batch + (size_t)m * p.ldc + nl;
         if (p.bias)
 #pragma unroll
@@ -667,6 +874,19 @@ __global__ __launch_bounds__(64 * WN * WM, 2) void k_dense_gemm(GemmArgsD p, int
     }
 }
 
+template <int T, int ST>
+static hipError_t grouped_go(const GemmArgsD &a, hipStream_t s) {
+    const int tn = (a.n + T - 1) / T;
+    constexpr size_t lds = (size_t)ST * T * 256;
+    auto fn = k_dense_gemm<T, T, 2, 2, ST, false, true>;
+    if (lds > 65536) {
+        const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(fn), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+        if (e != hipSuccess) return e;
+    }
+    hipLaunchKernelGGL(fn, dim3((tn * a.max_tiles + 7) / 8 * 8), dim3(256), lds, s, a, tn, 0, 0);
+    return hipGetLastError();
+}
+
 template <int T, int WN, int WM, int ST>
 static hipError_t gemm_go(const GemmArgsD &a, hipStream_t s) {
     const int tn = (a.n + T - 1) / T, tm = (a.m + T - 1) / T, swz = (tn * tm) % 8 == 0 ? 1 : 0;
@@ -681,15 +901,25 @@ static hipError_t gemm_go(const GemmArgsD &a, hipStream_t s) {
 }
 
 // f32 activations: f32 multiply-adds on a 64 x 64 tile, 4 x 4 per thread
+template <bool GROUPED>
 __global__ __launch_bounds__(256) void k_dense_gemm_f32(GemmArgsD p) {
     __shared__ float sa[16][68], sw[16][68];
     const int tid = threadIdx.x, tx = tid & 15, ty = tid >> 4;
-    const int m0 = blockIdx.y * 64, n0 = blockIdx.x * 64;
+    int m0 = blockIdx.y * 64, m_end = p.m;
+    const int n0 = blockIdx.x * 64;
     const float *A = (const float *)p.a + (size_t)blockIdx.z * p.a_batch;
     const uint16_t *W = p.w + (size_t)blockIdx.z * p.w_batch;
+    if (GROUPED) {
+        if ((int)blockIdx.y >= *p.n_tiles) return;
+        const int4 tile = p.tiles[blockIdx.y];
+        m0 = tile.y, m_end = tile.y + tile.z;
+        W += (size_t)tile.x * p.w_batch;
+    }
     float acc[4][4] = {};
     const int lr = tid >> 2, lk = (tid & 3) * 4;
-    const int ar = m0 + lr < p.m ? m0 + lr : p.m - 1, wr = n0 + lr < p.n ? n0 + lr : p.n - 1;
+    int ar = m0 + lr < m_end ? m0 + lr : m_end - 1;
+    if (GROUPED && p.gather) ar = p.gather[ar];
+    const int wr = n0 + lr < p.n ? n0 + lr : p.n - 1;
     for (int k0 = 0; k0 < p.k; k0 += 16) {
         const f32x4 av = *reinterpret_cast<const f32x4 *>(A + (size_t)ar * p.lda + k0 + lk);
         const u32x2 wv = *reinterpret_cast<const u32x2 *>(W + (size_t)wr * p.ldw + k0 + lk);
@@ -710,7 +940,7 @@ __global__ __launch_bounds__(256) void k_dense_gemm_f32(GemmArgsD p) {
     }
     for (int i = 0; i < 4; ++i) {
         const int m = m0 + ty * 4 + i;
-        if (m >= p.m) break;
+        if (m >= m_end) break;
         for (int j = 0; j < 4; ++j) {
             const int n = n0 + tx * 4 + j;
             if (n >= p.n) break;
@@ -728,8 +958,17 @@ hipError_t launch_dense_gemm(const GemmArgsD &args, hipStream_t s) {
     GemmArgsD a = args;
     if (a.m <= 0 || a.n <= 0) return hipSuccess;
     if (a.act_split == 0) a.act_split = a.n;
+    if (a.tiles) {
+        if (a.a_f32) {
+            if (a.tile != 64) return hipErrorInvalidValue;
+            hipLaunchKernelGGL(k_dense_gemm_f32<true>, dim3((a.n + 63) / 64, a.max_tiles, 1), dim3(256), 0, s, a);
+            return hipGetLastError();
+        }
+        if (a.c_f32) return hipErrorInvalidValue;
+        return a.tile == 128 ? grouped_go<128, 2>(a, s) : a.tile == 64 ? grouped_go<64, 4>(a, s) : hipErrorInvalidValue;
+    }
     if (a.a_f32) {
-        hipLaunchKernelGGL(k_dense_gemm_f32, dim3((a.n + 63) / 64, (a.m + 63) / 64, a.batch), dim3(256), 0, s, a);
+        hipLaunchKernelGGL(k_dense_gemm_f32<false>, dim3((a.n + 63) / 64, (a.m + 63) / 64, a.batch), dim3(256), 0, s, a);
         return hipGetLastError();
     }
     auto tiles = [&](int t) { return (long)((a.n + t - 1) / t) * ((a.m + t - 1) / t) * a.batch; };

@@ -1,0 +1,339 @@
+// kernels_experts.hip -- mixture of experts (gfx950): the choice of a token's experts, the row lists of the grouped products
+// (kernels_dense.hip) and the matrix-vector products of the decode step.
+//
+// The router's logits, scores and weights are f32.  A prompt's choices become slots: an expert's slots lie side by side, cut into tiles of rows
+// (expert, first slot, slots); a slot's token is its activation row on the way up, the slot itself is the row on the way down.
+#include "dense.hpp"
+
+namespace bitnet_hip {
+
+// A wave chooses one token's experts: lane k < top receives the k-th one and its weight.  Lanes hold neighbouring experts, so that among equal
+// scores the lowest lane has the lowest index.
+constexpr int kPerLane = kMaxExperts / 64;
+__device__ __forceinline__ void choose(const float *z, int experts, int top, float scale, int &id, float &weight) {
+    const int lane = threadIdx.x & 63, per = (experts + 63) / 64;
+    float s[kPerLane], m = -INFINITY;
+#pragma unroll
+    for (int j = 0; j < kPerLane; ++j) {
+        const int e = lane * per + j;
+        s[j] = j < per && e < experts ? z[e] : -INFINITY;
+        m = fmaxf(m, s[j]);
+    }
+    m = rows_max(row_max(m));
+    float sum = 0.f;
+#pragma unroll
+    for (int j = 0; j < kPerLane; ++j) {
+        s[j] = s[j] == -INFINITY ? 0.f : expf(s[j] - m);
+        sum += s[j];
+    }
+    sum = wave_sum(sum);
+#pragma unroll
+    for (int j = 0; j < kPerLane; ++j) s[j] = j < per && lane * per + j < experts ? s[j] / sum : -1.0f;  // (-1: not there, or taken)
+    id = 0, weight = 0.f;
+    float chosen = 0.f;
+    for (int k = 0; k < top; ++k) {
+        float best = -1.0f;
+        int at = 0;
+#pragma unroll
+        for (int j = 0; j < kPerLane; ++j)
+            if (s[j] > best) best = s[j], at = j;
+        const float w = rows_max(row_max(best));
+        const unsigned long long who = __ballot(best == w);
+        const int winner = who ? __builtin_ctzll(who) : 0;  // (no score compares equal to itself if a logit is not a number)
+        const int e = min(__builtin_amdgcn_readlane(lane * per + at, winner), experts - 1);
+        if (lane == k) id = e, weight = w;
+        chosen += w;
+        if (lane == winner)
+#pragma unroll
+            for (int j = 0; j < kPerLane; ++j)
+                if (j == at) s[j] = -1.0f;
+    }
+    weight = weight / (chosen + 1e-20f) * scale;
+}
+
+// ---- a prompt's choices -----------------------------------------------------------------------------------------------
+constexpr int kRouteTokens = 32;  // per workgroup; its choices are counted in LDS first
+
+__global__ __launch_bounds__(256) void k_route(const float *__restrict__ z, size_t ldz, float scale, ExpertsPlan p) {
+    __shared__ int hist[kMaxExperts];
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, experts = (int)p.experts, top = (int)p.top, m = (int)p.m;
+    constexpr int PER = kRouteTokens / 4;
+    for (int e = tid; e < experts; e += 256) hist[e] = 0;
+    __syncthreads();
+    int id[PER], rank[PER];
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+        const int t = blockIdx.x * kRouteTokens + wave * PER + i;
+        id[i] = rank[i] = 0;
+        if (t >= m) continue;
+        float w;
+        choose(z + (size_t)t * ldz, experts, top, scale, id[i], w);
+        if (lane < top) {
+            rank[i] = atomicAdd(&hist[id[i]], 1);
+            p.ids[(size_t)t * top + lane] = id[i];
+            p.weights[(size_t)t * top + lane] = w;
+        }
+    }
+    __syncthreads();
+    for (int e = tid; e < experts; e += 256) {
+        const int c = hist[e];
+        hist[e] = c ? atomicAdd(&p.counts[e], c) : 0;
+    }
+    __syncthreads();
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+        const int t = blockIdx.x * kRouteTokens + wave * PER + i;
+        if (t < m && lane < top) p.slots[(size_t)t * top + lane] = rank[i] + hist[id[i]];  // within its expert so far
+    }
+}
+
+// first slot and tiles of every expert; the counts are left at zero for the next portion
+__global__ __launch_bounds__(1024) void k_route_tiles(ExpertsPlan p) {
+    __shared__ int2 sums[kMaxExperts];
+    const int e = threadIdx.x, experts = (int)p.experts, tile = (int)p.tile;
+    const int count = e < experts ? p.counts[e] : 0, tiles = (count + tile - 1) / tile;
+    sums[e] = make_int2(count, tiles);
+    __syncthreads();
+    for (int off = 1; off < kMaxExperts; off <<= 1) {
+        const int2 mine = sums[e], other = e >= off ? sums[e - off] : make_int2(0, 0);
+        __syncthreads();
+        sums[e] = make_int2(mine.x + other.x, mine.y + other.y);
+        __syncthreads();
+    }
+    if (e < experts) {
+        const int first = sums[e].x - count, t0 = sums[e].y - tiles;
+        p.offsets[e] = first;
+        p.counts[e] = 0;
+        for (int i = 0; i < tiles; ++i)
+            if (t0 + i < (int)p.max_tiles) reinterpret_cast<int4 *>(p.tiles)[t0 + i] = make_int4(e, first + i * tile, min(tile, count - i * tile), 0);
+    }
+    if (e == 0) *p.n_tiles = min(sums[kMaxExperts - 1].y, (int)p.max_tiles);
+}
+
+__global__ __launch_bounds__(256) void k_route_slots(ExpertsPlan p) {
+    const int i = blockIdx.x * 256 + threadIdx.x;
+    if (i >= (int)(p.m * p.top)) return;
+    const int s = p.offsets[p.ids[i]] + p.slots[i];
+    p.slots[i] = s;
+    p.tokens[s] = i / (int)p.top;
+}
+
+hipError_t launch_experts_route(const float *logits, size_t ldz, float scale, const ExpertsPlan &p, hipStream_t s) {
+    hipLaunchKernelGGL(k_route, dim3((p.m + kRouteTokens - 1) / kRouteTokens), dim3(256), 0, s, logits, ldz, scale, p);
+    hipLaunchKernelGGL(k_route_tiles, dim3(1), dim3(1024), 0, s, p);
+    hipLaunchKernelGGL(k_route_slots, dim3((p.m * p.top + 255) / 256), dim3(256), 0, s, p);
+    return hipGetLastError();
+}
+
+// ---- one token --------------------------------------------------------------------------------------------------------
+// Both products in the manner of k_dense_gemv: LPR lanes per row, 16 bytes of weights per lane and chunk of LPR * 8 columns, R rows x U chunks in
+// flight, the input vector in LDS with every segment padded to whole chunks.
+__device__ __forceinline__ void stage(const float *x, int cols, int padded, float *dst) {
+    for (int i = threadIdx.x; i < padded; i += 256) dst[i] = i < cols ? x[i] : 0.f;
+}
+
+template <int R>
+__device__ __forceinline__ void multiply8(const u32x4 (&w)[R], const float *x, float (&acc)[R]) {
+    const f32x4 x0 = *reinterpret_cast<const f32x4 *>(x), x1 = *reinterpret_cast<const f32x4 *>(x + 4);
+#pragma unroll
+    for (int r = 0; r < R; ++r) {
+        acc[r] = fmaf(x0.x, __builtin_bit_cast(float, w[r].x << 16), acc[r]);
+        acc[r] = fmaf(x0.y, __builtin_bit_cast(float, w[r].x & 0xffff0000u), acc[r]);
+        acc[r] = fmaf(x0.z, __builtin_bit_cast(float, w[r].y << 16), acc[r]);
+        acc[r] = fmaf(x0.w, __builtin_bit_cast(float, w[r].y & 0xffff0000u), acc[r]);
+        acc[r] = fmaf(x1.x, __builtin_bit_cast(float, w[r].z << 16), acc[r]);
+        acc[r] = fmaf(x1.y, __builtin_bit_cast(float, w[r].z & 0xffff0000u), acc[r]);
+        acc[r] = fmaf(x1.z, __builtin_bit_cast(float, w[r].w << 16), acc[r]);
+        acc[r] = fmaf(x1.w, __builtin_bit_cast(float, w[r].w & 0xffff0000u), acc[r]);
+    }
+}
+template <int LPR>
+__device__ __forceinline__ float lanes_sum(float v) {
+    v = row_sum(v);
+    return LPR == 64 ? rows_sum(v) : v;
+}
+
+struct UpK {
+    ExpertsUp a;
+    int kp, groups;
+};
+
+template <int LPR, int R, int U>
+__global__ __launch_bounds__(256) void k_experts_up(UpK p) {
+    extern __shared__ __attribute__((aligned(16))) float xs[];
+    const ExpertsUp &a = p.a;
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, b = blockIdx.y, sub = lane / LPR, l = lane % LPR;
+    constexpr int G = 64 / LPR, CH = LPR * 8;
+    stage(a.x, a.cols, p.kp, xs);
+    int mine;
+    float weight;
+    choose(a.logits, a.experts, a.top, a.scale, mine, weight);
+    if (blockIdx.x == 0 && b == 0 && wave == 0 && lane < a.top) a.ids[lane] = mine;
+    const int e = __builtin_amdgcn_readlane(mine, b);
+    const float scale = __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, weight), b));
+    const uint16_t *wb = a.w + (size_t)e * a.rows * a.ld;
+    const int last = a.cols - 8;
+    u32x4 w[U][R];
+    auto fetch = [&](int grp, int k0) {
+#pragma unroll
+        for (int r = 0; r < R; ++r) {
+            const uint16_t *wr = wb + (size_t)min((grp * G + sub) * R + r, a.rows - 1) * a.ld;
+#pragma unroll
+            for (int u = 0; u < U; ++u) w[u][r] = __builtin_nontemporal_load(reinterpret_cast<const u32x4 *>(wr + min(k0 + (u * LPR + l) * 8, last)));
+        }
+    };
+    int g = blockIdx.x * 4 + wave;
+    if (g < p.groups) fetch(g, 0);
+    __syncthreads();
+    const int n_wg = gridDim.x;
+    for (; g < p.groups; g += n_wg * 4) {
+        float acc[R];
+#pragma unroll
+        for (int r = 0; r < R; ++r) acc[r] = 0.f;
+        for (int k0 = 0; k0 < p.kp; k0 += CH * U) {
+            u32x4 c[U][R];
+#pragma unroll
+            for (int u = 0; u < U; ++u)
+#pragma unroll
+                for (int r = 0; r < R; ++r) c[u][r] = w[u][r];
+            if (k0 + CH * U < p.kp)
+                fetch(g, k0 + CH * U);
+            else if (g + n_wg * 4 < p.groups)
+                fetch(g + n_wg * 4, 0);
+#pragma unroll
+            for (int u = 0; u < U; ++u) multiply8<R>(c[u], xs + k0 + (u * LPR + l) * 8, acc);
+        }
+#pragma unroll
+        for (int r = 0; r < R; ++r) {
+            const float v = lanes_sum<LPR>(acc[r]);
+            const int row = (g * G + sub) * R + r;
+            if (l == 0 && row < a.rows) a.y[(size_t)b * a.ldy + row] = scale * activate(v, a.act);
+        }
+    }
+}
+
+struct OutK {
+    ExpertsOut a;
+    int c0, ce, chunks;  // chunks of the first segment, of an expert's, of all (rounded up to whole steps)
+    unsigned magic;      // ceil(2^20 / ce)
+    int groups;
+};
+
+template <int LPR, int R, int U>
+__global__ __launch_bounds__(256) void k_experts_out(OutK p) {
+    extern __shared__ __attribute__((aligned(16))) float xs[];
+    const ExpertsOut &a = p.a;
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, sub = lane / LPR, l = lane % LPR;
+    constexpr int G = 64 / LPR, CH = LPR * 8;
+    const int ids = lane < a.top ? a.ids[lane] : 0;
+    u32x4 w[U][R];
+    auto fetch = [&](int grp, int chunk0) {
+#pragma unroll
+        for (int u = 0; u < U; ++u) {
+            const int c = chunk0 + u, x = max(c - p.c0, 0);
+            const int q = min((int)((unsigned)x * p.magic >> 20), a.top - 1), e = __builtin_amdgcn_readlane(ids, q);
+            const bool first = c < p.c0;
+            const uint16_t *base = first ? a.w0 : a.w1 + (size_t)e * a.rows * a.ld1;
+            const int ld = first ? a.ld0 : a.ld1, col = min((first ? c : x - q * p.ce) * CH + l * 8, (first ? a.cols0 : a.cols1) - 8);
+#pragma unroll
+            for (int r = 0; r < R; ++r)
+                w[u][r] = __builtin_nontemporal_load(reinterpret_cast<const u32x4 *>(base + (size_t)min((grp * G + sub) * R + r, a.rows - 1) * ld + col));
+        }
+    };
+    int g = blockIdx.x * 4 + wave;
+    if (g < p.groups) fetch(g, 0);
+    stage(a.x0, a.cols0, p.c0 * CH, xs);
+    for (int k = 0; k < a.top; ++k) stage(a.x1 + (size_t)k * a.ldx1, a.cols1, p.ce * CH, xs + (p.c0 + k * p.ce) * CH);
+    for (int i = (p.c0 + a.top * p.ce) * CH + tid; i < p.chunks * CH; i += 256) xs[i] = 0.f;
+    __syncthreads();
+    const int n_wg = gridDim.x;
+    for (; g < p.groups; g += n_wg * 4) {
+        float acc[R];
+#pragma unroll
+        for (int r = 0; r < R; ++r) acc[r] = 0.f;
+        for (int c0 = 0; c0 < p.chunks; c0 += U) {
+            u32x4 c[U][R];
+#pragma unroll
+            for (int u = 0; u < U; ++u)
+#pragma unroll
+                for (int r = 0; r < R; ++r) c[u][r] = w[u][r];
+            if (c0 + U < p.chunks)
+                fetch(g, c0 + U);
+            else if (g + n_wg * 4 < p.groups)
+                fetch(g + n_wg * 4, 0);
+#pragma unroll
+            for (int u = 0; u < U; ++u) multiply8<R>(c[u], xs + (c0 + u) * CH + l * 8, acc);
+        }
+#pragma unroll
+        for (int r = 0; r < R; ++r) {
+            const float v = lanes_sum<LPR>(acc[r]);
+            const int row = (g * G + sub) * R + r;
+            if (l == 0 && row < a.rows) a.y[row] = v + (a.bias ? a.bias[row] : 0.f);
+        }
+    }
+}
+
+// workgroups of a product: all of them at once up to three per CU, whole rounds of row groups beyond
+static int gemv_grid(int groups, int share) {
+    int n = (groups + 3) / 4;
+    const int cap = share > 1 ? (768 + share - 1) / share : 768;
+    if (n > cap) {
+        const int rounds = (n + cap - 1) / cap;
+        n = (n + rounds - 1) / rounds;
+    }
+    return n;
+}
+
+template <int LPR, int R>
+static hipError_t up_go(const ExpertsUp &a, int chunks, hipStream_t s) {
+    UpK k;
+    k.a = a;
+    const int u = chunks % 5 == 0 ? 5 : chunks >= 3 ? 3 : chunks;
+    k.kp = (chunks + u - 1) / u * u * LPR * 8;
+    k.groups = (a.rows + 64 / LPR * R - 1) / (64 / LPR * R);
+    if ((size_t)k.kp * 4 > 150 * 1024) return hipErrorInvalidValue;
+    auto fn = u == 1 ? k_experts_up<LPR, R, 1> : u == 2 ? k_experts_up<LPR, R, 2> : u == 3 ? k_experts_up<LPR, R, 3> : k_experts_up<LPR, R, 5>;
+    const size_t lds = (size_t)k.kp * 4;
+    if (lds > 65536) {
+        const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(fn), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+        if (e != hipSuccess) return e;
+    }
+    hipLaunchKernelGGL(fn, dim3(gemv_grid(k.groups, a.top), a.top), dim3(256), lds, s, k);
+    return hipGetLastError();
+}
+
+hipError_t launch_experts_up(const ExpertsUp &a, hipStream_t s) {
+    if (a.cols <= 256) return up_go<16, 1>(a, (a.cols + 127) / 128, s);
+    const int chunks = (a.cols + 511) / 512;
+    return (long)a.rows * a.top >= 4096 ? up_go<64, 2>(a, chunks, s) : up_go<64, 1>(a, chunks, s);
+}
+
+template <int LPR, int R>
+static hipError_t out_go(const ExpertsOut &a, hipStream_t s) {
+    OutK k;
+    k.a = a;
+    constexpr int CH = LPR * 8;
+    k.c0 = (a.cols0 + CH - 1) / CH, k.ce = (a.cols1 + CH - 1) / CH;
+    const int chunks = k.c0 + a.top * k.ce, u = chunks >= 4 ? 4 : chunks == 3 ? 3 : 2;
+    k.chunks = (chunks + u - 1) / u * u;
+    k.magic = ((1u << 20) + k.ce - 1) / k.ce;
+    k.groups = (a.rows + 64 / LPR * R - 1) / (64 / LPR * R);
+    const size_t lds = (size_t)k.chunks * CH * 4;
+    // (the quotient by multiplication holds while chunks * ce stays below 2^20)
+    if (lds > 150 * 1024 || (long)k.chunks * k.ce >= 1 << 20) return hipErrorInvalidValue;
+    auto fn = u == 2 ? k_experts_out<LPR, R, 2> : u == 3 ? k_experts_out<LPR, R, 3> : k_experts_out<LPR, R, 4>;
+    if (lds > 65536) {
+        const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(fn), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+        if (e != hipSuccess) return e;
+    }
+    hipLaunchKernelGGL(fn, dim3(gemv_grid(k.groups, 1)), dim3(256), lds, s, k);
+    return hipGetLastError();
+}
+
+hipError_t launch_experts_out(const ExpertsOut &a, hipStream_t s) {
+    auto waste = [&](int ch) { return (double)((a.cols0 + ch - 1) / ch * ch + (long)a.top * ((a.cols1 + ch - 1) / ch * ch)) / (a.cols0 + (double)a.top * a.cols1); };
+    // whole-wave rows unless their chunks are mostly padding
+    return waste(512) > 1.6 * waste(128) ? out_go<16, 1>(a, s) : out_go<64, 1>(a, s);
+}
+
+}  // namespace bitnet_hip

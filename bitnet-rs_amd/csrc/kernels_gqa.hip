@@ -1,0 +1,594 @@
+// kernels_gqa.hip -- causal attention whose query heads share keys and values in groups, with one softmax map per head or two (gfx950).
+//
+// Two maps (differential attention) weigh the same values; a head's output is a1 - lambda a2, divided by its root mean square over the value
+// columns.  Caches: keys [kv head][map][capacity][dimp], values transposed [kv head][vdimp][capacity].
+//   k_gqa_rows     rows of projections: query and key norms, the query's factor at its position, keys and values into the caches
+//   k_gqa_prefill  a prompt's portion: flash attention on S^T = K Q^T and O^T = V^T P^T, both maps of a query tile in one wave
+//   k_gqa_step     the decode step: norms and append in the same launch, 32 keys per wave and step on the matrix cores
+//   k_gqa_any      any size, f32 or bf16 cache, one wave per key
+//   k_gqa_merge    records of the decode forms -> output
+// Scores, maxima, sums and weights are f32; a weight (and the decode step's query) enters the matrix cores as a (high, low) pair of bf16 values.
+// Scores are kept in base 2: the score times log2(e).
+#include "dense.hpp"
+
+namespace bitnet_hip {
+
+constexpr float kLog2e = 1.44269504088896f;
+
+__device__ __forceinline__ void gqa_split(int n_keys, int &per, int &used) {
+    const int tiles = (n_keys + kGqaTile - 1) / kGqaTile;
+    per = (tiles + kGqaSplits - 1) / kGqaSplits;
+    used = (tiles + per - 1) / per;
+}
+
+size_t gqa_scratch_floats(size_t heads, size_t maps, size_t vdimp, size_t nq) { return nq * heads * maps * kGqaSplits * (kGqaRecHead + vdimp); }
+bool gqa_supported(int dimp, int vdimp) { return dimp <= 256 && vdimp <= 256; }
+
+// ---- rows of projections ----------------------------------------------------------------------------------------------
+// blockIdx.y: query heads x maps, key heads x maps, value heads; 64 tokens per workgroup
+template <class TR, class TC>
+__global__ __launch_bounds__(256) void k_gqa_rows(Gqa p, TR *rows, size_t ld, const int *pos_ptr, int n) {
+    extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, pos0 = *pos_ptr, t0 = blockIdx.x * 64;
+    const int nq = (int)(p.heads * p.maps), nk = (int)(p.kv_heads * p.maps), dim = (int)p.dim, dimp = (int)p.dimp, vdimp = (int)p.vdimp;
+    int y = blockIdx.y;
+    if (y < nq + nk) {
+        const bool key = y >= nq;
+        const float *w = key ? p.k_weight : p.q_weight;
+        TC *cache = key ? (TC *)p.kcache + (size_t)(y - nq) * p.capacity * dimp : nullptr;
+        for (int t = t0 + wave; t < min(t0 + 64, n); t += 4) {
+            TR *row = rows + (size_t)t * ld + (size_t)y * dimp;
+            float ss = 0.f;
+            for (int i = lane; i < dimp; i += 64) {
+                const float v = ld_act(row, i);
+                ss += v * v;
+            }
+            const float norm = w ? 1.0f / sqrtf(wave_sum(ss) / (float)dim + p.eps) : 1.0f;
+            const float factor = key ? norm : norm * p.q_factor[pos0 + t];
+            for (int i = lane; i < dimp; i += 64) {
+                const float v = ld_act(row, i) * factor * (w && i < dim ? w[i] : 1.0f);  // (padding columns hold zeros)
+                if (key)
+                    st_act(cache + (size_t)(pos0 + t) * dimp, i, v);
+                else
+                    st_act(row, i, v);
+            }
+        }
+        return;
+    }
+    y -= nq + nk;
+    TR *tile = (TR *)lds;  // [64][vdimp + 2]
+    const int stride = vdimp + 2, count = min(64, n - t0);
+    const TR *src = rows + (size_t)(nq + nk) * dimp + (size_t)y * vdimp;
+    for (int i = tid; i < count * vdimp; i += 256) {
+        const int t = i / vdimp, v = i - t * vdimp;
+        tile[t * stride + v] = src[(size_t)(t0 + t) * ld + v];
+    }
+    __syncthreads();
+    TC *cache = (TC *)p.vcache + (size_t)y * vdimp * p.capacity + pos0 + t0;
+    if (lane < count)
+        for (int v = wave; v < vdimp; v += 4) st_act(cache + (size_t)v * p.capacity, lane, ld_act(tile, lane * stride + v));
+}
+
+hipError_t launch_gqa_rows(const Gqa &g, void *rows, size_t ld, int rows_f32, int cache_f32, const int *pos, int n, hipStream_t s) {
+    const dim3 grid((n + 63) / 64, g.heads * g.maps + g.kv_heads * g.maps + g.kv_heads);
+    const size_t lds = 64 * (g.vdimp + 2) * (rows_f32 ? 4 : 2);
+    if (lds > 160 * 1024) return hipErrorInvalidValue;
+    auto go = [&](auto fn, auto *r) {
+        if (lds > 65536) {
+            const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(fn), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+            if (e != hipSuccess) return e;
+        }
+        hipLaunchKernelGGL(fn, grid, dim3(256), lds, s, g, r, ld, pos, n);
+        return hipGetLastError();
+    };
+    if (rows_f32) return cache_f32 ? go(k_gqa_rows<float, float>, (float *)rows) : go(k_gqa_rows<float, uint16_t>, (float *)rows);
+    return cache_f32 ? hipErrorInvalidValue : go(k_gqa_rows<uint16_t, uint16_t>, (uint16_t *)rows);
+}
+
+// ---- any size ---------------------------------------------------------------------------------------------------------
+// One workgroup per (record, head and map, query); a wave takes every fourth key, its lanes the columns.
+template <class TQ, class TC, int ND, int NV>
+__global__ __launch_bounds__(256) void k_gqa_any(Gqa p, const TQ *q, size_t ldq, const int *pos_ptr, int q0, float *scratch) {
+    extern __shared__ __attribute__((aligned(16))) float vec[];  // [4][vdimp]
+    __shared__ float sm[4], sl[4];
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, hm = blockIdx.y, qi = blockIdx.z;
+    const int maps = (int)p.maps, h = hm / maps, map = hm - h * maps, kv = h / (int)(p.heads / p.kv_heads), dimp = (int)p.dimp, vdimp = (int)p.vdimp;
+    const int n_keys = *pos_ptr + q0 + qi + 1;
+    int per, used;
+    gqa_split(n_keys, per, used);
+    if ((int)blockIdx.x >= used) return;
+    const int k0 = blockIdx.x * per * kGqaTile, k1 = min(k0 + per * kGqaTile, n_keys);
+    const TQ *qr = q + (size_t)qi * ldq + (size_t)hm * dimp;
+    const TC *K = (const TC *)p.kcache + (size_t)(kv * maps + map) * p.capacity * dimp, *V = (const TC *)p.vcache + (size_t)kv * vdimp * p.capacity;
+    float qv[ND], acc[NV];
+#pragma unroll
+    for (int j = 0; j < ND; ++j) qv[j] = lane + 64 * j < dimp ? ld_act(qr, lane + 64 * j) : 0.f;
+#pragma unroll
+    for (int j = 0; j < NV; ++j) acc[j] = 0.f;
+    float m = -INFINITY, l = 0.f;
+    for (int key = k0 + wave; key < k1; key += 4) {
+        float s = 0.f;
+#pragma unroll
+        for (int j = 0; j < ND; ++j)
+            if (lane + 64 * j < dimp) s += qv[j] * ld_act(K + (size_t)key * dimp, lane + 64 * j);
+        s = wave_sum(s) * kLog2e;
+        const float mn = fmaxf(m, s), al = exp2f(m - mn), w = exp2f(s - mn);
+        l = l * al + w;
+        m = mn;
+#pragma unroll
+        for (int j = 0; j < NV; ++j)
+            if (lane + 64 * j < vdimp) acc[j] = acc[j] * al + w * ld_act(V + (size_t)(lane + 64 * j) * p.capacity, key);
+    }
+    if (lane == 0) sm[wave] = m, sl[wave] = l;
+#pragma unroll
+    for (int j = 0; j < NV; ++j)
+        if (lane + 64 * j < vdimp) vec[wave * vdimp + lane + 64 * j] = acc[j];
+    __syncthreads();
+    const float M = fmaxf(fmaxf(sm[0], sm[1]), fmaxf(sm[2], sm[3]));
+    float w[4], L = 0.f;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {
+        w[i] = sm[i] == -INFINITY ? 0.f : exp2f(sm[i] - M);
+        L += w[i] * sl[i];
+    }
+    float *rec = scratch + (((size_t)qi * p.heads * maps + hm) * kGqaSplits + blockIdx.x) * (kGqaRecHead + vdimp);
+    for (int i = tid; i < vdimp; i += 256)
+        rec[kGqaRecHead + i] = (w[0] * vec[i] + w[1] * vec[vdimp + i]) + (w[2] * vec[2 * vdimp + i] + w[3] * vec[3 * vdimp + i]);
+    if (tid == 0) rec[0] = M, rec[1] = L;
+}
+
+template <class TQ, class TC>
+static hipError_t any_go(const Gqa &g, const void *q, size_t ldq, const int *pos, int q0, int nq, float *scratch, hipStream_t s) {
+    const int splits = min(kGqaSplits, (int)((g.capacity + kGqaTile - 1) / kGqaTile));
+    const size_t lds = 4 * g.vdimp * sizeof(float);
+    if (g.dimp > 1024 || g.vdimp > 1024) return hipErrorInvalidValue;
+    auto fn = g.dimp <= 64 && g.vdimp <= 64 ? k_gqa_any<TQ, TC, 1, 1> : g.dimp <= 256 && g.vdimp <= 256 ? k_gqa_any<TQ, TC, 4, 4> : k_gqa_any<TQ, TC, 16, 16>;
+    hipLaunchKernelGGL(fn, dim3(splits, g.heads * g.maps, nq), dim3(256), lds, s, g, (const TQ *)q, ldq, pos, q0, scratch);
+    return hipGetLastError();
+}
+
+hipError_t launch_gqa_any(const Gqa &g, const void *q, size_t ldq, int q_f32, int cache_f32, const int *pos, int q0, int nq, float *scratch, hipStream_t s) {
+    if (q_f32) return cache_f32 ? any_go<float, float>(g, q, ldq, pos, q0, nq, scratch, s) : any_go<float, uint16_t>(g, q, ldq, pos, q0, nq, scratch, s);
+    return cache_f32 ? hipErrorInvalidValue : any_go<uint16_t, uint16_t>(g, q, ldq, pos, q0, nq, scratch, s);
+}
+
+// ---- decode step, matrix cores ----------------------------------------------------------------------------------------
+// One workgroup per (record, kv head and 16 of its query heads), four waves; a wave takes every fourth block of 32 keys by itself, with maximum,
+// sum and output of its own, and the four meet at the end.  S^T = K Q^T: row 4 g + e of score tile t is key 8 g + 4 t + e of the block, so that a
+// lane's weights of both tiles are the eight consecutive keys 8 g .. 8 g + 7 which it needs as an operand of O^T = V^T P^T.
+template <int NK, int NV, int MAPS>
+__global__ __launch_bounds__(256, NV > 8 ? 1 : 2) void k_gqa_step(Gqa p, GqaStep a) {
+    extern __shared__ __attribute__((aligned(16))) float area[];  // queries [maps][16][NK * 32]; then the waves' outputs
+    __shared__ float sm[4][MAPS][16], sl[4][MAPS][16];
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r16 = lane & 15, g = lane >> 4;
+    const int group = (int)(p.heads / p.kv_heads), ht = (group + 15) / 16, kv = blockIdx.y / ht, h0 = kv * group + (blockIdx.y - kv * ht) * 16;
+    const int nh = min(16, (kv + 1) * group - h0), dim = (int)p.dim, dimp = (int)p.dimp, vdimp = (int)p.vdimp;
+    constexpr int QS = NK * 32 + 4;
+    const int pos = *a.pos, n_keys = pos + 1;
+    int per, used;
+    gqa_split(n_keys, per, used);
+    if ((int)blockIdx.x >= used) return;
+    const int k0 = blockIdx.x * per * kGqaTile, k1 = min(k0 + per * kGqaTile, n_keys);
+    uint16_t *K = (uint16_t *)p.kcache + (size_t)kv * MAPS * p.capacity * dimp, *V = (uint16_t *)p.vcache + (size_t)kv * vdimp * p.capacity;
+    const float *kraw = a.row + (p.heads * MAPS + (size_t)kv * MAPS) * dimp, *vraw = a.row + (p.heads + p.kv_heads) * MAPS * dimp + (size_t)kv * vdimp;
+    if (k1 == n_keys) {  // the record that holds the new position appends it
+        if (wave < MAPS) {
+            float v[NK], ss = 0.f;
+#pragma unroll
+            for (int j = 0; j < (NK + 1) / 2; ++j) {
+                v[j] = lane + 64 * j < dimp ? kraw[wave * dimp + lane + 64 * j] : 0.f;
+                ss += v[j] * v[j];
+            }
+            const float norm = p.k_weight ? 1.0f / sqrtf(wave_sum(ss) / (float)dim + p.eps) : 1.0f;
+#pragma unroll
+            for (int j = 0; j < (NK + 1) / 2; ++j) {
+                const int i = lane + 64 * j;
+                if (i < dimp) K[((size_t)wave * p.capacity + pos) * dimp + i] = f2bf(v[j] * norm * (p.k_weight && i < dim ? p.k_weight[i] : 1.0f));
+            }
+        }
+        for (int i = tid; i < vdimp; i += 256) V[(size_t)i * p.capacity + pos] = f2bf(vraw[i]);
+    }
+    {
+        const float factor = p.q_factor[pos];
+        for (int r = wave; r < MAPS * 16; r += 4) {
+            const int map = r >> 4, hh = r & 15;
+            const float *q = a.row + ((size_t)(h0 + min(hh, nh - 1)) * MAPS + map) * dimp;
+            float v[NK], ss = 0.f;
+#pragma unroll
+            for (int j = 0; j < (NK + 1) / 2; ++j) {
+                v[j] = lane + 64 * j < dimp && hh < nh ? q[lane + 64 * j] : 0.f;
+                ss += v[j] * v[j];
+            }
+            const float norm = (p.q_weight ? 1.0f / sqrtf(wave_sum(ss) / (float)dim + p.eps) : 1.0f) * factor;
+#pragma unroll
+            for (int j = 0; j < (NK + 1) / 2; ++j) {
+                const int i = lane + 64 * j;
+                if (i < NK * 32) area[r * QS + i] = v[j] * norm * (p.q_weight && i < dim ? p.q_weight[i] : 1.0f);
+            }
+        }
+    }
+    __syncthreads();  // queries; and the appended rows are there for every wave of this workgroup
+    SplitFrag q[MAPS][NK];
+#pragma unroll
+    for (int m = 0; m < MAPS; ++m)
+#pragma unroll
+        for (int kk = 0; kk < NK; ++kk) {
+            const float *src = area + (m * 16 + r16) * QS + kk * 32 + g * 8;
+            q[m][kk] = split8(*reinterpret_cast<const f32x4 *>(src), *reinterpret_cast<const f32x4 *>(src + 4));
+        }
+    __syncthreads();  // (the area is used again)
+    f32x4 o[NV][MAPS];
+    float m[MAPS], l[MAPS];
+#pragma unroll
+    for (int j = 0; j < MAPS; ++j) {
+        m[j] = -INFINITY, l[j] = 0.f;
+#pragma unroll
+        for (int v = 0; v < NV; ++v) o[v][j] = f32x4{0.f, 0.f, 0.f, 0.f};
+    }
+    for (int kb = k0 + wave * 32; kb < k1; kb += 128) {  // (blocks lie below the capacity, a multiple of 128)
+        u32x4 kf[2][MAPS][NK], vf[NV];
+#pragma unroll
+        for (int t = 0; t < 2; ++t)
+#pragma unroll
+            for (int j = 0; j < MAPS; ++j)
+#pragma unroll
+                for (int kk = 0; kk < NK; ++kk)
+                    kf[t][j][kk] = *reinterpret_cast<const u32x4 *>(K + ((size_t)j * p.capacity + kb + (r16 >> 2) * 8 + t * 4 + (r16 & 3)) * dimp + min(kk * 32, dimp - 32) + g * 8);
+#pragma unroll
+        for (int v = 0; v < NV; ++v) vf[v] = *reinterpret_cast<const u32x4 *>(V + (size_t)min(v * 16 + r16, vdimp - 1) * p.capacity + kb + g * 8);
+#pragma unroll
+        for (int j = 0; j < MAPS; ++j) {
+            f32x4 s[2];
+#pragma unroll
+            for (int t = 0; t < 2; ++t) {
+                f32x4 hi = f32x4{0.f, 0.f, 0.f, 0.f}, lo = hi;
+#pragma unroll
+                for (int kk = 0; kk < NK; ++kk) {  // (steps past dimp: the query is zero there)
+                    hi = mfma_bf16(__builtin_bit_cast(bf16x8, kf[t][j][kk]), q[j][kk].hi, hi);
+                    lo = mfma_bf16(__builtin_bit_cast(bf16x8, kf[t][j][kk]), q[j][kk].lo, lo);
+                }
+                s[t] = (hi + lo) * kLog2e;
+#pragma unroll
+                for (int e = 0; e < 4; ++e) s[t][e] = kb + g * 8 + t * 4 + e < k1 ? s[t][e] : -INFINITY;
+            }
+            float mx = fmaxf(fmaxf(fmaxf(s[0][0], s[0][1]), fmaxf(s[0][2], s[0][3])), fmaxf(fmaxf(s[1][0], s[1][1]), fmaxf(s[1][2], s[1][3])));
+            mx = fmaxf(m[j], rows_max(mx));
+            const float al = exp2f(m[j] - mx);
+            m[j] = mx;
+            f32x4 w[2];
+#pragma unroll
+            for (int t = 0; t < 2; ++t)
+#pragma unroll
+                for (int e = 0; e < 4; ++e) w[t][e] = exp2f(s[t][e] - mx);
+            l[j] = l[j] * al + ((w[0][0] + w[0][1]) + (w[0][2] + w[0][3])) + ((w[1][0] + w[1][1]) + (w[1][2] + w[1][3]));
+            const SplitFrag pf = split8(w[0], w[1]);
+#pragma unroll
+            for (int v = 0; v < NV; ++v) {
+                o[v][j] *= al;
+                o[v][j] = mfma_bf16(__builtin_bit_cast(bf16x8, vf[v]), pf.hi, o[v][j]);
+                o[v][j] = mfma_bf16(__builtin_bit_cast(bf16x8, vf[v]), pf.lo, o[v][j]);
+            }
+        }
+    }
+#pragma unroll
+    for (int j = 0; j < MAPS; ++j) {
+        const float t = rows_sum(l[j]);
+        if (g == 0) sm[wave][j][r16] = m[j], sl[wave][j][r16] = t;
+    }
+    __syncthreads();
+#pragma unroll
+    for (int j = 0; j < MAPS; ++j) {
+        const float M = fmaxf(fmaxf(sm[0][j][r16], sm[1][j][r16]), fmaxf(sm[2][j][r16], sm[3][j][r16]));
+        const float w = m[j] == -INFINITY ? 0.f : exp2f(m[j] - M);
+        if (r16 < nh)
+#pragma unroll
+            for (int v = 0; v < NV; ++v)
+                if (v * 16 < vdimp) *reinterpret_cast<f32x4 *>(area + ((size_t)(wave * MAPS + j) * nh + r16) * vdimp + v * 16 + g * 4) = o[v][j] * w;
+    }
+    __syncthreads();
+    const int v4 = vdimp / 4, rows = MAPS * nh;
+    for (int i = tid; i < rows * v4; i += 256) {
+        const int r = i / v4, c = (i - r * v4) * 4, j = r / nh, hh = r - j * nh;
+        const float *src = area + (size_t)r * vdimp + c;
+        const size_t step = (size_t)rows * vdimp;
+        const f32x4 sum = (*reinterpret_cast<const f32x4 *>(src) + *reinterpret_cast<const f32x4 *>(src + step)) +
+                          (*reinterpret_cast<const f32x4 *>(src + 2 * step) + *reinterpret_cast<const f32x4 *>(src + 3 * step));
+        float *rec = a.scratch + ((size_t)((h0 + hh) * MAPS + j) * kGqaSplits + blockIdx.x) * (kGqaRecHead + vdimp);
+        *reinterpret_cast<f32x4 *>(rec + kGqaRecHead + c) = sum;
+        if (c == 0) {
+            const float M = fmaxf(fmaxf(sm[0][j][hh], sm[1][j][hh]), fmaxf(sm[2][j][hh], sm[3][j][hh]));
+            float L = 0.f;
+#pragma unroll
+            for (int w = 0; w < 4; ++w) L += sm[w][j][hh] == -INFINITY ? 0.f : exp2f(sm[w][j][hh] - M) * sl[w][j][hh];
+            rec[0] = M, rec[1] = L;
+        }
+    }
+}
+
+template <int NK, int NV>
+static hipError_t step_go(const Gqa &g, const GqaStep &a, hipStream_t s) {
+    const int splits = min(kGqaSplits, (int)((g.capacity + kGqaTile - 1) / kGqaTile)), group = (int)(g.heads / g.kv_heads), nh = min(16, group);
+    const size_t queries = g.maps * 16 * (NK * 32 + 4), outs = 4 * g.maps * nh * g.vdimp, lds = (queries > outs ? queries : outs) * sizeof(float);
+    auto fn = g.maps == 2 ? k_gqa_step<NK, NV, 2> : k_gqa_step<NK, NV, 1>;
+    if (lds > 65536) {
+        const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(fn), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+        if (e != hipSuccess) return e;
+    }
+    hipLaunchKernelGGL(fn, dim3(splits, g.kv_heads * ((group + 15) / 16)), dim3(256), lds, s, g, a);
+    return hipGetLastError();
+}
+
+hipError_t launch_gqa_step(const Gqa &g, const GqaStep &a, hipStream_t s) {
+    if (!gqa_supported((int)g.dimp, (int)g.vdimp)) return hipErrorInvalidValue;
+    if (g.dimp <= 64 && g.vdimp <= 64) return step_go<2, 4>(g, a, s);
+    if (g.dimp <= 64 && g.vdimp <= 128) return step_go<2, 8>(g, a, s);
+    if (g.dimp <= 128 && g.vdimp <= 128) return step_go<4, 8>(g, a, s);
+    return step_go<8, 16>(g, a, s);
+}
+
+// ---- records -> output ------------------------------------------------------------------------------------------------
+template <class TO>
+__global__ __launch_bounds__(256) void k_gqa_merge(Gqa p, const int *pos_ptr, int q0, const float *scratch, TO *out, size_t ldo) {
+    extern __shared__ __attribute__((aligned(16))) float part[];  // [maps][2][vdimp]
+    static_assert(kGqaSplits == 128, "two records per lane of a wave");
+    __shared__ float ws[2][kGqaSplits], sinv[2], slot[4];
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, h = blockIdx.x, qi = blockIdx.z, maps = (int)p.maps, vdimp = (int)p.vdimp;
+    int per, used;
+    gqa_split(*pos_ptr + q0 + qi + 1, per, used);
+    const size_t stride = kGqaRecHead + vdimp;
+    const float *rec = scratch + ((size_t)qi * p.heads + h) * maps * kGqaSplits * stride;
+    if (wave < maps) {
+        const float *r = rec + (size_t)wave * kGqaSplits * stride;
+        float mv[2], lv[2];
+#pragma unroll
+        for (int e = 0; e < 2; ++e) {
+            const int i = lane + 64 * e;
+            mv[e] = i < used ? r[i * stride] : -INFINITY;
+            lv[e] = i < used ? r[i * stride + 1] : 0.f;
+        }
+        const float M = rows_max(row_max(fmaxf(mv[0], mv[1])));
+        float den = 0.f;
+#pragma unroll
+        for (int e = 0; e < 2; ++e) {
+            const float w = lane + 64 * e < used ? exp2f(mv[e] - M) : 0.f;
+            ws[wave][lane + 64 * e] = w;
+            den += w * lv[e];
+        }
+        den = wave_sum(den);
+        if (lane == 0) sinv[wave] = 1.0f / den;
+    }
+    __syncthreads();
+    // 32 lanes of four columns; eight groups share maps and records
+    const int grp = tid >> 5, gm = maps == 2 ? grp & 1 : 0, gs = maps == 2 ? grp >> 1 : grp, gn = maps == 2 ? 4 : 8;
+    for (int i = (tid & 31) * 4; i < vdimp; i += 128) {
+        const float *r = rec + (size_t)gm * kGqaSplits * stride + kGqaRecHead + i;
+        f32x4 acc = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll 8
+        for (int k = gs; k < used; k += gn) acc += ws[gm][k] * *reinterpret_cast<const f32x4 *>(r + k * stride);
+        *reinterpret_cast<f32x4 *>(part + (size_t)grp * vdimp + i) = acc;
+    }
+    __syncthreads();
+    float v = 0.f;
+    const bool live = tid < vdimp;  // (vdimp <= 256; wider heads loop below)
+    TO *dst = out + (size_t)qi * ldo + (size_t)h * vdimp;
+    auto value = [&](int i) {
+        if (maps == 1) {
+            float t = 0.f;
+#pragma unroll
+            for (int k = 0; k < 8; ++k) t += part[k * vdimp + i];
+            return t * sinv[0];
+        }
+        const float a = (part[i] + part[2 * vdimp + i]) + (part[4 * vdimp + i] + part[6 * vdimp + i]);
+        const float b = (part[vdimp + i] + part[3 * vdimp + i]) + (part[5 * vdimp + i] + part[7 * vdimp + i]);
+        return a * sinv[0] - p.lambda * (b * sinv[1]);
+    };
+    if (vdimp <= 256) {
+        v = live ? value(tid) : 0.f;
+        if (maps == 2) v *= p.out_scale / sqrtf(group_sum<4>(v * v, slot) / (float)p.vdim + p.eps);
+        if (live) st_act(dst, tid, v);
+        return;
+    }
+    float ss = 0.f, f = 1.0f;
+    for (int i = tid; i < vdimp; i += 256) v = value(i), ss += v * v;
+    if (maps == 2) f = p.out_scale / sqrtf(group_sum<4>(ss, slot) / (float)p.vdim + p.eps);
+    for (int i = tid; i < vdimp; i += 256) st_act(dst, i, value(i) * f);
+}
+
+hipError_t launch_gqa_merge(const Gqa &g, const int *pos, int q0, int nq, const float *scratch, void *out, size_t ldo, int out_bf16, hipStream_t s) {
+    const size_t lds = 8 * g.vdimp * sizeof(float);
+    if (lds > 65536) return hipErrorInvalidValue;
+    if (out_bf16)
+        hipLaunchKernelGGL(k_gqa_merge<uint16_t>, dim3(g.heads, 1, nq), dim3(256), lds, s, g, pos, q0, scratch, (uint16_t *)out, ldo);
+    else
+        hipLaunchKernelGGL(k_gqa_merge<float>, dim3(g.heads, 1, nq), dim3(256), lds, s, g, pos, q0, scratch, (float *)out, ldo);
+    return hipGetLastError();
+}
+
+// ---- prompt -----------------------------------------------------------------------------------------------------------
+// One workgroup: one head, four waves; a wave holds two slots of 16 queries: both maps of one query tile, or two tiles of the only map.  Key tiles
+// of 64 (every map's) and the values of the tile staged through registers into LDS one step ahead.
+template <int NK, int NV, int MAPS>
+__global__ __launch_bounds__(256, NV > 8 || NK > 4 ? 1 : 2) void k_gqa_prefill(Gqa p, const uint16_t *Q, size_t ldq, int n_ctx, int nq, uint16_t *out, size_t ldo, int n_qb) {
+    extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
+    constexpr int SLOTS = 2, QW = 16 * SLOTS / MAPS, KS = NK * 64 + 16, VS = 64 * 2 + 16, NVL = NV / 2;
+    uint8_t *lk = lds, *lv = lds + MAPS * 64 * KS;
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r16 = lane & 15, g = lane >> 4;
+    const int heads = (int)p.heads, dimp = (int)p.dimp, vdimp = (int)p.vdimp;
+    // Consecutive workgroups go to the eight XCDs in turn.  Longest blocks first; an XCD keeps heads / 8 neighbouring heads of its own (their keys
+    // and values stay in its L2), the heads left over move from XCD to XCD with the block so that all eight carry the same work.
+    const int x = blockIdx.x & 7, rest = blockIdx.x >> 3, own = heads >> 3, left = heads & 7, per = own + (left ? 1 : 0);
+    const int level = rest / per, slot = rest - level * per, r = (x + 8 * left - (level % 8) * left) & 7;
+    if (slot == own && r >= left) return;
+    const int h = slot < own ? x * own + slot : 8 * own + r, qb = n_qb - 1 - level;
+    const int kv = h / (int)(p.heads / p.kv_heads), q0 = qb * 4 * QW, pos0 = n_ctx - nq, qw = q0 + wave * QW;
+    bf16x8 qf[SLOTS][NK];
+    int qpos[SLOTS];
+#pragma unroll
+    for (int t = 0; t < SLOTS; ++t) {
+        const int tile = t / MAPS, map = t % MAPS, qi = min(qw + tile * 16 + r16, nq - 1);
+        qpos[t] = pos0 + qw + tile * 16 + r16;
+        const uint16_t *q = Q + (size_t)qi * ldq + (size_t)(h * MAPS + map) * dimp;
+#pragma unroll
+        for (int kk = 0; kk < NK; ++kk) {
+            u32x4 v = *reinterpret_cast<const u32x4 *>(q + min(kk * 32, dimp - 32) + g * 8);
+            const uint32_t keep = kk * 32 < dimp ? 0xffffffffu : 0u;
+            qf[t][kk] = __builtin_bit_cast(bf16x8, u32x4{v.x & keep, v.y & keep, v.z & keep, v.w & keep});
+        }
+    }
+    f32x4 o[NV][SLOTS];
+    float m[SLOTS], l[SLOTS];
+#pragma unroll
+    for (int t = 0; t < SLOTS; ++t) {
+        m[t] = -INFINITY, l[t] = 0.f;
+#pragma unroll
+        for (int v = 0; v < NV; ++v) o[v][t] = f32x4{0.f, 0.f, 0.f, 0.f};
+    }
+    const uint16_t *K = (const uint16_t *)p.kcache + (size_t)kv * MAPS * p.capacity * dimp, *V = (const uint16_t *)p.vcache + (size_t)kv * vdimp * p.capacity;
+    u32x4 kreg[MAPS][NK], vreg[NVL];
+    const unsigned koff = (unsigned)((tid >> 2) * dimp * 2 + (tid & 3) * 16);
+    const size_t voff = (size_t)(tid >> 3) * p.capacity * 2 + (tid & 7) * 16;
+#pragma unroll
+    for (int j = 0; j < NVL; ++j) vreg[j] = u32x4{0u, 0u, 0u, 0u};
+    auto fetch = [&](int key0) {  // (whole tiles: the capacity is a multiple of 64)
+#pragma unroll
+        for (int mp = 0; mp < MAPS; ++mp) {
+            const char *kb = (const char *)(K + ((size_t)mp * p.capacity + key0) * dimp);
+#pragma unroll
+            for (int j = 0; j < NK; ++j) kreg[mp][j] = *reinterpret_cast<const u32x4 *>(kb + min(j * 64, dimp * 2 - 64) + koff);
+        }
+        const char *vb = (const char *)(V + key0);
+#pragma unroll
+        for (int j = 0; j < NVL; ++j)
+            if (j * 32 < vdimp) vreg[j] = *reinterpret_cast<const u32x4 *>(vb + (size_t)j * 64 * p.capacity + voff);
+    };
+    const int n_tiles = (min(n_ctx, pos0 + q0 + 4 * QW) + 63) / 64;
+    fetch(0);
+    for (int kt0 = 0; kt0 < n_tiles; ++kt0) {
+        const int key0 = kt0 * 64;
+        __syncthreads();
+#pragma unroll
+        for (int mp = 0; mp < MAPS; ++mp)
+#pragma unroll
+            for (int j = 0; j < NK; ++j) *reinterpret_cast<u32x4 *>(lk + (mp * 64 + (tid >> 2)) * KS + j * 64 + (tid & 3) * 16) = kreg[mp][j];
+#pragma unroll
+        for (int j = 0; j < NVL; ++j) *reinterpret_cast<u32x4 *>(lv + ((tid >> 3) + 32 * j) * VS + (tid & 7) * 16) = vreg[j];
+        __syncthreads();
+        if (kt0 + 1 < n_tiles) fetch(key0 + 64);
+        if (key0 > pos0 + qw + QW - 1) continue;  // every key of the tile lies ahead of this wave's queries
+        f32x4 s[4][SLOTS];
+#pragma unroll
+        for (int kt = 0; kt < 4; ++kt) {
+#pragma unroll
+            for (int t = 0; t < SLOTS; ++t) s[kt][t] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+            for (int kk = 0; kk < NK; ++kk)
+#pragma unroll
+                for (int t = 0; t < SLOTS; ++t) {
+                    const bf16x8 a = *reinterpret_cast<const bf16x8 *>(lk + ((t % MAPS) * 64 + kt * 16 + r16) * KS + kk * 64 + g * 16);
+                    s[kt][t] = mfma_bf16(a, qf[t][kk], s[kt][t]);
+                }
+        }
+        if (key0 + 63 > pos0 + qw)  // the diagonal
+#pragma unroll
+            for (int t = 0; t < SLOTS; ++t)
+#pragma unroll
+                for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) s[kt][t][i] = key0 + kt * 16 + g * 4 + i > qpos[t] ? -INFINITY : s[kt][t][i];
+        float mn[SLOTS];
+        bool grows = false;
+#pragma unroll
+        for (int t = 0; t < SLOTS; ++t) {
+            float mx = fmaxf(fmaxf(s[0][t][0], s[0][t][1]), fmaxf(s[0][t][2], s[0][t][3]));
+#pragma unroll
+            for (int kt = 1; kt < 4; ++kt) mx = fmaxf(mx, fmaxf(fmaxf(s[kt][t][0], s[kt][t][1]), fmaxf(s[kt][t][2], s[kt][t][3])));
+            // (tile 0 holds a visible key for every query, so the maximum is finite from the first tile on)
+            mn[t] = fmaxf(m[t], rows_max(mx) * kLog2e);
+            grows = grows || mn[t] > m[t];
+        }
+        if (__any(grows)) {
+#pragma unroll
+            for (int t = 0; t < SLOTS; ++t) {
+                const float al = __builtin_amdgcn_exp2f(m[t] - mn[t]);
+                m[t] = mn[t];
+                l[t] *= al;
+#pragma unroll
+                for (int v = 0; v < NV; ++v) o[v][t] *= al;
+            }
+        }
+        SplitFrag pf[2][SLOTS];
+#pragma unroll
+        for (int ks = 0; ks < 2; ++ks)
+#pragma unroll
+            for (int t = 0; t < SLOTS; ++t) {
+                f32x4 w[2];
+#pragma unroll
+                for (int j = 0; j < 2; ++j) {
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) w[j][i] = __builtin_amdgcn_exp2f(fmaf(s[2 * ks + j][t][i], kLog2e, -m[t]));
+                    l[t] += (w[j][0] + w[j][1]) + (w[j][2] + w[j][3]);
+                }
+                pf[ks][t] = split8(w[0], w[1]);
+            }
+#pragma unroll
+        for (int v = 0; v < NV; ++v)
+#pragma unroll
+            for (int ks = 0; ks < 2; ++ks) {
+                const uint8_t *row = lv + (v * 16 + r16) * VS + ks * 64 + g * 8;
+                const u32x2 a0 = *reinterpret_cast<const u32x2 *>(row), a1 = *reinterpret_cast<const u32x2 *>(row + 32);
+                const bf16x8 a = __builtin_bit_cast(bf16x8, u32x4{a0.x, a0.y, a1.x, a1.y});
+#pragma unroll
+                for (int t = 0; t < SLOTS; ++t) {
+                    o[v][t] = mfma_bf16(a, pf[ks][t].hi, o[v][t]);
+                    o[v][t] = mfma_bf16(a, pf[ks][t].lo, o[v][t]);
+                }
+            }
+    }
+    float inv[SLOTS];
+#pragma unroll
+    for (int t = 0; t < SLOTS; ++t) inv[t] = 1.0f / rows_sum(l[t]);
+    if (MAPS == 2) {
+        float ss = 0.f;
+#pragma unroll
+        for (int v = 0; v < NV; ++v) {
+            o[v][0] = o[v][0] * inv[0] - (p.lambda * inv[1]) * o[v][1];
+            ss += (o[v][0].x * o[v][0].x + o[v][0].y * o[v][0].y) + (o[v][0].z * o[v][0].z + o[v][0].w * o[v][0].w);
+        }
+        inv[0] = p.out_scale / sqrtf(rows_sum(ss) / (float)p.vdim + p.eps);
+    }
+#pragma unroll
+    for (int t = 0; t < SLOTS / MAPS; ++t) {
+        const int qi = qw + t * 16 + r16;
+        if (qi >= nq) continue;
+        uint16_t *dst = out + (size_t)qi * ldo + (size_t)h * vdimp + g * 4;
+#pragma unroll
+        for (int v = 0; v < NV; ++v)
+            if (v * 16 < vdimp) {
+                const f32x4 q = o[v][t] * inv[t];
+                *reinterpret_cast<bf16x4 *>(dst + v * 16) = bf16x4{(__bf16)q.x, (__bf16)q.y, (__bf16)q.z, (__bf16)q.w};
+            }
+    }
+}
+
+template <int NK, int NV>
+static hipError_t gqa_prefill_go(const Gqa &g, const uint16_t *q, size_t ldq, int n_ctx, int nq, uint16_t *out, size_t ldo, hipStream_t s) {
+    const int rows = g.maps == 2 ? 64 : 128, n_qb = (nq + rows - 1) / rows;
+    const size_t lds = (size_t)g.maps * 64 * (NK * 64 + 16) + (size_t)NV * 16 * (64 * 2 + 16);
+    auto fn = g.maps == 2 ? k_gqa_prefill<NK, NV, 2> : k_gqa_prefill<NK, NV, 1>;
+    if (lds > 65536) {
+        const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(fn), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
+        if (e != hipSuccess) return e;
+    }
+    hipLaunchKernelGGL(fn, dim3(8 * ((g.heads + 7) / 8) * n_qb), dim3(256), lds, s, g, q, ldq, n_ctx, nq, out, ldo, n_qb);
+    return hipGetLastError();
+}
+
+hipError_t launch_gqa_prefill(const Gqa &g, const uint16_t *q, size_t ldq, int n_ctx, int nq, uint16_t *out, size_t ldo, hipStream_t s) {
+    if (!gqa_supported((int)g.dimp, (int)g.vdimp)) return hipErrorInvalidValue;
+    if (g.dimp <= 64 && g.vdimp <= 64) return gqa_prefill_go<2, 4>(g, q, ldq, n_ctx, nq, out, ldo, s);
+    if (g.dimp <= 64 && g.vdimp <= 128) return gqa_prefill_go<2, 8>(g, q, ldq, n_ctx, nq, out, ldo, s);
+    if (g.dimp <= 128 && g.vdimp <= 128) return gqa_prefill_go<4, 8>(g, q, ldq, n_ctx, nq, out, ldo, s);
+    return gqa_prefill_go<8, 16>(g, q, ldq, n_ctx, nq, out, ldo, s);
+}
+
+}  // namespace bitnet_hip

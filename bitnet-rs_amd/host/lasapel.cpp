@@ -104,7 +104,7 @@ Sequence *open_lasapel(const Json &config, const std::string &dir, const OpenOpt
     }
     std::vector<float> final_norm;
     const uint16_t *embed = t.matrix("embed", s.vocab, s.width, err), *head = embed ? t.matrix("head", s.vocab, s.width, err) : nullptr;
-    if (!head || !t.vector("final.norm", s.width, final_norm, err) || model->set_globals(embed, final_norm, head) != 0) return failed();
+    if (!head || !t.vector("final.norm", s.width, final_norm, err) || model->set_globals(embed, final_norm, {}, head, nullptr) != 0) return failed();
     return model.release();
 }
 

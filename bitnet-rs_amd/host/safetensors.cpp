@@ -107,8 +107,7 @@ bool SafeTensors::vector(const std::string &name, size_t n, std::vector<float> &
         for (size_t i = 0; i < n; ++i) {
             uint16_t h;
             memcpy(&h, t->data + 2 * i, 2);
-            const uint32_t u = (uint32_t)h << 16;
-            memcpy(&out[i], &u, 4);
+            out[i] = bf16_value(h);
         }
     }
     return true;

@@ -4,11 +4,19 @@
 
 #include <cstddef>
 #include <cstdint>
+#include <cstring>
 #include <map>
 #include <string>
 #include <vector>
 
 namespace bitnet_host {
+
+inline float bf16_value(uint16_t h) {
+    const uint32_t u = (uint32_t)h << 16;
+    float v;
+    memcpy(&v, &u, 4);
+    return v;
+}
 
 struct SafeTensor {
     std::string dtype;

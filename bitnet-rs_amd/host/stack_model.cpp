@@ -10,7 +10,7 @@
 namespace bitnet_host {
 
 namespace {
-constexpr size_t kDecodeSlice = 64;  // queries per latent-space attention call of a portion
+constexpr size_t kDecodeSlice = 64;  // queries per call where a portion takes a decode form of its attention
 size_t up_to(size_t v, size_t a) { return (v + a - 1) / a * a; }
 }  // namespace
 
@@ -35,9 +35,20 @@ StackModel::StackModel(const StackSpec &spec, bool f32, int max_pos) : spec_(spe
         err_ = "stack: empty model";
         return;
     }
+    if (plan_runs() != 0) return;
+    for (size_t i = 0; i < layers_.size(); ++i) {
+        const LayerSpec &S = spec_.layers[i];
+        const bool own = S.mixer == LayerSpec::Attention || S.mixer == LayerSpec::Delta;
+        if (S.parallel && !own) {
+            err_ = "stack: layer " + std::to_string(i) + ": side by side with the feed-forward stand attention and delta mixers only";
+            return;
+        }
+        if (own && plan_block(i, 0, true, S.parallel) != 0) return;
+        if (!S.parallel && S.experts.count > 0 && plan_block(i, 1, false, true) != 0) return;
+    }
     if (init_sequence(spec.vocab, spec.width, max_pos) != 0) return;
-    cap_ = up_to((size_t)max_pos + 1, 64);
-    size_t z = 64, q = 64, qabs = 64, att = 64, act = 64, lin = 64, lino = 64, scratch = 64;
+    cap_ = up_to((size_t)max_pos + 1, 128);
+    size_t row = 64, eact = 64, z = 64, q = 64, qabs = 64, att = 64, act = 64, lin = 64, lino = 64, scratch = 64;
     const size_t es = f32_ ? 4 : 2;
     for (size_t i = 0; i < layers_.size(); ++i) {
         Layer &L = layers_[i];
@@ -50,7 +61,8 @@ StackModel::StackModel(const StackSpec &spec, bool f32, int max_pos) : spec_(spe
             }
             if (m.kv_from >= 0) {
                 const LayerSpec *src = (size_t)m.kv_from < i ? &spec_.layers[(size_t)m.kv_from] : nullptr;
-                if (!src || src->mixer != LayerSpec::Latent || src->latent.kv_from >= 0 || src->latent.kv_rank != m.kv_rank || !(src->latent.rot == m.rot)) {
+                if (!src || src->mixer != LayerSpec::Latent || src->latent.kv_from >= 0 || src->latent.kv_rank != m.kv_rank || !(src->latent.rot == m.rot) ||
+                    layers_[(size_t)m.kv_from].slots.size() != L.slots.size()) {
                     err_ = "stack: layer " + std::to_string(i) + " reads the cache of layer " + std::to_string(m.kv_from) + ", which has none that fits";
                     return;
                 }
@@ -65,7 +77,7 @@ StackModel::StackModel(const StackSpec &spec, bool f32, int max_pos) : spec_(spe
             qabs = std::max(qabs, (size_t)m.heads * L.ldc);
             att = std::max(att, (size_t)m.heads * L.vdimp);
             scratch = std::max(scratch, bitnet_hip_latent_scratch_bytes(m.heads, L.ldc, 1) / 4);
-        } else {
+        } else if (S.mixer == LayerSpec::Linear) {
             const LinearSpec &m = S.linear;
             L.dimp = (int)up_to(m.dim, 32), L.vdimp = (int)up_to(m.vdim, 32);
             if (L.dimp > 512 || m.decay.size() != (size_t)m.heads) {
@@ -74,25 +86,38 @@ StackModel::StackModel(const StackSpec &spec, bool f32, int max_pos) : spec_(spe
             }
             lin = std::max(lin, (size_t)m.heads * 2 * (L.dimp + L.vdimp));
             lino = std::max(lino, (size_t)m.heads * L.vdimp);
+        } else if (S.mixer == LayerSpec::Attention) {
+            scratch = std::max(scratch, bitnet_hip_gqa_scratch_bytes(S.attention.heads, S.attention.maps, L.vdimp, 1) / 4);
         }
+        for (const Block &B : L.block)
+            if (B.used) {
+                row = std::max(row, (size_t)B.ko + B.fs + B.main + B.tail);
+                eact = std::max(eact, (size_t)S.experts.top * up_to(S.experts.ff, 64));
+            }
         act = std::max(act, (size_t)S.ff);
     }
-    auto alloc = [&](void **p, size_t bytes) {
-        if (hipMalloc(p, bytes) != hipSuccess || hipMemset(*p, 0, bytes) != hipSuccess) return false;
-        owned_.push_back(*p);
-        return true;
-    };
     auto vec = [&](float **p, size_t n) { return alloc((void **)p, up_to(n, 64) * 4); };
     bool ok = vec(&x_[0], width_) && vec(&x_[1], width_) && vec(&y_[0], width_) && vec(&y_[1], width_) && vec(&z_, z) && vec(&q_, q) && vec(&qabs_, qabs) &&
-              vec(&att_, att) && vec(&act_, act) && vec(&lin_, lin) && vec(&lino_, lino) && vec(&scratch_, scratch) && alloc(&argmax_, 8192);
+              vec(&att_, att) && vec(&act_, act) && vec(&lin_, lin) && vec(&lino_, lino) && vec(&scratch_, scratch) && alloc(&argmax_, 8192) && vec(&x0_, width_) && vec(&row_, row) && vec(&h_, width_) && vec(&eact_, eact) &&
+              alloc((void **)&eids_, 256);
     for (size_t i = 0; ok && i < layers_.size(); ++i) {
         Layer &L = layers_[i];
         const LayerSpec &S = spec_.layers[i];
-        if (S.mixer == LayerSpec::Latent) {
-            if (S.latent.kv_from < 0) ok = alloc(&L.cache.c, cap_ * L.ldc * es) && alloc(&L.cache.r, cap_ * L.rotp * es);
-            ok = ok && rope_tables(S.latent.rot, &L.cos, &L.sin) == 0;
-        } else {
-            ok = alloc((void **)&L.state, (size_t)S.linear.heads * L.dimp * L.vdimp * 4);
+        if (S.mixer == LayerSpec::Latent) ok = rope_tables(S.latent.rot, &L.cos, &L.sin) == 0;
+        if (S.mixer == LayerSpec::Attention) ok = query_factors(S.attention, &L.q_factor) == 0;
+        for (Slot &slot : L.slots) {
+            if (!ok) break;
+            if (S.mixer == LayerSpec::Latent && S.latent.kv_from < 0) {
+                ok = alloc(&slot.c, cap_ * L.ldc * es) && alloc(&slot.r, cap_ * L.rotp * es);
+            } else if (S.mixer == LayerSpec::Attention) {
+                const AttentionSpec &m = S.attention;
+                ok = alloc(&slot.k, cap_ * m.kv_heads * m.maps * L.dimp * es) && alloc(&slot.v, cap_ * m.kv_heads * L.vdimp * es);
+            } else if (S.mixer == LayerSpec::Linear || S.mixer == LayerSpec::Delta) {
+                const bool delta = S.mixer == LayerSpec::Delta;
+                slot.state_bytes = (size_t)(delta ? S.delta.heads : S.linear.heads) * L.dimp * L.vdimp * 4;
+                ok = alloc((void **)&slot.state, slot.state_bytes);
+                if (delta) ok = ok && alloc((void **)&slot.ring, (size_t)S.delta.taps * (2 * S.delta.kv_heads * L.dimp + S.delta.heads * L.vdimp) * 4);
+            }
         }
     }
     if (!ok) {
@@ -107,8 +132,77 @@ StackModel::~StackModel() {
     drop_graphs();
     for (void *p : owned_) hipFree(p);
     for (Buffer *b : {&px_, &ph_, &pz_, &pcq_, &pq_, &pqf_, &pqabs_, &patt_, &py_, &pact_, &pk_, &pvt_, &plin_, &plinf_, &plino_, &pgate_, &pscratch_, &plws_,
-                      &pwant_, &pxw_, &phw_, &plog_})
+                      &pwant_, &pxw_, &phw_, &plog_, &px0_, &pcat_, &prow_, &ptail_, &pqk_, &pv_, &pgates_, &pplan_, &peact_, &peout_})
         if (b->p) hipFree(b->p);
+}
+
+bool StackModel::alloc(void **p, size_t bytes) {
+    *p = nullptr;
+    if (hipMalloc(p, bytes) != hipSuccess) return false;
+    owned_.push_back(*p);
+    return hipMemset(*p, 0, bytes) == hipSuccess;
+}
+
+// the order in which layers run, and every layer's number of passes
+int StackModel::plan_runs() {
+    const int n = (int)layers_.size();
+    const LoopSpec &loop = spec_.loop;
+    if (loop.times != 0 && (loop.times < 1 || loop.start < 0 || loop.stop <= loop.start || loop.stop > n))
+        return fail_arg("stack: a loop's range does not lie within the layers");
+    for (int i = 0; i < n; ++i) {
+        if (loop.times == 0 || i != loop.start) {
+            runs_.push_back({(size_t)i, 0, false});
+            layers_[(size_t)i].slots.resize(1);
+            continue;
+        }
+        for (int t = 0; t < loop.times; ++t)
+            for (int k = loop.start; k < loop.stop; ++k) runs_.push_back({(size_t)k, t, k == loop.start});
+        for (int k = loop.start; k < loop.stop; ++k) layers_[(size_t)k].slots.resize((size_t)loop.times);
+        i = loop.stop - 1;
+    }
+    return 0;
+}
+
+// sizes of a block and of its mixer's padded heads
+int StackModel::plan_block(size_t i, int which, bool mixer, bool ff) {
+    Layer &L = layers_[i];
+    Block &B = L.block[which];
+    const LayerSpec &S = spec_.layers[i];
+    const std::string where = "stack: layer " + std::to_string(i) + ": ";
+    B.used = true, B.mixer = mixer;
+    if (mixer && S.mixer == LayerSpec::Attention) {
+        const AttentionSpec &m = S.attention;
+        L.dimp = (int)up_to(m.dim, 32), L.vdimp = (int)up_to(m.vdim, 32);
+        if (m.heads < 1 || m.kv_heads < 1 || m.heads % m.kv_heads || m.maps < 1 || m.maps > 2 || L.dimp > 1024 || L.vdimp > 1024 || !(m.temp_every > 0.0))
+            return err_ = where + "attention: query heads in whole groups, one or two maps, heads of up to 1024 columns", BITNET_HIP_ERR_INVALID_ARGUMENT;
+        B.ko = (int)up_to((size_t)m.heads * L.vdimp, 64);
+        B.main = (m.heads + m.kv_heads) * m.maps * L.dimp + m.kv_heads * L.vdimp;
+    } else if (mixer) {
+        const DeltaSpec &m = S.delta;
+        L.dimp = (int)up_to(m.dim, 32), L.vdimp = (int)up_to(m.vdim, 32);
+        if (m.heads < 1 || m.kv_heads < 1 || m.heads % m.kv_heads || !bitnet_hip_delta_supported(L.dimp, L.vdimp) || m.taps < 1 || m.taps > 64)
+            return err_ = where + "delta: value heads in whole groups, heads of up to 256 columns, at most 64 taps", BITNET_HIP_ERR_INVALID_ARGUMENT;
+        B.ko = (int)up_to((size_t)m.heads * L.vdimp, 64);
+        B.main = 2 * m.kv_heads * L.dimp + 2 * m.heads * L.vdimp;
+        B.tail = B.gates = 2 * m.heads;
+    }
+    if (ff) {
+        const ExpertsSpec &e = S.experts;
+        B.fs = (int)up_to(S.ff, 64);
+        if (e.count > 0) {
+            if (e.top < 1 || e.top > e.count || e.top > 32 || e.count > 1024 || e.ff < 1)
+                return err_ = where + "experts: at most 32 of 1024, and not more than there are", BITNET_HIP_ERR_INVALID_ARGUMENT;
+            B.tail += e.count;
+        }
+    }
+    if (B.ko + B.fs == 0) B.fs = 64;  // routed experts alone: the product back is theirs, over columns of zeros
+    return 0;
+}
+
+int StackModel::query_factors(const AttentionSpec &a, float **out) {
+    std::vector<float> f(cap_);
+    for (size_t p = 0; p < cap_; ++p) f[p] = (float)(a.scale * (1.0 + a.temp_coef * std::log(std::floor((double)(p + 1) / a.temp_every) + 1.0)));
+    return upload(out, f);
 }
 
 int StackModel::grow(Buffer &b, size_t bytes) {
@@ -188,6 +282,17 @@ std::vector<uint16_t> pad_cols(const uint16_t *w, size_t rows, size_t groups, si
         for (size_t g = 0; g < groups; ++g) memcpy(&o[(r * groups + g) * to], w + (r * groups + g) * from, from * 2);
     return o;
 }
+// short convolution weights [groups][from channels][taps] into rows [taps][channels] at column `at`
+void put_taps(std::vector<float> &rows, size_t channels, size_t at, const std::vector<float> &w, size_t groups, size_t from, size_t to, size_t taps) {
+    for (size_t g = 0; g < groups; ++g)
+        for (size_t c = 0; c < from; ++c)
+            for (size_t j = 0; j < taps; ++j) rows[j * channels + at + g * to + c] = w[(g * from + c) * taps + j];
+}
+double dot(const std::vector<float> &a, const std::vector<float> &b) {
+    double s = 0.0;
+    for (size_t i = 0; i < a.size(); ++i) s += (double)a[i] * b[i];
+    return s;
+}
 std::vector<uint16_t> take(const uint16_t *w, size_t n) { return std::vector<uint16_t>(w, w + n); }
 void append(std::vector<uint16_t> &a, const std::vector<uint16_t> &b) { a.insert(a.end(), b.begin(), b.end()); }
 }  // namespace
@@ -203,8 +308,12 @@ int StackModel::set_layer(int layer, const StackLayerWeights &w) {
     const LayerSpec &S = spec_.layers[(size_t)layer];
     const size_t W = width_;
     if (L.set) return fail_arg("the layer already holds weights");
-    if (w.norm1.size() != W || w.norm1b.size() != W || (!w.ls1.empty() && w.ls1.size() != W)) return fail_arg("stack: norm of the wrong size");
-    TRY(upload(&L.norm1, w.norm1));
+    auto sized = [&](const std::vector<float> &v) { return v.empty() || v.size() == W; };
+    if (w.norm1.size() != W || !sized(w.norm1b) || !sized(w.ls1) || !sized(w.norm1_bias) || (!w.ls1.empty() && w.norm1b.empty()))
+        return fail_arg("stack: norm of the wrong size");
+    const size_t before = weight_bytes_;
+    TRY(upload(&L.norm1.w, w.norm1));
+    TRY(upload(&L.norm1.bias, w.norm1_bias));
     TRY(upload(&L.norm1b, w.norm1b));
     TRY(upload(&L.ls1, w.ls1));
     if (S.mixer == LayerSpec::Latent) {
@@ -237,7 +346,7 @@ int StackModel::set_layer(int layer, const StackLayerWeights &w) {
         TRY(upload(&L.dq_norm, w.dq_norm));
         TRY(upload(&L.dkv_norm, w.dkv_norm));
         TRY(upload(&L.sink, w.sink));
-    } else {
+    } else if (S.mixer == LayerSpec::Linear) {
         const LinearSpec &m = S.linear;
         const size_t H = m.heads, D = m.dim, V = m.vdim;
         if (!w.q || !w.k || !w.v || !w.g || !w.o || w.out_norm.size() != H * V) return fail_arg("stack: incomplete linear attention weights");
@@ -256,68 +365,188 @@ int StackModel::set_layer(int layer, const StackLayerWeights &w) {
         TRY(upload(&L.out_norm, n));
         TRY(upload(&L.decay_pow, pw));
     }
-    if (S.ff > 0) {
-        const size_t F = S.ff;
-        if (w.norm2.size() != W || w.norm2b.size() != W || (!w.ls2.empty() && w.ls2.size() != W) || !w.up || !w.down || (!w.up_b.empty() && w.up_b.size() != F) ||
-            (!w.down_b.empty() && w.down_b.size() != W))
-            return fail_arg("stack: incomplete feed-forward weights");
-        TRY(upload(&L.norm2, w.norm2));
+    if (!S.parallel && (S.ff > 0 || S.experts.count > 0)) {
+        if (w.norm2.size() != W || !sized(w.norm2b) || !sized(w.ls2) || !sized(w.norm2_bias) || (!w.ls2.empty() && w.norm2b.empty()))
+            return fail_arg("stack: norm of the wrong size");
+        TRY(upload(&L.norm2.w, w.norm2));
+        TRY(upload(&L.norm2.bias, w.norm2_bias));
         TRY(upload(&L.norm2b, w.norm2b));
         TRY(upload(&L.ls2, w.ls2));
+    }
+    for (int b = 0; b < 2; ++b)
+        if (L.block[b].used) TRY(set_block((size_t)layer, b, w));
+    if (!S.parallel && S.ff > 0 && S.experts.count == 0) {
+        const size_t F = S.ff;
+        if (!w.up || !w.down || (!w.up_b.empty() && w.up_b.size() != F) || (!w.down_b.empty() && w.down_b.size() != W))
+            return fail_arg("stack: incomplete feed-forward weights");
         TRY(upload_matrix(L.up, take(w.up, F * W), (int)F, (int)W));
         TRY(upload_matrix(L.down, take(w.down, W * F), (int)W, (int)F));
         TRY(upload(&L.up_b, w.up_b));
         TRY(upload(&L.down_b, w.down_b));
     }
+    weight_bytes_ = before + (weight_bytes_ - before) * L.slots.size();  // every pass reads them
     L.set = true;
     ++layers_set_;
     return 0;
 }
 
-int StackModel::set_globals(const uint16_t *embed, const std::vector<float> &final_norm, const uint16_t *head) {
-    if (!embed || final_norm.size() != (size_t)width_ || !head) return fail_arg("stack: incomplete globals");
+int StackModel::set_block(size_t i, int which, const StackLayerWeights &w) {
+    Layer &L = layers_[i];
+    Block &B = L.block[which];
+    const LayerSpec &S = spec_.layers[i];
+    const size_t W = width_, F = B.mixer && !S.parallel ? 0 : S.ff;
+    const ExpertsSpec E = B.mixer && !S.parallel ? ExpertsSpec() : S.experts;
+    B.norm = which == 0 ? L.norm1 : L.norm2;
+    std::vector<uint16_t> in((size_t)B.fs * W, 0), out(W * (B.ko + B.fs), 0);
+    auto into_out = [&](const uint16_t *m, size_t at, size_t groups, size_t from, size_t to) {
+        for (size_t r = 0; r < W; ++r)
+            for (size_t g = 0; g < groups; ++g) memcpy(&out[r * (B.ko + B.fs) + at + g * to], m + (r * groups + g) * from, from * 2);
+    };
+    if (F > 0) {
+        if (!w.up || !w.down || (!w.up_b.empty() && w.up_b.size() != F) || (!w.down_b.empty() && w.down_b.size() != W)) return fail_arg("stack: incomplete feed-forward weights");
+        memcpy(in.data(), w.up, F * W * 2);
+        into_out(w.down, B.ko, 1, F, F);
+    }
+    if (B.mixer && S.mixer == LayerSpec::Attention) {
+        const AttentionSpec &m = S.attention;
+        const size_t H = m.heads, G = m.kv_heads, M = m.maps, D = m.dim, V = m.vdim;
+        const bool two = M == 2 && w.lq1.size() == D && w.lk1.size() == D && w.lq2.size() == D && w.lk2.size() == D;
+        if (!w.q || !w.k || !w.v || !w.o || (!w.q_norm.empty() && w.q_norm.size() != D) || (!w.k_norm.empty() && w.k_norm.size() != D) || (M == 2 && !two))
+            return fail_arg("stack: incomplete attention weights");
+        append(in, pad_rows(w.q, H * M, D, L.dimp, W));
+        append(in, pad_rows(w.k, G * M, D, L.dimp, W));
+        append(in, pad_rows(w.v, G, V, L.vdimp, W));
+        into_out(w.o, 0, H, V, L.vdimp);
+        TRY(upload(&L.q_norm, w.q_norm));
+        TRY(upload(&L.k_norm, w.k_norm));
+        if (two) L.lambda = (float)(std::exp(dot(w.lq1, w.lk1)) - std::exp(dot(w.lq2, w.lk2)) + m.diff);
+    } else if (B.mixer) {
+        const DeltaSpec &m = S.delta;
+        const size_t H = m.heads, G = m.kv_heads, D = m.dim, V = m.vdim, T = m.taps, C = 2 * G * L.dimp + H * L.vdimp;
+        if (!w.q || !w.k || !w.v || !w.g || !w.o || !w.b || !w.a || w.q_conv.size() != G * D * T || w.k_conv.size() != G * D * T || w.v_conv.size() != H * V * T ||
+            w.a_log.size() != H || w.dt_bias.size() != H || w.out_norm.size() != V)
+            return fail_arg("stack: incomplete delta weights");
+        append(in, pad_rows(w.q, G, D, L.dimp, W));
+        append(in, pad_rows(w.k, G, D, L.dimp, W));
+        append(in, pad_rows(w.v, H, V, L.vdimp, W));
+        append(in, pad_rows(w.g, H, V, L.vdimp, W));
+        append(in, take(w.b, H * W));
+        append(in, take(w.a, H * W));
+        into_out(w.o, 0, H, V, L.vdimp);
+        std::vector<float> conv(T * C, 0.f), rate(H), norm(L.vdimp, 0.f);
+        put_taps(conv, C, 0, w.q_conv, G, D, L.dimp, T);
+        put_taps(conv, C, G * L.dimp, w.k_conv, G, D, L.dimp, T);
+        put_taps(conv, C, 2 * G * L.dimp, w.v_conv, H, V, L.vdimp, T);
+        for (size_t h = 0; h < H; ++h) rate[h] = (float)std::exp((double)w.a_log[h]);
+        std::copy(w.out_norm.begin(), w.out_norm.end(), norm.begin());
+        TRY(upload(&L.conv, conv));
+        TRY(upload(&L.decay_rate, rate));
+        TRY(upload(&L.dt_bias, w.dt_bias));
+        TRY(upload(&L.out_norm, norm));
+    }
+    if (E.count > 0) {
+        const size_t N = E.count, R = E.ff;
+        if (!w.router || w.expert_up.size() != N || w.expert_down.size() != N) return fail_arg("stack: incomplete experts");
+        append(in, take(w.router, N * W));
+        std::vector<uint16_t> up, down;
+        for (size_t e = 0; e < N; ++e) {
+            if (!w.expert_up[e] || !w.expert_down[e]) return fail_arg("stack: incomplete experts");
+            up.insert(up.end(), w.expert_up[e], w.expert_up[e] + R * W);
+            down.insert(down.end(), w.expert_down[e], w.expert_down[e] + W * R);
+        }
+        TRY(upload_matrix(B.expert_up, up, (int)(N * R), (int)W));
+        TRY(upload_matrix(B.expert_down, down, (int)(N * W), (int)R));
+        weight_bytes_ -= (N - E.top) * R * W * 4;  // a token reads `top` of them
+    }
+    TRY(upload_matrix(B.in, in, B.fs + B.main + B.tail, (int)W));
+    TRY(upload_matrix(B.out, out, (int)W, B.ko + B.fs));
+    if (F > 0 && !w.up_b.empty()) {
+        std::vector<float> bias(B.in.rows, 0.f);
+        std::copy(w.up_b.begin(), w.up_b.end(), bias.begin());
+        TRY(upload(&B.in_bias, bias));
+    }
+    if (F > 0) TRY(upload(&B.out_bias, w.down_b));
+    return 0;
+}
+
+int StackModel::set_globals(const uint16_t *embed, const std::vector<float> &final_norm, const std::vector<float> &final_bias, const uint16_t *head,
+                            const uint16_t *loop_in) {
+    if (!embed || final_norm.size() != (size_t)width_ || (!final_bias.empty() && final_bias.size() != (size_t)width_) || !head ||
+        (spec_.loop.times > 0) != (loop_in != nullptr))
+        return fail_arg("stack: incomplete globals");
     if (head_) return fail_arg("the model already holds its globals");
     const size_t n = (size_t)vocab_ * width_;
     TRY(upload_matrix(embed_, take(embed, n), vocab_, width_));
     weight_bytes_ -= n * 2;  // a row of it is read per token
     TRY(upload_matrix(head_m_, take(head, n), vocab_, width_));
-    TRY(upload(&final_norm_, final_norm));
+    TRY(upload(&final_norm_.w, final_norm));
+    TRY(upload(&final_norm_.bias, final_bias));
+    if (loop_in) {
+        TRY(upload_matrix(loop_in_, take(loop_in, 2 * (size_t)width_ * width_), width_, 2 * width_));
+        weight_bytes_ += (size_t)(spec_.loop.times - 1) * 4 * width_ * width_;
+    }
     head_ = head_m_.w;
     return 0;
 }
 
 int StackModel::clear_state() {
     // the caches need no clearing: a position is read only after it was written, what lies past it meets a zero weight
-    for (size_t i = 0; i < layers_.size(); ++i)
-        if (layers_[i].state)
-            HCHK(hipMemsetAsync(layers_[i].state, 0, (size_t)spec_.layers[i].linear.heads * layers_[i].dimp * layers_[i].vdimp * 4, (hipStream_t)stream_));
+    // (a convolution's earlier inputs are read for positions of this sequence only)
+    for (const Layer &L : layers_)
+        for (const Slot &slot : L.slots)
+            if (slot.state) HCHK(hipMemsetAsync(slot.state, 0, slot.state_bytes, (hipStream_t)stream_));
     HCHK(hipStreamSynchronize((hipStream_t)stream_));
     hidden_ = nullptr;
     return 0;
 }
 
-void StackModel::attention_args(size_t i, bitnet_hip_latent_attention &a) const {
-    const Layer &L = layers_[i], &K = kv_layer(i);
+bitnet_hip_gqa StackModel::gqa_args(size_t i, int pass) const {
+    const Layer &L = layers_[i];
+    const AttentionSpec &m = spec_.layers[i].attention;
+    const Slot &slot = L.slots[(size_t)pass];
+    bitnet_hip_gqa a;
+    memset(&a, 0, sizeof(a));
+    a.heads = m.heads, a.kv_heads = m.kv_heads, a.maps = m.maps, a.dim = m.dim, a.dimp = L.dimp, a.vdim = m.vdim, a.vdimp = L.vdimp, a.capacity = cap_;
+    a.eps = spec_.eps, a.lambda = L.lambda, a.out_scale = 1.0f - m.diff, a.q_weight = L.q_norm, a.k_weight = L.k_norm, a.q_factor = L.q_factor;
+    a.kcache = slot.k, a.vcache = slot.v;
+    return a;
+}
+
+bitnet_hip_delta StackModel::delta_args(size_t i, int pass) const {
+    const Layer &L = layers_[i];
+    const DeltaSpec &m = spec_.layers[i].delta;
+    const Slot &slot = L.slots[(size_t)pass];
+    bitnet_hip_delta d;
+    memset(&d, 0, sizeof(d));
+    d.heads = m.heads, d.kv_heads = m.kv_heads, d.dim = m.dim, d.dimp = L.dimp, d.vdim = m.vdim, d.vdimp = L.vdimp, d.taps = m.taps;
+    d.conv = L.conv, d.decay_rate = L.decay_rate, d.dt_bias = L.dt_bias, d.norm = L.out_norm;
+    d.q_scale = (float)(1.0 / std::sqrt((double)m.dim)), d.unit_eps = m.unit_eps, d.eps = spec_.eps, d.state = slot.state, d.ring = slot.ring;
+    return d;
+}
+
+void StackModel::attention_args(size_t i, int pass, bitnet_hip_latent_attention &a) const {
+    const Layer &L = layers_[i];
+    const Slot &K = kv_slot(i, pass);
     const LatentSpec &m = spec_.layers[i].latent;
     a.heads = m.heads, a.dimp = L.dimp, a.qd = L.dimp + L.rotp, a.vdimp = L.vdimp, a.kv_rank = m.kv_rank, a.rot_dim = m.rot_dim;
-    a.scale = m.scale, a.sink = L.sink, a.ccache = K.cache.c, a.rcache = K.cache.r, a.ldc = L.ldc, a.ldr = L.rotp, a.capacity = cap_;
+    a.scale = m.scale, a.sink = L.sink, a.ccache = K.c, a.rcache = K.r, a.ldc = L.ldc, a.ldr = L.rotp, a.capacity = cap_;
     a.rope_cos = L.cos, a.rope_sin = L.sin;
 }
 
-void StackModel::latent_args(size_t i, const float *z, size_t ldz, void *cq, size_t ldcq, bitnet_hip_latent_rows &r) const {
+void StackModel::latent_args(size_t i, int pass, const float *z, size_t ldz, void *cq, size_t ldcq, bitnet_hip_latent_rows &r) const {
     const Layer &L = layers_[i];
     const LatentSpec &m = spec_.layers[i].latent;
     memset(&r, 0, sizeof(r));
     r.z = z, r.ldz = ldz, r.q_rank = m.q_rank, r.q_weight = L.dq_norm, r.eps = spec_.eps, r.cq = cq, r.ldcq = ldcq, r.pos = pos_;
     if (m.kv_from < 0) {
         r.kv_rank = m.kv_rank, r.rot_dim = m.rot_dim, r.kv_weight = L.dkv_norm;
-        r.ccache = L.cache.c, r.rcache = L.cache.r, r.ldc = L.ldc, r.ldr = L.rotp, r.rope_cos = L.cos, r.rope_sin = L.sin;
+        r.ccache = L.slots[(size_t)pass].c, r.rcache = L.slots[(size_t)pass].r, r.ldc = L.ldc, r.ldr = L.rotp, r.rope_cos = L.cos, r.rope_sin = L.sin;
     }
 }
 
 // ---- one token --------------------------------------------------------------------------------------------------------
-// x_[cur_] is the residual stream up to the pending sublayer; the launch that normalises it for the next sublayer adds the pending
-// output on the way and leaves the sum in the other buffer.
+// *cur_ is the residual stream up to the pending sublayer; the launch that normalises it for the next sublayer adds the pending
+// output on the way and leaves the sum in another buffer.
 
 int StackModel::gemv(const bitnet_hip_vector_input &in, const Matrix &m, const float *bias, int act0, int act1, size_t split, float *y,
                      const bitnet_hip_latent_rows *latent) {
@@ -333,68 +562,121 @@ static bitnet_hip_vector_input plain_input(const float *x) {
     return in;
 }
 
-bitnet_hip_vector_input StackModel::block_input(const float *norm) {
-    bitnet_hip_vector_input in = plain_input(x_[cur_]);
+void StackModel::add_pending(bitnet_hip_vector_input &in) {
+    if (!pending_.y) return;
+    cur_ = in.x_out = next_x();
+    in.y = pending_.y, in.post_weight = pending_.w, in.scale = pending_.scale, in.mult = spec_.residual_mult;
+    pending_ = Pending();
+}
+
+bitnet_hip_vector_input StackModel::block_input(const Norm &norm) {
+    bitnet_hip_vector_input in = plain_input(cur_);
     in.kind = BITNET_HIP_IN_RESIDUAL_NORM;
-    in.eps = spec_.eps, in.weight_offset = spec_.norm_offset, in.weight = norm, in.n = width_;
-    if (pending_.y) {
-        cur_ ^= 1;
-        in.y = pending_.y, in.post_weight = pending_.w, in.scale = pending_.scale, in.x_out = x_[cur_];
-        pending_ = Pending();
-    }
+    in.eps = spec_.eps, in.weight_offset = spec_.norm_offset, in.weight = norm.w, in.bias = norm.bias, in.center = spec_.center, in.n = width_;
+    add_pending(in);
     return in;
 }
 
-int StackModel::step_latent(size_t i) {
+// x <- W_in [x; embedding output]
+int StackModel::step_loop_in() {
+    bitnet_hip_vector_input in = plain_input(cur_);
+    in.kind = BITNET_HIP_IN_CONCAT, in.n = width_, in.x2 = x0_;
+    add_pending(in);
+    in.x_out = nullptr;  // (nobody else reads the sum)
+    float *x = in.x == x_[0] ? x_[1] : x_[0];
+    TRY(gemv(in, loop_in_, nullptr, 0, 0, 0, x));
+    cur_ = x;
+    return 0;
+}
+
+// the sublayers of a block; their sum is left in y_[which]
+int StackModel::step_block(size_t i, int pass, int which) {
+    const Layer &L = layers_[i];
+    const Block &B = L.block[which];
+    const LayerSpec &S = spec_.layers[i];
+    const bool routed = B.expert_up.w != nullptr;
+    const int act = S.act_ff;
+    bitnet_hip_vector_input in = block_input(B.norm);
+    if (routed) in.h_out = h_;
+    float *proj = row_ + B.ko + B.fs, *tail = proj + B.main;
+    TRY(gemv(in, B.in, B.in_bias, B.fs ? act : 0, 0, B.fs, row_ + B.ko));
+    if (B.mixer && S.mixer == LayerSpec::Attention) {
+        const bitnet_hip_gqa a = gqa_args(i, pass);
+        if (!f32_ && bitnet_hip_gqa_supported(a.dimp, a.vdimp)) {
+            BCHK(bitnet_hip_gqa_step_dev(&a, proj, pos_, scratch_, stream_));
+        } else {
+            BCHK(bitnet_hip_gqa_rows_dev(&a, proj, B.main, 1, f32_, pos_, 1, stream_));
+            BCHK(bitnet_hip_gqa_any_dev(&a, proj, B.main, 1, f32_, pos_, 0, 1, scratch_, stream_));
+        }
+        BCHK(bitnet_hip_gqa_merge_dev(&a, pos_, 0, 1, scratch_, row_, B.ko, 0, stream_));
+    } else if (B.mixer) {
+        const bitnet_hip_delta d = delta_args(i, pass);
+        BCHK(bitnet_hip_delta_step_dev(&d, proj, tail, pos_, row_, stream_));
+    }
+    if (!routed) return gemv(plain_input(row_), B.out, B.out_bias, 0, 0, 0, y_[which]);
+    const ExpertsSpec &e = S.experts;
+    BCHK(bitnet_hip_experts_up_dev(tail + B.gates, e.count, e.top, e.scale, h_, B.expert_up.w, e.ff, B.expert_up.cols, B.expert_up.ld, e.act, eact_, B.expert_down.ld,
+                                   eids_, stream_));
+    BCHK(bitnet_hip_experts_out_dev(row_, B.out.w, B.out.cols, B.out.ld, B.out_bias, eact_, B.expert_down.ld, B.expert_down.w, B.expert_down.cols, B.expert_down.ld, eids_,
+                                    e.top, width_, y_[which], stream_));
+    return 0;
+}
+
+int StackModel::step_latent(size_t i, int pass) {
     const Layer &L = layers_[i];
     const LatentSpec &m = spec_.layers[i].latent;
     TRY(gemv(block_input(L.norm1), L.down_q, nullptr, 0, 0, 0, z_));
     bitnet_hip_vector_input in = plain_input(z_);
     in.kind = BITNET_HIP_IN_NORM, in.eps = spec_.eps, in.weight = L.dq_norm, in.n = m.q_rank;
     bitnet_hip_latent_rows r;
-    latent_args(i, z_, L.down_q.rows, nullptr, 0, r);
+    latent_args(i, pass, z_, L.down_q.rows, nullptr, 0, r);
     TRY(gemv(in, L.uq, nullptr, 0, 0, 0, q_, m.kv_from < 0 ? &r : nullptr));
     const size_t qd = L.dimp + L.rotp;
     const bitnet_hip_vector_input qi = plain_input(q_);
     BCHK(bitnet_hip_dense_gemv_dev(&qi, L.uk_t.w, L.ldc, L.dimp, L.uk_t.ld, nullptr, 0, 0, 0, qabs_, m.heads, (size_t)L.ldc * L.uk_t.ld, qd, L.ldc, nullptr, 0,
                                    stream_));
     bitnet_hip_latent_attention a;
-    attention_args(i, a);
+    attention_args(i, pass, a);
     BCHK(bitnet_hip_latent_decode_dev(&a, q_, qabs_, pos_, 0, 1, f32_, scratch_, stream_));
     BCHK(bitnet_hip_latent_merge_dev(&a, L.uv.w, pos_, 0, 1, scratch_, att_, (size_t)m.heads * L.vdimp, 0, stream_));
     return gemv(plain_input(att_), L.o, nullptr, 0, 0, 0, y_[0]);
 }
 
-int StackModel::step_linear(size_t i) {
+int StackModel::step_linear(size_t i, int pass) {
     const Layer &L = layers_[i];
     const LinearSpec &m = spec_.layers[i].linear;
     const size_t split = (size_t)m.heads * (2 * L.dimp + L.vdimp);
     TRY(gemv(block_input(L.norm1), L.qkvg, nullptr, m.act_qkv, m.act_gate, split, lin_));
-    BCHK(bitnet_hip_linear_recurrent_dev(lin_, L.qkvg.rows, 1, m.heads, L.dimp, L.vdimp, L.decay_pow, L.state, lino_, (size_t)m.heads * L.vdimp, stream_));
+    BCHK(bitnet_hip_linear_recurrent_dev(lin_, L.qkvg.rows, 1, m.heads, L.dimp, L.vdimp, L.decay_pow, L.slots[(size_t)pass].state, lino_, (size_t)m.heads * L.vdimp, stream_));
     bitnet_hip_vector_input in = plain_input(lino_);
     in.kind = BITNET_HIP_IN_NORM, in.eps = spec_.eps, in.weight = L.out_norm, in.gate = lin_ + split, in.n = m.heads * L.vdimp, in.mean_n = m.heads * m.vdim;
     return gemv(in, L.o, nullptr, 0, 0, 0, y_[0]);
 }
 
 int StackModel::step(bool with_logits, int) {
-    cur_ = 0;
+    cur_ = x0_;
     pending_ = Pending();
-    BCHK(bitnet_hip_embed_bf16_dev(embed_.w, embed_.ld, history_, pos_, 1, width_, vocab_, x_[0], stream_));
-    for (size_t i = 0; i < layers_.size(); ++i) {
+    BCHK(bitnet_hip_embed_bf16_dev(embed_.w, embed_.ld, history_, pos_, 1, width_, vocab_, spec_.embed_scale, x0_, stream_));
+    for (const Run &run : runs_) {
+        const size_t i = run.layer;
         const Layer &L = layers_[i];
         const LayerSpec &S = spec_.layers[i];
-        TRY(S.mixer == LayerSpec::Latent ? step_latent(i) : step_linear(i));
+        if (run.enters) TRY(step_loop_in());
+        TRY(L.block[0].used ? step_block(i, run.pass, 0) : S.mixer == LayerSpec::Latent ? step_latent(i, run.pass) : step_linear(i, run.pass));
         pending_ = {y_[0], L.norm1b, L.ls1};
-        if (S.ff > 0) {
+        if (S.parallel || (S.ff == 0 && S.experts.count == 0)) continue;
+        if (L.block[1].used) {
+            TRY(step_block(i, run.pass, 1));
+        } else {
             TRY(gemv(block_input(L.norm2), L.up, L.up_b, S.act_ff, 0, 0, act_));
             TRY(gemv(plain_input(act_), L.down, L.down_b, 0, 0, 0, y_[1]));
-            pending_ = {y_[1], L.norm2b, L.ls2};
         }
+        pending_ = {y_[1], L.norm2b, L.ls2};
     }
     if (with_logits) {
         const bitnet_hip_vector_input in = block_input(final_norm_);
         BCHK(bitnet_hip_dense_logits_dev(&in, head_m_.w, vocab_, head_m_.cols, head_m_.ld, logits_, argmax_, token_, pos_, history_, n_forced_, stream_));
-        hidden_ = x_[cur_];
+        hidden_ = cur_;
     } else {
         BCHK(bitnet_hip_advance_pos_dev(pos_, stream_));
         hidden_ = nullptr;  // the last sublayer's output was not added: nobody asked for it
@@ -409,6 +691,7 @@ int StackModel::portion_buffers(size_t n) {
     n = up_to(n, 64);
     const size_t es = f32_ ? 4 : 2;
     size_t z = 0, cq = 0, q = 0, qabs = 0, att = 0, act = 0, k = 0, vt = 0, lin = 0, linf = 0, lino = 0, gate = 0, ws = 0, scratch = 0, qf = 0;
+    size_t row = 0, tail = 0, qk = 0, v = 0, gates = 0, plan = 0, eact = 0, eout = 0;
     for (size_t i = 0; i < layers_.size(); ++i) {
         const Layer &L = layers_[i];
         const LayerSpec &S = spec_.layers[i];
@@ -426,6 +709,15 @@ int StackModel::portion_buffers(size_t n) {
                 qabs = std::max(qabs, (size_t)m.heads * L.ldc);
                 scratch = std::max(scratch, bitnet_hip_latent_scratch_bytes(m.heads, L.ldc, kDecodeSlice));
             }
+        } else if (S.mixer == LayerSpec::Attention) {
+            const AttentionSpec &m = S.attention;
+            if (f32_ || !bitnet_hip_gqa_supported(L.dimp, L.vdimp)) scratch = std::max(scratch, bitnet_hip_gqa_scratch_bytes(m.heads, m.maps, L.vdimp, kDecodeSlice));
+        } else if (S.mixer == LayerSpec::Delta) {
+            const DeltaSpec &m = S.delta;
+            qk = std::max(qk, (size_t)2 * m.kv_heads * L.dimp);
+            v = std::max(v, (size_t)m.heads * L.vdimp);
+            gates = std::max(gates, (size_t)2 * m.heads);
+            if (!f32_ && bitnet_hip_delta_chunked_supported(L.dimp, L.vdimp)) ws = std::max(ws, bitnet_hip_delta_workspace_bytes(n, m.heads, L.dimp, L.vdimp));
         } else {
             const LinearSpec &m = S.linear;
             lino = std::max(lino, (size_t)m.heads * L.vdimp);
@@ -437,9 +729,31 @@ int StackModel::portion_buffers(size_t n) {
                 linf = std::max(linf, (size_t)L.qkvg.rows);
             }
         }
-        act = std::max(act, S.ff ? (size_t)L.down.ld : 0);
+        for (const Block &B : L.block) {
+            if (!B.used) continue;
+            row = std::max(row, up_to((size_t)B.ko + B.fs + B.main, 64));
+            tail = std::max(tail, up_to(B.tail, 64));
+            if (!B.expert_up.w) continue;
+            const ExpertsSpec &e = S.experts;
+            plan = std::max(plan, bitnet_hip_experts_plan_bytes(n, e.count, e.top));
+            eact = std::max(eact, (size_t)e.top * B.expert_down.ld);
+            eout = std::max(eout, (size_t)e.top * up_to(width_, 64));
+        }
+        act = std::max(act, (size_t)L.down.ld);
     }
     rows_cap_ = 0;
+    if (spec_.loop.times > 0) {
+        TRY(grow(px0_, n * width_ * 4));
+        TRY(grow(pcat_, n * loop_in_.ld * es));
+    }
+    TRY(grow(prow_, n * row * es));
+    TRY(grow(ptail_, n * tail * 4));
+    TRY(grow(pqk_, n * qk * 4));
+    TRY(grow(pv_, n * v * es));
+    TRY(grow(pgates_, n * gates * 4));
+    TRY(grow(pplan_, plan));
+    TRY(grow(peact_, n * eact * es));
+    TRY(grow(peout_, n * eout * es));
     TRY(grow(px_, n * width_ * 4));
     TRY(grow(ph_, n * up_to(width_, 64) * es));
     TRY(grow(py_, n * width_ * 4));
@@ -468,21 +782,99 @@ int StackModel::matmul(const void *a, size_t lda, bool a_f32, const Matrix &m, c
     return 0;
 }
 
-int StackModel::portion_latent(size_t i, size_t n, size_t pos0) {
-    const Layer &L = layers_[i], &K = kv_layer(i);
+// The pending sublayer is added to the n rows of px_; h (nullable) receives their norm, or -- x2 given -- [x; x2].
+int StackModel::portion_norm(size_t n, const Norm *norm, const float *x2, void *h, size_t ldh) {
+    const Pending p = pending_;
+    pending_ = Pending();
+    const bool post = p.y && p.w, own = spec_.center || x2 || !h;
+    if (post) {  // the norm behind the sublayer, and the next one with it where it is of the same kind
+        BCHK(bitnet_hip_residual_norm_rows_dev((float *)px_.p, p.y, width_, p.w, p.scale, own ? nullptr : norm->w, spec_.norm_offset, spec_.eps, n, width_,
+                                               own ? nullptr : h, ldh, f32_, stream_));
+        if (!own || !h) return 0;
+    }
+    bitnet_hip_sum_rows r;
+    memset(&r, 0, sizeof(r));
+    r.x = (float *)px_.p, r.m = n, r.width = width_, r.mult = spec_.residual_mult, r.eps = spec_.eps, r.weight_offset = spec_.norm_offset;
+    r.center = spec_.center, r.h_f32 = f32_, r.h = h, r.ldh = ldh, r.x2 = x2;
+    if (norm) r.weight = norm->w, r.bias = norm->bias;
+    if (p.y && !post) {
+        r.y = p.y, r.ldy = width_;
+        if (p.experts) r.expert_rows = peout_.p, r.ld_expert = up_to(width_, 64), r.top = plan_.top, r.slots = plan_.slots, r.slot_weights = plan_.weights;
+    }
+    BCHK(bitnet_hip_sum_norm_rows_dev(&r, stream_));
+    return 0;
+}
+
+int StackModel::portion_loop_in(size_t n) {
+    TRY(portion_norm(n, nullptr, (const float *)px0_.p, pcat_.p, loop_in_.ld));
+    return matmul(pcat_.p, loop_in_.ld, f32_, loop_in_, nullptr, n, 0, 0, 0, px_.p, width_, true);
+}
+
+// the sublayers of a block: py_ holds the sum of those that every token takes, the routed experts' rows lie in peout_ by slot
+int StackModel::portion_block(size_t i, int pass, int which, size_t n, size_t pos0) {
+    const Layer &L = layers_[i];
+    const Block &B = L.block[which];
+    const LayerSpec &S = spec_.layers[i];
+    const size_t ldh = up_to(width_, 64), ld = up_to((size_t)B.ko + B.fs + B.main, 64), ldt = up_to(B.tail, 64), es = f32_ ? 4 : 2;
+    const bool routed = B.expert_up.w != nullptr;
+    char *row = (char *)prow_.p, *proj = row + (size_t)(B.ko + B.fs) * es;
+    float *tail = (float *)ptail_.p;
+    if (B.fs + B.main > 0)
+        BCHK(bitnet_hip_dense_matmul_dev(ph_.p, ldh, f32_, B.in.w, B.in.ld, B.in_bias, n, B.fs + B.main, B.in.ld, B.fs ? S.act_ff : 0, 0, B.fs, row + (size_t)B.ko * es, ld,
+                                         f32_, 1, 0, 0, 0, stream_));
+    if (B.tail > 0)
+        BCHK(bitnet_hip_dense_matmul_dev(ph_.p, ldh, f32_, B.in.w + (size_t)(B.fs + B.main) * B.in.ld, B.in.ld, nullptr, n, B.tail, B.in.ld, 0, 0, 0, tail, ldt, 1, 1, 0, 0,
+                                         0, stream_));
+    if (B.mixer && S.mixer == LayerSpec::Attention) {
+        const bitnet_hip_gqa a = gqa_args(i, pass);
+        BCHK(bitnet_hip_gqa_rows_dev(&a, proj, ld, f32_, f32_, pos_, n, stream_));
+        if (!f32_ && bitnet_hip_gqa_supported(a.dimp, a.vdimp)) {
+            BCHK(bitnet_hip_gqa_prefill_dev(&a, (const uint16_t *)proj, ld, pos0 + n, n, (uint16_t *)row, ld, stream_));
+        } else {
+            for (size_t s = 0; s < n; s += kDecodeSlice) {
+                const size_t k = std::min(kDecodeSlice, n - s);
+                BCHK(bitnet_hip_gqa_any_dev(&a, proj + s * ld * es, ld, f32_, f32_, pos_, s, k, (float *)pscratch_.p, stream_));
+                BCHK(bitnet_hip_gqa_merge_dev(&a, pos_, s, k, (const float *)pscratch_.p, row + s * ld * es, ld, !f32_, stream_));
+            }
+        }
+    } else if (B.mixer) {
+        const bitnet_hip_delta d = delta_args(i, pass);
+        float *qk = (float *)pqk_.p, *gates = (float *)pgates_.p;
+        BCHK(bitnet_hip_delta_rows_dev(&d, proj, ld, f32_, tail, ldt, pos_, n, qk, pv_.p, gates, stream_));
+        BCHK(bitnet_hip_delta_keep_dev(&d, proj, ld, f32_, pos_, n, stream_));
+        if (!f32_ && bitnet_hip_delta_chunked_supported(L.dimp, L.vdimp))
+            BCHK(bitnet_hip_delta_chunked_dev(&d, qk, (const uint16_t *)pv_.p, gates, (const uint16_t *)proj, ld, n, (uint16_t *)row, ld, plws_.p, plws_.bytes, stream_));
+        else
+            BCHK(bitnet_hip_delta_recurrent_dev(&d, qk, pv_.p, gates, proj, ld, f32_, n, row, ld, stream_));
+    }
+    TRY(matmul(row, ld, f32_, B.out, B.out_bias, n, 0, 0, 0, py_.p, width_, true));
+    if (!routed) return 0;
+    const ExpertsSpec &e = S.experts;
+    const size_t tile = !f32_ && n * e.top >= (size_t)96 * e.count ? 128 : 64;
+    BCHK(bitnet_hip_experts_plan_make(pplan_.p, pplan_.bytes, n, e.count, e.top, tile, &plan_));
+    BCHK(bitnet_hip_experts_route_dev(tail + B.gates, ldt, e.scale, &plan_, stream_));
+    BCHK(bitnet_hip_experts_matmul_dev(&plan_, 1, ph_.p, ldh, f32_, B.expert_up.w, e.ff, B.expert_up.ld, B.expert_up.ld, e.act, peact_.p, B.expert_down.ld, f32_, stream_));
+    BCHK(bitnet_hip_experts_matmul_dev(&plan_, 0, peact_.p, B.expert_down.ld, f32_, B.expert_down.w, width_, B.expert_down.ld, B.expert_down.ld, 0, peout_.p, up_to(width_, 64),
+                                       f32_, stream_));
+    return 0;
+}
+
+int StackModel::portion_latent(size_t i, int pass, size_t n, size_t pos0) {
+    const Layer &L = layers_[i];
+    const Slot &K = kv_slot(i, pass);
     const LatentSpec &m = spec_.layers[i].latent;
     const size_t ldh = up_to(width_, 64), ldcq = up_to(m.q_rank, 64), qd = L.dimp + L.rotp, lda = L.o.ld, ctx = pos0 + n;
     TRY(matmul(ph_.p, ldh, f32_, L.down_q, nullptr, n, 0, 0, 0, pz_.p, L.down_q.rows, true));
     bitnet_hip_latent_rows r;
-    latent_args(i, (const float *)pz_.p, L.down_q.rows, pcq_.p, ldcq, r);
+    latent_args(i, pass, (const float *)pz_.p, L.down_q.rows, pcq_.p, ldcq, r);
     BCHK(bitnet_hip_latent_rows_dev(&r, n, f32_, stream_));
     bitnet_hip_latent_attention a;
-    attention_args(i, a);
+    attention_args(i, pass, a);
     if (!f32_ && bitnet_hip_latent_prefill_supported(qd, L.vdimp)) {
         TRY(matmul(pcq_.p, ldcq, false, L.uq, nullptr, n, 0, 0, 0, pq_.p, L.uq.rows, false));
-        TRY(matmul(K.cache.c, L.ldc, false, L.uk, nullptr, ctx, 0, 0, 0, pk_.p, L.uk.rows, false));
+        TRY(matmul(K.c, L.ldc, false, L.uk, nullptr, ctx, 0, 0, 0, pk_.p, L.uk.rows, false));
         // the values transposed: W_uv's rows are the product's rows, the cache its "weights"
-        BCHK(bitnet_hip_dense_matmul_dev(L.uv.w, L.uv.ld, 0, (const uint16_t *)K.cache.c, L.ldc, nullptr, L.uv.rows, up_to(ctx, 64), L.ldc, 0, 0, 0, pvt_.p, cap_, 0,
+        BCHK(bitnet_hip_dense_matmul_dev(L.uv.w, L.uv.ld, 0, (const uint16_t *)K.c, L.ldc, nullptr, L.uv.rows, up_to(ctx, 64), L.ldc, 0, 0, 0, pvt_.p, cap_, 0,
                                          1, 0, 0, 0, stream_));
         BCHK(bitnet_hip_latent_prefill_dev(&a, (const uint16_t *)pq_.p, (const uint16_t *)pk_.p, (const uint16_t *)pvt_.p, cap_, ctx, n, (uint16_t *)patt_.p, lda,
                                            stream_));
@@ -501,8 +893,9 @@ int StackModel::portion_latent(size_t i, size_t n, size_t pos0) {
     return matmul(patt_.p, lda, f32_, L.o, nullptr, n, 0, 0, 0, py_.p, width_, true);
 }
 
-int StackModel::portion_linear(size_t i, size_t n) {
+int StackModel::portion_linear(size_t i, int pass, size_t n) {
     const Layer &L = layers_[i];
+    float *state = L.slots[(size_t)pass].state;
     const LinearSpec &m = spec_.layers[i].linear;
     const size_t ldh = up_to(width_, 64), ld = L.qkvg.rows, no = (size_t)m.heads * L.vdimp, split = (size_t)m.heads * (2 * L.dimp + L.vdimp);
     const bool chunked = !f32_ && bitnet_hip_linear_chunked_supported(L.dimp, L.vdimp);
@@ -510,10 +903,10 @@ int StackModel::portion_linear(size_t i, size_t n) {
     TRY(matmul(ph_.p, ldh, f32_, L.qkvg, nullptr, n, m.act_qkv, m.act_gate, split, lin, ld, !chunked));
     const void *gate = chunked ? (const void *)((const uint16_t *)lin + split) : (const void *)((const float *)lin + split);
     if (chunked)
-        BCHK(bitnet_hip_linear_chunked_dev((const uint16_t *)lin, ld, n, m.heads, L.dimp, L.vdimp, L.decay_pow, L.state, (float *)plino_.p, no, plws_.p, plws_.bytes,
+        BCHK(bitnet_hip_linear_chunked_dev((const uint16_t *)lin, ld, n, m.heads, L.dimp, L.vdimp, L.decay_pow, state, (float *)plino_.p, no, plws_.p, plws_.bytes,
                                            stream_));
     else
-        BCHK(bitnet_hip_linear_recurrent_dev((const float *)lin, ld, n, m.heads, L.dimp, L.vdimp, L.decay_pow, L.state, (float *)plino_.p, no, stream_));
+        BCHK(bitnet_hip_linear_recurrent_dev((const float *)lin, ld, n, m.heads, L.dimp, L.vdimp, L.decay_pow, state, (float *)plino_.p, no, stream_));
     BCHK(bitnet_hip_gated_norm_rows_dev((const float *)plino_.p, no, L.out_norm, gate, ld, spec_.eps, !chunked, n, no, (size_t)m.heads * m.vdim, pgate_.p, L.o.ld,
                                         f32_, stream_));
     return matmul(pgate_.p, L.o.ld, f32_, L.o, nullptr, n, 0, 0, 0, py_.p, width_, true);
@@ -525,23 +918,28 @@ int StackModel::portion(int rows, int pos0) {
     TRY(portion_buffers(n));
     float *x = (float *)px_.p;
     const float *y = (const float *)py_.p;
-    BCHK(bitnet_hip_embed_bf16_dev(embed_.w, embed_.ld, history_, pos_, n, width_, vocab_, x, stream_));
-    const float *post = nullptr, *scale = nullptr;
-    bool have = false;
-    for (size_t i = 0; i < layers_.size(); ++i) {
+    BCHK(bitnet_hip_embed_bf16_dev(embed_.w, embed_.ld, history_, pos_, n, width_, vocab_, spec_.embed_scale, x, stream_));
+    if (spec_.loop.times > 0) BCHK(bitnet_hip_embed_bf16_dev(embed_.w, embed_.ld, history_, pos_, n, width_, vocab_, spec_.embed_scale, (float *)px0_.p, stream_));
+    pending_ = Pending();
+    for (const Run &run : runs_) {
+        const size_t i = run.layer;
         const Layer &L = layers_[i];
         const LayerSpec &S = spec_.layers[i];
-        BCHK(bitnet_hip_residual_norm_rows_dev(x, have ? y : nullptr, width_, post, scale, L.norm1, spec_.norm_offset, spec_.eps, n, width_, ph_.p, ldh, f32_, stream_));
-        TRY(S.mixer == LayerSpec::Latent ? portion_latent(i, n, pos0) : portion_linear(i, n));
-        have = true, post = L.norm1b, scale = L.ls1;
-        if (S.ff > 0) {
-            BCHK(bitnet_hip_residual_norm_rows_dev(x, y, width_, post, scale, L.norm2, spec_.norm_offset, spec_.eps, n, width_, ph_.p, ldh, f32_, stream_));
+        if (run.enters) TRY(portion_loop_in(n));
+        TRY(portion_norm(n, &L.norm1, nullptr, ph_.p, ldh));
+        TRY(L.block[0].used ? portion_block(i, run.pass, 0, n, pos0) : S.mixer == LayerSpec::Latent ? portion_latent(i, run.pass, n, pos0) : portion_linear(i, run.pass, n));
+        pending_ = {y, L.norm1b, L.ls1, L.block[0].expert_up.w != nullptr};
+        if (S.parallel || (S.ff == 0 && S.experts.count == 0)) continue;
+        TRY(portion_norm(n, &L.norm2, nullptr, ph_.p, ldh));
+        if (L.block[1].used) {
+            TRY(portion_block(i, run.pass, 1, n, pos0));
+        } else {
             TRY(matmul(ph_.p, ldh, f32_, L.up, L.up_b, n, S.act_ff, 0, 0, pact_.p, L.down.ld, f32_));
             TRY(matmul(pact_.p, L.down.ld, f32_, L.down, L.down_b, n, 0, 0, 0, py_.p, width_, true));
-            post = L.norm2b, scale = L.ls2;
         }
+        pending_ = {y, L.norm2b, L.ls2, L.block[1].expert_up.w != nullptr};
     }
-    BCHK(bitnet_hip_residual_norm_rows_dev(x, y, width_, post, scale, nullptr, spec_.norm_offset, spec_.eps, n, width_, nullptr, 0, 0, stream_));
+    TRY(portion_norm(n, nullptr, nullptr, nullptr, 0));
     hidden_ = x + (n - 1) * (size_t)width_;
     return 0;
 }
@@ -569,7 +967,7 @@ int StackModel::prefill(int n, bool with_logits, int, float *elapsed_ms) {
     if (with_logits) {
         bitnet_hip_vector_input in = plain_input(hidden_);
         in.kind = BITNET_HIP_IN_NORM;
-        in.eps = spec_.eps, in.weight_offset = spec_.norm_offset, in.weight = final_norm_, in.n = width_;
+        in.eps = spec_.eps, in.weight_offset = spec_.norm_offset, in.weight = final_norm_.w, in.bias = final_norm_.bias, in.center = spec_.center, in.n = width_;
         BCHK(bitnet_hip_dense_logits_dev(&in, head_m_.w, vocab_, head_m_.cols, head_m_.ld, logits_, argmax_, token_, pos_, history_, n_forced_, s));
     }
     HCHK(hipEventRecord(e1.e, s));
@@ -596,7 +994,11 @@ int StackModel::forward(const int32_t *tokens, int n, const int32_t *want, int n
     hipStream_t s = (hipStream_t)stream_;
     HCHK(hipMemcpy(pwant_.p, want, k * 4, hipMemcpyHostToDevice));
     BCHK(bitnet_hip_gather_rows_dev((const float *)px_.p, (const int32_t *)pwant_.p, k, width_, (float *)pxw_.p, s));
-    BCHK(bitnet_hip_residual_norm_rows_dev((float *)pxw_.p, nullptr, 0, nullptr, nullptr, final_norm_, spec_.norm_offset, spec_.eps, k, width_, phw_.p, ldh, f32_, s));
+    bitnet_hip_sum_rows r;
+    memset(&r, 0, sizeof(r));
+    r.x = (float *)pxw_.p, r.m = k, r.width = width_, r.eps = spec_.eps, r.weight_offset = spec_.norm_offset, r.center = spec_.center, r.h_f32 = f32_;
+    r.weight = final_norm_.w, r.bias = final_norm_.bias, r.h = phw_.p, r.ldh = ldh;
+    BCHK(bitnet_hip_sum_norm_rows_dev(&r, s));
     TRY(matmul(phw_.p, ldh, f32_, head_m_, nullptr, k, 0, 0, 0, plog_.p, vocab_, true));
     HCHK(hipStreamSynchronize(s));
     HCHK(hipMemcpy(logits, plog_.p, k * vocab_ * 4, hipMemcpyDeviceToHost));

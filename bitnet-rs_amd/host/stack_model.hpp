@@ -1,9 +1,12 @@
-// stack_model.hpp -- a decoder made of a list of layers, each a sequence mixer and an optional feed-forward, with norms ahead of
-// and behind every sublayer.  The mechanisms are parameters (mixer kinds and their sizes, norm offset, layer scale, activations):
-// a design fills a StackSpec and hands its tensors over (see lasapel.cpp), the stack owns the device layout, the caches and
+// stack_model.hpp -- a decoder made of a list of layers, each a sequence mixer and an optional feed-forward.  The mechanisms are
+// parameters (mixer kinds and their sizes, kind of norm, layer scale, activations, experts, layers that run several times):
+// a design fills a StackSpec and hands its tensors over (see lasapel.cpp, mimolix.cpp), the stack owns the device layout, the caches and
 // states of the live sequence, the launches of a step and of a prompt's portions.
 //
-//   x <- x + ls1 * norm1b(mixer(norm1(x)));  x <- x + ls2 * norm2b(ff(norm2(x)))
+//   one sublayer behind the other   x <- x + ls1 * norm1b(mixer(norm1(x)));  x <- x + ls2 * norm2b(ff(norm2(x)))
+//   side by side                    x <- x + m * (mixer(norm1(x)) + ff(norm1(x)))
+// (no norm behind a sublayer: m takes the place of ls * norm).  A loop runs a range of layers several times with the same weights, every
+// pass with caches and states of its own and, ahead of its first layer, x <- W_in [x; embedding output].
 #pragma once
 
 #include <memory>
@@ -37,29 +40,59 @@ struct LinearSpec {  // linear attention with a constant decay per head (bitnet_
     std::vector<double> decay;
     int act_qkv = BITNET_HIP_ACT_SILU, act_gate = BITNET_HIP_ACT_SIGMOID;
 };
+struct AttentionSpec {  // keys and values of its own, shared by groups of query heads; one softmax map per head or two (bitnet_hip_gqa_*)
+    int heads = 0, kv_heads = 0, dim = 0, vdim = 0, maps = 1;
+    float scale = 1.f;
+    double temp_coef = 0.0, temp_every = 1.0;  // a query at position p is multiplied by 1 + coef ln(floor((p + 1) / every) + 1)
+    float diff = 0.f;                          // two maps: constant part of lambda, and 1 - diff scales the normed difference
+};
+struct DeltaSpec {  // gated delta rule (bitnet_hip_delta_*)
+    int heads = 0, kv_heads = 0, dim = 0, vdim = 0, taps = 1;
+    float unit_eps = 1e-6f;
+};
+struct ExpertsSpec {  // routed experts (bitnet_hip_experts_*); count 0: none
+    int count = 0, top = 0, ff = 0, act = BITNET_HIP_ACT_NONE;
+    float scale = 1.f;
+};
 struct LayerSpec {
-    enum Mixer { Latent, Linear } mixer = Latent;
+    enum Mixer { Latent, Linear, Attention, Delta } mixer = Latent;
     LatentSpec latent;
     LinearSpec linear;
-    int ff = 0;  // 0: no feed-forward
+    AttentionSpec attention;
+    DeltaSpec delta;
+    bool parallel = false;  // mixer and feed-forward side by side behind one norm (attention and delta mixers)
+    int ff = 0;             // every token's feed-forward: dense, or the expert shared by all; 0: none
     int act_ff = BITNET_HIP_ACT_NONE;
+    ExpertsSpec experts;
+};
+struct LoopSpec {  // layers start .. stop - 1 run `times` times in a row
+    int start = 0, stop = 0, times = 0;  // times 0: no loop
 };
 struct StackSpec {
     int width = 0, vocab = 0;
     float eps = 1e-6f;
-    float norm_offset = 0.f;  // block norms multiply by norm_offset + weight
+    float norm_offset = 0.f;     // block norms multiply by norm_offset + weight
+    bool center = false;         // block norms are layer norms, with a bias
+    float embed_scale = 1.f;
+    float residual_mult = 1.f;   // on a sublayer without a norm behind it
+    LoopSpec loop;
     std::vector<LayerSpec> layers;
 };
 
 // One layer's tensors as the loader hands them over: bf16 matrices [out, in], f32 vectors.
 struct StackLayerWeights {
-    std::vector<float> norm1, norm1b, ls1, norm2, norm2b, ls2;  // empty ls: no layer scale
+    std::vector<float> norm1, norm1b, ls1, norm2, norm2b, ls2;  // empty ls: no layer scale; empty norm1b, norm2b: no norm behind the sublayer
+    std::vector<float> norm1_bias, norm2_bias;
     const uint16_t *dq = nullptr, *uq = nullptr, *dkv = nullptr, *uk = nullptr, *uv = nullptr, *o = nullptr;
     std::vector<float> dq_norm, dkv_norm, sink;
     const uint16_t *q = nullptr, *k = nullptr, *v = nullptr, *g = nullptr;
     std::vector<float> out_norm;
-    const uint16_t *up = nullptr, *down = nullptr;
+    std::vector<float> q_norm, k_norm, lq1, lk1, lq2, lk2;              // attention; empty q_norm, k_norm: no norm
+    const uint16_t *b = nullptr, *a = nullptr;                          // delta: step size and decay, one row per head
+    std::vector<float> q_conv, k_conv, v_conv, a_log, dt_bias;          // [channels][taps]
+    const uint16_t *up = nullptr, *down = nullptr, *router = nullptr;
     std::vector<float> up_b, down_b;
+    std::vector<const uint16_t *> expert_up, expert_down;
 };
 
 class StackModel : public Sequence {
@@ -68,7 +101,8 @@ class StackModel : public Sequence {
     ~StackModel() override;
 
     int set_layer(int layer, const StackLayerWeights &w);
-    int set_globals(const uint16_t *embed, const std::vector<float> &final_norm, const uint16_t *head);
+    int set_globals(const uint16_t *embed, const std::vector<float> &final_norm, const std::vector<float> &final_bias, const uint16_t *head,
+                    const uint16_t *loop_in);
 
     int prefill(int n, bool with_logits, int digits, float *elapsed_ms) override;
     int forward(const int32_t *tokens, int n, const int32_t *want, int n_want, float *logits) override;
@@ -85,19 +119,42 @@ class StackModel : public Sequence {
         uint16_t *w = nullptr;
         int rows = 0, cols = 0, ld = 0;  // cols: padded to a multiple of 8 for the matrix-vector product
     };
-    struct Cache {  // one layer's latent cache
-        void *c = nullptr, *r = nullptr;
+    struct Slot {  // what one pass of a layer carries from token to token
+        void *c = nullptr, *r = nullptr;       // latent: rows, rotated parts
+        void *k = nullptr, *v = nullptr;       // attention: keys, transposed values
+        float *state = nullptr, *ring = nullptr;  // linear, delta: state; delta: the last inputs of its convolution
+        size_t state_bytes = 0;
+    };
+    struct Norm {
+        float *w = nullptr, *bias = nullptr;
+    };
+    // Sublayers that read one norm and whose outputs add up, as two products and what lies between them.  A row of activations is
+    // [mixer output, ko | feed-forward, fs | the mixer's projections]; `in` makes everything behind the mixer's output from the normed row (and
+    // the tail: rows whose results stay f32 in a prompt), `out` takes the first ko + fs columns back to the residual stream.
+    struct Block {
+        bool used = false, mixer = false;
+        Norm norm;
+        Matrix in, out, expert_up, expert_down;
+        int ko = 0, fs = 0, main = 0, tail = 0, gates = 0;  // gates: rows of the tail ahead of the router
+        float *in_bias = nullptr, *out_bias = nullptr;
     };
     struct Layer {
-        float *norm1 = nullptr, *norm1b = nullptr, *ls1 = nullptr, *norm2 = nullptr, *norm2b = nullptr, *ls2 = nullptr;
+        Norm norm1, norm2;
+        float *norm1b = nullptr, *ls1 = nullptr, *norm2b = nullptr, *ls2 = nullptr;
+        std::vector<Slot> slots;  // one per pass
+        Block block[2];
+        // attention
+        float *q_norm = nullptr, *k_norm = nullptr, *q_factor = nullptr;
+        float lambda = 0.f;
+        // delta
+        float *conv = nullptr, *decay_rate = nullptr, *dt_bias = nullptr;
         // latent
         int dimp = 0, rotp = 0, vdimp = 0, ldc = 0;
         Matrix down_q, uq, uk, uk_t, uv, o;  // down_q: dq, followed by dkv where the layer has one
         float *dq_norm = nullptr, *dkv_norm = nullptr, *sink = nullptr, *cos = nullptr, *sin = nullptr;
-        Cache cache;
-        // linear
+        // linear (out_norm: delta too)
         Matrix qkvg;
-        float *out_norm = nullptr, *decay_pow = nullptr, *state = nullptr;
+        float *out_norm = nullptr, *decay_pow = nullptr;
         // feed-forward
         Matrix up, down;
         float *up_b = nullptr, *down_b = nullptr;
@@ -110,6 +167,12 @@ class StackModel : public Sequence {
     // the sublayer whose output is still to be added to the residual stream
     struct Pending {
         const float *y = nullptr, *w = nullptr, *scale = nullptr;
+        bool experts = false;  // a portion's routed rows join in
+    };
+    struct Run {
+        size_t layer;
+        int pass;
+        bool enters;  // the first layer of a pass of the loop
     };
 
     int grow(Buffer &b, size_t bytes);
@@ -117,32 +180,46 @@ class StackModel : public Sequence {
     int upload(T **dst, const std::vector<T> &src);
     int upload_matrix(Matrix &m, const std::vector<uint16_t> &rows, int n_rows, int cols);
     int rope_tables(const RotarySpec &r, float **cos, float **sin);
-    const Layer &kv_layer(size_t i) const { return layers_[spec_.layers[i].latent.kv_from >= 0 ? (size_t)spec_.layers[i].latent.kv_from : i]; }
-    void attention_args(size_t i, bitnet_hip_latent_attention &a) const;
-    void latent_args(size_t i, const float *z, size_t ldz, void *cq, size_t ldcq, bitnet_hip_latent_rows &r) const;
+    int query_factors(const AttentionSpec &a, float **out);
+    int plan_runs();
+    int plan_block(size_t i, int which, bool mixer, bool ff);
+    bool alloc(void **p, size_t bytes);
+    int set_block(size_t i, int which, const StackLayerWeights &w);
+    const Slot &kv_slot(size_t i, int pass) const { return layers_[spec_.layers[i].latent.kv_from >= 0 ? (size_t)spec_.layers[i].latent.kv_from : i].slots[(size_t)pass]; }
+    void attention_args(size_t i, int pass, bitnet_hip_latent_attention &a) const;
+    void latent_args(size_t i, int pass, const float *z, size_t ldz, void *cq, size_t ldcq, bitnet_hip_latent_rows &r) const;
+    bitnet_hip_gqa gqa_args(size_t i, int pass) const;
+    bitnet_hip_delta delta_args(size_t i, int pass) const;
     // single token
     int gemv(const bitnet_hip_vector_input &in, const Matrix &m, const float *bias, int act0, int act1, size_t split, float *y,
              const bitnet_hip_latent_rows *latent = nullptr);
-    bitnet_hip_vector_input block_input(const float *norm);
-    int step_latent(size_t i);
-    int step_linear(size_t i);
+    bitnet_hip_vector_input block_input(const Norm &norm);
+    void add_pending(bitnet_hip_vector_input &in);
+    int step_latent(size_t i, int pass);
+    int step_linear(size_t i, int pass);
+    int step_block(size_t i, int pass, int which);
+    int step_loop_in();
     // portion of n tokens
     int matmul(const void *a, size_t lda, bool a_f32, const Matrix &m, const float *bias, size_t n, int act0, int act1, size_t split, void *c, size_t ldc,
                bool c_f32);
     int portion(int n, int pos0);
-    int portion_latent(size_t i, size_t n, size_t pos0);
-    int portion_linear(size_t i, size_t n);
+    int portion_norm(size_t n, const Norm *norm, const float *x2, void *h, size_t ldh);
+    int portion_latent(size_t i, int pass, size_t n, size_t pos0);
+    int portion_linear(size_t i, int pass, size_t n);
+    int portion_block(size_t i, int pass, int which, size_t n, size_t pos0);
+    int portion_loop_in(size_t n);
     int portion_buffers(size_t n);
     int set_position(int p);
 
     StackSpec spec_;
     bool f32_ = false;
-    size_t cap_ = 0;  // positions the caches hold, a multiple of 64
+    size_t cap_ = 0;  // positions the caches hold, a multiple of 128
     std::vector<Layer> layers_;
+    std::vector<Run> runs_;
     size_t layers_set_ = 0;
-    Matrix embed_, head_m_;
+    Matrix embed_, head_m_, loop_in_;
     const uint16_t *head_ = nullptr;
-    float *final_norm_ = nullptr;
+    Norm final_norm_;
     size_t weight_bytes_ = 0;
     std::vector<void *> owned_;  // every fixed allocation
     struct RopeTable {
@@ -150,16 +227,21 @@ class StackModel : public Sequence {
         float *cos, *sin;
     };
     std::vector<RopeTable> ropes_;
-    // single-token vectors (f32)
+    // single-token vectors (f32); x0_: the embedding output
+    float *x0_ = nullptr, *row_ = nullptr, *h_ = nullptr, *eact_ = nullptr;
+    int32_t *eids_ = nullptr;
     float *x_[2] = {nullptr, nullptr}, *z_ = nullptr, *q_ = nullptr, *qabs_ = nullptr, *att_ = nullptr, *y_[2] = {nullptr, nullptr}, *act_ = nullptr,
           *lin_ = nullptr, *lino_ = nullptr, *scratch_ = nullptr;
     void *argmax_ = nullptr;
-    int cur_ = 0;  // which x_ the step's residual stream is in
+    const float *cur_ = nullptr;  // where the step's residual stream is
+    float *next_x() const { return cur_ == x_[0] ? x_[1] : x_[0]; }
     Pending pending_;
     const float *hidden_ = nullptr;  // residual stream of the last position run
     // portion buffers; T = bf16, or f32 in 32-bit mode
     size_t rows_cap_ = 0;
     Buffer px_, ph_, pz_, pcq_, pq_, pqf_, pqabs_, patt_, py_, pact_, pk_, pvt_, plin_, plinf_, plino_, pgate_, pscratch_, plws_, pwant_, pxw_, phw_, plog_;
+    Buffer px0_, pcat_, prow_, ptail_, pqk_, pv_, pgates_, pplan_, peact_, peout_;
+    bitnet_hip_experts_plan plan_;
 };
 
 }  // namespace bitnet_host

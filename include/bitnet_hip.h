@@ -573,14 +573,34 @@ int bitnet_hip_hbm_read_ceiling(size_t bytes, int iters, double *best_gbs, doubl
 #define BITNET_HIP_ACT_SIGMOID 2
 #define BITNET_HIP_ACT_RELU2 3 /* square of relu */
 
-/* out[i][width] = table[tokens[*offset + i]] as f32 (offset NULL = 0) */
+/* out[i][width] = scale * table[tokens[*offset + i]] as f32 (offset NULL = 0) */
 int bitnet_hip_embed_bf16_dev(const uint16_t *table_dev, size_t ld, const int32_t *tokens_dev, const int32_t *offset_dev, size_t n,
-                              size_t width, size_t vocab, float *out_dev, void *stream);
+                              size_t width, size_t vocab, float scale, float *out_dev, void *stream);
 /* x[i] += scale * norm(y[i]; post_weight) (y NULL: skipped), then h[i] = norm(x[i]; next_weight) (h NULL: skipped), padding columns of h
  * zero; norm(v; w) = v / sqrt(mean(v^2) + eps) * (weight_offset + w). */
 int bitnet_hip_residual_norm_rows_dev(float *x_dev, const float *y_dev, size_t ldy, const float *post_weight_dev, const float *scale_dev,
                                       const float *next_weight_dev, float weight_offset, float eps, size_t m, size_t width, void *h_dev,
                                       size_t ldh, int h_f32, void *stream);
+/* Rows of a block whose sublayers' outputs add up: x[i] += mult * (y[i] + sum over k < top of slot_weights[i][k] * expert_rows[slots[i][k]])
+ * (y NULL: nothing is added; top 0: no experts), then h[i] (NULL: skipped) = norm(x[i]; weight), padding columns zero, or -- x2 given --
+ * the unnormed [x[i]; x2[i]].  center: layer norm, (v - mean) / sqrt(variance + eps) * weight + bias. */
+typedef struct bitnet_hip_sum_rows {
+    float *x;
+    size_t m, width;
+    const float *y;
+    size_t ldy;
+    float mult;
+    const void *expert_rows; /* f32 with h_f32, else bf16 */
+    size_t ld_expert, top;
+    const int32_t *slots;
+    const float *slot_weights;
+    const float *weight, *bias, *x2;
+    float weight_offset, eps;
+    int32_t center, h_f32;
+    void *h;
+    size_t ldh;
+} bitnet_hip_sum_rows;
+int bitnet_hip_sum_norm_rows_dev(const bitnet_hip_sum_rows *rows, void *stream);
 /* h[i] = norm(o[i]; weight) * gate[i] over n columns; the mean divides by mean_n (padded heads hold zeros). */
 int bitnet_hip_gated_norm_rows_dev(const float *o_dev, size_t ldo, const float *weight_dev, const void *gate_dev, size_t ldg, float eps,
                                    int gate_f32, size_t m, size_t n, size_t mean_n, void *h_dev, size_t ldh, int h_f32,
@@ -597,6 +617,7 @@ int bitnet_hip_dense_matmul_dev(const void *a_dev, size_t lda, int a_f32, const 
 #define BITNET_HIP_IN_PLAIN 0
 #define BITNET_HIP_IN_NORM 1          /* norm(x; weight) [* gate] */
 #define BITNET_HIP_IN_RESIDUAL_NORM 2 /* x' = x + scale * norm(y; post_weight) -> x_out (not x itself); norm(x'; weight) */
+#define BITNET_HIP_IN_CONCAT 3        /* [x'; x2], n elements each */
 typedef struct bitnet_hip_vector_input {
     const float *x;
     int32_t kind;
@@ -604,6 +625,11 @@ typedef struct bitnet_hip_vector_input {
     const float *weight, *y, *post_weight, *scale, *gate; /* y NULL: nothing is added; scale, gate NULL: 1 */
     float *x_out;                                         /* NULL: not stored */
     int32_t n, mean_n;                                    /* elements, and what the mean divides by (0 = n) */
+    /* post_weight NULL: x' = x + mult * y.  center: norm(x') is a layer norm with bias.  h_out (nullable): the vector formed is stored */
+    float mult;
+    int32_t center;
+    const float *bias, *x2;
+    float *h_out;
 } bitnet_hip_vector_input;
 /* The latent rows of a down-projection output z [m][ldz] = [q_rank | kv_rank | rot_dim]: cq[i] = norm(first q_rank; q_weight) (cq NULL:
  * skipped), and at position p = *pos + i of the caches the latent norm(next kv_rank; kv_weight) and the last rot_dim rotated by the
@@ -670,6 +696,93 @@ int bitnet_hip_linear_chunked_supported(size_t dimp, size_t vdimp);
 int bitnet_hip_linear_chunked_dev(const uint16_t *qkv_dev, size_t ld, size_t n, size_t heads, size_t dimp, size_t vdimp,
                                   const float *decay_pow_dev, float *state_dev, float *out_dev, size_t ldo, void *workspace_dev,
                                   size_t workspace_bytes, void *stream);
+
+/* Attention with heads of its own keys and values, query heads sharing them in groups of heads / kv_heads; causal.  maps = 2: differential
+ * attention -- queries and keys of a head are [map 1 | map 2], both maps weigh the same values, and the output is
+ * o = a1 - lambda a2, then o / sqrt(mean(o^2) + eps) * out_scale over the head's vdim values.  maps = 1: a1.
+ * A row of projections is [heads * maps * dimp | kv_heads * maps * dimp | kv_heads * vdimp], heads zero-padded to multiples of 32.
+ * Queries and keys are normed per head and map (rms over dim, plain weight; NULL: not at all), a query at position p is then multiplied by
+ * q_factor[p] (score scale and whatever depends on the position).  Caches: keys [kv_heads][maps][capacity][dimp], values transposed
+ * [kv_heads][vdimp][capacity], bf16 or f32, zero-filled once. */
+typedef struct bitnet_hip_gqa {
+    size_t heads, kv_heads, maps, dim, dimp, vdim, vdimp, capacity; /* capacity % 128 == 0 */
+    float eps, lambda, out_scale;
+    const float *q_weight, *k_weight; /* [dim] */
+    const float *q_factor;            /* [capacity] */
+    void *kcache, *vcache;
+} bitnet_hip_gqa;
+size_t bitnet_hip_gqa_scratch_bytes(size_t heads, size_t maps, size_t vdimp, size_t nq);
+/* n rows of projections from position *pos on: queries in place, keys and values into the caches. */
+int bitnet_hip_gqa_rows_dev(const bitnet_hip_gqa *attn, void *rows_dev, size_t ld, int rows_f32, int cache_f32, const int32_t *pos_dev, size_t n,
+                            void *stream);
+/* The decode step on a bf16 cache: one raw f32 row of projections at *pos, appended by the same launch; leaves records in scratch.
+ * dimp <= 256, vdimp <= 256 (bitnet_hip_gqa_supported). */
+int bitnet_hip_gqa_supported(size_t dimp, size_t vdimp);
+int bitnet_hip_gqa_step_dev(const bitnet_hip_gqa *attn, const float *row_dev, const int32_t *pos_dev, float *scratch_dev, void *stream);
+/* Any size and either cache: queries (as gqa_rows leaves them) at *pos + q0 + i; records in scratch. */
+int bitnet_hip_gqa_any_dev(const bitnet_hip_gqa *attn, const void *q_dev, size_t ldq, int q_f32, int cache_f32, const int32_t *pos_dev, size_t q0,
+                           size_t nq, float *scratch_dev, void *stream);
+/* The records of nq queries -> out [nq][ldo], f32 or bf16. */
+int bitnet_hip_gqa_merge_dev(const bitnet_hip_gqa *attn, const int32_t *pos_dev, size_t q0, size_t nq, const float *scratch_dev, void *out_dev,
+                             size_t ldo, int out_bf16, void *stream);
+/* A portion of a prompt, bf16: the LAST nq of n_ctx positions attend (all of them in the caches); q as gqa_rows leaves it. */
+int bitnet_hip_gqa_prefill_dev(const bitnet_hip_gqa *attn, const uint16_t *q_dev, size_t ldq, size_t n_ctx, size_t nq, uint16_t *out_dev, size_t ldo,
+                               void *stream);
+
+/* Gated delta rule.  A row of projections is [q kv_heads * dimp | k kv_heads * dimp | v heads * vdimp | gate heads * vdimp], and apart from it
+ * [b heads | a heads] f32; heads zero-padded to multiples of 32.  q, k, v pass a causal convolution of `taps` tokens per channel and
+ * silu; q and k are divided by sqrt(sum of squares + unit_eps) per head, q multiplied by q_scale; head h uses q/k head
+ * h / (heads / kv_heads).  beta = sigmoid(b), g = exp(-decay_rate * softplus(a + dt_bias)).
+ *   S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q
+ * out = o / sqrt(mean(o^2 over vdim) + eps) * norm * silu(gate).  state f32 [heads][dimp][vdimp]; ring f32 [taps][channels]: the inputs of
+ * position p at p % taps (positions before the start are not read). */
+typedef struct bitnet_hip_delta {
+    size_t heads, kv_heads, dim, dimp, vdim, vdimp, taps;
+    const float *conv;                /* [taps][2 kv_heads dimp + heads vdimp], last row = the current token */
+    const float *decay_rate, *dt_bias; /* [heads] */
+    const float *norm;                /* [vdimp] */
+    float q_scale, unit_eps, eps;
+    float *state, *ring;
+} bitnet_hip_delta;
+int bitnet_hip_delta_supported(size_t dimp, size_t vdimp);         /* <= 256 each */
+int bitnet_hip_delta_chunked_supported(size_t dimp, size_t vdimp); /* dimp <= 128, vdimp <= 256 */
+/* one token: f32 row and gates; out f32 [heads * vdimp] */
+int bitnet_hip_delta_step_dev(const bitnet_hip_delta *d, const float *row_dev, const float *ba_dev, const int32_t *pos_dev, float *out_dev, void *stream);
+/* n tokens from *pos on: qk f32 [n][2 kv_heads dimp] (unit vectors), v [n][heads vdimp] (type of the rows), gates f32 [n][2 heads] =
+ * (log g, beta) of each head */
+int bitnet_hip_delta_rows_dev(const bitnet_hip_delta *d, const void *rows_dev, size_t ld, int rows_f32, const float *ba_dev, size_t ldba,
+                              const int32_t *pos_dev, size_t n, float *qk_dev, void *v_dev, float *gates_dev, void *stream);
+/* the last inputs of a portion into the ring, behind delta_rows */
+int bitnet_hip_delta_keep_dev(const bitnet_hip_delta *d, const void *rows_dev, size_t ld, int rows_f32, const int32_t *pos_dev, size_t n, void *stream);
+/* those n tokens through the recurrence, out [n][ldo] of the rows' type: token by token, or in chunks of 64 on the matrix cores (bf16 rows) */
+int bitnet_hip_delta_recurrent_dev(const bitnet_hip_delta *d, const float *qk_dev, const void *v_dev, const float *gates_dev, const void *rows_dev,
+                                   size_t ld, int rows_f32, size_t n, void *out_dev, size_t ldo, void *stream);
+size_t bitnet_hip_delta_workspace_bytes(size_t n, size_t heads, size_t dimp, size_t vdimp);
+int bitnet_hip_delta_chunked_dev(const bitnet_hip_delta *d, const float *qk_dev, const uint16_t *v_dev, const float *gates_dev, const uint16_t *rows_dev,
+                                 size_t ld, size_t n, uint16_t *out_dev, size_t ldo, void *workspace_dev, size_t workspace_bytes, void *stream);
+
+/* Mixture of experts.  scores = softmax(logits); the `top` largest (lower index first among equals) get weights score / (their sum + 1e-20) *
+ * scale.  experts <= 1024, top <= 32. */
+typedef struct bitnet_hip_experts_plan { /* where m tokens' choices lie in a workspace */
+    int32_t *counts, *offsets, *n_tiles, *tiles; /* tiles: (expert, first slot, slots, 0) */
+    int32_t *ids, *slots, *tokens;               /* [m][top], [m][top], [m * top]: slot -> token */
+    float *weights;                              /* [m][top] */
+    size_t m, experts, top, tile, max_tiles;
+} bitnet_hip_experts_plan;
+size_t bitnet_hip_experts_plan_bytes(size_t m, size_t experts, size_t top);
+/* lays a plan out in memory that was zero-filled once (plans of other sizes may have used it); tile: rows of a product's tile (64 or 128) */
+int bitnet_hip_experts_plan_make(void *workspace_dev, size_t bytes, size_t m, size_t experts, size_t top, size_t tile, bitnet_hip_experts_plan *plan);
+int bitnet_hip_experts_route_dev(const float *logits_dev, size_t ldz, float scale, const bitnet_hip_experts_plan *plan, void *stream);
+/* C[slot] = act(A[row of slot] . W[expert of slot]^T): rows are the slot's token (gather) or the slot itself.  W bf16 [experts][n][ldw] */
+int bitnet_hip_experts_matmul_dev(const bitnet_hip_experts_plan *plan, int gather, const void *a_dev, size_t lda, int a_f32, const uint16_t *w_dev,
+                                  size_t n, size_t k, size_t ldw, int act, void *c_dev, size_t ldc, int c_f32, void *stream);
+/* One token: y[k][ldy] = weight_k * act(W[expert k] . x), the choice made from the logits by the same launch and stored in ids [top]. */
+int bitnet_hip_experts_up_dev(const float *logits_dev, size_t experts, size_t top, float scale, const float *x_dev, const uint16_t *w_dev, size_t rows,
+                              size_t cols, size_t ld, int act, float *y_dev, size_t ldy, int32_t *ids_dev, void *stream);
+/* y = W0 . x0 + bias + sum over k of W1[ids[k]] . x1[k]; W1 bf16 [experts][rows][ld1] */
+int bitnet_hip_experts_out_dev(const float *x0_dev, const uint16_t *w0_dev, size_t cols0, size_t ld0, const float *bias_dev, const float *x1_dev,
+                               size_t ldx1, const uint16_t *w1_dev, size_t cols1, size_t ld1, const int32_t *ids_dev, size_t top, size_t rows,
+                               float *y_dev, void *stream);
 
 #ifdef __cplusplus
 }
