@@ -130,6 +130,25 @@ def query_temperature(p, m):
     return 1.0 + s["coef"] * math.log(math.floor((p + 1) / s["every"]) + 1.0)
 
 
+def softmax_maps(q, k, v):
+    """q [n, heads, maps, dim], k [n, kv heads, maps, dim], v [n, kv heads, vdim]: causal softmax of q.k over the values, per head and map"""
+    n, H, M, _ = q.shape
+    out = np.zeros((n, H, M, v.shape[2]), F)
+    for a in range(H):
+        g = a // (H // k.shape[1])
+        for j in range(M):
+            s = q[:, a, j] @ k[:, g, j].T
+            s[np.triu_indices(n, 1)] = -np.inf
+            e = np.exp(s - s.max(axis=1, keepdims=True))
+            out[:, a, j] = e / e.sum(axis=1, keepdims=True) @ v[:, g]
+    return out
+
+
+def difference(maps, lam, diff, eps):
+    """[..., 2, vdim] -> [..., vdim]"""
+    return rms_divide(maps[..., 0, :] - lam * maps[..., 1, :], eps) * (1.0 - diff)
+
+
 def differential_attention(h, t, p, m, eps):
     """two softmax maps per head over the same values; the second, weighted, is taken from the first"""
     n, H, G, D, V = len(h), m["heads"], m["kv_heads"], m["dim"], m["vdim"]
@@ -137,17 +156,8 @@ def differential_attention(h, t, p, m, eps):
     k = norm_plain((h @ t[p + "k"].T).reshape(n, G, 2, D), t[p + "k.norm"], eps)
     v = (h @ t[p + "v"].T).reshape(n, G, V)
     lam = math.exp(t[p + "lq1"] @ t[p + "lk1"]) - math.exp(t[p + "lq2"] @ t[p + "lk2"]) + m["diff"]
-    temp = np.array([query_temperature(i, m) for i in range(n)])
-    out = np.zeros((n, H, V), F)
-    for a in range(H):
-        g = a // (H // G)
-        maps = []
-        for j in range(2):
-            s = (q[:, a, j] * temp[:, None]) @ k[:, g, j].T * m["scale"]
-            s[np.triu_indices(n, 1)] = -np.inf
-            e = np.exp(s - s.max(axis=1, keepdims=True))
-            maps.append(e / e.sum(axis=1, keepdims=True) @ v[:, g])
-        out[:, a] = rms_divide(maps[0] - lam * maps[1], eps) * (1.0 - m["diff"])
+    factor = np.array([query_temperature(i, m) * m["scale"] for i in range(n)])
+    out = difference(softmax_maps(q * factor[:, None, None, None], k, v), lam, m["diff"], eps)
     return out.reshape(n, H * V) @ t[p + "o"].T
 
 
@@ -166,6 +176,16 @@ def unit(x):
     return x / np.sqrt(np.sum(x * x, axis=-1, keepdims=True) + 1e-6)
 
 
+def delta_rule(q, k, v, decay, beta, S):
+    """one head: q, k [n, dim], v [n, vdim], S [dim, vdim] -> outputs, S behind the last token"""
+    o = np.zeros_like(v)
+    for i in range(len(q)):
+        S = decay[i] * S
+        S = S + np.outer(k[i], beta[i] * (v[i] - S.T @ k[i]))
+        o[i] = S.T @ q[i]
+    return o, S
+
+
 def gated_delta(h, t, p, m, eps):
     n, H, G, D, V = len(h), m["heads"], m["kv_heads"], m["dim"], m["vdim"]
     q, k, v = (silu(short_convolution(h @ t[p + x].T, t[p + x + ".conv"])) for x in "qkv")
@@ -175,11 +195,7 @@ def gated_delta(h, t, p, m, eps):
     o = np.zeros((n, H, V), F)
     for a in range(H):
         g = a // (H // G)
-        S = np.zeros((D, V), F)
-        for i in range(n):
-            S = decay[i, a] * S
-            S = S + np.outer(k[i, g], beta[i, a] * (v[i, a] - S.T @ k[i, g]))
-            o[i, a] = S.T @ q[i, g]
+        o[:, a], _ = delta_rule(q[:, g], k[:, g], v[:, a], decay[:, a], beta[:, a], np.zeros((D, V), F))
     y = norm_plain(o, t[p + "norm"], eps).reshape(n, H * V) * silu(h @ t[p + "g"].T)
     return y @ t[p + "o"].T
 

@@ -69,7 +69,107 @@ def lasapel(layers, width=112, vocab=150, eps=1e-5) -> dict:
     return {"architecture": "Lasapel", "vocab": vocab, "width": width, "norm": {"eps": eps}, "layers": layers}
 
 
+def expert_mlp(experts=6, top=3, ff=24, scale=1.7, shared=40) -> dict:
+    m = {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": experts, "scale": scale, "top": top}}
+    if shared:
+        m["shared"] = {"ff": shared}
+    return m
+
+
+def attention_layer(heads=6, kv_heads=3, dim=20, vdim=28, scale=0.31, diff=0.2, coef=0.4, every=8, mlp=None) -> dict:
+    return {"type": "attention", "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": scale, "diff": diff,
+                                           "q_temp": {"coef": coef, "every": every}}, "mlp": mlp}
+
+
+def delta_layer(heads=4, kv_heads=2, dim=24, vdim=40, conv=4, mlp=None) -> dict:
+    return {"type": "delta", "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "conv": conv}, "mlp": mlp}
+
+
+def mimolix(layers, width=112, vocab=150, eps=1e-5, mult=0.4, embed=3.0, loop=None) -> dict:
+    c = {"architecture": "Mimolix", "vocab": vocab, "width": width, "norm": {"eps": eps}, "residual_mult": mult, "embedding": {"scale": embed}, "layers": layers}
+    if loop:
+        c["loop"] = dict(zip(("start", "stop", "times"), loop))
+    return c
+
+
+def random_mimolix(config: dict, seed: int) -> dict:
+    """bf16-representable weights, everything away from its neutral value.  A router's choice must not hang on the last bit of its input: the
+    first columns of an embedding row say which experts the token takes (well apart from each other and from the rest), nothing is added to these
+    columns behind the embedding, and the router reads them (and a little of the rest)."""
+    g = np.random.default_rng(seed)
+    W, V = config["width"], config["vocab"]
+    codes = max([layer["mlp"]["router"]["experts"] for layer in config["layers"] if layer["mlp"]], default=0)
+    tops = max([layer["mlp"]["router"]["top"] for layer in config["layers"] if layer["mlp"]], default=0)
+    t = {}
+
+    def mat(name, rows, cols, gain=1.0):
+        t[name] = rounded(g.standard_normal((rows, cols)) * gain / np.sqrt(cols))
+
+    def back(name, cols):  # a matrix back to the residual stream
+        mat(name, W, cols)
+        t[name][:codes] = 0.0
+
+    def around(name, n, centre, spread):
+        t[name] = rounded(centre + spread * g.standard_normal(n))
+
+    def norm(name):
+        around(name, W, 1.0, 0.2)
+        around(name + ".b", W, 0.0, 0.2)
+        t[name][:codes], t[name + ".b"][:codes] = 1.0, 0.0
+
+    t["embed"] = g.standard_normal((V, W)) / config["embedding"]["scale"]
+    for i in range(V):
+        order = g.permutation(codes)
+        t["embed"][i, order] = (-0.5 - g.random(codes)) / config["embedding"]["scale"]
+        first = order[:tops + 1]
+        t["embed"][i, first] = (2.5 - 0.7 * np.arange(len(first))) / config["embedding"]["scale"]
+    t["embed"] = rounded(t["embed"])
+    for i, layer in enumerate(config["layers"]):
+        p, m = f"l{i}.", layer["mixer"]
+        H, G, D, VD, q = m["heads"], m["kv_heads"], m["dim"], m["vdim"], f"l{i}.mix."
+        norm(p + "norm1")
+        if layer["type"] == "attention":
+            for name, rows in (("q", H * 2 * D), ("k", G * 2 * D), ("v", G * VD)):
+                mat(q + name, rows, W)
+            around(q + "q.norm", D, 1.2, 0.3)
+            around(q + "k.norm", D, 1.2, 0.3)
+            for name in ("lq1", "lk1", "lq2", "lk2"):
+                around(q + name, D, 0.0, 0.15)
+        else:
+            for name, rows in (("q", G * D), ("k", G * D), ("v", H * VD)):
+                mat(q + name, rows, W)
+                t[q + name + ".conv"] = rounded(0.5 * g.standard_normal((rows, m["conv"])))
+            for name, rows in (("b", H), ("a", H), ("g", H * VD)):
+                mat(q + name, rows, W)
+            around(q + "A_log", H, -0.5, 0.7)
+            t[q + "A_log"][0] = -5.0  # one head that forgets slowly
+            around(q + "dt_bias", H, -1.0, 0.7)
+            around(q + "norm", VD, 1.0, 0.3)
+        back(q + "o", H * VD)
+        if layer["mlp"]:
+            f, r = p + "mlp.", layer["mlp"]["router"]
+            t[f + "router"] = rounded(np.concatenate([2.0 * np.eye(r["experts"], codes), 0.02 * g.standard_normal((r["experts"], W - codes))], axis=1))
+            parts = {f"e{e}.": layer["mlp"]["expert"]["ff"] for e in range(r["experts"])}
+            if "shared" in layer["mlp"]:
+                parts["shared."] = layer["mlp"]["shared"]["ff"]
+            for name, ff in parts.items():
+                mat(f + name + "up", ff, W)
+                back(f + name + "down", ff)
+    if config.get("loop"):
+        t["loop.in"] = g.standard_normal((W, 2 * W)) * 0.6 / np.sqrt(W)
+        t["loop.in"][:codes] = 0.0
+        t["loop.in"][:codes, :codes] = t["loop.in"][:codes, W:W + codes] = 0.5 * np.eye(codes)
+        t["loop.in"] = rounded(t["loop.in"])
+    norm("final.norm")
+    mat("head", V, W)
+    return t
+
+
 def random_tensors(config: dict, seed: int) -> dict:
+    return {"Lasapel": random_lasapel, "Mimolix": random_mimolix}[config["architecture"]](config, seed)
+
+
+def random_lasapel(config: dict, seed: int) -> dict:
     """bf16-representable weights; every norm, scale, bias and sink away from its neutral value"""
     g = np.random.default_rng(seed)
     W, V = config["width"], config["vocab"]

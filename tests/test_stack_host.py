@@ -23,7 +23,32 @@ BASE = u.lasapel([u.latent_layer(ff=24), u.lightning_layer()], width=40, vocab=2
 
 def test_registry_names(built):
     names = built.registered_models()
-    assert "Lasapel" in names and ".gguf" in names
+    assert "Lasapel" in names and "Mimolix" in names and ".gguf" in names
+
+
+PARALLEL = u.mimolix([u.delta_layer(mlp=u.expert_mlp()), u.attention_layer()], width=40, vocab=20, loop=(0, 1, 2))
+
+
+@pytest.mark.parametrize("change,message", [
+    (lambda c: c.pop("residual_mult"), "residual_mult: missing"),
+    (lambda c: c["embedding"].pop("scale"), "embedding.scale: missing"),
+    (lambda c: c["loop"].update(stop=3), "loop's range"),
+    (lambda c: c["loop"].update(times=0), "loop.times: not an integer"),
+    (lambda c: c["layers"][0].update(type="latent_attention"), r"layers\[0\].type: unknown mixer"),
+    (lambda c: c["layers"][0]["mixer"].pop("conv"), r"layers\[0\].mixer.conv: missing"),
+    (lambda c: c["layers"][0]["mixer"].update(dim=300), "layer 0: delta"),
+    (lambda c: c["layers"][0]["mlp"].update(kind="dense"), r"layers\[0\].mlp.kind: unknown"),
+    (lambda c: c["layers"][0]["mlp"]["router"].update(top=7), "layer 0: experts"),
+    (lambda c: c["layers"][1]["mixer"].update(kv_heads=4), "layer 1: attention"),
+    (lambda c: c["layers"][1]["mixer"]["q_temp"].pop("every"), r"layers\[1\].mixer.q_temp.every: missing"),
+    (lambda c: c["layers"][1]["mixer"].pop("diff"), r"layers\[1\].mixer.diff: missing"),
+])
+def test_bad_parallel_configurations_say_why(built, tmp_path, change, message):
+    c = copy.deepcopy(PARALLEL)
+    change(c)
+    path = u.save_model(str(tmp_path), c, u.random_tensors(PARALLEL, 1))
+    with pytest.raises(built.BitNetHipError, match=message):
+        built.open_model(path)
 
 
 def broken(change):
@@ -85,6 +110,14 @@ def test_entry_points_check_shapes_before_any_launch(built):
         (lambda: hip.dense_gemv_dev(8, 8, 4, 64, 64, 8, kind=built.IN_RESIDUAL_NORM, weight=8, res=8, post_weight=8, x_out=8, n=64), "buffer of its own"),
         (lambda: hip.linear_recurrent_dev(8, 96, 1, 1, 32, 24, 8, 8, 8, 32), "bad shape"),
         (lambda: hip.linear_chunked_dev(8, 96, 1, 1, 32, 32, 8, 8, 8, 32, 8, 16), "workspace"),
+        (lambda: hip.gqa_step_dev(built.Gqa(6, 4, 2, 16, 32, 16, 32, 128, 1e-5, 0.1, 0.9, 8, 8, 8, 8, 8), 8, 8, 8), "gqa: bad shape"),
+        (lambda: hip.gqa_any_dev(built.Gqa(4, 4, 2, 16, 32, 16, 32, 128, 1e-5, 0.1, 0.9, 8, 8, 8, 8, 8), 8, 128, True, True, 8, 0, 1, 8), "gqa_any"),
+        (lambda: hip.delta_step_dev(built.Delta(4, 2, 16, 32, 16, 48, 4, 8, 8, 8, 8, 1.0, 1e-6, 1e-5, 8, 8), 8, 8, 8, 8), "delta: bad shape"),
+        (lambda: hip.delta_chunked_dev(built.Delta(4, 2, 16, 32, 16, 32, 4, 8, 8, 8, 8, 1.0, 1e-6, 1e-5, 8, 8), 8, 8, 8, 8, 512, 9, 8, 128, 8, 64), "workspace"),
+        (lambda: hip.experts_plan_make(16, 1 << 20, 4, 8, 9, 64), "experts_plan"),
+        (lambda: hip.experts_up_dev(8, 8, 2, 1.0, 8, 8, 16, 12, 64, 0, 8, 16, 8), "experts_up"),
+        (lambda: hip.experts_out_dev(8, 8, 64, 64, None, 8, 8, 8, 16, 64, 8, 2, 16, 8), "experts_out"),
+        (lambda: hip.sum_norm_rows_dev(built.SumRows(x=8, m=1, width=8, h=8, ldh=8)), "sum_norm_rows"),
         (lambda: hip.latent_decode_dev(built.LatentAttention(1, 20, 52, 16, 64, 16, 1.0, 8, 8, 8, 64, 32, 64, 8, 8), 8, 8, 8, 0, 1, True, 8), "bad shape"),
     ]
     for call, message in bad:
@@ -139,6 +172,34 @@ def test_oracle_sink_takes_a_share():
     q = so.norm_plain(h @ t[p + "dq"].T, t[p + "dq.norm"], 1e-6) @ t[p + "uq"].T
     s = (q[0, :4] @ (t[p + "uk"] @ c[0]) + q[0, 4:] @ kr[0]) * m["scale"]
     assert np.allclose(outs[0.3], outs[-50.0] * np.exp(s) / (np.exp(s) + np.exp(0.3)))
+
+
+def test_oracle_delta_rule_by_hand():
+    """two tokens, keys alike: the second write replaces what the first one left, as far as its step size goes"""
+    k, v = np.array([[1.0, 0.0], [1.0, 0.0]]), np.array([[2.0], [6.0]])
+    o, S = so.delta_rule(k, k, v, np.array([1.0, 0.5]), np.array([1.0, 0.25]), np.zeros((2, 1)))
+    assert np.allclose(o[:, 0], [2.0, 1.0 + 0.25 * (6.0 - 1.0)]) and np.allclose(S[:, 0], [2.25, 0.0])
+
+
+def test_oracle_convolution_and_routing():
+    x = np.array([[1.0], [2.0], [3.0]])
+    assert np.allclose(so.short_convolution(x, np.array([[10.0, 1.0]]))[:, 0], [1.0, 12.0, 23.0])
+    ids, w = so.route(np.eye(3)[:1], np.array([[0.0, 0, 0], [2.0, 0, 0], [1.0, 0, 0], [2.0, 0, 0]]), 3, 2.0)
+    assert ids.tolist() == [[1, 3, 2]] and np.isclose(w.sum(), 2.0) and np.isclose(w[0, 0] / w[0, 2], math.e)
+    assert [so.query_temperature(p, {"q_temp": {"coef": 1.0, "every": 4}}) for p in (2, 3, 6, 7)] == [1.0, 1.0 + math.log(2), 1.0 + math.log(2), 1.0 + math.log(3)]
+
+
+def test_oracle_difference_of_maps():
+    """one token: both maps give its own value, whatever the scores"""
+    v = np.array([[[3.0, -4.0]]])
+    a = so.softmax_maps(np.ones((1, 2, 2, 3)), np.ones((1, 1, 2, 3)), v)
+    assert np.allclose(a, np.broadcast_to(v[0], (1, 2, 2, 2)))
+    assert np.allclose(so.difference(a, 0.25, 0.5, 0.0)[0, 0], 0.5 * v[0, 0] / math.sqrt(12.5))
+
+
+def test_oracle_loop_order():
+    c = u.mimolix([u.delta_layer()] * 4, loop=(1, 3, 2))
+    assert so.layer_runs(c) == [(0, False), (1, True), (2, False), (1, True), (2, False), (3, False)]
 
 
 def test_trace_runner_refuses_bad_use(built):

@@ -22,8 +22,20 @@ MODELS = {
                              u.lightning_layer(heads=1, dim=200, vdim=136)], width=200, vocab=64),
     "huge_heads": u.lasapel([u.latent_layer(heads=1, dim=230, rot_dim=40, vdim=270, q_rank=40, kv_rank=600), u.lightning_layer(heads=1, dim=290, vdim=48)],
                             width=88, vocab=70),
+    # layers side by side with experts, a loop around two kinds of mixer, a layer without feed-forward
+    "mimolix": u.mimolix([u.delta_layer(mlp=u.expert_mlp()), u.attention_layer(mlp=u.expert_mlp(experts=5, top=1, ff=40, scale=0.8)),
+                          u.delta_layer(heads=3, kv_heads=3, dim=40, vdim=24, conv=2), u.attention_layer(heads=2, kv_heads=1, dim=36, vdim=12, every=50, mlp=u.expert_mlp())],
+                         width=120, vocab=170, loop=(1, 3, 2)),
+    "mimolix_delta": u.mimolix([u.delta_layer(heads=6, kv_heads=1, dim=8, vdim=64, conv=1, mlp=u.expert_mlp(experts=9, top=9, ff=16, shared=0))], width=90, vocab=101, mult=1.0,
+                               embed=1.0, loop=(0, 1, 3)),
+    "mimolix_attention": u.mimolix([u.attention_layer(heads=5, kv_heads=5, dim=64, vdim=8, coef=0.0, mlp=u.expert_mlp(experts=70, top=5, ff=8, shared=72))], width=200, vocab=64,
+                                   eps=1e-3),
+    "mimolix_wide": u.mimolix([u.attention_layer(heads=20, kv_heads=1, dim=150, vdim=200, scale=0.1), u.delta_layer(heads=2, kv_heads=1, dim=130, vdim=230, conv=3),
+                               u.delta_layer(heads=2, kv_heads=2, dim=100, vdim=160, mlp=u.expert_mlp(experts=4, top=2, ff=100, shared=130))], width=136, vocab=77),
+    "mimolix_huge": u.mimolix([u.attention_layer(heads=2, kv_heads=2, dim=300, vdim=270, scale=0.05), u.attention_layer(heads=4, kv_heads=2, dim=8, vdim=300)], width=64, vocab=50),
     "many_heads": u.lasapel([u.latent_layer(heads=19, dim=16, rot_dim=8, vdim=16, q_rank=40, kv_rank=136, ff=16)], width=64, vocab=500),
 }
+SEQUENCES = ["mixed", "mimolix"]  # the models of the tests about sequences
 LIMIT = {"float32": 2e-5, "bfloat16": 6e-2}
 
 
@@ -95,19 +107,21 @@ def test_prompt_and_decoding(cases, name, dtype):
     assert error(in_portions(c.model(dtype), t, [1]), want) < LIMIT[dtype]
 
 
+@pytest.mark.parametrize("name", SEQUENCES)
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
 @pytest.mark.parametrize("sizes", [[2], [3, 1, 2], [64, 1], [63, 2, 65], [127, 2, 1, 130], [129], [40, 100, 2, 1, 1]])
-def test_portions(cases, dtype, sizes):
-    c = cases("mixed")
+def test_portions(cases, dtype, sizes, name):
+    c = cases(name)
     t = tokens_of(c.config, 290)
     want = c.oracle(t)[0]
     assert error(in_portions(c.model(dtype), t, sizes), want) < LIMIT[dtype]
 
 
+@pytest.mark.parametrize("name", SEQUENCES)
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-def test_first_tokens(cases, dtype):
+def test_first_tokens(cases, dtype, name):
     """sequences of one, two and three tokens: the sink weighs most there, states are empty"""
-    c = cases("mixed")
+    c = cases(name)
     for n in (1, 2, 3):
         t = tokens_of(c.config, n, 5)
         want = c.oracle(t)[0]
@@ -115,27 +129,32 @@ def test_first_tokens(cases, dtype):
         assert error(in_portions(c.model(dtype), t, [1]), want) < LIMIT[dtype]
 
 
+@pytest.mark.parametrize("name", SEQUENCES)
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-def test_residual_stream_after_each_layer(cases, pkg, tmp_path, dtype):
+def test_residual_stream_after_each_layer(cases, pkg, tmp_path, dtype, name):
     """the model cut after each of its layers: the stream ahead of the final norm, from the prompt and from a step"""
-    c = cases("mixed")
+    c = cases(name)
     t = tokens_of(c.config, 21)
-    after = c.oracle(t)[1]
     for k in range(1, len(c.config["layers"]) + 1):
         config = dict(c.config, layers=c.config["layers"][:k])
+        loop = config.pop("loop", None)
+        if loop and loop["start"] < k:
+            config["loop"] = dict(loop, stop=min(loop["stop"], k))
+        after = so.forward(config, c.tensors, t)[1]
         m = pkg.open_model(u.save_model(str(tmp_path / str(k)), config, c.tensors), dtype, 64)
         m.feed(t)
         m.prefill(20, with_logits=False)
-        assert u.rms_error(m.last_hidden(), after[k - 1, 19]) < LIMIT[dtype]
+        assert u.rms_error(m.last_hidden(), after[-1, 19]) < LIMIT[dtype]
         m.run(1)
-        assert u.rms_error(m.last_hidden(), after[k - 1, 20]) < LIMIT[dtype]
+        assert u.rms_error(m.last_hidden(), after[-1, 20]) < LIMIT[dtype]
         m.close()
 
 
+@pytest.mark.parametrize("name", SEQUENCES)
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-def test_long_decoding(cases, dtype):
+def test_long_decoding(cases, dtype, name):
     """300 steps behind a short prompt: several cache tiles, states carried all the way"""
-    c = cases("mixed")
+    c = cases(name)
     t = tokens_of(c.config, 310, 3)
     want = c.oracle(t)[0]
     m = c.model(dtype)
@@ -143,10 +162,11 @@ def test_long_decoding(cases, dtype):
     assert error(np.concatenate(got), want) < LIMIT[dtype]
 
 
+@pytest.mark.parametrize("name", SEQUENCES)
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-def test_requests_follow_one_another(cases, dtype):
+def test_requests_follow_one_another(cases, dtype, name):
     """a slot used again: nothing of the longer sequence before shows in the next one, and a repeat is bit for bit the same"""
-    c = cases("mixed")
+    c = cases(name)
     long, short = tokens_of(c.config, 200, 1), tokens_of(c.config, 30, 2)
     m = c.model(dtype)
     first = m.forward(short, range(30))
@@ -159,9 +179,10 @@ def test_requests_follow_one_another(cases, dtype):
     assert error(first, c.oracle(short)[0]) < LIMIT[dtype]
 
 
+@pytest.mark.parametrize("name", SEQUENCES)
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-def test_graph_replays_match_eager_steps(cases, dtype):
-    c = cases("mixed")
+def test_graph_replays_match_eager_steps(cases, dtype, name):
+    c = cases(name)
     t = tokens_of(c.config, 40, 4)
     out = []
     for use_graph in (True, False):
@@ -177,7 +198,7 @@ def test_graph_replays_match_eager_steps(cases, dtype):
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-@pytest.mark.parametrize("name", ["mixed", "lightning_only", "many_heads"])
+@pytest.mark.parametrize("name", ["mixed", "lightning_only", "many_heads", "mimolix", "mimolix_delta"])
 def test_greedy_generation(cases, name, dtype):
     """generate(): each token is the argmax of the oracle's logits over what was generated so far (or as good as it)"""
     c = cases(name)
@@ -239,6 +260,92 @@ def test_one_far_key(pkg, hip, tmp_path, dtype, far):
     m.close()
 
 
+def one_key_differential(root, far):
+    """One differential layer in which a marked token's first map scores one other marked token far above all others; the second map sees them
+    all alike."""
+    W, V, D = 32, 40, 8
+    config = u.mimolix([u.attention_layer(heads=2, kv_heads=1, dim=D, vdim=24, scale=3.0, diff=0.3, every=64)], width=W, vocab=V, eps=1e-6, embed=1.0, mult=1.0)
+    t = u.random_tensors(config, 12)
+    t["embed"] = u.rounded(np.random.default_rng(9).standard_normal((V, W)) * 0.3)
+    t["embed"][:, :3] = 0.0
+    t["embed"][1, 1] = 8.0   # the token looked for
+    t["embed"][2, 2] = 8.0   # the token that looks
+    t["l0.norm1"][:], t["l0.norm1.b"][:] = 1.0, 0.0
+    t["l0.norm1.b"][0] = 1.0  # every token
+    for k in ("q", "k"):
+        t["l0.mix." + k] *= 0.02
+        t["l0.mix." + k + ".norm"][:] = 1.0
+    for head in range(2):  # map 1 of both heads; keys of other tokens point elsewhere
+        t["l0.mix.q"][head * 2 * D, 2] = 4.0
+    t["l0.mix.k"][0, 1], t["l0.mix.k"][1, 0] = 4.0, 2.0
+    t = {k: u.rounded(v) for k, v in t.items()}
+    return config, t, u.save_model(str(root / f"diff{far}"), config, t)
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("far", [0, 1, 31, 32, 63, 64, 126, 127, 128, 129, 255, 256, 300, 398])
+def test_one_far_key_of_one_map(pkg, hip, tmp_path, dtype, far):
+    config, t, path = one_key_differential(tmp_path, far)
+    n = 400
+    base = np.random.default_rng(far).integers(3, 40, n).astype(np.int32)
+    base[-1] = 2
+    marked = base.copy()
+    marked[far] = 1
+    m = pkg.open_model(path, dtype, n + 8)
+    for tokens in (base, marked):
+        want = so.forward(config, t, tokens)[0][-1:]
+        m.reset()
+        assert error(m.forward(tokens, [n - 1]), want) < LIMIT[dtype]
+        m.reset()
+        m.forward(tokens[:-1], [])
+        assert error(m.forward(tokens[-1:], [0]), want) < LIMIT[dtype]
+    a, b = so.forward(config, t, base)[0][-1], so.forward(config, t, marked)[0][-1]
+    assert u.rms_error(a - a.mean(), b - b.mean()) > 0.2  # the key shows
+    m.close()
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_query_temperature_steps(pkg, hip, tmp_path, dtype):
+    """a temperature that changes much from step to step: the positions around every step, prompt and decoded"""
+    config = u.mimolix([u.attention_layer(heads=2, kv_heads=1, dim=16, vdim=16, coef=3.0, every=7, scale=0.4)], width=48, vocab=60)
+    t = u.random_tensors(config, 21)
+    m = pkg.open_model(u.save_model(str(tmp_path), config, t), dtype, 80)
+    tokens = tokens_of(config, 64, 11)
+    want = so.forward(config, t, tokens)[0]
+    assert error(m.forward(tokens, range(64)), want) < LIMIT[dtype]
+    m.reset()
+    assert error(in_portions(m, tokens, [6, 1, 1]), want) < LIMIT[dtype]
+    m.close()
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_slow_decay_carries_the_first_tokens(pkg, hip, tmp_path, dtype):
+    """a state that forgets next to nothing over several chunks: the first token still shows in the last logits, in a prompt and decoded"""
+    config = u.mimolix([u.delta_layer(heads=2, kv_heads=1, dim=32, vdim=16, conv=3)], width=48, vocab=60, mult=1.0)
+    t = u.random_tensors(config, 31)
+    t["l0.mix.A_log"][:], t["l0.mix.dt_bias"][:] = -8.0, -2.0
+    t["l0.mix.b"][:] = 0.0
+    t["l0.mix.b"][:, 0] = u.rounded(np.array([-3.0, -2.0]))  # step sizes well below one, except after a marked token
+    t["embed"][:, 0] = 1.0
+    t["embed"][1, 0] = -2.0
+    t = {k: u.rounded(v) for k, v in t.items()}
+    n = 200
+    m = pkg.open_model(u.save_model(str(tmp_path), config, t), dtype, n + 8)
+    base = np.random.default_rng(1).integers(2, 60, n).astype(np.int32)
+    marked = base.copy()
+    marked[0] = 1
+    rows = []
+    for tokens in (base, marked):
+        want = so.forward(config, t, tokens)[0]
+        rows.append(want[-1] - want[-1].mean())
+        m.reset()
+        assert error(m.forward(tokens, range(n)), want) < LIMIT[dtype]
+        m.reset()
+        assert error(in_portions(m, tokens, [70, 1, 2, 64, 1]), want) < LIMIT[dtype]
+    assert u.rms_error(rows[0], rows[1]) > 3 * LIMIT[dtype]
+    m.close()
+
+
 def test_errors_leave_a_usable_model(cases, pkg):
     c = cases("lightning_only")
     m = c.model("bfloat16")
@@ -263,12 +370,13 @@ def test_command_line_generates(cases, capsys):
     assert capsys.readouterr().out.strip() == ",".join(map(str, c.model("bfloat16").generate(p, 6)))
 
 
-def test_trace_runner_matches_the_library(cases, pkg, tmp_path):
+@pytest.mark.parametrize("name", SEQUENCES)
+def test_trace_runner_matches_the_library(cases, pkg, tmp_path, name):
     """the program's logits are those of the same portions through the library, bit for bit"""
     import json
     import subprocess
 
-    c = cases("mixed")
+    c = cases(name)
     prog = pkg._load_build_module().build_program("trace_run")
     a, b = tokens_of(c.config, 20, 8), tokens_of(c.config, 7, 9)
     steps = [("a", a[:12], [0, 11], []), ("a", a[12:13], [], []), ("a", a[13:], [6, 1], ["a"]), ("b", b, [6], ["b"])]
@@ -276,8 +384,8 @@ def test_trace_runner_matches_the_library(cases, pkg, tmp_path):
     p = subprocess.run([prog, "--model", c.path, "--dtype", "float32", "--out", str(tmp_path), "--max-tokens", "64"], input=text, capture_output=True, text=True, timeout=60)
     assert p.returncode == 0 and p.stdout.split("\n")[:4] == [f"done {i}" for i in range(4)], p.stderr
     m = c.model("float32")
-    for i, (name, t, w, _) in enumerate(steps):
-        if name == "b":
+    for i, (request, t, w, _) in enumerate(steps):
+        if request == "b":
             m.reset()
         want = m.forward(t, w)
         if w:
