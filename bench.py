@@ -634,22 +634,33 @@ def timed_model(model, prompt, steps: int, warmup: int, digits: int = 2) -> dict
             "decode_ms_per_token": round(ms / steps, 4), "decode_tok_s": round(steps / ms * 1e3, 1)}
 
 
+STACK_DESIGNS = {"lasapel": ("Lasapel", "write_lasapel", "lasapel_config"), "mimolix": ("Mimolix", "write_mimolix", "mimolix_config")}
+
+
 def bench_stack(args, pkg, synth):
-    """--workload lasapel: prompt and decode throughput of the Lasapel design at sizes that resemble a real model's layers, beside the
-    library's BitNet model (QK256) with the same width, feed-forward, heads, vocabulary and number of layers."""
+    """--workload lasapel | mimolix: prompt and decode throughput of a layer-stack design at sizes that resemble a real model's layers, beside the
+    library's closest other model with the same width, (active) feed-forward, heads, vocabulary and number of layer runs: BitNet (QK256) for
+    Lasapel, Lasapel for Mimolix."""
     import tempfile
 
     rows = []
     max_pos = 4096 + 64 + args.steps + args.warmup
+
+    def stack(row, design, size):
+        _, write, config = STACK_DESIGNS[design]
+        with tempfile.TemporaryDirectory() as tmp:
+            model = pkg.open_model(getattr(synth, write)(tmp, getattr(synth, config)(size, row["layers"])), "bfloat16", max_pos)
+            row[design] = [timed_model(model, synth.prompt(n, row["vocab"], 1), args.steps, args.warmup) for n in (128, 4096)]
+            row[design + "_weight_bytes"] = model.weight_bytes()
+            model.close()
+
     for size in args.sizes.split(","):
         s = synth.STACK_SIZES[size]
         row = {"size": size, "layers": args.layers or 8, **{k: s[k] for k in ("width", "ff", "heads", "vocab")}}
-        with tempfile.TemporaryDirectory() as tmp:
-            model = pkg.open_model(synth.write_lasapel(tmp, synth.lasapel_config(size, row["layers"])), "bfloat16", max_pos)
-            row["lasapel"] = [timed_model(model, synth.prompt(n, s["vocab"], 1), args.steps, args.warmup) for n in (128, 4096)]
-            row["lasapel_weight_bytes"] = model.weight_bytes()
-            model.close()
-        if not args.no_also:
+        stack(row, args.workload, size)
+        if not args.no_also and args.workload == "mimolix":
+            stack(row, "lasapel", size)
+        elif not args.no_also:
             cfg = synth.ModelConfig(hidden=s["width"], n_layers=row["layers"], n_heads=s["heads"], n_kv_heads=s["n_kv"], ffn=s["ff"], vocab=s["vocab"], max_pos=max_pos)
             dec = pkg.HostDecoder(cfg)
             layer = synth.make_layer(cfg, 0, fmt="qk256")
@@ -661,10 +672,10 @@ def bench_stack(args, pkg, synth):
             dec.close()
         rows.append(row)
         print(f"{size} done", file=sys.stderr, flush=True)
-    first = rows[0]["lasapel"][0]
-    return {"metric": "Lasapel decode tokens/s (128-token prompt)", "value": first["decode_tok_s"], "unit": "tokens/s", "n_gpus": 1, "steps": args.steps,
+    first, name = rows[0][args.workload][0], STACK_DESIGNS[args.workload][0]
+    return {"metric": f"{name} decode tokens/s (128-token prompt)", "value": first["decode_tok_s"], "unit": "tokens/s", "n_gpus": 1, "steps": args.steps,
             "warmup": args.warmup, "ms_per_step": first["decode_ms_per_token"], "higher_is_better": True, "scaling": "weak", "vs_baseline": None, "dtype": "bf16",
-            "data": "synthetic", "config": {"model": f"Lasapel {rows[0]['size']}", "layers": rows[0]["layers"], "sizes": args.sizes}, "sizes": rows}
+            "data": "synthetic", "config": {"model": f"{name} {rows[0]['size']}", "layers": rows[0]["layers"], "sizes": args.sizes}, "sizes": rows}
 
 
 def main():
@@ -672,8 +683,8 @@ def main():
     ap.add_argument("--gpus", type=int, default=1)
     ap.add_argument("--steps", type=int, default=None, help="timed steps (default 256; 512 for --workload c4: BASELINE configs[3] = 4k-token prefill + 512 decode)")
     ap.add_argument("--warmup", type=int, default=16)
-    ap.add_argument("--workload", default="c2", choices=["c2", "c3", "c4", "c5", "stream", "lasapel"])
-    ap.add_argument("--sizes", default="2b,1b,3b", help="lasapel workload: which of the model sizes (synth.STACK_SIZES)")
+    ap.add_argument("--workload", default="c2", choices=["c2", "c3", "c4", "c5", "stream", *STACK_DESIGNS])
+    ap.add_argument("--sizes", default="2b,1b,3b", help="lasapel and mimolix workloads: which of the model sizes (synth.STACK_SIZES)")
     ap.add_argument("--stream-layers", type=int, default=64, help="i2s_stream: gate|up matrices laid end to end (64 = 708 MB BitNet32-F16 / 566 MB QK256)")
     ap.add_argument("--stream-launches", type=int, default=None, help="stream workload only: a fixed number of launches and no timing (profiler counter passes)")
     ap.add_argument("--stream-format", default="i2s", choices=["i2s", "qk256"])
@@ -732,7 +743,7 @@ def main():
     hip = pkg.load()
     hip.init(local_rank)
 
-    if args.workload == "lasapel":
+    if args.workload in STACK_DESIGNS:
         line = bench_stack(args, pkg, synth)
         if rank == 0:
             print(json.dumps(line), flush=True)

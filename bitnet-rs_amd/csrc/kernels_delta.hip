@@ -90,11 +90,24 @@ __global__ __launch_bounds__(kStepThreads) void k_delta_step(Delta p, const floa
     for (int j = 0; j < NJ; ++j) s[j] = live && sl + SL * j < dimp ? st[(size_t)(sl + SL * j) * vdimp + v] : 0.f;
     const int part = tid >> 8, c = tid & 255, pos = *pos_ptr;
     const int off = part == 0 ? kv * dimp + c : part == 1 ? (kvh + kv) * dimp + c : 2 * kvh * dimp + h * vdimp + c;
+    const float gate = row[C + (size_t)h * vdimp + min(tid, vdimp - 1)], weight = p.norm[min(tid, vdimp - 1)], araw = ba[heads + h], braw = ba[h];
     float y = 0.f;
     if (part < 3 && c < (part == 2 ? vdimp : dimp)) {
         const float x = row[off];
         y = x * p.conv[(size_t)(taps - 1) * C + off];
-        for (int j = 1; j < taps && j <= pos; ++j) y += p.conv[(size_t)(taps - 1 - j) * C + off] * p.ring[(size_t)((pos - j) % taps) * C + off];
+        constexpr int AH = 4;  // earlier inputs in flight
+        for (int j0 = 1; j0 < taps; j0 += AH) {
+            float f[AH], in[AH];
+#pragma unroll
+            for (int e = 0; e < AH; ++e) {
+                const int j = min(j0 + e, taps - 1);
+                f[e] = p.conv[(size_t)(taps - 1 - j) * C + off];
+                in[e] = p.ring[(size_t)((pos - j + taps) % taps) * C + off];
+            }
+#pragma unroll
+            for (int e = 0; e < AH; ++e)
+                if (j0 + e < taps && j0 + e <= pos) y += f[e] * in[e];
+        }
         // (the slot written is none of those read: taps slots, taps - 1 earlier tokens)
         if (part == 2 || h == kv * per) p.ring[(size_t)(pos % taps) * C + off] = x;
         y = silu(y);
@@ -112,14 +125,14 @@ __global__ __launch_bounds__(kStepThreads) void k_delta_step(Delta p, const floa
     } else if (part == 2) {
         w.v[c] = y;
     }
-    const float g = expf(log_decay(p, h, ba[heads + h])), beta = 1.0f / (1.0f + expf(-ba[h]));
+    const float g = expf(log_decay(p, h, araw)), beta = 1.0f / (1.0f + expf(-braw));
     __syncthreads();
     const float o = delta_token<NJ>(w, s, dimp, vdimp, v, sl, SL, live, g, beta);
 #pragma unroll
     for (int j = 0; j < NJ; ++j)
         if (live && sl + SL * j < dimp) st[(size_t)(sl + SL * j) * vdimp + v] = s[j];
     const float inv = 1.0f / sqrtf(head_sum(o * o, w.slot) / (float)p.vdim + p.eps);
-    if (tid < vdimp) out[(size_t)h * vdimp + tid] = o * inv * p.norm[tid] * silu(row[C + (size_t)h * vdimp + tid]);
+    if (tid < vdimp) out[(size_t)h * vdimp + tid] = o * inv * weight * silu(gate);
 }
 
 template <int NJ, class T>
@@ -186,77 +199,113 @@ hipError_t launch_delta_recurrent(const Delta &d, const float *qk, const void *v
 }
 
 // ---- rows of a portion ------------------------------------------------------------------------------------------------
-// A wave: one head's slice (q, k or v) of four neighbouring tokens, two columns per lane and step.
-constexpr int kRowTokens = 16;
+// A wave: one head's slice (q, k or v) of neighbouring tokens, two columns per lane and step; the window of earlier inputs moves along in
+// registers.
+constexpr int kRowTokens = 32, kRowTaps = 4;
 
-template <class T>
-__device__ __forceinline__ float2 ld2(const T *p, size_t i);
-template <>
-__device__ __forceinline__ float2 ld2(const float *p, size_t i) {
-    return *reinterpret_cast<const float2 *>(p + i);
-}
-template <>
+__device__ __forceinline__ float2 ld2(const float *p, size_t i) { return *reinterpret_cast<const float2 *>(p + i); }
+__device__ __forceinline__ void st2(float *p, size_t i, float2 v) { *reinterpret_cast<float2 *>(p + i) = v; }
+__device__ __forceinline__ void st2(uint16_t *p, size_t i, float2 v) { *reinterpret_cast<uint32_t *>(p + i) = (uint32_t)f2bf(v.x) | (uint32_t)f2bf(v.y) << 16; }
 __device__ __forceinline__ float2 ld2(const uint16_t *p, size_t i) {
     const uint32_t v = *reinterpret_cast<const uint32_t *>(p + i);
     return make_float2(bf2f(v & 0xffffu), __builtin_bit_cast(float, v & 0xffff0000u));
 }
 
-template <class T>
+// TAPS: the convolution's taps, 0: more than kRowTaps
+template <class T, int TAPS>
 __global__ __launch_bounds__(256) void k_delta_rows(Delta p, const T *rows, size_t ld, const float *ba, size_t ldba, const int *pos_ptr, int n, float *qk, T *vo,
                                                     float *gates) {
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, y = blockIdx.y, pos0 = *pos_ptr;
-    const int heads = (int)p.heads, kvh = (int)p.kv_heads, dimp = (int)p.dimp, vdimp = (int)p.vdimp, taps = (int)p.taps, C = 2 * kvh * dimp + heads * vdimp;
+    const int heads = (int)p.heads, kvh = (int)p.kv_heads, dimp = (int)p.dimp, vdimp = (int)p.vdimp, taps = TAPS ? TAPS : (int)p.taps, C = 2 * kvh * dimp + heads * vdimp;
     const bool value = y >= 2 * kvh;
     const int width = value ? vdimp : dimp, off = value ? 2 * kvh * dimp + (y - 2 * kvh) * vdimp : y * dimp;
-    for (int i = 0; i < kRowTokens / 4; ++i) {
-        const int t = blockIdx.x * kRowTokens + wave * (kRowTokens / 4) + i;
-        if (t >= n) return;
-        float2 x[2];
-        float ss = 0.f;
+    constexpr int PER = kRowTokens / 4, NT = TAPS ? TAPS : 1;
+    const int t0 = blockIdx.x * kRowTokens + wave * PER, count = min(PER, n - t0);
+    if (count <= 0) return;
+    auto input = [&](int t, int col) {  // token t of the portion, or one ahead of it
+        if (pos0 + t < 0) return make_float2(0.f, 0.f);
+        return t >= 0 ? ld2(rows + (size_t)t * ld, col) : ld2(p.ring + (size_t)((pos0 + t) % taps) * C, col);
+    };
+    float2 x[PER][2];
 #pragma unroll
-        for (int c = 0; c < 2; ++c) {
-            const int col = off + lane * 2 + 128 * c;
-            x[c] = make_float2(0.f, 0.f);
-            if (lane * 2 + 128 * c >= width) continue;
-            for (int j = 0; j < taps && j <= pos0 + t; ++j) {
-                const float2 f = ld2(p.conv + (size_t)(taps - 1 - j) * C, col);
-                const float2 in = j <= t ? ld2(rows + (size_t)(t - j) * ld, col) : ld2(p.ring + (size_t)((pos0 + t - j) % taps) * C, col);
-                x[c].x += f.x * in.x, x[c].y += f.y * in.y;
-            }
-            x[c].x = silu(x[c].x), x[c].y = silu(x[c].y);
-            ss += x[c].x * x[c].x + x[c].y * x[c].y;
+    for (int c = 0; c < 2; ++c) {
+        const int lc = lane * 2 + 128 * c, col = off + min(lc, width - 2);
+        if (128 * c >= width) {
+#pragma unroll
+            for (int i = 0; i < PER; ++i) x[i][c] = make_float2(0.f, 0.f);
+            continue;
         }
+        if (TAPS) {
+            float2 in[PER + NT - 1], f[NT];
+#pragma unroll
+            for (int j = 0; j < NT; ++j) f[j] = ld2(p.conv + (size_t)j * C, col);
+#pragma unroll
+            for (int i = 0; i < PER; ++i) in[NT - 1 + i] = ld2(rows + (size_t)min(t0 + i, n - 1) * ld, col);
+#pragma unroll
+            for (int j = 0; j < NT - 1; ++j) in[j] = input(t0 + j - (NT - 1), col);
+#pragma unroll
+            for (int i = 0; i < PER; ++i) {
+                x[i][c] = make_float2(0.f, 0.f);
+#pragma unroll
+                for (int j = 0; j < NT; ++j) x[i][c].x += f[j].x * in[i + j].x, x[i][c].y += f[j].y * in[i + j].y;
+            }
+        } else {
+            for (int i = 0; i < count; ++i) {
+                float2 s = make_float2(0.f, 0.f);
+                for (int j = 0; j < taps; ++j) {
+                    const float2 f = ld2(p.conv + (size_t)(taps - 1 - j) * C, col), in = input(t0 + i - j, col);
+                    s.x += f.x * in.x, s.y += f.y * in.y;
+                }
+#pragma unroll
+                for (int k = 0; k < PER; ++k)
+                    if (k == i) x[k][c] = s;
+            }
+        }
+#pragma unroll
+        for (int i = 0; i < PER; ++i) {
+            const float live = lc < width ? 1.0f : 0.0f;
+            x[i][c].x = live * silu(x[i][c].x), x[i][c].y = live * silu(x[i][c].y);
+        }
+    }
+#pragma unroll
+    for (int i = 0; i < PER; ++i) {
+        if (i >= count) break;
+        const int t = t0 + i;
         if (value) {
             T *dst = vo + (size_t)t * heads * vdimp + (size_t)(y - 2 * kvh) * vdimp;
 #pragma unroll
-            for (int c = 0; c < 2; ++c) {
-                const int col = lane * 2 + 128 * c;
-                if (col < width) st_act(dst, col, x[c].x), st_act(dst, col + 1, x[c].y);
-            }
-            if (lane == 0) {
-                const int h = y - 2 * kvh;
-                gates[(size_t)t * 2 * heads + h] = log_decay(p, h, ba[(size_t)t * ldba + heads + h]);
-                gates[(size_t)t * 2 * heads + heads + h] = 1.0f / (1.0f + expf(-ba[(size_t)t * ldba + h]));
-            }
+            for (int c = 0; c < 2; ++c)
+                if (lane * 2 + 128 * c < width) st2(dst, lane * 2 + 128 * c, x[i][c]);
         } else {
-            const float inv = 1.0f / sqrtf(wave_sum(ss) + p.unit_eps) * (y < kvh ? p.q_scale : 1.0f);
+            const float ss = wave_sum((x[i][0].x * x[i][0].x + x[i][0].y * x[i][0].y) + (x[i][1].x * x[i][1].x + x[i][1].y * x[i][1].y));
+            const float inv = 1.0f / sqrtf(ss + p.unit_eps) * (y < kvh ? p.q_scale : 1.0f);
             float *dst = qk + (size_t)t * 2 * kvh * dimp + (size_t)y * dimp;
 #pragma unroll
-            for (int c = 0; c < 2; ++c) {
-                const int col = lane * 2 + 128 * c;
-                if (col < width) *reinterpret_cast<float2 *>(dst + col) = make_float2(x[c].x * inv, x[c].y * inv);
-            }
+            for (int c = 0; c < 2; ++c)
+                if (lane * 2 + 128 * c < width) st2(dst, lane * 2 + 128 * c, make_float2(x[i][c].x * inv, x[i][c].y * inv));
         }
     }
+    if (value && lane < count) {
+        const int h = y - 2 * kvh, t = t0 + lane;
+        gates[(size_t)t * 2 * heads + h] = log_decay(p, h, ba[(size_t)t * ldba + heads + h]);
+        gates[(size_t)t * 2 * heads + heads + h] = 1.0f / (1.0f + expf(-ba[(size_t)t * ldba + h]));
+    }
+}
+
+template <class T>
+static void rows_go(const Delta &d, const T *rows, size_t ld, const float *ba, size_t ldba, const int *pos, int n, float *qk, T *v, float *gates, hipStream_t s) {
+    const dim3 grid((n + kRowTokens - 1) / kRowTokens, 2 * d.kv_heads + d.heads);
+    auto fn = d.taps == 1 ? k_delta_rows<T, 1> : d.taps == 2 ? k_delta_rows<T, 2> : d.taps == 3 ? k_delta_rows<T, 3> : d.taps == kRowTaps ? k_delta_rows<T, kRowTaps>
+                                                                                                                               : k_delta_rows<T, 0>;
+    hipLaunchKernelGGL(fn, grid, dim3(256), 0, s, d, rows, ld, ba, ldba, pos, n, qk, v, gates);
 }
 
 hipError_t launch_delta_rows(const Delta &d, const void *rows, size_t ld, int rows_f32, const float *ba, size_t ldba, const int *pos, int n, float *qk,
                              void *v, float *gates, hipStream_t s) {
-    const dim3 grid((n + kRowTokens - 1) / kRowTokens, 2 * d.kv_heads + d.heads);
     if (rows_f32)
-        hipLaunchKernelGGL(k_delta_rows<float>, grid, dim3(256), 0, s, d, (const float *)rows, ld, ba, ldba, pos, n, qk, (float *)v, gates);
+        rows_go(d, (const float *)rows, ld, ba, ldba, pos, n, qk, (float *)v, gates, s);
     else
-        hipLaunchKernelGGL(k_delta_rows<uint16_t>, grid, dim3(256), 0, s, d, (const uint16_t *)rows, ld, ba, ldba, pos, n, qk, (uint16_t *)v, gates);
+        rows_go(d, (const uint16_t *)rows, ld, ba, ldba, pos, n, qk, (uint16_t *)v, gates, s);
     return hipGetLastError();
 }
 

@@ -7,45 +7,60 @@
 
 namespace bitnet_hip {
 
-// A wave chooses one token's experts: lane k < top receives the k-th one and its weight.  Lanes hold neighbouring experts, so that among equal
-// scores the lowest lane has the lowest index.
-constexpr int kPerLane = kMaxExperts / 64;
-__device__ __forceinline__ void choose(const float *z, int experts, int top, float scale, int &id, float &weight) {
-    const int lane = threadIdx.x & 63, per = (experts + 63) / 64;
-    float s[kPerLane], m = -INFINITY;
+// LT lanes choose one token's experts: lane k < top of them receives the k-th one and its weight.  A lane holds PL neighbouring experts, so that
+// among equal scores the lowest lane has the lowest index.
+template <int LT>
+__device__ __forceinline__ float token_max(float v) {
+    v = row_max(v);
+    return LT == 64 ? rows_max(v) : v;
+}
+template <int LT>
+__device__ __forceinline__ float token_sum(float v) {
+    v = row_sum(v);
+    return LT == 64 ? rows_sum(v) : v;
+}
+
+template <int LT, int PL>
+__device__ __forceinline__ void choose_load(const float *z, int experts, float (&s)[PL]) {
+    const int l = threadIdx.x & (LT - 1);
 #pragma unroll
-    for (int j = 0; j < kPerLane; ++j) {
-        const int e = lane * per + j;
-        s[j] = j < per && e < experts ? z[e] : -INFINITY;
-        m = fmaxf(m, s[j]);
-    }
-    m = rows_max(row_max(m));
-    float sum = 0.f;
+    for (int j = 0; j < PL; ++j) s[j] = l * PL + j < experts ? z[l * PL + j] : -INFINITY;
+}
+
+template <int LT, int PL>
+__device__ __forceinline__ void choose(float (&s)[PL], int experts, int top, float scale, int &id, float &weight) {
+    const int lane = threadIdx.x & 63, l = lane & (LT - 1), base = lane & ~(LT - 1);
+    float m = -INFINITY, sum = 0.f;
 #pragma unroll
-    for (int j = 0; j < kPerLane; ++j) {
+    for (int j = 0; j < PL; ++j) m = fmaxf(m, s[j]);
+    m = token_max<LT>(m);
+#pragma unroll
+    for (int j = 0; j < PL; ++j) {
         s[j] = s[j] == -INFINITY ? 0.f : expf(s[j] - m);
         sum += s[j];
     }
-    sum = wave_sum(sum);
+    sum = token_sum<LT>(sum);
 #pragma unroll
-    for (int j = 0; j < kPerLane; ++j) s[j] = j < per && lane * per + j < experts ? s[j] / sum : -1.0f;  // (-1: not there, or taken)
+    for (int j = 0; j < PL; ++j) s[j] = l * PL + j < experts ? s[j] / sum : -1.0f;  // (-1: not there, or taken)
     id = 0, weight = 0.f;
     float chosen = 0.f;
     for (int k = 0; k < top; ++k) {
         float best = -1.0f;
         int at = 0;
 #pragma unroll
-        for (int j = 0; j < kPerLane; ++j)
+        for (int j = 0; j < PL; ++j)
             if (s[j] > best) best = s[j], at = j;
-        const float w = rows_max(row_max(best));
-        const unsigned long long who = __ballot(best == w);
+        const float w = token_max<LT>(best);
+        unsigned long long who = __ballot(best == w) >> base;
+        if (LT < 64) who &= (1ull << LT) - 1;
         const int winner = who ? __builtin_ctzll(who) : 0;  // (no score compares equal to itself if a logit is not a number)
-        const int e = min(__builtin_amdgcn_readlane(lane * per + at, winner), experts - 1);
-        if (lane == k) id = e, weight = w;
+        const int mine = l * PL + at;
+        const int e = min(LT == 64 ? __builtin_amdgcn_readlane(mine, winner) : __shfl(mine, base + winner, 64), experts - 1);
+        if (l == k) id = e, weight = w;
         chosen += w;
-        if (lane == winner)
+        if (l == winner)
 #pragma unroll
-            for (int j = 0; j < kPerLane; ++j)
+            for (int j = 0; j < PL; ++j)
                 if (j == at) s[j] = -1.0f;
     }
     weight = weight / (chosen + 1e-20f) * scale;
@@ -54,24 +69,27 @@ __device__ __forceinline__ void choose(const float *z, int experts, int top, flo
 // ---- a prompt's choices -----------------------------------------------------------------------------------------------
 constexpr int kRouteTokens = 32;  // per workgroup; its choices are counted in LDS first
 
+template <int LT, int PL>
 __global__ __launch_bounds__(256) void k_route(const float *__restrict__ z, size_t ldz, float scale, ExpertsPlan p) {
     __shared__ int hist[kMaxExperts];
-    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, experts = (int)p.experts, top = (int)p.top, m = (int)p.m;
-    constexpr int PER = kRouteTokens / 4;
+    const int tid = threadIdx.x, grp = tid / LT, l = tid & (LT - 1), experts = (int)p.experts, top = (int)p.top, m = (int)p.m;
+    constexpr int PER = kRouteTokens * LT / 256;  // (top <= LT)
+    const int t0 = blockIdx.x * kRouteTokens + grp * PER;
+    float s[PER][PL];
+#pragma unroll
+    for (int i = 0; i < PER; ++i) choose_load<LT, PL>(z + (size_t)min(t0 + i, m - 1) * ldz, experts, s[i]);
     for (int e = tid; e < experts; e += 256) hist[e] = 0;
     __syncthreads();
     int id[PER], rank[PER];
 #pragma unroll
     for (int i = 0; i < PER; ++i) {
-        const int t = blockIdx.x * kRouteTokens + wave * PER + i;
-        id[i] = rank[i] = 0;
-        if (t >= m) continue;
         float w;
-        choose(z + (size_t)t * ldz, experts, top, scale, id[i], w);
-        if (lane < top) {
+        choose<LT, PL>(s[i], experts, top, scale, id[i], w);
+        rank[i] = 0;
+        if (t0 + i < m && l < top) {
             rank[i] = atomicAdd(&hist[id[i]], 1);
-            p.ids[(size_t)t * top + lane] = id[i];
-            p.weights[(size_t)t * top + lane] = w;
+            p.ids[(size_t)(t0 + i) * top + l] = id[i];
+            p.weights[(size_t)(t0 + i) * top + l] = w;
         }
     }
     __syncthreads();
@@ -81,10 +99,8 @@ __global__ __launch_bounds__(256) void k_route(const float *__restrict__ z, size
     }
     __syncthreads();
 #pragma unroll
-    for (int i = 0; i < PER; ++i) {
-        const int t = blockIdx.x * kRouteTokens + wave * PER + i;
-        if (t < m && lane < top) p.slots[(size_t)t * top + lane] = rank[i] + hist[id[i]];  // within its expert so far
-    }
+    for (int i = 0; i < PER; ++i)
+        if (t0 + i < m && l < top) p.slots[(size_t)(t0 + i) * top + l] = rank[i] + hist[id[i]];  // within its expert so far
 }
 
 // first slot and tiles of every expert; the counts are left at zero for the next portion
@@ -119,7 +135,10 @@ __global__ __launch_bounds__(256) void k_route_slots(ExpertsPlan p) {
 }
 
 hipError_t launch_experts_route(const float *logits, size_t ldz, float scale, const ExpertsPlan &p, hipStream_t s) {
-    hipLaunchKernelGGL(k_route, dim3((p.m + kRouteTokens - 1) / kRouteTokens), dim3(256), 0, s, logits, ldz, scale, p);
+    const bool row = p.top <= 16;  // sixteen lanes per token
+    const int e = (int)p.experts;
+    auto fn = row && e <= 16 ? k_route<16, 1> : row && e <= 64 ? k_route<16, 4> : row && e <= 128 ? k_route<16, 8> : e <= 256 ? k_route<64, 4> : k_route<64, 16>;
+    hipLaunchKernelGGL(fn, dim3((p.m + kRouteTokens - 1) / kRouteTokens), dim3(256), 0, s, logits, ldz, scale, p);
     hipLaunchKernelGGL(k_route_tiles, dim3(1), dim3(1024), 0, s, p);
     hipLaunchKernelGGL(k_route_slots, dim3((p.m * p.top + 255) / 256), dim3(256), 0, s, p);
     return hipGetLastError();
@@ -128,9 +147,7 @@ hipError_t launch_experts_route(const float *logits, size_t ldz, float scale, co
 // ---- one token --------------------------------------------------------------------------------------------------------
 // Both products in the manner of k_dense_gemv: LPR lanes per row, 16 bytes of weights per lane and chunk of LPR * 8 columns, R rows x U chunks in
 // flight, the input vector in LDS with every segment padded to whole chunks.
-__device__ __forceinline__ void stage(const float *x, int cols, int padded, float *dst) {
-    for (int i = threadIdx.x; i < padded; i += 256) dst[i] = i < cols ? x[i] : 0.f;
-}
+constexpr int kStage = 4;  // sixteen-byte loads in flight per thread while the vector is staged (rows and segments start on 16 bytes)
 
 template <int R>
 __device__ __forceinline__ void multiply8(const u32x4 (&w)[R], const float *x, float (&acc)[R]) {
@@ -150,7 +167,13 @@ __device__ __forceinline__ void multiply8(const u32x4 (&w)[R], const float *x, f
 template <int LPR>
 __device__ __forceinline__ float lanes_sum(float v) {
     v = row_sum(v);
-    return LPR == 64 ? rows_sum(v) : v;
+    if (LPR == 64) return rows_sum(v);
+    if (LPR == 32) {
+        float w = v;
+        swap_rows16(v, w);
+        v += w;
+    }
+    return v;
 }
 
 struct UpK {
@@ -158,16 +181,30 @@ struct UpK {
     int kp, groups;
 };
 
-template <int LPR, int R, int U>
+template <int LPR, int R, int U, int PL>
 __global__ __launch_bounds__(256) void k_experts_up(UpK p) {
     extern __shared__ __attribute__((aligned(16))) float xs[];
     const ExpertsUp &a = p.a;
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, b = blockIdx.y, sub = lane / LPR, l = lane % LPR;
     constexpr int G = 64 / LPR, CH = LPR * 8;
-    stage(a.x, a.cols, p.kp, xs);
+    float z[PL];
+    choose_load<64, PL>(a.logits, a.experts, z);
+    f32x4 xv[kStage];
+    auto load = [&](int i0) {
+#pragma unroll
+        for (int j = 0; j < kStage; ++j) xv[j] = reinterpret_cast<const f32x4 *>(a.x)[min(i0 + 256 * j, a.cols / 4 - 1)];
+    };
+    auto store = [&](int i0) {
+#pragma unroll
+        for (int j = 0; j < kStage; ++j) {
+            const int i = i0 + 256 * j;
+            if (i < p.kp / 4) reinterpret_cast<f32x4 *>(xs)[i] = i < a.cols / 4 ? xv[j] : f32x4{0.f, 0.f, 0.f, 0.f};
+        }
+    };
+    load(tid);
     int mine;
     float weight;
-    choose(a.logits, a.experts, a.top, a.scale, mine, weight);
+    choose<64, PL>(z, a.experts, a.top, a.scale, mine, weight);
     if (blockIdx.x == 0 && b == 0 && wave == 0 && lane < a.top) a.ids[lane] = mine;
     const int e = __builtin_amdgcn_readlane(mine, b);
     const float scale = __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, weight), b));
@@ -184,6 +221,11 @@ __global__ __launch_bounds__(256) void k_experts_up(UpK p) {
     };
     int g = blockIdx.x * 4 + wave;
     if (g < p.groups) fetch(g, 0);
+    store(tid);
+    for (int i0 = tid + 256 * kStage; i0 < p.kp / 4; i0 += 256 * kStage) {
+        load(i0);
+        store(i0);
+    }
     __syncthreads();
     const int n_wg = gridDim.x;
     for (; g < p.groups; g += n_wg * 4) {
@@ -242,9 +284,22 @@ __global__ __launch_bounds__(256) void k_experts_out(OutK p) {
     };
     int g = blockIdx.x * 4 + wave;
     if (g < p.groups) fetch(g, 0);
-    stage(a.x0, a.cols0, p.c0 * CH, xs);
-    for (int k = 0; k < a.top; ++k) stage(a.x1 + (size_t)k * a.ldx1, a.cols1, p.ce * CH, xs + (p.c0 + k * p.ce) * CH);
-    for (int i = (p.c0 + a.top * p.ce) * CH + tid; i < p.chunks * CH; i += 256) xs[i] = 0.f;
+    const int total = p.chunks * CH / 4;
+    for (int i0 = tid; i0 < total; i0 += 256 * kStage) {
+        f32x4 v[kStage];
+        bool in[kStage];
+#pragma unroll
+        for (int j = 0; j < kStage; ++j) {
+            const int i = i0 + 256 * j, c = i / (CH / 4), x = max(c - p.c0, 0), q = min((int)((unsigned)x * p.magic >> 20), a.top - 1);
+            const bool first = c < p.c0;
+            const int col = (first ? i : i - (p.c0 + q * p.ce) * (CH / 4)) * 4, cols = first ? a.cols0 : a.cols1;
+            in[j] = col < cols;
+            v[j] = *reinterpret_cast<const f32x4 *>((first ? a.x0 : a.x1 + (size_t)q * a.ldx1) + min(col, cols - 4));
+        }
+#pragma unroll
+        for (int j = 0; j < kStage; ++j)
+            if (i0 + 256 * j < total) reinterpret_cast<f32x4 *>(xs)[i0 + 256 * j] = in[j] ? v[j] : f32x4{0.f, 0.f, 0.f, 0.f};
+    }
     __syncthreads();
     const int n_wg = gridDim.x;
     for (; g < p.groups; g += n_wg * 4) {
@@ -292,7 +347,11 @@ static hipError_t up_go(const ExpertsUp &a, int chunks, hipStream_t s) {
     k.kp = (chunks + u - 1) / u * u * LPR * 8;
     k.groups = (a.rows + 64 / LPR * R - 1) / (64 / LPR * R);
     if ((size_t)k.kp * 4 > 150 * 1024) return hipErrorInvalidValue;
-    auto fn = u == 1 ? k_experts_up<LPR, R, 1> : u == 2 ? k_experts_up<LPR, R, 2> : u == 3 ? k_experts_up<LPR, R, 3> : k_experts_up<LPR, R, 5>;
+    auto pick = [&](auto f64, auto f256, auto f1024) { return a.experts <= 64 ? f64 : a.experts <= 256 ? f256 : f1024; };
+    auto fn = u == 1   ? pick(k_experts_up<LPR, R, 1, 1>, k_experts_up<LPR, R, 1, 4>, k_experts_up<LPR, R, 1, 16>)
+              : u == 2 ? pick(k_experts_up<LPR, R, 2, 1>, k_experts_up<LPR, R, 2, 4>, k_experts_up<LPR, R, 2, 16>)
+              : u == 3 ? pick(k_experts_up<LPR, R, 3, 1>, k_experts_up<LPR, R, 3, 4>, k_experts_up<LPR, R, 3, 16>)
+                       : pick(k_experts_up<LPR, R, 5, 1>, k_experts_up<LPR, R, 5, 4>, k_experts_up<LPR, R, 5, 16>);
     const size_t lds = (size_t)k.kp * 4;
     if (lds > 65536) {
         const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(fn), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
@@ -332,8 +391,8 @@ static hipError_t out_go(const ExpertsOut &a, hipStream_t s) {
 
 hipError_t launch_experts_out(const ExpertsOut &a, hipStream_t s) {
     auto waste = [&](int ch) { return (double)((a.cols0 + ch - 1) / ch * ch + (long)a.top * ((a.cols1 + ch - 1) / ch * ch)) / (a.cols0 + (double)a.top * a.cols1); };
-    // whole-wave rows unless their chunks are mostly padding
-    return waste(512) > 1.6 * waste(128) ? out_go<16, 1>(a, s) : out_go<64, 1>(a, s);
+    // the longest rows of lanes whose chunks are not padding for the most part
+    return waste(512) <= 1.1 * waste(256) ? out_go<64, 1>(a, s) : waste(256) <= 1.3 * waste(128) ? out_go<32, 1>(a, s) : out_go<16, 1>(a, s);
 }
 
 }  // namespace bitnet_hip

@@ -171,7 +171,22 @@ __global__ __launch_bounds__(256, NV > 8 ? 1 : 2) void k_gqa_step(Gqa p, GqaStep
     const int k0 = blockIdx.x * per * kGqaTile, k1 = min(k0 + per * kGqaTile, n_keys);
     uint16_t *K = (uint16_t *)p.kcache + (size_t)kv * MAPS * p.capacity * dimp, *V = (uint16_t *)p.vcache + (size_t)kv * vdimp * p.capacity;
     const float *kraw = a.row + (p.heads * MAPS + (size_t)kv * MAPS) * dimp, *vraw = a.row + (p.heads + p.kv_heads) * MAPS * dimp + (size_t)kv * vdimp;
-    if (k1 == n_keys) {  // the record that holds the new position appends it
+    u32x4 kf[2][MAPS][NK], vf[NV];
+    auto fetch = [&](int kb) {  // (blocks lie below the capacity, a multiple of 128)
+#pragma unroll
+        for (int t = 0; t < 2; ++t)
+#pragma unroll
+            for (int j = 0; j < MAPS; ++j)
+#pragma unroll
+                for (int kk = 0; kk < NK; ++kk)
+                    kf[t][j][kk] = *reinterpret_cast<const u32x4 *>(K + ((size_t)j * p.capacity + kb + (r16 >> 2) * 8 + t * 4 + (r16 & 3)) * dimp + min(kk * 32, dimp - 32) + g * 8);
+#pragma unroll
+        for (int v = 0; v < NV; ++v) vf[v] = *reinterpret_cast<const u32x4 *>(V + (size_t)min(v * 16 + r16, vdimp - 1) * p.capacity + kb + g * 8);
+    };
+    constexpr bool kAhead = NK <= 4;  // the first block is requested ahead of the norms (registers allow it)
+    const bool owner = k1 == n_keys;
+    if (kAhead && !owner) fetch(k0 + wave * 32);
+    if (owner) {  // the record that holds the new position appends it
         if (wave < MAPS) {
             float v[NK], ss = 0.f;
 #pragma unroll
@@ -225,17 +240,8 @@ __global__ __launch_bounds__(256, NV > 8 ? 1 : 2) void k_gqa_step(Gqa p, GqaStep
 #pragma unroll
         for (int v = 0; v < NV; ++v) o[v][j] = f32x4{0.f, 0.f, 0.f, 0.f};
     }
-    for (int kb = k0 + wave * 32; kb < k1; kb += 128) {  // (blocks lie below the capacity, a multiple of 128)
-        u32x4 kf[2][MAPS][NK], vf[NV];
-#pragma unroll
-        for (int t = 0; t < 2; ++t)
-#pragma unroll
-            for (int j = 0; j < MAPS; ++j)
-#pragma unroll
-                for (int kk = 0; kk < NK; ++kk)
-                    kf[t][j][kk] = *reinterpret_cast<const u32x4 *>(K + ((size_t)j * p.capacity + kb + (r16 >> 2) * 8 + t * 4 + (r16 & 3)) * dimp + min(kk * 32, dimp - 32) + g * 8);
-#pragma unroll
-        for (int v = 0; v < NV; ++v) vf[v] = *reinterpret_cast<const u32x4 *>(V + (size_t)min(v * 16 + r16, vdimp - 1) * p.capacity + kb + g * 8);
+    for (int kb = k0 + wave * 32; kb < k1; kb += 128) {
+        if (!kAhead || owner || kb >= k0 + 128) fetch(kb);
 #pragma unroll
         for (int j = 0; j < MAPS; ++j) {
             f32x4 s[2];

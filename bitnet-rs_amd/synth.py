@@ -135,9 +135,49 @@ def lasapel_config(size: str, n_layers: int) -> dict:
     return {"architecture": "Lasapel", "vocab": s["vocab"], "width": s["width"], "norm": {"eps": 1e-6}, "layers": layers}
 
 
+MIMOLIX_EXPERTS = {"1b": (448, 512), "2b": (768, 768), "3b": (896, 1024)}  # columns of one of 64 experts, of the shared one: 8 and 1 make up the size's ff
+
+
+def mimolix_config(size: str, runs: int) -> dict:
+    """delta rule (heads of 128 / 128, two on one q / k head) and differential attention (heads of 2 x 64 / 128, kv heads of the size) in turn,
+    64 experts of which a token takes 8, one shared; `runs` layer runs, four of them two layers run twice."""
+    s = STACK_SIZES[size]
+    ff, shared = MIMOLIX_EXPERTS[size]
+    mlp = {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": 64, "scale": 2.5, "top": 8}, "shared": {"ff": shared}}
+    delta = {"type": "delta", "mixer": {"heads": s["heads"], "kv_heads": s["heads"] // 2, "dim": 128, "vdim": 128, "conv": 4}, "mlp": mlp}
+    attention = {"type": "attention", "mixer": {"heads": s["heads"], "kv_heads": s["n_kv"], "dim": 64, "vdim": 128, "scale": 0.125, "diff": 0.5,
+                                                "q_temp": {"coef": 0.1, "every": 2048}}, "mlp": mlp}
+    return {"architecture": "Mimolix", "vocab": s["vocab"], "width": s["width"], "norm": {"eps": 1e-6}, "residual_mult": 0.5, "embedding": {"scale": 4.0},
+            "loop": {"start": 0, "stop": 2, "times": 2}, "layers": [delta, attention] * ((runs - 2) // 2)}
+
+
+def mimolix_shapes(config: dict) -> dict:
+    W = config["width"]
+    shapes = {"embed": (config["vocab"], W), "head": (config["vocab"], W), "final.norm": (W,), "final.norm.b": (W,), "loop.in": (W, 2 * W)}
+    for i, layer in enumerate(config["layers"]):
+        p, m, f = f"l{i}.", layer["mixer"], layer["mlp"]
+        q, H, G, D, V = p + "mix.", m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+        shapes.update({p + "norm1": (W,), p + "norm1.b": (W,), q + "o": (W, H * V)})
+        if layer["type"] == "attention":
+            shapes.update({q + "q": (H * 2 * D, W), q + "k": (G * 2 * D, W), q + "v": (G * V, W)})
+            shapes.update({q + n: (D,) for n in ("q.norm", "k.norm", "lq1", "lk1", "lq2", "lk2")})
+        else:
+            for n, c in (("q", G * D), ("k", G * D), ("v", H * V)):
+                shapes.update({q + n: (c, W), q + n + ".conv": (c, m["conv"])})
+            shapes.update({q + "b": (H, W), q + "a": (H, W), q + "g": (H * V, W), q + "A_log": (H,), q + "dt_bias": (H,), q + "norm": (V,)})
+        for e in [f"e{k}" for k in range(f["router"]["experts"])] + ["shared"]:
+            ff = (f["shared"] if e == "shared" else f["expert"])["ff"]
+            shapes.update({f"{p}mlp.{e}.up": (ff, W), f"{p}mlp.{e}.down": (W, ff)})
+        shapes[p + "mlp.router"] = (f["router"]["experts"], W)
+    return shapes
+
+
+def write_mimolix(folder: str, config: dict, seed: int = 42) -> str:
+    ones = ("norm1", "q.norm", "k.norm", "mix.norm", "final.norm")
+    return write_random(folder, config, mimolix_shapes(config), seed, lambda name: 1.0 if name.endswith(ones) else -1.0 if name.endswith(("A_log", "dt_bias")) else 0.0)
+
+
 def write_lasapel(folder: str, config: dict, seed: int = 42) -> str:
-    """config.json + model.safetensors with random bf16 weights (slices of one random block, scaled per tensor)."""
-    block = _stream(seed, 7).standard_normal(1 << 22, dtype=np.float32)
     shapes = {"embed": (config["vocab"], config["width"]), "head": (config["vocab"], config["width"]), "final.norm": (config["width"],)}
     W = config["width"]
     for i, layer in enumerate(config["layers"]):
@@ -154,6 +194,14 @@ def write_lasapel(folder: str, config: dict, seed: int = 42) -> str:
             shapes.update({q + "norm": (H * m["vdim"],), q + "o": (W, H * m["vdim"])})
         f = layer["mlp"]["ff"]
         shapes.update({p + "mlp.up": (f, W), p + "mlp.up.b": (f,), p + "mlp.down": (W, f), p + "mlp.down.b": (W,)})
+    return write_random(folder, config, shapes, seed,
+                        lambda name: 1.0 if name.endswith("q.norm") or name.endswith("v.norm") or name.endswith("mix.norm") else 0.5 if ".ls" in name else 0.0)
+
+
+def write_random(folder: str, config: dict, shapes: dict, seed: int, centre) -> str:
+    """config.json + model.safetensors with random bf16 weights: slices of one random block, matrices scaled to unit gain, vectors around
+    centre(name)."""
+    block = _stream(seed, 7).standard_normal(1 << 22, dtype=np.float32)
     os.makedirs(folder, exist_ok=True)
     with open(os.path.join(folder, "config.json"), "w") as fh:
         json.dump(config, fh)
@@ -165,15 +213,13 @@ def write_lasapel(folder: str, config: dict, seed: int = 42) -> str:
     h = json.dumps(head).encode()
     with open(os.path.join(folder, "model.safetensors"), "wb") as fh:
         fh.write(struct.pack("<Q", len(h)) + h)
+        made = {}
         for k, (name, shape) in enumerate(shapes.items()):
             n = int(np.prod(shape))
-            if len(shape) == 2:
-                gain, centre = (1.0 if name == "embed" else 1.0 / np.sqrt(shape[1])), 0.0
-            else:
-                gain, centre = 0.1, (1.0 if name.endswith("q.norm") or name.endswith("v.norm") or name.endswith("mix.norm") else 0.5 if ".ls" in name else 0.0)
-            bits = ((block * np.float32(gain) + np.float32(centre)).view(np.uint32) >> 16).astype(np.uint16)
-            start = (k * 9973) % block.size
-            bits = np.roll(bits, -start)
+            gain, mid = ((1.0 if name == "embed" else 1.0 / np.sqrt(shape[1])), 0.0) if len(shape) == 2 else (0.1, centre(name))
+            if (gain, mid) not in made:
+                made[gain, mid] = np.tile(((block * np.float32(gain) + np.float32(mid)).view(np.uint32) >> 16).astype(np.uint16), 2)
+            bits, start = made[gain, mid], (k * 9973) % block.size
             for a in range(0, n, block.size):
-                fh.write(bits[: min(block.size, n - a)].tobytes())
+                fh.write(bits[start: start + min(block.size, n - a)].data)
     return folder
