@@ -9,8 +9,8 @@
 //   (I + L) U = diag(beta) V - diag(beta e^G) K S0,
 // so with T = (I + L)^-1:  U = T diag(beta) V - (T diag(beta e^G) K) S0,  S' = e^G_end S0 + sum_j e^(G_end - G_j) k_j u_j^T,
 //   o_i = e^G_i S0^T q_i + sum_{j <= i} e^(G_i - G_j) (k_j.q_i) u_j.
-// k_delta_chunk forms T and the products with it for all chunks at once, k_delta_scan walks the chunks (one wave per 16 value columns, operands
-// straight from memory in the order the matrix cores want them), k_delta_out forms the outputs of all chunks.
+// k_delta_chunk forms T and the products with it for all chunks at once, k_delta_scan walks the chunks (one workgroup per 16 value columns,
+// operands straight from memory in the order the matrix cores want them), k_delta_out forms the outputs of all chunks.
 // f32 operands enter the matrix cores as (high, low) pairs of bf16 values; L and T are f32 throughout.
 #include "dense.hpp"
 
@@ -484,91 +484,121 @@ __global__ __launch_bounds__(256, 2) void k_delta_chunk(Delta p, const float *qk
     }
 }
 
-// one wave: one head, 16 value columns; the next chunk's operands are requested half a step ahead of their use
+// One workgroup: one head, 16 value columns.  Wave w takes token tile w of U and key tiles 2 w, 2 w + 1 of the state; state and U meet in LDS as
+// fragments, twice per chunk.  Operands come straight from memory, requested two chunks ahead.
 template <int NK>
-__global__ __launch_bounds__(64, 1) void k_delta_scan(Delta p, DeltaWs w) {
-    const int lane = threadIdx.x, r16 = lane & 15, g = lane >> 4;
+__global__ __launch_bounds__(256, 1) void k_delta_scan(Delta p, DeltaWs w) {
+    __shared__ u32x4 ss[NK][2][64], su[2][2][64];
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), r16 = lane & 15, g = lane >> 4;
     // consecutive workgroups go to the eight XCDs in turn: a head's value tiles stay on one of them, whose L2 then holds its operands
     const int x = blockIdx.x & 7, rest = blockIdx.x >> 3, h = (rest / w.nv) * 8 + x, vt = rest % w.nv;
     if (h >= (int)p.heads) return;
-    const int vdimp = (int)p.vdimp;
+    // (waves past the state's tiles repeat the last ones, stores included: no store stands behind a branch, which would keep hipcc from counting
+    // the loads in flight)
+    const int vdimp = (int)p.vdimp, kt = min(wave, NK - 1);
     float *st = p.state + (size_t)h * p.dimp * vdimp + vt * 16 + r16;
-    f32x4 s[2 * NK];
+    f32x4 s[2];
 #pragma unroll
-    for (int dt = 0; dt < 2 * NK; ++dt)
+    for (int d = 0; d < 2; ++d)
 #pragma unroll
-        for (int e = 0; e < 4; ++e) s[dt][e] = st[(size_t)(dt * 16 + g * 4 + e) * vdimp];
-    u32x4 wf[4][NK][2], kf[2 * NK][2][2];
-    f32x4 u[4], un[4];
-    float ge, gn;
-    auto fetch_w = [&](int c) {
-        const size_t ch = (size_t)h * w.nc + c;
+        for (int e = 0; e < 4; ++e) s[d][e] = st[(size_t)((2 * kt + d) * 16 + g * 4 + e) * vdimp];
+    u32x4 wf[2][NK][2], kf[2][2][2][2];
+    f32x4 ut[2];
+    float ge[2];
+    auto fetch_w = [&](int b, int c) {
+        const size_t ch = (size_t)h * w.nc + min(c, w.nc - 1);
 #pragma unroll
-        for (int it = 0; it < 4; ++it) {
+        for (int kk = 0; kk < NK; ++kk)
 #pragma unroll
-            for (int kk = 0; kk < NK; ++kk)
-#pragma unroll
-                for (int e = 0; e < 2; ++e) wf[it][kk][e] = w.w[(((ch * 4 + it) * NK + kk) * 2 + e) * 64 + lane];
-            un[it] = w.ut[((ch * w.nv + vt) * 4 + it) * 64 + lane];
-        }
-        gn = w.g[ch * 64 + 63];
+            for (int e = 0; e < 2; ++e) wf[b][kk][e] = w.w[(((ch * 4 + wave) * NK + kk) * 2 + e) * 64 + lane];
+        ut[b] = w.ut[((ch * w.nv + vt) * 4 + wave) * 64 + lane];
     };
-    fetch_w(0);
-    for (int c = 0; c < w.nc; ++c) {
-        const size_t ch = (size_t)h * w.nc + c;
+    auto fetch_k = [&](int b, int c) {
+        const size_t ch = (size_t)h * w.nc + min(c, w.nc - 1);
 #pragma unroll
-        for (int dt = 0; dt < 2 * NK; ++dt)
+        for (int d = 0; d < 2; ++d)
 #pragma unroll
             for (int k2 = 0; k2 < 2; ++k2)
 #pragma unroll
-                for (int e = 0; e < 2; ++e) kf[dt][k2][e] = w.k[(((ch * 2 * NK + dt) * 2 + k2) * 2 + e) * 64 + lane];
+                for (int e = 0; e < 2; ++e) kf[b][d][k2][e] = w.k[(((ch * 2 * NK + 2 * kt + d) * 2 + k2) * 2 + e) * 64 + lane];
+        ge[b] = w.g[ch * 64 + 63];
+    };
+    auto chunk = [&](int b, int c) {
+        const size_t ch = (size_t)h * w.nc + c;
+        {
+            const SplitFrag f = split8(s[0], s[1]);
+            ss[kt][0][lane] = __builtin_bit_cast(u32x4, f.hi);
+            ss[kt][1][lane] = __builtin_bit_cast(u32x4, f.lo);
+            u32x4 *dst = w.s + (((ch * w.nv + vt) * NK + kt) * 2) * 64 + lane;
+            dst[0] = __builtin_bit_cast(u32x4, f.hi);
+            dst[64] = __builtin_bit_cast(u32x4, f.lo);
+        }
+        __syncthreads();
+        f32x4 a[3] = {ut[b], f32x4{0.f, 0.f, 0.f, 0.f}, f32x4{0.f, 0.f, 0.f, 0.f}};
+        u32x4 sf[NK][2];
 #pragma unroll
-        for (int it = 0; it < 4; ++it) u[it] = un[it];
-        ge = expf(gn);
+        for (int kk = 0; kk < NK; ++kk) sf[kk][0] = ss[kk][0][lane], sf[kk][1] = ss[kk][1][lane];
         __builtin_amdgcn_sched_barrier(0);
 #pragma unroll
         for (int kk = 0; kk < NK; ++kk) {
-            const SplitFrag b = split8(s[2 * kk], s[2 * kk + 1]);
-            u32x4 *dst = w.s + (((ch * w.nv + vt) * NK + kk) * 2) * 64;
-            dst[lane] = __builtin_bit_cast(u32x4, b.hi);
-            dst[64 + lane] = __builtin_bit_cast(u32x4, b.lo);
-#pragma unroll
-            for (int it = 0; it < 4; ++it) u[it] = mfma_bf16(__builtin_bit_cast(bf16x8, wf[it][kk][0]), b.hi, u[it]);
-#pragma unroll
-            for (int it = 0; it < 4; ++it) u[it] = mfma_bf16(__builtin_bit_cast(bf16x8, wf[it][kk][0]), b.lo, u[it]);
-#pragma unroll
-            for (int it = 0; it < 4; ++it) u[it] = mfma_bf16(__builtin_bit_cast(bf16x8, wf[it][kk][1]), b.hi, u[it]);
+            const bf16x8 hi = __builtin_bit_cast(bf16x8, sf[kk][0]), lo = __builtin_bit_cast(bf16x8, sf[kk][1]);
+            a[0] = mfma_bf16(__builtin_bit_cast(bf16x8, wf[b][kk][0]), hi, a[0]);
+            a[1] = mfma_bf16(__builtin_bit_cast(bf16x8, wf[b][kk][0]), lo, a[1]);
+            a[2] = mfma_bf16(__builtin_bit_cast(bf16x8, wf[b][kk][1]), hi, a[2]);
+        }
+        const f32x4 u = a[0] + (a[1] + a[2]);
+        {
+            uint32_t h0, l0, h1, l1;
+            split2(u.x, u.y, h0, l0);
+            split2(u.z, u.w, h1, l1);
+            reinterpret_cast<u32x2 *>(&su[wave >> 1][0][lane])[wave & 1] = u32x2{h0, h1};
+            reinterpret_cast<u32x2 *>(&su[wave >> 1][1][lane])[wave & 1] = u32x2{l0, l1};
         }
         __builtin_amdgcn_sched_barrier(0);
-        if (c + 1 < w.nc) fetch_w(c + 1);
+        fetch_w(b, c + 2);
+        __syncthreads();
+        const u32x4 uf[2][2] = {{su[0][0][lane], su[0][1][lane]}, {su[1][0][lane], su[1][1][lane]}};
+        w.u[(((ch * w.nv + vt) * 2 + (wave >> 1)) * 2 + (wave & 1)) * 64 + lane] = su[wave >> 1][wave & 1][lane];
         __builtin_amdgcn_sched_barrier(0);
+        const float end = expf(ge[b]);
+        f32x4 d0[2], d1[2];
 #pragma unroll
-        for (int dt = 0; dt < 2 * NK; ++dt) s[dt] *= ge;
+        for (int d = 0; d < 2; ++d) d0[d] = s[d] * end, d1[d] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
         for (int k2 = 0; k2 < 2; ++k2) {
-            const SplitFrag b = split8(u[2 * k2], u[2 * k2 + 1]);
-            u32x4 *dst = w.u + (((ch * w.nv + vt) * 2 + k2) * 2) * 64;
-            dst[lane] = __builtin_bit_cast(u32x4, b.hi);
-            dst[64 + lane] = __builtin_bit_cast(u32x4, b.lo);
+            const bf16x8 hi = __builtin_bit_cast(bf16x8, uf[k2][0]), lo = __builtin_bit_cast(bf16x8, uf[k2][1]);
 #pragma unroll
-            for (int dt = 0; dt < 2 * NK; ++dt) s[dt] = mfma_bf16(__builtin_bit_cast(bf16x8, kf[dt][k2][0]), b.hi, s[dt]);
+            for (int d = 0; d < 2; ++d) {
+                d0[d] = mfma_bf16(__builtin_bit_cast(bf16x8, kf[b][d][k2][0]), hi, d0[d]);
+                d1[d] = mfma_bf16(__builtin_bit_cast(bf16x8, kf[b][d][k2][0]), lo, d1[d]);
+            }
 #pragma unroll
-            for (int dt = 0; dt < 2 * NK; ++dt) s[dt] = mfma_bf16(__builtin_bit_cast(bf16x8, kf[dt][k2][0]), b.lo, s[dt]);
-#pragma unroll
-            for (int dt = 0; dt < 2 * NK; ++dt) s[dt] = mfma_bf16(__builtin_bit_cast(bf16x8, kf[dt][k2][1]), b.hi, s[dt]);
+            for (int d = 0; d < 2; ++d) d1[d] = mfma_bf16(__builtin_bit_cast(bf16x8, kf[b][d][k2][1]), hi, d1[d]);
         }
+#pragma unroll
+        for (int d = 0; d < 2; ++d) s[d] = d0[d] + d1[d];
+        __builtin_amdgcn_sched_barrier(0);
+        fetch_k(b, c + 2);
+    };
+    fetch_w(0, 0), fetch_k(0, 0), fetch_w(1, 1), fetch_k(1, 1);
+    int c = 0;
+    for (; c + 1 < w.nc; c += 2) {
+        chunk(0, c);
+        chunk(1, c + 1);
     }
+    if (c < w.nc) chunk(0, c);
 #pragma unroll
-    for (int dt = 0; dt < 2 * NK; ++dt)
+    for (int d = 0; d < 2; ++d)
 #pragma unroll
-        for (int e = 0; e < 4; ++e) st[(size_t)(dt * 16 + g * 4 + e) * vdimp] = s[dt][e];
+        for (int e = 0; e < 4; ++e) st[(size_t)((2 * kt + d) * 16 + g * 4 + e) * vdimp] = s[d][e];
 }
 
-// outputs of a chunk and head: wave = token tile; O^T = S^T Q^T and U^T P^T, then norm and gate
+// Outputs of a chunk and head, two waves of two token tiles each (the first and the last, the two between): O^T = S^T Q^T and U^T P^T, then norm
+// and gate.  A value tile's operands are requested one tile ahead.
 template <int NK, int NV>
-__global__ __launch_bounds__(256, 2) void k_delta_out(Delta p, const float *qk, const uint16_t *rows, size_t ld, int n, DeltaWs w, uint16_t *out, size_t ldo) {
+__global__ __launch_bounds__(128, NV > 8 ? 1 : 2) void k_delta_out(Delta p, const float *qk, const uint16_t *rows, size_t ld, int n, DeltaWs w, uint16_t *out, size_t ldo) {
     __shared__ float sG[64];
-    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r16 = lane & 15, g = lane >> 4;
+    const int tid = threadIdx.x, lane = tid & 63, wave = __builtin_amdgcn_readfirstlane(tid >> 6), r16 = lane & 15, g = lane >> 4;
     const int c = blockIdx.x, h = blockIdx.y, heads = (int)p.heads, kvh = (int)p.kv_heads, dimp = (int)p.dimp, vdimp = (int)p.vdimp, kv = h / (heads / kvh);
     const int t0 = c * kDeltaChunk, len = min(kDeltaChunk, n - t0), C = 2 * kvh * dimp + heads * vdimp;
     const size_t ch = (size_t)h * w.nc + c, ldq = (size_t)2 * kvh * dimp;
@@ -580,66 +610,113 @@ __global__ __launch_bounds__(256, 2) void k_delta_out(Delta p, const float *qk, 
         const float *src = m + (size_t)min(t, len - 1) * ldq + kk * 32 + g * 4;
         return split8(*reinterpret_cast<const f32x4 *>(src), *reinterpret_cast<const f32x4 *>(src + 16));
     };
-    const int i = wave * 16 + r16;
-    SplitFrag q[NK];
-#pragma unroll
-    for (int kk = 0; kk < NK; ++kk) q[kk] = load(Q, i, kk);
-    f32x4 o[NV];
-    const float Gi = sG[i], ei = expf(Gi);
-#pragma unroll
-    for (int v = 0; v < NV; ++v) {
-        o[v] = f32x4{0.f, 0.f, 0.f, 0.f};
+    const int tile[2] = {wave, 3 - wave};
+    int i[2];
+    float Gi[2];
+    SplitFrag q[2][NK];
+    u32x4 sf[2][NK][2];
+    auto request = [&](int v) {
         const u32x4 *src = w.s + ((ch * w.nv + min(v, w.nv - 1)) * NK * 2) * 64 + lane;
 #pragma unroll
-        for (int kk = 0; kk < NK; ++kk) {
-            const bf16x8 hi = __builtin_bit_cast(bf16x8, src[kk * 128]), lo = __builtin_bit_cast(bf16x8, src[kk * 128 + 64]);
-            o[v] = mfma_bf16(hi, q[kk].hi, o[v]);
-            o[v] = mfma_bf16(hi, q[kk].lo, o[v]);
-            o[v] = mfma_bf16(lo, q[kk].hi, o[v]);
-        }
-        o[v] *= ei;
+        for (int kk = 0; kk < NK; ++kk) sf[v & 1][kk][0] = src[kk * 128], sf[v & 1][kk][1] = src[kk * 128 + 64];
+    };
+    request(0);
+#pragma unroll
+    for (int t = 0; t < 2; ++t) {
+        i[t] = tile[t] * 16 + r16;
+        Gi[t] = sG[i[t]];
+#pragma unroll
+        for (int kk = 0; kk < NK; ++kk) q[t][kk] = load(Q, i[t], kk);
     }
-    for (int k2 = 0; k2 <= wave / 2; ++k2) {
-        f32x4 s[2];
+    f32x4 o[NV][2];
+    const float ei[2] = {expf(Gi[0]), expf(Gi[1])};
+#pragma unroll
+    for (int v = 0; v < NV; ++v) {
+        if (v + 1 < NV) request(v + 1);
+        __builtin_amdgcn_sched_barrier(0);
+#pragma unroll
+        for (int t = 0; t < 2; ++t) o[v][t] = f32x4{0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+        for (int kk = 0; kk < NK; ++kk) {
+            const bf16x8 hi = __builtin_bit_cast(bf16x8, sf[v & 1][kk][0]), lo = __builtin_bit_cast(bf16x8, sf[v & 1][kk][1]);
+#pragma unroll
+            for (int t = 0; t < 2; ++t) o[v][t] = mfma_bf16(hi, q[t][kk].hi, o[v][t]);
+#pragma unroll
+            for (int t = 0; t < 2; ++t) o[v][t] = mfma_bf16(hi, q[t][kk].lo, o[v][t]);
+#pragma unroll
+            for (int t = 0; t < 2; ++t) o[v][t] = mfma_bf16(lo, q[t][kk].hi, o[v][t]);
+        }
+#pragma unroll
+        for (int t = 0; t < 2; ++t) o[v][t] *= ei[t];
+        __builtin_amdgcn_sched_barrier(0);
+    }
+    // tokens 32 k2 .. 32 k2 + 31: both tiles look at the first half, the later one at the second
+#pragma unroll
+    for (int k2 = 0; k2 < 2; ++k2) {
+        SplitFrag b[2];
+        f32x4 s[2][2];
 #pragma unroll
         for (int j = 0; j < 2; ++j) {
-            s[j] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-            for (int kk = 0; kk < NK; ++kk) s[j] = mfma_split(load(K, (k2 * 2 + j) * 16 + r16, kk), q[kk], s[j]);
+            for (int t = k2; t < 2; ++t) s[t][j] = f32x4{0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-            for (int e = 0; e < 4; ++e) {
-                const int t = (k2 * 2 + j) * 16 + g * 4 + e;
-                s[j][e] = t <= i ? s[j][e] * expf(Gi - sG[t]) : 0.f;
+            for (int kk = 0; kk < NK; ++kk) {
+                const SplitFrag k = load(K, (k2 * 2 + j) * 16 + r16, kk);
+#pragma unroll
+                for (int t = k2; t < 2; ++t) s[t][j] = mfma_split(k, q[t][kk], s[t][j]);
             }
+#pragma unroll
+            for (int t = k2; t < 2; ++t)
+#pragma unroll
+                for (int e = 0; e < 4; ++e) {
+                    const int at = (k2 * 2 + j) * 16 + g * 4 + e;
+                    s[t][j][e] = at <= i[t] ? s[t][j][e] * expf(Gi[t] - sG[at]) : 0.f;
+                }
         }
-        const SplitFrag b = split8(s[0], s[1]);
+#pragma unroll
+        for (int t = k2; t < 2; ++t) b[t] = split8(s[t][0], s[t][1]);
+        u32x4 uf[2][2];
+        auto request_u = [&](int v) {
+            const u32x4 *src = w.u + (((ch * w.nv + min(v, w.nv - 1)) * 2 + k2) * 2) * 64 + lane;
+            uf[v & 1][0] = src[0], uf[v & 1][1] = src[64];
+        };
+        request_u(0);
 #pragma unroll
         for (int v = 0; v < NV; ++v) {
-            const u32x4 *src = w.u + (((ch * w.nv + min(v, w.nv - 1)) * 2 + k2) * 2) * 64 + lane;
-            const bf16x8 hi = __builtin_bit_cast(bf16x8, src[0]), lo = __builtin_bit_cast(bf16x8, src[64]);
-            o[v] = mfma_bf16(hi, b.hi, o[v]);
-            o[v] = mfma_bf16(hi, b.lo, o[v]);
-            o[v] = mfma_bf16(lo, b.hi, o[v]);
+            if (v + 1 < NV) request_u(v + 1);
+            __builtin_amdgcn_sched_barrier(0);
+            const bf16x8 hi = __builtin_bit_cast(bf16x8, uf[v & 1][0]), lo = __builtin_bit_cast(bf16x8, uf[v & 1][1]);
+#pragma unroll
+            for (int t = k2; t < 2; ++t) {
+                o[v][t] = mfma_bf16(hi, b[t].hi, o[v][t]);
+                o[v][t] = mfma_bf16(hi, b[t].lo, o[v][t]);
+                o[v][t] = mfma_bf16(lo, b[t].hi, o[v][t]);
+            }
+            __builtin_amdgcn_sched_barrier(0);
         }
     }
-    float ss = 0.f;
 #pragma unroll
-    for (int v = 0; v < NV; ++v)
-        if (v < w.nv) ss += (o[v].x * o[v].x + o[v].y * o[v].y) + (o[v].z * o[v].z + o[v].w * o[v].w);
-    const float inv = 1.0f / sqrtf(rows_sum(ss) / (float)p.vdim + p.eps);
-    if (i >= len) return;
-    const uint16_t *gate = rows + (size_t)(t0 + i) * ld + C + (size_t)h * vdimp + g * 4;
-    uint16_t *dst = out + (size_t)(t0 + i) * ldo + (size_t)h * vdimp + g * 4;
+    for (int t = 0; t < 2; ++t) {
+        float ss = 0.f;
 #pragma unroll
-    for (int v = 0; v < NV; ++v)
-        if (v < w.nv) {
-            const u32x2 gb = *reinterpret_cast<const u32x2 *>(gate + v * 16);
-            const f32x4 nw = *reinterpret_cast<const f32x4 *>(p.norm + v * 16 + g * 4), ga = f32x4{bf2f(gb.x & 0xffffu), bf2f(gb.x >> 16), bf2f(gb.y & 0xffffu), bf2f(gb.y >> 16)};
-            f32x4 r = o[v] * inv * nw;
+        for (int v = 0; v < NV; ++v)
+            if (v < w.nv) ss += (o[v][t].x * o[v][t].x + o[v][t].y * o[v][t].y) + (o[v][t].z * o[v][t].z + o[v][t].w * o[v][t].w);
+        const float inv = 1.0f / sqrtf(rows_sum(ss) / (float)p.vdim + p.eps);
+        if (i[t] >= len) continue;
+        const uint16_t *gate = rows + (size_t)(t0 + i[t]) * ld + C + (size_t)h * vdimp + g * 4;
+        uint16_t *dst = out + (size_t)(t0 + i[t]) * ldo + (size_t)h * vdimp + g * 4;
 #pragma unroll
-            for (int e = 0; e < 4; ++e) r[e] *= ga[e] * __builtin_amdgcn_rcpf(1.0f + __expf(-ga[e]));
-            *reinterpret_cast<bf16x4 *>(dst + v * 16) = bf16x4{(__bf16)r.x, (__bf16)r.y, (__bf16)r.z, (__bf16)r.w};
-        }
+        for (int v = 0; v < NV; ++v)
+            if (v < w.nv) {
+                const u32x2 gb = *reinterpret_cast<const u32x2 *>(gate + v * 16);
+                const f32x4 nw = *reinterpret_cast<const f32x4 *>(p.norm + v * 16 + g * 4);
+                const f32x4 ga = f32x4{bf2f(gb.x & 0xffffu), bf2f(gb.x >> 16), bf2f(gb.y & 0xffffu), bf2f(gb.y >> 16)};
+                f32x4 r = o[v][t] * inv * nw;
+#pragma unroll
+                for (int e = 0; e < 4; ++e) r[e] *= ga[e] * __builtin_amdgcn_rcpf(1.0f + __expf(-ga[e]));
+                *reinterpret_cast<bf16x4 *>(dst + v * 16) = bf16x4{(__bf16)r.x, (__bf16)r.y, (__bf16)r.z, (__bf16)r.w};
+            }
+    }
 }
 
 // bytes of one chunk and head: w, k (same size), ut, s, u, g
@@ -653,7 +730,7 @@ size_t delta_workspace_bytes(size_t n, size_t heads, size_t dimp, size_t vdimp) 
 template <int NK>
 static hipError_t out_nv(const Delta &d, const float *qk, const uint16_t *rows, size_t ld, int n, const DeltaWs &w, uint16_t *out, size_t ldo, hipStream_t s) {
     auto fn = w.nv <= 4 ? k_delta_out<NK, 4> : w.nv <= 8 ? k_delta_out<NK, 8> : k_delta_out<NK, 16>;
-    hipLaunchKernelGGL(fn, dim3(w.nc, d.heads), dim3(256), 0, s, d, qk, rows, ld, n, w, out, ldo);
+    hipLaunchKernelGGL(fn, dim3(w.nc, d.heads), dim3(128), 0, s, d, qk, rows, ld, n, w, out, ldo);
     return hipGetLastError();
 }
 
@@ -682,7 +759,7 @@ hipError_t launch_delta_chunked(const Delta &d, const float *qk, const uint16_t 
         hipLaunchKernelGGL(k_delta_chunk, dim3(w.nc, d.heads), dim3(256), lds, s, d, q, vv, gt, m, w);
         const dim3 grid(8 * ((d.heads + 7) / 8) * w.nv);
         auto scan = nk == 1 ? k_delta_scan<1> : nk == 2 ? k_delta_scan<2> : nk == 3 ? k_delta_scan<3> : k_delta_scan<4>;
-        hipLaunchKernelGGL(scan, grid, dim3(64), 0, s, d, w);
+        hipLaunchKernelGGL(scan, grid, dim3(256), 0, s, d, w);
         const hipError_t e = nk == 1 ? out_nv<1>(d, q, rr, ld, m, w, oo, ldo, s) : nk == 2 ? out_nv<2>(d, q, rr, ld, m, w, oo, ldo, s)
                            : nk == 3 ? out_nv<3>(d, q, rr, ld, m, w, oo, ldo, s) : out_nv<4>(d, q, rr, ld, m, w, oo, ldo, s);
         if (e != hipSuccess) return e;

@@ -285,11 +285,12 @@ __global__ __launch_bounds__(256) void k_experts_out(OutK p) {
     int g = blockIdx.x * 4 + wave;
     if (g < p.groups) fetch(g, 0);
     const int total = p.chunks * CH / 4;
-    for (int i0 = tid; i0 < total; i0 += 256 * kStage) {
-        f32x4 v[kStage];
-        bool in[kStage];
+    constexpr int AH = 12;
+    for (int i0 = tid; i0 < total; i0 += 256 * AH) {
+        f32x4 v[AH];
+        bool in[AH];
 #pragma unroll
-        for (int j = 0; j < kStage; ++j) {
+        for (int j = 0; j < AH; ++j) {
             const int i = i0 + 256 * j, c = i / (CH / 4), x = max(c - p.c0, 0), q = min((int)((unsigned)x * p.magic >> 20), a.top - 1);
             const bool first = c < p.c0;
             const int col = (first ? i : i - (p.c0 + q * p.ce) * (CH / 4)) * 4, cols = first ? a.cols0 : a.cols1;
@@ -297,7 +298,7 @@ __global__ __launch_bounds__(256) void k_experts_out(OutK p) {
             v[j] = *reinterpret_cast<const f32x4 *>((first ? a.x0 : a.x1 + (size_t)q * a.ldx1) + min(col, cols - 4));
         }
 #pragma unroll
-        for (int j = 0; j < kStage; ++j)
+        for (int j = 0; j < AH; ++j)
             if (i0 + 256 * j < total) reinterpret_cast<f32x4 *>(xs)[i0 + 256 * j] = in[j] ? v[j] : f32x4{0.f, 0.f, 0.f, 0.f};
     }
     __syncthreads();
@@ -373,14 +374,14 @@ static hipError_t out_go(const ExpertsOut &a, hipStream_t s) {
     k.a = a;
     constexpr int CH = LPR * 8;
     k.c0 = (a.cols0 + CH - 1) / CH, k.ce = (a.cols1 + CH - 1) / CH;
-    const int chunks = k.c0 + a.top * k.ce, u = chunks >= 4 ? 4 : chunks == 3 ? 3 : 2;
+    const int chunks = k.c0 + a.top * k.ce, u = chunks >= 8 ? 8 : chunks >= 4 ? 4 : 2;
     k.chunks = (chunks + u - 1) / u * u;
     k.magic = ((1u << 20) + k.ce - 1) / k.ce;
     k.groups = (a.rows + 64 / LPR * R - 1) / (64 / LPR * R);
     const size_t lds = (size_t)k.chunks * CH * 4;
     // (the quotient by multiplication holds while chunks * ce stays below 2^20)
     if (lds > 150 * 1024 || (long)k.chunks * k.ce >= 1 << 20) return hipErrorInvalidValue;
-    auto fn = u == 2 ? k_experts_out<LPR, R, 2> : u == 3 ? k_experts_out<LPR, R, 3> : k_experts_out<LPR, R, 4>;
+    auto fn = u == 2 ? k_experts_out<LPR, R, 2> : u == 4 ? k_experts_out<LPR, R, 4> : k_experts_out<LPR, R, 8>;
     if (lds > 65536) {
         const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(fn), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
         if (e != hipSuccess) return e;

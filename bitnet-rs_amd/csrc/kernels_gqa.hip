@@ -157,9 +157,10 @@ hipError_t launch_gqa_any(const Gqa &g, const void *q, size_t ldq, int q_f32, in
 // sum and output of its own, and the four meet at the end.  S^T = K Q^T: row 4 g + e of score tile t is key 8 g + 4 t + e of the block, so that a
 // lane's weights of both tiles are the eight consecutive keys 8 g .. 8 g + 7 which it needs as an operand of O^T = V^T P^T.
 template <int NK, int NV, int MAPS>
-__global__ __launch_bounds__(256, NV > 8 ? 1 : 2) void k_gqa_step(Gqa p, GqaStep a) {
+__global__ __launch_bounds__(256, NV > 8 || NK * MAPS >= 8 ? 1 : 2) void k_gqa_step(Gqa p, GqaStep a) {
     extern __shared__ __attribute__((aligned(16))) float area[];  // queries [maps][16][NK * 32]; then the waves' outputs
     __shared__ float sm[4][MAPS][16], sl[4][MAPS][16];
+    __shared__ __attribute__((aligned(16))) uint16_t newk[MAPS][NK * 32], newv[NV * 16];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, r16 = lane & 15, g = lane >> 4;
     const int group = (int)(p.heads / p.kv_heads), ht = (group + 15) / 16, kv = blockIdx.y / ht, h0 = kv * group + (blockIdx.y - kv * ht) * 16;
     const int nh = min(16, (kv + 1) * group - h0), dim = (int)p.dim, dimp = (int)p.dimp, vdimp = (int)p.vdimp;
@@ -185,8 +186,8 @@ __global__ __launch_bounds__(256, NV > 8 ? 1 : 2) void k_gqa_step(Gqa p, GqaStep
     };
     constexpr bool kAhead = NK <= 4;  // the first block is requested ahead of the norms (registers allow it)
     const bool owner = k1 == n_keys;
-    if (kAhead && !owner) fetch(k0 + wave * 32);
-    if (owner) {  // the record that holds the new position appends it
+    if (kAhead) fetch(k0 + wave * 32);
+    if (owner) {  // the record that holds the new position appends it (and puts it into its own fragments below)
         if (wave < MAPS) {
             float v[NK], ss = 0.f;
 #pragma unroll
@@ -198,20 +199,32 @@ __global__ __launch_bounds__(256, NV > 8 ? 1 : 2) void k_gqa_step(Gqa p, GqaStep
 #pragma unroll
             for (int j = 0; j < (NK + 1) / 2; ++j) {
                 const int i = lane + 64 * j;
-                if (i < dimp) K[((size_t)wave * p.capacity + pos) * dimp + i] = f2bf(v[j] * norm * (p.k_weight && i < dim ? p.k_weight[i] : 1.0f));
+                if (i < dimp) {
+                    const uint16_t b = f2bf(v[j] * norm * (p.k_weight && i < dim ? p.k_weight[i] : 1.0f));
+                    K[((size_t)wave * p.capacity + pos) * dimp + i] = b;
+                    newk[wave][i] = b;
+                }
             }
         }
-        for (int i = tid; i < vdimp; i += 256) V[(size_t)i * p.capacity + pos] = f2bf(vraw[i]);
+        for (int i = tid; i < vdimp; i += 256) {
+            const uint16_t b = f2bf(vraw[i]);
+            V[(size_t)i * p.capacity + pos] = b;
+            newv[i] = b;
+        }
     }
     {
         const float factor = p.q_factor[pos];
         for (int r = wave; r < MAPS * 16; r += 4) {
             const int map = r >> 4, hh = r & 15;
-            const float *q = a.row + ((size_t)(h0 + min(hh, nh - 1)) * MAPS + map) * dimp;
+            if (hh >= nh) {
+                for (int i = lane; i < NK * 32; i += 64) area[r * QS + i] = 0.f;
+                continue;
+            }
+            const float *q = a.row + ((size_t)(h0 + hh) * MAPS + map) * dimp;
             float v[NK], ss = 0.f;
 #pragma unroll
             for (int j = 0; j < (NK + 1) / 2; ++j) {
-                v[j] = lane + 64 * j < dimp && hh < nh ? q[lane + 64 * j] : 0.f;
+                v[j] = lane + 64 * j < dimp ? q[lane + 64 * j] : 0.f;
                 ss += v[j] * v[j];
             }
             const float norm = (p.q_weight ? 1.0f / sqrtf(wave_sum(ss) / (float)dim + p.eps) : 1.0f) * factor;
@@ -222,7 +235,7 @@ __global__ __launch_bounds__(256, NV > 8 ? 1 : 2) void k_gqa_step(Gqa p, GqaStep
             }
         }
     }
-    __syncthreads();  // queries; and the appended rows are there for every wave of this workgroup
+    __syncthreads();
     SplitFrag q[MAPS][NK];
 #pragma unroll
     for (int m = 0; m < MAPS; ++m)
@@ -241,7 +254,29 @@ __global__ __launch_bounds__(256, NV > 8 ? 1 : 2) void k_gqa_step(Gqa p, GqaStep
         for (int v = 0; v < NV; ++v) o[v][j] = f32x4{0.f, 0.f, 0.f, 0.f};
     }
     for (int kb = k0 + wave * 32; kb < k1; kb += 128) {
-        if (!kAhead || owner || kb >= k0 + 128) fetch(kb);
+        if (!kAhead || kb >= k0 + 128) fetch(kb);
+        if (owner && pos - kb < 32) {  // the new position, which memory need not show yet
+            const int at = pos - kb, t = (at >> 2) & 1;
+            const bool mine = r16 == (at >> 3) * 4 + (at & 3);
+#pragma unroll
+            for (int j = 0; j < MAPS; ++j)
+#pragma unroll
+                for (int kk = 0; kk < NK; ++kk) {
+                    const u32x4 k = *reinterpret_cast<const u32x4 *>(&newk[j][min(kk * 32, dimp - 32) + g * 8]);
+                    if (mine && t == 0) kf[0][j][kk] = k;
+                    if (mine && t == 1) kf[1][j][kk] = k;
+                }
+            if (g == at >> 3) {
+                const uint32_t keep = (at & 1) ? 0xffffu : 0xffff0000u, sh = (at & 1) * 16;
+#pragma unroll
+                for (int v = 0; v < NV; ++v) {
+                    const uint32_t n = (uint32_t)newv[min(v * 16 + r16, vdimp - 1)] << sh;
+#pragma unroll
+                    for (int e = 0; e < 4; ++e)
+                        if (e == (at & 7) >> 1) vf[v][e] = (vf[v][e] & keep) | n;
+                }
+            }
+        }
 #pragma unroll
         for (int j = 0; j < MAPS; ++j) {
             f32x4 s[2];
