@@ -168,7 +168,7 @@ constexpr int kGqaTile = 128;      // keys per workgroup and step of the decode 
 constexpr int kGqaSplits = 128;    // most records per (query, head, map)
 constexpr int kGqaRecHead = 4;     // floats ahead of a record's vector: running maximum (of base-2 scores), sum, unused
 constexpr int kDeltaChunk = 64;    // tokens per chunk of the delta rule
-constexpr int kDeltaSegment = 4096;  // tokens per pass over the workspace
+constexpr int kDeltaUnits = 512;   // chunks x heads per pass over the workspace: one round of workgroups, and small enough to stay in the caches
 constexpr int kMaxExperts = 1024, kMaxTop = 32;
 
 hipError_t launch_embed_bf16(const uint16_t *table, size_t ld, const int *tokens, const int *offset, int n, int width, int vocab, float scale, float *out,

@@ -12,6 +12,8 @@
 // k_delta_chunk forms T and the products with it for all chunks at once, k_delta_scan walks the chunks (one workgroup per 16 value columns,
 // operands straight from memory in the order the matrix cores want them), k_delta_out forms the outputs of all chunks.
 // f32 operands enter the matrix cores as (high, low) pairs of bf16 values; L and T are f32 throughout.
+#include <algorithm>
+
 #include "dense.hpp"
 
 namespace bitnet_hip {
@@ -722,9 +724,10 @@ __global__ __launch_bounds__(128, NV > 8 ? 1 : 2) void k_delta_out(Delta p, cons
 // bytes of one chunk and head: w, k (same size), ut, s, u, g
 static size_t chunk_bytes(size_t nk, size_t nv) { return 2 * (4 * nk * 2048) + nv * 4096 + nv * nk * 2048 + nv * 4096 + 256; }
 
+static size_t segment_chunks(size_t heads) { return std::max((size_t)kDeltaUnits / heads, (size_t)4); }
+
 size_t delta_workspace_bytes(size_t n, size_t heads, size_t dimp, size_t vdimp) {
-    const size_t m = n < (size_t)kDeltaSegment ? n : (size_t)kDeltaSegment;
-    return (m + kDeltaChunk - 1) / kDeltaChunk * heads * chunk_bytes(dimp / 32, vdimp / 16);
+    return std::min((n + kDeltaChunk - 1) / kDeltaChunk, segment_chunks(heads)) * heads * chunk_bytes(dimp / 32, vdimp / 16);
 }
 
 template <int NK>
@@ -742,8 +745,9 @@ hipError_t launch_delta_chunked(const Delta &d, const float *qk, const uint16_t 
         const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(k_delta_chunk), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
         if (e != hipSuccess) return e;
     }
-    for (int t0 = 0; t0 < n; t0 += kDeltaSegment) {
-        const int m = min(kDeltaSegment, n - t0);
+    const int segment = (int)segment_chunks(d.heads) * kDeltaChunk;
+    for (int t0 = 0; t0 < n; t0 += segment) {
+        const int m = min(segment, n - t0);
         DeltaWs w;
         w.nc = (m + kDeltaChunk - 1) / kDeltaChunk, w.nk = (int)d.dimp / 32, w.nv = (int)d.vdimp / 16;
         const size_t ch = (size_t)w.nc * d.heads, nk = w.nk, nv = w.nv;

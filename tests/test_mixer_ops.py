@@ -326,7 +326,7 @@ def test_delta_chunks_hold_32_bits(hip, pkg):
 
 
 def test_delta_more_than_one_segment(hip, pkg):
-    a, b = (DeltaCase(pkg, 2048 + 70, 2, 1, 32, 32, 4, False) for _ in range(2))
+    a, b = (DeltaCase(pkg, 700, 64, 32, 16, 16, 4, False) for _ in range(2))  # (eight chunks of 64 heads per pass)
     x, y = a.portion(hip, 0, a.n, True), b.portion(hip, 0, b.n, False)
     assert u.rms_error(x, y) < 8e-3 and u.rms_error(u.host(a.keep[4]), u.host(b.keep[4])) < 1e-4
 
