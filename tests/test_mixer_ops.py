@@ -407,7 +407,7 @@ def test_experts_of_a_portion(hip, pkg, m, experts, top, tile, width, ff, f32):
     assert u.rms_error(got, want) < (F32_TOL if f32 else 8e-3)
 
 
-@pytest.mark.parametrize("experts,top,width,ff,cols0", [(4, 1, 64, 24, 8), (6, 6, 112, 40, 200), (16, 2, 256, 64, 160), (64, 8, 1000, 520, 1032), (128, 4, 2560, 768, 3328), (9, 3, 90, 16, 64)])
+@pytest.mark.parametrize("experts,top,width,ff,cols0", [(4, 1, 64, 24, 8), (6, 6, 112, 40, 200), (12, 3, 320, 72, 160), (64, 8, 1000, 520, 1032), (128, 4, 2560, 768, 3328), (9, 3, 90, 16, 64)])
 def test_experts_of_one_token(hip, pkg, experts, top, width, ff, cols0):
     g = rng(experts, width, ff)
     z, ids, w = routing(1, experts, top, 2)
