@@ -50,6 +50,10 @@ def softplus(z):
     return np.maximum(z, 0.0) + np.log1p(np.exp(-np.abs(z)))
 
 
+def gelu_tanh(z):
+    return 0.5 * z * (1.0 + np.tanh(math.sqrt(2.0 / math.pi) * (z + 0.044715 * z ** 3)))
+
+
 # ---- rotary positions ------------------------------------------------------------------------------------------------
 def rotary_frequencies(rot):
     """(frequency per pair, factor on cos and sin)"""
@@ -80,6 +84,33 @@ def rotate(v, positions, rot):
         u, w = v[t][..., :half], v[t][..., half:2 * half]
         out[t][..., :half] = u * c - w * s
         out[t][..., half:2 * half] = w * c + u * s
+    return out
+
+
+def banded_frequencies(rot):
+    """frequency per pair: slow pairs (long wavelengths) divided by the factor, fast ones kept, a line between the two bands"""
+    out, s = [], rot.get("scaling")
+    for i in range(rot["dims"] // 2):
+        f = float(rot["base"]) ** (-2.0 * i / rot["dims"])
+        if s:
+            turns = s["original"] * f / (2.0 * math.pi)  # within the original length
+            if turns < s["low"]:
+                f = f / s["factor"]
+            elif turns <= s["high"]:
+                keep = (turns - s["low"]) / (s["high"] - s["low"])
+                f = (1.0 - keep) * f / s["factor"] + keep * f
+        out.append(f)
+    return np.array(out, F)
+
+
+def rotate_neighbours(v, rot):
+    """v [tokens, heads, dim]: elements 2i and 2i + 1 turn together, elements from rot["dims"] on stay"""
+    out, f = np.array(v, F), banded_frequencies(rot)
+    for p in range(len(v)):
+        for i, fi in enumerate(f):
+            c, s = math.cos(p * fi), math.sin(p * fi)
+            a, b = v[p, :, 2 * i], v[p, :, 2 * i + 1]
+            out[p, :, 2 * i], out[p, :, 2 * i + 1] = a * c - b * s, b * c + a * s
     return out
 
 
@@ -161,6 +192,31 @@ def differential_attention(h, t, p, m, eps):
     return out.reshape(n, H * V) @ t[p + "o"].T
 
 
+def chunk_softmax(q, k, v, scale, chunk):
+    """q [n, heads, dim], k [n, kv heads, dim], v [n, kv heads, vdim]: a token sees what lies ahead of it in its own chunk of positions; the
+    softmax's denominator holds one more"""
+    n, H, _ = q.shape
+    out = np.zeros((n, H, v.shape[2]), F)
+    for a in range(H):
+        g = a // (H // k.shape[1])
+        for i in range(n):
+            first = i // chunk * chunk
+            s = k[first:i + 1, g] @ q[i, a] * scale
+            top = max(s.max(), 0.0)
+            e = np.exp(s - top)
+            out[i, a] = e @ v[first:i + 1, g] / (math.exp(-top) + e.sum())
+    return out
+
+
+def chunk_attention(h, t, p, m, eps):
+    n, H, G, D = len(h), m["heads"], m["kv_heads"], m["dim"]
+    q, k = (h @ t[p + "q"].T).reshape(n, H, D), (h @ t[p + "k"].T).reshape(n, G, D)
+    qr, kr = (rms_divide(rotate_neighbours(x, m["rot"]), eps) for x in (q, k))
+    o = chunk_softmax(qr, kr, k, m["scale"], m["mask"]["size"])
+    o = o * sigmoid(h @ t[p + "g"].T)[:, :, None]
+    return o.reshape(n, H * D) @ t[p + "o"].T
+
+
 def short_convolution(x, w):
     """x [tokens, channels], w [channels, taps]: the last tap meets the current token, zeros stand ahead of the first"""
     taps = w.shape[1]
@@ -230,11 +286,35 @@ def expert_mlp(h, t, p, f):
     return out
 
 
+def gated_mlp(h, t, p, act):
+    return (act(h @ t[p + "gate"].T) * (h @ t[p + "up"].T)) @ t[p + "down"].T
+
+
+def route_corrected(h, router, correction, top):
+    """per token: the experts with the largest corrected scores, and their uncorrected scores"""
+    z = h @ router.T
+    s = np.exp(z - z.max(axis=1, keepdims=True))
+    s /= s.sum(axis=1, keepdims=True)
+    ids = np.argsort(-(s + correction), axis=1, kind="stable")[:, :top]
+    return ids, np.take_along_axis(s, ids, 1)
+
+
+def expert_or_identity_mlp(h, t, p, f):
+    """experts behind the last one with tensors hand their input through"""
+    r = f["router"]
+    ids, w = route_corrected(h, t[p + "router"], t[p + "correction"], r["top"])
+    out = np.zeros_like(h)
+    for i in range(len(h)):
+        for e, x in zip(ids[i], w[i]):
+            out[i] += x * (gated_mlp(h[i:i + 1], t, p + f"e{e}.", silu)[0] if e < r["experts"] else h[i])
+    return out
+
+
 # ---- the stack -------------------------------------------------------------------------------------------------------
 def forward(config, tensors, tokens):
     """(logits [n, vocab], residual stream after every layer run [runs, n, width])"""
     t = {k: np.asarray(v, F) for k, v in tensors.items()}
-    return {"Lasapel": forward_lasapel, "Mimolix": forward_mimolix}[config["architecture"]](config, t, tokens)
+    return {"Lasapel": forward_lasapel, "Mimolix": forward_mimolix, "Lurepel": forward_lurepel}[config["architecture"]](config, t, tokens)
 
 
 def layer_runs(config):
@@ -282,3 +362,17 @@ def forward_lasapel(config, t, tokens):
             x = x + norm_around_zero(y, t[p + "norm2b"], eps) * t[p + "ls2"]
         after.append(x)
     return norm_around_zero(x, t["final.norm"], eps) @ t["head"].T, np.stack(after)
+
+
+def forward_lurepel(config, t, tokens):
+    eps = config["norm"]["eps"]
+    x = norm_plain(t["embed"][np.asarray(tokens)], t["embed.norm"], eps)
+    after = []
+    for i, layer in enumerate(config["layers"]):
+        p, f = f"l{i}.", layer.get("mlp")
+        x = x + norm_plain(chunk_attention(x, t, p + "mix.", layer["mixer"], eps), t[p + "norm1"], eps)
+        if f:
+            y = gated_mlp(x, t, p + "mlp.", gelu_tanh) if f["kind"] == "dense" else expert_or_identity_mlp(x, t, p + "mlp.", f)
+            x = x + norm_plain(y, t[p + "norm2"], eps)
+        after.append(x)
+    return norm_plain(x, t["final.norm"], eps) @ t["head"].T, np.stack(after)
