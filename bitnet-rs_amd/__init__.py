@@ -95,8 +95,8 @@ def _addr(t):
     return None if t is None else (t if isinstance(t, int) else t.data_ptr())
 
 
-ACT_NONE, ACT_SILU, ACT_SIGMOID, ACT_RELU2 = 0, 1, 2, 3
-IN_PLAIN, IN_NORM, IN_RESIDUAL_NORM, IN_CONCAT = 0, 1, 2, 3
+ACT_NONE, ACT_SILU, ACT_SIGMOID, ACT_RELU2, ACT_GELU_TANH, ACT_GATED = 0, 1, 2, 3, 4, 0x100
+IN_PLAIN, IN_NORM, IN_RESIDUAL_NORM, IN_CONCAT, IN_RESIDUAL = 0, 1, 2, 3, 4
 LINEAR_BLOCK = 128
 
 
@@ -109,18 +109,24 @@ class VectorInput(C.Structure):
 class SumRows(C.Structure):
     _fields_ = [("x", _vp), ("m", _sz), ("width", _sz), ("y", _vp), ("ldy", _sz), ("mult", C.c_float), ("expert_rows", _vp), ("ld_expert", _sz), ("top", _sz),
                 ("slots", _vp), ("slot_weights", _vp), ("weight", _vp), ("bias", _vp), ("x2", _vp), ("weight_offset", C.c_float), ("eps", C.c_float),
-                ("center", C.c_int32), ("h_f32", C.c_int32), ("h", _vp), ("ldh", _sz)]
+                ("center", C.c_int32), ("h_f32", C.c_int32), ("h", _vp), ("ldh", _sz), ("post_weight", _vp), ("scale", _vp), ("input", _vp), ("ld_input", _sz)]
 
 
 class Gqa(C.Structure):
     _fields_ = [(n, _sz) for n in ("heads", "kv_heads", "maps", "dim", "dimp", "vdim", "vdimp", "capacity")] + [
-        ("eps", C.c_float), ("lam", C.c_float), ("out_scale", C.c_float), ("q_weight", _vp), ("k_weight", _vp), ("q_factor", _vp), ("kcache", _vp), ("vcache", _vp)]
+        ("eps", C.c_float), ("lam", C.c_float), ("out_scale", C.c_float), ("q_weight", _vp), ("k_weight", _vp), ("q_factor", _vp), ("kcache", _vp), ("vcache", _vp),
+        ("unit_norm", C.c_int32), ("values_are_keys", C.c_int32), ("rot_dims", _sz), ("chunk", _sz), ("rope_cos", _vp), ("rope_sin", _vp), ("sink", _vp), ("gate", _vp),
+        ("ldgate", _sz), ("gate_f32", C.c_int32)]
 
 
 class Delta(C.Structure):
     _fields_ = [(n, _sz) for n in ("heads", "kv_heads", "dim", "dimp", "vdim", "vdimp", "taps")] + [
         ("conv", _vp), ("decay_rate", _vp), ("dt_bias", _vp), ("norm", _vp), ("q_scale", C.c_float), ("unit_eps", C.c_float), ("eps", C.c_float), ("state", _vp),
         ("ring", _vp)]
+
+
+class Router(C.Structure):
+    _fields_ = [("experts", _sz), ("identity", _sz), ("top", _sz), ("scale", C.c_float), ("raw", C.c_int32), ("correction", _vp)]
 
 
 class ExpertsPlan(C.Structure):
@@ -580,6 +586,11 @@ class HipLib:
     def embed_bf16_dev(self, table, ld: int, tokens, out, n: int, width: int, vocab: int, offset=None, scale: float = 1.0, stream: int = 0) -> None:
         self._call("embed_bf16_dev", _ptr(table), _sz(ld), _ptr(tokens), _optr(offset), _sz(n), _sz(width), _sz(vocab), C.c_float(scale), _ptr(out), _vp(stream))
 
+    def embed_norm_bf16_dev(self, table, ld: int, tokens, norm_weight, eps: float, out, n: int, width: int, vocab: int, offset=None, scale: float = 1.0,
+                            stream: int = 0) -> None:
+        self._call("embed_norm_bf16_dev", _ptr(table), _sz(ld), _ptr(tokens), _optr(offset), _sz(n), _sz(width), _sz(vocab), C.c_float(scale), _ptr(norm_weight),
+                   C.c_float(eps), _ptr(out), _vp(stream))
+
     def sum_norm_rows_dev(self, rows: "SumRows", stream: int = 0) -> None:
         self._call("sum_norm_rows_dev", C.byref(rows), _vp(stream))
 
@@ -632,21 +643,22 @@ class HipLib:
         self._call("experts_plan_make", _ptr(workspace), _sz(nbytes), _sz(m), _sz(experts), _sz(top), _sz(tile), C.byref(p))
         return p
 
-    def experts_route_dev(self, logits, ldz: int, scale: float, plan: "ExpertsPlan", stream: int = 0) -> None:
-        self._call("experts_route_dev", _ptr(logits), _sz(ldz), C.c_float(scale), C.byref(plan), _vp(stream))
+    def experts_route_dev(self, logits, ldz: int, router: "Router", plan: "ExpertsPlan", stream: int = 0) -> None:
+        self._call("experts_route_dev", _ptr(logits), _sz(ldz), C.byref(router), C.byref(plan), _vp(stream))
 
     def experts_matmul_dev(self, plan: "ExpertsPlan", gather: bool, a, lda: int, a_f32: bool, w, n: int, k: int, ldw: int, act: int, c, ldc: int, c_f32: bool,
                            stream: int = 0) -> None:
         self._call("experts_matmul_dev", C.byref(plan), C.c_int(gather), _ptr(a), _sz(lda), C.c_int(a_f32), _ptr(w), _sz(n), _sz(k), _sz(ldw), C.c_int(act), _ptr(c),
                    _sz(ldc), C.c_int(c_f32), _vp(stream))
 
-    def experts_up_dev(self, logits, experts: int, top: int, scale: float, x, w, rows: int, cols: int, ld: int, act: int, y, ldy: int, ids, stream: int = 0) -> None:
-        self._call("experts_up_dev", _ptr(logits), _sz(experts), _sz(top), C.c_float(scale), _ptr(x), _ptr(w), _sz(rows), _sz(cols), _sz(ld), C.c_int(act), _ptr(y),
-                   _sz(ldy), _ptr(ids), _vp(stream))
+    def experts_up_dev(self, logits, router: "Router", x, w, rows: int, cols: int, ld: int, act: int, y, ldy: int, ids, identity=None, stream: int = 0) -> None:
+        self._call("experts_up_dev", _ptr(logits), C.byref(router), _ptr(x), _ptr(w), _sz(rows), _sz(cols), _sz(ld), C.c_int(act), _ptr(y), _sz(ldy), _ptr(ids),
+                   _optr(identity), _vp(stream))
 
-    def experts_out_dev(self, x0, w0, cols0: int, ld0: int, bias, x1, ldx1: int, w1, cols1: int, ld1: int, ids, top: int, rows: int, y, stream: int = 0) -> None:
-        self._call("experts_out_dev", _ptr(x0), _ptr(w0), _sz(cols0), _sz(ld0), _optr(bias), _ptr(x1), _sz(ldx1), _ptr(w1), _sz(cols1), _sz(ld1), _ptr(ids), _sz(top),
-                   _sz(rows), _ptr(y), _vp(stream))
+    def experts_out_dev(self, x0, w0, cols0: int, ld0: int, bias, x1, ldx1: int, w1, cols1: int, ld1: int, ids, top: int, rows: int, y, identity=None, input=None,
+                        stream: int = 0) -> None:
+        self._call("experts_out_dev", _optr(x0), _optr(w0), _sz(cols0), _sz(ld0), _optr(bias), _ptr(x1), _sz(ldx1), _ptr(w1), _sz(cols1), _sz(ld1), _ptr(ids), _sz(top),
+                   _sz(rows), _optr(identity), _optr(input), _ptr(y), _vp(stream))
 
     def residual_norm_rows_dev(self, x, m: int, width: int, eps: float, weight_offset: float, y=None, ldy: int = 0, post_weight=None, scale=None,
                                next_weight=None, h=None, ldh: int = 0, h_f32: bool = True, stream: int = 0) -> None:

@@ -12,7 +12,7 @@ static_assert(kLinBlock == BITNET_HIP_LINEAR_BLOCK, "the decay table's length is
     } while (0)
 
 namespace {
-bool act_ok(int a) { return a >= BITNET_HIP_ACT_NONE && a <= BITNET_HIP_ACT_RELU2; }
+bool act_ok(int a) { return a >= BITNET_HIP_ACT_NONE && a <= BITNET_HIP_ACT_GELU_TANH; }
 
 int to_latent_rows(const bitnet_hip_latent_rows *r, size_t m, int f32, LatentRows &o) {
     BH_REQUIRE(r && r->z && r->pos, "latent_rows: null pointer");
@@ -32,12 +32,12 @@ int to_latent_rows(const bitnet_hip_latent_rows *r, size_t m, int f32, LatentRow
 
 int to_vec_in(const bitnet_hip_vector_input *in, size_t cols, VecIn &o) {
     BH_REQUIRE(in && in->x, "vector input: null pointer");
-    BH_REQUIRE(in->kind >= BITNET_HIP_IN_PLAIN && in->kind <= BITNET_HIP_IN_CONCAT, "vector input: unknown kind %d", in->kind);
+    BH_REQUIRE(in->kind >= BITNET_HIP_IN_PLAIN && in->kind <= BITNET_HIP_IN_RESIDUAL, "vector input: unknown kind %d", in->kind);
     if (in->kind != BITNET_HIP_IN_PLAIN) {
         if (in->kind == BITNET_HIP_IN_CONCAT)
             BH_REQUIRE(in->x2 && in->n > 0 && 2 * (size_t)in->n <= cols, "vector input: bad second half");
         else
-            BH_REQUIRE(in->weight && in->n > 0 && (size_t)in->n <= cols && in->mean_n >= 0, "vector input: bad norm");
+            BH_REQUIRE((in->weight || in->kind == BITNET_HIP_IN_RESIDUAL) && in->n > 0 && (size_t)in->n <= cols && in->mean_n >= 0, "vector input: bad norm");
         if (in->kind >= BITNET_HIP_IN_RESIDUAL_NORM && in->y)
             BH_REQUIRE((in->post_weight || in->mult != 0.f) && (!in->x_out || (in->x_out != in->x && in->x_out != in->y)),
                        "vector input: the residual needs a norm or a factor, and a buffer of its own");
@@ -68,7 +68,18 @@ int bitnet_hip_embed_bf16_dev(const uint16_t *table, size_t ld, const int32_t *t
     BH_REQUIRE(table && tokens && out, "Null pointer passed to embed_bf16_dev");
     BH_REQUIRE(n > 0 && width > 0 && vocab > 0 && ld >= width, "embed_bf16: bad shape");
     BH_CHECK_DIMS(n, width);
-    BH_HIP_TRY(launch_embed_bf16(table, ld, tokens, offset, (int)n, (int)width, (int)vocab, scale, out, (hipStream_t)stream));
+    BH_HIP_TRY(launch_embed_bf16(table, ld, tokens, offset, (int)n, (int)width, (int)vocab, scale, nullptr, 0.f, out, (hipStream_t)stream));
+    return BITNET_HIP_OK;
+    BH_GUARD_END
+}
+
+int bitnet_hip_embed_norm_bf16_dev(const uint16_t *table, size_t ld, const int32_t *tokens, const int32_t *offset, size_t n, size_t width, size_t vocab,
+                                   float scale, const float *norm_weight, float eps, float *out, void *stream) {
+    BH_GUARD_BEGIN
+    BH_REQUIRE(table && tokens && norm_weight && out, "Null pointer passed to embed_norm_bf16_dev");
+    BH_REQUIRE(n > 0 && width > 0 && vocab > 0 && ld >= width, "embed_norm_bf16: bad shape");
+    BH_CHECK_DIMS(n, width);
+    BH_HIP_TRY(launch_embed_bf16(table, ld, tokens, offset, (int)n, (int)width, (int)vocab, scale, norm_weight, eps, out, (hipStream_t)stream));
     return BITNET_HIP_OK;
     BH_GUARD_END
 }
@@ -76,7 +87,7 @@ int bitnet_hip_embed_bf16_dev(const uint16_t *table, size_t ld, const int32_t *t
 int bitnet_hip_residual_norm_rows_dev(float *x, const float *y, size_t ldy, const float *post_weight, const float *scale, const float *next_weight,
                                       float weight_offset, float eps, size_t m, size_t width, void *h, size_t ldh, int h_f32, void *stream) {
     BH_GUARD_BEGIN
-    BH_REQUIRE(x && (!y || (post_weight && ldy >= width)) && (!h || (next_weight && ldh >= width)), "residual_norm_rows: bad arguments");
+    BH_REQUIRE(x && (!y || (post_weight && ldy >= width)) && (!h || ldh >= width), "residual_norm_rows: bad arguments");
     BH_REQUIRE(m > 0 && width > 0, "residual_norm_rows: empty");
     BH_CHECK_DIMS(m, width);
     BH_HIP_TRY(launch_residual_norm_rows(x, y, ldy, post_weight, scale, next_weight, weight_offset, eps, (int)m, (int)width, h, ldh, h_f32,
@@ -110,15 +121,18 @@ int bitnet_hip_dense_matmul_dev(const void *a, size_t lda, int a_f32, const uint
     BH_GUARD_BEGIN
     BH_REQUIRE(a && w && c, "Null pointer passed to dense_matmul_dev");
     BH_REQUIRE(m > 0 && n > 0 && k > 0 && batch > 0 && batch < 65536, "dense_matmul: empty");
-    BH_REQUIRE(k % 64 == 0 && lda >= k && ldw >= k && lda % 8 == 0 && ldw % 8 == 0 && ldc >= n, "dense_matmul: k %zu must be a multiple of 64 inside lda %zu, ldw %zu; ldc %zu >= n %zu",
+    const int gated = act0 & BITNET_HIP_ACT_GATED;
+    act0 &= ~BITNET_HIP_ACT_GATED;
+    BH_REQUIRE(k % 64 == 0 && lda >= k && ldw >= k && lda % 8 == 0 && ldw % 8 == 0 && ldc >= (gated ? n / 2 : n), "dense_matmul: k %zu must be a multiple of 64 inside lda %zu, ldw %zu; ldc %zu >= n %zu",
                k, lda, ldw, ldc, n);
     BH_REQUIRE(act_ok(act0) && act_ok(act1) && a_batch % 8 == 0 && w_batch % 8 == 0, "dense_matmul: bad activation or batch stride");
+    BH_REQUIRE(!gated || (n % 2 == 0 && act_split == 0 && (a_f32 || !c_f32)), "dense_matmul: gated columns come in pairs, with one activation, in the activations' type");
     BH_CHECK_DIMS(m, lda);
     BH_CHECK_DIMS(n, ldw);
     BH_CHECK_DIMS(m, ldc);
     GemmArgsD g;
     g.a = a, g.w = w, g.bias = bias, g.c = c, g.m = (int)m, g.n = (int)n, g.k = (int)k, g.lda = lda, g.ldw = ldw, g.ldc = ldc;
-    g.act0 = act0, g.act1 = act1, g.act_split = (int)act_split, g.a_f32 = a_f32, g.c_f32 = c_f32;
+    g.act0 = act0, g.act1 = act1, g.act_split = (int)act_split, g.gated = gated != 0, g.a_f32 = a_f32, g.c_f32 = c_f32;
     g.batch = (int)batch, g.a_batch = a_batch, g.w_batch = w_batch, g.c_batch = c_batch;
     BH_HIP_TRY(launch_dense_gemm(g, (hipStream_t)stream));
     return BITNET_HIP_OK;
@@ -150,10 +164,13 @@ int bitnet_hip_dense_gemv_dev(const bitnet_hip_vector_input *input, const uint16
     BH_GUARD_BEGIN
     GemvArgs g;
     if (int rc = gemv_args(input, w, rows, cols, ld, y, g)) return rc;
+    const int gated = act0 & BITNET_HIP_ACT_GATED;
+    act0 &= ~BITNET_HIP_ACT_GATED;
     BH_REQUIRE(act_ok(act0) && act_ok(act1), "dense_gemv: unknown activation");
+    BH_REQUIRE(!gated || (rows % 2 == 0 && act_split == 0), "dense_gemv: gated rows come in pairs, with one activation");
     BH_REQUIRE(batch > 0 && batch < 65536 && (batch == 1 || (g.in.kind == BITNET_HIP_IN_PLAIN && !latent)) && w_batch % 8 == 0, "dense_gemv: bad batch");
     BH_CHECK_DIMS(batch, rows, ld);
-    g.bias = bias, g.act0 = act0, g.act1 = act1, g.act_split = (int)act_split;
+    g.bias = bias, g.act0 = act0, g.act1 = act1, g.act_split = (int)act_split, g.gated = gated != 0;
     g.batch = (int)batch, g.w_batch = w_batch, g.x_batch = x_batch, g.y_batch = y_batch;
     LatentRows r;
     if (latent) {

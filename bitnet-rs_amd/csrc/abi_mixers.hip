@@ -11,7 +11,7 @@ using namespace bitnet_hip;
     } while (0)
 
 namespace {
-bool act_ok(int a) { return a >= BITNET_HIP_ACT_NONE && a <= BITNET_HIP_ACT_RELU2; }
+bool act_ok(int a) { return a >= BITNET_HIP_ACT_NONE && a <= BITNET_HIP_ACT_GELU_TANH; }
 
 int check_gqa(const bitnet_hip_gqa *a) {
     BH_REQUIRE(a && a->q_factor && a->kcache && a->vcache, "gqa: null pointer");
@@ -20,11 +20,15 @@ int check_gqa(const bitnet_hip_gqa *a) {
                    a->capacity > 0 && a->capacity % kGqaTile == 0,
                "gqa: bad shape (%zu heads on %zu, %zu maps of %zu in %zu, values %zu in %zu, capacity %zu)", a->heads, a->kv_heads, a->maps, a->dim, a->dimp,
                a->vdim, a->vdimp, a->capacity);
+    BH_REQUIRE(a->rot_dims % 2 == 0 && a->rot_dims <= a->dim && (a->rot_dims == 0 || (a->rope_cos && a->rope_sin)), "gqa: bad rotation of %zu dimensions", a->rot_dims);
+    BH_REQUIRE(a->chunk < (size_t(1) << 30) && (!a->sink || a->maps == 1) && (!a->values_are_keys || (a->maps == 1 && a->vdim == a->dim && a->vdimp == a->dimp)) &&
+                   (!a->gate || a->ldgate >= a->heads),
+               "gqa: bad chunk, sink, values or gate");
     BH_CHECK_DIMS(a->capacity, a->kv_heads * a->maps, a->dimp);
     BH_CHECK_DIMS(a->capacity, a->kv_heads, a->vdimp);
     return 0;
 }
-size_t gqa_row(const bitnet_hip_gqa *a) { return (a->heads + a->kv_heads) * a->maps * a->dimp + a->kv_heads * a->vdimp; }
+size_t gqa_row(const bitnet_hip_gqa *a) { return (a->heads + a->kv_heads) * a->maps * a->dimp + (a->values_are_keys ? 0 : a->kv_heads * a->vdimp); }
 
 int check_delta(const bitnet_hip_delta *d) {
     BH_REQUIRE(d && d->conv && d->decay_rate && d->dt_bias && d->norm && d->state && d->ring, "delta: null pointer");
@@ -37,10 +41,15 @@ size_t delta_row(const bitnet_hip_delta *d) { return 2 * d->kv_heads * d->dimp +
 
 int check_plan(const bitnet_hip_experts_plan *p) {
     BH_REQUIRE(p && p->counts && p->offsets && p->n_tiles && p->tiles && p->ids && p->slots && p->tokens && p->weights, "experts: no plan");
-    BH_REQUIRE(p->m > 0 && p->experts > 0 && p->experts <= (size_t)kMaxExperts && p->top > 0 && p->top <= (size_t)kMaxTop && p->top <= p->experts &&
-                   (p->tile == 64 || p->tile == 128),
+    BH_REQUIRE(p->m > 0 && p->experts > 0 && p->experts <= (size_t)kMaxExperts && p->top > 0 && p->top <= (size_t)kMaxTop && (p->tile == 64 || p->tile == 128),
                "experts: bad plan");
     BH_CHECK_DIMS(p->m, p->top);
+    return 0;
+}
+int check_router(const bitnet_hip_router *r) {
+    BH_REQUIRE(r && r->experts > 0 && r->experts <= (size_t)kMaxExperts && r->identity <= (size_t)kMaxExperts && r->experts + r->identity <= (size_t)kMaxExperts && r->top > 0 &&
+                   r->top <= (size_t)kMaxTop && r->top <= r->experts + r->identity,
+               "experts: bad router");
     return 0;
 }
 // tiles of a plan at most: every expert's last tile may be short
@@ -52,8 +61,9 @@ extern "C" {
 int bitnet_hip_sum_norm_rows_dev(const bitnet_hip_sum_rows *r, void *stream) {
     BH_GUARD_BEGIN
     BH_REQUIRE(r && r->x && r->m > 0 && r->width > 0 && (!r->y || r->ldy >= r->width), "sum_norm_rows: bad arguments");
-    BH_REQUIRE(!r->h || (r->x2 ? r->ldh >= 2 * r->width : r->weight && r->ldh >= r->width), "sum_norm_rows: bad output");
-    BH_REQUIRE(r->top == 0 || (r->y && r->expert_rows && r->slots && r->slot_weights && r->ld_expert >= r->width), "sum_norm_rows: bad expert rows");
+    BH_REQUIRE(!r->h || (r->ldh >= (r->x2 ? 2 * r->width : r->width)), "sum_norm_rows: bad output");
+    BH_REQUIRE(r->top == 0 || (r->expert_rows && r->slots && r->slot_weights && r->ld_expert >= r->width && (!r->input || r->ld_input >= r->width)),
+               "sum_norm_rows: bad expert rows");
     BH_CHECK_DIMS(r->m, r->width);
     BH_HIP_TRY(launch_sum_norm_rows(*r, (hipStream_t)stream));
     return BITNET_HIP_OK;
@@ -186,7 +196,7 @@ size_t bitnet_hip_experts_plan_bytes(size_t m, size_t experts, size_t top) {
 
 int bitnet_hip_experts_plan_make(void *workspace, size_t bytes, size_t m, size_t experts, size_t top, size_t tile, bitnet_hip_experts_plan *plan) {
     BH_GUARD_BEGIN
-    BH_REQUIRE(workspace && plan && m > 0 && experts > 0 && experts <= (size_t)kMaxExperts && top > 0 && top <= (size_t)kMaxTop && top <= experts,
+    BH_REQUIRE(workspace && plan && m > 0 && experts > 0 && experts <= (size_t)kMaxExperts && top > 0 && top <= (size_t)kMaxTop,
                "experts_plan: %zu of %zu experts (at most %d of %d)", top, experts, kMaxTop, kMaxExperts);
     BH_CHECK_DIMS(m, top);
     BH_REQUIRE((tile == 64 || tile == 128) && bytes >= bitnet_hip_experts_plan_bytes(m, experts, top) && (uintptr_t)workspace % 16 == 0, "experts_plan: bad workspace");
@@ -204,12 +214,13 @@ int bitnet_hip_experts_plan_make(void *workspace, size_t bytes, size_t m, size_t
     BH_GUARD_END
 }
 
-int bitnet_hip_experts_route_dev(const float *logits, size_t ldz, float scale, const bitnet_hip_experts_plan *plan, void *stream) {
+int bitnet_hip_experts_route_dev(const float *logits, size_t ldz, const bitnet_hip_router *router, const bitnet_hip_experts_plan *plan, void *stream) {
     BH_GUARD_BEGIN
     if (int rc = check_plan(plan)) return rc;
-    BH_REQUIRE(logits && ldz >= plan->experts, "experts_route: bad arguments");
+    if (int rc = check_router(router)) return rc;
+    BH_REQUIRE(logits && ldz >= router->experts + router->identity && plan->experts == router->experts && plan->top == router->top, "experts_route: bad arguments");
     BH_CHECK_DIMS(plan->m, ldz);
-    BH_HIP_TRY(launch_experts_route(logits, ldz, scale, *plan, (hipStream_t)stream));
+    BH_HIP_TRY(launch_experts_route(logits, ldz, *router, *plan, (hipStream_t)stream));
     return BITNET_HIP_OK;
     BH_GUARD_END
 }
@@ -218,7 +229,10 @@ int bitnet_hip_experts_matmul_dev(const bitnet_hip_experts_plan *plan, int gathe
                                   size_t ldw, int act, void *c, size_t ldc, int c_f32, void *stream) {
     BH_GUARD_BEGIN
     if (int rc = check_plan(plan)) return rc;
-    BH_REQUIRE(a && w && c && n > 0 && k > 0 && k % 64 == 0 && lda >= k && ldw >= k && lda % 8 == 0 && ldw % 8 == 0 && ldc >= n && act_ok(act) && (a_f32 || !c_f32) &&
+    const int gated = act & BITNET_HIP_ACT_GATED;
+    act &= ~BITNET_HIP_ACT_GATED;
+    BH_REQUIRE(!gated || n % 2 == 0, "experts_matmul: gated columns come in pairs");
+    BH_REQUIRE(a && w && c && n > 0 && k > 0 && k % 64 == 0 && lda >= k && ldw >= k && lda % 8 == 0 && ldw % 8 == 0 && ldc >= (gated ? n / 2 : n) && act_ok(act) && (a_f32 || !c_f32) &&
                    (!a_f32 || plan->tile == 64),
                "experts_matmul: bad arguments");
     BH_CHECK_DIMS(plan->experts, n, ldw);
@@ -228,7 +242,7 @@ int bitnet_hip_experts_matmul_dev(const bitnet_hip_experts_plan *plan, int gathe
     BH_CHECK_DIMS(plan->m * plan->top, lda);
     GemmArgsD g;
     g.a = a, g.w = w, g.c = c, g.m = (int)(plan->m * plan->top), g.n = (int)n, g.k = (int)k, g.lda = lda, g.ldw = ldw, g.ldc = ldc;
-    g.act0 = g.act1 = act, g.a_f32 = a_f32, g.c_f32 = c_f32, g.w_batch = n * ldw;
+    g.act0 = g.act1 = act, g.gated = gated != 0, g.a_f32 = a_f32, g.c_f32 = c_f32, g.w_batch = n * ldw;
     g.tiles = reinterpret_cast<const int4 *>(plan->tiles), g.n_tiles = plan->n_tiles, g.max_tiles = (int)plan->max_tiles, g.tile = (int)plan->tile;
     g.gather = gather ? plan->tokens : nullptr;
     BH_HIP_TRY(launch_dense_gemm(g, (hipStream_t)stream));
@@ -236,32 +250,36 @@ int bitnet_hip_experts_matmul_dev(const bitnet_hip_experts_plan *plan, int gathe
     BH_GUARD_END
 }
 
-int bitnet_hip_experts_up_dev(const float *logits, size_t experts, size_t top, float scale, const float *x, const uint16_t *w, size_t rows, size_t cols, size_t ld,
-                              int act, float *y, size_t ldy, int32_t *ids, void *stream) {
+int bitnet_hip_experts_up_dev(const float *logits, const bitnet_hip_router *router, const float *x, const uint16_t *w, size_t rows, size_t cols, size_t ld, int act,
+                              float *y, size_t ldy, int32_t *ids, float *identity, void *stream) {
     BH_GUARD_BEGIN
-    BH_REQUIRE(logits && x && w && y && ids && experts > 0 && experts <= (size_t)kMaxExperts && top > 0 && top <= (size_t)kMaxTop && top <= experts && rows > 0 &&
-                   cols >= 8 && cols % 8 == 0 && cols <= ld && ld % 8 == 0 && cols <= 32768 && ldy >= rows && act_ok(act),
+    if (int rc = check_router(router)) return rc;
+    const int gated = act & BITNET_HIP_ACT_GATED;
+    act &= ~BITNET_HIP_ACT_GATED;
+    BH_REQUIRE(logits && x && w && y && ids && rows > 0 && cols >= 8 && cols % 8 == 0 && cols <= ld && ld % 8 == 0 && cols <= 32768 && ldy >= (gated ? rows / 2 : rows) &&
+                   act_ok(act) && (!gated || rows % 2 == 0) && (identity || router->identity == 0),
                "experts_up: bad arguments");
-    BH_CHECK_DIMS(experts, rows, ld);
+    BH_CHECK_DIMS(router->experts, rows, ld);
     ExpertsUp a;
-    a.logits = logits, a.experts = (int)experts, a.top = (int)top, a.scale = scale, a.x = x, a.w = w, a.rows = (int)rows, a.cols = (int)cols, a.ld = (int)ld;
-    a.act = act, a.y = y, a.ldy = (int)ldy, a.ids = ids;
+    a.logits = logits, a.r = *router, a.x = x, a.w = w, a.rows = (int)rows, a.cols = (int)cols, a.ld = (int)ld;
+    a.act = act, a.gated = gated != 0, a.y = y, a.ldy = (int)ldy, a.ids = ids, a.identity = identity;
     BH_HIP_TRY(launch_experts_up(a, (hipStream_t)stream));
     return BITNET_HIP_OK;
     BH_GUARD_END
 }
 
 int bitnet_hip_experts_out_dev(const float *x0, const uint16_t *w0, size_t cols0, size_t ld0, const float *bias, const float *x1, size_t ldx1, const uint16_t *w1,
-                               size_t cols1, size_t ld1, const int32_t *ids, size_t top, size_t rows, float *y, void *stream) {
+                               size_t cols1, size_t ld1, const int32_t *ids, size_t top, size_t rows, const float *identity, const float *input, float *y, void *stream) {
     BH_GUARD_BEGIN
-    BH_REQUIRE(x0 && w0 && x1 && w1 && ids && y && top > 0 && top <= (size_t)kMaxTop && rows > 0 && cols0 >= 8 && cols0 % 8 == 0 && cols0 <= ld0 && ld0 % 8 == 0 &&
-                   cols1 >= 8 && cols1 % 8 == 0 && cols1 <= ld1 && ld1 % 8 == 0 && ldx1 >= cols1,
+    if (!x0) w0 = nullptr, cols0 = ld0 = 0;
+    BH_REQUIRE((!x0 || (w0 && cols0 >= 8)) && x1 && w1 && ids && y && top > 0 && top <= (size_t)kMaxTop && rows > 0 && cols0 % 8 == 0 && cols0 <= ld0 && ld0 % 8 == 0 &&
+                   (!identity || input) && cols1 >= 8 && cols1 % 8 == 0 && cols1 <= ld1 && ld1 % 8 == 0 && ldx1 >= cols1,
                "experts_out: bad arguments");
     BH_CHECK_DIMS(rows, ld0);
     BH_CHECK_DIMS(rows, ld1);
     ExpertsOut a;
     a.x0 = x0, a.x1 = x1, a.bias = bias, a.w0 = w0, a.w1 = w1, a.cols0 = (int)cols0, a.ld0 = (int)ld0, a.cols1 = (int)cols1, a.ld1 = (int)ld1, a.ldx1 = (int)ldx1;
-    a.top = (int)top, a.rows = (int)rows, a.ids = ids, a.y = y;
+    a.top = (int)top, a.rows = (int)rows, a.ids = ids, a.identity = identity, a.input = input, a.y = y;
     const hipError_t e = launch_experts_out(a, (hipStream_t)stream);
     if (e == hipErrorInvalidValue) return set_error(BITNET_HIP_ERR_UNSUPPORTED, "experts_out: %zu + %zu x %zu columns do not fit a workgroup's memory", cols0, top, cols1);
     BH_HIP_TRY(e);

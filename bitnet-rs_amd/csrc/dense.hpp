@@ -41,6 +41,7 @@ struct GemvArgs {
     size_t w_batch = 0, x_batch = 0, y_batch = 0;  // elements between consecutive batch members
     const float *bias = nullptr;
     int act0 = 0, act1 = 0, act_split = 0;         // rows < act_split take act0, the others act1
+    int gated = 0;                                 // rows 2 i and 2 i + 1 make element i: act0(row 2 i) * row 2 i + 1
     float *y = nullptr;
     float *best_val = nullptr;                     // argmax partial per workgroup (batch 1)
     int *best_idx = nullptr;
@@ -56,6 +57,7 @@ struct GemmArgsD {
     int m = 0, n = 0, k = 0;   // k: multiple of 64, <= lda and ldw
     size_t lda = 0, ldw = 0, ldc = 0;
     int act0 = 0, act1 = 0, act_split = 0;
+    int gated = 0;             // columns 2 i and 2 i + 1 make column i of c: act0(column 2 i) * column 2 i + 1 (n: columns ahead of that)
     int a_f32 = 0, c_f32 = 0;
     int batch = 1;
     size_t a_batch = 0, w_batch = 0, c_batch = 0;
@@ -70,6 +72,7 @@ typedef bitnet_hip_sum_rows SumRows;
 typedef bitnet_hip_gqa Gqa;
 typedef bitnet_hip_delta Delta;
 typedef bitnet_hip_experts_plan ExpertsPlan;
+typedef bitnet_hip_router Router;
 
 struct GqaStep {
     const float *row = nullptr;    // raw projections of the token
@@ -79,14 +82,15 @@ struct GqaStep {
 
 struct ExpertsUp {
     const float *logits = nullptr;
-    int experts = 0, top = 0;
-    float scale = 1.f;
+    Router r;
     const float *x = nullptr;
     const uint16_t *w = nullptr;
     int rows = 0, cols = 0, ld = 0, act = 0;
+    int gated = 0;                 // rows 2 i and 2 i + 1 make column i
     float *y = nullptr;
     int ldy = 0;
     int *ids = nullptr;
+    float *identity = nullptr;
 };
 
 struct ExpertsOut {
@@ -94,6 +98,7 @@ struct ExpertsOut {
     const uint16_t *w0 = nullptr, *w1 = nullptr;
     int cols0 = 0, ld0 = 0, cols1 = 0, ld1 = 0, ldx1 = 0, top = 0, rows = 0;
     const int *ids = nullptr;
+    const float *identity = nullptr, *input = nullptr;
     float *y = nullptr;
 };
 
@@ -171,8 +176,8 @@ constexpr int kDeltaChunk = 64;    // tokens per chunk of the delta rule
 constexpr int kDeltaUnits = 512;   // chunks x heads per pass over the workspace: one round of workgroups, and small enough to stay in the caches
 constexpr int kMaxExperts = 1024, kMaxTop = 32;
 
-hipError_t launch_embed_bf16(const uint16_t *table, size_t ld, const int *tokens, const int *offset, int n, int width, int vocab, float scale, float *out,
-                             hipStream_t s);
+hipError_t launch_embed_bf16(const uint16_t *table, size_t ld, const int *tokens, const int *offset, int n, int width, int vocab, float scale,
+                             const float *norm_w, float eps, float *out, hipStream_t s);
 hipError_t launch_sum_norm_rows(const SumRows &a, hipStream_t s);
 hipError_t launch_residual_norm_rows(float *x, const float *y, size_t ldy, const float *post_w, const float *scale, const float *next_w,
                                      float offset, float eps, int m, int width, void *h, size_t ldh, int h_f32, hipStream_t s);
@@ -209,7 +214,7 @@ hipError_t launch_delta_recurrent(const Delta &d, const float *qk, const void *v
                                   void *out, size_t ldo, hipStream_t s);
 hipError_t launch_delta_chunked(const Delta &d, const float *qk, const uint16_t *v, const float *gates, const uint16_t *rows, size_t ld, int n,
                                 uint16_t *out, size_t ldo, void *workspace, hipStream_t s);
-hipError_t launch_experts_route(const float *logits, size_t ldz, float scale, const ExpertsPlan &p, hipStream_t s);
+hipError_t launch_experts_route(const float *logits, size_t ldz, const Router &r, const ExpertsPlan &p, hipStream_t s);
 hipError_t launch_experts_up(const ExpertsUp &a, hipStream_t s);
 hipError_t launch_experts_out(const ExpertsOut &a, hipStream_t s);
 
@@ -275,6 +280,7 @@ __device__ __forceinline__ float group_sum(float v, float *slot) {
     return t;
 }
 
+__device__ __forceinline__ float gelu_argument(float v) { return 0.7978845608028654f * (v + 0.044715f * v * v * v); }  // sqrt(2 / pi)
 // BITNET_HIP_ACT_*
 __device__ __forceinline__ float activate(float v, int act) {
     switch (act) {
@@ -284,6 +290,7 @@ __device__ __forceinline__ float activate(float v, int act) {
             const float r = fmaxf(v, 0.0f);
             return r * r;
         }
+        case BITNET_HIP_ACT_GELU_TANH: return v / (1.0f + expf(-2.0f * gelu_argument(v)));  // (1 + tanh z) / 2 = 1 / (1 + exp(-2 z))
         default: return v;
     }
 }

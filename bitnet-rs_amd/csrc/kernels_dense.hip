@@ -11,15 +11,27 @@ namespace bitnet_hip {
 
 // ---- embedding rows ---------------------------------------------------------------------------------------------------
 __global__ void k_embed_bf16(const uint16_t *__restrict__ table, size_t ld, const int *__restrict__ tokens, const int *__restrict__ offset,
-                             int width, int vocab, float scale, float *__restrict__ out) {
+                             int width, int vocab, float scale, const float *__restrict__ norm_w, float eps, float *__restrict__ out) {
+    __shared__ float slot[4];
     int tok = tokens[(offset ? *offset : 0) + blockIdx.x];
     tok = tok < 0 ? 0 : (tok >= vocab ? vocab - 1 : tok);
+    if (norm_w) {
+        const uint16_t *row = table + (size_t)tok * ld;
+        float ss = 0.f;
+        for (int i = threadIdx.x; i < width; i += 256) {
+            const float v = scale * bf2f(row[i]);
+            ss += v * v;
+        }
+        const float inv = 1.0f / sqrtf(group_sum<4>(ss, slot) / (float)width + eps);
+        for (int i = threadIdx.x; i < width; i += 256) out[(size_t)blockIdx.x * width + i] = scale * bf2f(row[i]) * inv * norm_w[i];
+        return;
+    }
     for (int i = threadIdx.x; i < width; i += blockDim.x) out[(size_t)blockIdx.x * width + i] = scale * bf2f(table[(size_t)tok * ld + i]);
 }
 
-hipError_t launch_embed_bf16(const uint16_t *table, size_t ld, const int *tokens, const int *offset, int n, int width, int vocab, float scale, float *out,
-                             hipStream_t s) {
-    hipLaunchKernelGGL(k_embed_bf16, dim3(n), dim3(256), 0, s, table, ld, tokens, offset, width, vocab, scale, out);
+hipError_t launch_embed_bf16(const uint16_t *table, size_t ld, const int *tokens, const int *offset, int n, int width, int vocab, float scale,
+                             const float *norm_w, float eps, float *out, hipStream_t s) {
+    hipLaunchKernelGGL(k_embed_bf16, dim3(n), dim3(256), 0, s, table, ld, tokens, offset, width, vocab, scale, norm_w, eps, out);
     return hipGetLastError();
 }
 
@@ -34,7 +46,7 @@ hipError_t launch_gather_rows(const float *x, const int *rows, int n, int width,
 }
 
 // ---- residual + norm rows ---------------------------------------------------------------------------------------------
-// x += scale * norm(y; post_w); h = norm(x; next_w).  One workgroup per row; rows of up to 4096 columns stay in registers.
+// x += scale * norm(y; post_w); h = norm(x; next_w), or x itself without next_w.  One workgroup per row; rows of up to 4096 columns stay in registers.
 constexpr int kRowRegs = 16;
 
 template <class TH>
@@ -85,8 +97,19 @@ __global__ __launch_bounds__(256) void k_residual_norm_rows(float *__restrict__ 
     } else {
         for (int i = tid; i < width; i += 256) ss += xr[i] * xr[i];
     }
-    const float inv = 1.0f / sqrtf(group_sum<4>(ss, slot) / (float)width + eps);
     TH *hr = h + (size_t)blockIdx.x * ldh;
+    if (!next_w) {
+        if (regs) {
+#pragma unroll
+            for (int j = 0; j < kRowRegs; ++j)
+                if (tid + 256 * j < width) st_act(hr, tid + 256 * j, xv[j]);
+        } else {
+            for (int i = tid; i < width; i += 256) st_act(hr, i, xr[i]);
+        }
+        for (int i = width + tid; i < (int)ldh; i += 256) st_act(hr, i, 0.f);
+        return;
+    }
+    const float inv = 1.0f / sqrtf(group_sum<4>(ss, slot) / (float)width + eps);
     if (regs) {
 #pragma unroll
         for (int j = 0; j < kRowRegs; ++j) {
@@ -108,7 +131,7 @@ hipError_t launch_residual_norm_rows(float *x, const float *y, size_t ldy, const
     return hipGetLastError();
 }
 
-// Rows of a block whose sublayers add up: x += mult * (y + the chosen experts' rows); h = norm(x) or [x; x2].  Four columns at a time, rows of up to
+// Rows of a block whose sublayers add up: t = y + the chosen experts' rows, x += mult * t or scale * norm(t); h = norm(x), x or [x; x2].  Four columns at a time, rows of up to
 // 4096 columns in registers.
 __device__ __forceinline__ f32x4 ld4(const float *p, size_t i) { return *reinterpret_cast<const f32x4 *>(p + i); }
 __device__ __forceinline__ f32x4 ld4(const uint16_t *p, size_t i) {
@@ -132,6 +155,8 @@ __global__ __launch_bounds__(256) void k_sum_norm_rows(SumRows p) {
     const int *slots = p.slots + (size_t)blockIdx.x * p.top;
     const float *sw = p.slot_weights + (size_t)blockIdx.x * p.top;
     const float *x2 = p.x2 ? p.x2 + (size_t)blockIdx.x * width : nullptr;
+    const T *input = p.input ? (const T *)p.input + (size_t)blockIdx.x * p.ld_input : nullptr;  // (may be h: a thread reads its columns ahead of writing them)
+    const int top = (int)p.top;
     if (VEC) {
         f32x4 v[kSumRegs];
         const int n4 = width >> 2;
@@ -141,27 +166,50 @@ __global__ __launch_bounds__(256) void k_sum_norm_rows(SumRows p) {
             v[j] = f32x4{0.f, 0.f, 0.f, 0.f};
             if (i < n4) v[j] = ld4(x, 4 * i);
         }
-        if (y) {
+        if (y || top) {
             f32x4 a[kSumRegs];
 #pragma unroll
             for (int j = 0; j < kSumRegs; ++j) {
                 const int i = tid + 256 * j;
-                if (i < n4) a[j] = ld4(y, 4 * i);
+                a[j] = f32x4{0.f, 0.f, 0.f, 0.f};
+                if (y && i < n4) a[j] = ld4(y, 4 * i);
             }
-            for (int k = 0; k < (int)p.top; ++k) {
-                const T *row = er + (size_t)slots[k] * p.ld_expert;
+            for (int k = 0; k < top; ++k) {
+                const int slot_k = slots[k];
                 const float w = sw[k];
+                if (slot_k < 0) {
+#pragma unroll
+                    for (int j = 0; j < kSumRegs; ++j) {
+                        const int i = tid + 256 * j;
+                        if (i < n4) a[j] += w * (input ? ld4(input, 4 * i) : v[j]);
+                    }
+                    continue;
+                }
+                const T *row = er + (size_t)slot_k * p.ld_expert;
 #pragma unroll
                 for (int j = 0; j < kSumRegs; ++j) {
                     const int i = tid + 256 * j;
                     if (i < n4) a[j] += w * ld4(row, 4 * i);
                 }
             }
+            float post = 0.f;
+            if (p.post_weight) {
+                float ss = 0.f;
+#pragma unroll
+                for (int j = 0; j < kSumRegs; ++j) ss += (a[j].x * a[j].x + a[j].y * a[j].y) + (a[j].z * a[j].z + a[j].w * a[j].w);
+                post = 1.0f / sqrtf(group_sum<4>(ss, slot) / (float)width + p.eps);
+            }
 #pragma unroll
             for (int j = 0; j < kSumRegs; ++j) {
                 const int i = tid + 256 * j;
                 if (i < n4) {
-                    v[j] += p.mult * a[j];
+                    if (p.post_weight) {
+                        f32x4 r = a[j] * post * (p.weight_offset + ld4(p.post_weight, 4 * i));
+                        if (p.scale) r *= ld4(p.scale, 4 * i);
+                        v[j] += r;
+                    } else {
+                        v[j] += p.mult * a[j];
+                    }
                     st4(x, 4 * i, v[j]);
                 }
             }
@@ -176,6 +224,10 @@ __global__ __launch_bounds__(256) void k_sum_norm_rows(SumRows p) {
                     st4(h, width + 4 * i, ld4(x2, 4 * i));
                 }
             }
+        } else if (!p.weight) {
+#pragma unroll
+            for (int j = 0; j < kSumRegs; ++j)
+                if (tid + 256 * j < n4) st4(h, 4 * (tid + 256 * j), v[j]);
         } else {
             float mean = 0.f, ss = 0.f;
             if (p.center) {
@@ -201,18 +253,32 @@ __global__ __launch_bounds__(256) void k_sum_norm_rows(SumRows p) {
             }
         }
     } else {  // (a thread comes back to its own columns only)
-        if (y)
-            for (int i = tid; i < width; i += 256) {
-                float a = y[i];
-                for (int k = 0; k < (int)p.top; ++k) a += sw[k] * ld_act(er + (size_t)slots[k] * p.ld_expert, i);
-                x[i] += p.mult * a;
+        if (y || top) {
+            auto sum = [&](int i) {
+                float a = y ? y[i] : 0.f;
+                for (int k = 0; k < top; ++k) a += sw[k] * (slots[k] >= 0 ? ld_act(er + (size_t)slots[k] * p.ld_expert, i) : input ? ld_act(input, i) : x[i]);
+                return a;
+            };
+            float post = 0.f;
+            if (p.post_weight) {
+                float ss = 0.f;
+                for (int i = tid; i < width; i += 256) {
+                    const float a = sum(i);
+                    ss += a * a;
+                }
+                post = 1.0f / sqrtf(group_sum<4>(ss, slot) / (float)width + p.eps);
             }
+            for (int i = tid; i < width; i += 256)
+                x[i] += p.post_weight ? (p.scale ? p.scale[i] : 1.0f) * (sum(i) * post * (p.weight_offset + p.post_weight[i])) : p.mult * sum(i);
+        }
         if (!h) return;
         if (x2) {
             for (int i = tid; i < width; i += 256) {
                 st_act(h, i, x[i]);
                 st_act(h, width + i, x2[i]);
             }
+        } else if (!p.weight) {
+            for (int i = tid; i < width; i += 256) st_act(h, i, x[i]);
         } else {
             float mean = 0.f, ss = 0.f;
             if (p.center) {
@@ -230,7 +296,7 @@ __global__ __launch_bounds__(256) void k_sum_norm_rows(SumRows p) {
 
 hipError_t launch_sum_norm_rows(const SumRows &a, hipStream_t s) {
     // (four columns at a time: every row of every operand starts on its own alignment)
-    const bool vec = a.width % 4 == 0 && a.width <= 1024 * kSumRegs && a.ldy % 4 == 0 && a.ld_expert % 4 == 0 && a.ldh % 4 == 0;
+    const bool vec = a.width % 4 == 0 && a.width <= 1024 * kSumRegs && a.ldy % 4 == 0 && a.ld_expert % 4 == 0 && a.ldh % 4 == 0 && a.ld_input % 4 == 0;
     auto fn = a.h_f32 ? (vec ? k_sum_norm_rows<float, true> : k_sum_norm_rows<float, false>) : (vec ? k_sum_norm_rows<uint16_t, true> : k_sum_norm_rows<uint16_t, false>);
     hipLaunchKernelGGL(fn, dim3(a.m), dim3(256), 0, s, a);
     return hipGetLastError();
@@ -395,15 +461,16 @@ __device__ void form_input(const VecIn &in, const float *x, int cols, int kp, fl
                 if (writer && in.x_out) reinterpret_cast<f32x4 *>(in.x_out)[i] = xv[j];
             }
         }
-        if (in.kind == BITNET_HIP_IN_CONCAT) {
+        if (in.kind >= BITNET_HIP_IN_CONCAT) {
+            const bool two = in.kind == BITNET_HIP_IN_CONCAT;
 #pragma unroll
             for (int j = 0; j < NR; ++j) {
                 const int i = tid + 256 * j;
                 if (i >= n4) continue;
                 reinterpret_cast<f32x4 *>(xs)[i] = xv[j];
-                reinterpret_cast<f32x4 *>(xs)[n4 + i] = reinterpret_cast<const f32x4 *>(in.x2)[i];
+                if (two) reinterpret_cast<f32x4 *>(xs)[n4 + i] = reinterpret_cast<const f32x4 *>(in.x2)[i];
             }
-            for (int i = 2 * n + tid; i < kp; i += 256) xs[i] = 0.f;
+            for (int i = (two ? 2 : 1) * n + tid; i < kp; i += 256) xs[i] = 0.f;
             __syncthreads();
             return;
         }
@@ -469,9 +536,10 @@ __device__ void form_input(const VecIn &in, const float *x, int cols, int kp, fl
                 ss += x[i] * x[i];
             }
         }
-        if (in.kind == BITNET_HIP_IN_CONCAT) {
-            for (int i = tid; i < n; i += 256) xs[n + i] = in.x2[i];
-            for (int i = 2 * n + tid; i < kp; i += 256) xs[i] = 0.f;
+        if (in.kind >= BITNET_HIP_IN_CONCAT) {
+            const bool two = in.kind == BITNET_HIP_IN_CONCAT;
+            for (int i = tid; two && i < n; i += 256) xs[n + i] = in.x2[i];
+            for (int i = (two ? 2 : 1) * n + tid; i < kp; i += 256) xs[i] = 0.f;
             __syncthreads();
             return;
         }
@@ -578,7 +646,16 @@ __global__ __launch_bounds__(256) void k_dense_gemv(GemvK p) {
             }
             if (LPR == 64) acc[r] = rows_sum(acc[r]);
         }
-        if (l == 0) {
+        if (R > 1 && a.gated) {
+            if (l == 0)
+#pragma unroll
+                for (int r = 0; r + 1 < R; r += 2) {
+                    const int row = row0 + r;  // (even, and so is the number of rows)
+                    if (row >= a.rows) continue;
+                    const float b0 = a.bias ? a.bias[row] : 0.f, b1 = a.bias ? a.bias[row + 1] : 0.f;
+                    a.y[(size_t)b * a.y_batch + (row >> 1)] = activate(acc[r] + b0, a.act0) * (acc[r + 1] + b1);
+                }
+        } else if (l == 0) {
 #pragma unroll
             for (int r = 0; r < R; ++r) {
                 const int row = row0 + r;
@@ -654,7 +731,7 @@ hipError_t launch_dense_gemv(const GemvArgs &a, int *n_wg_out, hipStream_t s) {
     auto wgs = [&](int r) { return ((long)a.rows + 4l * per * r - 1) / (4l * per * r) * a.batch; };
     int r = 1;
     if (wgs(4) >= 1024) r = 4;
-    else if (wgs(2) >= 512) r = 2;
+    else if (wgs(2) >= 512 || a.gated) r = 2;
     k.groups = (a.rows + per * r - 1) / (per * r);
     int n_wg = (k.groups + 3) / 4;
     const int cap = 768;  // three workgroups per CU: each forms the whole input again (measured: 512 and 1024 are slower)
@@ -702,7 +779,8 @@ __device__ __forceinline__ int weight_key(int row) {
 }
 
 // GROUPED: the row tiles come from a device list, (matrix, first row, rows) each; a matrix's tiles follow one another.
-template <int TN, int TM, int WN, int WM, int ST, bool CF32, bool GROUPED = false>
+// GATED (bf16 outputs): columns 2 i and 2 i + 1 make column i of the output.
+template <int TN, int TM, int WN, int WM, int ST, bool CF32, bool GROUPED = false, bool GATED = false>
 __global__ __launch_bounds__(64 * WN * WM, 2) void k_dense_gemm(GemmArgsD p, int tiles_n, int tiles_m, int swizzle) {
     extern __shared__ __attribute__((aligned(1024))) uint8_t lds[];
     constexpr int NW = WN * WM, DN = TN / NW / 8, DM = TM / NW / 8;  // DMA instructions per wave and step (eight rows each)
@@ -826,6 +904,29 @@ __global__ __launch_bounds__(64 * WN * WM, 2) void k_dense_gemm(GemmArgsD p, int
             for (int i = 0; i < FN; ++i)
 #pragma unroll
                 for (int e = 0; e < 4; ++e) acc[i][j][e] += p.bias[min(nl + i * FS + e, p.n - 1)];
+        if (GATED) {
+            float r[2 * FN];
+#pragma unroll
+            for (int i = 0; i < FN; ++i)
+#pragma unroll
+                for (int e = 0; e < 4; e += 2) {
+                    const float v = acc[i][j][e], z = p.act0 == BITNET_HIP_ACT_GELU_TANH ? 2.0f * gelu_argument(v) : v;
+                    const float sg = __builtin_amdgcn_rcpf(1.0f + __expf(-z));
+                    r[2 * i + e / 2] = (p.act0 == BITNET_HIP_ACT_SILU || p.act0 == BITNET_HIP_ACT_GELU_TANH ? v * sg : activate(v, p.act0)) * acc[i][j][e + 1];
+                }
+            uint16_t *dst = (uint16_t *)p.c + (size_t)blockIdx.y * p.c_batch + (size_t)m * p.ldc + nl / 2;
+#pragma unroll
+            for (int i = 0; i < 2 * FN; i += 4) {
+                if (vec && nl + 2 * i + 7 < p.n) {
+                    *reinterpret_cast<bf16x4 *>(dst + i) = bf16x4{(__bf16)r[i], (__bf16)r[i + 1], (__bf16)r[i + 2], (__bf16)r[i + 3]};
+                } else {
+#pragma unroll
+                    for (int e = 0; e < 4; ++e)
+                        if (nl + 2 * (i + e) < p.n) dst[i + e] = f2bf(r[i + e]);
+                }
+            }
+            continue;
+        }
         auto apply = [&](auto f) {
 #pragma unroll
             for (int i = 0; i < FN; ++i)
@@ -836,7 +937,7 @@ __global__ __launch_bounds__(64 * WN * WM, 2) void k_dense_gemm(GemmArgsD p, int
             apply([&](float v, int n) {
                 const int f = n < p.act_split ? p.act0 : p.act1;
                 const float sg = __builtin_amdgcn_rcpf(1.0f + __expf(-v)), r = fmaxf(v, 0.0f);
-                return f == BITNET_HIP_ACT_SILU ? v * sg : f == BITNET_HIP_ACT_SIGMOID ? sg : f == BITNET_HIP_ACT_RELU2 ? r * r : v;
+                return f == BITNET_HIP_ACT_SILU ? v * sg : f == BITNET_HIP_ACT_SIGMOID ? sg : f == BITNET_HIP_ACT_RELU2 ? r * r : activate(v, f);
             });
         else if (act == BITNET_HIP_ACT_SILU)
             apply([](float v, int) { return v * __builtin_amdgcn_rcpf(1.0f + __expf(-v)); });
@@ -844,6 +945,8 @@ __global__ __launch_bounds__(64 * WN * WM, 2) void k_dense_gemm(GemmArgsD p, int
             apply([](float v, int) { return __builtin_amdgcn_rcpf(1.0f + __expf(-v)); });
         else if (act == BITNET_HIP_ACT_RELU2)
             apply([](float v, int) { return activate(v, BITNET_HIP_ACT_RELU2); });
+        else if (act == BITNET_HIP_ACT_GELU_TANH)
+            apply([](float v, int) { return v * __builtin_amdgcn_rcpf(1.0f + __expf(-2.0f * gelu_argument(v))); });
         if (CF32) {
 #pragma unroll
             for (int i = 0; i < FN; ++i) {
@@ -878,7 +981,7 @@ template <int T, int ST>
 static hipError_t grouped_go(const GemmArgsD &a, hipStream_t s) {
     const int tn = (a.n + T - 1) / T;
     constexpr size_t lds = (size_t)ST * T * 256;
-    auto fn = k_dense_gemm<T, T, 2, 2, ST, false, true>;
+    auto fn = a.gated ? k_dense_gemm<T, T, 2, 2, ST, false, true, true> : k_dense_gemm<T, T, 2, 2, ST, false, true>;
     if (lds > 65536) {
         const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(fn), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
         if (e != hipSuccess) return e;
@@ -891,7 +994,9 @@ template <int T, int WN, int WM, int ST>
 static hipError_t gemm_go(const GemmArgsD &a, hipStream_t s) {
     const int tn = (a.n + T - 1) / T, tm = (a.m + T - 1) / T, swz = (tn * tm) % 8 == 0 ? 1 : 0;
     constexpr size_t lds = (size_t)ST * T * 256;
-    auto fn = a.c_f32 ? k_dense_gemm<T, T, WN, WM, ST, true> : k_dense_gemm<T, T, WN, WM, ST, false>;
+    auto fn = a.gated   ? k_dense_gemm<T, T, WN, WM, ST, false, false, true>
+              : a.c_f32 ? k_dense_gemm<T, T, WN, WM, ST, true>
+                        : k_dense_gemm<T, T, WN, WM, ST, false>;
     if (lds > 65536) {
         const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(fn), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
         if (e != hipSuccess) return e;
@@ -944,8 +1049,13 @@ __global__ __launch_bounds__(256) void k_dense_gemm_f32(GemmArgsD p) {
         for (int j = 0; j < 4; ++j) {
             const int n = n0 + tx * 4 + j;
             if (n >= p.n) break;
-            const float v = activate(acc[i][j] + (p.bias ? p.bias[n] : 0.f), n < p.act_split ? p.act0 : p.act1);
-            const size_t o = (size_t)blockIdx.z * p.c_batch + (size_t)m * p.ldc + n;
+            if (p.gated && (j & 1)) continue;
+            float v = activate(acc[i][j] + (p.bias ? p.bias[n] : 0.f), n < p.act_split ? p.act0 : p.act1);
+            size_t o = (size_t)blockIdx.z * p.c_batch + (size_t)m * p.ldc + n;
+            if (p.gated) {  // (n is even here, and so is the number of columns)
+                v *= acc[i][j < 3 ? j + 1 : 3] + (p.bias ? p.bias[n + 1] : 0.f);
+                o -= n / 2;
+            }
             if (p.c_f32)
                 ((float *)p.c)[o] = v;
             else
@@ -958,6 +1068,7 @@ hipError_t launch_dense_gemm(const GemmArgsD &args, hipStream_t s) {
     GemmArgsD a = args;
     if (a.m <= 0 || a.n <= 0) return hipSuccess;
     if (a.act_split == 0) a.act_split = a.n;
+    if (a.gated && !a.a_f32 && a.c_f32) return hipErrorInvalidValue;
     if (a.tiles) {
         if (a.a_f32) {
             if (a.tile != 64) return hipErrorInvalidValue;

@@ -28,7 +28,8 @@ __device__ __forceinline__ void choose_load(const float *z, int experts, float (
 }
 
 template <int LT, int PL>
-__device__ __forceinline__ void choose(float (&s)[PL], int experts, int top, float scale, int &id, float &weight) {
+__device__ __forceinline__ void choose(float (&s)[PL], const Router &r, int &id, float &weight) {
+    const int experts = (int)(r.experts + r.identity), top = (int)r.top;
     const int lane = threadIdx.x & 63, l = lane & (LT - 1), base = lane & ~(LT - 1);
     float m = -INFINITY, sum = 0.f;
 #pragma unroll
@@ -41,53 +42,60 @@ __device__ __forceinline__ void choose(float (&s)[PL], int experts, int top, flo
     }
     sum = token_sum<LT>(sum);
 #pragma unroll
-    for (int j = 0; j < PL; ++j) s[j] = l * PL + j < experts ? s[j] / sum : -1.0f;  // (-1: not there, or taken)
+    for (int j = 0; j < PL; ++j) s[j] = l * PL + j < experts ? s[j] / sum : -INFINITY;  // (-infinity: not there, or taken)
+    float score[PL];  // without the correction
+#pragma unroll
+    for (int j = 0; j < PL; ++j) {
+        score[j] = s[j];
+        if (r.correction) s[j] += r.correction[min(l * PL + j, experts - 1)];
+    }
     id = 0, weight = 0.f;
     float chosen = 0.f;
     for (int k = 0; k < top; ++k) {
-        float best = -1.0f;
+        float best = -INFINITY, mine_w = 0.f;
         int at = 0;
 #pragma unroll
         for (int j = 0; j < PL; ++j)
-            if (s[j] > best) best = s[j], at = j;
-        const float w = token_max<LT>(best);
+            if (s[j] > best) best = s[j], mine_w = score[j], at = j;
+        float w = token_max<LT>(best);
         unsigned long long who = __ballot(best == w) >> base;
         if (LT < 64) who &= (1ull << LT) - 1;
         const int winner = who ? __builtin_ctzll(who) : 0;  // (no score compares equal to itself if a logit is not a number)
         const int mine = l * PL + at;
         const int e = min(LT == 64 ? __builtin_amdgcn_readlane(mine, winner) : __shfl(mine, base + winner, 64), experts - 1);
+        if (r.correction) w = __shfl(mine_w, base + winner, 64);
         if (l == k) id = e, weight = w;
         chosen += w;
         if (l == winner)
 #pragma unroll
             for (int j = 0; j < PL; ++j)
-                if (j == at) s[j] = -1.0f;
+                if (j == at) s[j] = -INFINITY;
     }
-    weight = weight / (chosen + 1e-20f) * scale;
+    weight = (r.raw ? weight : weight / (chosen + 1e-20f)) * r.scale;
 }
 
 // ---- a prompt's choices -----------------------------------------------------------------------------------------------
 constexpr int kRouteTokens = 32;  // per workgroup; its choices are counted in LDS first
 
 template <int LT, int PL>
-__global__ __launch_bounds__(256) void k_route(const float *__restrict__ z, size_t ldz, float scale, ExpertsPlan p) {
+__global__ __launch_bounds__(256) void k_route(const float *__restrict__ z, size_t ldz, Router r, ExpertsPlan p) {
     __shared__ int hist[kMaxExperts];
-    const int tid = threadIdx.x, grp = tid / LT, l = tid & (LT - 1), experts = (int)p.experts, top = (int)p.top, m = (int)p.m;
+    const int tid = threadIdx.x, grp = tid / LT, l = tid & (LT - 1), experts = (int)p.experts, outputs = (int)(r.experts + r.identity), top = (int)p.top, m = (int)p.m;
     constexpr int PER = kRouteTokens * LT / 256;  // (top <= LT)
     const int t0 = blockIdx.x * kRouteTokens + grp * PER;
     float s[PER][PL];
 #pragma unroll
-    for (int i = 0; i < PER; ++i) choose_load<LT, PL>(z + (size_t)min(t0 + i, m - 1) * ldz, experts, s[i]);
+    for (int i = 0; i < PER; ++i) choose_load<LT, PL>(z + (size_t)min(t0 + i, m - 1) * ldz, outputs, s[i]);
     for (int e = tid; e < experts; e += 256) hist[e] = 0;
     __syncthreads();
     int id[PER], rank[PER];
 #pragma unroll
     for (int i = 0; i < PER; ++i) {
         float w;
-        choose<LT, PL>(s[i], experts, top, scale, id[i], w);
+        choose<LT, PL>(s[i], r, id[i], w);
         rank[i] = 0;
         if (t0 + i < m && l < top) {
-            rank[i] = atomicAdd(&hist[id[i]], 1);
+            if (id[i] < experts) rank[i] = atomicAdd(&hist[id[i]], 1);
             p.ids[(size_t)(t0 + i) * top + l] = id[i];
             p.weights[(size_t)(t0 + i) * top + l] = w;
         }
@@ -100,7 +108,7 @@ __global__ __launch_bounds__(256) void k_route(const float *__restrict__ z, size
     __syncthreads();
 #pragma unroll
     for (int i = 0; i < PER; ++i)
-        if (t0 + i < m && l < top) p.slots[(size_t)(t0 + i) * top + l] = rank[i] + hist[id[i]];  // within its expert so far
+        if (t0 + i < m && l < top) p.slots[(size_t)(t0 + i) * top + l] = id[i] < experts ? rank[i] + hist[id[i]] : -1;  // within its expert so far
 }
 
 // first slot and tiles of every expert; the counts are left at zero for the next portion
@@ -129,16 +137,17 @@ __global__ __launch_bounds__(1024) void k_route_tiles(ExpertsPlan p) {
 __global__ __launch_bounds__(256) void k_route_slots(ExpertsPlan p) {
     const int i = blockIdx.x * 256 + threadIdx.x;
     if (i >= (int)(p.m * p.top)) return;
+    if (p.ids[i] >= (int)p.experts) return;  // (an identity expert)
     const int s = p.offsets[p.ids[i]] + p.slots[i];
     p.slots[i] = s;
     p.tokens[s] = i / (int)p.top;
 }
 
-hipError_t launch_experts_route(const float *logits, size_t ldz, float scale, const ExpertsPlan &p, hipStream_t s) {
+hipError_t launch_experts_route(const float *logits, size_t ldz, const Router &r, const ExpertsPlan &p, hipStream_t s) {
     const bool row = p.top <= 16;  // sixteen lanes per token
-    const int e = (int)p.experts;
+    const int e = (int)(r.experts + r.identity);
     auto fn = row && e <= 16 ? k_route<16, 1> : row && e <= 64 ? k_route<16, 4> : row && e <= 128 ? k_route<16, 8> : e <= 256 ? k_route<64, 4> : k_route<64, 16>;
-    hipLaunchKernelGGL(fn, dim3((p.m + kRouteTokens - 1) / kRouteTokens), dim3(256), 0, s, logits, ldz, scale, p);
+    hipLaunchKernelGGL(fn, dim3((p.m + kRouteTokens - 1) / kRouteTokens), dim3(256), 0, s, logits, ldz, r, p);
     hipLaunchKernelGGL(k_route_tiles, dim3(1), dim3(1024), 0, s, p);
     hipLaunchKernelGGL(k_route_slots, dim3((p.m * p.top + 255) / 256), dim3(256), 0, s, p);
     return hipGetLastError();
@@ -188,7 +197,7 @@ __global__ __launch_bounds__(256) void k_experts_up(UpK p) {
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, b = blockIdx.y, sub = lane / LPR, l = lane % LPR;
     constexpr int G = 64 / LPR, CH = LPR * 8;
     float z[PL];
-    choose_load<64, PL>(a.logits, a.experts, z);
+    choose_load<64, PL>(a.logits, (int)(a.r.experts + a.r.identity), z);
     f32x4 xv[kStage];
     auto load = [&](int i0) {
 #pragma unroll
@@ -204,10 +213,28 @@ __global__ __launch_bounds__(256) void k_experts_up(UpK p) {
     load(tid);
     int mine;
     float weight;
-    choose<64, PL>(z, a.experts, a.top, a.scale, mine, weight);
-    if (blockIdx.x == 0 && b == 0 && wave == 0 && lane < a.top) a.ids[lane] = mine;
-    const int e = __builtin_amdgcn_readlane(mine, b);
-    const float scale = __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, weight), b));
+    choose<64, PL>(z, a.r, mine, weight);
+    // member b of the launch takes the b-th chosen expert that is no identity
+    const unsigned long long real = __ballot(lane < (int)a.r.top && mine < (int)a.r.experts);
+    const int n_real = __popcll(real);
+    if (blockIdx.x == 0 && b == 0 && wave == 0) {
+        const int rank = __popcll(real & ((1ull << lane) - 1));
+        if (real >> lane & 1) a.ids[rank] = mine;
+        if (lane >= n_real && lane < (int)a.r.top) a.ids[lane] = -1;
+        if (a.identity) {
+            const float sum = wave_sum(lane < (int)a.r.top && mine >= (int)a.r.experts ? weight : 0.f);
+            if (lane == 0) *a.identity = sum;
+        }
+    }
+    if (b >= n_real) return;
+    int from = b;  // the b-th lane of those
+    if (n_real < (int)a.r.top) {
+        unsigned long long left = real;
+        for (int i = 0; i < b; ++i) left &= left - 1;
+        from = __builtin_ctzll(left);
+    }
+    const int e = __builtin_amdgcn_readlane(mine, from);
+    const float scale = __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, weight), from));
     const uint16_t *wb = a.w + (size_t)e * a.rows * a.ld;
     const int last = a.cols - 8;
     u32x4 w[U][R];
@@ -245,11 +272,20 @@ __global__ __launch_bounds__(256) void k_experts_up(UpK p) {
 #pragma unroll
             for (int u = 0; u < U; ++u) multiply8<R>(c[u], xs + k0 + (u * LPR + l) * 8, acc);
         }
+        if (R > 1 && a.gated) {
 #pragma unroll
-        for (int r = 0; r < R; ++r) {
-            const float v = lanes_sum<LPR>(acc[r]);
-            const int row = (g * G + sub) * R + r;
-            if (l == 0 && row < a.rows) a.y[(size_t)b * a.ldy + row] = scale * activate(v, a.act);
+            for (int r = 0; r + 1 < R; r += 2) {
+                const float v = lanes_sum<LPR>(acc[r]), u = lanes_sum<LPR>(acc[r + 1]);
+                const int row = (g * G + sub) * R + r;
+                if (l == 0 && row < a.rows) a.y[(size_t)b * a.ldy + (row >> 1)] = scale * (activate(v, a.act) * u);
+            }
+        } else {
+#pragma unroll
+            for (int r = 0; r < R; ++r) {
+                const float v = lanes_sum<LPR>(acc[r]);
+                const int row = (g * G + sub) * R + r;
+                if (l == 0 && row < a.rows) a.y[(size_t)b * a.ldy + row] = scale * activate(v, a.act);
+            }
         }
     }
 }
@@ -267,13 +303,13 @@ __global__ __launch_bounds__(256) void k_experts_out(OutK p) {
     const ExpertsOut &a = p.a;
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, sub = lane / LPR, l = lane % LPR;
     constexpr int G = 64 / LPR, CH = LPR * 8;
-    const int ids = lane < a.top ? a.ids[lane] : 0;
+    const int ids = lane < a.top ? a.ids[lane] : -1, n_real = __popcll(__ballot(ids >= 0)), end = p.c0 + n_real * p.ce;
     u32x4 w[U][R];
     auto fetch = [&](int grp, int chunk0) {
 #pragma unroll
         for (int u = 0; u < U; ++u) {
             const int c = chunk0 + u, x = max(c - p.c0, 0);
-            const int q = min((int)((unsigned)x * p.magic >> 20), a.top - 1), e = __builtin_amdgcn_readlane(ids, q);
+            const int q = min((int)((unsigned)x * p.magic >> 20), max(n_real - 1, 0)), e = max(__builtin_amdgcn_readlane(ids, q), 0);
             const bool first = c < p.c0;
             const uint16_t *base = first ? a.w0 : a.w1 + (size_t)e * a.rows * a.ld1;
             const int ld = first ? a.ld0 : a.ld1, col = min((first ? c : x - q * p.ce) * CH + l * 8, (first ? a.cols0 : a.cols1) - 8);
@@ -284,17 +320,18 @@ __global__ __launch_bounds__(256) void k_experts_out(OutK p) {
     };
     int g = blockIdx.x * 4 + wave;
     if (g < p.groups) fetch(g, 0);
-    const int total = p.chunks * CH / 4;
+    const int steps = (end + U - 1) / U * U, total = steps * CH / 4;  // (identity experts have no columns)
+    const float through = a.identity ? *a.identity : 0.f;
     constexpr int AH = 12;
     for (int i0 = tid; i0 < total; i0 += 256 * AH) {
         f32x4 v[AH];
         bool in[AH];
 #pragma unroll
         for (int j = 0; j < AH; ++j) {
-            const int i = i0 + 256 * j, c = i / (CH / 4), x = max(c - p.c0, 0), q = min((int)((unsigned)x * p.magic >> 20), a.top - 1);
+            const int i = i0 + 256 * j, c = i / (CH / 4), x = max(c - p.c0, 0), q = min((int)((unsigned)x * p.magic >> 20), max(n_real - 1, 0));
             const bool first = c < p.c0;
             const int col = (first ? i : i - (p.c0 + q * p.ce) * (CH / 4)) * 4, cols = first ? a.cols0 : a.cols1;
-            in[j] = col < cols;
+            in[j] = col < cols && c < end;
             v[j] = *reinterpret_cast<const f32x4 *>((first ? a.x0 : a.x1 + (size_t)q * a.ldx1) + min(col, cols - 4));
         }
 #pragma unroll
@@ -307,13 +344,13 @@ __global__ __launch_bounds__(256) void k_experts_out(OutK p) {
         float acc[R];
 #pragma unroll
         for (int r = 0; r < R; ++r) acc[r] = 0.f;
-        for (int c0 = 0; c0 < p.chunks; c0 += U) {
+        for (int c0 = 0; c0 < steps; c0 += U) {
             u32x4 c[U][R];
 #pragma unroll
             for (int u = 0; u < U; ++u)
 #pragma unroll
                 for (int r = 0; r < R; ++r) c[u][r] = w[u][r];
-            if (c0 + U < p.chunks)
+            if (c0 + U < steps)
                 fetch(g, c0 + U);
             else if (g + n_wg * 4 < p.groups)
                 fetch(g + n_wg * 4, 0);
@@ -324,7 +361,7 @@ __global__ __launch_bounds__(256) void k_experts_out(OutK p) {
         for (int r = 0; r < R; ++r) {
             const float v = lanes_sum<LPR>(acc[r]);
             const int row = (g * G + sub) * R + r;
-            if (l == 0 && row < a.rows) a.y[row] = v + (a.bias ? a.bias[row] : 0.f);
+            if (l == 0 && row < a.rows) a.y[row] = v + (a.bias ? a.bias[row] : 0.f) + (a.identity ? through * a.input[row] : 0.f);
         }
     }
 }
@@ -348,7 +385,8 @@ static hipError_t up_go(const ExpertsUp &a, int chunks, hipStream_t s) {
     k.kp = (chunks + u - 1) / u * u * LPR * 8;
     k.groups = (a.rows + 64 / LPR * R - 1) / (64 / LPR * R);
     if ((size_t)k.kp * 4 > 150 * 1024) return hipErrorInvalidValue;
-    auto pick = [&](auto f64, auto f256, auto f1024) { return a.experts <= 64 ? f64 : a.experts <= 256 ? f256 : f1024; };
+    const int outputs = (int)(a.r.experts + a.r.identity), top = (int)a.r.top;
+    auto pick = [&](auto f64, auto f256, auto f1024) { return outputs <= 64 ? f64 : outputs <= 256 ? f256 : f1024; };
     auto fn = u == 1   ? pick(k_experts_up<LPR, R, 1, 1>, k_experts_up<LPR, R, 1, 4>, k_experts_up<LPR, R, 1, 16>)
               : u == 2 ? pick(k_experts_up<LPR, R, 2, 1>, k_experts_up<LPR, R, 2, 4>, k_experts_up<LPR, R, 2, 16>)
               : u == 3 ? pick(k_experts_up<LPR, R, 3, 1>, k_experts_up<LPR, R, 3, 4>, k_experts_up<LPR, R, 3, 16>)
@@ -358,14 +396,14 @@ static hipError_t up_go(const ExpertsUp &a, int chunks, hipStream_t s) {
         const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(fn), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
         if (e != hipSuccess) return e;
     }
-    hipLaunchKernelGGL(fn, dim3(gemv_grid(k.groups, a.top), a.top), dim3(256), lds, s, k);
+    hipLaunchKernelGGL(fn, dim3(gemv_grid(k.groups, top), top), dim3(256), lds, s, k);
     return hipGetLastError();
 }
 
 hipError_t launch_experts_up(const ExpertsUp &a, hipStream_t s) {
-    if (a.cols <= 256) return up_go<16, 1>(a, (a.cols + 127) / 128, s);
+    if (a.cols <= 256) return a.gated ? up_go<16, 2>(a, (a.cols + 127) / 128, s) : up_go<16, 1>(a, (a.cols + 127) / 128, s);
     const int chunks = (a.cols + 511) / 512;
-    return (long)a.rows * a.top >= 4096 ? up_go<64, 2>(a, chunks, s) : up_go<64, 1>(a, chunks, s);
+    return a.gated || (long)a.rows * (long)a.r.top >= 4096 ? up_go<64, 2>(a, chunks, s) : up_go<64, 1>(a, chunks, s);
 }
 
 template <int LPR, int R>

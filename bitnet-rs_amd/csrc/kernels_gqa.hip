@@ -1,4 +1,6 @@
 // kernels_gqa.hip -- causal attention whose query heads share keys and values in groups, with one softmax map per head or two (gfx950).
+// Optionally rotated queries and keys, chunks of positions that do not see each other, a sink in the softmax's denominator, keys that are the
+// values too, and a gate per head on the output.
 //
 // Two maps (differential attention) weigh the same values; a head's output is a1 - lambda a2, divided by its root mean square over the value
 // columns.  Caches: keys [kv head][map][capacity][dimp], values transposed [kv head][vdimp][capacity].
@@ -15,10 +17,41 @@ namespace bitnet_hip {
 
 constexpr float kLog2e = 1.44269504088896f;
 
-__device__ __forceinline__ void gqa_split(int n_keys, int &per, int &used) {
-    const int tiles = (n_keys + kGqaTile - 1) / kGqaTile;
-    per = (tiles + kGqaSplits - 1) / kGqaSplits;
-    used = (tiles + per - 1) / per;
+// the first key a query at this position sees
+__device__ __forceinline__ int gqa_first(const Gqa &p, int pos) { return p.chunk ? pos - (int)((unsigned)pos % (unsigned)p.chunk) : 0; }
+
+// The records of a query at `pos`: tiles of keys from `base` (the tile that holds its first key) on, `per` tiles each.
+struct GqaRange {
+    int first, base, per, used;
+};
+__device__ __forceinline__ GqaRange gqa_range(const Gqa &p, int pos) {
+    GqaRange r;
+    r.first = gqa_first(p, pos);
+    r.base = r.first & ~(kGqaTile - 1);
+    const int tiles = (pos + 1 - r.base + kGqaTile - 1) / kGqaTile;
+    r.per = (tiles + kGqaSplits - 1) / kGqaSplits;
+    r.used = (tiles + r.per - 1) / r.per;
+    return r;
+}
+// records a launch has to provide for
+static int gqa_records(const Gqa &g) {
+    size_t keys = g.capacity;
+    if (g.chunk && g.chunk + kGqaTile < keys) keys = g.chunk + kGqaTile;  // (a chunk may start inside a tile)
+    return (int)min((size_t)kGqaSplits, (keys + kGqaTile - 1) / kGqaTile);
+}
+
+// element i of a head at a position, v being its own and the lane's neighbour holding the other element of the pair; cs, sn: the tables' row
+__device__ __forceinline__ float turn_neighbours(float v, int i, const float *cs, const float *sn, int dims) {
+    const float o = dpp<0xb1>(v);  // quad_perm [1,0,3,2]
+    if (i >= dims) return v;
+    const float c = cs[i >> 1], s = sn[i >> 1];
+    return (i & 1) ? v * c + o * s : v * c - o * s;
+}
+__device__ __forceinline__ float head_gate(const Gqa &p, int row, int h) {
+    if (!p.gate) return 1.0f;
+    const size_t i = (size_t)row * p.ldgate + h;
+    const float z = p.gate_f32 ? ((const float *)p.gate)[i] : bf2f(((const uint16_t *)p.gate)[i]);
+    return 1.0f / (1.0f + expf(-z));
 }
 
 size_t gqa_scratch_floats(size_t heads, size_t maps, size_t vdimp, size_t nq) { return nq * heads * maps * kGqaSplits * (kGqaRecHead + vdimp); }
@@ -35,6 +68,7 @@ __global__ __launch_bounds__(256) void k_gqa_rows(Gqa p, TR *rows, size_t ld, co
     if (y < nq + nk) {
         const bool key = y >= nq;
         const float *w = key ? p.k_weight : p.q_weight;
+        const int turned = (int)p.rot_dims, half = turned >> 1;
         TC *cache = key ? (TC *)p.kcache + (size_t)(y - nq) * p.capacity * dimp : nullptr;
         for (int t = t0 + wave; t < min(t0 + 64, n); t += 4) {
             TR *row = rows + (size_t)t * ld + (size_t)y * dimp;
@@ -43,10 +77,12 @@ __global__ __launch_bounds__(256) void k_gqa_rows(Gqa p, TR *rows, size_t ld, co
                 const float v = ld_act(row, i);
                 ss += v * v;
             }
-            const float norm = w ? 1.0f / sqrtf(wave_sum(ss) / (float)dim + p.eps) : 1.0f;
+            const float norm = w || p.unit_norm ? 1.0f / sqrtf(wave_sum(ss) / (float)dim + p.eps) : 1.0f;
             const float factor = key ? norm : norm * p.q_factor[pos0 + t];
+            const float *cs = p.rope_cos + (size_t)(pos0 + t) * half, *sn = p.rope_sin + (size_t)(pos0 + t) * half;
             for (int i = lane; i < dimp; i += 64) {
-                const float v = ld_act(row, i) * factor * (w && i < dim ? w[i] : 1.0f);  // (padding columns hold zeros)
+                float v = ld_act(row, i) * factor * (w && i < dim ? w[i] : 1.0f);  // (padding columns hold zeros)
+                if (turned) v = turn_neighbours(v, i, cs, sn, turned);
                 if (key)
                     st_act(cache + (size_t)(pos0 + t) * dimp, i, v);
                 else
@@ -58,7 +94,7 @@ __global__ __launch_bounds__(256) void k_gqa_rows(Gqa p, TR *rows, size_t ld, co
     y -= nq + nk;
     TR *tile = (TR *)lds;  // [64][vdimp + 2]
     const int stride = vdimp + 2, count = min(64, n - t0);
-    const TR *src = rows + (size_t)(nq + nk) * dimp + (size_t)y * vdimp;
+    const TR *src = rows + (size_t)(p.values_are_keys ? nq : nq + nk) * dimp + (size_t)y * vdimp;
     for (int i = tid; i < count * vdimp; i += 256) {
         const int t = i / vdimp, v = i - t * vdimp;
         tile[t * stride + v] = src[(size_t)(t0 + t) * ld + v];
@@ -93,11 +129,10 @@ __global__ __launch_bounds__(256) void k_gqa_any(Gqa p, const TQ *q, size_t ldq,
     __shared__ float sm[4], sl[4];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, hm = blockIdx.y, qi = blockIdx.z;
     const int maps = (int)p.maps, h = hm / maps, map = hm - h * maps, kv = h / (int)(p.heads / p.kv_heads), dimp = (int)p.dimp, vdimp = (int)p.vdimp;
-    const int n_keys = *pos_ptr + q0 + qi + 1;
-    int per, used;
-    gqa_split(n_keys, per, used);
-    if ((int)blockIdx.x >= used) return;
-    const int k0 = blockIdx.x * per * kGqaTile, k1 = min(k0 + per * kGqaTile, n_keys);
+    const int pos = *pos_ptr + q0 + qi;
+    const GqaRange range = gqa_range(p, pos);
+    if ((int)blockIdx.x >= range.used) return;
+    const int start = range.base + blockIdx.x * range.per * kGqaTile, k0 = max(start, range.first), k1 = min(start + range.per * kGqaTile, pos + 1);
     const TQ *qr = q + (size_t)qi * ldq + (size_t)hm * dimp;
     const TC *K = (const TC *)p.kcache + (size_t)(kv * maps + map) * p.capacity * dimp, *V = (const TC *)p.vcache + (size_t)kv * vdimp * p.capacity;
     float qv[ND], acc[NV];
@@ -139,7 +174,7 @@ __global__ __launch_bounds__(256) void k_gqa_any(Gqa p, const TQ *q, size_t ldq,
 
 template <class TQ, class TC>
 static hipError_t any_go(const Gqa &g, const void *q, size_t ldq, const int *pos, int q0, int nq, float *scratch, hipStream_t s) {
-    const int splits = min(kGqaSplits, (int)((g.capacity + kGqaTile - 1) / kGqaTile));
+    const int splits = gqa_records(g);
     const size_t lds = 4 * g.vdimp * sizeof(float);
     if (g.dimp > 1024 || g.vdimp > 1024) return hipErrorInvalidValue;
     auto fn = g.dimp <= 64 && g.vdimp <= 64 ? k_gqa_any<TQ, TC, 1, 1> : g.dimp <= 256 && g.vdimp <= 256 ? k_gqa_any<TQ, TC, 4, 4> : k_gqa_any<TQ, TC, 16, 16>;
@@ -166,12 +201,14 @@ __global__ __launch_bounds__(256, NV > 8 || NK * MAPS >= 8 ? 1 : 2) void k_gqa_s
     const int nh = min(16, (kv + 1) * group - h0), dim = (int)p.dim, dimp = (int)p.dimp, vdimp = (int)p.vdimp;
     constexpr int QS = NK * 32 + 4;
     const int pos = *a.pos, n_keys = pos + 1;
-    int per, used;
-    gqa_split(n_keys, per, used);
-    if ((int)blockIdx.x >= used) return;
-    const int k0 = blockIdx.x * per * kGqaTile, k1 = min(k0 + per * kGqaTile, n_keys);
+    const GqaRange range = gqa_range(p, pos);
+    if ((int)blockIdx.x >= range.used) return;
+    const int k0 = range.base + blockIdx.x * range.per * kGqaTile, k1 = min(k0 + range.per * kGqaTile, n_keys);
     uint16_t *K = (uint16_t *)p.kcache + (size_t)kv * MAPS * p.capacity * dimp, *V = (uint16_t *)p.vcache + (size_t)kv * vdimp * p.capacity;
-    const float *kraw = a.row + (p.heads * MAPS + (size_t)kv * MAPS) * dimp, *vraw = a.row + (p.heads + p.kv_heads) * MAPS * dimp + (size_t)kv * vdimp;
+    const float *kraw = a.row + (p.heads * MAPS + (size_t)kv * MAPS) * dimp,
+                *vraw = p.values_are_keys ? kraw : a.row + (p.heads + p.kv_heads) * MAPS * dimp + (size_t)kv * vdimp;
+    const int turned = (int)p.rot_dims;
+    const float *cs = p.rope_cos + (size_t)pos * (turned >> 1), *sn = p.rope_sin + (size_t)pos * (turned >> 1);
     u32x4 kf[2][MAPS][NK], vf[NV];
     auto fetch = [&](int kb) {  // (blocks lie below the capacity, a multiple of 128)
 #pragma unroll
@@ -195,12 +232,14 @@ __global__ __launch_bounds__(256, NV > 8 || NK * MAPS >= 8 ? 1 : 2) void k_gqa_s
                 v[j] = lane + 64 * j < dimp ? kraw[wave * dimp + lane + 64 * j] : 0.f;
                 ss += v[j] * v[j];
             }
-            const float norm = p.k_weight ? 1.0f / sqrtf(wave_sum(ss) / (float)dim + p.eps) : 1.0f;
+            const float norm = p.k_weight || p.unit_norm ? 1.0f / sqrtf(wave_sum(ss) / (float)dim + p.eps) : 1.0f;
 #pragma unroll
             for (int j = 0; j < (NK + 1) / 2; ++j) {
                 const int i = lane + 64 * j;
+                float k = v[j] * norm * (p.k_weight && i < dim ? p.k_weight[i] : 1.0f);
+                if (turned) k = turn_neighbours(k, i, cs, sn, turned);
                 if (i < dimp) {
-                    const uint16_t b = f2bf(v[j] * norm * (p.k_weight && i < dim ? p.k_weight[i] : 1.0f));
+                    const uint16_t b = f2bf(k);
                     K[((size_t)wave * p.capacity + pos) * dimp + i] = b;
                     newk[wave][i] = b;
                 }
@@ -227,11 +266,13 @@ __global__ __launch_bounds__(256, NV > 8 || NK * MAPS >= 8 ? 1 : 2) void k_gqa_s
                 v[j] = lane + 64 * j < dimp ? q[lane + 64 * j] : 0.f;
                 ss += v[j] * v[j];
             }
-            const float norm = (p.q_weight ? 1.0f / sqrtf(wave_sum(ss) / (float)dim + p.eps) : 1.0f) * factor;
+            const float norm = (p.q_weight || p.unit_norm ? 1.0f / sqrtf(wave_sum(ss) / (float)dim + p.eps) : 1.0f) * factor;
 #pragma unroll
             for (int j = 0; j < (NK + 1) / 2; ++j) {
                 const int i = lane + 64 * j;
-                if (i < NK * 32) area[r * QS + i] = v[j] * norm * (p.q_weight && i < dim ? p.q_weight[i] : 1.0f);
+                float t = v[j] * norm * (p.q_weight && i < dim ? p.q_weight[i] : 1.0f);
+                if (turned) t = turn_neighbours(t, i, cs, sn, turned);
+                if (i < NK * 32) area[r * QS + i] = t;
             }
         }
     }
@@ -255,6 +296,7 @@ __global__ __launch_bounds__(256, NV > 8 || NK * MAPS >= 8 ? 1 : 2) void k_gqa_s
     }
     for (int kb = k0 + wave * 32; kb < k1; kb += 128) {
         if (!kAhead || kb >= k0 + 128) fetch(kb);
+        if (kb + 32 <= range.first) continue;  // (another chunk's keys)
         if (owner && pos - kb < 32) {  // the new position, which memory need not show yet
             const int at = pos - kb, t = (at >> 2) & 1;
             const bool mine = r16 == (at >> 3) * 4 + (at & 3);
@@ -290,7 +332,10 @@ __global__ __launch_bounds__(256, NV > 8 || NK * MAPS >= 8 ? 1 : 2) void k_gqa_s
                 }
                 s[t] = (hi + lo) * kLog2e;
 #pragma unroll
-                for (int e = 0; e < 4; ++e) s[t][e] = kb + g * 8 + t * 4 + e < k1 ? s[t][e] : -INFINITY;
+                for (int e = 0; e < 4; ++e) {
+                    const int key = kb + g * 8 + t * 4 + e;
+                    s[t][e] = key < k1 && key >= range.first ? s[t][e] : -INFINITY;
+                }
             }
             float mx = fmaxf(fmaxf(fmaxf(s[0][0], s[0][1]), fmaxf(s[0][2], s[0][3])), fmaxf(fmaxf(s[1][0], s[1][1]), fmaxf(s[1][2], s[1][3])));
             mx = fmaxf(m[j], rows_max(mx));
@@ -348,7 +393,7 @@ __global__ __launch_bounds__(256, NV > 8 || NK * MAPS >= 8 ? 1 : 2) void k_gqa_s
 
 template <int NK, int NV>
 static hipError_t step_go(const Gqa &g, const GqaStep &a, hipStream_t s) {
-    const int splits = min(kGqaSplits, (int)((g.capacity + kGqaTile - 1) / kGqaTile)), group = (int)(g.heads / g.kv_heads), nh = min(16, group);
+    const int splits = gqa_records(g), group = (int)(g.heads / g.kv_heads), nh = min(16, group);
     const size_t queries = g.maps * 16 * (NK * 32 + 4), outs = 4 * g.maps * nh * g.vdimp, lds = (queries > outs ? queries : outs) * sizeof(float);
     auto fn = g.maps == 2 ? k_gqa_step<NK, NV, 2> : k_gqa_step<NK, NV, 1>;
     if (lds > 65536) {
@@ -374,8 +419,8 @@ __global__ __launch_bounds__(256) void k_gqa_merge(Gqa p, const int *pos_ptr, in
     static_assert(kGqaSplits == 128, "two records per lane of a wave");
     __shared__ float ws[2][kGqaSplits], sinv[2], slot[4];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, h = blockIdx.x, qi = blockIdx.z, maps = (int)p.maps, vdimp = (int)p.vdimp;
-    int per, used;
-    gqa_split(*pos_ptr + q0 + qi + 1, per, used);
+    const int used = gqa_range(p, *pos_ptr + q0 + qi).used;
+    const float gate = head_gate(p, qi, h);
     const size_t stride = kGqaRecHead + vdimp;
     const float *rec = scratch + ((size_t)qi * p.heads + h) * maps * kGqaSplits * stride;
     if (wave < maps) {
@@ -387,7 +432,7 @@ __global__ __launch_bounds__(256) void k_gqa_merge(Gqa p, const int *pos_ptr, in
             mv[e] = i < used ? r[i * stride] : -INFINITY;
             lv[e] = i < used ? r[i * stride + 1] : 0.f;
         }
-        const float M = rows_max(row_max(fmaxf(mv[0], mv[1])));
+        const float sink = p.sink ? p.sink[h] * kLog2e : -INFINITY, M = fmaxf(sink, rows_max(row_max(fmaxf(mv[0], mv[1]))));
         float den = 0.f;
 #pragma unroll
         for (int e = 0; e < 2; ++e) {
@@ -395,8 +440,8 @@ __global__ __launch_bounds__(256) void k_gqa_merge(Gqa p, const int *pos_ptr, in
             ws[wave][lane + 64 * e] = w;
             den += w * lv[e];
         }
-        den = wave_sum(den);
-        if (lane == 0) sinv[wave] = 1.0f / den;
+        den = wave_sum(den) + (p.sink ? exp2f(sink - M) : 0.f);
+        if (lane == 0) sinv[wave] = (maps == 1 ? gate : 1.0f) / den;
     }
     __syncthreads();
     // 32 lanes of four columns; eight groups share maps and records
@@ -425,13 +470,13 @@ __global__ __launch_bounds__(256) void k_gqa_merge(Gqa p, const int *pos_ptr, in
     };
     if (vdimp <= 256) {
         v = live ? value(tid) : 0.f;
-        if (maps == 2) v *= p.out_scale / sqrtf(group_sum<4>(v * v, slot) / (float)p.vdim + p.eps);
+        if (maps == 2) v *= gate * p.out_scale / sqrtf(group_sum<4>(v * v, slot) / (float)p.vdim + p.eps);
         if (live) st_act(dst, tid, v);
         return;
     }
     float ss = 0.f, f = 1.0f;
     for (int i = tid; i < vdimp; i += 256) v = value(i), ss += v * v;
-    if (maps == 2) f = p.out_scale / sqrtf(group_sum<4>(ss, slot) / (float)p.vdim + p.eps);
+    if (maps == 2) f = gate * p.out_scale / sqrtf(group_sum<4>(ss, slot) / (float)p.vdim + p.eps);
     for (int i = tid; i < vdimp; i += 256) st_act(dst, i, value(i) * f);
 }
 
@@ -463,11 +508,12 @@ __global__ __launch_bounds__(256, NV > 8 || NK > 4 ? 1 : 2) void k_gqa_prefill(G
     const int h = slot < own ? x * own + slot : 8 * own + r, qb = n_qb - 1 - level;
     const int kv = h / (int)(p.heads / p.kv_heads), q0 = qb * 4 * QW, pos0 = n_ctx - nq, qw = q0 + wave * QW;
     bf16x8 qf[SLOTS][NK];
-    int qpos[SLOTS];
+    int qpos[SLOTS], qfirst[SLOTS];
 #pragma unroll
     for (int t = 0; t < SLOTS; ++t) {
         const int tile = t / MAPS, map = t % MAPS, qi = min(qw + tile * 16 + r16, nq - 1);
         qpos[t] = pos0 + qw + tile * 16 + r16;
+        qfirst[t] = gqa_first(p, qpos[t]);
         const uint16_t *q = Q + (size_t)qi * ldq + (size_t)(h * MAPS + map) * dimp;
 #pragma unroll
         for (int kk = 0; kk < NK; ++kk) {
@@ -480,7 +526,8 @@ __global__ __launch_bounds__(256, NV > 8 || NK > 4 ? 1 : 2) void k_gqa_prefill(G
     float m[SLOTS], l[SLOTS];
 #pragma unroll
     for (int t = 0; t < SLOTS; ++t) {
-        m[t] = -INFINITY, l[t] = 0.f;
+        // (finite: with chunks a tile may hold no key that a query sees; the sink counts once per query, four lanes share one)
+        m[t] = MAPS == 1 && p.sink ? p.sink[h] * kLog2e : -1e30f, l[t] = MAPS == 1 && p.sink && g == 0 ? 1.0f : 0.f;
 #pragma unroll
         for (int v = 0; v < NV; ++v) o[v][t] = f32x4{0.f, 0.f, 0.f, 0.f};
     }
@@ -503,8 +550,10 @@ __global__ __launch_bounds__(256, NV > 8 || NK > 4 ? 1 : 2) void k_gqa_prefill(G
             if (j * 32 < vdimp) vreg[j] = *reinterpret_cast<const u32x4 *>(vb + (size_t)j * 64 * p.capacity + voff);
     };
     const int n_tiles = (min(n_ctx, pos0 + q0 + 4 * QW) + 63) / 64;
-    fetch(0);
-    for (int kt0 = 0; kt0 < n_tiles; ++kt0) {
+    // tiles from the first key of the workgroup's first query on; a wave leaves out what lies ahead of its own first key
+    const int t_first = gqa_first(p, pos0 + q0) >> 6, w_first = gqa_first(p, pos0 + qw), w_last = gqa_first(p, pos0 + qw + QW - 1);
+    fetch(t_first * 64);
+    for (int kt0 = t_first; kt0 < n_tiles; ++kt0) {
         const int key0 = kt0 * 64;
         __syncthreads();
 #pragma unroll
@@ -515,7 +564,7 @@ __global__ __launch_bounds__(256, NV > 8 || NK > 4 ? 1 : 2) void k_gqa_prefill(G
         for (int j = 0; j < NVL; ++j) *reinterpret_cast<u32x4 *>(lv + ((tid >> 3) + 32 * j) * VS + (tid & 7) * 16) = vreg[j];
         __syncthreads();
         if (kt0 + 1 < n_tiles) fetch(key0 + 64);
-        if (key0 > pos0 + qw + QW - 1) continue;  // every key of the tile lies ahead of this wave's queries
+        if (key0 > pos0 + qw + QW - 1 || key0 + 63 < w_first) continue;  // no key of the tile is seen by this wave's queries
         f32x4 s[4][SLOTS];
 #pragma unroll
         for (int kt = 0; kt < 4; ++kt) {
@@ -536,6 +585,13 @@ __global__ __launch_bounds__(256, NV > 8 || NK > 4 ? 1 : 2) void k_gqa_prefill(G
                 for (int kt = 0; kt < 4; ++kt)
 #pragma unroll
                     for (int i = 0; i < 4; ++i) s[kt][t][i] = key0 + kt * 16 + g * 4 + i > qpos[t] ? -INFINITY : s[kt][t][i];
+        if (key0 < w_last)  // an earlier chunk of some of the queries
+#pragma unroll
+            for (int t = 0; t < SLOTS; ++t)
+#pragma unroll
+                for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) s[kt][t][i] = key0 + kt * 16 + g * 4 + i < qfirst[t] ? -INFINITY : s[kt][t][i];
         float mn[SLOTS];
         bool grows = false;
 #pragma unroll
@@ -543,7 +599,6 @@ __global__ __launch_bounds__(256, NV > 8 || NK > 4 ? 1 : 2) void k_gqa_prefill(G
             float mx = fmaxf(fmaxf(s[0][t][0], s[0][t][1]), fmaxf(s[0][t][2], s[0][t][3]));
 #pragma unroll
             for (int kt = 1; kt < 4; ++kt) mx = fmaxf(mx, fmaxf(fmaxf(s[kt][t][0], s[kt][t][1]), fmaxf(s[kt][t][2], s[kt][t][3])));
-            // (tile 0 holds a visible key for every query, so the maximum is finite from the first tile on)
             mn[t] = fmaxf(m[t], rows_max(mx) * kLog2e);
             grows = grows || mn[t] > m[t];
         }
@@ -585,9 +640,14 @@ __global__ __launch_bounds__(256, NV > 8 || NK > 4 ? 1 : 2) void k_gqa_prefill(G
                 }
             }
     }
-    float inv[SLOTS];
+    float inv[SLOTS], gate[SLOTS / MAPS];
+#pragma unroll
+    for (int t = 0; t < SLOTS / MAPS; ++t) gate[t] = 1.0f;
 #pragma unroll
     for (int t = 0; t < SLOTS; ++t) inv[t] = 1.0f / rows_sum(l[t]);
+    if (p.gate)
+#pragma unroll
+        for (int t = 0; t < SLOTS / MAPS; ++t) gate[t] = head_gate(p, min(qw + t * 16 + r16, nq - 1), h);
     if (MAPS == 2) {
         float ss = 0.f;
 #pragma unroll
@@ -605,7 +665,7 @@ __global__ __launch_bounds__(256, NV > 8 || NK > 4 ? 1 : 2) void k_gqa_prefill(G
 #pragma unroll
         for (int v = 0; v < NV; ++v)
             if (v * 16 < vdimp) {
-                const f32x4 q = o[v][t] * inv[t];
+                const f32x4 q = o[v][t] * (inv[t] * gate[t]);
                 *reinterpret_cast<bf16x4 *>(dst + v * 16) = bf16x4{(__bf16)q.x, (__bf16)q.y, (__bf16)q.z, (__bf16)q.w};
             }
     }

@@ -18,6 +18,11 @@ std::vector<double> rotary_frequencies(const RotarySpec &r, double *mult) {
     std::vector<double> f((size_t)r.dims / 2);
     for (size_t i = 0; i < f.size(); ++i) f[i] = std::pow(r.base, -2.0 * (double)i / r.dims);
     *mult = 1.0;
+    if (r.banded)
+        for (double &v : f) {
+            const double turns = r.original * v / (2.0 * M_PI), keep = std::min(std::max((turns - r.slow) / (r.fast - r.slow), 0.0), 1.0);
+            v = (1.0 - keep) * v / r.factor + keep * v;
+        }
     if (!r.yarn) return f;
     // pairs that turn `turns` times within the original length sit at this (fractional) index
     auto index_of = [&](double turns) { return r.dims * std::log(r.original / (2.0 * M_PI * turns)) / (2.0 * std::log(r.base)); };
@@ -104,7 +109,7 @@ StackModel::StackModel(const StackSpec &spec, bool f32, int max_pos) : spec_(spe
         Layer &L = layers_[i];
         const LayerSpec &S = spec_.layers[i];
         if (S.mixer == LayerSpec::Latent) ok = rope_tables(S.latent.rot, &L.cos, &L.sin) == 0;
-        if (S.mixer == LayerSpec::Attention) ok = query_factors(S.attention, &L.q_factor) == 0;
+        if (S.mixer == LayerSpec::Attention) ok = query_factors(S.attention, &L.q_factor) == 0 && (S.attention.rot.dims == 0 || rope_tables(S.attention.rot, &L.cos, &L.sin) == 0);
         for (Slot &slot : L.slots) {
             if (!ok) break;
             if (S.mixer == LayerSpec::Latent && S.latent.kv_from < 0) {
@@ -175,8 +180,13 @@ int StackModel::plan_block(size_t i, int which, bool mixer, bool ff) {
         L.dimp = (int)up_to(m.dim, 32), L.vdimp = (int)up_to(m.vdim, 32);
         if (m.heads < 1 || m.kv_heads < 1 || m.heads % m.kv_heads || m.maps < 1 || m.maps > 2 || L.dimp > 1024 || L.vdimp > 1024 || !(m.temp_every > 0.0))
             return err_ = where + "attention: query heads in whole groups, one or two maps, heads of up to 1024 columns", BITNET_HIP_ERR_INVALID_ARGUMENT;
+        if (m.rot.dims % 2 || m.rot.dims > m.dim || (m.rot.banded && !(m.rot.fast > m.rot.slow)))
+            return err_ = where + "attention: an even number of rotated columns within the head, bands in order", BITNET_HIP_ERR_INVALID_ARGUMENT;
+        if (m.values_are_keys && (m.vdim != m.dim || m.maps != 1))
+            return err_ = where + "attention: keys that are the values have their size, and one map", BITNET_HIP_ERR_INVALID_ARGUMENT;
         B.ko = (int)up_to((size_t)m.heads * L.vdimp, 64);
-        B.main = (m.heads + m.kv_heads) * m.maps * L.dimp + m.kv_heads * L.vdimp;
+        L.gate_at = (m.heads + m.kv_heads) * m.maps * L.dimp + (m.values_are_keys ? 0 : m.kv_heads * L.vdimp);
+        B.main = L.gate_at + (m.head_gate ? m.heads : 0);
     } else if (mixer) {
         const DeltaSpec &m = S.delta;
         L.dimp = (int)up_to(m.dim, 32), L.vdimp = (int)up_to(m.vdim, 32);
@@ -190,12 +200,12 @@ int StackModel::plan_block(size_t i, int which, bool mixer, bool ff) {
         const ExpertsSpec &e = S.experts;
         B.fs = (int)up_to(S.ff, 64);
         if (e.count > 0) {
-            if (e.top < 1 || e.top > e.count || e.top > 32 || e.count > 1024 || e.ff < 1)
+            if (e.identity < 0 || e.top < 1 || e.top > e.count + e.identity || e.top > 32 || e.count + e.identity > 1024 || e.ff < 1)
                 return err_ = where + "experts: at most 32 of 1024, and not more than there are", BITNET_HIP_ERR_INVALID_ARGUMENT;
-            B.tail += e.count;
+            B.tail += e.count + e.identity;
         }
+        if (S.gated && S.ff > 0) return err_ = where + "a gated feed-forward stands behind its mixer, without routed experts", BITNET_HIP_ERR_INVALID_ARGUMENT;
     }
-    if (B.ko + B.fs == 0) B.fs = 64;  // routed experts alone: the product back is theirs, over columns of zeros
     return 0;
 }
 
@@ -288,6 +298,13 @@ void put_taps(std::vector<float> &rows, size_t channels, size_t at, const std::v
         for (size_t c = 0; c < from; ++c)
             for (size_t j = 0; j < taps; ++j) rows[j * channels + at + g * to + c] = w[(g * from + c) * taps + j];
 }
+// rows of two matrices in turn
+void append_pairs(std::vector<uint16_t> &o, const uint16_t *a, const uint16_t *b, size_t rows, size_t cols) {
+    for (size_t r = 0; r < rows; ++r) {
+        o.insert(o.end(), a + r * cols, a + (r + 1) * cols);
+        o.insert(o.end(), b + r * cols, b + (r + 1) * cols);
+    }
+}
 double dot(const std::vector<float> &a, const std::vector<float> &b) {
     double s = 0.0;
     for (size_t i = 0; i < a.size(); ++i) s += (double)a[i] * b[i];
@@ -309,7 +326,7 @@ int StackModel::set_layer(int layer, const StackLayerWeights &w) {
     const size_t W = width_;
     if (L.set) return fail_arg("the layer already holds weights");
     auto sized = [&](const std::vector<float> &v) { return v.empty() || v.size() == W; };
-    if (w.norm1.size() != W || !sized(w.norm1b) || !sized(w.ls1) || !sized(w.norm1_bias) || (!w.ls1.empty() && w.norm1b.empty()))
+    if (!sized(w.norm1) || !sized(w.norm1b) || !sized(w.ls1) || !sized(w.norm1_bias) || (!w.ls1.empty() && w.norm1b.empty()))
         return fail_arg("stack: norm of the wrong size");
     const size_t before = weight_bytes_;
     TRY(upload(&L.norm1.w, w.norm1));
@@ -366,7 +383,7 @@ int StackModel::set_layer(int layer, const StackLayerWeights &w) {
         TRY(upload(&L.decay_pow, pw));
     }
     if (!S.parallel && (S.ff > 0 || S.experts.count > 0)) {
-        if (w.norm2.size() != W || !sized(w.norm2b) || !sized(w.ls2) || !sized(w.norm2_bias) || (!w.ls2.empty() && w.norm2b.empty()))
+        if (!sized(w.norm2) || !sized(w.norm2b) || !sized(w.ls2) || !sized(w.norm2_bias) || (!w.ls2.empty() && w.norm2b.empty()))
             return fail_arg("stack: norm of the wrong size");
         TRY(upload(&L.norm2.w, w.norm2));
         TRY(upload(&L.norm2.bias, w.norm2_bias));
@@ -377,9 +394,15 @@ int StackModel::set_layer(int layer, const StackLayerWeights &w) {
         if (L.block[b].used) TRY(set_block((size_t)layer, b, w));
     if (!S.parallel && S.ff > 0 && S.experts.count == 0) {
         const size_t F = S.ff;
-        if (!w.up || !w.down || (!w.up_b.empty() && w.up_b.size() != F) || (!w.down_b.empty() && w.down_b.size() != W))
+        if (!w.up || !w.down || S.gated != (w.gate != nullptr) || (!w.up_b.empty() && (S.gated || w.up_b.size() != F)) || (!w.down_b.empty() && w.down_b.size() != W))
             return fail_arg("stack: incomplete feed-forward weights");
-        TRY(upload_matrix(L.up, take(w.up, F * W), (int)F, (int)W));
+        if (S.gated) {
+            std::vector<uint16_t> t;
+            append_pairs(t, w.gate, w.up, F, W);
+            TRY(upload_matrix(L.up, t, (int)(2 * F), (int)W));
+        } else {
+            TRY(upload_matrix(L.up, take(w.up, F * W), (int)F, (int)W));
+        }
         TRY(upload_matrix(L.down, take(w.down, W * F), (int)W, (int)F));
         TRY(upload(&L.up_b, w.up_b));
         TRY(upload(&L.down_b, w.down_b));
@@ -411,12 +434,15 @@ int StackModel::set_block(size_t i, int which, const StackLayerWeights &w) {
         const AttentionSpec &m = S.attention;
         const size_t H = m.heads, G = m.kv_heads, M = m.maps, D = m.dim, V = m.vdim;
         const bool two = M == 2 && w.lq1.size() == D && w.lk1.size() == D && w.lq2.size() == D && w.lk2.size() == D;
-        if (!w.q || !w.k || !w.v || !w.o || (!w.q_norm.empty() && w.q_norm.size() != D) || (!w.k_norm.empty() && w.k_norm.size() != D) || (M == 2 && !two))
+        if (!w.q || !w.k || m.values_are_keys != (w.v == nullptr) || m.head_gate != (w.g != nullptr) || !w.o || (!w.q_norm.empty() && w.q_norm.size() != D) ||
+            (!w.k_norm.empty() && w.k_norm.size() != D) || (M == 2 && !two) || (!w.sink.empty() && (w.sink.size() != H || M == 2)))
             return fail_arg("stack: incomplete attention weights");
         append(in, pad_rows(w.q, H * M, D, L.dimp, W));
         append(in, pad_rows(w.k, G * M, D, L.dimp, W));
-        append(in, pad_rows(w.v, G, V, L.vdimp, W));
+        if (w.v) append(in, pad_rows(w.v, G, V, L.vdimp, W));
+        if (w.g) append(in, take(w.g, H * W));
         into_out(w.o, 0, H, V, L.vdimp);
+        TRY(upload(&L.sink, w.sink));
         TRY(upload(&L.q_norm, w.q_norm));
         TRY(upload(&L.k_norm, w.k_norm));
         if (two) L.lambda = (float)(std::exp(dot(w.lq1, w.lk1)) - std::exp(dot(w.lq2, w.lk2)) + m.diff);
@@ -446,20 +472,27 @@ int StackModel::set_block(size_t i, int which, const StackLayerWeights &w) {
     }
     if (E.count > 0) {
         const size_t N = E.count, R = E.ff;
-        if (!w.router || w.expert_up.size() != N || w.expert_down.size() != N) return fail_arg("stack: incomplete experts");
-        append(in, take(w.router, N * W));
+        const size_t outputs = N + E.identity, up_rows = E.gated ? 2 * R : R;
+        if (!w.router || w.expert_up.size() != N || w.expert_down.size() != N || w.expert_gate.size() != (E.gated ? N : 0) ||
+            (!w.router_correction.empty() && w.router_correction.size() != outputs))
+            return fail_arg("stack: incomplete experts");
+        append(in, take(w.router, outputs * W));
+        TRY(upload(&L.correction, w.router_correction));
         std::vector<uint16_t> up, down;
         for (size_t e = 0; e < N; ++e) {
-            if (!w.expert_up[e] || !w.expert_down[e]) return fail_arg("stack: incomplete experts");
-            up.insert(up.end(), w.expert_up[e], w.expert_up[e] + R * W);
+            if (!w.expert_up[e] || !w.expert_down[e] || (E.gated && !w.expert_gate[e])) return fail_arg("stack: incomplete experts");
+            if (E.gated)
+                append_pairs(up, w.expert_gate[e], w.expert_up[e], R, W);
+            else
+                up.insert(up.end(), w.expert_up[e], w.expert_up[e] + R * W);
             down.insert(down.end(), w.expert_down[e], w.expert_down[e] + W * R);
         }
-        TRY(upload_matrix(B.expert_up, up, (int)(N * R), (int)W));
+        TRY(upload_matrix(B.expert_up, up, (int)(N * up_rows), (int)W));
         TRY(upload_matrix(B.expert_down, down, (int)(N * W), (int)R));
-        weight_bytes_ -= (N - E.top) * R * W * 4;  // a token reads `top` of them
+        weight_bytes_ -= (N - std::min(N, (size_t)E.top)) * (up_rows + R) * W * 2;  // a token reads `top` of them (fewer where identities are chosen)
     }
     TRY(upload_matrix(B.in, in, B.fs + B.main + B.tail, (int)W));
-    TRY(upload_matrix(B.out, out, (int)W, B.ko + B.fs));
+    if (B.ko + B.fs > 0) TRY(upload_matrix(B.out, out, (int)W, B.ko + B.fs));
     if (F > 0 && !w.up_b.empty()) {
         std::vector<float> bias(B.in.rows, 0.f);
         std::copy(w.up_b.begin(), w.up_b.end(), bias.begin());
@@ -470,8 +503,8 @@ int StackModel::set_block(size_t i, int which, const StackLayerWeights &w) {
 }
 
 int StackModel::set_globals(const uint16_t *embed, const std::vector<float> &final_norm, const std::vector<float> &final_bias, const uint16_t *head,
-                            const uint16_t *loop_in) {
-    if (!embed || final_norm.size() != (size_t)width_ || (!final_bias.empty() && final_bias.size() != (size_t)width_) || !head ||
+                            const uint16_t *loop_in, const std::vector<float> &embed_norm) {
+    if (!embed || (!embed_norm.empty() && embed_norm.size() != (size_t)width_) || final_norm.size() != (size_t)width_ || (!final_bias.empty() && final_bias.size() != (size_t)width_) || !head ||
         (spec_.loop.times > 0) != (loop_in != nullptr))
         return fail_arg("stack: incomplete globals");
     if (head_) return fail_arg("the model already holds its globals");
@@ -479,6 +512,7 @@ int StackModel::set_globals(const uint16_t *embed, const std::vector<float> &fin
     TRY(upload_matrix(embed_, take(embed, n), vocab_, width_));
     weight_bytes_ -= n * 2;  // a row of it is read per token
     TRY(upload_matrix(head_m_, take(head, n), vocab_, width_));
+    TRY(upload(&embed_norm_, embed_norm));
     TRY(upload(&final_norm_.w, final_norm));
     TRY(upload(&final_norm_.bias, final_bias));
     if (loop_in) {
@@ -500,7 +534,8 @@ int StackModel::clear_state() {
     return 0;
 }
 
-bitnet_hip_gqa StackModel::gqa_args(size_t i, int pass) const {
+// proj: rows of projections (the heads' gates stay in them)
+bitnet_hip_gqa StackModel::gqa_args(size_t i, int pass, const void *proj, size_t ld, bool f32) const {
     const Layer &L = layers_[i];
     const AttentionSpec &m = spec_.layers[i].attention;
     const Slot &slot = L.slots[(size_t)pass];
@@ -509,7 +544,17 @@ bitnet_hip_gqa StackModel::gqa_args(size_t i, int pass) const {
     a.heads = m.heads, a.kv_heads = m.kv_heads, a.maps = m.maps, a.dim = m.dim, a.dimp = L.dimp, a.vdim = m.vdim, a.vdimp = L.vdimp, a.capacity = cap_;
     a.eps = spec_.eps, a.lambda = L.lambda, a.out_scale = 1.0f - m.diff, a.q_weight = L.q_norm, a.k_weight = L.k_norm, a.q_factor = L.q_factor;
     a.kcache = slot.k, a.vcache = slot.v;
+    a.unit_norm = m.unit_norm, a.values_are_keys = m.values_are_keys, a.rot_dims = m.rot.dims, a.chunk = m.chunk, a.rope_cos = L.cos, a.rope_sin = L.sin, a.sink = L.sink;
+    if (m.head_gate) a.gate = (const char *)proj + (size_t)L.gate_at * (f32 ? 4 : 2), a.ldgate = ld, a.gate_f32 = f32;
     return a;
+}
+
+bitnet_hip_router StackModel::router_args(size_t i) const {
+    const ExpertsSpec &e = spec_.layers[i].experts;
+    bitnet_hip_router r;
+    memset(&r, 0, sizeof(r));
+    r.experts = e.count, r.identity = e.identity, r.top = e.top, r.scale = e.scale, r.raw = e.raw, r.correction = layers_[i].correction;
+    return r;
 }
 
 bitnet_hip_delta StackModel::delta_args(size_t i, int pass) const {
@@ -571,7 +616,7 @@ void StackModel::add_pending(bitnet_hip_vector_input &in) {
 
 bitnet_hip_vector_input StackModel::block_input(const Norm &norm) {
     bitnet_hip_vector_input in = plain_input(cur_);
-    in.kind = BITNET_HIP_IN_RESIDUAL_NORM;
+    in.kind = norm.w ? BITNET_HIP_IN_RESIDUAL_NORM : BITNET_HIP_IN_RESIDUAL;
     in.eps = spec_.eps, in.weight_offset = spec_.norm_offset, in.weight = norm.w, in.bias = norm.bias, in.center = spec_.center, in.n = width_;
     add_pending(in);
     return in;
@@ -597,11 +642,12 @@ int StackModel::step_block(size_t i, int pass, int which) {
     const bool routed = B.expert_up.w != nullptr;
     const int act = S.act_ff;
     bitnet_hip_vector_input in = block_input(B.norm);
-    if (routed) in.h_out = h_;
+    const float *h = B.norm.w ? h_ : cur_;  // what the experts read
+    if (routed && B.norm.w) in.h_out = h_;
     float *proj = row_ + B.ko + B.fs, *tail = proj + B.main;
     TRY(gemv(in, B.in, B.in_bias, B.fs ? act : 0, 0, B.fs, row_ + B.ko));
     if (B.mixer && S.mixer == LayerSpec::Attention) {
-        const bitnet_hip_gqa a = gqa_args(i, pass);
+        const bitnet_hip_gqa a = gqa_args(i, pass, proj, B.main, true);
         if (!f32_ && bitnet_hip_gqa_supported(a.dimp, a.vdimp)) {
             BCHK(bitnet_hip_gqa_step_dev(&a, proj, pos_, scratch_, stream_));
         } else {
@@ -615,10 +661,12 @@ int StackModel::step_block(size_t i, int pass, int which) {
     }
     if (!routed) return gemv(plain_input(row_), B.out, B.out_bias, 0, 0, 0, y_[which]);
     const ExpertsSpec &e = S.experts;
-    BCHK(bitnet_hip_experts_up_dev(tail + B.gates, e.count, e.top, e.scale, h_, B.expert_up.w, e.ff, B.expert_up.cols, B.expert_up.ld, e.act, eact_, B.expert_down.ld,
-                                   eids_, stream_));
-    BCHK(bitnet_hip_experts_out_dev(row_, B.out.w, B.out.cols, B.out.ld, B.out_bias, eact_, B.expert_down.ld, B.expert_down.w, B.expert_down.cols, B.expert_down.ld, eids_,
-                                    e.top, width_, y_[which], stream_));
+    const bitnet_hip_router r = router_args(i);
+    float *identity = e.identity ? (float *)(eids_ + 32) : nullptr;
+    BCHK(bitnet_hip_experts_up_dev(tail + B.gates, &r, h, B.expert_up.w, e.gated ? 2 * e.ff : e.ff, B.expert_up.cols, B.expert_up.ld,
+                                   e.act | (e.gated ? BITNET_HIP_ACT_GATED : 0), eact_, B.expert_down.ld, eids_, identity, stream_));
+    BCHK(bitnet_hip_experts_out_dev(B.out.w ? row_ : nullptr, B.out.w, B.out.cols, B.out.ld, B.out_bias, eact_, B.expert_down.ld, B.expert_down.w, B.expert_down.cols,
+                                    B.expert_down.ld, eids_, e.top, width_, identity, h, y_[which], stream_));
     return 0;
 }
 
@@ -653,10 +701,19 @@ int StackModel::step_linear(size_t i, int pass) {
     return gemv(in, L.o, nullptr, 0, 0, 0, y_[0]);
 }
 
+// the embedding output of the n tokens from the position on
+int StackModel::embed_rows(size_t n, float *out) {
+    if (embed_norm_)
+        BCHK(bitnet_hip_embed_norm_bf16_dev(embed_.w, embed_.ld, history_, pos_, n, width_, vocab_, spec_.embed_scale, embed_norm_, spec_.eps, out, stream_));
+    else
+        BCHK(bitnet_hip_embed_bf16_dev(embed_.w, embed_.ld, history_, pos_, n, width_, vocab_, spec_.embed_scale, out, stream_));
+    return 0;
+}
+
 int StackModel::step(bool with_logits, int) {
     cur_ = x0_;
     pending_ = Pending();
-    BCHK(bitnet_hip_embed_bf16_dev(embed_.w, embed_.ld, history_, pos_, 1, width_, vocab_, spec_.embed_scale, x0_, stream_));
+    TRY(embed_rows(1, x0_));
     for (const Run &run : runs_) {
         const size_t i = run.layer;
         const Layer &L = layers_[i];
@@ -668,7 +725,7 @@ int StackModel::step(bool with_logits, int) {
         if (L.block[1].used) {
             TRY(step_block(i, run.pass, 1));
         } else {
-            TRY(gemv(block_input(L.norm2), L.up, L.up_b, S.act_ff, 0, 0, act_));
+            TRY(gemv(block_input(L.norm2), L.up, L.up_b, S.act_ff | (S.gated ? BITNET_HIP_ACT_GATED : 0), 0, 0, act_));
             TRY(gemv(plain_input(act_), L.down, L.down_b, 0, 0, 0, y_[1]));
         }
         pending_ = {y_[1], L.norm2b, L.ls2};
@@ -786,7 +843,7 @@ int StackModel::matmul(const void *a, size_t lda, bool a_f32, const Matrix &m, c
 int StackModel::portion_norm(size_t n, const Norm *norm, const float *x2, void *h, size_t ldh) {
     const Pending p = pending_;
     pending_ = Pending();
-    const bool post = p.y && p.w, own = spec_.center || x2 || !h;
+    const bool post = p.w && !p.experts, own = spec_.center || x2 || !h;
     if (post) {  // the norm behind the sublayer, and the next one with it where it is of the same kind
         BCHK(bitnet_hip_residual_norm_rows_dev((float *)px_.p, p.y, width_, p.w, p.scale, own ? nullptr : norm->w, spec_.norm_offset, spec_.eps, n, width_,
                                                own ? nullptr : h, ldh, f32_, stream_));
@@ -797,8 +854,8 @@ int StackModel::portion_norm(size_t n, const Norm *norm, const float *x2, void *
     r.x = (float *)px_.p, r.m = n, r.width = width_, r.mult = spec_.residual_mult, r.eps = spec_.eps, r.weight_offset = spec_.norm_offset;
     r.center = spec_.center, r.h_f32 = f32_, r.h = h, r.ldh = ldh, r.x2 = x2;
     if (norm) r.weight = norm->w, r.bias = norm->bias;
-    if (p.y && !post) {
-        r.y = p.y, r.ldy = width_;
+    if (!post) {
+        r.y = p.y, r.ldy = width_, r.post_weight = p.w, r.scale = p.scale, r.input = p.input, r.ld_input = p.input ? up_to(width_, 64) : 0;
         if (p.experts) r.expert_rows = peout_.p, r.ld_expert = up_to(width_, 64), r.top = plan_.top, r.slots = plan_.slots, r.slot_weights = plan_.weights;
     }
     BCHK(bitnet_hip_sum_norm_rows_dev(&r, stream_));
@@ -826,7 +883,7 @@ int StackModel::portion_block(size_t i, int pass, int which, size_t n, size_t po
         BCHK(bitnet_hip_dense_matmul_dev(ph_.p, ldh, f32_, B.in.w + (size_t)(B.fs + B.main) * B.in.ld, B.in.ld, nullptr, n, B.tail, B.in.ld, 0, 0, 0, tail, ldt, 1, 1, 0, 0,
                                          0, stream_));
     if (B.mixer && S.mixer == LayerSpec::Attention) {
-        const bitnet_hip_gqa a = gqa_args(i, pass);
+        bitnet_hip_gqa a = gqa_args(i, pass, proj, ld, f32_);
         BCHK(bitnet_hip_gqa_rows_dev(&a, proj, ld, f32_, f32_, pos_, n, stream_));
         if (!f32_ && bitnet_hip_gqa_supported(a.dimp, a.vdimp)) {
             BCHK(bitnet_hip_gqa_prefill_dev(&a, (const uint16_t *)proj, ld, pos0 + n, n, (uint16_t *)row, ld, stream_));
@@ -835,6 +892,7 @@ int StackModel::portion_block(size_t i, int pass, int which, size_t n, size_t po
                 const size_t k = std::min(kDecodeSlice, n - s);
                 BCHK(bitnet_hip_gqa_any_dev(&a, proj + s * ld * es, ld, f32_, f32_, pos_, s, k, (float *)pscratch_.p, stream_));
                 BCHK(bitnet_hip_gqa_merge_dev(&a, pos_, s, k, (const float *)pscratch_.p, row + s * ld * es, ld, !f32_, stream_));
+                if (a.gate) a.gate = (const char *)a.gate + kDecodeSlice * ld * es;
             }
         }
     } else if (B.mixer) {
@@ -847,13 +905,15 @@ int StackModel::portion_block(size_t i, int pass, int which, size_t n, size_t po
         else
             BCHK(bitnet_hip_delta_recurrent_dev(&d, qk, pv_.p, gates, proj, ld, f32_, n, row, ld, stream_));
     }
-    TRY(matmul(row, ld, f32_, B.out, B.out_bias, n, 0, 0, 0, py_.p, width_, true));
+    if (B.out.w) TRY(matmul(row, ld, f32_, B.out, B.out_bias, n, 0, 0, 0, py_.p, width_, true));
     if (!routed) return 0;
     const ExpertsSpec &e = S.experts;
+    const bitnet_hip_router r = router_args(i);
     const size_t tile = !f32_ && n * e.top >= (size_t)96 * e.count ? 128 : 64;
     BCHK(bitnet_hip_experts_plan_make(pplan_.p, pplan_.bytes, n, e.count, e.top, tile, &plan_));
-    BCHK(bitnet_hip_experts_route_dev(tail + B.gates, ldt, e.scale, &plan_, stream_));
-    BCHK(bitnet_hip_experts_matmul_dev(&plan_, 1, ph_.p, ldh, f32_, B.expert_up.w, e.ff, B.expert_up.ld, B.expert_up.ld, e.act, peact_.p, B.expert_down.ld, f32_, stream_));
+    BCHK(bitnet_hip_experts_route_dev(tail + B.gates, ldt, &r, &plan_, stream_));
+    BCHK(bitnet_hip_experts_matmul_dev(&plan_, 1, ph_.p, ldh, f32_, B.expert_up.w, e.gated ? 2 * e.ff : e.ff, B.expert_up.ld, B.expert_up.ld,
+                                       e.act | (e.gated ? BITNET_HIP_ACT_GATED : 0), peact_.p, B.expert_down.ld, f32_, stream_));
     BCHK(bitnet_hip_experts_matmul_dev(&plan_, 0, peact_.p, B.expert_down.ld, f32_, B.expert_down.w, width_, B.expert_down.ld, B.expert_down.ld, 0, peout_.p, up_to(width_, 64),
                                        f32_, stream_));
     return 0;
@@ -918,8 +978,8 @@ int StackModel::portion(int rows, int pos0) {
     TRY(portion_buffers(n));
     float *x = (float *)px_.p;
     const float *y = (const float *)py_.p;
-    BCHK(bitnet_hip_embed_bf16_dev(embed_.w, embed_.ld, history_, pos_, n, width_, vocab_, spec_.embed_scale, x, stream_));
-    if (spec_.loop.times > 0) BCHK(bitnet_hip_embed_bf16_dev(embed_.w, embed_.ld, history_, pos_, n, width_, vocab_, spec_.embed_scale, (float *)px0_.p, stream_));
+    TRY(embed_rows(n, x));
+    if (spec_.loop.times > 0) TRY(embed_rows(n, (float *)px0_.p));
     pending_ = Pending();
     for (const Run &run : runs_) {
         const size_t i = run.layer;
@@ -928,16 +988,17 @@ int StackModel::portion(int rows, int pos0) {
         if (run.enters) TRY(portion_loop_in(n));
         TRY(portion_norm(n, &L.norm1, nullptr, ph_.p, ldh));
         TRY(L.block[0].used ? portion_block(i, run.pass, 0, n, pos0) : S.mixer == LayerSpec::Latent ? portion_latent(i, run.pass, n, pos0) : portion_linear(i, run.pass, n));
-        pending_ = {y, L.norm1b, L.ls1, L.block[0].expert_up.w != nullptr};
+        pending_ = {y, L.norm1b, L.ls1, L.block[0].expert_up.w != nullptr, L.norm1.w ? ph_.p : nullptr};
         if (S.parallel || (S.ff == 0 && S.experts.count == 0)) continue;
         TRY(portion_norm(n, &L.norm2, nullptr, ph_.p, ldh));
         if (L.block[1].used) {
             TRY(portion_block(i, run.pass, 1, n, pos0));
         } else {
-            TRY(matmul(ph_.p, ldh, f32_, L.up, L.up_b, n, S.act_ff, 0, 0, pact_.p, L.down.ld, f32_));
+            TRY(matmul(ph_.p, ldh, f32_, L.up, L.up_b, n, S.act_ff | (S.gated ? BITNET_HIP_ACT_GATED : 0), 0, 0, pact_.p, L.down.ld, f32_));
             TRY(matmul(pact_.p, L.down.ld, f32_, L.down, L.down_b, n, 0, 0, 0, py_.p, width_, true));
         }
-        pending_ = {y, L.norm2b, L.ls2, L.block[1].expert_up.w != nullptr};
+        const bool routed = L.block[1].expert_up.w != nullptr;
+        pending_ = {routed && !L.block[1].out.w ? nullptr : y, L.norm2b, L.ls2, routed, L.norm2.w ? ph_.p : nullptr};
     }
     TRY(portion_norm(n, nullptr, nullptr, nullptr, 0));
     hidden_ = x + (n - 1) * (size_t)width_;

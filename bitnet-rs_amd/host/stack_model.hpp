@@ -1,11 +1,11 @@
 // stack_model.hpp -- a decoder made of a list of layers, each a sequence mixer and an optional feed-forward.  The mechanisms are
-// parameters (mixer kinds and their sizes, kind of norm, layer scale, activations, experts, layers that run several times):
-// a design fills a StackSpec and hands its tensors over (see lasapel.cpp, mimolix.cpp), the stack owns the device layout, the caches and
+// parameters (mixer kinds and their sizes, kind and place of norms, layer scale, activations, experts, layers that run several times):
+// a design fills a StackSpec and hands its tensors over (see lasapel.cpp, mimolix.cpp, lurepel.cpp), the stack owns the device layout, the caches and
 // states of the live sequence, the launches of a step and of a prompt's portions.
 //
 //   one sublayer behind the other   x <- x + ls1 * norm1b(mixer(norm1(x)));  x <- x + ls2 * norm2b(ff(norm2(x)))
 //   side by side                    x <- x + m * (mixer(norm1(x)) + ff(norm1(x)))
-// (no norm behind a sublayer: m takes the place of ls * norm).  A loop runs a range of layers several times with the same weights, every
+// (no norm behind a sublayer: m takes the place of ls * norm; no norm ahead of it: the sublayer reads x itself).  A loop runs a range of layers several times with the same weights, every
 // pass with caches and states of its own and, ahead of its first layer, x <- W_in [x; embedding output].
 #pragma once
 
@@ -21,9 +21,10 @@ struct RotarySpec {
     int dims = 0;
     double base = 10000.0;
     bool yarn = false;  // frequencies interpolated between f and f / factor, cos and sin scaled
+    bool banded = false;  // f / factor for pairs of fewer than `slow` turns within the original length, f for more than `fast`, a line in between
     double factor = 1.0, original = 0.0, fast = 0.0, slow = 0.0;
     bool operator==(const RotarySpec &o) const {
-        return dims == o.dims && base == o.base && yarn == o.yarn && factor == o.factor && original == o.original && fast == o.fast && slow == o.slow;
+        return dims == o.dims && base == o.base && yarn == o.yarn && banded == o.banded && factor == o.factor && original == o.original && fast == o.fast && slow == o.slow;
     }
 };
 // frequency of every pair and the factor on cos and sin
@@ -45,6 +46,11 @@ struct AttentionSpec {  // keys and values of its own, shared by groups of query
     float scale = 1.f;
     double temp_coef = 0.0, temp_every = 1.0;  // a query at position p is multiplied by 1 + coef ln(floor((p + 1) / every) + 1)
     float diff = 0.f;                          // two maps: constant part of lambda, and 1 - diff scales the normed difference
+    RotarySpec rot;                            // dims 0: none; neighbouring elements turn together
+    int chunk = 0;                             // positions see their own chunk only; 0: everything ahead of them
+    bool unit_norm = false;                    // queries and keys divided by their root mean square
+    bool values_are_keys = false;              // no values of their own
+    bool head_gate = false;                    // a factor per head from the layer's input
 };
 struct DeltaSpec {  // gated delta rule (bitnet_hip_delta_*)
     int heads = 0, kv_heads = 0, dim = 0, vdim = 0, taps = 1;
@@ -53,6 +59,9 @@ struct DeltaSpec {  // gated delta rule (bitnet_hip_delta_*)
 struct ExpertsSpec {  // routed experts (bitnet_hip_experts_*); count 0: none
     int count = 0, top = 0, ff = 0, act = BITNET_HIP_ACT_NONE;
     float scale = 1.f;
+    bool raw = false;    // weights as the scores are, not divided by the chosen ones' sum
+    bool gated = false;  // act(gate) * up
+    int identity = 0;    // experts behind these whose output is their input
 };
 struct LayerSpec {
     enum Mixer { Latent, Linear, Attention, Delta } mixer = Latent;
@@ -63,6 +72,7 @@ struct LayerSpec {
     bool parallel = false;  // mixer and feed-forward side by side behind one norm (attention and delta mixers)
     int ff = 0;             // every token's feed-forward: dense, or the expert shared by all; 0: none
     int act_ff = BITNET_HIP_ACT_NONE;
+    bool gated = false;     // act_ff(gate) * up (a feed-forward behind the mixer, without routed experts)
     ExpertsSpec experts;
 };
 struct LoopSpec {  // layers start .. stop - 1 run `times` times in a row
@@ -81,7 +91,7 @@ struct StackSpec {
 
 // One layer's tensors as the loader hands them over: bf16 matrices [out, in], f32 vectors.
 struct StackLayerWeights {
-    std::vector<float> norm1, norm1b, ls1, norm2, norm2b, ls2;  // empty ls: no layer scale; empty norm1b, norm2b: no norm behind the sublayer
+    std::vector<float> norm1, norm1b, ls1, norm2, norm2b, ls2;  // empty ls: no layer scale; other empty ones: no norm ahead of, behind the sublayer
     std::vector<float> norm1_bias, norm2_bias;
     const uint16_t *dq = nullptr, *uq = nullptr, *dkv = nullptr, *uk = nullptr, *uv = nullptr, *o = nullptr;
     std::vector<float> dq_norm, dkv_norm, sink;
@@ -90,9 +100,9 @@ struct StackLayerWeights {
     std::vector<float> q_norm, k_norm, lq1, lk1, lq2, lk2;              // attention; empty q_norm, k_norm: no norm
     const uint16_t *b = nullptr, *a = nullptr;                          // delta: step size and decay, one row per head
     std::vector<float> q_conv, k_conv, v_conv, a_log, dt_bias;          // [channels][taps]
-    const uint16_t *up = nullptr, *down = nullptr, *router = nullptr;
-    std::vector<float> up_b, down_b;
-    std::vector<const uint16_t *> expert_up, expert_down;
+    const uint16_t *gate = nullptr, *up = nullptr, *down = nullptr, *router = nullptr;
+    std::vector<float> up_b, down_b, router_correction;                  // empty correction: none
+    std::vector<const uint16_t *> expert_gate, expert_up, expert_down;
 };
 
 class StackModel : public Sequence {
@@ -102,7 +112,7 @@ class StackModel : public Sequence {
 
     int set_layer(int layer, const StackLayerWeights &w);
     int set_globals(const uint16_t *embed, const std::vector<float> &final_norm, const std::vector<float> &final_bias, const uint16_t *head,
-                    const uint16_t *loop_in);
+                    const uint16_t *loop_in, const std::vector<float> &embed_norm = {});
 
     int prefill(int n, bool with_logits, int digits, float *elapsed_ms) override;
     int forward(const int32_t *tokens, int n, const int32_t *want, int n_want, float *logits) override;
@@ -146,6 +156,9 @@ class StackModel : public Sequence {
         // attention
         float *q_norm = nullptr, *k_norm = nullptr, *q_factor = nullptr;
         float lambda = 0.f;
+        int gate_at = 0;  // where a row of projections holds the heads' gates
+        // experts
+        float *correction = nullptr;
         // delta
         float *conv = nullptr, *decay_rate = nullptr, *dt_bias = nullptr;
         // latent
@@ -167,7 +180,8 @@ class StackModel : public Sequence {
     // the sublayer whose output is still to be added to the residual stream
     struct Pending {
         const float *y = nullptr, *w = nullptr, *scale = nullptr;
-        bool experts = false;  // a portion's routed rows join in
+        bool experts = false;         // a portion's routed rows join in (y may be missing)
+        const void *input = nullptr;  // what those experts read, if not the residual stream
     };
     struct Run {
         size_t layer;
@@ -181,6 +195,8 @@ class StackModel : public Sequence {
     int upload_matrix(Matrix &m, const std::vector<uint16_t> &rows, int n_rows, int cols);
     int rope_tables(const RotarySpec &r, float **cos, float **sin);
     int query_factors(const AttentionSpec &a, float **out);
+    int embed_rows(size_t n, float *out);
+    bitnet_hip_router router_args(size_t i) const;
     int plan_runs();
     int plan_block(size_t i, int which, bool mixer, bool ff);
     bool alloc(void **p, size_t bytes);
@@ -188,7 +204,7 @@ class StackModel : public Sequence {
     const Slot &kv_slot(size_t i, int pass) const { return layers_[spec_.layers[i].latent.kv_from >= 0 ? (size_t)spec_.layers[i].latent.kv_from : i].slots[(size_t)pass]; }
     void attention_args(size_t i, int pass, bitnet_hip_latent_attention &a) const;
     void latent_args(size_t i, int pass, const float *z, size_t ldz, void *cq, size_t ldcq, bitnet_hip_latent_rows &r) const;
-    bitnet_hip_gqa gqa_args(size_t i, int pass) const;
+    bitnet_hip_gqa gqa_args(size_t i, int pass, const void *proj, size_t ld, bool f32) const;
     bitnet_hip_delta delta_args(size_t i, int pass) const;
     // single token
     int gemv(const bitnet_hip_vector_input &in, const Matrix &m, const float *bias, int act0, int act1, size_t split, float *y,
@@ -220,6 +236,7 @@ class StackModel : public Sequence {
     Matrix embed_, head_m_, loop_in_;
     const uint16_t *head_ = nullptr;
     Norm final_norm_;
+    float *embed_norm_ = nullptr;
     size_t weight_bytes_ = 0;
     std::vector<void *> owned_;  // every fixed allocation
     struct RopeTable {

@@ -572,18 +572,27 @@ int bitnet_hip_hbm_read_ceiling(size_t bytes, int iters, double *best_gbs, doubl
 #define BITNET_HIP_ACT_SILU 1
 #define BITNET_HIP_ACT_SIGMOID 2
 #define BITNET_HIP_ACT_RELU2 3 /* square of relu */
+#define BITNET_HIP_ACT_GELU_TANH 4 /* v / 2 (1 + tanh(sqrt(2 / pi) (v + 0.044715 v^3))) */
+/* added to an activation: rows 2 i and 2 i + 1 of W make ONE column, act(row 2 i) * (row 2 i + 1): the number of columns of the output is half
+ * the number of rows given (which is even) */
+#define BITNET_HIP_ACT_GATED 0x100
 
 /* out[i][width] = scale * table[tokens[*offset + i]] as f32 (offset NULL = 0) */
 int bitnet_hip_embed_bf16_dev(const uint16_t *table_dev, size_t ld, const int32_t *tokens_dev, const int32_t *offset_dev, size_t n,
                               size_t width, size_t vocab, float scale, float *out_dev, void *stream);
-/* x[i] += scale * norm(y[i]; post_weight) (y NULL: skipped), then h[i] = norm(x[i]; next_weight) (h NULL: skipped), padding columns of h
- * zero; norm(v; w) = v / sqrt(mean(v^2) + eps) * (weight_offset + w). */
+/* the same, every row divided by sqrt(mean(v^2) + eps) and multiplied by norm_weight */
+int bitnet_hip_embed_norm_bf16_dev(const uint16_t *table_dev, size_t ld, const int32_t *tokens_dev, const int32_t *offset_dev, size_t n,
+                                   size_t width, size_t vocab, float scale, const float *norm_weight_dev, float eps, float *out_dev, void *stream);
+/* x[i] += scale * norm(y[i]; post_weight) (y NULL: skipped), then h[i] = norm(x[i]; next_weight) (next_weight NULL: x[i] itself; h NULL:
+ * skipped), padding columns of h zero; norm(v; w) = v / sqrt(mean(v^2) + eps) * (weight_offset + w). */
 int bitnet_hip_residual_norm_rows_dev(float *x_dev, const float *y_dev, size_t ldy, const float *post_weight_dev, const float *scale_dev,
                                       const float *next_weight_dev, float weight_offset, float eps, size_t m, size_t width, void *h_dev,
                                       size_t ldh, int h_f32, void *stream);
-/* Rows of a block whose sublayers' outputs add up: x[i] += mult * (y[i] + sum over k < top of slot_weights[i][k] * expert_rows[slots[i][k]])
- * (y NULL: nothing is added; top 0: no experts), then h[i] (NULL: skipped) = norm(x[i]; weight), padding columns zero, or -- x2 given --
- * the unnormed [x[i]; x2[i]].  center: layer norm, (v - mean) / sqrt(variance + eps) * weight + bias. */
+/* Rows of a block whose sublayers' outputs add up: t = y[i] + sum over k < top of slot_weights[i][k] * expert_rows[slots[i][k]] (y NULL: the
+ * experts' rows alone; top 0: no experts; neither: nothing is added; a negative slot stands for the row input[i], or -- input NULL -- for x[i]
+ * as it was), x[i] += mult * t or -- post_weight given -- scale * t / sqrt(mean(t^2) + eps) * (weight_offset + post_weight).  Then h[i] (NULL:
+ * skipped) = norm(x[i]; weight) (weight NULL: x[i] itself), padding columns zero, or -- x2 given -- the unnormed [x[i]; x2[i]].  center: norm
+ * is a layer norm, (v - mean) / sqrt(variance + eps) * weight + bias. */
 typedef struct bitnet_hip_sum_rows {
     float *x;
     size_t m, width;
@@ -599,6 +608,9 @@ typedef struct bitnet_hip_sum_rows {
     int32_t center, h_f32;
     void *h;
     size_t ldh;
+    const float *post_weight, *scale; /* scale NULL: 1 */
+    const void *input;                /* of the expert rows' type; may be h */
+    size_t ld_input;
 } bitnet_hip_sum_rows;
 int bitnet_hip_sum_norm_rows_dev(const bitnet_hip_sum_rows *rows, void *stream);
 /* h[i] = norm(o[i]; weight) * gate[i] over n columns; the mean divides by mean_n (padded heads hold zeros). */
@@ -618,6 +630,7 @@ int bitnet_hip_dense_matmul_dev(const void *a_dev, size_t lda, int a_f32, const 
 #define BITNET_HIP_IN_NORM 1          /* norm(x; weight) [* gate] */
 #define BITNET_HIP_IN_RESIDUAL_NORM 2 /* x' = x + scale * norm(y; post_weight) -> x_out (not x itself); norm(x'; weight) */
 #define BITNET_HIP_IN_CONCAT 3        /* [x'; x2], n elements each */
+#define BITNET_HIP_IN_RESIDUAL 4      /* x' itself */
 typedef struct bitnet_hip_vector_input {
     const float *x;
     int32_t kind;
@@ -703,13 +716,25 @@ int bitnet_hip_linear_chunked_dev(const uint16_t *qkv_dev, size_t ld, size_t n, 
  * A row of projections is [heads * maps * dimp | kv_heads * maps * dimp | kv_heads * vdimp], heads zero-padded to multiples of 32.
  * Queries and keys are normed per head and map (rms over dim, plain weight; NULL: not at all), a query at position p is then multiplied by
  * q_factor[p] (score scale and whatever depends on the position).  Caches: keys [kv_heads][maps][capacity][dimp], values transposed
- * [kv_heads][vdimp][capacity], bf16 or f32, zero-filled once. */
+ * [kv_heads][vdimp][capacity], bf16 or f32, zero-filled once.
+ * unit_norm: queries and keys are divided by their root mean square without a weight.  rot_dims > 0: elements 2 i and 2 i + 1 below rot_dims are
+ * turned by the tables' row of their position, (u, v) -> (u c - v s, v c + u s), behind the norm and its weight (without a weight the order
+ * makes no difference).  chunk > 0: a query at position p sees the keys from floor(p / chunk) chunk on.  sink: the softmax's denominator also holds
+ * exp(sink[head]) (one map).  values_are_keys: a row of projections has no values, they are the keys as projected (vdimp = dimp).  gate: every head's
+ * output is multiplied by sigmoid(gate[query][head]), the queries counted from the call's first one. */
 typedef struct bitnet_hip_gqa {
     size_t heads, kv_heads, maps, dim, dimp, vdim, vdimp, capacity; /* capacity % 128 == 0 */
     float eps, lambda, out_scale;
     const float *q_weight, *k_weight; /* [dim] */
     const float *q_factor;            /* [capacity] */
     void *kcache, *vcache;
+    int32_t unit_norm, values_are_keys;
+    size_t rot_dims, chunk;
+    const float *rope_cos, *rope_sin; /* [capacity][rot_dims / 2] */
+    const float *sink;                /* [heads] */
+    const void *gate;                 /* [queries][ldgate], f32 or bf16 */
+    size_t ldgate;
+    int32_t gate_f32;
 } bitnet_hip_gqa;
 size_t bitnet_hip_gqa_scratch_bytes(size_t heads, size_t maps, size_t vdimp, size_t nq);
 /* n rows of projections from position *pos on: queries in place, keys and values into the caches. */
@@ -761,28 +786,37 @@ size_t bitnet_hip_delta_workspace_bytes(size_t n, size_t heads, size_t dimp, siz
 int bitnet_hip_delta_chunked_dev(const bitnet_hip_delta *d, const float *qk_dev, const uint16_t *v_dev, const float *gates_dev, const uint16_t *rows_dev,
                                  size_t ld, size_t n, uint16_t *out_dev, size_t ldo, void *workspace_dev, size_t workspace_bytes, void *stream);
 
-/* Mixture of experts.  scores = softmax(logits); the `top` largest (lower index first among equals) get weights score / (their sum + 1e-20) *
- * scale.  experts <= 1024, top <= 32. */
+/* Mixture of experts.  A router has one logit per expert and, behind them, one per identity expert, whose output is its input.  scores =
+ * softmax(logits); chosen are the `top` largest of score + correction (correction NULL: of the scores; lower index first among equals), their
+ * weights are score / (the chosen scores' sum + 1e-20) * scale, or -- raw -- score * scale.  experts + identity <= 1024, top <= 32. */
+typedef struct bitnet_hip_router {
+    size_t experts, identity, top;
+    float scale;
+    int32_t raw;
+    const float *correction; /* [experts + identity] */
+} bitnet_hip_router;
 typedef struct bitnet_hip_experts_plan { /* where m tokens' choices lie in a workspace */
     int32_t *counts, *offsets, *n_tiles, *tiles; /* tiles: (expert, first slot, slots, 0) */
-    int32_t *ids, *slots, *tokens;               /* [m][top], [m][top], [m * top]: slot -> token */
+    int32_t *ids, *slots, *tokens;               /* [m][top], [m][top] (an identity expert's: -1), [m * top]: slot -> token */
     float *weights;                              /* [m][top] */
     size_t m, experts, top, tile, max_tiles;
 } bitnet_hip_experts_plan;
 size_t bitnet_hip_experts_plan_bytes(size_t m, size_t experts, size_t top);
 /* lays a plan out in memory that was zero-filled once (plans of other sizes may have used it); tile: rows of a product's tile (64 or 128) */
 int bitnet_hip_experts_plan_make(void *workspace_dev, size_t bytes, size_t m, size_t experts, size_t top, size_t tile, bitnet_hip_experts_plan *plan);
-int bitnet_hip_experts_route_dev(const float *logits_dev, size_t ldz, float scale, const bitnet_hip_experts_plan *plan, void *stream);
+int bitnet_hip_experts_route_dev(const float *logits_dev, size_t ldz, const bitnet_hip_router *router, const bitnet_hip_experts_plan *plan, void *stream);
 /* C[slot] = act(A[row of slot] . W[expert of slot]^T): rows are the slot's token (gather) or the slot itself.  W bf16 [experts][n][ldw] */
 int bitnet_hip_experts_matmul_dev(const bitnet_hip_experts_plan *plan, int gather, const void *a_dev, size_t lda, int a_f32, const uint16_t *w_dev,
                                   size_t n, size_t k, size_t ldw, int act, void *c_dev, size_t ldc, int c_f32, void *stream);
-/* One token: y[k][ldy] = weight_k * act(W[expert k] . x), the choice made from the logits by the same launch and stored in ids [top]. */
-int bitnet_hip_experts_up_dev(const float *logits_dev, size_t experts, size_t top, float scale, const float *x_dev, const uint16_t *w_dev, size_t rows,
-                              size_t cols, size_t ld, int act, float *y_dev, size_t ldy, int32_t *ids_dev, void *stream);
-/* y = W0 . x0 + bias + sum over k of W1[ids[k]] . x1[k]; W1 bf16 [experts][rows][ld1] */
+/* One token: y[k][ldy] = weight_k * act(W[expert k] . x), the choice made from the logits by the same launch and stored in ids [top].  Identity
+ * experts are left out of y and ids (-1 behind the last one that is none); the sum of their weights goes to *identity (needed where the router has any). */
+int bitnet_hip_experts_up_dev(const float *logits_dev, const bitnet_hip_router *router, const float *x_dev, const uint16_t *w_dev, size_t rows, size_t cols,
+                              size_t ld, int act, float *y_dev, size_t ldy, int32_t *ids_dev, float *identity_dev, void *stream);
+/* y = W0 . x0 + bias + sum over k of W1[ids[k]] . x1[k] + *identity * input; W1 bf16 [experts][rows][ld1]; x0 NULL: no first product; identity NULL:
+ * no last term */
 int bitnet_hip_experts_out_dev(const float *x0_dev, const uint16_t *w0_dev, size_t cols0, size_t ld0, const float *bias_dev, const float *x1_dev,
                                size_t ldx1, const uint16_t *w1_dev, size_t cols1, size_t ld1, const int32_t *ids_dev, size_t top, size_t rows,
-                               float *y_dev, void *stream);
+                               const float *identity_dev, const float *input_dev, float *y_dev, void *stream);
 
 #ifdef __cplusplus
 }

@@ -357,13 +357,13 @@ def routing(m, experts, top, seed):
 
 
 @pytest.mark.parametrize("m,experts,top,tile", [(1, 4, 1, 64), (2, 16, 16, 64), (70, 6, 3, 64), (300, 64, 8, 64), (257, 100, 5, 128), (500, 3, 2, 128), (64, 1024, 32, 64)])
-def test_route(hip, m, experts, top, tile):
+def test_route(hip, pkg, m, experts, top, tile):
     z, ids, w = routing(m, experts, top, 0)
     nb = hip.experts_plan_bytes(m, experts, top)
     ws = u.dev(np.zeros(nb // 4 + 4, np.int32))
     for _ in range(2):  # (a plan leaves its workspace ready for the next one)
         plan = hip.experts_plan_make(ws, nb, m, experts, top, tile)
-        hip.experts_route_dev(u.dev_f32(z), experts, 1.7, plan)
+        hip.experts_route_dev(u.dev_f32(z), experts, pkg.Router(experts, 0, top, 1.7), plan)
         raw, base = u.host(ws), ws.data_ptr()
 
         def at(p, n):
@@ -396,7 +396,7 @@ def test_experts_of_a_portion(hip, pkg, m, experts, top, tile, width, ff, f32):
     nb = hip.experts_plan_bytes(m, experts, top)
     ws = u.dev(np.zeros(nb // 4 + 4, np.int32))
     plan = hip.experts_plan_make(ws, nb, m, experts, top, tile)
-    hip.experts_route_dev(u.dev_f32(z), experts, 1.0, plan)
+    hip.experts_route_dev(u.dev_f32(z), experts, pkg.Router(experts, 0, top, 1.0), plan)
     put, new = (u.dev_f32, u.zeros_f32) if f32 else (u.dev_bf16, u.zeros_bf16)
     act, rows = new(m * top, ldf), new(m * top, ldw)
     hip.experts_matmul_dev(plan, True, put(u.padded(x, ldw)), ldw, f32, u.dev_bf16(u.padded(up, ldw)), ff, ldw, ldw, pkg.ACT_RELU2, act, ldf, f32)
@@ -416,7 +416,7 @@ def test_experts_of_one_token(hip, pkg, experts, top, width, ff, cols0):
     w0, bias = u.rounded(g.standard_normal((width, cols0)) / np.sqrt(cols0)), g.standard_normal(width).astype(np.float32)
     x, x0 = g.standard_normal(width).astype(np.float32), g.standard_normal(cols0).astype(np.float32)
     act, idd, y = u.zeros_f32(top, ldf), u.dev(np.zeros(64, np.int32)), u.zeros_f32(width)
-    hip.experts_up_dev(u.dev_f32(z[0]), experts, top, 2.5, u.dev_f32(u.padded(x, cols)), u.dev_bf16(u.padded(up, ldw)), ff, cols, ldw, pkg.ACT_RELU2, act, ldf, idd)
+    hip.experts_up_dev(u.dev_f32(z[0]), pkg.Router(experts, 0, top, 2.5), u.dev_f32(u.padded(x, cols)), u.dev_bf16(u.padded(up, ldw)), ff, cols, ldw, pkg.ACT_RELU2, act, ldf, idd)
     assert np.array_equal(u.host(idd)[:top], ids[0])
     want = 2.5 * w[0][:, None] * np.stack([so.relu_squared(up[e].astype(np.float64) @ x) for e in ids[0]])
     assert u.rms_error(u.host(act)[:, :ff], want) < F32_TOL
