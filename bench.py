@@ -634,13 +634,15 @@ def timed_model(model, prompt, steps: int, warmup: int, digits: int = 2) -> dict
             "decode_ms_per_token": round(ms / steps, 4), "decode_tok_s": round(steps / ms * 1e3, 1)}
 
 
-STACK_DESIGNS = {"lasapel": ("Lasapel", "write_lasapel", "lasapel_config"), "mimolix": ("Mimolix", "write_mimolix", "mimolix_config")}
+STACK_DESIGNS = {"lasapel": ("Lasapel", "write_lasapel", "lasapel_config"), "mimolix": ("Mimolix", "write_mimolix", "mimolix_config"),
+                 "lurepel": ("Lurepel", "write_lurepel", "lurepel_config")}
+STACK_BESIDE = {"mimolix": "lasapel", "lurepel": "mimolix"}  # the closest other model; BitNet where there is none
 
 
 def bench_stack(args, pkg, synth):
-    """--workload lasapel | mimolix: prompt and decode throughput of a layer-stack design at sizes that resemble a real model's layers, beside the
+    """--workload lasapel | mimolix | lurepel: prompt and decode throughput of a layer-stack design at sizes that resemble a real model's layers, beside the
     library's closest other model with the same width, (active) feed-forward, heads, vocabulary and number of layer runs: BitNet (QK256) for
-    Lasapel, Lasapel for Mimolix."""
+    Lasapel, Lasapel for Mimolix, Mimolix for Lurepel."""
     import tempfile
 
     rows = []
@@ -658,8 +660,8 @@ def bench_stack(args, pkg, synth):
         s = synth.STACK_SIZES[size]
         row = {"size": size, "layers": args.layers or 8, **{k: s[k] for k in ("width", "ff", "heads", "vocab")}}
         stack(row, args.workload, size)
-        if not args.no_also and args.workload == "mimolix":
-            stack(row, "lasapel", size)
+        if not args.no_also and args.workload in STACK_BESIDE:
+            stack(row, STACK_BESIDE[args.workload], size)
         elif not args.no_also:
             cfg = synth.ModelConfig(hidden=s["width"], n_layers=row["layers"], n_heads=s["heads"], n_kv_heads=s["n_kv"], ffn=s["ff"], vocab=s["vocab"], max_pos=max_pos)
             dec = pkg.HostDecoder(cfg)
@@ -684,7 +686,7 @@ def main():
     ap.add_argument("--steps", type=int, default=None, help="timed steps (default 256; 512 for --workload c4: BASELINE configs[3] = 4k-token prefill + 512 decode)")
     ap.add_argument("--warmup", type=int, default=16)
     ap.add_argument("--workload", default="c2", choices=["c2", "c3", "c4", "c5", "stream", *STACK_DESIGNS])
-    ap.add_argument("--sizes", default="2b,1b,3b", help="lasapel and mimolix workloads: which of the model sizes (synth.STACK_SIZES)")
+    ap.add_argument("--sizes", default="2b,1b,3b", help="layer-stack workloads: which of the model sizes (synth.STACK_SIZES)")
     ap.add_argument("--stream-layers", type=int, default=64, help="i2s_stream: gate|up matrices laid end to end (64 = 708 MB BitNet32-F16 / 566 MB QK256)")
     ap.add_argument("--stream-launches", type=int, default=None, help="stream workload only: a fixed number of launches and no timing (profiler counter passes)")
     ap.add_argument("--stream-format", default="i2s", choices=["i2s", "qk256"])

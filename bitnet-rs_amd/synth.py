@@ -177,6 +177,38 @@ def write_mimolix(folder: str, config: dict, seed: int = 42) -> str:
     return write_random(folder, config, mimolix_shapes(config), seed, lambda name: 1.0 if name.endswith(ones) else -1.0 if name.endswith(("A_log", "dt_bias")) else 0.0)
 
 
+LUREPEL_FF = {"1b": 2688, "2b": 4608, "3b": 5440}  # three gated matrices of about the bytes of the size's two; 8 experts of an eighth each
+LUREPEL_CHUNK = 8192
+
+
+def lurepel_config(size: str, n_layers: int, chunk: int = LUREPEL_CHUNK) -> dict:
+    """attention within chunks (heads of 128, half of it rotated, kv heads of the size), dense gated feed-forwards and mixtures of 64 experts and 8
+    identity experts, of which a token takes 8, in turn."""
+    s, ff = STACK_SIZES[size], LUREPEL_FF[size]
+    mixer = {"heads": s["heads"], "kv_heads": s["n_kv"], "dim": 128, "vdim": 128, "scale": 0.0884, "mask": {"size": chunk},
+             "rot": {"base": 500000.0, "dims": 64, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 4096}}}
+    dense = {"kind": "dense", "ff": ff}
+    moe = {"kind": "moe", "expert": {"ff": ff // 8}, "router": {"experts": 64, "identity": 8, "top": 8}}
+    return {"architecture": "Lurepel", "vocab": s["vocab"], "width": s["width"], "norm": {"eps": 1e-6},
+            "layers": [{"type": "attention", "mixer": mixer, "mlp": moe if i % 2 else dense} for i in range(n_layers)]}
+
+
+def write_lurepel(folder: str, config: dict, seed: int = 42) -> str:
+    W = config["width"]
+    shapes = {"embed": (config["vocab"], W), "embed.norm": (W,), "head": (config["vocab"], W), "final.norm": (W,)}
+    for i, layer in enumerate(config["layers"]):
+        p, m, f = f"l{i}.", layer["mixer"], layer["mlp"]
+        H, G, D = m["heads"], m["kv_heads"], m["dim"]
+        shapes.update({p + "norm1": (W,), p + "norm2": (W,), p + "mix.q": (H * D, W), p + "mix.k": (G * D, W), p + "mix.g": (H, W), p + "mix.o": (W, H * D)})
+        parts = {"": f["ff"]} if f["kind"] == "dense" else {f"e{e}.": f["expert"]["ff"] for e in range(f["router"]["experts"])}
+        for e, ff in parts.items():
+            shapes.update({f"{p}mlp.{e}gate": (ff, W), f"{p}mlp.{e}up": (ff, W), f"{p}mlp.{e}down": (W, ff)})
+        if f["kind"] == "moe":
+            n = f["router"]["experts"] + f["router"]["identity"]
+            shapes.update({p + "mlp.router": (n, W), p + "mlp.correction": (n,)})
+    return write_random(folder, config, shapes, seed, lambda name: 0.0 if name.endswith("correction") else 1.0)
+
+
 def write_lasapel(folder: str, config: dict, seed: int = 42) -> str:
     shapes = {"embed": (config["vocab"], config["width"]), "head": (config["vocab"], config["width"]), "final.norm": (config["width"],)}
     W = config["width"]

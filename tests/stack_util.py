@@ -165,8 +165,91 @@ def random_mimolix(config: dict, seed: int) -> dict:
     return t
 
 
+BANDS = {"factor": 5.0, "low": 1.5, "high": 6.0, "original": 96}
+
+
+def chunk_layer(heads=6, kv_heads=3, dim=20, scale=0.27, chunk=37, dims=12, base=300.0, scaling=None, mlp=None) -> dict:
+    rot = {"base": base, "dims": dims}
+    if scaling:
+        rot["scaling"] = scaling
+    return {"type": "attention", "mixer": {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": dim, "scale": scale, "mask": {"size": chunk}, "rot": rot}, "mlp": mlp}
+
+
+def gated_mlp(ff=40) -> dict:
+    return {"kind": "dense", "ff": ff}
+
+
+def corrected_mlp(experts=6, identity=2, top=3, ff=24) -> dict:
+    return {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": experts, "identity": identity, "top": top}}
+
+
+def lurepel(layers, width=112, vocab=150, eps=1e-5) -> dict:
+    return {"architecture": "Lurepel", "vocab": vocab, "width": width, "norm": {"eps": eps}, "layers": layers}
+
+
+def random_lurepel(config: dict, seed: int) -> dict:
+    """bf16-representable weights, everything away from its neutral value.  As with the parallel design, the first columns of an embedding row say
+    which experts its token takes and no sublayer adds to them; rows are drawn again until, in every layer, what is chosen and what is not lie well
+    apart."""
+    g = np.random.default_rng(seed)
+    W, V, eps = config["width"], config["vocab"], config["norm"]["eps"]
+    routers = {i: layer["mlp"]["router"] for i, layer in enumerate(config["layers"]) if layer["mlp"] and layer["mlp"]["kind"] == "moe"}
+    codes = max([r["experts"] + r["identity"] for r in routers.values()], default=0)
+    t = {}
+
+    def mat(name, rows, cols, gain=1.0):
+        t[name] = rounded(g.standard_normal((rows, cols)) * gain / np.sqrt(cols))
+
+    def norm(name, keep):
+        t[name] = rounded(1.0 + 0.25 * g.standard_normal(W))
+        t[name][:codes] = keep
+
+    norm("embed.norm", 1.0)
+    for i, r in routers.items():
+        n = r["experts"] + r["identity"]
+        t[f"l{i}.mlp.router"] = rounded(np.concatenate([1.2 * np.eye(n)[g.permutation(n)], np.zeros((n, codes - n)), 0.0003 * g.standard_normal((n, W - codes))], axis=1))
+        t[f"l{i}.mlp.correction"] = rounded(g.uniform(-0.25, 0.25, n))
+
+    def apart(row):
+        x = row / np.sqrt(np.mean(row ** 2) + eps) * t["embed.norm"]
+        for i, r in routers.items():
+            z = t[f"l{i}.mlp.router"].astype(np.float64) @ x
+            s = np.exp(z - z.max())
+            choice = np.sort(s / s.sum() + t[f"l{i}.mlp.correction"])[::-1]
+            if r["top"] < len(choice) and choice[r["top"] - 1] - choice[r["top"]] < 0.02:
+                return False
+        return True
+
+    t["embed"] = np.zeros((V, W), np.float32)
+    for k in range(V):
+        while True:
+            row = rounded(np.concatenate([g.uniform(-1.0, 2.0, codes), 0.8 * g.standard_normal(W - codes)]))
+            if apart(row.astype(np.float64)):
+                break
+        t["embed"][k] = row
+    for i, layer in enumerate(config["layers"]):
+        p, m, f = f"l{i}.", layer["mixer"], layer["mlp"]
+        H, G, D = m["heads"], m["kv_heads"], m["dim"]
+        norm(p + "norm1", 0.0)
+        mat(p + "mix.q", H * D, W)
+        mat(p + "mix.k", G * D, W)
+        mat(p + "mix.g", H, W, 1.5)
+        mat(p + "mix.o", W, H * D)
+        if not f:
+            continue
+        norm(p + "norm2", 0.0)
+        parts = {"": f["ff"]} if f["kind"] == "dense" else {f"e{e}.": f["expert"]["ff"] for e in range(f["router"]["experts"])}
+        for e, ff in parts.items():
+            mat(f"{p}mlp.{e}gate", ff, W)
+            mat(f"{p}mlp.{e}up", ff, W)
+            mat(f"{p}mlp.{e}down", W, ff)
+    norm("final.norm", 1.0)
+    mat("head", V, W)
+    return t
+
+
 def random_tensors(config: dict, seed: int) -> dict:
-    return {"Lasapel": random_lasapel, "Mimolix": random_mimolix}[config["architecture"]](config, seed)
+    return {"Lasapel": random_lasapel, "Mimolix": random_mimolix, "Lurepel": random_lurepel}[config["architecture"]](config, seed)
 
 
 def random_lasapel(config: dict, seed: int) -> dict:

@@ -85,6 +85,124 @@ def test_sum_norm_rows(hip, pkg, width, f32):
     assert np.array_equal(xs, x) and u.rms_error(h[:, :width], so.layer_norm(x.astype(np.float64), nw, nb, eps)) < tol
 
 
+@pytest.mark.parametrize("width", [96, 90, 2560, 5000])
+@pytest.mark.parametrize("f32", [True, False])
+def test_sum_norm_rows_behind_experts(hip, pkg, width, f32):
+    """the experts' rows and the input of identity experts, normed together ahead of the stream; the next input is the stream itself or its norm,
+    and may take the place of the input that the identities hand through"""
+    g = rng(width, 3)
+    m, top, ldh, eps = 6, 4, u.up_to(width, 64), 1e-2
+    x, y = (g.standard_normal((m, width)).astype(np.float32) for _ in range(2))
+    e, inp = g.standard_normal((m * top, width)).astype(np.float32), g.standard_normal((m, width)).astype(np.float32)
+    put, new, tol = (u.dev_f32, u.zeros_f32, F32_TOL) if f32 else (u.dev_bf16, u.zeros_bf16, BF_TOL)
+    if not f32:
+        e, inp = u.rounded(e), u.rounded(inp)
+    slots, sw = g.permutation(m * top).astype(np.int32).reshape(m, top), g.random((m, top)).astype(np.float32)
+    slots[0, 1], slots[1], slots[4, 2:] = -1, -1, -1
+    pw, sc, nw = ((1.0 + 0.3 * g.standard_normal(width)).astype(np.float32) for _ in range(3))
+    keep = [put(u.padded(e, ldh)), u.dev(slots), u.dev_f32(sw), u.dev_f32(pw), u.dev_f32(sc), u.dev_f32(nw), u.dev_f32(y)]
+    p = [k.data_ptr() for k in keep]
+    f64 = np.float64
+
+    def summed(through, start):
+        out = np.array(start, f64)
+        for i in range(m):
+            for k in range(top):
+                out[i] += f64(sw[i, k]) * (e[slots[i, k]] if slots[i, k] >= 0 else through[i])
+        return out
+
+    def run(h, **kw):
+        xd = u.dev_f32(x)
+        r = pkg.SumRows(x=xd.data_ptr(), m=m, width=width, eps=eps, h_f32=f32, h=h.data_ptr(), ldh=ldh, expert_rows=p[0], ld_expert=ldh, top=top, slots=p[1],
+                        slot_weights=p[2], **kw)
+        hip.sum_norm_rows_dev(r)
+        return u.host(xd), u.host(h)
+
+    want = x + so.norm_plain(summed(x, np.zeros((m, width))), pw, eps)
+    xs, h = run(new(m, ldh) + 3, post_weight=p[3])
+    assert u.rms_error(xs, want) < F32_TOL and u.rms_error(h[:, :width], want) < tol and not h[:, width:].any()
+    want = x + sc * so.norm_plain(summed(inp, y), pw, eps)
+    h = put(u.padded(inp, ldh))
+    xs, h = run(h, post_weight=p[3], scale=p[4], y=p[6], ldy=width, weight=p[5], input=h.data_ptr(), ld_input=ldh)
+    assert u.rms_error(xs, want) < F32_TOL and u.rms_error(h[:, :width], so.norm_plain(want, nw, eps)) < tol
+    xs, h = run(new(m, ldh), mult=0.6)
+    assert u.rms_error(xs, x + 0.6 * summed(x, np.zeros((m, width)))) < F32_TOL
+
+
+@pytest.mark.parametrize("width", [40, 77, 2560, 4500])
+def test_norm_behind_the_embedding(hip, width):
+    g = rng(width, 4)
+    ld, tokens = u.up_to(width, 64), np.array([5, 0, 11, 11], np.int32)
+    table, w = u.rounded(g.standard_normal((12, width))), g.standard_normal(width).astype(np.float32)
+    out = u.zeros_f32(3, width)
+    hip.embed_norm_bf16_dev(u.dev_bf16(u.padded(table, ld)), ld, u.dev(tokens), u.dev_f32(w), 1e-2, out, 3, width, 12, offset=pos_dev(1), scale=0.3)
+    assert u.rms_error(u.host(out), so.norm_plain(0.3 * table[tokens[1:]].astype(np.float64), w, 1e-2)) < F32_TOL
+
+
+@pytest.mark.parametrize("n", [40, 77, 256, 2560, 4500])
+def test_gemv_reads_the_stream_itself(hip, pkg, n):
+    g = rng(n, 5)
+    rows, ld, cols, eps = 70, u.up_to(n, 64), u.up_to(n, 8), 1e-2
+    w = u.rounded(g.standard_normal((rows, n)) / np.sqrt(n))
+    x, y, pw = (g.standard_normal(n).astype(np.float32) for _ in range(3))
+    wd = u.dev_bf16(u.padded(w, ld))
+    out, xo = u.zeros_f32(rows), u.zeros_f32(n)
+    hip.dense_gemv_dev(u.dev_f32(x), wd, rows, cols, ld, out, kind=pkg.IN_RESIDUAL, eps=eps, res=u.dev_f32(y), post_weight=u.dev_f32(pw), x_out=xo, n=n)
+    want = x + so.norm_plain(y.astype(np.float64), pw, eps)
+    assert u.rms_error(u.host(xo), want) < F32_TOL and u.rms_error(u.host(out), w @ want) < F32_TOL
+    hip.dense_gemv_dev(u.dev_f32(x), wd, rows, cols, ld, out, kind=pkg.IN_RESIDUAL, n=n)
+    assert u.rms_error(u.host(out), w @ x.astype(np.float64)) < F32_TOL
+
+
+ACTS = {"ACT_GELU_TANH": so.gelu_tanh, "ACT_SILU": so.silu, "ACT_RELU2": so.relu_squared}
+
+
+@pytest.mark.parametrize("act", list(ACTS))
+@pytest.mark.parametrize("rows,cols", [(1, 40), (7, 64), (33, 200), (300, 2560), (3000, 520), (9000, 2048)])
+def test_gemv_of_gated_pairs(hip, pkg, rows, cols, act):
+    g = rng(rows, cols)
+    ld = u.up_to(cols, 64)
+    w = u.rounded(2.0 * g.standard_normal((2 * rows, cols)) / np.sqrt(cols))
+    x, bias = g.standard_normal(cols).astype(np.float32), g.standard_normal(2 * rows).astype(np.float32)
+    out = u.zeros_f32(rows + 1) + 7
+    hip.dense_gemv_dev(u.dev_f32(x), u.dev_bf16(u.padded(w, ld)), 2 * rows, cols, ld, out, bias=u.dev_f32(bias), act0=getattr(pkg, act) | pkg.ACT_GATED)
+    z, got = w @ x.astype(np.float64) + bias, u.host(out)
+    assert u.rms_error(got[:rows], ACTS[act](z[0::2]) * z[1::2]) < F32_TOL and got[rows] == 7
+
+
+@pytest.mark.parametrize("act", list(ACTS))
+@pytest.mark.parametrize("m,n,k", [(1, 1, 64), (5, 35, 128), (70, 64, 192), (130, 333, 64), (2100, 1100, 1088), (4096, 2816, 1152), (300, 9000, 2048)])
+@pytest.mark.parametrize("f32", [True, False])
+def test_matmul_of_gated_pairs(hip, pkg, m, n, k, f32, act):
+    """every tile form (64, 128, 256 columns), ragged ends; the padding behind a row of the output stays"""
+    if f32 and m * n * k > 1 << 28:
+        m = 150
+    g = rng(m, n, k)
+    w = u.rounded(2.0 * g.standard_normal((2 * n, k), np.float32) / np.sqrt(k))
+    x = g.standard_normal((m, k), np.float32)
+    x = x if f32 else u.rounded(x)
+    ldc = u.up_to(n + 1, 64)
+    out = (u.zeros_f32 if f32 else u.zeros_bf16)(m, ldc)
+    out[:, n:] = 3
+    hip.dense_matmul_dev((u.dev_f32 if f32 else u.dev_bf16)(x), k, f32, u.dev_bf16(w), k, m, 2 * n, k, out, ldc, f32, act0=getattr(pkg, act) | pkg.ACT_GATED)
+    some = np.unique(np.r_[0, m // 3, m // 2, m - 1, g.integers(0, m, 60)])
+    z = x[some].astype(np.float64) @ w.T.astype(np.float64)
+    assert u.rms_error(u.host(out)[some, :n], ACTS[act](z[:, 0::2]) * z[:, 1::2]) < (F32_TOL if f32 else 4e-3)
+    assert bool((out[:, n:] == 3).all())
+
+
+@pytest.mark.parametrize("f32", [True, False])
+def test_matmul_gelu(hip, pkg, f32):
+    g = rng(6)
+    x, w = u.rounded(g.standard_normal((90, 128))), u.rounded(3.0 * g.standard_normal((70, 128)) / np.sqrt(128))
+    z = x.astype(np.float64) @ w.T
+    out = u.zeros_f32(90, 70)
+    for split in (0, 33):
+        hip.dense_matmul_dev((u.dev_f32 if f32 else u.dev_bf16)(x), 128, f32, u.dev_bf16(w), 128, 90, 70, 128, out, 70, True, act0=pkg.ACT_GELU_TANH, act1=pkg.ACT_NONE, act_split=split)
+        want = np.where(np.arange(70) < (split or 70), so.gelu_tanh(z), z)
+        assert u.rms_error(u.host(out), want) < (F32_TOL if f32 else 2e-5)
+
+
 # ---- attention ---------------------------------------------------------------------------------------------------------
 class Attention:
     """random projections of n tokens in the library's layout, and the attention's output by definition"""
@@ -131,6 +249,115 @@ class Attention:
 
 
 SHAPES = [(4, 2, 24, 40, 2), (6, 6, 128, 128, 2), (20, 1, 64, 100, 2), (8, 2, 96, 64, 1), (2, 1, 200, 256, 2), (5, 1, 40, 16, 1), (34, 2, 16, 24, 2)]
+
+
+class ChunkAttention:
+    """as above for heads of one map with everything optional on: rotation, unit norms, chunks, a sink, keys as values and a gate behind them"""
+
+    def __init__(self, pkg, n, heads, kv, dim, rot, chunk, f32, seed=0, own_values=False):
+        g = rng(n, heads, dim, chunk, seed)
+        self.n, self.heads, self.f32, self.dim = n, heads, f32, dim
+        self.dimp = self.vdimp = u.up_to(dim, 32)
+        self.vdim, self.cap = dim, u.up_to(n, 128)
+        store = (lambda a: a.astype(np.float32)) if f32 else u.rounded
+        q, k = store(g.standard_normal((n, heads, dim))), store(g.standard_normal((n, kv, dim)))
+        v = store(g.standard_normal((n, kv, dim))) if own_values else k
+        gate = store(2.0 * g.standard_normal((n, heads)))
+        parts = [u.padded(a, self.dimp).reshape(n, -1) for a in ((q, k, v) if own_values else (q, k))]
+        self.gate_at = sum(a.shape[1] for a in parts)
+        self.rows = np.concatenate(parts + [gate], axis=1)
+        self.ld = u.up_to(self.rows.shape[1], 64)
+        self.rows = u.padded(self.rows, self.ld)
+        eps, f64 = 1e-3, np.float64
+        self.scale = 1.3 / np.sqrt(dim)
+        spec = {"dims": rot, "base": 50.0, "scaling": dict(u.BANDS, original=30)}
+        self.q, self.k = (so.rms_divide(so.rotate_neighbours(a.astype(f64), spec), eps) for a in (q, k))
+        sink = g.standard_normal(heads).astype(np.float32)
+        self.want = np.zeros((n, heads, dim))
+        for a in range(heads):
+            for i in range(n):
+                first = i // chunk * chunk if chunk else 0
+                s = np.exp(self.k[first:i + 1, a // (heads // kv)] @ self.q[i, a] * self.scale)
+                self.want[i, a] = s @ v[first:i + 1, a // (heads // kv)].astype(f64) / (s.sum() + np.exp(f64(sink[a]))) * so.sigmoid(f64(gate[i, a]))
+        f = so.banded_frequencies(spec)
+        angle = np.arange(self.cap)[:, None] * f
+        new = u.zeros_f32 if f32 else u.zeros_bf16
+        factor = np.full(self.cap, self.scale, np.float32)
+        self.keep = [u.dev_f32(factor), new(kv, self.cap, self.dimp), new(kv, self.vdimp, self.cap), u.dev_f32(np.cos(angle)), u.dev_f32(np.sin(angle)), u.dev_f32(sink)]
+        p = [t.data_ptr() for t in self.keep]
+        self.attn = pkg.Gqa(heads, kv, 1, dim, self.dimp, dim, self.vdimp, self.cap, eps, 0.0, 1.0, 0, 0, p[0], p[1], p[2], 1, 0 if own_values else 1, rot, chunk, p[3], p[4], p[5])
+
+    put, new, fill, check = Attention.put, Attention.new, Attention.fill, Attention.check
+
+    def gated(self, rows, first=0):
+        """the gates are read from these rows"""
+        self.attn.gate = rows.data_ptr() + (first * self.ld + self.gate_at) * (4 if rows.element_size() == 4 else 2)
+        self.attn.ldgate, self.attn.gate_f32 = self.ld, rows.element_size() == 4
+
+
+CHUNKED = [(4, 2, 24, 16, 37), (6, 6, 128, 128, 64), (20, 1, 64, 2, 1), (5, 1, 40, 0, 100), (34, 2, 16, 16, 129), (2, 1, 200, 64, 300), (8, 2, 96, 32, 0)]
+
+
+@pytest.mark.parametrize("own_values", [False, True])
+@pytest.mark.parametrize("f32", [True, False])
+def test_chunk_attention_rows(hip, pkg, f32, own_values):
+    t = ChunkAttention(pkg, 200, 4, 2, 24, 16, 37, f32, own_values=own_values)
+    tol = F32_TOL if f32 else BF_TOL
+    for n0, n1 in ((0, 3), (3, 130), (130, 200)):
+        rows = u.host(t.fill(hip, n0, n1))
+        got = rows[:, :4 * t.dimp].reshape(-1, 4, t.dimp)
+        assert u.rms_error(got[..., :24], t.q[n0:n1] * t.scale) < tol and not got[..., 24:].any()
+        assert np.array_equal(rows[:, 4 * t.dimp:], t.rows[n0:n1, 4 * t.dimp:])  # what lies behind the queries stays
+    k, v = u.host(t.keep[1]), u.host(t.keep[2])
+    at = (4 + (2 if own_values else 0)) * t.dimp
+    assert u.rms_error(k[:, :200, :24], t.k.transpose(1, 0, 2)) < tol and not k[..., 24:].any() and not k[:, 200:].any()
+    assert np.array_equal(v[:, :, :200], t.rows[:, at:at + 2 * t.dimp].reshape(200, 2, t.dimp).transpose(1, 2, 0))
+
+
+@pytest.mark.parametrize("own_values", [False, True])
+@pytest.mark.parametrize("n,nq", [(1, 1), (2, 2), (65, 65), (128, 128), (129, 2), (300, 37), (300, 300)])
+@pytest.mark.parametrize("shape", CHUNKED)
+def test_chunk_attention_portion(hip, pkg, shape, n, nq, own_values):
+    t = ChunkAttention(pkg, n, *shape, False, own_values=own_values)
+    t.fill(hip, 0, n)
+    rows = t.put(t.rows[n - nq:])
+    hip.gqa_rows_dev(t.attn, rows, t.ld, False, False, pos_dev(n - nq), nq)
+    t.gated(rows)
+    out = t.new(nq, t.heads * t.vdimp)
+    hip.gqa_prefill_dev(t.attn, rows, t.ld, n, nq, out, t.heads * t.vdimp)
+    t.check(out, n - nq, 2e-2)
+
+
+@pytest.mark.parametrize("f32", [True, False])
+@pytest.mark.parametrize("n,nq", [(1, 1), (130, 130), (300, 2)])
+@pytest.mark.parametrize("shape", CHUNKED + [(2, 1, 300, 210, 70)])
+def test_chunk_attention_of_any_size(hip, pkg, shape, n, nq, f32):
+    t = ChunkAttention(pkg, n, *shape, f32)
+    rows = t.fill(hip, 0, n)
+    t.gated(rows, n - nq)
+    scratch = u.zeros_f32(hip.gqa_scratch_bytes(t.heads, 1, t.vdimp, nq) // 4)
+    out = u.zeros_f32(nq, t.heads * t.vdimp)
+    hip.gqa_any_dev(t.attn, rows[n - nq:].contiguous(), t.ld, f32, f32, pos_dev(n - nq), 0, nq, scratch)
+    hip.gqa_merge_dev(t.attn, pos_dev(n - nq), 0, nq, scratch, out, t.heads * t.vdimp, False)
+    t.check(out, n - nq, 1e-5 if f32 else 2e-2)
+
+
+@pytest.mark.parametrize("n", [1, 2, 32, 33, 64, 65, 128, 129, 257, 700])
+@pytest.mark.parametrize("shape", CHUNKED)
+def test_chunk_attention_step(hip, pkg, shape, n):
+    t = ChunkAttention(pkg, n, *shape, False)
+    if n > 1:
+        t.fill(hip, 0, n - 1)
+    scratch = u.zeros_f32(hip.gqa_scratch_bytes(t.heads, 1, t.vdimp, 1) // 4)
+    out, row = u.zeros_f32(1, t.heads * t.vdimp), u.dev_f32(t.rows[n - 1])
+    t.gated(row)
+    hip.gqa_step_dev(t.attn, row, pos_dev(n - 1), scratch)
+    hip.gqa_merge_dev(t.attn, pos_dev(n - 1), 0, 1, scratch, out, t.heads * t.vdimp, False)
+    t.check(out, n - 1, 1e-2)
+    k, v = u.host(t.keep[1]), u.host(t.keep[2])
+    assert u.rms_error(k[:, n - 1, :t.dim], t.k[n - 1]) < BF_TOL and not k[:, n:].any()
+    at = t.heads * t.dimp
+    assert np.array_equal(v[:, :, n - 1], t.rows[n - 1, at:at + len(v) * t.dimp].reshape(len(v), t.dimp)) and not v[:, :, n:].any()
 
 
 @pytest.mark.parametrize("f32", [True, False])
@@ -422,4 +649,123 @@ def test_experts_of_one_token(hip, pkg, experts, top, width, ff, cols0):
     assert u.rms_error(u.host(act)[:, :ff], want) < F32_TOL
     hip.experts_out_dev(u.dev_f32(x0), u.dev_bf16(u.padded(w0, ld0)), cols0, ld0, u.dev_f32(bias), act, ldf, u.dev_bf16(u.padded(down, ldf)), colf, ldf, idd, top, width, y)
     want = w0.astype(np.float64) @ x0 + bias + sum(down[e].astype(np.float64) @ want[k] for k, e in enumerate(ids[0]))
+    assert u.rms_error(u.host(y), want) < F32_TOL
+
+
+# experts that hand their input through, choice by corrected scores, weights as the scores are, gated pairs
+def corrected(m, experts, identity, top, seed):
+    n = experts + identity
+    g = rng(m, n, top, seed, 9)
+    z, c = 1.5 * g.standard_normal((m, n)).astype(np.float32), g.uniform(-0.3, 0.3, n).astype(np.float32)
+    if m > 3:
+        z[3] = 30.0 * (np.arange(n) < 1)  # one takes all; the others by their corrections
+    s = np.exp(z.astype(np.float64) - z.max(axis=1, keepdims=True))
+    s /= s.sum(axis=1, keepdims=True)
+    order = np.argsort(-(s + c), axis=1, kind="stable")
+    return z, c, order[:, :top], np.take_along_axis(s, order[:, :top], 1)
+
+
+def same_choice(got, z, c, ids):
+    """the oracle's choice, up to choice scores that lie within rounding of each other"""
+    s = np.exp(z.astype(np.float64) - z.max(axis=1, keepdims=True))
+    choice = s / s.sum(axis=1, keepdims=True) + c
+    return np.abs(np.take_along_axis(choice, np.asarray(got, np.int64), 1) - np.take_along_axis(choice, ids, 1)).max() < 1e-6
+
+
+CORRECTED = [(1, 4, 2, 1, 64), (2, 16, 1, 17, 64), (70, 6, 3, 3, 64), (300, 56, 8, 8, 64), (257, 100, 30, 5, 128), (500, 3, 9, 2, 128), (64, 1000, 24, 32, 64), (90, 1, 5, 4, 64)]
+
+
+@pytest.mark.parametrize("m,experts,identity,top,tile", CORRECTED)
+def test_corrected_route(hip, pkg, m, experts, identity, top, tile):
+    z, c, ids, w = corrected(m, experts, identity, top, 0)
+    nb, ldz = hip.experts_plan_bytes(m, experts, top), experts + identity + 3
+    ws, cd = u.dev(np.zeros(nb // 4 + 4, np.int32)), u.dev_f32(c)
+    for raw_weights in (1, 0):
+        plan = hip.experts_plan_make(ws, nb, m, experts, top, tile)
+        hip.experts_route_dev(u.dev_f32(u.padded(z, ldz)), ldz, pkg.Router(experts, identity, top, 0.8, raw_weights, cd.data_ptr()), plan)
+        raw, base = u.host(ws), ws.data_ptr()
+
+        def at(p, n):
+            return raw[(p - base) // 4:(p - base) // 4 + n]
+
+        got = at(plan.ids, m * top).reshape(m, top)
+        assert same_choice(got, z, c, ids)
+        s = np.exp(z.astype(np.float64) - z.max(axis=1, keepdims=True))
+        want = np.take_along_axis(s / s.sum(axis=1, keepdims=True), got.astype(np.int64), 1)
+        want = want if raw_weights else want / want.sum(axis=1, keepdims=True)
+        assert u.rms_error(at(plan.weights, m * top).view(np.float32).reshape(m, top), 0.8 * want) < F32_TOL
+        slots, real = at(plan.slots, m * top).reshape(m, top), got < experts
+        assert (slots[~real] == -1).all() and sorted(slots[real]) == list(range(real.sum()))
+        assert np.array_equal(at(plan.tokens, m * top)[slots[real]], np.repeat(np.arange(m), top).reshape(m, top)[real])
+        tiles = at(plan.tiles, 4 * int(at(plan.n_tiles, 1)[0])).reshape(-1, 4)
+        expert_of = np.full(m * top, -1)
+        for e, first, count, _ in tiles:
+            assert 0 < count <= tile and (expert_of[first:first + count] == -1).all()
+            expert_of[first:first + count] = e
+        assert np.array_equal(expert_of[slots[real]], got[real]) and (expert_of[real.sum():] == -1).all()
+
+
+@pytest.mark.parametrize("m,experts,identity,top,tile", [(2, 6, 2, 3, 64), (130, 5, 1, 2, 64), (300, 6, 4, 4, 128), (90, 1, 5, 4, 64)])
+@pytest.mark.parametrize("width,ff", [(112, 24), (256, 135), (192, 300)])
+@pytest.mark.parametrize("f32", [True, False])
+def test_gated_experts_of_a_portion(hip, pkg, m, experts, identity, top, tile, width, ff, f32):
+    if f32 and tile == 128:
+        tile = 64
+    g = rng(m, experts, width, 8)
+    z, c, ids, _ = corrected(m, experts, identity, top, 1)
+    ldw, ldf = u.up_to(width, 64), u.up_to(ff, 64)
+    up, down = u.rounded(2.0 * g.standard_normal((experts, 2 * ff, width)) / np.sqrt(width)), u.rounded(g.standard_normal((experts, width, ff)) / np.sqrt(ff))
+    x = g.standard_normal((m, width)).astype(np.float32) if f32 else u.rounded(g.standard_normal((m, width)))
+    nb, cd = hip.experts_plan_bytes(m, experts, top), u.dev_f32(c)
+    ws = u.dev(np.zeros(nb // 4 + 4, np.int32))
+    plan = hip.experts_plan_make(ws, nb, m, experts, top, tile)
+    hip.experts_route_dev(u.dev_f32(z), experts + identity, pkg.Router(experts, identity, top, 1.0, 1, cd.data_ptr()), plan)
+    put, new = (u.dev_f32, u.zeros_f32) if f32 else (u.dev_bf16, u.zeros_bf16)
+    act, rows = new(m * top, ldf), new(m * top, ldw)
+    hip.experts_matmul_dev(plan, True, put(u.padded(x, ldw)), ldw, f32, u.dev_bf16(u.padded(up, ldw)), 2 * ff, ldw, ldw, pkg.ACT_SILU | pkg.ACT_GATED, act, ldf, f32)
+    hip.experts_matmul_dev(plan, False, act, ldf, f32, u.dev_bf16(u.padded(down, ldf)), width, ldf, ldf, pkg.ACT_NONE, rows, ldw, f32)
+    raw = u.host(ws)
+    slots, got_ids = (raw[(q - ws.data_ptr()) // 4:][:m * top].reshape(m, top) for q in (plan.slots, plan.ids))
+    got, want = [], []
+    for i in range(m):
+        for k in range(top):
+            e = got_ids[i, k]
+            if e >= experts:
+                continue
+            h = up[e].astype(np.float64) @ x[i]
+            want.append(down[e].astype(np.float64) @ (so.silu(h[0::2]) * h[1::2]))
+            got.append(u.host(rows[slots[i, k]])[:width])
+    if want:
+        assert u.rms_error(got, want) < (F32_TOL if f32 else 8e-3)
+
+
+@pytest.mark.parametrize("experts,identity,top,width,ff,cols0", [(4, 2, 1, 64, 24, 0), (6, 2, 8, 112, 40, 200), (12, 5, 3, 320, 72, 0), (64, 8, 8, 1000, 519, 0), (64, 8, 8, 2560, 576, 0),
+                                                                 (2, 60, 9, 90, 16, 64), (1, 9, 3, 200, 130, 0)])
+@pytest.mark.parametrize("seed", [2, 3, 4])
+def test_gated_experts_of_one_token(hip, pkg, experts, identity, top, width, ff, cols0, seed):
+    """also with none but identities among the chosen (few experts, many identities)"""
+    g = rng(experts, width, ff, 8)
+    z, c, ids, w = corrected(1, experts, identity, top, seed)
+    ldw, ldf, ld0, cols, colf = u.up_to(width, 64), u.up_to(ff, 64), u.up_to(cols0, 64), u.up_to(width, 8), u.up_to(ff, 8)
+    up, down = u.rounded(2.0 * g.standard_normal((experts, 2 * ff, width)) / np.sqrt(width)), u.rounded(g.standard_normal((experts, width, ff)) / np.sqrt(ff))
+    w0, bias = u.rounded(g.standard_normal((width, cols0)) / np.sqrt(max(cols0, 1))), g.standard_normal(width).astype(np.float32)
+    x, x0 = g.standard_normal(width).astype(np.float32), g.standard_normal(cols0).astype(np.float32)
+    act, idd, y, through, cd = u.zeros_f32(top, ldf), u.dev(np.full(64, 77, np.int32)), u.zeros_f32(width), u.zeros_f32(1), u.dev_f32(c)
+    xd = u.dev_f32(u.padded(x, cols))
+    hip.experts_up_dev(u.dev_f32(z[0]), pkg.Router(experts, identity, top, 2.5, 1, cd.data_ptr()), xd, u.dev_bf16(u.padded(up, ldw)), 2 * ff, cols, ldw, pkg.ACT_SILU | pkg.ACT_GATED,
+                       act, ldf, idd, through)
+    real = ids[0] < experts
+    n = int(real.sum())
+    got = u.host(idd)
+    assert np.array_equal(got[:n], ids[0][real]) and (got[n:top] == -1).all() and (got[top:] == 77).all()
+    assert abs(u.host(through)[0] - 2.5 * w[0][~real].sum()) < 1e-5
+    want = np.zeros((n, ff))
+    for k, (e, s) in enumerate(zip(ids[0][real], w[0][real])):
+        h = up[e].astype(np.float64) @ x
+        want[k] = 2.5 * s * so.silu(h[0::2]) * h[1::2]
+    if n:
+        assert u.rms_error(u.host(act)[:n, :ff], want) < F32_TOL
+    first = (u.dev_f32(x0), u.dev_bf16(u.padded(w0, ld0))) if cols0 else (None, None)
+    hip.experts_out_dev(*first, cols0, ld0, u.dev_f32(bias), act, ldf, u.dev_bf16(u.padded(down, ldf)), colf, ldf, idd, top, width, y, identity=through, input=xd)
+    want = w0.astype(np.float64) @ x0 + bias + 2.5 * w[0][~real].sum() * x.astype(np.float64) + sum(down[e].astype(np.float64) @ want[k] for k, e in enumerate(ids[0][real]))
     assert u.rms_error(u.host(y), want) < F32_TOL

@@ -23,7 +23,7 @@ BASE = u.lasapel([u.latent_layer(ff=24), u.lightning_layer()], width=40, vocab=2
 
 def test_registry_names(built):
     names = built.registered_models()
-    assert "Lasapel" in names and "Mimolix" in names and ".gguf" in names
+    assert {"Lasapel", "Mimolix", "Lurepel"} <= set(names) and ".gguf" in names
 
 
 PARALLEL = u.mimolix([u.delta_layer(mlp=u.expert_mlp()), u.attention_layer()], width=40, vocab=20, loop=(0, 1, 2))
@@ -47,6 +47,32 @@ def test_bad_parallel_configurations_say_why(built, tmp_path, change, message):
     c = copy.deepcopy(PARALLEL)
     change(c)
     path = u.save_model(str(tmp_path), c, u.random_tensors(PARALLEL, 1))
+    with pytest.raises(built.BitNetHipError, match=message):
+        built.open_model(path)
+
+
+CHUNKED = u.lurepel([u.chunk_layer(mlp=u.gated_mlp(), scaling=u.BANDS), u.chunk_layer(mlp=u.corrected_mlp()), u.chunk_layer()], width=40, vocab=20)
+
+
+@pytest.mark.parametrize("change,message", [
+    (lambda c: c["norm"].pop("eps"), "norm.eps: missing"),
+    (lambda c: c["layers"][0].update(type="delta"), r"layers\[0\].type: unknown mixer"),
+    (lambda c: c["layers"][0]["mixer"].pop("kv_heads"), r"layers\[0\].mixer.kv_heads: missing"),
+    (lambda c: c["layers"][0]["mixer"].update(kv_heads=4), "layer 0: attention: query heads in whole groups"),
+    (lambda c: c["layers"][0]["mixer"].update(vdim=24), "layer 0: attention: keys that are the values"),
+    (lambda c: c["layers"][0]["mixer"]["mask"].update(size=0), r"layers\[0\].mixer.mask.size: not an integer"),
+    (lambda c: c["layers"][0]["mixer"]["rot"].update(dims=22), "layer 0: attention: an even number of rotated columns"),
+    (lambda c: c["layers"][0]["mixer"]["rot"].update(dims=7), "layer 0: attention: an even number of rotated columns"),
+    (lambda c: c["layers"][0]["mixer"]["rot"]["scaling"].pop("high"), r"layers\[0\].mixer.rot.scaling.high: missing"),
+    (lambda c: c["layers"][0]["mixer"]["rot"]["scaling"].update(high=1.5), "bands in order"),
+    (lambda c: c["layers"][0]["mlp"].update(kind="sparse"), r"layers\[0\].mlp.kind: unknown"),
+    (lambda c: c["layers"][1]["mlp"]["router"].update(top=9), "layer 1: experts"),
+    (lambda c: c["layers"][1]["mlp"]["router"].update(identity=-1), r"layers\[1\].mlp.router.identity: not an integer"),
+])
+def test_bad_chunked_configurations_say_why(built, tmp_path, change, message):
+    c = copy.deepcopy(CHUNKED)
+    change(c)
+    path = u.save_model(str(tmp_path), c, u.random_tensors(CHUNKED, 1))
     with pytest.raises(built.BitNetHipError, match=message):
         built.open_model(path)
 
@@ -114,10 +140,16 @@ def test_entry_points_check_shapes_before_any_launch(built):
         (lambda: hip.gqa_any_dev(built.Gqa(4, 4, 2, 16, 32, 16, 32, 128, 1e-5, 0.1, 0.9, 8, 8, 8, 8, 8), 8, 128, True, True, 8, 0, 1, 8), "gqa_any"),
         (lambda: hip.delta_step_dev(built.Delta(4, 2, 16, 32, 16, 48, 4, 8, 8, 8, 8, 1.0, 1e-6, 1e-5, 8, 8), 8, 8, 8, 8), "delta: bad shape"),
         (lambda: hip.delta_chunked_dev(built.Delta(4, 2, 16, 32, 16, 32, 4, 8, 8, 8, 8, 1.0, 1e-6, 1e-5, 8, 8), 8, 8, 8, 8, 512, 9, 8, 128, 8, 64), "workspace"),
-        (lambda: hip.experts_plan_make(16, 1 << 20, 4, 8, 9, 64), "experts_plan"),
-        (lambda: hip.experts_up_dev(8, 8, 2, 1.0, 8, 8, 16, 12, 64, 0, 8, 16, 8), "experts_up"),
+        (lambda: hip.experts_plan_make(16, 1 << 20, 4, 8, 33, 64), "experts_plan"),
+        (lambda: hip.gqa_step_dev(built.Gqa(4, 2, 2, 16, 32, 16, 32, 128, 1e-5, 0.1, 0.9, 8, 8, 8, 8, 8, sink=8), 8, 8, 8), "gqa: bad chunk, sink"),
+        (lambda: hip.gqa_step_dev(built.Gqa(4, 2, 1, 16, 32, 24, 32, 128, 1e-5, 0.1, 0.9, 8, 8, 8, 8, 8, values_are_keys=1), 8, 8, 8), "gqa: bad chunk, sink"),
+        (lambda: hip.gqa_step_dev(built.Gqa(4, 2, 1, 16, 32, 16, 32, 128, 1e-5, 0.1, 0.9, 8, 8, 8, 8, 8, rot_dims=18, rope_cos=8, rope_sin=8), 8, 8, 8), "gqa: bad rotation"),
+        (lambda: hip.dense_matmul_dev(8, 64, False, 8, 64, 4, 7, 64, 8, 8, False, act0=built.ACT_GATED), "gated"),
+        (lambda: hip.experts_up_dev(8, built.Router(8, 4, 13, 1.0), 8, 8, 16, 8, 64, 0, 8, 16, 8), "bad router"),
+        (lambda: hip.experts_up_dev(8, built.Router(8, 4, 2, 1.0), 8, 8, 16, 8, 64, 0, 8, 16, 8), "experts_up"),
+        (lambda: hip.experts_up_dev(8, built.Router(8, 0, 2, 1.0), 8, 8, 16, 12, 64, 0, 8, 16, 8), "experts_up"),
         (lambda: hip.experts_out_dev(8, 8, 64, 64, None, 8, 8, 8, 16, 64, 8, 2, 16, 8), "experts_out"),
-        (lambda: hip.sum_norm_rows_dev(built.SumRows(x=8, m=1, width=8, h=8, ldh=8)), "sum_norm_rows"),
+        (lambda: hip.sum_norm_rows_dev(built.SumRows(x=8, m=1, width=8, h=8, ldh=7)), "sum_norm_rows"),
         (lambda: hip.latent_decode_dev(built.LatentAttention(1, 20, 52, 16, 64, 16, 1.0, 8, 8, 8, 64, 32, 64, 8, 8), 8, 8, 8, 0, 1, True, 8), "bad shape"),
     ]
     for call, message in bad:
@@ -179,6 +211,37 @@ def test_oracle_delta_rule_by_hand():
     k, v = np.array([[1.0, 0.0], [1.0, 0.0]]), np.array([[2.0], [6.0]])
     o, S = so.delta_rule(k, k, v, np.array([1.0, 0.5]), np.array([1.0, 0.25]), np.zeros((2, 1)))
     assert np.allclose(o[:, 0], [2.0, 1.0 + 0.25 * (6.0 - 1.0)]) and np.allclose(S[:, 0], [2.25, 0.0])
+
+
+def test_oracle_chunks_and_sink():
+    """scores of zero: the mean over what a chunk shows so far and the sink's nothing"""
+    v = np.arange(1.0, 6.0).reshape(5, 1, 1)
+    o = so.chunk_softmax(np.ones((5, 2, 3)), np.zeros((5, 1, 3)), v, 1.0, 3)
+    assert np.allclose(o[:, :, 0].T, [1.0 / 2, 3.0 / 3, 6.0 / 4, 4.0 / 2, 9.0 / 3])
+    o = so.chunk_softmax(np.ones((1, 1, 2)), np.ones((1, 1, 2)), np.ones((1, 1, 1)), 0.5, 9)
+    assert np.isclose(o[0, 0, 0], math.e / (1.0 + math.e))
+
+
+def test_oracle_neighbours_turn_and_bands():
+    rot = {"dims": 4, "base": 10.0}
+    v = np.arange(12.0).reshape(2, 1, 6)
+    o = so.rotate_neighbours(v, rot)
+    assert np.array_equal(o[0], v[0]) and np.array_equal(o[1, :, 4:], v[1, :, 4:])
+    for i, f in enumerate((1.0, 10.0 ** -0.5)):
+        assert np.isclose(complex(*o[1, 0, 2 * i:2 * i + 2]), complex(*v[1, 0, 2 * i:2 * i + 2]) * np.exp(1j * f))
+    plain = so.banded_frequencies({"dims": 40, "base": 1000.0})
+    bands = so.banded_frequencies({"dims": 40, "base": 1000.0, "scaling": {"factor": 8.0, "low": 1.0, "high": 4.0, "original": 200}})
+    turns = 200 * plain / (2 * math.pi)
+    assert np.array_equal(bands[turns > 4], plain[turns > 4]) and np.allclose(bands[turns < 1], plain[turns < 1] / 8) and (turns > 4).any() and (turns < 1).any()
+    between = (turns > 1) & (turns < 4)
+    assert between.any() and np.allclose(bands[between], plain[between] * ((turns[between] - 1) / 3 * 7 / 8 + 1 / 8))
+
+
+def test_oracle_corrected_choice():
+    z = np.log(np.array([[0.1, 0.2, 0.3, 0.4]]))
+    ids, w = so.route_corrected(np.ones((1, 1)), z.T, np.array([0.35, 0.0, 0.0, -0.15]), 2)
+    assert ids.tolist() == [[0, 2]] and np.allclose(w, [[0.1, 0.3]])
+    assert np.allclose(so.gelu_tanh(np.array([-50.0, 0.0, 50.0])), [0.0, 0.0, 50.0]) and np.isclose(so.gelu_tanh(1.0), 0.841192, atol=1e-6)
 
 
 def test_oracle_convolution_and_routing():

@@ -33,9 +33,20 @@ MODELS = {
     "mimolix_wide": u.mimolix([u.attention_layer(heads=20, kv_heads=1, dim=150, vdim=200, scale=0.1), u.delta_layer(heads=2, kv_heads=1, dim=130, vdim=230, conv=3),
                                u.delta_layer(heads=2, kv_heads=2, dim=100, vdim=160, mlp=u.expert_mlp(experts=4, top=2, ff=100, shared=130))], width=136, vocab=77),
     "mimolix_huge": u.mimolix([u.attention_layer(heads=2, kv_heads=2, dim=300, vdim=270, scale=0.05), u.attention_layer(heads=4, kv_heads=2, dim=8, vdim=300)], width=64, vocab=50),
+    # chunks of several sizes, banded and plain rotation, all kinds of feed-forward and none
+    "lurepel": u.lurepel([u.chunk_layer(mlp=u.gated_mlp(), scaling=u.BANDS), u.chunk_layer(heads=4, kv_heads=1, dim=36, dims=36, chunk=64, mlp=u.corrected_mlp()),
+                          u.chunk_layer(chunk=150, scaling=dict(u.BANDS, factor=2.0, original=40)),
+                          u.chunk_layer(heads=5, kv_heads=5, dim=16, dims=2, chunk=100, mlp=u.corrected_mlp(experts=5, identity=1, top=4, ff=72))], width=120, vocab=170),
+    "lurepel_identities": u.lurepel([u.chunk_layer(heads=3, kv_heads=1, dim=64, dims=32, chunk=1, mlp=u.corrected_mlp(experts=2, identity=6, top=5, ff=16)),
+                                     u.chunk_layer(chunk=7, mlp=u.corrected_mlp(experts=1, identity=9, top=1, ff=130))], width=90, vocab=101, eps=1e-3),
+    "lurepel_dense": u.lurepel([u.chunk_layer(heads=2, kv_heads=2, dim=128, dims=128, chunk=1000, mlp=u.gated_mlp(71)), u.chunk_layer(dims=0, mlp=u.gated_mlp(8))], width=77, vocab=64),
+    "lurepel_wide": u.lurepel([u.chunk_layer(heads=20, kv_heads=1, dim=150, dims=64, chunk=40, scale=0.1, mlp=u.corrected_mlp(experts=70, identity=30, top=20, ff=8))],
+                              width=200, vocab=77),
+    "lurepel_huge": u.lurepel([u.chunk_layer(heads=4, kv_heads=2, dim=300, dims=210, chunk=33, scale=0.05, scaling=u.BANDS, mlp=u.corrected_mlp(experts=4, identity=0, top=4, ff=100))],
+                              width=64, vocab=50),
     "many_heads": u.lasapel([u.latent_layer(heads=19, dim=16, rot_dim=8, vdim=16, q_rank=40, kv_rank=136, ff=16)], width=64, vocab=500),
 }
-SEQUENCES = ["mixed", "mimolix"]  # the models of the tests about sequences
+SEQUENCES = ["mixed", "mimolix", "lurepel"]  # the models of the tests about sequences
 LIMIT = {"float32": 2e-5, "bfloat16": 6e-2}
 
 
@@ -198,7 +209,7 @@ def test_graph_replays_match_eager_steps(cases, dtype, name):
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-@pytest.mark.parametrize("name", ["mixed", "lightning_only", "many_heads", "mimolix", "mimolix_delta"])
+@pytest.mark.parametrize("name", ["mixed", "lightning_only", "many_heads", "mimolix", "mimolix_delta", "lurepel", "lurepel_identities"])
 def test_greedy_generation(cases, name, dtype):
     """generate(): each token is the argmax of the oracle's logits over what was generated so far (or as good as it)"""
     c = cases(name)
@@ -301,6 +312,78 @@ def test_one_far_key_of_one_map(pkg, hip, tmp_path, dtype, far):
         assert error(m.forward(tokens[-1:], [0]), want) < LIMIT[dtype]
     a, b = so.forward(config, t, base)[0][-1], so.forward(config, t, marked)[0][-1]
     assert u.rms_error(a - a.mean(), b - b.mean()) > 0.2  # the key shows
+    m.close()
+
+
+def one_key_chunked(root, chunk):
+    """One layer in which a marked token's query scores one other marked token far above all others; queries and keys of unit length point where
+    a column says: every token's own way, or the mark's."""
+    W, V, D = 32, 40, 8
+    config = u.lurepel([u.chunk_layer(heads=2, kv_heads=1, dim=D, scale=1.5, chunk=chunk, dims=2, base=1e6)], width=W, vocab=V, eps=1e-6)
+    t = u.random_tensors(config, 13)
+    t["embed"] = u.rounded(np.random.default_rng(10).standard_normal((V, W)) * 0.3)
+    t["embed"][:, :3] = 0.0
+    t["embed"][:, 0] = 2.0   # every token
+    t["embed"][1, 1] = 8.0   # the token looked for
+    t["embed"][2, 2] = 8.0   # the token that looks
+    for k in ("q", "k"):
+        t["l0.mix." + k] *= 0.02
+    for head in range(2):
+        t["l0.mix.q"][head * D + 4, 2] = 4.0
+    t["l0.mix.k"][4, 1], t["l0.mix.k"][5, 0] = 4.0, 2.0
+    t = {k: u.rounded(v) for k, v in t.items()}
+    return config, t, u.save_model(str(root), config, t)
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("chunk", [1, 2, 31, 64, 96, 100, 128, 130, 257, 399, 400, 5000])
+def test_keys_at_the_edge_of_a_chunk(pkg, hip, tmp_path, dtype, chunk):
+    """a marked key at the chunk's first position, beside it and near its query shows; one position ahead of the chunk and far ahead of it, it changes
+    no bit -- in whole prompts, at the end of portions and decoded"""
+    config, t, path = one_key_chunked(tmp_path, chunk)
+    n, p = 400, 399
+    first = p // chunk * chunk
+    base = np.random.default_rng(chunk).integers(3, 40, n).astype(np.int32)
+    base[-1] = 2
+    m = pkg.open_model(path, dtype, n + 8)
+
+    def last(tokens):
+        rows = []
+        for cut in (0, n - 1, n - 2, max(first - 1, 1), min(first + 1, n - 1)):
+            m.reset()
+            if cut:
+                m.forward(tokens[:cut], [])
+            rows.append(m.forward(tokens[cut:], [n - cut - 1])[0])
+        return np.stack(rows)
+
+    plain = last(base)
+    want = so.forward(config, t, base)[0][-1]
+    assert error(plain, np.broadcast_to(want, plain.shape)) < LIMIT[dtype]
+    for far in {0, first - 2, first - 1, first, first + 1, p - 1}:
+        if not 0 <= far < p:
+            continue
+        marked = base.copy()
+        marked[far] = 1
+        got, truth = last(marked), so.forward(config, t, marked)[0][-1]
+        assert error(got, np.broadcast_to(truth, got.shape)) < LIMIT[dtype]
+        if far < first:
+            assert np.array_equal(got, plain)
+        else:
+            assert u.rms_error(truth - truth.mean(), want - want.mean()) > 0.2
+    m.close()
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_decoding_across_chunks(pkg, hip, tmp_path, dtype):
+    """single tokens through several chunks, each compared; portions that end inside, at and behind an edge"""
+    config = u.lurepel([u.chunk_layer(chunk=48, scaling=u.BANDS), u.chunk_layer(chunk=65, heads=4, kv_heads=2, mlp=u.gated_mlp())], width=72, vocab=60)
+    t = u.random_tensors(config, 41)
+    m = pkg.open_model(u.save_model(str(tmp_path), config, t), dtype, 260)
+    tokens = tokens_of(config, 250, 12)
+    want = so.forward(config, t, tokens)[0]
+    for sizes in ([1], [47, 1, 1], [48], [49, 2], [65, 63, 2], [130, 1, 119], [200, 50]):
+        m.reset()
+        assert error(in_portions(m, tokens, sizes), want) < LIMIT[dtype], sizes
     m.close()
 
 
