@@ -109,7 +109,7 @@ class VectorInput(C.Structure):
 class SumRows(C.Structure):
     _fields_ = [("x", _vp), ("m", _sz), ("width", _sz), ("y", _vp), ("ldy", _sz), ("mult", C.c_float), ("expert_rows", _vp), ("ld_expert", _sz), ("top", _sz),
                 ("slots", _vp), ("slot_weights", _vp), ("weight", _vp), ("bias", _vp), ("x2", _vp), ("weight_offset", C.c_float), ("eps", C.c_float),
-                ("center", C.c_int32), ("h_f32", C.c_int32), ("h", _vp), ("ldh", _sz), ("post_weight", _vp), ("scale", _vp), ("input", _vp), ("ld_input", _sz)]
+                ("center", C.c_int32), ("h_f32", C.c_int32), ("h", _vp), ("ldh", _sz), ("post_weight", _vp), ("scale", _vp), ("input", _vp), ("ld_input", _sz), ("identity", C.c_int32)]
 
 
 class Gqa(C.Structure):

@@ -17,13 +17,23 @@ __global__ void k_embed_bf16(const uint16_t *__restrict__ table, size_t ld, cons
     tok = tok < 0 ? 0 : (tok >= vocab ? vocab - 1 : tok);
     if (norm_w) {
         const uint16_t *row = table + (size_t)tok * ld;
-        float ss = 0.f;
-        for (int i = threadIdx.x; i < width; i += 256) {
-            const float v = scale * bf2f(row[i]);
-            ss += v * v;
+        constexpr int NR = 16;  // rows of up to 4096 columns in registers, what lies behind is read again
+        float ss = 0.f, v[NR], w[NR];
+#pragma unroll
+        for (int j = 0; j < NR; ++j) {
+            const int i = threadIdx.x + 256 * j;
+            v[j] = i < width ? scale * bf2f(row[i]) : 0.f;
+            w[j] = i < width ? norm_w[i] : 0.f;
         }
+#pragma unroll
+        for (int j = 0; j < NR; ++j) ss += v[j] * v[j];
+        for (int i = threadIdx.x + 256 * NR; i < width; i += 256) ss += scale * bf2f(row[i]) * (scale * bf2f(row[i]));
         const float inv = 1.0f / sqrtf(group_sum<4>(ss, slot) / (float)width + eps);
-        for (int i = threadIdx.x; i < width; i += 256) out[(size_t)blockIdx.x * width + i] = scale * bf2f(row[i]) * inv * norm_w[i];
+        float *o = out + (size_t)blockIdx.x * width;
+#pragma unroll
+        for (int j = 0; j < NR; ++j)
+            if ((int)threadIdx.x + 256 * j < width) o[threadIdx.x + 256 * j] = v[j] * inv * w[j];
+        for (int i = threadIdx.x + 256 * NR; i < width; i += 256) o[i] = scale * bf2f(row[i]) * inv * norm_w[i];
         return;
     }
     for (int i = threadIdx.x; i < width; i += blockDim.x) out[(size_t)blockIdx.x * width + i] = scale * bf2f(table[(size_t)tok * ld + i]);
@@ -144,7 +154,8 @@ __device__ __forceinline__ void st4(uint16_t *p, size_t i, f32x4 v) {
 }
 constexpr int kSumRegs = 4;
 
-template <class T, bool VEC>
+// IDENTITY: slots may be negative.
+template <class T, bool VEC, bool IDENTITY>
 __global__ __launch_bounds__(256) void k_sum_norm_rows(SumRows p) {
     __shared__ float slot[4];
     const int tid = threadIdx.x, width = (int)p.width;
@@ -174,22 +185,36 @@ __global__ __launch_bounds__(256) void k_sum_norm_rows(SumRows p) {
                 a[j] = f32x4{0.f, 0.f, 0.f, 0.f};
                 if (y && i < n4) a[j] = ld4(y, 4 * i);
             }
+            float through = 0.f;
+#pragma unroll 4
             for (int k = 0; k < top; ++k) {
-                const int slot_k = slots[k];
                 const float w = sw[k];
-                if (slot_k < 0) {
+                const T *row;
+                if (IDENTITY) {  // (without a branch: an identity's place is taken by some row, which is not added)
+                    const int s = slots[k];
+                    row = er + (size_t)max(s, 0) * p.ld_expert;
+                    through += s < 0 ? w : 0.f;
 #pragma unroll
                     for (int j = 0; j < kSumRegs; ++j) {
                         const int i = tid + 256 * j;
-                        if (i < n4) a[j] += w * (input ? ld4(input, 4 * i) : v[j]);
+                        const f32x4 e = ld4(row, 4 * min(i, n4 - 1));
+                        a[j] += s < 0 || i >= n4 ? f32x4{0.f, 0.f, 0.f, 0.f} : w * e;
                     }
                     continue;
                 }
-                const T *row = er + (size_t)slot_k * p.ld_expert;
+                row = er + (size_t)slots[k] * p.ld_expert;
 #pragma unroll
                 for (int j = 0; j < kSumRegs; ++j) {
                     const int i = tid + 256 * j;
-                    if (i < n4) a[j] += w * ld4(row, 4 * i);
+                    const f32x4 e = ld4(row, 4 * min(i, n4 - 1));  // (no branch around the load: the rows' loads overlap)
+                    a[j] += i < n4 ? w * e : f32x4{0.f, 0.f, 0.f, 0.f};
+                }
+            }
+            if (IDENTITY && through != 0.f) {
+#pragma unroll
+                for (int j = 0; j < kSumRegs; ++j) {
+                    const int i = tid + 256 * j;
+                    if (i < n4) a[j] += through * (input ? ld4(input, 4 * i) : v[j]);
                 }
             }
             float post = 0.f;
@@ -256,7 +281,7 @@ __global__ __launch_bounds__(256) void k_sum_norm_rows(SumRows p) {
         if (y || top) {
             auto sum = [&](int i) {
                 float a = y ? y[i] : 0.f;
-                for (int k = 0; k < top; ++k) a += sw[k] * (slots[k] >= 0 ? ld_act(er + (size_t)slots[k] * p.ld_expert, i) : input ? ld_act(input, i) : x[i]);
+                for (int k = 0; k < top; ++k) a += sw[k] * (!IDENTITY || slots[k] >= 0 ? ld_act(er + (size_t)slots[k] * p.ld_expert, i) : input ? ld_act(input, i) : x[i]);
                 return a;
             };
             float post = 0.f;
@@ -297,7 +322,10 @@ __global__ __launch_bounds__(256) void k_sum_norm_rows(SumRows p) {
 hipError_t launch_sum_norm_rows(const SumRows &a, hipStream_t s) {
     // (four columns at a time: every row of every operand starts on its own alignment)
     const bool vec = a.width % 4 == 0 && a.width <= 1024 * kSumRegs && a.ldy % 4 == 0 && a.ld_expert % 4 == 0 && a.ldh % 4 == 0 && a.ld_input % 4 == 0;
-    auto fn = a.h_f32 ? (vec ? k_sum_norm_rows<float, true> : k_sum_norm_rows<float, false>) : (vec ? k_sum_norm_rows<uint16_t, true> : k_sum_norm_rows<uint16_t, false>);
+    auto pick = [&](auto all, auto some) { return a.identity ? some : all; };
+    auto fn = a.h_f32 ? (vec ? pick(k_sum_norm_rows<float, true, false>, k_sum_norm_rows<float, true, true>) : pick(k_sum_norm_rows<float, false, false>, k_sum_norm_rows<float, false, true>))
+                      : (vec ? pick(k_sum_norm_rows<uint16_t, true, false>, k_sum_norm_rows<uint16_t, true, true>)
+                             : pick(k_sum_norm_rows<uint16_t, false, false>, k_sum_norm_rows<uint16_t, false, true>));
     hipLaunchKernelGGL(fn, dim3(a.m), dim3(256), 0, s, a);
     return hipGetLastError();
 }

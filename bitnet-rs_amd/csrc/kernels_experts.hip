@@ -341,9 +341,13 @@ __global__ __launch_bounds__(256) void k_experts_out(OutK p) {
     __syncthreads();
     const int n_wg = gridDim.x;
     for (; g < p.groups; g += n_wg * 4) {
-        float acc[R];
+        float acc[R], more[R];
 #pragma unroll
-        for (int r = 0; r < R; ++r) acc[r] = 0.f;
+        for (int r = 0; r < R; ++r) {
+            const int row = min((g * G + sub) * R + r, a.rows - 1);
+            acc[r] = 0.f;
+            more[r] = (a.bias ? a.bias[row] : 0.f) + (a.identity ? through * a.input[row] : 0.f);
+        }
         for (int c0 = 0; c0 < steps; c0 += U) {
             u32x4 c[U][R];
 #pragma unroll
@@ -361,7 +365,7 @@ __global__ __launch_bounds__(256) void k_experts_out(OutK p) {
         for (int r = 0; r < R; ++r) {
             const float v = lanes_sum<LPR>(acc[r]);
             const int row = (g * G + sub) * R + r;
-            if (l == 0 && row < a.rows) a.y[row] = v + (a.bias ? a.bias[row] : 0.f) + (a.identity ? through * a.input[row] : 0.f);
+            if (l == 0 && row < a.rows) a.y[row] = v + more[r];
         }
     }
 }
@@ -430,8 +434,9 @@ static hipError_t out_go(const ExpertsOut &a, hipStream_t s) {
 
 hipError_t launch_experts_out(const ExpertsOut &a, hipStream_t s) {
     auto waste = [&](int ch) { return (double)((a.cols0 + ch - 1) / ch * ch + (long)a.top * ((a.cols1 + ch - 1) / ch * ch)) / (a.cols0 + (double)a.top * a.cols1); };
-    // the longest rows of lanes whose chunks are not padding for the most part
-    return waste(512) <= 1.1 * waste(256) ? out_go<64, 1>(a, s) : waste(256) <= 1.3 * waste(128) ? out_go<32, 1>(a, s) : out_go<16, 1>(a, s);
+    auto fits = [&](int ch) { return ((a.cols0 + ch - 1) / ch + (long)a.top * ((a.cols1 + ch - 1) / ch) + 7) / 8 * 8 * ch * 4 <= 150 * 1024; };
+    // the longest rows of lanes whose chunks are not padding for the most part (lanes past a row's end load its last columns again: no traffic)
+    return waste(512) <= 1.4 * waste(256) && fits(512) ? out_go<64, 1>(a, s) : waste(256) <= 1.3 * waste(128) && fits(256) ? out_go<32, 1>(a, s) : out_go<16, 1>(a, s);
 }
 
 }  // namespace bitnet_hip

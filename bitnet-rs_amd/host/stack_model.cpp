@@ -855,7 +855,7 @@ int StackModel::portion_norm(size_t n, const Norm *norm, const float *x2, void *
     r.center = spec_.center, r.h_f32 = f32_, r.h = h, r.ldh = ldh, r.x2 = x2;
     if (norm) r.weight = norm->w, r.bias = norm->bias;
     if (!post) {
-        r.y = p.y, r.ldy = width_, r.post_weight = p.w, r.scale = p.scale, r.input = p.input, r.ld_input = p.input ? up_to(width_, 64) : 0;
+        r.y = p.y, r.ldy = width_, r.post_weight = p.w, r.scale = p.scale, r.identity = p.identity, r.input = p.input, r.ld_input = p.input ? up_to(width_, 64) : 0;
         if (p.experts) r.expert_rows = peout_.p, r.ld_expert = up_to(width_, 64), r.top = plan_.top, r.slots = plan_.slots, r.slot_weights = plan_.weights;
     }
     BCHK(bitnet_hip_sum_norm_rows_dev(&r, stream_));
@@ -988,7 +988,7 @@ int StackModel::portion(int rows, int pos0) {
         if (run.enters) TRY(portion_loop_in(n));
         TRY(portion_norm(n, &L.norm1, nullptr, ph_.p, ldh));
         TRY(L.block[0].used ? portion_block(i, run.pass, 0, n, pos0) : S.mixer == LayerSpec::Latent ? portion_latent(i, run.pass, n, pos0) : portion_linear(i, run.pass, n));
-        pending_ = {y, L.norm1b, L.ls1, L.block[0].expert_up.w != nullptr, L.norm1.w ? ph_.p : nullptr};
+        pending_ = {y, L.norm1b, L.ls1, L.block[0].expert_up.w != nullptr, L.norm1.w ? ph_.p : nullptr, S.experts.identity > 0};
         if (S.parallel || (S.ff == 0 && S.experts.count == 0)) continue;
         TRY(portion_norm(n, &L.norm2, nullptr, ph_.p, ldh));
         if (L.block[1].used) {
@@ -998,7 +998,7 @@ int StackModel::portion(int rows, int pos0) {
             TRY(matmul(pact_.p, L.down.ld, f32_, L.down, L.down_b, n, 0, 0, 0, py_.p, width_, true));
         }
         const bool routed = L.block[1].expert_up.w != nullptr;
-        pending_ = {routed && !L.block[1].out.w ? nullptr : y, L.norm2b, L.ls2, routed, L.norm2.w ? ph_.p : nullptr};
+        pending_ = {routed && !L.block[1].out.w ? nullptr : y, L.norm2b, L.ls2, routed, L.norm2.w ? ph_.p : nullptr, S.experts.identity > 0};
     }
     TRY(portion_norm(n, nullptr, nullptr, nullptr, 0));
     hidden_ = x + (n - 1) * (size_t)width_;

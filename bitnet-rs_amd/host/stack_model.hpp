@@ -182,6 +182,7 @@ class StackModel : public Sequence {
         const float *y = nullptr, *w = nullptr, *scale = nullptr;
         bool experts = false;         // a portion's routed rows join in (y may be missing)
         const void *input = nullptr;  // what those experts read, if not the residual stream
+        bool identity = false;        // some of them hand it through
     };
     struct Run {
         size_t layer;

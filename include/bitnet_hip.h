@@ -589,8 +589,8 @@ int bitnet_hip_residual_norm_rows_dev(float *x_dev, const float *y_dev, size_t l
                                       const float *next_weight_dev, float weight_offset, float eps, size_t m, size_t width, void *h_dev,
                                       size_t ldh, int h_f32, void *stream);
 /* Rows of a block whose sublayers' outputs add up: t = y[i] + sum over k < top of slot_weights[i][k] * expert_rows[slots[i][k]] (y NULL: the
- * experts' rows alone; top 0: no experts; neither: nothing is added; a negative slot stands for the row input[i], or -- input NULL -- for x[i]
- * as it was), x[i] += mult * t or -- post_weight given -- scale * t / sqrt(mean(t^2) + eps) * (weight_offset + post_weight).  Then h[i] (NULL:
+ * experts' rows alone; top 0: no experts; neither: nothing is added; with `identity` a negative slot stands for the row input[i], or -- input
+ * NULL -- for x[i] as it was), x[i] += mult * t or -- post_weight given -- scale * t / sqrt(mean(t^2) + eps) * (weight_offset + post_weight).  Then h[i] (NULL:
  * skipped) = norm(x[i]; weight) (weight NULL: x[i] itself), padding columns zero, or -- x2 given -- the unnormed [x[i]; x2[i]].  center: norm
  * is a layer norm, (v - mean) / sqrt(variance + eps) * weight + bias. */
 typedef struct bitnet_hip_sum_rows {
@@ -611,6 +611,7 @@ typedef struct bitnet_hip_sum_rows {
     const float *post_weight, *scale; /* scale NULL: 1 */
     const void *input;                /* of the expert rows' type; may be h */
     size_t ld_input;
+    int32_t identity;
 } bitnet_hip_sum_rows;
 int bitnet_hip_sum_norm_rows_dev(const bitnet_hip_sum_rows *rows, void *stream);
 /* h[i] = norm(o[i]; weight) * gate[i] over n columns; the mean divides by mean_n (padded heads hold zeros). */

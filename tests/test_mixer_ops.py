@@ -114,7 +114,7 @@ def test_sum_norm_rows_behind_experts(hip, pkg, width, f32):
     def run(h, **kw):
         xd = u.dev_f32(x)
         r = pkg.SumRows(x=xd.data_ptr(), m=m, width=width, eps=eps, h_f32=f32, h=h.data_ptr(), ldh=ldh, expert_rows=p[0], ld_expert=ldh, top=top, slots=p[1],
-                        slot_weights=p[2], **kw)
+                        slot_weights=p[2], identity=1, **kw)
         hip.sum_norm_rows_dev(r)
         return u.host(xd), u.host(h)
 
