@@ -77,7 +77,8 @@ int bitnet_hip_gqa_supported(size_t dimp, size_t vdimp) { return dimp <= 65536 &
 int bitnet_hip_gqa_rows_dev(const bitnet_hip_gqa *a, void *rows, size_t ld, int rows_f32, int cache_f32, const int32_t *pos, size_t n, void *stream) {
     BH_GUARD_BEGIN
     if (int rc = check_gqa(a)) return rc;
-    BH_REQUIRE(rows && pos && n > 0 && n <= a->capacity && ld >= gqa_row(a) && (rows_f32 || !cache_f32), "gqa_rows: bad arguments");
+    BH_REQUIRE(rows && pos && n > 0 && n <= a->capacity && ld >= gqa_row(a) && (n == 1 || ld % 8 == 0) && (uintptr_t)rows % 16 == 0 && (rows_f32 || !cache_f32), "gqa_rows: bad arguments");
+    BH_REQUIRE((a->heads + a->kv_heads) * a->maps + a->kv_heads * (a->vdimp / 32) < 65536, "gqa_rows: too many heads");
     BH_CHECK_DIMS(n, ld);
     BH_HIP_TRY(launch_gqa_rows(*a, rows, ld, rows_f32, cache_f32, pos, (int)n, (hipStream_t)stream));
     return BITNET_HIP_OK;

@@ -52,24 +52,33 @@ __device__ __forceinline__ void choose(float (&s)[PL], const Router &r, int &id,
     id = 0, weight = 0.f;
     float chosen = 0.f;
     for (int k = 0; k < top; ++k) {
-        float best = -INFINITY, mine_w = 0.f;
+        float best = -INFINITY;
         int at = 0;
 #pragma unroll
         for (int j = 0; j < PL; ++j)
-            if (s[j] > best) best = s[j], mine_w = score[j], at = j;
-        float w = token_max<LT>(best);
+            if (s[j] > best) best = s[j], at = j;
+        const float w = token_max<LT>(best);
         unsigned long long who = __ballot(best == w) >> base;
         if (LT < 64) who &= (1ull << LT) - 1;
         const int winner = who ? __builtin_ctzll(who) : 0;  // (no score compares equal to itself if a logit is not a number)
         const int mine = l * PL + at;
         const int e = min(LT == 64 ? __builtin_amdgcn_readlane(mine, winner) : __shfl(mine, base + winner, 64), experts - 1);
-        if (r.correction) w = __shfl(mine_w, base + winner, 64);
         if (l == k) id = e, weight = w;
         chosen += w;
         if (l == winner)
 #pragma unroll
             for (int j = 0; j < PL; ++j)
                 if (j == at) s[j] = -INFINITY;
+    }
+    if (r.correction) {  // the scores of what was chosen
+        float w = 0.f;
+#pragma unroll
+        for (int j = 0; j < PL; ++j) {
+            const float t = __shfl(score[j], base + id / PL, 64);
+            w = id % PL == j ? t : w;
+        }
+        weight = l < top ? w : 0.f;
+        chosen = token_sum<LT>(weight);
     }
     weight = (r.raw ? weight : weight / (chosen + 1e-20f)) * r.scale;
 }

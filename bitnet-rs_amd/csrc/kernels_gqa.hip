@@ -47,30 +47,92 @@ __device__ __forceinline__ float turn_neighbours(float v, int i, const float *cs
     const float c = cs[i >> 1], s = sn[i >> 1];
     return (i & 1) ? v * c + o * s : v * c - o * s;
 }
-__device__ __forceinline__ float head_gate(const Gqa &p, int row, int h) {
-    if (!p.gate) return 1.0f;
+// what a head's gate is the sigmoid of
+__device__ __forceinline__ float gate_logit(const Gqa &p, int row, int h) {
     const size_t i = (size_t)row * p.ldgate + h;
-    const float z = p.gate_f32 ? ((const float *)p.gate)[i] : bf2f(((const uint16_t *)p.gate)[i]);
-    return 1.0f / (1.0f + expf(-z));
+    return p.gate_f32 ? ((const float *)p.gate)[i] : bf2f(((const uint16_t *)p.gate)[i]);
 }
 
 size_t gqa_scratch_floats(size_t heads, size_t maps, size_t vdimp, size_t nq) { return nq * heads * maps * kGqaSplits * (kGqaRecHead + vdimp); }
 bool gqa_supported(int dimp, int vdimp) { return dimp <= 256 && vdimp <= 256; }
 
 // ---- rows of projections ----------------------------------------------------------------------------------------------
-// blockIdx.y: query heads x maps, key heads x maps, value heads; 64 tokens per workgroup
+// blockIdx.y: query heads x maps, key heads x maps (sixteen tokens per workgroup, four per wave), then value heads in groups of 32 columns (64
+// tokens, every fourth workgroup).
+constexpr int kRowTokens = 16, kRowCols = 32;
+
+// four tokens of a query or key head of up to 256 columns: a lane holds neighbouring elements, so that a pair turns within it
+template <class TR, class TC>
+__device__ __forceinline__ void head_rows(const Gqa &p, TR *rows, size_t ld, int pos0, int t0, int n, int y, bool key, TC *cache) {
+    constexpr int U = kRowTokens / 4, NJ = 2;
+    const int lane = threadIdx.x & 63, dim = (int)p.dim, dimp = (int)p.dimp, turned = (int)p.rot_dims, half = turned >> 1;
+    const float *w = key ? p.k_weight : p.q_weight;
+    float v[U][NJ][2], cs[U][NJ], sn[U][NJ], factor[U];
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+        const int t = min(t0 + u, n - 1);
+        const TR *row = rows + (size_t)t * ld + (size_t)y * dimp;
+        factor[u] = key ? 1.0f : p.q_factor[pos0 + t];
+#pragma unroll
+        for (int j = 0; j < NJ; ++j) {
+            const int i = min(2 * lane + 128 * j, dimp - 2);
+            v[u][j][0] = ld_act(row, i), v[u][j][1] = ld_act(row, i + 1);
+            cs[u][j] = 1.0f, sn[u][j] = 0.f;
+            if (turned && 2 * lane + 128 * j < turned) {
+                const size_t at = (size_t)(pos0 + t) * half + lane + 64 * j;
+                cs[u][j] = p.rope_cos[at], sn[u][j] = p.rope_sin[at];
+            }
+        }
+    }
+    float wv[NJ][2];
+#pragma unroll
+    for (int j = 0; j < NJ; ++j)
+#pragma unroll
+        for (int e = 0; e < 2; ++e) wv[j][e] = w && 2 * lane + 128 * j + e < dim ? w[2 * lane + 128 * j + e] : 1.0f;  // (padding columns hold zeros)
+#pragma unroll
+    for (int u = 0; u < U; ++u) {
+        if (w || p.unit_norm) {
+            float ss = 0.f;
+#pragma unroll
+            for (int j = 0; j < NJ; ++j) ss += 2 * lane + 128 * j < dimp ? v[u][j][0] * v[u][j][0] + v[u][j][1] * v[u][j][1] : 0.f;
+            factor[u] *= 1.0f / sqrtf(wave_sum(ss) / (float)dim + p.eps);
+        }
+        if (t0 + u >= n) continue;
+        TR *row = rows + (size_t)(t0 + u) * ld + (size_t)y * dimp;
+#pragma unroll
+        for (int j = 0; j < NJ; ++j) {
+            const int i = 2 * lane + 128 * j;
+            if (i >= dimp) continue;
+            const float a = v[u][j][0] * factor[u] * wv[j][0], b = v[u][j][1] * factor[u] * wv[j][1];
+            const float x = a * cs[u][j] - b * sn[u][j], z = b * cs[u][j] + a * sn[u][j];
+            if (key) {
+                TC *dst = cache + (size_t)(pos0 + t0 + u) * dimp;
+                st_act(dst, i, x), st_act(dst, i + 1, z);
+            } else {
+                st_act(row, i, x), st_act(row, i + 1, z);
+            }
+        }
+    }
+}
+
 template <class TR, class TC>
 __global__ __launch_bounds__(256) void k_gqa_rows(Gqa p, TR *rows, size_t ld, const int *pos_ptr, int n) {
-    extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
-    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, pos0 = *pos_ptr, t0 = blockIdx.x * 64;
+    constexpr int STRIDE = sizeof(TR) == 4 ? kRowCols + 1 : kRowCols + 2;
+    __shared__ __attribute__((aligned(16))) TR tile[64 * STRIDE];
+    const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, pos0 = *pos_ptr;
     const int nq = (int)(p.heads * p.maps), nk = (int)(p.kv_heads * p.maps), dim = (int)p.dim, dimp = (int)p.dimp, vdimp = (int)p.vdimp;
     int y = blockIdx.y;
     if (y < nq + nk) {
         const bool key = y >= nq;
         const float *w = key ? p.k_weight : p.q_weight;
-        const int turned = (int)p.rot_dims, half = turned >> 1;
+        const int turned = (int)p.rot_dims, half = turned >> 1, t0 = blockIdx.x * kRowTokens + wave * (kRowTokens / 4);
         TC *cache = key ? (TC *)p.kcache + (size_t)(y - nq) * p.capacity * dimp : nullptr;
-        for (int t = t0 + wave; t < min(t0 + 64, n); t += 4) {
+        if (t0 >= n) return;
+        if (dimp <= 256) {
+            head_rows<TR, TC>(p, rows, ld, pos0, t0, n, y, key, cache);
+            return;
+        }
+        for (int t = t0; t < min(t0 + kRowTokens / 4, n); ++t) {
             TR *row = rows + (size_t)t * ld + (size_t)y * dimp;
             float ss = 0.f;
             for (int i = lane; i < dimp; i += 64) {
@@ -81,7 +143,7 @@ __global__ __launch_bounds__(256) void k_gqa_rows(Gqa p, TR *rows, size_t ld, co
             const float factor = key ? norm : norm * p.q_factor[pos0 + t];
             const float *cs = p.rope_cos + (size_t)(pos0 + t) * half, *sn = p.rope_sin + (size_t)(pos0 + t) * half;
             for (int i = lane; i < dimp; i += 64) {
-                float v = ld_act(row, i) * factor * (w && i < dim ? w[i] : 1.0f);  // (padding columns hold zeros)
+                float v = ld_act(row, i) * factor * (w && i < dim ? w[i] : 1.0f);
                 if (turned) v = turn_neighbours(v, i, cs, sn, turned);
                 if (key)
                     st_act(cache + (size_t)(pos0 + t) * dimp, i, v);
@@ -91,30 +153,34 @@ __global__ __launch_bounds__(256) void k_gqa_rows(Gqa p, TR *rows, size_t ld, co
         }
         return;
     }
+    if (blockIdx.x % (64 / kRowTokens)) return;
     y -= nq + nk;
-    TR *tile = (TR *)lds;  // [64][vdimp + 2]
-    const int stride = vdimp + 2, count = min(64, n - t0);
-    const TR *src = rows + (size_t)(p.values_are_keys ? nq : nq + nk) * dimp + (size_t)y * vdimp;
-    for (int i = tid; i < count * vdimp; i += 256) {
-        const int t = i / vdimp, v = i - t * vdimp;
-        tile[t * stride + v] = src[(size_t)(t0 + t) * ld + v];
+    const int t0 = blockIdx.x * kRowTokens, groups = vdimp / kRowCols, head = y / groups, c0 = (y - head * groups) * kRowCols, count = min(64, n - t0);
+    const TR *src = rows + (size_t)(p.values_are_keys ? nq : nq + nk) * dimp + (size_t)head * vdimp + c0;
+    constexpr int V = 16 / sizeof(TR), PER = kRowCols / V;
+#pragma unroll
+    for (int j = 0; j < 64 * PER / 256; ++j) {
+        const int i = tid + 256 * j, t = i / PER, c = i % PER * V;
+        if (t < count) {
+            const u32x4 x = *reinterpret_cast<const u32x4 *>(src + (size_t)(t0 + t) * ld + c);
+            uint32_t *dst = reinterpret_cast<uint32_t *>(tile + t * STRIDE + c);
+            dst[0] = x.x, dst[1] = x.y, dst[2] = x.z, dst[3] = x.w;
+        }
     }
     __syncthreads();
-    TC *cache = (TC *)p.vcache + (size_t)y * vdimp * p.capacity + pos0 + t0;
+    TC *cache = (TC *)p.vcache + ((size_t)head * vdimp + c0) * p.capacity + pos0 + t0;
     if (lane < count)
-        for (int v = wave; v < vdimp; v += 4) st_act(cache + (size_t)v * p.capacity, lane, ld_act(tile, lane * stride + v));
+#pragma unroll
+        for (int j = 0; j < kRowCols / 4; ++j) {
+            const int v = wave * (kRowCols / 4) + j;
+            st_act(cache + (size_t)v * p.capacity, lane, ld_act(tile, lane * STRIDE + v));
+        }
 }
 
 hipError_t launch_gqa_rows(const Gqa &g, void *rows, size_t ld, int rows_f32, int cache_f32, const int *pos, int n, hipStream_t s) {
-    const dim3 grid((n + 63) / 64, g.heads * g.maps + g.kv_heads * g.maps + g.kv_heads);
-    const size_t lds = 64 * (g.vdimp + 2) * (rows_f32 ? 4 : 2);
-    if (lds > 160 * 1024) return hipErrorInvalidValue;
+    const dim3 grid((n + kRowTokens - 1) / kRowTokens, (g.heads + g.kv_heads) * g.maps + g.kv_heads * (g.vdimp / kRowCols));
     auto go = [&](auto fn, auto *r) {
-        if (lds > 65536) {
-            const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(fn), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
-            if (e != hipSuccess) return e;
-        }
-        hipLaunchKernelGGL(fn, grid, dim3(256), lds, s, g, r, ld, pos, n);
+        hipLaunchKernelGGL(fn, grid, dim3(256), 0, s, g, r, ld, pos, n);
         return hipGetLastError();
     };
     if (rows_f32) return cache_f32 ? go(k_gqa_rows<float, float>, (float *)rows) : go(k_gqa_rows<float, uint16_t>, (float *)rows);
@@ -419,8 +485,8 @@ __global__ __launch_bounds__(256) void k_gqa_merge(Gqa p, const int *pos_ptr, in
     static_assert(kGqaSplits == 128, "two records per lane of a wave");
     __shared__ float ws[2][kGqaSplits], sinv[2], slot[4];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, h = blockIdx.x, qi = blockIdx.z, maps = (int)p.maps, vdimp = (int)p.vdimp;
+    const float z = p.gate ? gate_logit(p, qi, h) : 0.f, sink = p.sink ? p.sink[h] * kLog2e : -INFINITY;  // (ahead of the chain that starts with the position)
     const int used = gqa_range(p, *pos_ptr + q0 + qi).used;
-    const float gate = head_gate(p, qi, h);
     const size_t stride = kGqaRecHead + vdimp;
     const float *rec = scratch + ((size_t)qi * p.heads + h) * maps * kGqaSplits * stride;
     if (wave < maps) {
@@ -432,7 +498,7 @@ __global__ __launch_bounds__(256) void k_gqa_merge(Gqa p, const int *pos_ptr, in
             mv[e] = i < used ? r[i * stride] : -INFINITY;
             lv[e] = i < used ? r[i * stride + 1] : 0.f;
         }
-        const float sink = p.sink ? p.sink[h] * kLog2e : -INFINITY, M = fmaxf(sink, rows_max(row_max(fmaxf(mv[0], mv[1]))));
+        const float M = fmaxf(sink, rows_max(row_max(fmaxf(mv[0], mv[1]))));
         float den = 0.f;
 #pragma unroll
         for (int e = 0; e < 2; ++e) {
@@ -441,9 +507,10 @@ __global__ __launch_bounds__(256) void k_gqa_merge(Gqa p, const int *pos_ptr, in
             den += w * lv[e];
         }
         den = wave_sum(den) + (p.sink ? exp2f(sink - M) : 0.f);
-        if (lane == 0) sinv[wave] = (maps == 1 ? gate : 1.0f) / den;
+        if (lane == 0) sinv[wave] = 1.0f / den;
     }
     __syncthreads();
+    const float gate = p.gate ? activate(z, BITNET_HIP_ACT_SIGMOID) : 1.0f;
     // 32 lanes of four columns; eight groups share maps and records
     const int grp = tid >> 5, gm = maps == 2 ? grp & 1 : 0, gs = maps == 2 ? grp >> 1 : grp, gn = maps == 2 ? 4 : 8;
     for (int i = (tid & 31) * 4; i < vdimp; i += 128) {
@@ -462,7 +529,7 @@ __global__ __launch_bounds__(256) void k_gqa_merge(Gqa p, const int *pos_ptr, in
             float t = 0.f;
 #pragma unroll
             for (int k = 0; k < 8; ++k) t += part[k * vdimp + i];
-            return t * sinv[0];
+            return t * (sinv[0] * gate);
         }
         const float a = (part[i] + part[2 * vdimp + i]) + (part[4 * vdimp + i] + part[6 * vdimp + i]);
         const float b = (part[vdimp + i] + part[3 * vdimp + i]) + (part[5 * vdimp + i] + part[7 * vdimp + i]);
@@ -647,7 +714,7 @@ __global__ __launch_bounds__(256, NV > 8 || NK > 4 ? 1 : 2) void k_gqa_prefill(G
     for (int t = 0; t < SLOTS; ++t) inv[t] = 1.0f / rows_sum(l[t]);
     if (p.gate)
 #pragma unroll
-        for (int t = 0; t < SLOTS / MAPS; ++t) gate[t] = head_gate(p, min(qw + t * 16 + r16, nq - 1), h);
+        for (int t = 0; t < SLOTS / MAPS; ++t) gate[t] = activate(gate_logit(p, min(qw + t * 16 + r16, nq - 1), h), BITNET_HIP_ACT_SIGMOID);
     if (MAPS == 2) {
         float ss = 0.f;
 #pragma unroll
