@@ -87,9 +87,6 @@ def build(force: bool = False, verbose: bool = False, diag: bool = False) -> str
             return _build(force, verbose, OBJ_DIR + "_sched_" + sf, LIB_PATH.replace(".so", f"_ablatesched{sf.replace('-', '')}.so"), ["-DBH_SCHED_VARIANT"])
         finally:
             EXTRA.pop("kernels_gemm.hip", None)
-    ab = os.environ.get("BH_ABLATE")  # developer builds of kernels_gemm.hip with parts of the loop removed (tools/ablate_gemm.py)
-    if ab:
-        obj_dir, lib_path, extra_all = OBJ_DIR + "_ablate" + ab, LIB_PATH.replace(".so", f"_ablate{ab}.so"), [f"-DBH_ABLATE={ab}", "-DBH_STAMPS"]
     return _build(force, verbose, obj_dir, lib_path, extra_all)
 
 

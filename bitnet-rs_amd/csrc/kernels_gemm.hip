@@ -711,11 +711,7 @@ __global__ __launch_bounds__(256 * CW, MINW) void k_gemm_mfma(GemmArgs p) {
             // reads the other buffer): stage tile blk + 1 there now, then start the loads of tile blk + 2
             bcur = bread + (blk & 1) * kBuf;
             uint8_t *nxt = lds + ((blk + 1) & 1) * kBuf;
-#if defined(BH_ABLATE) && (BH_ABLATE & 4)  // developer build: no LDS staging stores
-            if (blk + 1 < p.nblk && p.m < 0) {
-#else
             if (blk + 1 < p.nblk) {
-#endif
 #pragma unroll
                 for (int i = 0; i < NB; ++i) *reinterpret_cast<gv4u *>(nxt + bdst[i]) = bn[i];
             }
@@ -725,14 +721,10 @@ __global__ __launch_bounds__(256 * CW, MINW) void k_gemm_mfma(GemmArgs p) {
         for (int rt = 0; rt < 4; ++rt) wc[rt] = wn[rt];
         if (!WS) {
             const int n1 = blk + 1 < p.nblk ? blk + 1 : p.nblk - 1, n2 = blk + 2 < p.nblk ? blk + 2 : p.nblk - 1;
-#if !(defined(BH_ABLATE) && (BH_ABLATE & 32))  // developer build: no weight loads in the loop
 #pragma unroll
             for (int rt = 0; rt < 4; ++rt) wn[rt] = *reinterpret_cast<const gv4u *>(wptr[rt] + (size_t)n1 * 1024);  // next step's weights
-#endif
-#if !(defined(BH_ABLATE) && (BH_ABLATE & 8))  // developer build: no activation tile loads
 #pragma unroll
             for (int i = 0; i < NB; ++i) bn[i] = *reinterpret_cast<const gv4u *>(bsrc[i] + (size_t)n2 * 256);
-#endif
         }
         if (WS == 3) {
 #pragma unroll
@@ -794,19 +786,11 @@ __global__ __launch_bounds__(256 * CW, MINW) void k_gemm_mfma(GemmArgs p) {
 #pragma unroll
                 for (int rt = 0; rt < 4; ++rt) {
                     const uint32_t wd = m == 0 ? wc[rt].x : m == 1 ? wc[rt].y : m == 2 ? wc[rt].z : wc[rt].w;
-#if defined(BH_ABLATE) && (BH_ABLATE & 2)  // developer build: no code expansion
-                    a[rt] = (v4i){(int)wd, (int)(wd >> 1), (int)(wd >> 2), (int)(wd >> 3)};
-#else
                     a[rt] = gdecode16(wd, p.lut);
-#endif
                 }
 #pragma unroll
                 for (int ct = 0; ct < CT; ++ct) {
-#if defined(BH_ABLATE) && (BH_ABLATE & 1)  // developer build: no LDS operand reads
-                    const v4i b = (v4i){ct + blk, m, ct, 1};
-#else
                     const v4i b = *reinterpret_cast<const v4i *>(bcur + ct * 16 * CSTR + moff[m]);
-#endif
 #pragma unroll
                     for (int rt = 0; rt < 4; ++rt) acc[rt][ct] = __builtin_amdgcn_mfma_i32_16x16x64_i8(a[rt], b, acc[rt][ct], 0, 0, 0);
                 }
@@ -850,9 +834,7 @@ __global__ __launch_bounds__(256 * CW, MINW) void k_gemm_mfma(GemmArgs p) {
                 }
             }
         }
-#if !(defined(BH_ABLATE) && (BH_ABLATE & 16))  // developer build: no barrier per K step
         if (!WS) __syncthreads();  // every wave is done with buffer blk & 1
-#endif
         if (WS == 1) {
             // one f32 weight scale per (row, 256-block): fold this block's exact sums into f32
 #pragma unroll
@@ -1382,11 +1364,7 @@ __global__ __launch_bounds__(256, 2) void k_gemm_f16a(GemmArgs p, uint32_t lut_h
             for (int rt = 0; rt < RT; ++rt) wn[rt] = *reinterpret_cast<const gv4u *>(wptr[rt] + (size_t)n1 * 1024);
             if (FMT == 1) {
 #pragma unroll
-#if defined(BH_ABLATE) && (BH_ABLATE & 4)  // developer build: no scale loads in the loop
-                for (int rt = 0; rt < RT; ++rt) sn[rt] = 0x3C003C00u + (uint32_t)n1;
-#else
                 for (int rt = 0; rt < RT; ++rt) sn[rt] = sptr[rt][(size_t)n1 * 64];
-#endif
             }
 #pragma unroll
             for (int i = 0; i < NB; ++i) bn[i] = *reinterpret_cast<const gv4u *>(bsrc[i] + (size_t)n2 * 512);
@@ -1405,19 +1383,11 @@ __global__ __launch_bounds__(256, 2) void k_gemm_f16a(GemmArgs p, uint32_t lut_h
                     const uint32_t wd = m == 0 ? wc[rt].x : m == 1 ? wc[rt].y : m == 2 ? wc[rt].z : wc[rt].w;
                     // (s, s) of this lane's 32-block 2 g + (m >> 1): low / high half of its scale dword
                     const gh2 s2 = __builtin_bit_cast(gh2, __builtin_amdgcn_perm(0u, sc[rt], (m >> 1) ? 0x03020302u : 0x01000100u));
-#if defined(BH_ABLATE) && (BH_ABLATE & 2)  // developer build: no code expansion
-                    a[rt] = __builtin_bit_cast(gh8, (gv4u){wd, wd >> (h + 1), sc[rt], wd ^ lut_hi});
-#else
                     a[rt] = expand8_f16<FMT>(wd, h, lut_hi, s2);
-#endif
                 }
 #pragma unroll
                 for (int ct = 0; ct < TTW; ++ct) {
-#if defined(BH_ABLATE) && (BH_ABLATE & 1)  // developer build: no LDS operand reads
-                    const gh8 b = __builtin_bit_cast(gh8, (gv4u){(unsigned)(ct + blk), (unsigned)m, (unsigned)h, 1u});
-#else
                     const gh8 b = *reinterpret_cast<const gh8 *>(bcur + ct * 16 * ROWB + boff[2 * m + h]);
-#endif
 #pragma unroll
                     for (int rt = 0; rt < RT; ++rt) acc[rt][ct] = __builtin_amdgcn_mfma_f32_16x16x32_f16(a[rt], b, acc[rt][ct], 0, 0, 0);
                 }
@@ -1930,11 +1900,7 @@ __global__ __launch_bounds__(256, 2) void k_gemm_fp6w(GemmArgs p) {
     const int bread = (g * T + wt * 32 + c) * 144;
     for (int blk = 0; blk < p.nblk; ++blk) {
         const uint8_t *bcur = lds + (blk & 1) * kBuf + bread;
-#if defined(BH_ABLATE) && (BH_ABLATE & 128)
-        if (blk + 1 < p.nblk && p.m == 12345) stage(blk + 1, (blk + 1) & 1);
-#else
         if (blk + 1 < p.nblk) stage(blk + 1, (blk + 1) & 1);  // (every wave is past the barrier that ended step blk - 1: nobody reads that buffer)
-#endif
         v4i a[2][RT];
 #pragma unroll
         for (int rt = 0; rt < RT; ++rt)
@@ -1942,9 +1908,6 @@ __global__ __launch_bounds__(256, 2) void k_gemm_fp6w(GemmArgs p) {
             for (int m = 0; m < 2; ++m) a[m][rt] = wn[m][rt];
         {
             const int n1 = blk + 1 < p.nblk ? blk + 1 : p.nblk - 1;
-#if defined(BH_ABLATE) && (BH_ABLATE & 256)
-            if (p.m == 12345)
-#endif
 #pragma unroll
             for (int rt = 0; rt < RT; ++rt)
 #pragma unroll
@@ -1992,11 +1955,7 @@ __global__ __launch_bounds__(256, 2) void k_gemm_fp6w(GemmArgs p) {
             for (int rt = 0; rt < 4; ++rt)
 #pragma unroll
                 for (int j = 0; j < 4; ++j) val[rt][j] = acc[4 * hf + rt][tt][j] * is;
-#if defined(BH_ABLATE) && (BH_ABLATE & 64)
-            if (val[0][0] == 1234567.f) store_wave_tiles(p, val, tok0, c, g, bx * 16 + wr * 8 + 4 * hf);
-#else
             store_wave_tiles(p, val, tok0, c, g, bx * 16 + wr * 8 + 4 * hf);
-#endif
         }
     }
 }
