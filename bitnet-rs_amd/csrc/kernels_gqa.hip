@@ -489,6 +489,13 @@ __global__ __launch_bounds__(256) void k_gqa_merge(Gqa p, const int *pos_ptr, in
     const int used = gqa_range(p, *pos_ptr + q0 + qi).used;
     const size_t stride = kGqaRecHead + vdimp;
     const float *rec = scratch + ((size_t)qi * p.heads + h) * maps * kGqaSplits * stride;
+    // 32 lanes of four columns; eight groups share maps and records.  Each group's first records are requested ahead of the weights.
+    const int grp = tid >> 5, gm = maps == 2 ? grp & 1 : 0, gs = maps == 2 ? grp >> 1 : grp, gn = maps == 2 ? 4 : 8, i0 = (tid & 31) * 4;
+    const float *vec = rec + (size_t)gm * kGqaSplits * stride + kGqaRecHead;
+    constexpr int AHEAD = 4;
+    f32x4 first[AHEAD];
+#pragma unroll
+    for (int e = 0; e < AHEAD; ++e) first[e] = *reinterpret_cast<const f32x4 *>(vec + min(gs + e * gn, used - 1) * stride + min(i0, vdimp - 4));
     if (wave < maps) {
         const float *r = rec + (size_t)wave * kGqaSplits * stride;
         float mv[2], lv[2];
@@ -511,13 +518,17 @@ __global__ __launch_bounds__(256) void k_gqa_merge(Gqa p, const int *pos_ptr, in
     }
     __syncthreads();
     const float gate = p.gate ? activate(z, BITNET_HIP_ACT_SIGMOID) : 1.0f;
-    // 32 lanes of four columns; eight groups share maps and records
-    const int grp = tid >> 5, gm = maps == 2 ? grp & 1 : 0, gs = maps == 2 ? grp >> 1 : grp, gn = maps == 2 ? 4 : 8;
-    for (int i = (tid & 31) * 4; i < vdimp; i += 128) {
-        const float *r = rec + (size_t)gm * kGqaSplits * stride + kGqaRecHead + i;
+    for (int i = i0; i < vdimp; i += 128) {
+        const float *r = vec + i;
         f32x4 acc = f32x4{0.f, 0.f, 0.f, 0.f};
+        int k0 = gs;
+        if (i == i0) {
+#pragma unroll
+            for (int e = 0; e < AHEAD; ++e) acc += ws[gm][gs + e * gn] * first[e];  // (weights past the last record are zero)
+            k0 += AHEAD * gn;
+        }
 #pragma unroll 8
-        for (int k = gs; k < used; k += gn) acc += ws[gm][k] * *reinterpret_cast<const f32x4 *>(r + k * stride);
+        for (int k = k0; k < used; k += gn) acc += ws[gm][k] * *reinterpret_cast<const f32x4 *>(r + k * stride);
         *reinterpret_cast<f32x4 *>(part + (size_t)grp * vdimp + i) = acc;
     }
     __syncthreads();

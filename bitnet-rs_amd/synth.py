@@ -232,7 +232,7 @@ def write_lasapel(folder: str, config: dict, seed: int = 42) -> str:
 
 def write_random(folder: str, config: dict, shapes: dict, seed: int, centre) -> str:
     """config.json + model.safetensors with random bf16 weights: slices of one random block, matrices scaled to unit gain, vectors around
-    centre(name)."""
+    centre(name) (a router's correction: next to nothing, so that its experts carry like loads)."""
     block = _stream(seed, 7).standard_normal(1 << 22, dtype=np.float32)
     os.makedirs(folder, exist_ok=True)
     with open(os.path.join(folder, "config.json"), "w") as fh:
@@ -248,7 +248,7 @@ def write_random(folder: str, config: dict, shapes: dict, seed: int, centre) -> 
         made = {}
         for k, (name, shape) in enumerate(shapes.items()):
             n = int(np.prod(shape))
-            gain, mid = ((1.0 if name == "embed" else 1.0 / np.sqrt(shape[1])), 0.0) if len(shape) == 2 else (0.1, centre(name))
+            gain, mid = ((1.0 if name == "embed" else 1.0 / np.sqrt(shape[1])), 0.0) if len(shape) == 2 else (0.001 if name.endswith("correction") else 0.1, centre(name))
             if (gain, mid) not in made:
                 made[gain, mid] = np.tile(((block * np.float32(gain) + np.float32(mid)).view(np.uint32) >> 16).astype(np.uint16), 2)
             bits, start = made[gain, mid], (k * 9973) % block.size
