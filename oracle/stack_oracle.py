@@ -54,6 +54,13 @@ def gelu_tanh(z):
     return 0.5 * z * (1.0 + np.tanh(math.sqrt(2.0 / math.pi) * (z + 0.044715 * z ** 3)))
 
 
+def xielu(z, p, q):
+    """a parabola for positive arguments, an exponential for the others; the two numbers pass a softplus"""
+    up = softplus(p) * z * z + 0.5 * z
+    down = (0.5 + softplus(q)) * (np.expm1(np.minimum(z, 0.0)) - z) + 0.5 * z
+    return np.where(z > 0.0, up, down)
+
+
 # ---- rotary positions ------------------------------------------------------------------------------------------------
 def rotary_frequencies(rot):
     """(frequency per pair, factor on cos and sin)"""
@@ -84,6 +91,17 @@ def rotate(v, positions, rot):
         u, w = v[t][..., :half], v[t][..., half:2 * half]
         out[t][..., :half] = u * c - w * s
         out[t][..., half:2 * half] = w * c + u * s
+    return out
+
+
+def rotate_pairs(v, positions, rot):
+    """v [tokens, ..., dims]: elements 2i and 2i + 1 turn together, by the frequencies and the factor of rotary_frequencies"""
+    f, mult = rotary_frequencies(rot)
+    out = np.array(v, F)
+    for t, p in enumerate(positions):
+        c, s = np.cos(p * f) * mult, np.sin(p * f) * mult
+        a, b = v[t][..., 0::2], v[t][..., 1::2]
+        out[t][..., 0::2], out[t][..., 1::2] = a * c - b * s, b * c + a * s
     return out
 
 
@@ -256,6 +274,57 @@ def gated_delta(h, t, p, m, eps):
     return y @ t[p + "o"].T
 
 
+def latent_attention_direct(h, t, p, m, eps):
+    """queries straight from the input, pairs of neighbouring elements turn, no sink"""
+    n, H, D, R, V = len(h), m["heads"], m["dim"], m["rot_dim"], m["vdim"]
+    z = h @ t[p + "dkv"].T
+    c = norm_plain(z[:, :m["kv_rank"]], t[p + "dkv.norm"], eps)
+    kr = rotate_pairs(z[:, m["kv_rank"]:], range(n), m["rot"])
+    q = (h @ t[p + "q"].T).reshape(n, H, D + R)
+    qr = rotate_pairs(q[:, :, D:], range(n), m["rot"])
+    k, v = (c @ t[p + "uk"].T).reshape(n, H, D), (c @ t[p + "uv"].T).reshape(n, H, V)
+    out = np.zeros((n, H, V), F)
+    for a in range(H):
+        s = (q[:, a, :D] @ k[:, a].T + qr[:, a] @ kr.T) * m["scale"]
+        s[np.triu_indices(n, 1)] = -np.inf
+        e = np.exp(s - s.max(axis=1, keepdims=True))
+        out[:, a] = e / e.sum(axis=1, keepdims=True) @ v[:, a]
+    return out.reshape(n, H * V) @ t[p + "o"].T
+
+
+def distance_penalty(i, j, r1, r2):
+    return r1 * np.log(1.0 + r2 * (i - j))
+
+
+def window_softmax(q, k, v, scale, size, r1, r2):
+    """q [n, heads, dim], k [n, kv heads, dim], v [n, kv heads, vdim]: a token sees itself and the size - 1 tokens ahead of it, far ones with a
+    penalty that grows with the logarithm of the distance"""
+    n, H, _ = q.shape
+    out = np.zeros((n, H, v.shape[2]), F)
+    for a in range(H):
+        g = a // (H // k.shape[1])
+        for i in range(n):
+            j = np.arange(max(0, i - size + 1), i + 1)
+            s = k[j, g] @ q[i, a] * scale - distance_penalty(i, j, r1[a], r2[a])
+            e = np.exp(s - s.max())
+            out[i, a] = e @ v[j, g] / e.sum()
+    return out
+
+
+def convolved(h, t, name):
+    return short_convolution(h @ t[name].T + t[name + ".b"], t[name + ".conv"])
+
+
+def window_attention(h, t, p, m, shared=None):
+    """(output, (keys, values)); shared: the keys and values of another layer"""
+    n, H, G, D, V = len(h), m["heads"], m["kv_heads"], m["dim"], m["vdim"]
+    q = convolved(h, t, p + "q").reshape(n, H, D)
+    k, v = shared or (convolved(h, t, p + "k").reshape(n, G, D), convolved(h, t, p + "v").reshape(n, G, V))
+    size = m["mask"]["size"] if m.get("mask") else n
+    o = window_softmax(q, k, v, m["scale"], size, t[p + "r1"], t[p + "r2"]).reshape(n, H * V)
+    return (o * sigmoid(h @ t[p + "g"].T)) @ t[p + "o"].T, (k, v)
+
+
 # ---- feed-forward ----------------------------------------------------------------------------------------------------
 def dense_mlp(h, t, p):
     z = relu_squared(h @ t[p + "up"].T + t[p + "up.b"])
@@ -310,11 +379,55 @@ def expert_or_identity_mlp(h, t, p, f):
     return out
 
 
+def xielu_mlp(h, t, p):
+    return xielu(h @ t[p + "up"].T, *t[p + "act"]) @ t[p + "down"].T
+
+
+def route_in_groups(h, router, correction, top, groups=None):
+    """per token: the experts with the largest corrected scores among the best groups of neighbours, and their uncorrected scores"""
+    score = sigmoid(h @ router.T)
+    ids = np.zeros((len(h), top), int)
+    for i in range(len(h)):
+        choice = score[i] + correction
+        if groups:
+            part = choice.reshape(groups["count"], -1)
+            worth = np.sort(part, axis=1)[:, -2:].sum(axis=1)
+            keep = np.argsort(-worth, kind="stable")[:groups["keep"]]
+            masked = np.full_like(part, -np.inf)
+            masked[keep] = part[keep]
+            choice = masked.reshape(-1)
+        ids[i] = np.argsort(-choice, kind="stable")[:top]
+    return ids, np.take_along_axis(score, ids, 1)
+
+
+def grouped_expert_mlp(h, t, p, f):
+    r = f["router"]
+    ids, w = route_in_groups(h, t[p + "router"], t[p + "correction"], r["top"], r.get("groups"))
+    out = np.zeros_like(h)
+    if f.get("shared"):
+        out += gated_mlp(h, t, p + "shared.", silu) * sigmoid(h @ t[p + "shared.sg"].T)
+    for i in range(len(h)):
+        for e, x in zip(ids[i], w[i]):
+            out[i] += x * gated_mlp(h[i:i + 1], t, p + f"e{e}.", silu)[0]
+    return out
+
+
+# ---- what a token brings along ----
+def bigram_rows(tokens, b):
+    """row of the pair table per token: the first token of a sequence has a row of its own"""
+    return [b["buckets"] if i == 0 else (int(tokens[i - 1]) * b["mul_prev"] + int(tokens[i]) * b["mul_cur"]) % b["buckets"] for i in range(len(tokens))]
+
+
+def token_side_input(x, e, t, p, eps):
+    g = gelu_tanh(x @ t[p + "gate"].T) * e
+    return norm_plain(g @ t[p + "proj"].T, t[p + "norm"], eps)
+
+
 # ---- the stack -------------------------------------------------------------------------------------------------------
 def forward(config, tensors, tokens):
     """(logits [n, vocab], residual stream after every layer run [runs, n, width])"""
     t = {k: np.asarray(v, F) for k, v in tensors.items()}
-    return {"Lasapel": forward_lasapel, "Mimolix": forward_mimolix, "Lurepel": forward_lurepel}[config["architecture"]](config, t, tokens)
+    return {"Lasapel": forward_lasapel, "Mimolix": forward_mimolix, "Lurepel": forward_lurepel, "Sipelorn": forward_sipelorn}[config["architecture"]](config, t, tokens)
 
 
 def layer_runs(config):
@@ -376,3 +489,32 @@ def forward_lurepel(config, t, tokens):
             x = x + norm_plain(y, t[p + "norm2"], eps)
         after.append(x)
     return norm_plain(x, t["final.norm"], eps) @ t["head"].T, np.stack(after)
+
+
+def forward_sipelorn(config, t, tokens):
+    eps, tokens = config["norm"]["eps"], np.asarray(tokens)
+    x = t["embed"][tokens] * config["embedding"]["scale"]
+    if config["embedding"].get("bigram"):
+        x = x + t["bigram"][bigram_rows(tokens, config["embedding"]["bigram"])]
+    side = config["token_side"]["dim"] if config.get("token_side") else 0
+    after, shared = [], {}
+
+    def gated(y, h, name):
+        return y * sigmoid(h @ t[name].T + t[name + ".b"])
+
+    for i, layer in enumerate(config["layers"]):
+        p, m, f = f"l{i}.", layer["mixer"], layer.get("mlp")
+        h = layer_norm(x, t[p + "norm1"], t[p + "norm1.b"], eps)
+        if layer["type"] == "attention":
+            y, shared[i] = window_attention(h, t, p + "mix.", m, shared[m["kv_from"]] if m.get("kv_from") is not None else None)
+        else:
+            y = latent_attention_direct(h, t, p + "mix.", m, eps)
+        x = x + gated(y, h, p + "rg1")
+        if f:
+            h = layer_norm(x, t[p + "norm2"], t[p + "norm2.b"], eps)
+            y = xielu_mlp(h, t, p + "mlp.") if f["kind"] == "dense" else grouped_expert_mlp(h, t, p + "mlp.", f)
+            x = x + gated(y, h, p + "rg2")
+        if side:
+            x = x + token_side_input(x, t["side.embed"][tokens][:, i * side:(i + 1) * side], t, p + "side.", eps)
+        after.append(x)
+    return layer_norm(x, t["final.norm"], t["final.norm.b"], eps) @ t["head"].T, np.stack(after)
