@@ -635,14 +635,14 @@ def timed_model(model, prompt, steps: int, warmup: int, digits: int = 2) -> dict
 
 
 STACK_DESIGNS = {"lasapel": ("Lasapel", "write_lasapel", "lasapel_config"), "mimolix": ("Mimolix", "write_mimolix", "mimolix_config"),
-                 "lurepel": ("Lurepel", "write_lurepel", "lurepel_config")}
-STACK_BESIDE = {"mimolix": "lasapel", "lurepel": "mimolix"}  # the closest other model; BitNet where there is none
+                 "lurepel": ("Lurepel", "write_lurepel", "lurepel_config"), "sipelorn": ("Sipelorn", "write_sipelorn", "sipelorn_config")}
+STACK_BESIDE = {"mimolix": "lasapel", "lurepel": "mimolix", "sipelorn": "lurepel"}  # the closest other model; BitNet where there is none
 
 
 def bench_stack(args, pkg, synth):
-    """--workload lasapel | mimolix | lurepel: prompt and decode throughput of a layer-stack design at sizes that resemble a real model's layers, beside the
+    """--workload lasapel | mimolix | lurepel | sipelorn: prompt and decode throughput of a layer-stack design at sizes that resemble a real model's layers, beside the
     library's closest other model with the same width, (active) feed-forward, heads, vocabulary and number of layer runs: BitNet (QK256) for
-    Lasapel, Lasapel for Mimolix, Mimolix for Lurepel."""
+    Lasapel, Lasapel for Mimolix, Mimolix for Lurepel, Lurepel for Sipelorn."""
     import tempfile
 
     rows = []

@@ -95,7 +95,7 @@ def _addr(t):
     return None if t is None else (t if isinstance(t, int) else t.data_ptr())
 
 
-ACT_NONE, ACT_SILU, ACT_SIGMOID, ACT_RELU2, ACT_GELU_TANH, ACT_GATED = 0, 1, 2, 3, 4, 0x100
+ACT_NONE, ACT_SILU, ACT_SIGMOID, ACT_RELU2, ACT_GELU_TANH, ACT_XIELU, ACT_GATED = 0, 1, 2, 3, 4, 5, 0x100
 IN_PLAIN, IN_NORM, IN_RESIDUAL_NORM, IN_CONCAT, IN_RESIDUAL = 0, 1, 2, 3, 4
 LINEAR_BLOCK = 128
 
@@ -103,20 +103,27 @@ LINEAR_BLOCK = 128
 class VectorInput(C.Structure):
     _fields_ = [("x", _vp), ("kind", C.c_int32), ("eps", C.c_float), ("weight_offset", C.c_float), ("weight", _vp), ("y", _vp), ("post_weight", _vp),
                 ("scale", _vp), ("gate", _vp), ("x_out", _vp), ("n", C.c_int32), ("mean_n", C.c_int32),
-                ("mult", C.c_float), ("center", C.c_int32), ("bias", _vp), ("x2", _vp), ("h_out", _vp)]
+                ("mult", C.c_float), ("center", C.c_int32), ("bias", _vp), ("x2", _vp), ("h_out", _vp), ("y_gate", _vp)]
+
+
+class Epilogue(C.Structure):
+    _fields_ = [("act_a", C.c_float), ("act_b", C.c_float), ("pairs", _sz), ("act2_from", _sz), ("act2", C.c_int32), ("conv_from", _sz), ("channels", _sz), ("taps", _sz),
+                ("conv", _vp), ("ring", _vp), ("pos", _vp), ("mul", _vp), ("ld_mul", _sz), ("mul_rows", _sz), ("mul_tokens", _vp), ("mul_at", _vp)]
 
 
 class SumRows(C.Structure):
     _fields_ = [("x", _vp), ("m", _sz), ("width", _sz), ("y", _vp), ("ldy", _sz), ("mult", C.c_float), ("expert_rows", _vp), ("ld_expert", _sz), ("top", _sz),
                 ("slots", _vp), ("slot_weights", _vp), ("weight", _vp), ("bias", _vp), ("x2", _vp), ("weight_offset", C.c_float), ("eps", C.c_float),
-                ("center", C.c_int32), ("h_f32", C.c_int32), ("h", _vp), ("ldh", _sz), ("post_weight", _vp), ("scale", _vp), ("input", _vp), ("ld_input", _sz), ("identity", C.c_int32)]
+                ("center", C.c_int32), ("h_f32", C.c_int32), ("h", _vp), ("ldh", _sz), ("post_weight", _vp), ("scale", _vp), ("input", _vp), ("ld_input", _sz), ("identity", C.c_int32),
+                ("y_scale", _vp), ("ld_y_scale", _sz), ("gate", _vp), ("ld_gate", _sz)]
 
 
 class Gqa(C.Structure):
     _fields_ = [(n, _sz) for n in ("heads", "kv_heads", "maps", "dim", "dimp", "vdim", "vdimp", "capacity")] + [
         ("eps", C.c_float), ("lam", C.c_float), ("out_scale", C.c_float), ("q_weight", _vp), ("k_weight", _vp), ("q_factor", _vp), ("kcache", _vp), ("vcache", _vp),
         ("unit_norm", C.c_int32), ("values_are_keys", C.c_int32), ("rot_dims", _sz), ("chunk", _sz), ("rope_cos", _vp), ("rope_sin", _vp), ("sink", _vp), ("gate", _vp),
-        ("ldgate", _sz), ("gate_f32", C.c_int32)]
+        ("ldgate", _sz), ("gate_f32", C.c_int32), ("gate_columns", C.c_int32), ("queries_only", C.c_int32), ("window", _sz), ("taps", _sz), ("far_weight", _vp),
+        ("far_rate", _vp), ("conv", _vp), ("ring", _vp)]
 
 
 class Delta(C.Structure):
@@ -126,7 +133,8 @@ class Delta(C.Structure):
 
 
 class Router(C.Structure):
-    _fields_ = [("experts", _sz), ("identity", _sz), ("top", _sz), ("scale", C.c_float), ("raw", C.c_int32), ("correction", _vp)]
+    _fields_ = [("experts", _sz), ("identity", _sz), ("top", _sz), ("scale", C.c_float), ("raw", C.c_int32), ("correction", _vp), ("sigmoid", C.c_int32),
+                ("groups", _sz), ("keep", _sz)]
 
 
 class ExpertsPlan(C.Structure):
@@ -142,7 +150,8 @@ class LatentRows(C.Structure):
 
 class LatentAttention(C.Structure):
     _fields_ = [("heads", _sz), ("dimp", _sz), ("qd", _sz), ("vdimp", _sz), ("kv_rank", _sz), ("rot_dim", _sz), ("scale", C.c_float), ("sink", _vp),
-                ("ccache", _vp), ("rcache", _vp), ("ldc", _sz), ("ldr", _sz), ("capacity", _sz), ("rope_cos", _vp), ("rope_sin", _vp)]
+                ("ccache", _vp), ("rcache", _vp), ("ldc", _sz), ("ldr", _sz), ("capacity", _sz), ("rope_cos", _vp), ("rope_sin", _vp),
+                ("ldq", _sz)]
 
 
 class HipLib:
@@ -591,6 +600,11 @@ class HipLib:
         self._call("embed_norm_bf16_dev", _ptr(table), _sz(ld), _ptr(tokens), _optr(offset), _sz(n), _sz(width), _sz(vocab), C.c_float(scale), _ptr(norm_weight),
                    C.c_float(eps), _ptr(out), _vp(stream))
 
+    def embed_pairs_bf16_dev(self, table, ld: int, pairs, ld_pairs: int, buckets: int, mul_prev: int, mul_cur: int, tokens, out, n: int, width: int, vocab: int,
+                             offset=None, scale: float = 1.0, stream: int = 0) -> None:
+        self._call("embed_pairs_bf16_dev", _ptr(table), _sz(ld), _ptr(pairs), _sz(ld_pairs), _sz(buckets), C.c_uint64(mul_prev), C.c_uint64(mul_cur), _ptr(tokens),
+                   _optr(offset), _sz(n), _sz(width), _sz(vocab), C.c_float(scale), _ptr(out), _vp(stream))
+
     def sum_norm_rows_dev(self, rows: "SumRows", stream: int = 0) -> None:
         self._call("sum_norm_rows_dev", C.byref(rows), _vp(stream))
 
@@ -598,8 +612,11 @@ class HipLib:
         self.c.bitnet_hip_gqa_scratch_bytes.restype = _sz
         return int(self.c.bitnet_hip_gqa_scratch_bytes(_sz(heads), _sz(maps), _sz(vdimp), _sz(nq)))
 
-    def gqa_rows_dev(self, a: "Gqa", rows, ld: int, rows_f32: bool, cache_f32: bool, pos, n: int, stream: int = 0) -> None:
-        self._call("gqa_rows_dev", C.byref(a), _ptr(rows), _sz(ld), C.c_int(rows_f32), C.c_int(cache_f32), _ptr(pos), _sz(n), _vp(stream))
+    def gqa_rows_dev(self, a: "Gqa", rows, ld: int, rows_f32: bool, cache_f32: bool, pos, n: int, q=None, ldq: int = 0, stream: int = 0) -> None:
+        self._call("gqa_rows_dev", C.byref(a), _ptr(rows), _sz(ld), C.c_int(rows_f32), C.c_int(cache_f32), _ptr(pos), _sz(n), _optr(q), _sz(ldq), _vp(stream))
+
+    def conv_keep_dev(self, rows, ld: int, rows_f32: bool, channels: int, taps: int, ring, pos, n: int, stream: int = 0) -> None:
+        self._call("conv_keep_dev", _ptr(rows), _sz(ld), C.c_int(rows_f32), _sz(channels), _sz(taps), _ptr(ring), _ptr(pos), _sz(n), _vp(stream))
 
     def gqa_step_dev(self, a: "Gqa", row, pos, scratch, stream: int = 0) -> None:
         self._call("gqa_step_dev", C.byref(a), _ptr(row), _ptr(pos), _ptr(scratch), _vp(stream))
@@ -656,9 +673,9 @@ class HipLib:
                    _optr(identity), _vp(stream))
 
     def experts_out_dev(self, x0, w0, cols0: int, ld0: int, bias, x1, ldx1: int, w1, cols1: int, ld1: int, ids, top: int, rows: int, y, identity=None, input=None,
-                        stream: int = 0) -> None:
+                        x0_scale=None, stream: int = 0) -> None:
         self._call("experts_out_dev", _optr(x0), _optr(w0), _sz(cols0), _sz(ld0), _optr(bias), _ptr(x1), _sz(ldx1), _ptr(w1), _sz(cols1), _sz(ld1), _ptr(ids), _sz(top),
-                   _sz(rows), _optr(identity), _optr(input), _ptr(y), _vp(stream))
+                   _sz(rows), _optr(identity), _optr(input), _optr(x0_scale), _ptr(y), _vp(stream))
 
     def residual_norm_rows_dev(self, x, m: int, width: int, eps: float, weight_offset: float, y=None, ldy: int = 0, post_weight=None, scale=None,
                                next_weight=None, h=None, ldh: int = 0, h_f32: bool = True, stream: int = 0) -> None:
@@ -671,18 +688,22 @@ class HipLib:
                    _sz(mean_n), _ptr(h), _sz(ldh), C.c_int(h_f32), _vp(stream))
 
     def dense_matmul_dev(self, a, lda: int, a_f32: bool, w, ldw: int, m: int, n: int, k: int, c, ldc: int, c_f32: bool, bias=None, act0: int = 0,
-                         act1: int = 0, act_split: int = 0, batch: int = 1, a_batch: int = 0, w_batch: int = 0, c_batch: int = 0, stream: int = 0) -> None:
+                         act1: int = 0, act_split: int = 0, batch: int = 1, a_batch: int = 0, w_batch: int = 0, c_batch: int = 0, more: "Epilogue | None" = None,
+                         stream: int = 0) -> None:
         self._call("dense_matmul_dev", _ptr(a), _sz(lda), C.c_int(a_f32), _ptr(w), _sz(ldw), _optr(bias), _sz(m), _sz(n), _sz(k), C.c_int(act0),
-                   C.c_int(act1), _sz(act_split), _ptr(c), _sz(ldc), C.c_int(c_f32), _sz(batch), _sz(a_batch), _sz(w_batch), _sz(c_batch), _vp(stream))
+                   C.c_int(act1), _sz(act_split), _ptr(c), _sz(ldc), C.c_int(c_f32), _sz(batch), _sz(a_batch), _sz(w_batch), _sz(c_batch),
+                   C.byref(more) if more is not None else None, _vp(stream))
 
     def dense_gemv_dev(self, x, w, rows: int, cols: int, ld: int, y, kind: int = 0, eps: float = 0.0, weight_offset: float = 0.0, weight=None, res=None,
                        post_weight=None, scale=None, gate=None, x_out=None, n: int = 0, mean_n: int = 0, bias=None, act0: int = 0, act1: int = 0,
                        act_split: int = 0, batch: int = 1, w_batch: int = 0, x_batch: int = 0, y_batch: int = 0, latent=None, latent_f32: bool = False,
-                       mult: float = 1.0, center: bool = False, norm_bias=None, x2=None, h_out=None, stream: int = 0) -> None:
+                       mult: float = 1.0, center: bool = False, norm_bias=None, x2=None, h_out=None, y_gate=None,
+                       more: "Epilogue | None" = None, stream: int = 0) -> None:
         vi = VectorInput(_addr(x), kind, eps, weight_offset, _addr(weight), _addr(res), _addr(post_weight), _addr(scale), _addr(gate), _addr(x_out), n, mean_n, mult, int(center),
-                         _addr(norm_bias), _addr(x2), _addr(h_out))
+                         _addr(norm_bias), _addr(x2), _addr(h_out), _addr(y_gate))
         self._call("dense_gemv_dev", C.byref(vi), _ptr(w), _sz(rows), _sz(cols), _sz(ld), _optr(bias), C.c_int(act0), C.c_int(act1), _sz(act_split), _ptr(y),
-                   _sz(batch), _sz(w_batch), _sz(x_batch), _sz(y_batch), C.byref(latent) if latent is not None else None, C.c_int(latent_f32), _vp(stream))
+                   _sz(batch), _sz(w_batch), _sz(x_batch), _sz(y_batch), C.byref(latent) if latent is not None else None, C.c_int(latent_f32),
+                   C.byref(more) if more is not None else None, _vp(stream))
 
     def latent_rows_dev(self, rows, m: int, f32: bool, stream: int = 0) -> None:
         self._call("latent_rows_dev", C.byref(rows), _sz(m), C.c_int(f32), _vp(stream))

@@ -133,7 +133,7 @@ def _build(force: bool, verbose: bool, OBJ_DIR: str, LIB_PATH: str, extra_all: l
 # Programs linked from the same objects as the libraries: the kernels and host files of the models they serve, and no others.
 STACK_CSRC = ["abi_core.hip", "abi_dense.hip", "abi_mixers.hip", "kernels_decode.hip", "kernels_delta.hip", "kernels_dense.hip", "kernels_experts.hip",
               "kernels_gqa.hip", "kernels_latent.hip", "kernels_linear.hip"]
-STACK_HOST = ["sequence.cpp", "registry.cpp", "safetensors.cpp", "stack_model.cpp", "lasapel.cpp", "mimolix.cpp", "lurepel.cpp"]
+STACK_HOST = ["sequence.cpp", "registry.cpp", "safetensors.cpp", "stack_model.cpp", "lasapel.cpp", "mimolix.cpp", "lurepel.cpp", "sipelorn.cpp"]
 PROGRAMS = {"trace_run": (STACK_CSRC, STACK_HOST + ["trace_run.cpp"])}
 HOST_FLAGS = ["-O2", "-std=c++17", "-fPIC", "-Wall", "-Wno-unused-result", "-Wno-int-in-bool-context", "-D__HIP_PLATFORM_AMD__"]
 

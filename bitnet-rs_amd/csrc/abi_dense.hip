@@ -12,7 +12,7 @@ static_assert(kLinBlock == BITNET_HIP_LINEAR_BLOCK, "the decay table's length is
     } while (0)
 
 namespace {
-bool act_ok(int a) { return a >= BITNET_HIP_ACT_NONE && a <= BITNET_HIP_ACT_GELU_TANH; }
+bool act_ok(int a) { return a >= BITNET_HIP_ACT_NONE && a <= BITNET_HIP_ACT_XIELU; }
 
 int to_latent_rows(const bitnet_hip_latent_rows *r, size_t m, int f32, LatentRows &o) {
     BH_REQUIRE(r && r->z && r->pos, "latent_rows: null pointer");
@@ -30,6 +30,25 @@ int to_latent_rows(const bitnet_hip_latent_rows *r, size_t m, int f32, LatentRow
     return 0;
 }
 
+// rows: those of W ahead of pairing; m: rows of the output
+int to_epilogue(const bitnet_hip_epilogue *e, size_t rows, Epilogue &o) {
+    if (!e) return 0;
+    BH_REQUIRE(act_ok(e->act2) && e->pairs <= rows && e->pairs % 4 == 0, "product: bad pairs or third activation");
+    if (e->taps) {
+        BH_REQUIRE(e->conv && e->ring && e->pos && e->channels > 0 && e->taps <= (size_t)kMaxTaps && e->conv_from + e->channels <= rows && e->conv_from >= e->pairs,
+                   "product: bad convolution (%zu taps, rows %zu + %zu of %zu)", e->taps, e->conv_from, e->channels, rows);
+        o.conv_from = (int)e->conv_from, o.channels = (int)e->channels, o.taps = (int)e->taps, o.conv = e->conv, o.ring = e->ring, o.pos = e->pos;
+    }
+    if (e->mul) {
+        BH_REQUIRE(e->pairs == 0 && e->mul_tokens && e->mul_at && e->mul_rows > 0 && e->ld_mul >= rows, "product: bad table of factors");
+        BH_CHECK_DIMS(e->mul_rows, e->ld_mul);
+        o.mul = e->mul, o.ld_mul = e->ld_mul, o.mul_rows = (int)e->mul_rows, o.mul_tokens = e->mul_tokens, o.mul_at = e->mul_at;
+    }
+    o.act_a = e->act_a, o.act_b = e->act_b, o.act2 = e->act2;
+    if (e->act2_from && e->act2_from < rows) o.act2_from = (int)e->act2_from;
+    return 0;
+}
+
 int to_vec_in(const bitnet_hip_vector_input *in, size_t cols, VecIn &o) {
     BH_REQUIRE(in && in->x, "vector input: null pointer");
     BH_REQUIRE(in->kind >= BITNET_HIP_IN_PLAIN && in->kind <= BITNET_HIP_IN_RESIDUAL, "vector input: unknown kind %d", in->kind);
@@ -44,15 +63,16 @@ int to_vec_in(const bitnet_hip_vector_input *in, size_t cols, VecIn &o) {
     }
     o.x = in->x, o.kind = in->kind, o.eps = in->eps, o.offset = in->weight_offset, o.weight = in->weight, o.y = in->y, o.post_weight = in->post_weight;
     o.scale = in->scale, o.gate = in->gate, o.x_out = in->y ? in->x_out : nullptr, o.n = in->n, o.mean_n = in->mean_n ? in->mean_n : in->n;
-    o.mult = in->mult, o.center = in->center, o.bias = in->bias, o.x2 = in->x2, o.h_out = in->h_out;
+    o.mult = in->mult, o.center = in->center, o.bias = in->bias, o.x2 = in->x2, o.h_out = in->h_out, o.y_gate = in->y_gate;
     return 0;
 }
 
 int to_attn(const bitnet_hip_latent_attention *a, LatentAttn &o) {
-    BH_REQUIRE(a && a->sink && a->ccache && a->rcache && a->rope_cos && a->rope_sin, "latent attention: null pointer");
+    BH_REQUIRE(a && a->ccache && a->rcache && a->rope_cos && a->rope_sin, "latent attention: null pointer");
     BH_REQUIRE(a->heads > 0 && a->heads < 65536 && a->dimp % 32 == 0 && a->ldr % 32 == 0 && a->qd == a->dimp + a->ldr && a->vdimp > 0 && a->vdimp % 16 == 0 &&
-                   a->ldc % 64 == 0 && a->kv_rank > 0 && a->kv_rank <= a->ldc && a->rot_dim <= a->ldr && a->rot_dim % 2 == 0 && a->capacity % 64 == 0,
+                   a->ldc % 64 == 0 && a->kv_rank > 0 && a->kv_rank <= a->ldc && a->rot_dim <= a->ldr && a->rot_dim % 2 == 0 && a->capacity % 64 == 0 && (a->ldq == 0 || a->ldq >= a->heads * a->qd),
                "latent attention: bad shape");
+    o.ldq = a->ldq ? a->ldq : a->heads * a->qd;
     o.ccache = a->ccache, o.rcache = a->rcache, o.ldc = (int)a->ldc, o.ldr = (int)a->ldr, o.kv_rank = (int)a->kv_rank, o.rot_dim = (int)a->rot_dim;
     o.heads = (int)a->heads, o.dimp = (int)a->dimp, o.qd = (int)a->qd, o.vdimp = (int)a->vdimp, o.scale = a->scale, o.sink = a->sink;
     o.rope_cos = a->rope_cos, o.rope_sin = a->rope_sin, o.capacity = (int)a->capacity;
@@ -68,7 +88,21 @@ int bitnet_hip_embed_bf16_dev(const uint16_t *table, size_t ld, const int32_t *t
     BH_REQUIRE(table && tokens && out, "Null pointer passed to embed_bf16_dev");
     BH_REQUIRE(n > 0 && width > 0 && vocab > 0 && ld >= width, "embed_bf16: bad shape");
     BH_CHECK_DIMS(n, width);
-    BH_HIP_TRY(launch_embed_bf16(table, ld, tokens, offset, (int)n, (int)width, (int)vocab, scale, nullptr, 0.f, out, (hipStream_t)stream));
+    BH_HIP_TRY(launch_embed_bf16(table, ld, tokens, offset, (int)n, (int)width, (int)vocab, scale, nullptr, 0.f, TokenPairs(), out, (hipStream_t)stream));
+    return BITNET_HIP_OK;
+    BH_GUARD_END
+}
+
+int bitnet_hip_embed_pairs_bf16_dev(const uint16_t *table, size_t ld, const uint16_t *pairs, size_t ld_pairs, size_t buckets, uint64_t mul_prev, uint64_t mul_cur,
+                                    const int32_t *tokens, const int32_t *offset, size_t n, size_t width, size_t vocab, float scale, float *out, void *stream) {
+    BH_GUARD_BEGIN
+    BH_REQUIRE(table && pairs && tokens && out, "Null pointer passed to embed_pairs_bf16_dev");
+    BH_REQUIRE(n > 0 && width > 0 && vocab > 0 && ld >= width && ld_pairs >= width && buckets > 0 && mul_prev < (uint64_t(1) << 31) && mul_cur < (uint64_t(1) << 31),
+               "embed_pairs_bf16: bad shape");
+    BH_CHECK_DIMS(n, width);
+    TokenPairs p;
+    p.table = pairs, p.ld = ld_pairs, p.buckets = buckets, p.mul_prev = mul_prev, p.mul_cur = mul_cur;
+    BH_HIP_TRY(launch_embed_bf16(table, ld, tokens, offset, (int)n, (int)width, (int)vocab, scale, nullptr, 0.f, p, out, (hipStream_t)stream));
     return BITNET_HIP_OK;
     BH_GUARD_END
 }
@@ -79,7 +113,7 @@ int bitnet_hip_embed_norm_bf16_dev(const uint16_t *table, size_t ld, const int32
     BH_REQUIRE(table && tokens && norm_weight && out, "Null pointer passed to embed_norm_bf16_dev");
     BH_REQUIRE(n > 0 && width > 0 && vocab > 0 && ld >= width, "embed_norm_bf16: bad shape");
     BH_CHECK_DIMS(n, width);
-    BH_HIP_TRY(launch_embed_bf16(table, ld, tokens, offset, (int)n, (int)width, (int)vocab, scale, norm_weight, eps, out, (hipStream_t)stream));
+    BH_HIP_TRY(launch_embed_bf16(table, ld, tokens, offset, (int)n, (int)width, (int)vocab, scale, norm_weight, eps, TokenPairs(), out, (hipStream_t)stream));
     return BITNET_HIP_OK;
     BH_GUARD_END
 }
@@ -117,7 +151,7 @@ int bitnet_hip_gather_rows_dev(const float *x, const int32_t *rows, size_t n, si
 
 int bitnet_hip_dense_matmul_dev(const void *a, size_t lda, int a_f32, const uint16_t *w, size_t ldw, const float *bias, size_t m, size_t n, size_t k,
                                 int act0, int act1, size_t act_split, void *c, size_t ldc, int c_f32, size_t batch, size_t a_batch, size_t w_batch,
-                                size_t c_batch, void *stream) {
+                                size_t c_batch, const bitnet_hip_epilogue *more, void *stream) {
     BH_GUARD_BEGIN
     BH_REQUIRE(a && w && c, "Null pointer passed to dense_matmul_dev");
     BH_REQUIRE(m > 0 && n > 0 && k > 0 && batch > 0 && batch < 65536, "dense_matmul: empty");
@@ -131,6 +165,9 @@ int bitnet_hip_dense_matmul_dev(const void *a, size_t lda, int a_f32, const uint
     BH_CHECK_DIMS(n, ldw);
     BH_CHECK_DIMS(m, ldc);
     GemmArgsD g;
+    if (int rc = to_epilogue(more, n, g.more)) return rc;
+    BH_REQUIRE(!more || (!g.more.conv && more->pairs == 0 && more->act2_from == 0 && (!more->mul || (batch == 1 && !gated && (a_f32 || !c_f32)))),
+               "dense_matmul: what a product of one row does, or a table of factors with pairs or f32 sums");
     g.a = a, g.w = w, g.bias = bias, g.c = c, g.m = (int)m, g.n = (int)n, g.k = (int)k, g.lda = lda, g.ldw = ldw, g.ldc = ldc;
     g.act0 = act0, g.act1 = act1, g.act_split = (int)act_split, g.gated = gated != 0, g.a_f32 = a_f32, g.c_f32 = c_f32;
     g.batch = (int)batch, g.a_batch = a_batch, g.w_batch = w_batch, g.c_batch = c_batch;
@@ -160,17 +197,19 @@ static int gemv_args(const bitnet_hip_vector_input *input, const uint16_t *w, si
 
 int bitnet_hip_dense_gemv_dev(const bitnet_hip_vector_input *input, const uint16_t *w, size_t rows, size_t cols, size_t ld, const float *bias, int act0,
                               int act1, size_t act_split, float *y, size_t batch, size_t w_batch, size_t x_batch, size_t y_batch,
-                              const bitnet_hip_latent_rows *latent, int latent_f32, void *stream) {
+                              const bitnet_hip_latent_rows *latent, int latent_f32, const bitnet_hip_epilogue *more, void *stream) {
     BH_GUARD_BEGIN
     GemvArgs g;
     if (int rc = gemv_args(input, w, rows, cols, ld, y, g)) return rc;
     const int gated = act0 & BITNET_HIP_ACT_GATED;
     act0 &= ~BITNET_HIP_ACT_GATED;
     BH_REQUIRE(act_ok(act0) && act_ok(act1), "dense_gemv: unknown activation");
-    BH_REQUIRE(!gated || (rows % 2 == 0 && act_split == 0), "dense_gemv: gated rows come in pairs, with one activation");
-    BH_REQUIRE(batch > 0 && batch < 65536 && (batch == 1 || (g.in.kind == BITNET_HIP_IN_PLAIN && !latent)) && w_batch % 8 == 0, "dense_gemv: bad batch");
+    if (int rc = to_epilogue(more, rows, g.more)) return rc;
+    const size_t pairs = gated ? (more && more->pairs ? more->pairs : rows) : 0;
+    BH_REQUIRE(!gated ? !more || more->pairs == 0 : pairs % 2 == 0 && (pairs < rows ? act_split >= pairs : act_split == 0), "dense_gemv: gated rows come in pairs, with one activation");
+    BH_REQUIRE(batch > 0 && batch < 65536 && (batch == 1 || (g.in.kind == BITNET_HIP_IN_PLAIN && !g.more.conv && !g.more.mul && pairs == 0)) && w_batch % 8 == 0, "dense_gemv: bad batch");
     BH_CHECK_DIMS(batch, rows, ld);
-    g.bias = bias, g.act0 = act0, g.act1 = act1, g.act_split = (int)act_split, g.gated = gated != 0;
+    g.bias = bias, g.act0 = act0, g.act1 = act1, g.act_split = (int)act_split, g.gated = (int)pairs;
     g.batch = (int)batch, g.w_batch = w_batch, g.x_batch = x_batch, g.y_batch = y_batch;
     LatentRows r;
     if (latent) {

@@ -11,7 +11,7 @@ using namespace bitnet_hip;
     } while (0)
 
 namespace {
-bool act_ok(int a) { return a >= BITNET_HIP_ACT_NONE && a <= BITNET_HIP_ACT_GELU_TANH; }
+bool act_ok(int a) { return a >= BITNET_HIP_ACT_NONE && a <= BITNET_HIP_ACT_GELU_TANH; }  // (no constants here)
 
 int check_gqa(const bitnet_hip_gqa *a) {
     BH_REQUIRE(a && a->q_factor && a->kcache && a->vcache, "gqa: null pointer");
@@ -22,13 +22,18 @@ int check_gqa(const bitnet_hip_gqa *a) {
                a->vdim, a->vdimp, a->capacity);
     BH_REQUIRE(a->rot_dims % 2 == 0 && a->rot_dims <= a->dim && (a->rot_dims == 0 || (a->rope_cos && a->rope_sin)), "gqa: bad rotation of %zu dimensions", a->rot_dims);
     BH_REQUIRE(a->chunk < (size_t(1) << 30) && (!a->sink || a->maps == 1) && (!a->values_are_keys || (a->maps == 1 && a->vdim == a->dim && a->vdimp == a->dimp)) &&
-                   (!a->gate || a->ldgate >= a->heads),
+                   (!a->gate || a->ldgate >= (a->gate_columns ? a->heads * a->vdimp : a->heads)) && (!a->gate_columns || a->maps == 1),
                "gqa: bad chunk, sink, values or gate");
+    BH_REQUIRE(a->window < (size_t(1) << 30) && !a->far_weight == !a->far_rate && (a->maps == 1 || (!a->far_weight && !a->queries_only)) && a->taps <= (size_t)kMaxTaps &&
+                   (a->taps == 0 || (a->conv && a->ring)),
+               "gqa: bad window, distance penalty, queries or convolution");
     BH_CHECK_DIMS(a->capacity, a->kv_heads * a->maps, a->dimp);
     BH_CHECK_DIMS(a->capacity, a->kv_heads, a->vdimp);
     return 0;
 }
-size_t gqa_row(const bitnet_hip_gqa *a) { return (a->heads + a->kv_heads) * a->maps * a->dimp + (a->values_are_keys ? 0 : a->kv_heads * a->vdimp); }
+size_t gqa_row(const bitnet_hip_gqa *a) {
+    return a->queries_only ? a->heads * a->dimp : (a->heads + a->kv_heads) * a->maps * a->dimp + (a->values_are_keys ? 0 : a->kv_heads * a->vdimp);
+}
 
 int check_delta(const bitnet_hip_delta *d) {
     BH_REQUIRE(d && d->conv && d->decay_rate && d->dt_bias && d->norm && d->state && d->ring, "delta: null pointer");
@@ -50,6 +55,8 @@ int check_router(const bitnet_hip_router *r) {
     BH_REQUIRE(r && r->experts > 0 && r->experts <= (size_t)kMaxExperts && r->identity <= (size_t)kMaxExperts && r->experts + r->identity <= (size_t)kMaxExperts && r->top > 0 &&
                    r->top <= (size_t)kMaxTop && r->top <= r->experts + r->identity,
                "experts: bad router");
+    BH_REQUIRE(r->groups == 0 || (r->identity == 0 && r->experts % r->groups == 0 && r->keep > 0 && r->keep <= r->groups && r->top <= r->keep * (r->experts / r->groups)),
+               "experts: bad groups");
     return 0;
 }
 // tiles of a plan at most: every expert's last tile may be short
@@ -64,6 +71,7 @@ int bitnet_hip_sum_norm_rows_dev(const bitnet_hip_sum_rows *r, void *stream) {
     BH_REQUIRE(!r->h || (r->ldh >= (r->x2 ? 2 * r->width : r->width)), "sum_norm_rows: bad output");
     BH_REQUIRE(r->top == 0 || (r->expert_rows && r->slots && r->slot_weights && r->ld_expert >= r->width && (!r->input || r->ld_input >= r->width)),
                "sum_norm_rows: bad expert rows");
+    BH_REQUIRE((!r->gate || r->ld_gate >= r->width) && (!r->y_scale || r->ld_y_scale > 0), "sum_norm_rows: bad gate or factors");
     BH_CHECK_DIMS(r->m, r->width);
     BH_HIP_TRY(launch_sum_norm_rows(*r, (hipStream_t)stream));
     return BITNET_HIP_OK;
@@ -74,13 +82,26 @@ int bitnet_hip_sum_norm_rows_dev(const bitnet_hip_sum_rows *r, void *stream) {
 size_t bitnet_hip_gqa_scratch_bytes(size_t heads, size_t maps, size_t vdimp, size_t nq) { return gqa_scratch_floats(heads, maps, vdimp, nq) * sizeof(float); }
 int bitnet_hip_gqa_supported(size_t dimp, size_t vdimp) { return dimp <= 65536 && vdimp <= 65536 && gqa_supported((int)dimp, (int)vdimp) ? 1 : 0; }
 
-int bitnet_hip_gqa_rows_dev(const bitnet_hip_gqa *a, void *rows, size_t ld, int rows_f32, int cache_f32, const int32_t *pos, size_t n, void *stream) {
+int bitnet_hip_gqa_rows_dev(const bitnet_hip_gqa *a, void *rows, size_t ld, int rows_f32, int cache_f32, const int32_t *pos, size_t n, void *q, size_t ldq, void *stream) {
     BH_GUARD_BEGIN
     if (int rc = check_gqa(a)) return rc;
+    if (!q) ldq = ld;
+    BH_REQUIRE((q || a->taps == 0) && (!q || q != rows) && ldq >= a->heads * a->maps * a->dimp, "gqa_rows: bad place of the queries");
     BH_REQUIRE(rows && pos && n > 0 && n <= a->capacity && ld >= gqa_row(a) && (n == 1 || ld % 8 == 0) && (uintptr_t)rows % 16 == 0 && (rows_f32 || !cache_f32), "gqa_rows: bad arguments");
     BH_REQUIRE((a->heads + a->kv_heads) * a->maps + a->kv_heads * (a->vdimp / 32) < 65536, "gqa_rows: too many heads");
     BH_CHECK_DIMS(n, ld);
-    BH_HIP_TRY(launch_gqa_rows(*a, rows, ld, rows_f32, cache_f32, pos, (int)n, (hipStream_t)stream));
+    BH_CHECK_DIMS(n, ldq);
+    BH_HIP_TRY(launch_gqa_rows(*a, rows, ld, rows_f32, cache_f32, pos, (int)n, q ? q : rows, ldq, (hipStream_t)stream));
+    return BITNET_HIP_OK;
+    BH_GUARD_END
+}
+
+int bitnet_hip_conv_keep_dev(const void *rows, size_t ld, int rows_f32, size_t channels, size_t taps, float *ring, const int32_t *pos, size_t n, void *stream) {
+    BH_GUARD_BEGIN
+    BH_REQUIRE(rows && ring && pos && n > 0 && channels > 0 && ld >= channels && taps > 0 && taps <= (size_t)kMaxTaps, "conv_keep: bad arguments");
+    BH_CHECK_DIMS(n, ld);
+    BH_CHECK_DIMS(taps, channels);
+    BH_HIP_TRY(launch_conv_keep(rows, ld, rows_f32, (int)channels, (int)taps, ring, pos, (int)n, (hipStream_t)stream));
     return BITNET_HIP_OK;
     BH_GUARD_END
 }
@@ -158,7 +179,8 @@ int bitnet_hip_delta_keep_dev(const bitnet_hip_delta *d, const void *rows, size_
     if (int rc = check_delta(d)) return rc;
     BH_REQUIRE(rows && pos && n > 0 && ld >= delta_row(d), "delta_keep: bad arguments");
     BH_CHECK_DIMS(n, ld);
-    BH_HIP_TRY(launch_delta_keep(*d, rows, ld, rows_f32, pos, (int)n, (hipStream_t)stream));
+    const size_t channels = 2 * d->kv_heads * d->dimp + d->heads * d->vdimp;
+    BH_HIP_TRY(launch_conv_keep(rows, ld, rows_f32, (int)channels, (int)d->taps, d->ring, pos, (int)n, (hipStream_t)stream));
     return BITNET_HIP_OK;
     BH_GUARD_END
 }
@@ -270,7 +292,8 @@ int bitnet_hip_experts_up_dev(const float *logits, const bitnet_hip_router *rout
 }
 
 int bitnet_hip_experts_out_dev(const float *x0, const uint16_t *w0, size_t cols0, size_t ld0, const float *bias, const float *x1, size_t ldx1, const uint16_t *w1,
-                               size_t cols1, size_t ld1, const int32_t *ids, size_t top, size_t rows, const float *identity, const float *input, float *y, void *stream) {
+                               size_t cols1, size_t ld1, const int32_t *ids, size_t top, size_t rows, const float *identity, const float *input, const float *x0_scale,
+                               float *y, void *stream) {
     BH_GUARD_BEGIN
     if (!x0) w0 = nullptr, cols0 = ld0 = 0;
     BH_REQUIRE((!x0 || (w0 && cols0 >= 8)) && x1 && w1 && ids && y && top > 0 && top <= (size_t)kMaxTop && rows > 0 && cols0 % 8 == 0 && cols0 <= ld0 && ld0 % 8 == 0 &&
@@ -280,7 +303,7 @@ int bitnet_hip_experts_out_dev(const float *x0, const uint16_t *w0, size_t cols0
     BH_CHECK_DIMS(rows, ld1);
     ExpertsOut a;
     a.x0 = x0, a.x1 = x1, a.bias = bias, a.w0 = w0, a.w1 = w1, a.cols0 = (int)cols0, a.ld0 = (int)ld0, a.cols1 = (int)cols1, a.ld1 = (int)ld1, a.ldx1 = (int)ldx1;
-    a.top = (int)top, a.rows = (int)rows, a.ids = ids, a.identity = identity, a.input = input, a.y = y;
+    a.top = (int)top, a.rows = (int)rows, a.ids = ids, a.identity = identity, a.input = input, a.x0_scale = x0_scale, a.y = y;
     const hipError_t e = launch_experts_out(a, (hipStream_t)stream);
     if (e == hipErrorInvalidValue) return set_error(BITNET_HIP_ERR_UNSUPPORTED, "experts_out: %zu + %zu x %zu columns do not fit a workgroup's memory", cols0, top, cols1);
     BH_HIP_TRY(e);

@@ -17,6 +17,20 @@ typedef uint32_t u32x2 __attribute__((ext_vector_type(2)));
 
 // ---- launch arguments ------------------------------------------------------------------------------------------------
 
+// What else a product does with its rows (bitnet_hip_epilogue).
+struct Epilogue {
+    float act_a = 0.f, act_b = 0.f;
+    int act2 = 0, act2_from = 0x7fffffff;
+    int conv_from = 0, channels = 0, taps = 0;
+    const float *conv = nullptr;
+    float *ring = nullptr;
+    const int *pos = nullptr;
+    const uint16_t *mul = nullptr;
+    size_t ld_mul = 0;
+    int mul_rows = 0;
+    const int *mul_tokens = nullptr, *mul_at = nullptr;
+};
+
 // How a matrix-vector product forms its input vector (bitnet_hip_vector_input).
 struct VecIn {
     const float *x = nullptr;
@@ -31,6 +45,7 @@ struct VecIn {
     int center = 0;               // layer norm, with bias
     const float *bias = nullptr, *x2 = nullptr;
     float *h_out = nullptr;       // the vector formed
+    const float *y_gate = nullptr;  // on what is added to x
 };
 
 struct GemvArgs {
@@ -41,7 +56,8 @@ struct GemvArgs {
     size_t w_batch = 0, x_batch = 0, y_batch = 0;  // elements between consecutive batch members
     const float *bias = nullptr;
     int act0 = 0, act1 = 0, act_split = 0;         // rows < act_split take act0, the others act1
-    int gated = 0;                                 // rows 2 i and 2 i + 1 make element i: act0(row 2 i) * row 2 i + 1
+    int gated = 0;                                 // rows 2 i and 2 i + 1 below this make element i: act0(row 2 i) * row 2 i + 1
+    Epilogue more;
     float *y = nullptr;
     float *best_val = nullptr;                     // argmax partial per workgroup (batch 1)
     int *best_idx = nullptr;
@@ -59,6 +75,7 @@ struct GemmArgsD {
     int act0 = 0, act1 = 0, act_split = 0;
     int gated = 0;             // columns 2 i and 2 i + 1 make column i of c: act0(column 2 i) * column 2 i + 1 (n: columns ahead of that)
     int a_f32 = 0, c_f32 = 0;
+    Epilogue more;
     int batch = 1;
     size_t a_batch = 0, w_batch = 0, c_batch = 0;
     // grouped form: the row tiles come from a list, (matrix, first row, rows) each; matrix i lies at w + i w_batch
@@ -98,8 +115,15 @@ struct ExpertsOut {
     const uint16_t *w0 = nullptr, *w1 = nullptr;
     int cols0 = 0, ld0 = 0, cols1 = 0, ld1 = 0, ldx1 = 0, top = 0, rows = 0;
     const int *ids = nullptr;
-    const float *identity = nullptr, *input = nullptr;
+    const float *identity = nullptr, *input = nullptr, *x0_scale = nullptr;
     float *y = nullptr;
+};
+
+// pairs of neighbouring tokens: the second table of an embedding (bitnet_hip_embed_pairs_bf16_dev)
+struct TokenPairs {
+    const uint16_t *table = nullptr;
+    size_t ld = 0;
+    uint64_t buckets = 0, mul_prev = 0, mul_cur = 0;
 };
 
 // rows of a down-projection output z -> normed query latent, normed key latent and rotated key part
@@ -119,6 +143,7 @@ struct LatentRows {
 };
 
 struct LatentAttn {
+    size_t ldq = 0;                // leading dimension of q, qb
     const float *q = nullptr;      // decode: f32 [nq][heads * qd] before rotation (the rotated part at [h * qd + dimp])
     const void *qb = nullptr;      // prompt: bf16 of the same
     const float *qabs = nullptr;   // decode: f32 [nq][heads * ldc] queries in latent space
@@ -171,13 +196,15 @@ constexpr int kLatentRecHead = 4;  // floats ahead of a record's vector: running
 
 constexpr int kGqaTile = 128;      // keys per workgroup and step of the decode attention
 constexpr int kGqaSplits = 128;    // most records per (query, head, map)
+constexpr int kMaxTaps = 64;       // of a convolution ahead of the attention
 constexpr int kGqaRecHead = 4;     // floats ahead of a record's vector: running maximum (of base-2 scores), sum, unused
 constexpr int kDeltaChunk = 64;    // tokens per chunk of the delta rule
 constexpr int kDeltaUnits = 512;   // chunks x heads per pass over the workspace: one round of workgroups, and small enough to stay in the caches
 constexpr int kMaxExperts = 1024, kMaxTop = 32;
 
 hipError_t launch_embed_bf16(const uint16_t *table, size_t ld, const int *tokens, const int *offset, int n, int width, int vocab, float scale,
-                             const float *norm_w, float eps, float *out, hipStream_t s);
+                             const float *norm_w, float eps, const TokenPairs &pairs, float *out, hipStream_t s);
+hipError_t launch_conv_keep(const void *rows, size_t ld, int rows_f32, int channels, int taps, float *ring, const int *pos, int n, hipStream_t s);
 hipError_t launch_sum_norm_rows(const SumRows &a, hipStream_t s);
 hipError_t launch_residual_norm_rows(float *x, const float *y, size_t ldy, const float *post_w, const float *scale, const float *next_w,
                                      float offset, float eps, int m, int width, void *h, size_t ldh, int h_f32, hipStream_t s);
@@ -198,7 +225,7 @@ hipError_t launch_linear_recurrent(const LinearAttn &a, hipStream_t s);
 hipError_t launch_linear_chunked(const LinearAttn &a, hipStream_t s);
 size_t gqa_scratch_floats(size_t heads, size_t maps, size_t vdimp, size_t nq);
 bool gqa_supported(int dimp, int vdimp);
-hipError_t launch_gqa_rows(const Gqa &g, void *rows, size_t ld, int rows_f32, int cache_f32, const int *pos, int n, hipStream_t s);
+hipError_t launch_gqa_rows(const Gqa &g, void *rows, size_t ld, int rows_f32, int cache_f32, const int *pos, int n, void *q, size_t ldq, hipStream_t s);
 hipError_t launch_gqa_step(const Gqa &g, const GqaStep &a, hipStream_t s);
 hipError_t launch_gqa_any(const Gqa &g, const void *q, size_t ldq, int q_f32, int cache_f32, const int *pos, int q0, int nq, float *scratch, hipStream_t s);
 hipError_t launch_gqa_merge(const Gqa &g, const int *pos, int q0, int nq, const float *scratch, void *out, size_t ldo, int out_bf16, hipStream_t s);
@@ -209,7 +236,6 @@ size_t delta_workspace_bytes(size_t n, size_t heads, size_t dimp, size_t vdimp);
 hipError_t launch_delta_step(const Delta &d, const float *row, const float *ba, const int *pos, float *out, hipStream_t s);
 hipError_t launch_delta_rows(const Delta &d, const void *rows, size_t ld, int rows_f32, const float *ba, size_t ldba, const int *pos, int n, float *qk,
                              void *v, float *gates, hipStream_t s);
-hipError_t launch_delta_keep(const Delta &d, const void *rows, size_t ld, int rows_f32, const int *pos, int n, hipStream_t s);
 hipError_t launch_delta_recurrent(const Delta &d, const float *qk, const void *v, const float *gates, const void *rows, size_t ld, int rows_f32, int n,
                                   void *out, size_t ldo, hipStream_t s);
 hipError_t launch_delta_chunked(const Delta &d, const float *qk, const uint16_t *v, const float *gates, const uint16_t *rows, size_t ld, int n,
@@ -282,7 +308,7 @@ __device__ __forceinline__ float group_sum(float v, float *slot) {
 
 __device__ __forceinline__ float gelu_argument(float v) { return 0.7978845608028654f * (v + 0.044715f * v * v * v); }  // sqrt(2 / pi)
 // BITNET_HIP_ACT_*
-__device__ __forceinline__ float activate(float v, int act) {
+__device__ __forceinline__ float activate(float v, int act, float a = 0.f, float b = 0.f) {
     switch (act) {
         case BITNET_HIP_ACT_SILU: return v / (1.0f + expf(-v));
         case BITNET_HIP_ACT_SIGMOID: return 1.0f / (1.0f + expf(-v));
@@ -291,6 +317,7 @@ __device__ __forceinline__ float activate(float v, int act) {
             return r * r;
         }
         case BITNET_HIP_ACT_GELU_TANH: return v / (1.0f + expf(-2.0f * gelu_argument(v)));  // (1 + tanh z) / 2 = 1 / (1 + exp(-2 z))
+        case BITNET_HIP_ACT_XIELU: return 0.5f * v + (v > 0.f ? a * v * v : b * (expm1f(v) - v));
         default: return v;
     }
 }

@@ -2,7 +2,7 @@
 //   S <- g S;  u = beta (v - S^T k);  S <- S + k u^T;  o = S^T q,
 // behind a short causal convolution with silu and unit norms of q and k, ahead of a norm per head and a gate.
 //   k_delta_step       one token: convolution, norms, recurrence, output norm and gate in one launch
-//   k_delta_rows       a portion's convolution, unit norms, decays and step sizes;  k_delta_keep: its last inputs, for what follows
+//   k_delta_rows       a portion's convolution, unit norms, decays and step sizes (its last inputs, for what follows: k_conv_keep)
 //   k_delta_recurrent  those rows token by token
 //   chunks of 64 tokens on the matrix cores: k_delta_chunk, k_delta_scan, k_delta_out
 // With G_i the sum of log g up to token i of a chunk and L_ij = beta_i e^(G_i - G_j) k_i.k_j (j < i), the chunk's u satisfy
@@ -308,22 +308,6 @@ hipError_t launch_delta_rows(const Delta &d, const void *rows, size_t ld, int ro
         rows_go(d, (const float *)rows, ld, ba, ldba, pos, n, qk, (float *)v, gates, s);
     else
         rows_go(d, (const uint16_t *)rows, ld, ba, ldba, pos, n, qk, (uint16_t *)v, gates, s);
-    return hipGetLastError();
-}
-
-template <class T>
-__global__ __launch_bounds__(256) void k_delta_keep(Delta p, const T *rows, size_t ld, const int *pos_ptr, int n) {
-    const int C = (int)(2 * p.kv_heads * p.dimp + p.heads * p.vdimp), taps = (int)p.taps, i = blockIdx.x * 256 + threadIdx.x, pos0 = *pos_ptr;
-    if (i >= C) return;
-    for (int t = max(0, n - (taps - 1)); t < n; ++t) p.ring[(size_t)((pos0 + t) % taps) * C + i] = ld_act(rows + (size_t)t * ld, i);
-}
-
-hipError_t launch_delta_keep(const Delta &d, const void *rows, size_t ld, int rows_f32, const int *pos, int n, hipStream_t s) {
-    const int C = (int)(2 * d.kv_heads * d.dimp + d.heads * d.vdimp);
-    if (rows_f32)
-        hipLaunchKernelGGL(k_delta_keep<float>, dim3((C + 255) / 256), dim3(256), 0, s, d, (const float *)rows, ld, pos, n);
-    else
-        hipLaunchKernelGGL(k_delta_keep<uint16_t>, dim3((C + 255) / 256), dim3(256), 0, s, d, (const uint16_t *)rows, ld, pos, n);
     return hipGetLastError();
 }
 

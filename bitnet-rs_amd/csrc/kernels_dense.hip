@@ -11,10 +11,17 @@ namespace bitnet_hip {
 
 // ---- embedding rows ---------------------------------------------------------------------------------------------------
 __global__ void k_embed_bf16(const uint16_t *__restrict__ table, size_t ld, const int *__restrict__ tokens, const int *__restrict__ offset,
-                             int width, int vocab, float scale, const float *__restrict__ norm_w, float eps, float *__restrict__ out) {
+                             int width, int vocab, float scale, const float *__restrict__ norm_w, float eps, TokenPairs pairs, float *__restrict__ out) {
     __shared__ float slot[4];
-    int tok = tokens[(offset ? *offset : 0) + blockIdx.x];
-    tok = tok < 0 ? 0 : (tok >= vocab ? vocab - 1 : tok);
+    const int at = (offset ? *offset : 0) + blockIdx.x;
+    auto token = [&](int i) { return min(max(tokens[i], 0), vocab - 1); };
+    const int tok = token(at);
+    if (pairs.table) {
+        const uint64_t pair = at == 0 ? pairs.buckets : ((uint64_t)token(max(at - 1, 0)) * pairs.mul_prev + (uint64_t)tok * pairs.mul_cur) % pairs.buckets;
+        const uint16_t *a = table + (size_t)tok * ld, *b = pairs.table + (size_t)pair * pairs.ld;
+        for (int i = threadIdx.x; i < width; i += blockDim.x) out[(size_t)blockIdx.x * width + i] = scale * bf2f(a[i]) + bf2f(b[i]);
+        return;
+    }
     if (norm_w) {
         const uint16_t *row = table + (size_t)tok * ld;
         constexpr int NR = 16;  // rows of up to 4096 columns in registers, what lies behind is read again
@@ -40,8 +47,8 @@ __global__ void k_embed_bf16(const uint16_t *__restrict__ table, size_t ld, cons
 }
 
 hipError_t launch_embed_bf16(const uint16_t *table, size_t ld, const int *tokens, const int *offset, int n, int width, int vocab, float scale,
-                             const float *norm_w, float eps, float *out, hipStream_t s) {
-    hipLaunchKernelGGL(k_embed_bf16, dim3(n), dim3(256), 0, s, table, ld, tokens, offset, width, vocab, scale, norm_w, eps, out);
+                             const float *norm_w, float eps, const TokenPairs &pairs, float *out, hipStream_t s) {
+    hipLaunchKernelGGL(k_embed_bf16, dim3(n), dim3(256), 0, s, table, ld, tokens, offset, width, vocab, scale, norm_w, eps, pairs, out);
     return hipGetLastError();
 }
 
@@ -52,6 +59,23 @@ __global__ void k_gather_rows(const float *__restrict__ x, const int *__restrict
 
 hipError_t launch_gather_rows(const float *x, const int *rows, int n, int width, float *out, hipStream_t s) {
     hipLaunchKernelGGL(k_gather_rows, dim3(n), dim3(256), 0, s, x, rows, width, out);
+    return hipGetLastError();
+}
+
+// the last inputs of a portion into the ring of a causal convolution (position p in row p % taps)
+template <class T>
+__global__ __launch_bounds__(256) void k_conv_keep(const T *rows, size_t ld, int channels, int taps, float *ring, const int *pos_ptr, int n) {
+    const int i = blockIdx.x * 256 + threadIdx.x, pos0 = *pos_ptr;
+    if (i >= channels) return;
+    for (int t = max(0, n - (taps - 1)); t < n; ++t) ring[(size_t)((pos0 + t) % taps) * channels + i] = ld_act(rows + (size_t)t * ld, i);
+}
+
+hipError_t launch_conv_keep(const void *rows, size_t ld, int rows_f32, int channels, int taps, float *ring, const int *pos, int n, hipStream_t s) {
+    const dim3 grid((channels + 255) / 256);
+    if (rows_f32)
+        hipLaunchKernelGGL(k_conv_keep<float>, grid, dim3(256), 0, s, (const float *)rows, ld, channels, taps, ring, pos, n);
+    else
+        hipLaunchKernelGGL(k_conv_keep<uint16_t>, grid, dim3(256), 0, s, (const uint16_t *)rows, ld, channels, taps, ring, pos, n);
     return hipGetLastError();
 }
 
@@ -166,6 +190,8 @@ __global__ __launch_bounds__(256) void k_sum_norm_rows(SumRows p) {
     const int *slots = p.slots + (size_t)blockIdx.x * p.top;
     const float *sw = p.slot_weights + (size_t)blockIdx.x * p.top;
     const float *x2 = p.x2 ? p.x2 + (size_t)blockIdx.x * width : nullptr;
+    const T *gate = p.gate ? (const T *)p.gate + (size_t)blockIdx.x * p.ld_gate : nullptr;
+    const float ys = p.y_scale ? p.y_scale[(size_t)blockIdx.x * p.ld_y_scale] : 1.0f;
     const T *input = p.input ? (const T *)p.input + (size_t)blockIdx.x * p.ld_input : nullptr;  // (may be h: a thread reads its columns ahead of writing them)
     const int top = (int)p.top;
     if (VEC) {
@@ -183,7 +209,7 @@ __global__ __launch_bounds__(256) void k_sum_norm_rows(SumRows p) {
             for (int j = 0; j < kSumRegs; ++j) {
                 const int i = tid + 256 * j;
                 a[j] = f32x4{0.f, 0.f, 0.f, 0.f};
-                if (y && i < n4) a[j] = ld4(y, 4 * i);
+                if (y && i < n4) a[j] = ys * ld4(y, 4 * i);
             }
             float through = 0.f;
 #pragma unroll 4
@@ -228,13 +254,15 @@ __global__ __launch_bounds__(256) void k_sum_norm_rows(SumRows p) {
             for (int j = 0; j < kSumRegs; ++j) {
                 const int i = tid + 256 * j;
                 if (i < n4) {
+                    f32x4 r;
                     if (p.post_weight) {
-                        f32x4 r = a[j] * post * (p.weight_offset + ld4(p.post_weight, 4 * i));
+                        r = a[j] * post * (p.weight_offset + ld4(p.post_weight, 4 * i));
                         if (p.scale) r *= ld4(p.scale, 4 * i);
-                        v[j] += r;
                     } else {
-                        v[j] += p.mult * a[j];
+                        r = p.mult * a[j];
                     }
+                    if (gate) r *= ld4(gate, 4 * i);
+                    v[j] += r;
                     st4(x, 4 * i, v[j]);
                 }
             }
@@ -280,7 +308,7 @@ __global__ __launch_bounds__(256) void k_sum_norm_rows(SumRows p) {
     } else {  // (a thread comes back to its own columns only)
         if (y || top) {
             auto sum = [&](int i) {
-                float a = y ? y[i] : 0.f;
+                float a = y ? ys * y[i] : 0.f;
                 for (int k = 0; k < top; ++k) a += sw[k] * (!IDENTITY || slots[k] >= 0 ? ld_act(er + (size_t)slots[k] * p.ld_expert, i) : input ? ld_act(input, i) : x[i]);
                 return a;
             };
@@ -294,7 +322,8 @@ __global__ __launch_bounds__(256) void k_sum_norm_rows(SumRows p) {
                 post = 1.0f / sqrtf(group_sum<4>(ss, slot) / (float)width + p.eps);
             }
             for (int i = tid; i < width; i += 256)
-                x[i] += p.post_weight ? (p.scale ? p.scale[i] : 1.0f) * (sum(i) * post * (p.weight_offset + p.post_weight[i])) : p.mult * sum(i);
+                x[i] += (gate ? ld_act(gate, i) : 1.0f) *
+                        (p.post_weight ? (p.scale ? p.scale[i] : 1.0f) * (sum(i) * post * (p.weight_offset + p.post_weight[i])) : p.mult * sum(i));
         }
         if (!h) return;
         if (x2) {
@@ -321,7 +350,7 @@ __global__ __launch_bounds__(256) void k_sum_norm_rows(SumRows p) {
 
 hipError_t launch_sum_norm_rows(const SumRows &a, hipStream_t s) {
     // (four columns at a time: every row of every operand starts on its own alignment)
-    const bool vec = a.width % 4 == 0 && a.width <= 1024 * kSumRegs && a.ldy % 4 == 0 && a.ld_expert % 4 == 0 && a.ldh % 4 == 0 && a.ld_input % 4 == 0;
+    const bool vec = a.width % 4 == 0 && a.width <= 1024 * kSumRegs && a.ldy % 4 == 0 && a.ld_expert % 4 == 0 && a.ldh % 4 == 0 && a.ld_input % 4 == 0 && a.ld_gate % 4 == 0;
     auto pick = [&](auto all, auto some) { return a.identity ? some : all; };
     auto fn = a.h_f32 ? (vec ? pick(k_sum_norm_rows<float, true, false>, k_sum_norm_rows<float, true, true>) : pick(k_sum_norm_rows<float, false, false>, k_sum_norm_rows<float, false, true>))
                       : (vec ? pick(k_sum_norm_rows<uint16_t, true, false>, k_sum_norm_rows<uint16_t, true, true>)
@@ -450,14 +479,17 @@ __device__ void form_input(const VecIn &in, const float *x, int cols, int kp, fl
             xv[j] = v * (i < n4 ? 1.0f : 0.0f);
         }
         if (in.kind >= BITNET_HIP_IN_RESIDUAL_NORM && in.y && !in.post_weight) {
-            f32x4 yv[NR];
+            f32x4 yv[NR], yg[NR];
 #pragma unroll
-            for (int j = 0; j < NR; ++j) yv[j] = reinterpret_cast<const f32x4 *>(in.y)[min(tid + 256 * j, n4 - 1)];
+            for (int j = 0; j < NR; ++j) {
+                yv[j] = reinterpret_cast<const f32x4 *>(in.y)[min(tid + 256 * j, n4 - 1)];
+                yg[j] = in.y_gate ? reinterpret_cast<const f32x4 *>(in.y_gate)[min(tid + 256 * j, n4 - 1)] : f32x4{1.f, 1.f, 1.f, 1.f};
+            }
 #pragma unroll
             for (int j = 0; j < NR; ++j) {
                 const int i = tid + 256 * j;
                 if (i >= n4) continue;
-                xv[j] += in.mult * yv[j];
+                xv[j] += in.mult * yv[j] * yg[j];
                 if (writer && in.x_out) reinterpret_cast<f32x4 *>(in.x_out)[i] = xv[j];
             }
         } else if (in.kind >= BITNET_HIP_IN_RESIDUAL_NORM && in.y) {
@@ -478,6 +510,9 @@ __device__ void form_input(const VecIn &in, const float *x, int cols, int kp, fl
 #pragma unroll
                 for (int j = 0; j < NR; ++j) sc[j] = f32x4{1.f, 1.f, 1.f, 1.f};
             }
+            if (in.y_gate)
+#pragma unroll
+                for (int j = 0; j < NR; ++j) sc[j] *= reinterpret_cast<const f32x4 *>(in.y_gate)[min(tid + 256 * j, n4 - 1)];
 #pragma unroll
             for (int j = 0; j < NR; ++j) ss += yv[j].x * yv[j].x + yv[j].y * yv[j].y + yv[j].z * yv[j].z + yv[j].w * yv[j].w;
             const float inv = 1.0f / sqrtf(group_sum<4>(ss, slot) / (float)in.mean_n + in.eps);
@@ -543,7 +578,7 @@ __device__ void form_input(const VecIn &in, const float *x, int cols, int kp, fl
         float ss = 0.f;
         if (in.kind >= BITNET_HIP_IN_RESIDUAL_NORM && in.y && !in.post_weight) {
             for (int i = tid; i < n; i += 256) {
-                const float v = x[i] + in.mult * in.y[i];
+                const float v = x[i] + in.mult * in.y[i] * (in.y_gate ? in.y_gate[i] : 1.0f);
                 xs[i] = v;
                 if (writer && in.x_out) in.x_out[i] = v;
                 ss += v * v;
@@ -553,7 +588,7 @@ __device__ void form_input(const VecIn &in, const float *x, int cols, int kp, fl
             const float inv = 1.0f / sqrtf(group_sum<4>(ss, slot) / (float)in.mean_n + in.eps);
             ss = 0.f;
             for (int i = tid; i < n; i += 256) {
-                const float v = x[i] + (in.scale ? in.scale[i] : 1.0f) * (in.y[i] * inv * (in.offset + in.post_weight[i]));
+                const float v = x[i] + (in.scale ? in.scale[i] : 1.0f) * (in.y_gate ? in.y_gate[i] : 1.0f) * (in.y[i] * inv * (in.offset + in.post_weight[i]));
                 xs[i] = v;
                 if (writer && in.x_out) in.x_out[i] = v;
                 ss += v * v;
@@ -591,6 +626,17 @@ __device__ void form_input(const VecIn &in, const float *x, int cols, int kp, fl
     __syncthreads();
 }
 
+template <int LPR>
+__device__ __forceinline__ float lanes_total(float v) {
+    if (LPR == 8) {
+        v += dpp<0x141>(v);       // row_half_mirror
+        v += dpp<0xb1>(v);        // quad_perm [1,0,3,2]
+        return v + dpp<0x4e>(v);  // quad_perm [2,3,0,1]
+    }
+    v = row_sum(v);
+    return LPR == 64 ? rows_sum(v) : v;
+}
+
 template <int LPR, int R, int U>
 __global__ __launch_bounds__(256) void k_dense_gemv(GemvK p) {
     extern __shared__ __attribute__((aligned(16))) float xs[];
@@ -600,6 +646,7 @@ __global__ __launch_bounds__(256) void k_dense_gemv(GemvK p) {
     const GemvArgs &a = p.a;
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     if ((int)blockIdx.x == p.lat_wg) {  // (the whole workgroup)
+        if (blockIdx.y > 0) return;
         if (p.lat.f32)
             latent_row<float>(p.lat, 0, slot);
         else
@@ -628,7 +675,24 @@ __global__ __launch_bounds__(256) void k_dense_gemv(GemvK p) {
             }
         }
     };
+    // the earlier positions of a convolution's rows, a tap per lane; summed behind the product
+    const Epilogue &e = a.more;
+    const int pos = e.conv ? *e.pos : 0, mul_at = e.mul ? *e.mul_at : 0;
+    float past[R];
+    auto fetch_past = [&](int grp) {
+#pragma unroll
+        for (int r = 0; r < R; ++r) {
+            const int ch = (grp * G + sub) * R + r - e.conv_from;
+            past[r] = 0.f;
+            if (ch < 0 || ch >= e.channels) continue;
+            for (int j = l; j < e.taps - 1; j += LPR) {
+                const int at = pos - (e.taps - 1) + j;
+                if (at >= 0) past[r] += e.conv[(size_t)j * e.channels + ch] * e.ring[(size_t)(at % e.taps) * e.channels + ch];
+            }
+        }
+    };
     if (g < p.groups) fetch(g, 0);
+    if (e.conv && g < p.groups) fetch_past(g);
     form_input(a.in, a.in.x + (size_t)b * a.x_batch, a.cols, p.kp, xs, slot, blockIdx.x == 0 && b == 0);
     float bv = -INFINITY;
     int bi = 0x7fffffff;
@@ -666,32 +730,40 @@ __global__ __launch_bounds__(256) void k_dense_gemv(GemvK p) {
         }
         const int row0 = (g * G + sub) * R;
 #pragma unroll
-        for (int r = 0; r < R; ++r) {
-            acc[r] = LPR == 8 ? acc[r] + dpp<0x141>(acc[r]) : row_sum(acc[r]);  // (8 lanes: row_half_mirror first)
-            if (LPR == 8) {
-                acc[r] += dpp<0xb1>(acc[r]);  // quad_perm [1,0,3,2]
-                acc[r] += dpp<0x4e>(acc[r]);  // quad_perm [2,3,0,1]
+        for (int r = 0; r < R; ++r) acc[r] = lanes_total<LPR>(acc[r]);
+        if (e.conv) {
+            float f[R];
+#pragma unroll
+            for (int r = 0; r < R; ++r) f[r] = lanes_total<LPR>(past[r]);
+#pragma unroll
+            for (int r = 0; r < R; ++r) {
+                const int row = row0 + r, ch = row - e.conv_from;
+                if (ch < 0 || ch >= e.channels || row >= a.rows) continue;
+                if (a.bias) acc[r] += a.bias[row];
+                if (l == 0) e.ring[(size_t)(pos % e.taps) * e.channels + ch] = acc[r];  // (no earlier position's slot)
+                acc[r] = acc[r] * e.conv[(size_t)(e.taps - 1) * e.channels + ch] + f[r];
             }
-            if (LPR == 64) acc[r] = rows_sum(acc[r]);
+            if (g + n_wg * 4 < p.groups) fetch_past(g + n_wg * 4);
         }
-        if (R > 1 && a.gated) {
+        if (R > 1 && row0 < a.gated) {
             if (l == 0)
 #pragma unroll
                 for (int r = 0; r + 1 < R; r += 2) {
-                    const int row = row0 + r;  // (even, and so is the number of rows)
+                    const int row = row0 + r;  // (even, and so is the number of rows in pairs, in whole groups)
                     if (row >= a.rows) continue;
                     const float b0 = a.bias ? a.bias[row] : 0.f, b1 = a.bias ? a.bias[row + 1] : 0.f;
-                    a.y[(size_t)b * a.y_batch + (row >> 1)] = activate(acc[r] + b0, a.act0) * (acc[r + 1] + b1);
+                    a.y[(size_t)b * a.y_batch + (row >> 1)] = activate(acc[r] + b0, a.act0, e.act_a, e.act_b) * (acc[r + 1] + b1);
                 }
         } else if (l == 0) {
 #pragma unroll
             for (int r = 0; r < R; ++r) {
-                const int row = row0 + r;
+                const int row = row0 + r, ch = row - e.conv_from;
                 if (row >= a.rows) continue;
                 float v = acc[r];
-                if (a.bias) v += a.bias[row];
-                v = activate(v, row < a.act_split ? a.act0 : a.act1);
-                a.y[(size_t)b * a.y_batch + row] = v;
+                if (a.bias && (!e.conv || ch < 0 || ch >= e.channels)) v += a.bias[row];
+                v = activate(v, row >= e.act2_from ? e.act2 : row < a.act_split ? a.act0 : a.act1, e.act_a, e.act_b);
+                if (e.mul) v *= bf2f(e.mul[(size_t)min(max(e.mul_tokens[mul_at], 0), e.mul_rows - 1) * e.ld_mul + row]);
+                a.y[(size_t)b * a.y_batch + row - (a.gated >> 1)] = v;
                 if (a.best_val) {
                     const float t = v != v ? -INFINITY : v;
                     if (t > bv || (t == bv && row < bi)) {
@@ -808,7 +880,8 @@ __device__ __forceinline__ int weight_key(int row) {
 
 // GROUPED: the row tiles come from a device list, (matrix, first row, rows) each; a matrix's tiles follow one another.
 // GATED (bf16 outputs): columns 2 i and 2 i + 1 make column i of the output.
-template <int TN, int TM, int WN, int WM, int ST, bool CF32, bool GROUPED = false, bool GATED = false>
+// MUL (bf16 outputs): row i of the output is multiplied by a table's row, the one of its token.
+template <int TN, int TM, int WN, int WM, int ST, bool CF32, bool GROUPED = false, bool GATED = false, bool MUL = false>
 __global__ __launch_bounds__(64 * WN * WM, 2) void k_dense_gemm(GemmArgsD p, int tiles_n, int tiles_m, int swizzle) {
     extern __shared__ __attribute__((aligned(1024))) uint8_t lds[];
     constexpr int NW = WN * WM, DN = TN / NW / 8, DM = TM / NW / 8;  // DMA instructions per wave and step (eight rows each)
@@ -965,7 +1038,7 @@ __global__ __launch_bounds__(64 * WN * WM, 2) void k_dense_gemm(GemmArgsD p, int
             apply([&](float v, int n) {
                 const int f = n < p.act_split ? p.act0 : p.act1;
                 const float sg = __builtin_amdgcn_rcpf(1.0f + __expf(-v)), r = fmaxf(v, 0.0f);
-                return f == BITNET_HIP_ACT_SILU ? v * sg : f == BITNET_HIP_ACT_SIGMOID ? sg : f == BITNET_HIP_ACT_RELU2 ? r * r : activate(v, f);
+                return f == BITNET_HIP_ACT_SILU ? v * sg : f == BITNET_HIP_ACT_SIGMOID ? sg : f == BITNET_HIP_ACT_RELU2 ? r * r : activate(v, f, p.more.act_a, p.more.act_b);
             });
         else if (act == BITNET_HIP_ACT_SILU)
             apply([](float v, int) { return v * __builtin_amdgcn_rcpf(1.0f + __expf(-v)); });
@@ -975,6 +1048,13 @@ __global__ __launch_bounds__(64 * WN * WM, 2) void k_dense_gemm(GemmArgsD p, int
             apply([](float v, int) { return activate(v, BITNET_HIP_ACT_RELU2); });
         else if (act == BITNET_HIP_ACT_GELU_TANH)
             apply([](float v, int) { return v * __builtin_amdgcn_rcpf(1.0f + __expf(-2.0f * gelu_argument(v))); });
+        else if (act == BITNET_HIP_ACT_XIELU)  // (exp(v) - 1 loses what a bf16 output does not keep)
+            apply([&](float v, int) { return 0.5f * v + (v > 0.f ? p.more.act_a * v * v : p.more.act_b * (__expf(v) - 1.0f - v)); });
+        if (MUL) {
+            const int token = min(max(p.more.mul_tokens[*p.more.mul_at + m], 0), p.more.mul_rows - 1);
+            const uint16_t *mul = p.more.mul + (size_t)token * p.more.ld_mul;
+            apply([&](float v, int n) { return v * bf2f(mul[min(n, p.n - 1)]); });
+        }
         if (CF32) {
 #pragma unroll
             for (int i = 0; i < FN; ++i) {
@@ -1018,11 +1098,12 @@ static hipError_t grouped_go(const GemmArgsD &a, hipStream_t s) {
     return hipGetLastError();
 }
 
-template <int T, int WN, int WM, int ST>
+template <int T, int WN, int WM, int ST, bool MUL = false>
 static hipError_t gemm_go(const GemmArgsD &a, hipStream_t s) {
     const int tn = (a.n + T - 1) / T, tm = (a.m + T - 1) / T, swz = (tn * tm) % 8 == 0 ? 1 : 0;
     constexpr size_t lds = (size_t)ST * T * 256;
-    auto fn = a.gated   ? k_dense_gemm<T, T, WN, WM, ST, false, false, true>
+    auto fn = MUL       ? k_dense_gemm<T, T, WN, WM, ST, false, false, false, MUL>
+              : a.gated ? k_dense_gemm<T, T, WN, WM, ST, false, false, true>
               : a.c_f32 ? k_dense_gemm<T, T, WN, WM, ST, true>
                         : k_dense_gemm<T, T, WN, WM, ST, false>;
     if (lds > 65536) {
@@ -1078,7 +1159,8 @@ __global__ __launch_bounds__(256) void k_dense_gemm_f32(GemmArgsD p) {
             const int n = n0 + tx * 4 + j;
             if (n >= p.n) break;
             if (p.gated && (j & 1)) continue;
-            float v = activate(acc[i][j] + (p.bias ? p.bias[n] : 0.f), n < p.act_split ? p.act0 : p.act1);
+            float v = activate(acc[i][j] + (p.bias ? p.bias[n] : 0.f), n < p.act_split ? p.act0 : p.act1, p.more.act_a, p.more.act_b);
+            if (p.more.mul) v *= bf2f(p.more.mul[(size_t)min(max(p.more.mul_tokens[*p.more.mul_at + m], 0), p.more.mul_rows - 1) * p.more.ld_mul + n]);
             size_t o = (size_t)blockIdx.z * p.c_batch + (size_t)m * p.ldc + n;
             if (p.gated) {  // (n is even here, and so is the number of columns)
                 v *= acc[i][j < 3 ? j + 1 : 3] + (p.bias ? p.bias[n + 1] : 0.f);
@@ -1110,6 +1192,7 @@ hipError_t launch_dense_gemm(const GemmArgsD &args, hipStream_t s) {
         hipLaunchKernelGGL(k_dense_gemm_f32<false>, dim3((a.n + 63) / 64, (a.m + 63) / 64, a.batch), dim3(256), 0, s, a);
         return hipGetLastError();
     }
+    if (a.more.mul) return a.c_f32 || a.gated ? hipErrorInvalidValue : gemm_go<64, 2, 2, 4, true>(a, s);
     auto tiles = [&](int t) { return (long)((a.n + t - 1) / t) * ((a.m + t - 1) / t) * a.batch; };
     if (a.k <= 1024 && tiles(64) >= 1024) return gemm_go<64, 2, 2, 2>(a, s);  // few steps: what counts is how many workgroups overlap their ends
     if (tiles(128) >= 200) {

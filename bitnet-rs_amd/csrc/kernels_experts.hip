@@ -27,28 +27,98 @@ __device__ __forceinline__ void choose_load(const float *z, int experts, float (
     for (int j = 0; j < PL; ++j) s[j] = l * PL + j < experts ? z[l * PL + j] : -INFINITY;
 }
 
+// the two largest of the pairs (a1 >= a2) and (b1 >= b2)
+__device__ __forceinline__ void two_largest(float &a1, float &a2, float b1, float b2) {
+    const float low = fmaxf(fminf(a1, b1), fmaxf(a2, b2));
+    a1 = fmaxf(a1, b1), a2 = low;
+}
+
+// Choice scores s of a token: those of the groups that are not among the best become minus infinity.
+template <int LT, int PL>
+__device__ __forceinline__ void keep_groups(float (&s)[PL], const Router &r) {
+    const int groups = (int)r.groups, keep = (int)r.keep, size = (int)r.experts / groups;
+    const int lane = threadIdx.x & 63, l = lane & (LT - 1), base = lane & ~(LT - 1);
+    auto worth = [&](float a1, float a2) { return size > 1 ? a1 + a2 : a1; };
+    const int span = size / PL;  // lanes of a group, where it fills them and they are a power of two
+    if (span * PL == size && (span & (span - 1)) == 0) {
+        float a1 = -INFINITY, a2 = -INFINITY;
+#pragma unroll
+        for (int j = 0; j < PL; ++j) two_largest(a1, a2, s[j], -INFINITY);
+        for (int off = 1; off < span; off <<= 1) {
+            const float b1 = __shfl_xor(a1, off, 64), b2 = __shfl_xor(a2, off, 64);
+            two_largest(a1, a2, b1, b2);
+        }
+        const float w = worth(a1, a2);
+        const int mine = l / span;
+        int ahead = 0;
+        for (int g = 0; g < groups; ++g) {
+            const float o = __shfl(w, base + g * span, 64);
+            ahead += o > w || (o == w && g < mine);
+        }
+#pragma unroll
+        for (int j = 0; j < PL; ++j) s[j] = ahead < keep ? s[j] : -INFINITY;
+        return;
+    }
+    // groups that do not: each one's worth by itself; a lane keeps the worth of every expert's group
+    float w[PL];
+    int ahead[PL];
+#pragma unroll
+    for (int j = 0; j < PL; ++j) w[j] = -INFINITY, ahead[j] = 0;
+    auto of_group = [&](int g) {
+        float a1 = -INFINITY, a2 = -INFINITY;
+#pragma unroll
+        for (int j = 0; j < PL; ++j) {
+            const int e = l * PL + j;
+            two_largest(a1, a2, e >= g * size && e < (g + 1) * size ? s[j] : -INFINITY, -INFINITY);
+        }
+        for (int off = 1; off < LT; off <<= 1) {
+            const float b1 = __shfl_xor(a1, off, 64), b2 = __shfl_xor(a2, off, 64);
+            two_largest(a1, a2, b1, b2);
+        }
+        return worth(a1, a2);
+    };
+    for (int g = 0; g < groups; ++g) {
+        const float o = of_group(g);
+#pragma unroll
+        for (int j = 0; j < PL; ++j) w[j] = (l * PL + j) / size == g ? o : w[j];
+    }
+    for (int g = 0; g < groups; ++g) {
+        const float o = of_group(g);
+#pragma unroll
+        for (int j = 0; j < PL; ++j) ahead[j] += o > w[j] || (o == w[j] && g < (l * PL + j) / size);
+    }
+#pragma unroll
+    for (int j = 0; j < PL; ++j) s[j] = ahead[j] < keep ? s[j] : -INFINITY;
+}
+
 template <int LT, int PL>
 __device__ __forceinline__ void choose(float (&s)[PL], const Router &r, int &id, float &weight) {
     const int experts = (int)(r.experts + r.identity), top = (int)r.top;
     const int lane = threadIdx.x & 63, l = lane & (LT - 1), base = lane & ~(LT - 1);
-    float m = -INFINITY, sum = 0.f;
+    if (r.sigmoid) {
 #pragma unroll
-    for (int j = 0; j < PL; ++j) m = fmaxf(m, s[j]);
-    m = token_max<LT>(m);
+        for (int j = 0; j < PL; ++j) s[j] = l * PL + j < experts ? 1.0f / (1.0f + expf(-s[j])) : -INFINITY;
+    } else {
+        float m = -INFINITY, sum = 0.f;
 #pragma unroll
-    for (int j = 0; j < PL; ++j) {
-        s[j] = s[j] == -INFINITY ? 0.f : expf(s[j] - m);
-        sum += s[j];
+        for (int j = 0; j < PL; ++j) m = fmaxf(m, s[j]);
+        m = token_max<LT>(m);
+#pragma unroll
+        for (int j = 0; j < PL; ++j) {
+            s[j] = s[j] == -INFINITY ? 0.f : expf(s[j] - m);
+            sum += s[j];
+        }
+        sum = token_sum<LT>(sum);
+#pragma unroll
+        for (int j = 0; j < PL; ++j) s[j] = l * PL + j < experts ? s[j] / sum : -INFINITY;  // (-infinity: not there, or taken)
     }
-    sum = token_sum<LT>(sum);
-#pragma unroll
-    for (int j = 0; j < PL; ++j) s[j] = l * PL + j < experts ? s[j] / sum : -INFINITY;  // (-infinity: not there, or taken)
     float score[PL];  // without the correction
 #pragma unroll
     for (int j = 0; j < PL; ++j) {
         score[j] = s[j];
         if (r.correction) s[j] += r.correction[min(l * PL + j, experts - 1)];
     }
+    if (r.groups) keep_groups<LT, PL>(s, r);
     id = 0, weight = 0.f;
     float chosen = 0.f;
     for (int k = 0; k < top; ++k) {
@@ -330,22 +400,22 @@ __global__ __launch_bounds__(256) void k_experts_out(OutK p) {
     int g = blockIdx.x * 4 + wave;
     if (g < p.groups) fetch(g, 0);
     const int steps = (end + U - 1) / U * U, total = steps * CH / 4;  // (identity experts have no columns)
-    const float through = a.identity ? *a.identity : 0.f;
+    const float through = a.identity ? *a.identity : 0.f, scale0 = a.x0_scale ? *a.x0_scale : 1.0f;
     constexpr int AH = 12;
     for (int i0 = tid; i0 < total; i0 += 256 * AH) {
         f32x4 v[AH];
-        bool in[AH];
+        float in[AH];  // zero: past a segment's columns
 #pragma unroll
         for (int j = 0; j < AH; ++j) {
             const int i = i0 + 256 * j, c = i / (CH / 4), x = max(c - p.c0, 0), q = min((int)((unsigned)x * p.magic >> 20), max(n_real - 1, 0));
             const bool first = c < p.c0;
             const int col = (first ? i : i - (p.c0 + q * p.ce) * (CH / 4)) * 4, cols = first ? a.cols0 : a.cols1;
-            in[j] = col < cols && c < end;
+            in[j] = col < cols && c < end ? (first ? scale0 : 1.0f) : 0.f;
             v[j] = *reinterpret_cast<const f32x4 *>((first ? a.x0 : a.x1 + (size_t)q * a.ldx1) + min(col, cols - 4));
         }
 #pragma unroll
         for (int j = 0; j < AH; ++j)
-            if (i0 + 256 * j < total) reinterpret_cast<f32x4 *>(xs)[i0 + 256 * j] = in[j] ? v[j] : f32x4{0.f, 0.f, 0.f, 0.f};
+            if (i0 + 256 * j < total) reinterpret_cast<f32x4 *>(xs)[i0 + 256 * j] = in[j] != 0.f ? in[j] * v[j] : f32x4{0.f, 0.f, 0.f, 0.f};
     }
     __syncthreads();
     const int n_wg = gridDim.x;

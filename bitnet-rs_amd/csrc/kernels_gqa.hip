@@ -1,10 +1,10 @@
 // kernels_gqa.hip -- causal attention whose query heads share keys and values in groups, with one softmax map per head or two (gfx950).
-// Optionally rotated queries and keys, chunks of positions that do not see each other, a sink in the softmax's denominator, keys that are the
-// values too, and a gate per head on the output.
+// Optionally rotated queries and keys, chunks of positions that do not see each other, a window, a penalty that grows with the distance, a sink in the
+// softmax's denominator, keys that are the values too, short convolutions ahead of it all, and a gate per head or column on the output.
 //
 // Two maps (differential attention) weigh the same values; a head's output is a1 - lambda a2, divided by its root mean square over the value
 // columns.  Caches: keys [kv head][map][capacity][dimp], values transposed [kv head][vdimp][capacity].
-//   k_gqa_rows     rows of projections: query and key norms, the query's factor at its position, keys and values into the caches
+//   k_gqa_rows     rows of projections: convolution, query and key norms, the query's factor at its position, keys and values into the caches
 //   k_gqa_prefill  a prompt's portion: flash attention on S^T = K Q^T and O^T = V^T P^T, both maps of a query tile in one wave
 //   k_gqa_step     the decode step: norms and append in the same launch, 32 keys per wave and step on the matrix cores
 //   k_gqa_any      any size, f32 or bf16 cache, one wave per key
@@ -18,7 +18,10 @@ namespace bitnet_hip {
 constexpr float kLog2e = 1.44269504088896f;
 
 // the first key a query at this position sees
-__device__ __forceinline__ int gqa_first(const Gqa &p, int pos) { return p.chunk ? pos - (int)((unsigned)pos % (unsigned)p.chunk) : 0; }
+__device__ __forceinline__ int gqa_first(const Gqa &p, int pos) {
+    const int first = p.chunk ? pos - (int)((unsigned)pos % (unsigned)p.chunk) : 0;
+    return p.window ? max(first, pos - (int)p.window + 1) : first;
+}
 
 // The records of a query at `pos`: tiles of keys from `base` (the tile that holds its first key) on, `per` tiles each.
 struct GqaRange {
@@ -37,6 +40,7 @@ __device__ __forceinline__ GqaRange gqa_range(const Gqa &p, int pos) {
 static int gqa_records(const Gqa &g) {
     size_t keys = g.capacity;
     if (g.chunk && g.chunk + kGqaTile < keys) keys = g.chunk + kGqaTile;  // (a chunk may start inside a tile)
+    if (g.window && g.window + kGqaTile < keys) keys = g.window + kGqaTile;
     return (int)min((size_t)kGqaSplits, (keys + kGqaTile - 1) / kGqaTile);
 }
 
@@ -47,10 +51,32 @@ __device__ __forceinline__ float turn_neighbours(float v, int i, const float *cs
     const float c = cs[i >> 1], s = sn[i >> 1];
     return (i & 1) ? v * c + o * s : v * c - o * s;
 }
-// what a head's gate is the sigmoid of
-__device__ __forceinline__ float gate_logit(const Gqa &p, int row, int h) {
-    const size_t i = (size_t)row * p.ldgate + h;
+// what a head's gate (or that of a column of it) is the sigmoid of
+__device__ __forceinline__ float gate_logit(const Gqa &p, int row, int h, int column) {
+    const size_t i = (size_t)row * p.ldgate + (p.gate_columns ? (size_t)h * p.vdimp + column : (size_t)h);
     return p.gate_f32 ? ((const float *)p.gate)[i] : bf2f(((const uint16_t *)p.gate)[i]);
+}
+// a head's distance penalty: what is taken off the natural score is weight * log2(1 + rate * distance)
+struct FarPenalty {
+    float weight, rate;
+};
+__device__ __forceinline__ FarPenalty far_penalty(const Gqa &p, int h) {
+    FarPenalty f{0.f, 0.f};
+    if (p.far_weight) f.weight = p.far_weight[h] * 0.69314718055994531f, f.rate = p.far_rate[h];
+    return f;
+}
+__device__ __forceinline__ float nearer(float score, const FarPenalty &f, int distance) { return fmaf(-f.weight, __log2f(fmaf(f.rate, (float)distance, 1.0f)), score); }
+// columns of a row of projections that a convolution covers
+__host__ __device__ __forceinline__ int gqa_channels(const Gqa &p) {
+    if (p.queries_only) return (int)(p.heads * p.maps * p.dimp);
+    return (int)((p.heads + p.kv_heads) * p.maps * p.dimp + (p.values_are_keys ? 0 : p.kv_heads * p.vdimp));
+}
+// column c of the row of projections t (negative: an earlier portion's; zero ahead of the sequence)
+template <class TR>
+__device__ __forceinline__ float raw_value(const Gqa &p, const TR *rows, size_t ld, int pos0, int t, int c, int channels) {
+    if (t >= 0) return ld_act(rows + (size_t)t * ld, c);
+    const int at = pos0 + t;
+    return at >= 0 ? p.ring[(size_t)(at % (int)p.taps) * channels + c] : 0.f;
 }
 
 size_t gqa_scratch_floats(size_t heads, size_t maps, size_t vdimp, size_t nq) { return nq * heads * maps * kGqaSplits * (kGqaRecHead + vdimp); }
@@ -62,8 +88,8 @@ bool gqa_supported(int dimp, int vdimp) { return dimp <= 256 && vdimp <= 256; }
 constexpr int kRowTokens = 16, kRowCols = 32;
 
 // four tokens of a query or key head of up to 256 columns: a lane holds neighbouring elements, so that a pair turns within it
-template <class TR, class TC>
-__device__ __forceinline__ void head_rows(const Gqa &p, TR *rows, size_t ld, int pos0, int t0, int n, int y, bool key, TC *cache) {
+template <class TR, class TC, bool CONV>
+__device__ __forceinline__ void head_rows(const Gqa &p, const TR *rows, size_t ld, int pos0, int t0, int n, int y, bool key, TC *cache, TR *queries, size_t ldq) {
     constexpr int U = kRowTokens / 4, NJ = 2;
     const int lane = threadIdx.x & 63, dim = (int)p.dim, dimp = (int)p.dimp, turned = (int)p.rot_dims, half = turned >> 1;
     const float *w = key ? p.k_weight : p.q_weight;
@@ -76,12 +102,36 @@ __device__ __forceinline__ void head_rows(const Gqa &p, TR *rows, size_t ld, int
 #pragma unroll
         for (int j = 0; j < NJ; ++j) {
             const int i = min(2 * lane + 128 * j, dimp - 2);
-            v[u][j][0] = ld_act(row, i), v[u][j][1] = ld_act(row, i + 1);
+            if (CONV)
+                v[u][j][0] = v[u][j][1] = 0.f;
+            else
+                v[u][j][0] = ld_act(row, i), v[u][j][1] = ld_act(row, i + 1);
             cs[u][j] = 1.0f, sn[u][j] = 0.f;
             if (turned && 2 * lane + 128 * j < turned) {
                 const size_t at = (size_t)(pos0 + t) * half + lane + 64 * j;
                 cs[u][j] = p.rope_cos[at], sn[u][j] = p.rope_sin[at];
             }
+        }
+    }
+    if (CONV) {
+        const int taps = (int)p.taps, channels = gqa_channels(p);
+        auto add = [&](int k, auto value) {  // tap k of the four tokens
+#pragma unroll
+            for (int j = 0; j < NJ; ++j) {
+                const int c = y * dimp + min(2 * lane + 128 * j, dimp - 2);
+                const float f0 = p.conv[(size_t)k * channels + c], f1 = p.conv[(size_t)k * channels + c + 1];
+#pragma unroll
+                for (int u = 0; u < U; ++u) {
+                    const int t = min(t0 + u, n - 1) - (taps - 1) + k;
+                    v[u][j][0] += f0 * value(t, c), v[u][j][1] += f1 * value(t, c + 1);
+                }
+            }
+        };
+        for (int k = 0; k < taps; ++k) {
+            if (t0 - (taps - 1) + k >= 0)
+                add(k, [&](int t, int c) { return ld_act(rows + (size_t)t * ld, c); });
+            else
+                add(k, [&](int t, int c) { return raw_value(p, rows, ld, pos0, t, c, channels); });
         }
     }
     float wv[NJ][2];
@@ -98,7 +148,7 @@ __device__ __forceinline__ void head_rows(const Gqa &p, TR *rows, size_t ld, int
             factor[u] *= 1.0f / sqrtf(wave_sum(ss) / (float)dim + p.eps);
         }
         if (t0 + u >= n) continue;
-        TR *row = rows + (size_t)(t0 + u) * ld + (size_t)y * dimp;
+        TR *row = queries + (size_t)(t0 + u) * ldq + (size_t)y * dimp;
 #pragma unroll
         for (int j = 0; j < NJ; ++j) {
             const int i = 2 * lane + 128 * j;
@@ -115,10 +165,11 @@ __device__ __forceinline__ void head_rows(const Gqa &p, TR *rows, size_t ld, int
     }
 }
 
-template <class TR, class TC>
-__global__ __launch_bounds__(256) void k_gqa_rows(Gqa p, TR *rows, size_t ld, const int *pos_ptr, int n) {
+// CONV: every column passes a convolution over time first, and the queries go to a place of their own
+template <class TR, class TC, bool CONV>
+__global__ __launch_bounds__(256) void k_gqa_rows(Gqa p, const TR *rows, size_t ld, const int *pos_ptr, int n, TR *queries, size_t ldq) {
     constexpr int STRIDE = sizeof(TR) == 4 ? kRowCols + 1 : kRowCols + 2;
-    __shared__ __attribute__((aligned(16))) TR tile[64 * STRIDE];
+    __shared__ __attribute__((aligned(16))) TR tile[(64 + (CONV ? kMaxTaps - 1 : 0)) * STRIDE];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, pos0 = *pos_ptr;
     const int nq = (int)(p.heads * p.maps), nk = (int)(p.kv_heads * p.maps), dim = (int)p.dim, dimp = (int)p.dimp, vdimp = (int)p.vdimp;
     int y = blockIdx.y;
@@ -129,21 +180,29 @@ __global__ __launch_bounds__(256) void k_gqa_rows(Gqa p, TR *rows, size_t ld, co
         TC *cache = key ? (TC *)p.kcache + (size_t)(y - nq) * p.capacity * dimp : nullptr;
         if (t0 >= n) return;
         if (dimp <= 256) {
-            head_rows<TR, TC>(p, rows, ld, pos0, t0, n, y, key, cache);
+            head_rows<TR, TC, CONV>(p, rows, ld, pos0, t0, n, y, key, cache, queries, ldq);
             return;
         }
+        const int channels = gqa_channels(p), taps = (int)p.taps;
         for (int t = t0; t < min(t0 + kRowTokens / 4, n); ++t) {
-            TR *row = rows + (size_t)t * ld + (size_t)y * dimp;
+            TR *row = queries + (size_t)t * ldq + (size_t)y * dimp;
+            auto value = [&](int i) {
+                if (!CONV) return ld_act(rows + (size_t)t * ld + (size_t)y * dimp, i);
+                float v = 0.f;
+                for (int k = 0; k < taps; ++k) v += p.conv[(size_t)k * channels + y * dimp + i] * raw_value(p, rows, ld, pos0, t - (taps - 1) + k, y * dimp + i, channels);
+                return v;
+            };
             float ss = 0.f;
-            for (int i = lane; i < dimp; i += 64) {
-                const float v = ld_act(row, i);
-                ss += v * v;
-            }
+            if (w || p.unit_norm)
+                for (int i = lane; i < dimp; i += 64) {
+                    const float v = value(i);
+                    ss += v * v;
+                }
             const float norm = w || p.unit_norm ? 1.0f / sqrtf(wave_sum(ss) / (float)dim + p.eps) : 1.0f;
             const float factor = key ? norm : norm * p.q_factor[pos0 + t];
             const float *cs = p.rope_cos + (size_t)(pos0 + t) * half, *sn = p.rope_sin + (size_t)(pos0 + t) * half;
             for (int i = lane; i < dimp; i += 64) {
-                float v = ld_act(row, i) * factor * (w && i < dim ? w[i] : 1.0f);
+                float v = value(i) * factor * (w && i < dim ? w[i] : 1.0f);
                 if (turned) v = turn_neighbours(v, i, cs, sn, turned);
                 if (key)
                     st_act(cache + (size_t)(pos0 + t) * dimp, i, v);
@@ -156,8 +215,16 @@ __global__ __launch_bounds__(256) void k_gqa_rows(Gqa p, TR *rows, size_t ld, co
     if (blockIdx.x % (64 / kRowTokens)) return;
     y -= nq + nk;
     const int t0 = blockIdx.x * kRowTokens, groups = vdimp / kRowCols, head = y / groups, c0 = (y - head * groups) * kRowCols, count = min(64, n - t0);
-    const TR *src = rows + (size_t)(p.values_are_keys ? nq : nq + nk) * dimp + (size_t)head * vdimp + c0;
+    const int column = (p.values_are_keys ? nq : nq + nk) * dimp + head * vdimp + c0;
+    const TR *src = rows + column;
     constexpr int V = 16 / sizeof(TR), PER = kRowCols / V;
+    const int taps = CONV ? (int)p.taps : 1, channels = gqa_channels(p);
+    if (CONV) {  // the tokens ahead of the first one in the tile's last rows
+        for (int i = tid; i < (taps - 1) * kRowCols; i += 256) {
+            const int k = i / kRowCols, c = i % kRowCols;
+            st_act(tile, (64 + k) * STRIDE + c, raw_value(p, rows, ld, pos0, t0 - (taps - 1) + k, column + c, channels));
+        }
+    }
 #pragma unroll
     for (int j = 0; j < 64 * PER / 256; ++j) {
         const int i = tid + 256 * j, t = i / PER, c = i % PER * V;
@@ -173,18 +240,32 @@ __global__ __launch_bounds__(256) void k_gqa_rows(Gqa p, TR *rows, size_t ld, co
 #pragma unroll
         for (int j = 0; j < kRowCols / 4; ++j) {
             const int v = wave * (kRowCols / 4) + j;
-            st_act(cache + (size_t)v * p.capacity, lane, ld_act(tile, lane * STRIDE + v));
+            float x;
+            if (CONV) {
+                x = 0.f;
+                for (int k = 0; k < taps; ++k) {
+                    const int t = lane - (taps - 1) + k;
+                    x += p.conv[(size_t)k * channels + column + v] * ld_act(tile, (t >= 0 ? t : 64 + taps - 1 + t) * STRIDE + v);
+                }
+            } else {
+                x = ld_act(tile, lane * STRIDE + v);
+            }
+            st_act(cache + (size_t)v * p.capacity, lane, x);
         }
 }
 
-hipError_t launch_gqa_rows(const Gqa &g, void *rows, size_t ld, int rows_f32, int cache_f32, const int *pos, int n, hipStream_t s) {
-    const dim3 grid((n + kRowTokens - 1) / kRowTokens, (g.heads + g.kv_heads) * g.maps + g.kv_heads * (g.vdimp / kRowCols));
-    auto go = [&](auto fn, auto *r) {
-        hipLaunchKernelGGL(fn, grid, dim3(256), 0, s, g, r, ld, pos, n);
-        return hipGetLastError();
-    };
-    if (rows_f32) return cache_f32 ? go(k_gqa_rows<float, float>, (float *)rows) : go(k_gqa_rows<float, uint16_t>, (float *)rows);
-    return cache_f32 ? hipErrorInvalidValue : go(k_gqa_rows<uint16_t, uint16_t>, (uint16_t *)rows);
+template <class TR, class TC>
+static hipError_t rows_go(const Gqa &g, const void *rows, size_t ld, const int *pos, int n, void *q, size_t ldq, hipStream_t s) {
+    const int keys = g.queries_only ? 0 : (int)(g.kv_heads * g.maps + g.kv_heads * (g.vdimp / kRowCols));
+    const dim3 grid((n + kRowTokens - 1) / kRowTokens, (int)(g.heads * g.maps) + keys);
+    auto fn = g.taps > 0 ? k_gqa_rows<TR, TC, true> : k_gqa_rows<TR, TC, false>;
+    hipLaunchKernelGGL(fn, grid, dim3(256), 0, s, g, (const TR *)rows, ld, pos, n, (TR *)q, ldq);
+    return hipGetLastError();
+}
+
+hipError_t launch_gqa_rows(const Gqa &g, void *rows, size_t ld, int rows_f32, int cache_f32, const int *pos, int n, void *q, size_t ldq, hipStream_t s) {
+    if (rows_f32) return cache_f32 ? rows_go<float, float>(g, rows, ld, pos, n, q, ldq, s) : rows_go<float, uint16_t>(g, rows, ld, pos, n, q, ldq, s);
+    return cache_f32 ? hipErrorInvalidValue : rows_go<uint16_t, uint16_t>(g, rows, ld, pos, n, q, ldq, s);
 }
 
 // ---- any size ---------------------------------------------------------------------------------------------------------
@@ -206,13 +287,14 @@ __global__ __launch_bounds__(256) void k_gqa_any(Gqa p, const TQ *q, size_t ldq,
     for (int j = 0; j < ND; ++j) qv[j] = lane + 64 * j < dimp ? ld_act(qr, lane + 64 * j) : 0.f;
 #pragma unroll
     for (int j = 0; j < NV; ++j) acc[j] = 0.f;
+    const FarPenalty far = far_penalty(p, h);
     float m = -INFINITY, l = 0.f;
     for (int key = k0 + wave; key < k1; key += 4) {
         float s = 0.f;
 #pragma unroll
         for (int j = 0; j < ND; ++j)
             if (lane + 64 * j < dimp) s += qv[j] * ld_act(K + (size_t)key * dimp, lane + 64 * j);
-        s = wave_sum(s) * kLog2e;
+        s = nearer(wave_sum(s), far, pos - key) * kLog2e;
         const float mn = fmaxf(m, s), al = exp2f(m - mn), w = exp2f(s - mn);
         l = l * al + w;
         m = mn;
@@ -288,7 +370,7 @@ __global__ __launch_bounds__(256, NV > 8 || NK * MAPS >= 8 ? 1 : 2) void k_gqa_s
         for (int v = 0; v < NV; ++v) vf[v] = *reinterpret_cast<const u32x4 *>(V + (size_t)min(v * 16 + r16, vdimp - 1) * p.capacity + kb + g * 8);
     };
     constexpr bool kAhead = NK <= 4;  // the first block is requested ahead of the norms (registers allow it)
-    const bool owner = k1 == n_keys;
+    const bool owner = k1 == n_keys && !p.queries_only;
     if (kAhead) fetch(k0 + wave * 32);
     if (owner) {  // the record that holds the new position appends it (and puts it into its own fragments below)
         if (wave < MAPS) {
@@ -352,6 +434,7 @@ __global__ __launch_bounds__(256, NV > 8 || NK * MAPS >= 8 ? 1 : 2) void k_gqa_s
             q[m][kk] = split8(*reinterpret_cast<const f32x4 *>(src), *reinterpret_cast<const f32x4 *>(src + 4));
         }
     __syncthreads();  // (the area is used again)
+    const FarPenalty far = far_penalty(p, min(h0 + r16, (int)p.heads - 1));
     f32x4 o[NV][MAPS];
     float m[MAPS], l[MAPS];
 #pragma unroll
@@ -396,7 +479,11 @@ __global__ __launch_bounds__(256, NV > 8 || NK * MAPS >= 8 ? 1 : 2) void k_gqa_s
                     hi = mfma_bf16(__builtin_bit_cast(bf16x8, kf[t][j][kk]), q[j][kk].hi, hi);
                     lo = mfma_bf16(__builtin_bit_cast(bf16x8, kf[t][j][kk]), q[j][kk].lo, lo);
                 }
-                s[t] = (hi + lo) * kLog2e;
+                s[t] = hi + lo;
+                if (MAPS == 1 && p.far_weight)
+#pragma unroll
+                    for (int e = 0; e < 4; ++e) s[t][e] = nearer(s[t][e], far, pos - (kb + g * 8 + t * 4 + e));
+                s[t] *= kLog2e;
 #pragma unroll
                 for (int e = 0; e < 4; ++e) {
                     const int key = kb + g * 8 + t * 4 + e;
@@ -485,7 +572,7 @@ __global__ __launch_bounds__(256) void k_gqa_merge(Gqa p, const int *pos_ptr, in
     static_assert(kGqaSplits == 128, "two records per lane of a wave");
     __shared__ float ws[2][kGqaSplits], sinv[2], slot[4];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, h = blockIdx.x, qi = blockIdx.z, maps = (int)p.maps, vdimp = (int)p.vdimp;
-    const float z = p.gate ? gate_logit(p, qi, h) : 0.f, sink = p.sink ? p.sink[h] * kLog2e : -INFINITY;  // (ahead of the chain that starts with the position)
+    const float z = p.gate ? gate_logit(p, qi, h, min(tid, vdimp - 1)) : 0.f, sink = p.sink ? p.sink[h] * kLog2e : -INFINITY;  // (ahead of the chain that starts with the position)
     const int used = gqa_range(p, *pos_ptr + q0 + qi).used;
     const size_t stride = kGqaRecHead + vdimp;
     const float *rec = scratch + ((size_t)qi * p.heads + h) * maps * kGqaSplits * stride;
@@ -540,7 +627,8 @@ __global__ __launch_bounds__(256) void k_gqa_merge(Gqa p, const int *pos_ptr, in
             float t = 0.f;
 #pragma unroll
             for (int k = 0; k < 8; ++k) t += part[k * vdimp + i];
-            return t * (sinv[0] * gate);
+            const float own = p.gate_columns && vdimp > 256 ? activate(gate_logit(p, qi, h, i), BITNET_HIP_ACT_SIGMOID) : gate;
+            return t * (sinv[0] * own);
         }
         const float a = (part[i] + part[2 * vdimp + i]) + (part[4 * vdimp + i] + part[6 * vdimp + i]);
         const float b = (part[vdimp + i] + part[3 * vdimp + i]) + (part[5 * vdimp + i] + part[7 * vdimp + i]);
@@ -628,6 +716,7 @@ __global__ __launch_bounds__(256, NV > 8 || NK > 4 ? 1 : 2) void k_gqa_prefill(G
             if (j * 32 < vdimp) vreg[j] = *reinterpret_cast<const u32x4 *>(vb + (size_t)j * 64 * p.capacity + voff);
     };
     const int n_tiles = (min(n_ctx, pos0 + q0 + 4 * QW) + 63) / 64;
+    const FarPenalty far = far_penalty(p, h);
     // tiles from the first key of the workgroup's first query on; a wave leaves out what lies ahead of its own first key
     const int t_first = gqa_first(p, pos0 + q0) >> 6, w_first = gqa_first(p, pos0 + qw), w_last = gqa_first(p, pos0 + qw + QW - 1);
     fetch(t_first * 64);
@@ -656,6 +745,13 @@ __global__ __launch_bounds__(256, NV > 8 || NK > 4 ? 1 : 2) void k_gqa_prefill(G
                     s[kt][t] = mfma_bf16(a, qf[t][kk], s[kt][t]);
                 }
         }
+        if (MAPS == 1 && p.far_weight)
+#pragma unroll
+            for (int t = 0; t < SLOTS; ++t)
+#pragma unroll
+                for (int kt = 0; kt < 4; ++kt)
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) s[kt][t][i] = nearer(s[kt][t][i], far, qpos[t] - (key0 + kt * 16 + g * 4 + i));
         if (key0 + 63 > pos0 + qw)  // the diagonal
 #pragma unroll
             for (int t = 0; t < SLOTS; ++t)
@@ -723,9 +819,9 @@ __global__ __launch_bounds__(256, NV > 8 || NK > 4 ? 1 : 2) void k_gqa_prefill(G
     for (int t = 0; t < SLOTS / MAPS; ++t) gate[t] = 1.0f;
 #pragma unroll
     for (int t = 0; t < SLOTS; ++t) inv[t] = 1.0f / rows_sum(l[t]);
-    if (p.gate)
+    if (p.gate && !p.gate_columns)
 #pragma unroll
-        for (int t = 0; t < SLOTS / MAPS; ++t) gate[t] = activate(gate_logit(p, min(qw + t * 16 + r16, nq - 1), h), BITNET_HIP_ACT_SIGMOID);
+        for (int t = 0; t < SLOTS / MAPS; ++t) gate[t] = activate(gate_logit(p, min(qw + t * 16 + r16, nq - 1), h, 0), BITNET_HIP_ACT_SIGMOID);
     if (MAPS == 2) {
         float ss = 0.f;
 #pragma unroll
@@ -743,7 +839,14 @@ __global__ __launch_bounds__(256, NV > 8 || NK > 4 ? 1 : 2) void k_gqa_prefill(G
 #pragma unroll
         for (int v = 0; v < NV; ++v)
             if (v * 16 < vdimp) {
-                const f32x4 q = o[v][t] * (inv[t] * gate[t]);
+                f32x4 q = o[v][t] * (inv[t] * gate[t]);
+                if (p.gate_columns) {
+                    float z[4];
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) z[i] = gate_logit(p, qi, h, v * 16 + g * 4 + i);
+#pragma unroll
+                    for (int i = 0; i < 4; ++i) q[i] *= __builtin_amdgcn_rcpf(1.0f + __expf(-z[i]));
+                }
                 *reinterpret_cast<bf16x4 *>(dst + v * 16) = bf16x4{(__bf16)q.x, (__bf16)q.y, (__bf16)q.z, (__bf16)q.w};
             }
     }

@@ -7,7 +7,7 @@
 //   prompt  keys and values of the context are expanded once per layer (matmuls), then k_latent_prefill: flash attention on
 //           S^T = K Q^T and O^T = V^T P^T, probabilities staying in registers.
 // Scores, running maximum, sum and the weights themselves are f32: a weight enters the matrix cores as a (high, low) pair of
-// bf16 values.  A learned sink per head joins the denominator only.
+// bf16 values.  A learned sink per head (where there is one) joins the denominator only.
 #include "dense.hpp"
 
 namespace bitnet_hip {
@@ -51,7 +51,7 @@ __global__ __launch_bounds__(256) void k_latent_decode_any(LatentAttn p) {
     const int k0 = blockIdx.x * per * kLatentTile, k1 = min(k0 + per * kLatentTile, n_keys);
     const int half = p.rot_dim / 2;
     const float *qa = p.qabs + ((size_t)qi * p.heads + h) * p.ldc;
-    const float *qr = p.q + ((size_t)qi * p.heads + h) * p.qd + p.dimp;
+    const float *qr = p.q + (size_t)qi * p.ldq + (size_t)h * p.qd + p.dimp;
     constexpr int NR = 4;
     float q[NJ], r[NR], acc[NJ];
 #pragma unroll
@@ -152,7 +152,7 @@ __global__ __launch_bounds__(512) void k_latent_decode(LatentAttn p) {
         // the query rows, 32 threads each: latent part, then the rotated part
         const int half = p.rot_dim / 2, row = tid >> 5, c4 = (tid & 31) * 4, h = min(h0 + row, p.heads - 1);
         const float *qa = p.qabs + ((size_t)qi * p.heads + h) * ldc;
-        const float *qr = p.q + ((size_t)qi * p.heads + h) * p.qd + p.dimp;
+        const float *qr = p.q + (size_t)qi * p.ldq + (size_t)h * p.qd + p.dimp;
         const float *cs = p.rope_cos + (size_t)pos * half, *sn = p.rope_sin + (size_t)pos * half;
         constexpr int NQ = NCK ? (NCK + 3) / 4 : kDecNT;  // 128 columns at a time
         f32x4 v[NQ];
@@ -320,7 +320,7 @@ __global__ __launch_bounds__(512) void k_latent_merge(LatentMerge p) {
     const size_t stride = kLatentRecHead + p.ldc;
     const float *rec = p.scratch + ((size_t)qi * p.heads + h) * kLatentSplits * stride;
     if (wave == 0) {
-        const float sink = p.sink[h];
+        const float sink = p.sink ? p.sink[h] : -INFINITY;
         float mv[2], lv[2], M = sink;
 #pragma unroll
         for (int e = 0; e < 2; ++e) {
@@ -407,7 +407,7 @@ __global__ __launch_bounds__(256, NV > 8 ? 1 : QT == 1 ? 3 : 2) void k_latent_pr
         const int qi = min(qw + t * 16 + r16, p.nq - 1);
         qpos[t] = pos0 + qw + t * 16 + r16;
         const float sign = p.scale < 0.f ? -1.0f : 1.0f;
-        const uint16_t *q = (const uint16_t *)p.qb + (size_t)qi * p.heads * p.qd + (size_t)h * p.qd;
+        const uint16_t *q = (const uint16_t *)p.qb + (size_t)qi * p.ldq + (size_t)h * p.qd;
         const float *cs = p.rope_cos + (size_t)(pos0 + qi) * half, *sn = p.rope_sin + (size_t)(pos0 + qi) * half;
 #pragma unroll
         for (int kk = 0; kk < NK; ++kk) {
@@ -425,13 +425,13 @@ __global__ __launch_bounds__(256, NV > 8 ? 1 : QT == 1 ? 3 : 2) void k_latent_pr
     }
     // scores stay unscaled up to the exponential (their maximum is then the maximum of the scaled ones: a negative scale's sign goes
     // into the query)
-    const float c2 = fabsf(p.scale) * 1.44269504088896f, sink2 = p.sink[h] * 1.44269504088896f;
+    const float c2 = fabsf(p.scale) * 1.44269504088896f, sink2 = p.sink ? p.sink[h] * 1.44269504088896f : -1e30f;  // (every query sees the first tile's first key)
     f32x4 o[NV][QT];
     float m[QT], l[QT];
 #pragma unroll
     for (int t = 0; t < QT; ++t) {
         m[t] = sink2;
-        l[t] = g == 0 ? 1.0f : 0.0f;
+        l[t] = p.sink && g == 0 ? 1.0f : 0.0f;
 #pragma unroll
         for (int v = 0; v < NV; ++v) o[v][t] = f32x4{0.f, 0.f, 0.f, 0.f};
     }

@@ -104,10 +104,9 @@ Sequence *open_lurepel(const Json &config, const std::string &dir, const OpenOpt
         StackLayerWeights w;
         if (!read_layer(t, s, i, w, err) || model->set_layer((int)i, w) != 0) return failed();
     }
-    std::vector<float> embed_norm, final_norm;
-    const uint16_t *embed = t.matrix("embed", s.vocab, s.width, err), *head = embed ? t.matrix("head", s.vocab, s.width, err) : nullptr;
-    if (!head || !t.vector("embed.norm", s.width, embed_norm, err) || !t.vector("final.norm", s.width, final_norm, err) ||
-        model->set_globals(embed, final_norm, {}, head, nullptr, embed_norm) != 0)
+    StackGlobalWeights g;
+    g.embed = t.matrix("embed", s.vocab, s.width, err), g.head = g.embed ? t.matrix("head", s.vocab, s.width, err) : nullptr;
+    if (!g.head || !t.vector("embed.norm", s.width, g.embed_norm, err) || !t.vector("final.norm", s.width, g.final_norm, err) || model->set_globals(g) != 0)
         return failed();
     return model.release();
 }

@@ -120,11 +120,10 @@ Sequence *open_mimolix(const Json &config, const std::string &dir, const OpenOpt
         StackLayerWeights w;
         if (!read_layer(t, s, i, w, err) || model->set_layer((int)i, w) != 0) return failed();
     }
-    std::vector<float> norm, bias;
-    const uint16_t *embed = t.matrix("embed", s.vocab, s.width, err), *head = embed ? t.matrix("head", s.vocab, s.width, err) : nullptr;
-    const uint16_t *loop_in = head && s.loop.times > 0 ? t.matrix("loop.in", s.width, 2 * (size_t)s.width, err) : nullptr;
-    if (!head || !err.empty() || !t.vector("final.norm", s.width, norm, err) || !t.vector("final.norm.b", s.width, bias, err) ||
-        model->set_globals(embed, norm, bias, head, loop_in) != 0)
+    StackGlobalWeights g;
+    g.embed = t.matrix("embed", s.vocab, s.width, err), g.head = g.embed ? t.matrix("head", s.vocab, s.width, err) : nullptr;
+    g.loop_in = g.head && s.loop.times > 0 ? t.matrix("loop.in", s.width, 2 * (size_t)s.width, err) : nullptr;
+    if (!g.head || !err.empty() || !t.vector("final.norm", s.width, g.final_norm, err) || !t.vector("final.norm.b", s.width, g.final_bias, err) || model->set_globals(g) != 0)
         return failed();
     return model.release();
 }

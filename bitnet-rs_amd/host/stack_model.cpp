@@ -43,13 +43,13 @@ StackModel::StackModel(const StackSpec &spec, bool f32, int max_pos) : spec_(spe
     if (plan_runs() != 0) return;
     for (size_t i = 0; i < layers_.size(); ++i) {
         const LayerSpec &S = spec_.layers[i];
-        const bool own = S.mixer == LayerSpec::Attention || S.mixer == LayerSpec::Delta;
-        if (S.parallel && !own) {
-            err_ = "stack: layer " + std::to_string(i) + ": side by side with the feed-forward stand attention and delta mixers only";
+        const bool own = S.mixer == LayerSpec::Attention || S.mixer == LayerSpec::Delta || (S.mixer == LayerSpec::Latent && S.latent.q_rank == 0);
+        if ((S.parallel || spec_.residual_gate) && !own) {
+            err_ = "stack: layer " + std::to_string(i) + ": side by side with the feed-forward, and gated, stand attention, delta and latent mixers without a query latent only";
             return;
         }
         if (own && plan_block(i, 0, true, S.parallel) != 0) return;
-        if (!S.parallel && S.experts.count > 0 && plan_block(i, 1, false, true) != 0) return;
+        if (!S.parallel && (S.experts.count > 0 || (spec_.residual_gate && S.ff > 0)) && plan_block(i, 1, false, true) != 0) return;
     }
     if (init_sequence(spec.vocab, spec.width, max_pos) != 0) return;
     cap_ = up_to((size_t)max_pos + 1, 128);
@@ -64,13 +64,9 @@ StackModel::StackModel(const StackSpec &spec, bool f32, int max_pos) : spec_(spe
                 err_ = "stack: the rotated part must be even, at most 256 and rotated whole";
                 return;
             }
-            if (m.kv_from >= 0) {
-                const LayerSpec *src = (size_t)m.kv_from < i ? &spec_.layers[(size_t)m.kv_from] : nullptr;
-                if (!src || src->mixer != LayerSpec::Latent || src->latent.kv_from >= 0 || src->latent.kv_rank != m.kv_rank || !(src->latent.rot == m.rot) ||
-                    layers_[(size_t)m.kv_from].slots.size() != L.slots.size()) {
-                    err_ = "stack: layer " + std::to_string(i) + " reads the cache of layer " + std::to_string(m.kv_from) + ", which has none that fits";
-                    return;
-                }
+            if (!fits_source(i)) {
+                err_ = "stack: layer " + std::to_string(i) + " reads the cache of layer " + std::to_string(m.kv_from) + ", which has none that fits";
+                return;
             }
             L.dimp = (int)up_to(m.dim, 32), L.rotp = (int)up_to(std::max(m.rot_dim, 1), 32), L.vdimp = (int)up_to(m.vdim, 32), L.ldc = (int)up_to(m.kv_rank, 64);
             if (L.ldc > 1024) {
@@ -92,18 +88,23 @@ StackModel::StackModel(const StackSpec &spec, bool f32, int max_pos) : spec_(spe
             lin = std::max(lin, (size_t)m.heads * 2 * (L.dimp + L.vdimp));
             lino = std::max(lino, (size_t)m.heads * L.vdimp);
         } else if (S.mixer == LayerSpec::Attention) {
+            if (!fits_source(i)) {
+                err_ = "stack: layer " + std::to_string(i) + " reads the cache of layer " + std::to_string(S.attention.kv_from) + ", which has none that fits";
+                return;
+            }
             scratch = std::max(scratch, bitnet_hip_gqa_scratch_bytes(S.attention.heads, S.attention.maps, L.vdimp, 1) / 4);
         }
         for (const Block &B : L.block)
             if (B.used) {
-                row = std::max(row, (size_t)B.ko + B.fs + B.main + B.tail);
+                row = std::max(row, (size_t)B.ko + B.fs + B.rg + B.main + B.tail);
                 eact = std::max(eact, (size_t)S.experts.top * up_to(S.experts.ff, 64));
             }
         act = std::max(act, (size_t)S.ff);
     }
+    act = std::max(act, up_to(spec_.side_dim, 8));
     auto vec = [&](float **p, size_t n) { return alloc((void **)p, up_to(n, 64) * 4); };
     bool ok = vec(&x_[0], width_) && vec(&x_[1], width_) && vec(&y_[0], width_) && vec(&y_[1], width_) && vec(&z_, z) && vec(&q_, q) && vec(&qabs_, qabs) &&
-              vec(&att_, att) && vec(&act_, act) && vec(&lin_, lin) && vec(&lino_, lino) && vec(&scratch_, scratch) && alloc(&argmax_, 8192) && vec(&x0_, width_) && vec(&row_, row) && vec(&h_, width_) && vec(&eact_, eact) &&
+              vec(&att_, att) && vec(&act_, act) && vec(&lin_, lin) && vec(&lino_, lino) && vec(&scratch_, scratch) && alloc(&argmax_, 8192) && vec(&x0_, width_) && vec(&row_[0], row) && vec(&row_[1], row) && vec(&h_, width_) && vec(&eact_, eact) &&
               alloc((void **)&eids_, 256);
     for (size_t i = 0; ok && i < layers_.size(); ++i) {
         Layer &L = layers_[i];
@@ -116,7 +117,8 @@ StackModel::StackModel(const StackSpec &spec, bool f32, int max_pos) : spec_(spe
                 ok = alloc(&slot.c, cap_ * L.ldc * es) && alloc(&slot.r, cap_ * L.rotp * es);
             } else if (S.mixer == LayerSpec::Attention) {
                 const AttentionSpec &m = S.attention;
-                ok = alloc(&slot.k, cap_ * m.kv_heads * m.maps * L.dimp * es) && alloc(&slot.v, cap_ * m.kv_heads * L.vdimp * es);
+                if (m.kv_from < 0) ok = alloc(&slot.k, cap_ * m.kv_heads * m.maps * L.dimp * es) && alloc(&slot.v, cap_ * m.kv_heads * L.vdimp * es);
+                if (m.taps > 0) ok = ok && alloc((void **)&slot.ring, (size_t)m.taps * L.channels * 4);
             } else if (S.mixer == LayerSpec::Linear || S.mixer == LayerSpec::Delta) {
                 const bool delta = S.mixer == LayerSpec::Delta;
                 slot.state_bytes = (size_t)(delta ? S.delta.heads : S.linear.heads) * L.dimp * L.vdimp * 4;
@@ -137,7 +139,7 @@ StackModel::~StackModel() {
     drop_graphs();
     for (void *p : owned_) hipFree(p);
     for (Buffer *b : {&px_, &ph_, &pz_, &pcq_, &pq_, &pqf_, &pqabs_, &patt_, &py_, &pact_, &pk_, &pvt_, &plin_, &plinf_, &plino_, &pgate_, &pscratch_, &plws_,
-                      &pwant_, &pxw_, &phw_, &plog_, &px0_, &pcat_, &prow_, &ptail_, &pqk_, &pv_, &pgates_, &pplan_, &peact_, &peout_})
+                      &pwant_, &pxw_, &phw_, &plog_, &px0_, &pcat_, &prow_, &ptail_, &pqk_, &pv_, &pgates_, &pplan_, &peact_, &peout_, &pqc_})
         if (b->p) hipFree(b->p);
 }
 
@@ -168,6 +170,20 @@ int StackModel::plan_runs() {
     return 0;
 }
 
+// a layer that reads the keys and values of an earlier one needs them in its own sizes
+bool StackModel::fits_source(size_t i) const {
+    const LayerSpec &S = spec_.layers[i];
+    const int from = S.mixer == LayerSpec::Latent ? S.latent.kv_from : S.attention.kv_from;
+    if (from < 0) return true;
+    if ((size_t)from >= i || spec_.layers[(size_t)from].mixer != S.mixer || layers_[(size_t)from].slots.size() != layers_[i].slots.size()) return false;
+    if (S.mixer == LayerSpec::Latent) {
+        const LatentSpec &a = S.latent, &b = spec_.layers[(size_t)from].latent;
+        return b.kv_from < 0 && a.kv_rank == b.kv_rank && a.rot == b.rot && a.neighbours == b.neighbours;
+    }
+    const AttentionSpec &a = S.attention, &b = spec_.layers[(size_t)from].attention;
+    return b.kv_from < 0 && a.kv_heads == b.kv_heads && a.dim == b.dim && a.vdim == b.vdim && a.maps == b.maps && a.rot == b.rot && a.values_are_keys == b.values_are_keys;
+}
+
 // sizes of a block and of its mixer's padded heads
 int StackModel::plan_block(size_t i, int which, bool mixer, bool ff) {
     Layer &L = layers_[i];
@@ -175,6 +191,7 @@ int StackModel::plan_block(size_t i, int which, bool mixer, bool ff) {
     const LayerSpec &S = spec_.layers[i];
     const std::string where = "stack: layer " + std::to_string(i) + ": ";
     B.used = true, B.mixer = mixer;
+    if (spec_.residual_gate) B.rg = (int)up_to(spec_.width, 64);
     if (mixer && S.mixer == LayerSpec::Attention) {
         const AttentionSpec &m = S.attention;
         L.dimp = (int)up_to(m.dim, 32), L.vdimp = (int)up_to(m.vdim, 32);
@@ -184,9 +201,18 @@ int StackModel::plan_block(size_t i, int which, bool mixer, bool ff) {
             return err_ = where + "attention: an even number of rotated columns within the head, bands in order", BITNET_HIP_ERR_INVALID_ARGUMENT;
         if (m.values_are_keys && (m.vdim != m.dim || m.maps != 1))
             return err_ = where + "attention: keys that are the values have their size, and one map", BITNET_HIP_ERR_INVALID_ARGUMENT;
+        if (m.maps != 1 && (m.far_penalty || m.kv_from >= 0 || m.column_gate))
+            return err_ = where + "attention: distance penalties, another layer's keys and gates per column go with one map", BITNET_HIP_ERR_INVALID_ARGUMENT;
+        if (m.taps < 0 || m.taps > 64 || (m.column_gate && m.head_gate)) return err_ = where + "attention: at most 64 taps, and gates of one kind", BITNET_HIP_ERR_INVALID_ARGUMENT;
         B.ko = (int)up_to((size_t)m.heads * L.vdimp, 64);
-        L.gate_at = (m.heads + m.kv_heads) * m.maps * L.dimp + (m.values_are_keys ? 0 : m.kv_heads * L.vdimp);
-        B.main = L.gate_at + (m.head_gate ? m.heads : 0);
+        L.channels = L.gate_at = m.kv_from >= 0 ? m.heads * L.dimp : (m.heads + m.kv_heads) * m.maps * L.dimp + (m.values_are_keys ? 0 : m.kv_heads * L.vdimp);
+        B.main = L.gate_at + (m.head_gate ? m.heads : m.column_gate ? m.heads * L.vdimp : 0);
+    } else if (mixer && S.mixer == LayerSpec::Latent) {
+        const LatentSpec &m = S.latent;
+        L.dimp = (int)up_to(m.dim, 32), L.rotp = (int)up_to(std::max(m.rot_dim, 1), 32), L.vdimp = (int)up_to(m.vdim, 32);
+        B.ko = (int)up_to((size_t)m.heads * L.vdimp, 64);
+        B.main = m.heads * (L.dimp + L.rotp);
+        B.tail = B.gates = m.kv_from < 0 ? m.kv_rank + m.rot_dim : 0;
     } else if (mixer) {
         const DeltaSpec &m = S.delta;
         L.dimp = (int)up_to(m.dim, 32), L.vdimp = (int)up_to(m.vdim, 32);
@@ -198,13 +224,18 @@ int StackModel::plan_block(size_t i, int which, bool mixer, bool ff) {
     }
     if (ff) {
         const ExpertsSpec &e = S.experts;
-        B.fs = (int)up_to(S.ff, 64);
+        B.fs = (int)up_to(S.ff, 64), B.gated = S.gated && S.ff > 0;
+        if (S.shared_gate) {
+            if (mixer || S.ff == 0 || e.count == 0) return err_ = where + "a gated shared expert stands beside routed ones, behind the mixer", BITNET_HIP_ERR_INVALID_ARGUMENT;
+            B.shared = B.tail = B.gates = 1;
+        }
         if (e.count > 0) {
             if (e.identity < 0 || e.top < 1 || e.top > e.count + e.identity || e.top > 32 || e.count + e.identity > 1024 || e.ff < 1)
                 return err_ = where + "experts: at most 32 of 1024, and not more than there are", BITNET_HIP_ERR_INVALID_ARGUMENT;
+            if (e.groups < 0 || (e.groups > 0 && (e.identity > 0 || e.count % e.groups || e.keep < 1 || e.keep > e.groups || e.top > e.keep * (e.count / e.groups))))
+                return err_ = where + "experts: equal groups, and enough experts in those that are kept", BITNET_HIP_ERR_INVALID_ARGUMENT;
             B.tail += e.count + e.identity;
         }
-        if (S.gated && S.ff > 0) return err_ = where + "a gated feed-forward stands behind its mixer, without routed experts", BITNET_HIP_ERR_INVALID_ARGUMENT;
     }
     return 0;
 }
@@ -298,6 +329,12 @@ void put_taps(std::vector<float> &rows, size_t channels, size_t at, const std::v
         for (size_t c = 0; c < from; ++c)
             for (size_t j = 0; j < taps; ++j) rows[j * channels + at + g * to + c] = w[(g * from + c) * taps + j];
 }
+// a vector [groups][from] at `at` of another one, [groups][to]
+void put_heads(std::vector<float> &o, size_t at, const std::vector<float> &v, size_t groups, size_t from, size_t to) {
+    for (size_t g = 0; g < groups; ++g) std::copy(v.begin() + g * from, v.begin() + (g + 1) * from, o.begin() + at + g * to);
+}
+// where the j-th row of a rotated part of n rows comes from: pairs of neighbours lie half of the part apart on the device
+size_t rotated_row(bool neighbours, size_t n, size_t j) { return !neighbours ? j : j < n / 2 ? 2 * j : 2 * (j - n / 2) + 1; }
 // rows of two matrices in turn
 void append_pairs(std::vector<uint16_t> &o, const uint16_t *a, const uint16_t *b, size_t rows, size_t cols) {
     for (size_t r = 0; r < rows; ++r) {
@@ -333,9 +370,11 @@ int StackModel::set_layer(int layer, const StackLayerWeights &w) {
     TRY(upload(&L.norm1.bias, w.norm1_bias));
     TRY(upload(&L.norm1b, w.norm1b));
     TRY(upload(&L.ls1, w.ls1));
-    if (S.mixer == LayerSpec::Latent) {
+    L.act_a = w.act_a, L.act_b = w.act_b;
+    if (S.mixer == LayerSpec::Latent && S.latent.q_rank > 0) {
         const LatentSpec &m = S.latent;
         const size_t H = m.heads, D = m.dim, R = m.rot_dim, V = m.vdim;
+        if (m.neighbours) return fail_arg("stack: neighbours turn together in queries straight from the input only");
         if (!w.dq || !w.uq || !w.uk || !w.uv || !w.o || (m.kv_from < 0) != (w.dkv != nullptr) || w.dq_norm.size() != (size_t)m.q_rank || w.sink.size() != H ||
             (m.kv_from < 0 && w.dkv_norm.size() != (size_t)m.kv_rank))
             return fail_arg("stack: incomplete latent attention weights");
@@ -350,19 +389,9 @@ int StackModel::set_layer(int layer, const StackLayerWeights &w) {
             memcpy(&t[(h * qd + L.dimp) * m.q_rank], w.uq + (h * (D + R) + D) * m.q_rank, R * m.q_rank * 2);
         }
         TRY(upload_matrix(L.uq, t, (int)(H * qd), m.q_rank));
-        // W_uk twice: as it is (the prompt expands keys) and per head transposed (a step takes the query into latent space)
-        TRY(upload_matrix(L.uk, pad_rows(w.uk, H, D, L.dimp, m.kv_rank), (int)(H * L.dimp), m.kv_rank));
-        t.assign(H * L.ldc * L.dimp, 0);
-        for (size_t h = 0; h < H; ++h)
-            for (size_t d = 0; d < D; ++d)
-                for (size_t c = 0; c < (size_t)m.kv_rank; ++c) t[(h * L.ldc + c) * L.dimp + d] = w.uk[(h * D + d) * m.kv_rank + c];
-        TRY(upload_matrix(L.uk_t, t, (int)(H * L.ldc), L.dimp));
-        weight_bytes_ -= t.size() * 2;  // one of the two copies is read per token
-        TRY(upload_matrix(L.uv, pad_rows(w.uv, H, V, L.vdimp, m.kv_rank), (int)(H * L.vdimp), m.kv_rank));
+        TRY(set_latent(L, m, w));
         TRY(upload_matrix(L.o, pad_cols(w.o, W, H, V, L.vdimp), (int)W, (int)(H * L.vdimp)));
         TRY(upload(&L.dq_norm, w.dq_norm));
-        TRY(upload(&L.dkv_norm, w.dkv_norm));
-        TRY(upload(&L.sink, w.sink));
     } else if (S.mixer == LayerSpec::Linear) {
         const LinearSpec &m = S.linear;
         const size_t H = m.heads, D = m.dim, V = m.vdim;
@@ -392,7 +421,15 @@ int StackModel::set_layer(int layer, const StackLayerWeights &w) {
     }
     for (int b = 0; b < 2; ++b)
         if (L.block[b].used) TRY(set_block((size_t)layer, b, w));
-    if (!S.parallel && S.ff > 0 && S.experts.count == 0) {
+    if (spec_.side_dim > 0) {
+        if (!w.side_gate || !w.side_proj || w.side_norm.size() != W) return fail_arg("stack: incomplete token input");
+        TRY(upload_matrix(L.side_gate, take(w.side_gate, (size_t)spec_.side_dim * W), spec_.side_dim, (int)W));
+        TRY(upload_matrix(L.side_proj, take(w.side_proj, W * spec_.side_dim), (int)W, spec_.side_dim));
+        std::vector<float> norm = w.side_norm;  // (a plain weight, whatever the model's norms have)
+        for (float &v : norm) v -= spec_.norm_offset;
+        TRY(upload(&L.side_norm, norm));
+    }
+    if (!S.parallel && S.ff > 0 && S.experts.count == 0 && !L.block[1].used) {
         const size_t F = S.ff;
         if (!w.up || !w.down || S.gated != (w.gate != nullptr) || (!w.up_b.empty() && (S.gated || w.up_b.size() != F)) || (!w.down_b.empty() && w.down_b.size() != W))
             return fail_arg("stack: incomplete feed-forward weights");
@@ -413,6 +450,22 @@ int StackModel::set_layer(int layer, const StackLayerWeights &w) {
     return 0;
 }
 
+// what latent attention needs besides its down-projections and its output
+int StackModel::set_latent(Layer &L, const LatentSpec &m, const StackLayerWeights &w) {
+    const size_t H = m.heads, D = m.dim, V = m.vdim;
+    // W_uk twice: as it is (the prompt expands keys) and per head transposed (a step takes the query into latent space)
+    TRY(upload_matrix(L.uk, pad_rows(w.uk, H, D, L.dimp, m.kv_rank), (int)(H * L.dimp), m.kv_rank));
+    std::vector<uint16_t> t(H * L.ldc * L.dimp, 0);
+    for (size_t h = 0; h < H; ++h)
+        for (size_t d = 0; d < D; ++d)
+            for (size_t c = 0; c < (size_t)m.kv_rank; ++c) t[(h * L.ldc + c) * L.dimp + d] = w.uk[(h * D + d) * m.kv_rank + c];
+    TRY(upload_matrix(L.uk_t, t, (int)(H * L.ldc), L.dimp));
+    weight_bytes_ -= t.size() * 2;  // one of the two copies is read per token
+    TRY(upload_matrix(L.uv, pad_rows(w.uv, H, V, L.vdimp, m.kv_rank), (int)(H * L.vdimp), m.kv_rank));
+    TRY(upload(&L.dkv_norm, w.dkv_norm));
+    return upload(&L.sink, w.sink);
+}
+
 int StackModel::set_block(size_t i, int which, const StackLayerWeights &w) {
     Layer &L = layers_[i];
     Block &B = L.block[which];
@@ -420,32 +473,93 @@ int StackModel::set_block(size_t i, int which, const StackLayerWeights &w) {
     const size_t W = width_, F = B.mixer && !S.parallel ? 0 : S.ff;
     const ExpertsSpec E = B.mixer && !S.parallel ? ExpertsSpec() : S.experts;
     B.norm = which == 0 ? L.norm1 : L.norm2;
-    std::vector<uint16_t> in((size_t)B.fs * W, 0), out(W * (B.ko + B.fs), 0);
+    std::vector<uint16_t> in, out(W * (B.ko + B.fs), 0);
+    std::vector<float> bias((size_t)B.ff_rows() + B.rg + B.main + B.tail, 0.f);
+    bool biased = false;
+    auto put_bias = [&](size_t at, const std::vector<float> &v, size_t groups, size_t from, size_t to) {
+        if (!v.empty()) put_heads(bias, at, v, groups, from, to), biased = true;
+    };
     auto into_out = [&](const uint16_t *m, size_t at, size_t groups, size_t from, size_t to) {
         for (size_t r = 0; r < W; ++r)
             for (size_t g = 0; g < groups; ++g) memcpy(&out[r * (B.ko + B.fs) + at + g * to], m + (r * groups + g) * from, from * 2);
     };
     if (F > 0) {
-        if (!w.up || !w.down || (!w.up_b.empty() && w.up_b.size() != F) || (!w.down_b.empty() && w.down_b.size() != W)) return fail_arg("stack: incomplete feed-forward weights");
-        memcpy(in.data(), w.up, F * W * 2);
+        if (!w.up || !w.down || B.gated != (w.gate != nullptr) || (!w.up_b.empty() && (B.gated || w.up_b.size() != F)) || (!w.down_b.empty() && w.down_b.size() != W) ||
+            (B.shared != 0) != (w.shared_gate != nullptr))
+            return fail_arg("stack: incomplete feed-forward weights");
+        if (B.gated)
+            append_pairs(in, w.gate, w.up, F, W);
+        else
+            append(in, take(w.up, F * W));
+        in.resize((size_t)B.ff_rows() * W, 0);
+        put_bias(0, w.up_b, 1, F, F);
         into_out(w.down, B.ko, 1, F, F);
     }
+    if (B.rg > 0) {
+        const uint16_t *m = which == 0 ? w.rg1 : w.rg2;
+        const std::vector<float> &b = which == 0 ? w.rg1_b : w.rg2_b;
+        if (!m || (!b.empty() && b.size() != W)) return fail_arg("stack: incomplete residual gate");
+        append(in, take(m, W * W));
+        in.resize((size_t)(B.ff_rows() + B.rg) * W, 0);
+        put_bias(B.ff_rows(), b, 1, W, W);
+    }
+    const size_t proj = B.ff_rows() + B.rg;  // rows ahead of the mixer's
     if (B.mixer && S.mixer == LayerSpec::Attention) {
         const AttentionSpec &m = S.attention;
         const size_t H = m.heads, G = m.kv_heads, M = m.maps, D = m.dim, V = m.vdim;
         const bool two = M == 2 && w.lq1.size() == D && w.lk1.size() == D && w.lq2.size() == D && w.lk2.size() == D;
-        if (!w.q || !w.k || m.values_are_keys != (w.v == nullptr) || m.head_gate != (w.g != nullptr) || !w.o || (!w.q_norm.empty() && w.q_norm.size() != D) ||
-            (!w.k_norm.empty() && w.k_norm.size() != D) || (M == 2 && !two) || (!w.sink.empty() && (w.sink.size() != H || M == 2)))
+        const bool owns = m.kv_from < 0, values = owns && !m.values_are_keys;
+        auto sized = [](const std::vector<float> &v, size_t n) { return v.empty() || v.size() == n; };
+        if (!w.q || owns != (w.k != nullptr) || values != (w.v != nullptr) || (m.head_gate || m.column_gate) != (w.g != nullptr) || !w.o || !sized(w.q_norm, D) ||
+            !sized(w.k_norm, D) || (M == 2 && !two) || (!w.sink.empty() && (w.sink.size() != H || M == 2)) || !sized(w.q_b, H * M * D) || !sized(w.k_b, owns ? G * M * D : 0) ||
+            !sized(w.v_b, values ? G * V : 0) || (m.far_penalty && (w.far_weight.size() != H || w.far_rate.size() != H)))
             return fail_arg("stack: incomplete attention weights");
         append(in, pad_rows(w.q, H * M, D, L.dimp, W));
-        append(in, pad_rows(w.k, G * M, D, L.dimp, W));
+        if (w.k) append(in, pad_rows(w.k, G * M, D, L.dimp, W));
         if (w.v) append(in, pad_rows(w.v, G, V, L.vdimp, W));
-        if (w.g) append(in, take(w.g, H * W));
+        if (w.g) append(in, m.column_gate ? pad_rows(w.g, H, V, L.vdimp, W) : take(w.g, H * W));
+        const size_t k_at = H * M * L.dimp, v_at = k_at + G * M * L.dimp;
+        put_bias(proj, w.q_b, H * M, D, L.dimp);
+        put_bias(proj + k_at, w.k_b, G * M, D, L.dimp);
+        put_bias(proj + v_at, w.v_b, G, V, L.vdimp);
+        if (m.taps > 0) {
+            const size_t T = m.taps, C = L.channels;
+            if (w.q_conv.size() != H * M * D * T || w.k_conv.size() != (owns ? G * M * D * T : 0) || w.v_conv.size() != (values ? G * V * T : 0))
+                return fail_arg("stack: incomplete convolutions");
+            std::vector<float> conv(T * C, 0.f);
+            put_taps(conv, C, 0, w.q_conv, H * M, D, L.dimp, T);
+            if (owns) put_taps(conv, C, k_at, w.k_conv, G * M, D, L.dimp, T);
+            if (values) put_taps(conv, C, v_at, w.v_conv, G, V, L.vdimp, T);
+            TRY(upload(&L.conv, conv));
+        }
+        if (m.far_penalty) {
+            TRY(upload(&L.far_weight, w.far_weight));
+            TRY(upload(&L.far_rate, w.far_rate));
+        }
         into_out(w.o, 0, H, V, L.vdimp);
         TRY(upload(&L.sink, w.sink));
         TRY(upload(&L.q_norm, w.q_norm));
         TRY(upload(&L.k_norm, w.k_norm));
         if (two) L.lambda = (float)(std::exp(dot(w.lq1, w.lk1)) - std::exp(dot(w.lq2, w.lk2)) + m.diff);
+    } else if (B.mixer && S.mixer == LayerSpec::Latent) {
+        const LatentSpec &m = S.latent;
+        const size_t H = m.heads, D = m.dim, R = m.rot_dim, V = m.vdim, qd = L.dimp + L.rotp;
+        if (!w.q || !w.uk || !w.uv || !w.o || (m.kv_from < 0) != (w.dkv != nullptr) || (!w.sink.empty() && w.sink.size() != H) ||
+            (m.kv_from < 0 && w.dkv_norm.size() != (size_t)m.kv_rank))
+            return fail_arg("stack: incomplete latent attention weights");
+        // every head's unrotated part, then its rotated part, each padded on its own
+        std::vector<uint16_t> t(H * qd * W, 0);
+        for (size_t h = 0; h < H; ++h) {
+            memcpy(&t[h * qd * W], w.q + h * (D + R) * W, D * W * 2);
+            for (size_t j = 0; j < R; ++j) memcpy(&t[(h * qd + L.dimp + j) * W], w.q + (h * (D + R) + D + rotated_row(m.neighbours, R, j)) * W, W * 2);
+        }
+        append(in, t);
+        if (w.dkv) {
+            append(in, take(w.dkv, m.kv_rank * W));
+            for (size_t j = 0; j < R; ++j) append(in, take(w.dkv + (m.kv_rank + rotated_row(m.neighbours, R, j)) * W, W));
+        }
+        into_out(w.o, 0, H, V, L.vdimp);
+        TRY(set_latent(L, m, w));
     } else if (B.mixer) {
         const DeltaSpec &m = S.delta;
         const size_t H = m.heads, G = m.kv_heads, D = m.dim, V = m.vdim, T = m.taps, C = 2 * G * L.dimp + H * L.vdimp;
@@ -476,6 +590,7 @@ int StackModel::set_block(size_t i, int which, const StackLayerWeights &w) {
         if (!w.router || w.expert_up.size() != N || w.expert_down.size() != N || w.expert_gate.size() != (E.gated ? N : 0) ||
             (!w.router_correction.empty() && w.router_correction.size() != outputs))
             return fail_arg("stack: incomplete experts");
+        if (B.shared) append(in, take(w.shared_gate, W));
         append(in, take(w.router, outputs * W));
         TRY(upload(&L.correction, w.router_correction));
         std::vector<uint16_t> up, down;
@@ -491,33 +606,37 @@ int StackModel::set_block(size_t i, int which, const StackLayerWeights &w) {
         TRY(upload_matrix(B.expert_down, down, (int)(N * W), (int)R));
         weight_bytes_ -= (N - std::min(N, (size_t)E.top)) * (up_rows + R) * W * 2;  // a token reads `top` of them (fewer where identities are chosen)
     }
-    TRY(upload_matrix(B.in, in, B.fs + B.main + B.tail, (int)W));
+    if (in.size() != bias.size() * W) return fail_arg("stack: a block's rows do not add up");
+    TRY(upload_matrix(B.in, in, (int)bias.size(), (int)W));
     if (B.ko + B.fs > 0) TRY(upload_matrix(B.out, out, (int)W, B.ko + B.fs));
-    if (F > 0 && !w.up_b.empty()) {
-        std::vector<float> bias(B.in.rows, 0.f);
-        std::copy(w.up_b.begin(), w.up_b.end(), bias.begin());
-        TRY(upload(&B.in_bias, bias));
-    }
+    if (biased) TRY(upload(&B.in_bias, bias));
     if (F > 0) TRY(upload(&B.out_bias, w.down_b));
     return 0;
 }
 
-int StackModel::set_globals(const uint16_t *embed, const std::vector<float> &final_norm, const std::vector<float> &final_bias, const uint16_t *head,
-                            const uint16_t *loop_in, const std::vector<float> &embed_norm) {
-    if (!embed || (!embed_norm.empty() && embed_norm.size() != (size_t)width_) || final_norm.size() != (size_t)width_ || (!final_bias.empty() && final_bias.size() != (size_t)width_) || !head ||
-        (spec_.loop.times > 0) != (loop_in != nullptr))
+int StackModel::set_globals(const StackGlobalWeights &w) {
+    const size_t W = width_;
+    if (!w.embed || (!w.embed_norm.empty() && w.embed_norm.size() != W) || w.final_norm.size() != W || (!w.final_bias.empty() && w.final_bias.size() != W) || !w.head ||
+        (spec_.loop.times > 0) != (w.loop_in != nullptr) || (spec_.pairs.buckets > 0) != (w.pairs != nullptr) || (spec_.side_dim > 0) != (w.side != nullptr) ||
+        (w.pairs && !w.embed_norm.empty()))
         return fail_arg("stack: incomplete globals");
     if (head_) return fail_arg("the model already holds its globals");
-    const size_t n = (size_t)vocab_ * width_;
-    TRY(upload_matrix(embed_, take(embed, n), vocab_, width_));
-    weight_bytes_ -= n * 2;  // a row of it is read per token
-    TRY(upload_matrix(head_m_, take(head, n), vocab_, width_));
-    TRY(upload(&embed_norm_, embed_norm));
-    TRY(upload(&final_norm_.w, final_norm));
-    TRY(upload(&final_norm_.bias, final_bias));
-    if (loop_in) {
-        TRY(upload_matrix(loop_in_, take(loop_in, 2 * (size_t)width_ * width_), width_, 2 * width_));
-        weight_bytes_ += (size_t)(spec_.loop.times - 1) * 4 * width_ * width_;
+    const size_t n = (size_t)vocab_ * W;
+    const size_t before = weight_bytes_;
+    TRY(upload_matrix(embed_, take(w.embed, n), vocab_, width_));
+    if (w.pairs) TRY(upload_matrix(pairs_, take(w.pairs, (spec_.pairs.buckets + 1) * W), (int)spec_.pairs.buckets + 1, width_));
+    if (w.side) {
+        const size_t cols = layers_.size() * (size_t)spec_.side_dim;
+        TRY(upload_matrix(side_, take(w.side, vocab_ * cols), vocab_, (int)cols));
+    }
+    weight_bytes_ = before;  // a row of each is read per token
+    TRY(upload_matrix(head_m_, take(w.head, n), vocab_, width_));
+    TRY(upload(&embed_norm_, w.embed_norm));
+    TRY(upload(&final_norm_.w, w.final_norm));
+    TRY(upload(&final_norm_.bias, w.final_bias));
+    if (w.loop_in) {
+        TRY(upload_matrix(loop_in_, take(w.loop_in, 2 * W * W), width_, 2 * width_));
+        weight_bytes_ += (size_t)(spec_.loop.times - 1) * 4 * W * W;
     }
     head_ = head_m_.w;
     return 0;
@@ -538,14 +657,15 @@ int StackModel::clear_state() {
 bitnet_hip_gqa StackModel::gqa_args(size_t i, int pass, const void *proj, size_t ld, bool f32) const {
     const Layer &L = layers_[i];
     const AttentionSpec &m = spec_.layers[i].attention;
-    const Slot &slot = L.slots[(size_t)pass];
+    const Slot &slot = kv_slot(i, pass);
     bitnet_hip_gqa a;
     memset(&a, 0, sizeof(a));
     a.heads = m.heads, a.kv_heads = m.kv_heads, a.maps = m.maps, a.dim = m.dim, a.dimp = L.dimp, a.vdim = m.vdim, a.vdimp = L.vdimp, a.capacity = cap_;
     a.eps = spec_.eps, a.lambda = L.lambda, a.out_scale = 1.0f - m.diff, a.q_weight = L.q_norm, a.k_weight = L.k_norm, a.q_factor = L.q_factor;
     a.kcache = slot.k, a.vcache = slot.v;
     a.unit_norm = m.unit_norm, a.values_are_keys = m.values_are_keys, a.rot_dims = m.rot.dims, a.chunk = m.chunk, a.rope_cos = L.cos, a.rope_sin = L.sin, a.sink = L.sink;
-    if (m.head_gate) a.gate = (const char *)proj + (size_t)L.gate_at * (f32 ? 4 : 2), a.ldgate = ld, a.gate_f32 = f32;
+    a.window = m.window, a.queries_only = m.kv_from >= 0, a.far_weight = L.far_weight, a.far_rate = L.far_rate, a.gate_columns = m.column_gate;
+    if (m.head_gate || m.column_gate) a.gate = (const char *)proj + (size_t)L.gate_at * (f32 ? 4 : 2), a.ldgate = ld, a.gate_f32 = f32;
     return a;
 }
 
@@ -554,6 +674,7 @@ bitnet_hip_router StackModel::router_args(size_t i) const {
     bitnet_hip_router r;
     memset(&r, 0, sizeof(r));
     r.experts = e.count, r.identity = e.identity, r.top = e.top, r.scale = e.scale, r.raw = e.raw, r.correction = layers_[i].correction;
+    r.sigmoid = e.sigmoid, r.groups = e.groups, r.keep = e.keep;
     return r;
 }
 
@@ -575,7 +696,7 @@ void StackModel::attention_args(size_t i, int pass, bitnet_hip_latent_attention 
     const LatentSpec &m = spec_.layers[i].latent;
     a.heads = m.heads, a.dimp = L.dimp, a.qd = L.dimp + L.rotp, a.vdimp = L.vdimp, a.kv_rank = m.kv_rank, a.rot_dim = m.rot_dim;
     a.scale = m.scale, a.sink = L.sink, a.ccache = K.c, a.rcache = K.r, a.ldc = L.ldc, a.ldr = L.rotp, a.capacity = cap_;
-    a.rope_cos = L.cos, a.rope_sin = L.sin;
+    a.rope_cos = L.cos, a.rope_sin = L.sin, a.ldq = 0;
 }
 
 void StackModel::latent_args(size_t i, int pass, const float *z, size_t ldz, void *cq, size_t ldcq, bitnet_hip_latent_rows &r) const {
@@ -594,8 +715,8 @@ void StackModel::latent_args(size_t i, int pass, const float *z, size_t ldz, voi
 // output on the way and leaves the sum in another buffer.
 
 int StackModel::gemv(const bitnet_hip_vector_input &in, const Matrix &m, const float *bias, int act0, int act1, size_t split, float *y,
-                     const bitnet_hip_latent_rows *latent) {
-    BCHK(bitnet_hip_dense_gemv_dev(&in, m.w, m.rows, m.cols, m.ld, bias, act0, act1, split, y, 1, 0, 0, 0, latent, f32_, stream_));
+                     const bitnet_hip_latent_rows *latent, const bitnet_hip_epilogue *more) {
+    BCHK(bitnet_hip_dense_gemv_dev(&in, m.w, m.rows, m.cols, m.ld, bias, act0, act1, split, y, 1, 0, 0, 0, latent, f32_, more, stream_));
     return 0;
 }
 
@@ -610,7 +731,7 @@ static bitnet_hip_vector_input plain_input(const float *x) {
 void StackModel::add_pending(bitnet_hip_vector_input &in) {
     if (!pending_.y) return;
     cur_ = in.x_out = next_x();
-    in.y = pending_.y, in.post_weight = pending_.w, in.scale = pending_.scale, in.mult = spec_.residual_mult;
+    in.y = pending_.y, in.post_weight = pending_.w, in.scale = pending_.scale, in.mult = spec_.residual_mult, in.y_gate = (const float *)pending_.gate;
     pending_ = Pending();
 }
 
@@ -640,33 +761,50 @@ int StackModel::step_block(size_t i, int pass, int which) {
     const Block &B = L.block[which];
     const LayerSpec &S = spec_.layers[i];
     const bool routed = B.expert_up.w != nullptr;
-    const int act = S.act_ff;
     bitnet_hip_vector_input in = block_input(B.norm);
     const float *h = B.norm.w ? h_ : cur_;  // what the experts read
     if (routed && B.norm.w) in.h_out = h_;
-    float *proj = row_ + B.ko + B.fs, *tail = proj + B.main;
-    TRY(gemv(in, B.in, B.in_bias, B.fs ? act : 0, 0, B.fs, row_ + B.ko));
-    if (B.mixer && S.mixer == LayerSpec::Attention) {
+    row_at_ ^= 1;
+    float *row = row_[row_at_], *proj = row + B.ko + B.fs + B.rg, *tail = proj + B.main;
+    // feed-forward | residual gate and the shared expert's number | the rest
+    bitnet_hip_epilogue more = {};
+    const int gates = B.rg + B.shared, gate_act = gates ? BITNET_HIP_ACT_SIGMOID : 0;
+    more.act_a = L.act_a, more.act_b = L.act_b;
+    if (B.gated) more.pairs = B.ff_rows();
+    if (B.fs && gates) more.act2_from = B.ff_rows() + gates;
+    if (B.mixer && S.mixer == LayerSpec::Attention && S.attention.taps > 0) {
+        more.conv_from = B.ff_rows() + B.rg, more.channels = L.channels, more.taps = S.attention.taps;
+        more.conv = L.conv, more.ring = L.slots[(size_t)pass].ring, more.pos = pos_;
+    }
+    if (B.fs)
+        TRY(gemv(in, B.in, B.in_bias, S.act_ff | (B.gated ? BITNET_HIP_ACT_GATED : 0), gate_act, B.ff_rows(), row + B.ko, nullptr, &more));
+    else
+        TRY(gemv(in, B.in, B.in_bias, gate_act, 0, gates, row + B.ko, nullptr, &more));
+    if (B.mixer && S.mixer == LayerSpec::Latent) {
+        bitnet_hip_latent_rows r;
+        latent_args(i, pass, tail, B.tail, nullptr, 0, r);
+        TRY(step_attend_latent(i, pass, proj, S.latent.kv_from < 0 ? &r : nullptr, row, B.ko));
+    } else if (B.mixer && S.mixer == LayerSpec::Attention) {
         const bitnet_hip_gqa a = gqa_args(i, pass, proj, B.main, true);
         if (!f32_ && bitnet_hip_gqa_supported(a.dimp, a.vdimp)) {
             BCHK(bitnet_hip_gqa_step_dev(&a, proj, pos_, scratch_, stream_));
         } else {
-            BCHK(bitnet_hip_gqa_rows_dev(&a, proj, B.main, 1, f32_, pos_, 1, stream_));
+            BCHK(bitnet_hip_gqa_rows_dev(&a, proj, B.main, 1, f32_, pos_, 1, nullptr, 0, stream_));
             BCHK(bitnet_hip_gqa_any_dev(&a, proj, B.main, 1, f32_, pos_, 0, 1, scratch_, stream_));
         }
-        BCHK(bitnet_hip_gqa_merge_dev(&a, pos_, 0, 1, scratch_, row_, B.ko, 0, stream_));
+        BCHK(bitnet_hip_gqa_merge_dev(&a, pos_, 0, 1, scratch_, row, B.ko, 0, stream_));
     } else if (B.mixer) {
         const bitnet_hip_delta d = delta_args(i, pass);
-        BCHK(bitnet_hip_delta_step_dev(&d, proj, tail, pos_, row_, stream_));
+        BCHK(bitnet_hip_delta_step_dev(&d, proj, tail, pos_, row, stream_));
     }
-    if (!routed) return gemv(plain_input(row_), B.out, B.out_bias, 0, 0, 0, y_[which]);
+    if (!routed) return gemv(plain_input(row), B.out, B.out_bias, 0, 0, 0, y_[which]);
     const ExpertsSpec &e = S.experts;
     const bitnet_hip_router r = router_args(i);
     float *identity = e.identity ? (float *)(eids_ + 32) : nullptr;
     BCHK(bitnet_hip_experts_up_dev(tail + B.gates, &r, h, B.expert_up.w, e.gated ? 2 * e.ff : e.ff, B.expert_up.cols, B.expert_up.ld,
                                    e.act | (e.gated ? BITNET_HIP_ACT_GATED : 0), eact_, B.expert_down.ld, eids_, identity, stream_));
-    BCHK(bitnet_hip_experts_out_dev(B.out.w ? row_ : nullptr, B.out.w, B.out.cols, B.out.ld, B.out_bias, eact_, B.expert_down.ld, B.expert_down.w, B.expert_down.cols,
-                                    B.expert_down.ld, eids_, e.top, width_, identity, h, y_[which], stream_));
+    BCHK(bitnet_hip_experts_out_dev(B.out.w ? row : nullptr, B.out.w, B.out.cols, B.out.ld, B.out_bias, eact_, B.expert_down.ld, B.expert_down.w, B.expert_down.cols,
+                                    B.expert_down.ld, eids_, e.top, width_, identity, h, B.shared ? tail : nullptr, y_[which], stream_));
     return 0;
 }
 
@@ -679,15 +817,33 @@ int StackModel::step_latent(size_t i, int pass) {
     bitnet_hip_latent_rows r;
     latent_args(i, pass, z_, L.down_q.rows, nullptr, 0, r);
     TRY(gemv(in, L.uq, nullptr, 0, 0, 0, q_, m.kv_from < 0 ? &r : nullptr));
-    const size_t qd = L.dimp + L.rotp;
-    const bitnet_hip_vector_input qi = plain_input(q_);
-    BCHK(bitnet_hip_dense_gemv_dev(&qi, L.uk_t.w, L.ldc, L.dimp, L.uk_t.ld, nullptr, 0, 0, 0, qabs_, m.heads, (size_t)L.ldc * L.uk_t.ld, qd, L.ldc, nullptr, 0,
-                                   stream_));
+    TRY(step_attend_latent(i, pass, q_, nullptr, att_, (size_t)m.heads * L.vdimp));
+    return gemv(plain_input(att_), L.o, nullptr, 0, 0, 0, y_[0]);
+}
+
+// one query q over the latent cache; rows: the position's latent row, still to be written
+int StackModel::step_attend_latent(size_t i, int pass, const float *q, const bitnet_hip_latent_rows *rows, float *out, size_t ldo) {
+    const Layer &L = layers_[i];
+    const bitnet_hip_vector_input qi = plain_input(q);
+    BCHK(bitnet_hip_dense_gemv_dev(&qi, L.uk_t.w, L.ldc, L.dimp, L.uk_t.ld, nullptr, 0, 0, 0, qabs_, spec_.layers[i].latent.heads, (size_t)L.ldc * L.uk_t.ld, L.dimp + L.rotp,
+                                   L.ldc, rows, f32_, nullptr, stream_));
     bitnet_hip_latent_attention a;
     attention_args(i, pass, a);
-    BCHK(bitnet_hip_latent_decode_dev(&a, q_, qabs_, pos_, 0, 1, f32_, scratch_, stream_));
-    BCHK(bitnet_hip_latent_merge_dev(&a, L.uv.w, pos_, 0, 1, scratch_, att_, (size_t)m.heads * L.vdimp, 0, stream_));
-    return gemv(plain_input(att_), L.o, nullptr, 0, 0, 0, y_[0]);
+    BCHK(bitnet_hip_latent_decode_dev(&a, q, qabs_, pos_, 0, 1, f32_, scratch_, stream_));
+    BCHK(bitnet_hip_latent_merge_dev(&a, L.uv.w, pos_, 0, 1, scratch_, out, ldo, 0, stream_));
+    return 0;
+}
+
+// what the token brings along: norm(W_proj (gelu(W_gate x) * its part of the table's row)) is left to be added
+int StackModel::step_side(size_t i) {
+    const Layer &L = layers_[i];
+    bitnet_hip_epilogue more = {};
+    more.mul = side_.w + i * (size_t)spec_.side_dim, more.ld_mul = side_.ld, more.mul_rows = vocab_, more.mul_tokens = history_, more.mul_at = pos_;
+    TRY(gemv(block_input(Norm()), L.side_gate, nullptr, BITNET_HIP_ACT_GELU_TANH, 0, 0, act_, nullptr, &more));
+    TRY(gemv(plain_input(act_), L.side_proj, nullptr, 0, 0, 0, y_[0]));
+    pending_ = Pending();
+    pending_.y = y_[0], pending_.w = L.side_norm;
+    return 0;
 }
 
 int StackModel::step_linear(size_t i, int pass) {
@@ -703,7 +859,10 @@ int StackModel::step_linear(size_t i, int pass) {
 
 // the embedding output of the n tokens from the position on
 int StackModel::embed_rows(size_t n, float *out) {
-    if (embed_norm_)
+    if (pairs_.w)
+        BCHK(bitnet_hip_embed_pairs_bf16_dev(embed_.w, embed_.ld, pairs_.w, pairs_.ld, spec_.pairs.buckets, spec_.pairs.mul_prev, spec_.pairs.mul_cur, history_, pos_, n, width_,
+                                             vocab_, spec_.embed_scale, out, stream_));
+    else if (embed_norm_)
         BCHK(bitnet_hip_embed_norm_bf16_dev(embed_.w, embed_.ld, history_, pos_, n, width_, vocab_, spec_.embed_scale, embed_norm_, spec_.eps, out, stream_));
     else
         BCHK(bitnet_hip_embed_bf16_dev(embed_.w, embed_.ld, history_, pos_, n, width_, vocab_, spec_.embed_scale, out, stream_));
@@ -712,6 +871,7 @@ int StackModel::embed_rows(size_t n, float *out) {
 
 int StackModel::step(bool with_logits, int) {
     cur_ = x0_;
+    row_at_ = 0;
     pending_ = Pending();
     TRY(embed_rows(1, x0_));
     for (const Run &run : runs_) {
@@ -720,15 +880,25 @@ int StackModel::step(bool with_logits, int) {
         const LayerSpec &S = spec_.layers[i];
         if (run.enters) TRY(step_loop_in());
         TRY(L.block[0].used ? step_block(i, run.pass, 0) : S.mixer == LayerSpec::Latent ? step_latent(i, run.pass) : step_linear(i, run.pass));
-        pending_ = {y_[0], L.norm1b, L.ls1};
-        if (S.parallel || (S.ff == 0 && S.experts.count == 0)) continue;
-        if (L.block[1].used) {
-            TRY(step_block(i, run.pass, 1));
-        } else {
-            TRY(gemv(block_input(L.norm2), L.up, L.up_b, S.act_ff | (S.gated ? BITNET_HIP_ACT_GATED : 0), 0, 0, act_));
-            TRY(gemv(plain_input(act_), L.down, L.down_b, 0, 0, 0, y_[1]));
+        auto leave = [&](int which, const float *norm, const float *scale) {
+            const Block &B = L.block[which];
+            pending_ = Pending();
+            pending_.y = y_[which], pending_.w = norm, pending_.scale = scale;
+            if (B.rg) pending_.gate = row_[row_at_] + B.ko + B.fs;
+        };
+        leave(0, L.norm1b, L.ls1);
+        if (!S.parallel && (S.ff > 0 || S.experts.count > 0)) {
+            if (L.block[1].used) {
+                TRY(step_block(i, run.pass, 1));
+            } else {
+                bitnet_hip_epilogue more = {};
+                more.act_a = L.act_a, more.act_b = L.act_b;
+                TRY(gemv(block_input(L.norm2), L.up, L.up_b, S.act_ff | (S.gated ? BITNET_HIP_ACT_GATED : 0), 0, 0, act_, nullptr, &more));
+                TRY(gemv(plain_input(act_), L.down, L.down_b, 0, 0, 0, y_[1]));
+            }
+            leave(1, L.norm2b, L.ls2);
         }
-        pending_ = {y_[1], L.norm2b, L.ls2};
+        if (spec_.side_dim > 0) TRY(step_side(i));
     }
     if (with_logits) {
         const bitnet_hip_vector_input in = block_input(final_norm_);
@@ -748,26 +918,30 @@ int StackModel::portion_buffers(size_t n) {
     n = up_to(n, 64);
     const size_t es = f32_ ? 4 : 2;
     size_t z = 0, cq = 0, q = 0, qabs = 0, att = 0, act = 0, k = 0, vt = 0, lin = 0, linf = 0, lino = 0, gate = 0, ws = 0, scratch = 0, qf = 0;
-    size_t row = 0, tail = 0, qk = 0, v = 0, gates = 0, plan = 0, eact = 0, eout = 0;
+    size_t row = 0, tail = 0, qk = 0, v = 0, gates = 0, plan = 0, eact = 0, eout = 0, qc = 0;
     for (size_t i = 0; i < layers_.size(); ++i) {
         const Layer &L = layers_[i];
         const LayerSpec &S = spec_.layers[i];
         if (S.mixer == LayerSpec::Latent) {
             const LatentSpec &m = S.latent;
-            z = std::max(z, (size_t)L.down_q.rows);
-            cq = std::max(cq, up_to(m.q_rank, 64));
-            att = std::max(att, (size_t)L.o.ld);
+            const bool direct = m.q_rank == 0;  // (queries in the block's rows)
+            if (!direct) {
+                z = std::max(z, (size_t)L.down_q.rows);
+                cq = std::max(cq, up_to(m.q_rank, 64));
+                att = std::max(att, (size_t)L.o.ld);
+            }
             if (!f32_ && bitnet_hip_latent_prefill_supported(L.dimp + L.rotp, L.vdimp)) {
-                q = std::max(q, (size_t)L.uq.rows);
+                if (!direct) q = std::max(q, (size_t)L.uq.rows);
                 k = std::max(k, (size_t)L.uk.rows);
                 vt = std::max(vt, (size_t)L.uv.rows);
             } else {
-                qf = std::max(qf, (size_t)L.uq.rows);
+                if (!direct || !f32_) qf = std::max(qf, (size_t)m.heads * (L.dimp + L.rotp));
                 qabs = std::max(qabs, (size_t)m.heads * L.ldc);
                 scratch = std::max(scratch, bitnet_hip_latent_scratch_bytes(m.heads, L.ldc, kDecodeSlice));
             }
         } else if (S.mixer == LayerSpec::Attention) {
             const AttentionSpec &m = S.attention;
+            if (m.taps > 0) qc = std::max(qc, (size_t)m.heads * m.maps * L.dimp);
             if (f32_ || !bitnet_hip_gqa_supported(L.dimp, L.vdimp)) scratch = std::max(scratch, bitnet_hip_gqa_scratch_bytes(m.heads, m.maps, L.vdimp, kDecodeSlice));
         } else if (S.mixer == LayerSpec::Delta) {
             const DeltaSpec &m = S.delta;
@@ -788,7 +962,7 @@ int StackModel::portion_buffers(size_t n) {
         }
         for (const Block &B : L.block) {
             if (!B.used) continue;
-            row = std::max(row, up_to((size_t)B.ko + B.fs + B.main, 64));
+            row = std::max(row, up_to((size_t)B.ko + B.fs + B.rg + B.main, 64));
             tail = std::max(tail, up_to(B.tail, 64));
             if (!B.expert_up.w) continue;
             const ExpertsSpec &e = S.experts;
@@ -796,14 +970,15 @@ int StackModel::portion_buffers(size_t n) {
             eact = std::max(eact, (size_t)e.top * B.expert_down.ld);
             eout = std::max(eout, (size_t)e.top * up_to(width_, 64));
         }
-        act = std::max(act, (size_t)L.down.ld);
+        act = std::max(act, (size_t)std::max(L.down.ld, L.side_proj.ld));
     }
     rows_cap_ = 0;
     if (spec_.loop.times > 0) {
         TRY(grow(px0_, n * width_ * 4));
         TRY(grow(pcat_, n * loop_in_.ld * es));
     }
-    TRY(grow(prow_, n * row * es));
+    TRY(grow(prow_, n * row * es + 256));  // (the latent-space product of f32 rows reads up to 32 columns past a head)
+    TRY(grow(pqc_, n * qc * es));
     TRY(grow(ptail_, n * tail * 4));
     TRY(grow(pqk_, n * qk * 4));
     TRY(grow(pv_, n * v * es));
@@ -834,8 +1009,17 @@ int StackModel::portion_buffers(size_t n) {
 }
 
 int StackModel::matmul(const void *a, size_t lda, bool a_f32, const Matrix &m, const float *bias, size_t n, int act0, int act1, size_t split, void *c,
-                       size_t ldc, bool c_f32) {
-    BCHK(bitnet_hip_dense_matmul_dev(a, lda, a_f32, m.w, m.ld, bias, n, m.rows, m.ld, act0, act1, split, c, ldc, c_f32, 1, 0, 0, 0, stream_));
+                       size_t ldc, bool c_f32, const bitnet_hip_epilogue *more) {
+    BCHK(bitnet_hip_dense_matmul_dev(a, lda, a_f32, m.w, m.ld, bias, n, m.rows, m.ld, act0, act1, split, c, ldc, c_f32, 1, 0, 0, 0, more, stream_));
+    return 0;
+}
+
+// rows first .. first + rows - 1 of a block's first product, from ph_
+int StackModel::block_matmul(const Layer &L, const Block &B, int first, int rows, size_t n, int act0, int act1, int split, void *c, size_t ldc, bool c_f32) {
+    bitnet_hip_epilogue more = {};
+    more.act_a = L.act_a, more.act_b = L.act_b;
+    BCHK(bitnet_hip_dense_matmul_dev(ph_.p, up_to(width_, 64), f32_, B.in.w + (size_t)first * B.in.ld, B.in.ld, B.in_bias ? B.in_bias + first : nullptr, n, rows, B.in.ld, act0,
+                                     act1, split, c, ldc, c_f32, 1, 0, 0, 0, &more, stream_));
     return 0;
 }
 
@@ -843,21 +1027,19 @@ int StackModel::matmul(const void *a, size_t lda, bool a_f32, const Matrix &m, c
 int StackModel::portion_norm(size_t n, const Norm *norm, const float *x2, void *h, size_t ldh) {
     const Pending p = pending_;
     pending_ = Pending();
-    const bool post = p.w && !p.experts, own = spec_.center || x2 || !h;
-    if (post) {  // the norm behind the sublayer, and the next one with it where it is of the same kind
-        BCHK(bitnet_hip_residual_norm_rows_dev((float *)px_.p, p.y, width_, p.w, p.scale, own ? nullptr : norm->w, spec_.norm_offset, spec_.eps, n, width_,
-                                               own ? nullptr : h, ldh, f32_, stream_));
-        if (!own || !h) return 0;
+    // the norm behind the sublayer, and the next one with it where it is of the same kind
+    if (p.w && !p.experts && !p.gate && !spec_.center && !x2 && !(h && !norm)) {
+        BCHK(bitnet_hip_residual_norm_rows_dev((float *)px_.p, p.y, width_, p.w, p.scale, h ? norm->w : nullptr, spec_.norm_offset, spec_.eps, n, width_, h, ldh, f32_, stream_));
+        return 0;
     }
     bitnet_hip_sum_rows r;
     memset(&r, 0, sizeof(r));
     r.x = (float *)px_.p, r.m = n, r.width = width_, r.mult = spec_.residual_mult, r.eps = spec_.eps, r.weight_offset = spec_.norm_offset;
     r.center = spec_.center, r.h_f32 = f32_, r.h = h, r.ldh = ldh, r.x2 = x2;
     if (norm) r.weight = norm->w, r.bias = norm->bias;
-    if (!post) {
-        r.y = p.y, r.ldy = width_, r.post_weight = p.w, r.scale = p.scale, r.identity = p.identity, r.input = p.input, r.ld_input = p.input ? up_to(width_, 64) : 0;
-        if (p.experts) r.expert_rows = peout_.p, r.ld_expert = up_to(width_, 64), r.top = plan_.top, r.slots = plan_.slots, r.slot_weights = plan_.weights;
-    }
+    r.y = p.y, r.ldy = width_, r.post_weight = p.w, r.scale = p.scale, r.identity = p.identity, r.input = p.input, r.ld_input = p.input ? up_to(width_, 64) : 0;
+    r.y_scale = p.y_scale, r.ld_y_scale = p.ld_y_scale, r.gate = p.gate, r.ld_gate = p.ld_gate;
+    if (p.experts) r.expert_rows = peout_.p, r.ld_expert = up_to(width_, 64), r.top = plan_.top, r.slots = plan_.slots, r.slot_weights = plan_.weights;
     BCHK(bitnet_hip_sum_norm_rows_dev(&r, stream_));
     return 0;
 }
@@ -872,38 +1054,57 @@ int StackModel::portion_block(size_t i, int pass, int which, size_t n, size_t po
     const Layer &L = layers_[i];
     const Block &B = L.block[which];
     const LayerSpec &S = spec_.layers[i];
-    const size_t ldh = up_to(width_, 64), ld = up_to((size_t)B.ko + B.fs + B.main, 64), ldt = up_to(B.tail, 64), es = f32_ ? 4 : 2;
+    const size_t ldh = up_to(width_, 64), ld = up_to((size_t)B.ko + B.fs + B.rg + B.main, 64), ldt = up_to(B.tail, 64), es = f32_ ? 4 : 2;
     const bool routed = B.expert_up.w != nullptr;
-    char *row = (char *)prow_.p, *proj = row + (size_t)(B.ko + B.fs) * es;
+    char *row = (char *)prow_.p, *gates = row + (size_t)(B.ko + B.fs) * es, *proj = gates + (size_t)B.rg * es;
     float *tail = (float *)ptail_.p;
-    if (B.fs + B.main > 0)
-        BCHK(bitnet_hip_dense_matmul_dev(ph_.p, ldh, f32_, B.in.w, B.in.ld, B.in_bias, n, B.fs + B.main, B.in.ld, B.fs ? S.act_ff : 0, 0, B.fs, row + (size_t)B.ko * es, ld,
-                                         f32_, 1, 0, 0, 0, stream_));
-    if (B.tail > 0)
-        BCHK(bitnet_hip_dense_matmul_dev(ph_.p, ldh, f32_, B.in.w + (size_t)(B.fs + B.main) * B.in.ld, B.in.ld, nullptr, n, B.tail, B.in.ld, 0, 0, 0, tail, ldt, 1, 1, 0, 0,
-                                         0, stream_));
-    if (B.mixer && S.mixer == LayerSpec::Attention) {
+    const bool prefill_latent = !f32_ && bitnet_hip_latent_prefill_supported(L.dimp + L.rotp, L.vdimp);
+    const bool latent = B.mixer && S.mixer == LayerSpec::Latent;
+    const int main = latent && !f32_ && !prefill_latent ? 0 : B.main, sig = B.rg ? BITNET_HIP_ACT_SIGMOID : 0;
+    if (B.gated) {
+        TRY(block_matmul(L, B, 0, B.ff_rows(), n, S.act_ff | BITNET_HIP_ACT_GATED, 0, 0, row + (size_t)B.ko * es, ld, f32_));
+        if (B.rg + main > 0) TRY(block_matmul(L, B, B.ff_rows(), B.rg + main, n, sig, 0, B.rg, gates, ld, f32_));
+    } else if (B.fs && B.rg && main) {
+        TRY(block_matmul(L, B, 0, B.fs + B.rg, n, S.act_ff, sig, B.fs, row + (size_t)B.ko * es, ld, f32_));
+        TRY(block_matmul(L, B, B.fs + B.rg, main, n, 0, 0, 0, proj, ld, f32_));
+    } else if (B.fs + B.rg + main > 0) {
+        TRY(block_matmul(L, B, 0, B.fs + B.rg + main, n, B.fs ? S.act_ff : sig, B.fs ? sig : 0, B.fs ? B.fs : B.rg, row + (size_t)B.ko * es, ld, f32_));
+    }
+    if (B.tail > 0) TRY(block_matmul(L, B, B.ff_rows() + B.rg + B.main, B.tail, n, B.shared ? BITNET_HIP_ACT_SIGMOID : 0, 0, B.shared, tail, ldt, true));
+    if (latent) {
+        bitnet_hip_latent_rows r;
+        latent_args(i, pass, tail, ldt, nullptr, 0, r);
+        if (S.latent.kv_from < 0) BCHK(bitnet_hip_latent_rows_dev(&r, n, f32_, stream_));
+        const float *qf = f32_ ? (const float *)proj : (const float *)pqf_.p;
+        if (main == 0) TRY(block_matmul(L, B, B.ff_rows() + B.rg, B.main, n, 0, 0, 0, pqf_.p, B.main, true));
+        TRY(portion_attend_latent(i, pass, n, pos0, (const uint16_t *)proj, qf, main ? ld : (size_t)B.main, row, ld));
+    } else if (B.mixer && S.mixer == LayerSpec::Attention) {
         bitnet_hip_gqa a = gqa_args(i, pass, proj, ld, f32_);
-        BCHK(bitnet_hip_gqa_rows_dev(&a, proj, ld, f32_, f32_, pos_, n, stream_));
+        const bool conv = S.attention.taps > 0;
+        const size_t ldq = conv ? a.heads * a.maps * a.dimp : ld;
+        const char *q = conv ? (const char *)pqc_.p : proj;
+        if (conv) a.taps = S.attention.taps, a.conv = L.conv, a.ring = L.slots[(size_t)pass].ring;
+        BCHK(bitnet_hip_gqa_rows_dev(&a, proj, ld, f32_, f32_, pos_, n, conv ? pqc_.p : nullptr, ldq, stream_));
+        if (conv) BCHK(bitnet_hip_conv_keep_dev(proj, ld, f32_, L.channels, a.taps, L.slots[(size_t)pass].ring, pos_, n, stream_));
         if (!f32_ && bitnet_hip_gqa_supported(a.dimp, a.vdimp)) {
-            BCHK(bitnet_hip_gqa_prefill_dev(&a, (const uint16_t *)proj, ld, pos0 + n, n, (uint16_t *)row, ld, stream_));
+            BCHK(bitnet_hip_gqa_prefill_dev(&a, (const uint16_t *)q, ldq, pos0 + n, n, (uint16_t *)row, ld, stream_));
         } else {
             for (size_t s = 0; s < n; s += kDecodeSlice) {
                 const size_t k = std::min(kDecodeSlice, n - s);
-                BCHK(bitnet_hip_gqa_any_dev(&a, proj + s * ld * es, ld, f32_, f32_, pos_, s, k, (float *)pscratch_.p, stream_));
+                BCHK(bitnet_hip_gqa_any_dev(&a, q + s * ldq * es, ldq, f32_, f32_, pos_, s, k, (float *)pscratch_.p, stream_));
                 BCHK(bitnet_hip_gqa_merge_dev(&a, pos_, s, k, (const float *)pscratch_.p, row + s * ld * es, ld, !f32_, stream_));
                 if (a.gate) a.gate = (const char *)a.gate + kDecodeSlice * ld * es;
             }
         }
     } else if (B.mixer) {
         const bitnet_hip_delta d = delta_args(i, pass);
-        float *qk = (float *)pqk_.p, *gates = (float *)pgates_.p;
-        BCHK(bitnet_hip_delta_rows_dev(&d, proj, ld, f32_, tail, ldt, pos_, n, qk, pv_.p, gates, stream_));
+        float *qk = (float *)pqk_.p, *decays = (float *)pgates_.p;
+        BCHK(bitnet_hip_delta_rows_dev(&d, proj, ld, f32_, tail, ldt, pos_, n, qk, pv_.p, decays, stream_));
         BCHK(bitnet_hip_delta_keep_dev(&d, proj, ld, f32_, pos_, n, stream_));
         if (!f32_ && bitnet_hip_delta_chunked_supported(L.dimp, L.vdimp))
-            BCHK(bitnet_hip_delta_chunked_dev(&d, qk, (const uint16_t *)pv_.p, gates, (const uint16_t *)proj, ld, n, (uint16_t *)row, ld, plws_.p, plws_.bytes, stream_));
+            BCHK(bitnet_hip_delta_chunked_dev(&d, qk, (const uint16_t *)pv_.p, decays, (const uint16_t *)proj, ld, n, (uint16_t *)row, ld, plws_.p, plws_.bytes, stream_));
         else
-            BCHK(bitnet_hip_delta_recurrent_dev(&d, qk, pv_.p, gates, proj, ld, f32_, n, row, ld, stream_));
+            BCHK(bitnet_hip_delta_recurrent_dev(&d, qk, pv_.p, decays, proj, ld, f32_, n, row, ld, stream_));
     }
     if (B.out.w) TRY(matmul(row, ld, f32_, B.out, B.out_bias, n, 0, 0, 0, py_.p, width_, true));
     if (!routed) return 0;
@@ -921,36 +1122,57 @@ int StackModel::portion_block(size_t i, int pass, int which, size_t n, size_t po
 
 int StackModel::portion_latent(size_t i, int pass, size_t n, size_t pos0) {
     const Layer &L = layers_[i];
-    const Slot &K = kv_slot(i, pass);
     const LatentSpec &m = spec_.layers[i].latent;
-    const size_t ldh = up_to(width_, 64), ldcq = up_to(m.q_rank, 64), qd = L.dimp + L.rotp, lda = L.o.ld, ctx = pos0 + n;
+    const size_t ldh = up_to(width_, 64), ldcq = up_to(m.q_rank, 64), lda = L.o.ld;
     TRY(matmul(ph_.p, ldh, f32_, L.down_q, nullptr, n, 0, 0, 0, pz_.p, L.down_q.rows, true));
     bitnet_hip_latent_rows r;
     latent_args(i, pass, (const float *)pz_.p, L.down_q.rows, pcq_.p, ldcq, r);
     BCHK(bitnet_hip_latent_rows_dev(&r, n, f32_, stream_));
+    const bool prefill = !f32_ && bitnet_hip_latent_prefill_supported(L.dimp + L.rotp, L.vdimp);
+    TRY(matmul(pcq_.p, ldcq, f32_, L.uq, nullptr, n, 0, 0, 0, prefill ? pq_.p : pqf_.p, L.uq.rows, !prefill));
+    TRY(portion_attend_latent(i, pass, n, pos0, (const uint16_t *)pq_.p, (const float *)pqf_.p, L.uq.rows, patt_.p, lda));
+    return matmul(patt_.p, lda, f32_, L.o, nullptr, n, 0, 0, 0, py_.p, width_, true);
+}
+
+// n queries over the latent cache: q (bf16) where the prompt form covers the heads, qf (f32) elsewhere, both ldq apart
+int StackModel::portion_attend_latent(size_t i, int pass, size_t n, size_t pos0, const uint16_t *q, const float *qf, size_t ldq, void *out, size_t ldo) {
+    const Layer &L = layers_[i];
+    const Slot &K = kv_slot(i, pass);
+    const LatentSpec &m = spec_.layers[i].latent;
+    const size_t qd = L.dimp + L.rotp, ctx = pos0 + n;
     bitnet_hip_latent_attention a;
     attention_args(i, pass, a);
+    a.ldq = ldq;
     if (!f32_ && bitnet_hip_latent_prefill_supported(qd, L.vdimp)) {
-        TRY(matmul(pcq_.p, ldcq, false, L.uq, nullptr, n, 0, 0, 0, pq_.p, L.uq.rows, false));
         TRY(matmul(K.c, L.ldc, false, L.uk, nullptr, ctx, 0, 0, 0, pk_.p, L.uk.rows, false));
         // the values transposed: W_uv's rows are the product's rows, the cache its "weights"
         BCHK(bitnet_hip_dense_matmul_dev(L.uv.w, L.uv.ld, 0, (const uint16_t *)K.c, L.ldc, nullptr, L.uv.rows, up_to(ctx, 64), L.ldc, 0, 0, 0, pvt_.p, cap_, 0,
-                                         1, 0, 0, 0, stream_));
-        BCHK(bitnet_hip_latent_prefill_dev(&a, (const uint16_t *)pq_.p, (const uint16_t *)pk_.p, (const uint16_t *)pvt_.p, cap_, ctx, n, (uint16_t *)patt_.p, lda,
-                                           stream_));
-    } else {
-        // in latent space, a slice of queries at a time
-        const size_t es = f32_ ? 4 : 2, ldq = L.uq.rows, ldqa = (size_t)m.heads * L.ldc;
-        TRY(matmul(pcq_.p, ldcq, f32_, L.uq, nullptr, n, 0, 0, 0, pqf_.p, ldq, true));
-        BCHK(bitnet_hip_dense_matmul_dev(pqf_.p, ldq, 1, L.uk_t.w, L.uk_t.ld, nullptr, n, L.ldc, L.uk_t.ld, 0, 0, 0, pqabs_.p, ldqa, 1, m.heads, qd,
-                                         (size_t)L.ldc * L.uk_t.ld, L.ldc, stream_));
-        for (size_t s = 0; s < n; s += kDecodeSlice) {
-            const size_t k = std::min(kDecodeSlice, n - s);
-            BCHK(bitnet_hip_latent_decode_dev(&a, (const float *)pqf_.p + s * ldq, (const float *)pqabs_.p + s * ldqa, pos_, s, k, f32_, (float *)pscratch_.p, stream_));
-            BCHK(bitnet_hip_latent_merge_dev(&a, L.uv.w, pos_, s, k, (const float *)pscratch_.p, (char *)patt_.p + s * lda * es, lda, !f32_, stream_));
-        }
+                                         1, 0, 0, 0, nullptr, stream_));
+        BCHK(bitnet_hip_latent_prefill_dev(&a, q, (const uint16_t *)pk_.p, (const uint16_t *)pvt_.p, cap_, ctx, n, (uint16_t *)out, ldo, stream_));
+        return 0;
     }
-    return matmul(patt_.p, lda, f32_, L.o, nullptr, n, 0, 0, 0, py_.p, width_, true);
+    // in latent space, a slice of queries at a time
+    const size_t es = f32_ ? 4 : 2, ldqa = (size_t)m.heads * L.ldc;
+    BCHK(bitnet_hip_dense_matmul_dev(qf, ldq, 1, L.uk_t.w, L.uk_t.ld, nullptr, n, L.ldc, L.uk_t.ld, 0, 0, 0, pqabs_.p, ldqa, 1, m.heads, qd, (size_t)L.ldc * L.uk_t.ld, L.ldc,
+                                     nullptr, stream_));
+    for (size_t s = 0; s < n; s += kDecodeSlice) {
+        const size_t k = std::min(kDecodeSlice, n - s);
+        BCHK(bitnet_hip_latent_decode_dev(&a, qf + s * ldq, (const float *)pqabs_.p + s * ldqa, pos_, s, k, f32_, (float *)pscratch_.p, stream_));
+        BCHK(bitnet_hip_latent_merge_dev(&a, L.uv.w, pos_, s, k, (const float *)pscratch_.p, (char *)out + s * ldo * es, ldo, !f32_, stream_));
+    }
+    return 0;
+}
+
+int StackModel::portion_side(size_t i, size_t n) {
+    const Layer &L = layers_[i];
+    TRY(portion_norm(n, nullptr, nullptr, ph_.p, up_to(width_, 64)));
+    bitnet_hip_epilogue more = {};
+    more.mul = side_.w + i * (size_t)spec_.side_dim, more.ld_mul = side_.ld, more.mul_rows = vocab_, more.mul_tokens = history_, more.mul_at = pos_;
+    TRY(matmul(ph_.p, up_to(width_, 64), f32_, L.side_gate, nullptr, n, BITNET_HIP_ACT_GELU_TANH, 0, 0, pact_.p, L.side_proj.ld, f32_, &more));
+    TRY(matmul(pact_.p, L.side_proj.ld, f32_, L.side_proj, nullptr, n, 0, 0, 0, py_.p, width_, true));
+    pending_ = Pending();
+    pending_.y = (const float *)py_.p, pending_.w = L.side_norm;
+    return 0;
 }
 
 int StackModel::portion_linear(size_t i, int pass, size_t n) {
@@ -988,17 +1210,30 @@ int StackModel::portion(int rows, int pos0) {
         if (run.enters) TRY(portion_loop_in(n));
         TRY(portion_norm(n, &L.norm1, nullptr, ph_.p, ldh));
         TRY(L.block[0].used ? portion_block(i, run.pass, 0, n, pos0) : S.mixer == LayerSpec::Latent ? portion_latent(i, run.pass, n, pos0) : portion_linear(i, run.pass, n));
-        pending_ = {y, L.norm1b, L.ls1, L.block[0].expert_up.w != nullptr, L.norm1.w ? ph_.p : nullptr, S.experts.identity > 0};
-        if (S.parallel || (S.ff == 0 && S.experts.count == 0)) continue;
-        TRY(portion_norm(n, &L.norm2, nullptr, ph_.p, ldh));
-        if (L.block[1].used) {
-            TRY(portion_block(i, run.pass, 1, n, pos0));
-        } else {
-            TRY(matmul(ph_.p, ldh, f32_, L.up, L.up_b, n, S.act_ff | (S.gated ? BITNET_HIP_ACT_GATED : 0), 0, 0, pact_.p, L.down.ld, f32_));
-            TRY(matmul(pact_.p, L.down.ld, f32_, L.down, L.down_b, n, 0, 0, 0, py_.p, width_, true));
+        auto leave = [&](int which, const Norm &ahead, const float *norm, const float *scale) {
+            const Block &B = L.block[which];
+            const bool routed = B.expert_up.w != nullptr;
+            Pending p;
+            p.y = routed && !B.out.w ? nullptr : y, p.w = norm, p.scale = scale;
+            p.experts = routed, p.input = ahead.w ? ph_.p : nullptr, p.identity = S.experts.identity > 0;
+            if (B.rg) p.gate = (const char *)prow_.p + (size_t)(B.ko + B.fs) * (f32_ ? 4 : 2), p.ld_gate = up_to((size_t)B.ko + B.fs + B.rg + B.main, 64);
+            if (B.shared) p.y_scale = (const float *)ptail_.p, p.ld_y_scale = up_to(B.tail, 64);
+            pending_ = p;
+        };
+        leave(0, L.norm1, L.norm1b, L.ls1);
+        if (!S.parallel && (S.ff > 0 || S.experts.count > 0)) {
+            TRY(portion_norm(n, &L.norm2, nullptr, ph_.p, ldh));
+            if (L.block[1].used) {
+                TRY(portion_block(i, run.pass, 1, n, pos0));
+            } else {
+                bitnet_hip_epilogue more = {};
+                more.act_a = L.act_a, more.act_b = L.act_b;
+                TRY(matmul(ph_.p, ldh, f32_, L.up, L.up_b, n, S.act_ff | (S.gated ? BITNET_HIP_ACT_GATED : 0), 0, 0, pact_.p, L.down.ld, f32_, &more));
+                TRY(matmul(pact_.p, L.down.ld, f32_, L.down, L.down_b, n, 0, 0, 0, py_.p, width_, true));
+            }
+            leave(1, L.norm2, L.norm2b, L.ls2);
         }
-        const bool routed = L.block[1].expert_up.w != nullptr;
-        pending_ = {routed && !L.block[1].out.w ? nullptr : y, L.norm2b, L.ls2, routed, L.norm2.w ? ph_.p : nullptr, S.experts.identity > 0};
+        if (spec_.side_dim > 0) TRY(portion_side(i, n));
     }
     TRY(portion_norm(n, nullptr, nullptr, nullptr, 0));
     hidden_ = x + (n - 1) * (size_t)width_;

@@ -1,11 +1,12 @@
 // stack_model.hpp -- a decoder made of a list of layers, each a sequence mixer and an optional feed-forward.  The mechanisms are
 // parameters (mixer kinds and their sizes, kind and place of norms, layer scale, activations, experts, layers that run several times):
-// a design fills a StackSpec and hands its tensors over (see lasapel.cpp, mimolix.cpp, lurepel.cpp), the stack owns the device layout, the caches and
+// a design fills a StackSpec and hands its tensors over (see lasapel.cpp, mimolix.cpp, lurepel.cpp, sipelorn.cpp), the stack owns the device layout, the caches and
 // states of the live sequence, the launches of a step and of a prompt's portions.
 //
 //   one sublayer behind the other   x <- x + ls1 * norm1b(mixer(norm1(x)));  x <- x + ls2 * norm2b(ff(norm2(x)))
 //   side by side                    x <- x + m * (mixer(norm1(x)) + ff(norm1(x)))
-// (no norm behind a sublayer: m takes the place of ls * norm; no norm ahead of it: the sublayer reads x itself).  A loop runs a range of layers several times with the same weights, every
+// (no norm behind a sublayer: m takes the place of ls * norm; no norm ahead of it: the sublayer reads x itself).  What a sublayer adds may be gated column by
+// column from its input, and behind its sublayers a layer may add what the token itself brings along (a part of a table's row, weighed by x).  A loop runs a range of layers several times with the same weights, every
 // pass with caches and states of its own and, ahead of its first layer, x <- W_in [x; embedding output].
 #pragma once
 
@@ -31,7 +32,8 @@ struct RotarySpec {
 std::vector<double> rotary_frequencies(const RotarySpec &r, double *mult);
 
 struct LatentSpec {  // attention over a shared latent (bitnet_hip_latent_*)
-    int heads = 0, dim = 0, rot_dim = 0, vdim = 0, q_rank = 0, kv_rank = 0;
+    int heads = 0, dim = 0, rot_dim = 0, vdim = 0, q_rank = 0, kv_rank = 0;  // q_rank 0: queries straight from the layer's input
+    bool neighbours = false;  // elements 2 i and 2 i + 1 turn together, not i and i + rot_dim / 2
     float scale = 1.f;
     RotarySpec rot;
     int kv_from = -1;  // the layer whose cache is read instead of one of its own
@@ -51,6 +53,11 @@ struct AttentionSpec {  // keys and values of its own, shared by groups of query
     bool unit_norm = false;                    // queries and keys divided by their root mean square
     bool values_are_keys = false;              // no values of their own
     bool head_gate = false;                    // a factor per head from the layer's input
+    bool column_gate = false;                  // a factor per column of the heads' outputs
+    int window = 0;                            // a position sees itself and the window - 1 positions ahead of it; 0: no window
+    bool far_penalty = false;                  // weight ln(1 + rate * distance) taken off a score, two numbers per head
+    int taps = 0;                              // queries, keys and values pass a causal convolution over that many positions; 0: none
+    int kv_from = -1;                          // the layer whose keys and values are read instead of ones of its own
 };
 struct DeltaSpec {  // gated delta rule (bitnet_hip_delta_*)
     int heads = 0, kv_heads = 0, dim = 0, vdim = 0, taps = 1;
@@ -62,6 +69,8 @@ struct ExpertsSpec {  // routed experts (bitnet_hip_experts_*); count 0: none
     bool raw = false;    // weights as the scores are, not divided by the chosen ones' sum
     bool gated = false;  // act(gate) * up
     int identity = 0;    // experts behind these whose output is their input
+    bool sigmoid = false;        // scores: every logit by itself, not a softmax
+    int groups = 0, keep = 0;    // choice among the experts of the best `keep` of `groups` groups of neighbours; 0: among all
 };
 struct LayerSpec {
     enum Mixer { Latent, Linear, Attention, Delta } mixer = Latent;
@@ -72,11 +81,15 @@ struct LayerSpec {
     bool parallel = false;  // mixer and feed-forward side by side behind one norm (attention and delta mixers)
     int ff = 0;             // every token's feed-forward: dense, or the expert shared by all; 0: none
     int act_ff = BITNET_HIP_ACT_NONE;
-    bool gated = false;     // act_ff(gate) * up (a feed-forward behind the mixer, without routed experts)
+    bool gated = false;     // act_ff(gate) * up
+    bool shared_gate = false;  // the expert shared by all is multiplied by a number per token (not side by side with a mixer)
     ExpertsSpec experts;
 };
 struct LoopSpec {  // layers start .. stop - 1 run `times` times in a row
     int start = 0, stop = 0, times = 0;  // times 0: no loop
+};
+struct PairsSpec {  // a second embedding, of the previous and the current token: row (prev * mul_prev + cur * mul_cur) mod buckets; the first token: row `buckets`
+    uint64_t buckets = 0, mul_prev = 0, mul_cur = 0;  // buckets 0: none
 };
 struct StackSpec {
     int width = 0, vocab = 0;
@@ -85,6 +98,9 @@ struct StackSpec {
     bool center = false;         // block norms are layer norms, with a bias
     float embed_scale = 1.f;
     float residual_mult = 1.f;   // on a sublayer without a norm behind it
+    bool residual_gate = false;  // what a sublayer adds is multiplied by sigmoid(W h + b), h being its input
+    PairsSpec pairs;
+    int side_dim = 0;            // columns of the table of token inputs per layer; 0: no such inputs
     LoopSpec loop;
     std::vector<LayerSpec> layers;
 };
@@ -103,6 +119,19 @@ struct StackLayerWeights {
     const uint16_t *gate = nullptr, *up = nullptr, *down = nullptr, *router = nullptr;
     std::vector<float> up_b, down_b, router_correction;                  // empty correction: none
     std::vector<const uint16_t *> expert_gate, expert_up, expert_down;
+    std::vector<float> q_b, k_b, v_b, far_weight, far_rate;              // attention; empty biases: none
+    const uint16_t *rg1 = nullptr, *rg2 = nullptr;                       // residual gates [width, width]
+    std::vector<float> rg1_b, rg2_b;
+    float act_a = 0.f, act_b = 0.f;                                      // constants of act_ff
+    const uint16_t *shared_gate = nullptr;                               // [1, width]
+    const uint16_t *side_gate = nullptr, *side_proj = nullptr;           // [side_dim, width], [width, side_dim]
+    std::vector<float> side_norm;
+};
+struct StackGlobalWeights {
+    const uint16_t *embed = nullptr, *head = nullptr, *loop_in = nullptr;
+    const uint16_t *pairs = nullptr;  // [buckets + 1, width]
+    const uint16_t *side = nullptr;   // [vocab, layers * side_dim]
+    std::vector<float> final_norm, final_bias, embed_norm;  // empty bias, norm behind the embedding: none
 };
 
 class StackModel : public Sequence {
@@ -111,8 +140,7 @@ class StackModel : public Sequence {
     ~StackModel() override;
 
     int set_layer(int layer, const StackLayerWeights &w);
-    int set_globals(const uint16_t *embed, const std::vector<float> &final_norm, const std::vector<float> &final_bias, const uint16_t *head,
-                    const uint16_t *loop_in, const std::vector<float> &embed_norm = {});
+    int set_globals(const StackGlobalWeights &w);
 
     int prefill(int n, bool with_logits, int digits, float *elapsed_ms) override;
     int forward(const int32_t *tokens, int n, const int32_t *want, int n_want, float *logits) override;
@@ -132,20 +160,24 @@ class StackModel : public Sequence {
     struct Slot {  // what one pass of a layer carries from token to token
         void *c = nullptr, *r = nullptr;       // latent: rows, rotated parts
         void *k = nullptr, *v = nullptr;       // attention: keys, transposed values
-        float *state = nullptr, *ring = nullptr;  // linear, delta: state; delta: the last inputs of its convolution
+        float *state = nullptr, *ring = nullptr;  // linear, delta: state; delta, attention: the last inputs of the convolution
         size_t state_bytes = 0;
     };
     struct Norm {
         float *w = nullptr, *bias = nullptr;
     };
     // Sublayers that read one norm and whose outputs add up, as two products and what lies between them.  A row of activations is
-    // [mixer output, ko | feed-forward, fs | the mixer's projections]; `in` makes everything behind the mixer's output from the normed row (and
-    // the tail: rows whose results stay f32 in a prompt), `out` takes the first ko + fs columns back to the residual stream.
+    // [mixer output, ko | feed-forward, fs | residual gate, rg | the mixer's projections, main]; `in` makes everything behind the mixer's output from the
+    // normed row (and the tail: rows whose results stay f32 in a prompt -- the shared expert's number, the mixer's, the router's), `out` takes the first
+    // ko + fs columns back to the residual stream.
     struct Block {
         bool used = false, mixer = false;
+        bool gated = false;  // the feed-forward's rows of `in` come in pairs
         Norm norm;
         Matrix in, out, expert_up, expert_down;
-        int ko = 0, fs = 0, main = 0, tail = 0, gates = 0;  // gates: rows of the tail ahead of the router
+        int ko = 0, fs = 0, rg = 0, main = 0, tail = 0, gates = 0;  // gates: rows of the tail ahead of the router
+        int shared = 0;                                             // 1: the tail's first row is the shared expert's number
+        int ff_rows() const { return gated ? 2 * fs : fs; }
         float *in_bias = nullptr, *out_bias = nullptr;
     };
     struct Layer {
@@ -157,10 +189,12 @@ class StackModel : public Sequence {
         float *q_norm = nullptr, *k_norm = nullptr, *q_factor = nullptr;
         float lambda = 0.f;
         int gate_at = 0;  // where a row of projections holds the heads' gates
+        int channels = 0;  // columns of it that a convolution covers
+        float *far_weight = nullptr, *far_rate = nullptr;
         // experts
         float *correction = nullptr;
         // delta
-        float *conv = nullptr, *decay_rate = nullptr, *dt_bias = nullptr;
+        float *conv = nullptr /* attention too */, *decay_rate = nullptr, *dt_bias = nullptr;
         // latent
         int dimp = 0, rotp = 0, vdimp = 0, ldc = 0;
         Matrix down_q, uq, uk, uk_t, uv, o;  // down_q: dq, followed by dkv where the layer has one
@@ -171,6 +205,10 @@ class StackModel : public Sequence {
         // feed-forward
         Matrix up, down;
         float *up_b = nullptr, *down_b = nullptr;
+        float act_a = 0.f, act_b = 0.f;
+        // token input
+        Matrix side_gate, side_proj;
+        float *side_norm = nullptr;
         bool set = false;
     };
     struct Buffer {  // grown on demand, zero-filled: what a kernel reads past a matrix is finite
@@ -180,6 +218,10 @@ class StackModel : public Sequence {
     // the sublayer whose output is still to be added to the residual stream
     struct Pending {
         const float *y = nullptr, *w = nullptr, *scale = nullptr;
+        const void *gate = nullptr;   // one token: f32; a portion: rows of ld_gate, of the activations' type
+        size_t ld_gate = 0;
+        const float *y_scale = nullptr;  // a portion: a number per row on y, ld_y_scale apart
+        size_t ld_y_scale = 0;
         bool experts = false;         // a portion's routed rows join in (y may be missing)
         const void *input = nullptr;  // what those experts read, if not the residual stream
         bool identity = false;        // some of them hand it through
@@ -202,26 +244,37 @@ class StackModel : public Sequence {
     int plan_block(size_t i, int which, bool mixer, bool ff);
     bool alloc(void **p, size_t bytes);
     int set_block(size_t i, int which, const StackLayerWeights &w);
-    const Slot &kv_slot(size_t i, int pass) const { return layers_[spec_.layers[i].latent.kv_from >= 0 ? (size_t)spec_.layers[i].latent.kv_from : i].slots[(size_t)pass]; }
+    const Slot &kv_slot(size_t i, int pass) const {
+        const LayerSpec &S = spec_.layers[i];
+        const int from = S.mixer == LayerSpec::Latent ? S.latent.kv_from : S.mixer == LayerSpec::Attention ? S.attention.kv_from : -1;
+        return layers_[from >= 0 ? (size_t)from : i].slots[(size_t)pass];
+    }
+    bool fits_source(size_t i) const;
+    int set_latent(Layer &L, const LatentSpec &m, const StackLayerWeights &w);
     void attention_args(size_t i, int pass, bitnet_hip_latent_attention &a) const;
     void latent_args(size_t i, int pass, const float *z, size_t ldz, void *cq, size_t ldcq, bitnet_hip_latent_rows &r) const;
     bitnet_hip_gqa gqa_args(size_t i, int pass, const void *proj, size_t ld, bool f32) const;
     bitnet_hip_delta delta_args(size_t i, int pass) const;
     // single token
     int gemv(const bitnet_hip_vector_input &in, const Matrix &m, const float *bias, int act0, int act1, size_t split, float *y,
-             const bitnet_hip_latent_rows *latent = nullptr);
+             const bitnet_hip_latent_rows *latent = nullptr, const bitnet_hip_epilogue *more = nullptr);
     bitnet_hip_vector_input block_input(const Norm &norm);
     void add_pending(bitnet_hip_vector_input &in);
     int step_latent(size_t i, int pass);
+    int step_attend_latent(size_t i, int pass, const float *q, const bitnet_hip_latent_rows *rows, float *out, size_t ldo);
+    int step_side(size_t i);
     int step_linear(size_t i, int pass);
     int step_block(size_t i, int pass, int which);
     int step_loop_in();
     // portion of n tokens
     int matmul(const void *a, size_t lda, bool a_f32, const Matrix &m, const float *bias, size_t n, int act0, int act1, size_t split, void *c, size_t ldc,
-               bool c_f32);
+               bool c_f32, const bitnet_hip_epilogue *more = nullptr);
+    int block_matmul(const Layer &L, const Block &B, int first, int rows, size_t n, int act0, int act1, int split, void *c, size_t ldc, bool c_f32);
     int portion(int n, int pos0);
     int portion_norm(size_t n, const Norm *norm, const float *x2, void *h, size_t ldh);
     int portion_latent(size_t i, int pass, size_t n, size_t pos0);
+    int portion_attend_latent(size_t i, int pass, size_t n, size_t pos0, const uint16_t *q, const float *qf, size_t ldq, void *out, size_t ldo);
+    int portion_side(size_t i, size_t n);
     int portion_linear(size_t i, int pass, size_t n);
     int portion_block(size_t i, int pass, int which, size_t n, size_t pos0);
     int portion_loop_in(size_t n);
@@ -234,7 +287,7 @@ class StackModel : public Sequence {
     std::vector<Layer> layers_;
     std::vector<Run> runs_;
     size_t layers_set_ = 0;
-    Matrix embed_, head_m_, loop_in_;
+    Matrix embed_, head_m_, loop_in_, pairs_, side_;
     const uint16_t *head_ = nullptr;
     Norm final_norm_;
     float *embed_norm_ = nullptr;
@@ -246,11 +299,12 @@ class StackModel : public Sequence {
     };
     std::vector<RopeTable> ropes_;
     // single-token vectors (f32); x0_: the embedding output
-    float *x0_ = nullptr, *row_ = nullptr, *h_ = nullptr, *eact_ = nullptr;
+    float *x0_ = nullptr, *row_[2] = {nullptr, nullptr}, *h_ = nullptr, *eact_ = nullptr;
     int32_t *eids_ = nullptr;
     float *x_[2] = {nullptr, nullptr}, *z_ = nullptr, *q_ = nullptr, *qabs_ = nullptr, *att_ = nullptr, *y_[2] = {nullptr, nullptr}, *act_ = nullptr,
           *lin_ = nullptr, *lino_ = nullptr, *scratch_ = nullptr;
     void *argmax_ = nullptr;
+    int row_at_ = 0;  // the row the last block used: its residual gate is read while the next block's is written
     const float *cur_ = nullptr;  // where the step's residual stream is
     float *next_x() const { return cur_ == x_[0] ? x_[1] : x_[0]; }
     Pending pending_;
@@ -258,7 +312,7 @@ class StackModel : public Sequence {
     // portion buffers; T = bf16, or f32 in 32-bit mode
     size_t rows_cap_ = 0;
     Buffer px_, ph_, pz_, pcq_, pq_, pqf_, pqabs_, patt_, py_, pact_, pk_, pvt_, plin_, plinf_, plino_, pgate_, pscratch_, plws_, pwant_, pxw_, phw_, plog_;
-    Buffer px0_, pcat_, prow_, ptail_, pqk_, pv_, pgates_, pplan_, peact_, peout_;
+    Buffer px0_, pcat_, prow_, ptail_, pqk_, pv_, pgates_, pplan_, peact_, peout_, pqc_;
     bitnet_hip_experts_plan plan_;
 };
 

@@ -209,6 +209,55 @@ def write_lurepel(folder: str, config: dict, seed: int = 42) -> str:
     return write_random(folder, config, shapes, seed, lambda name: 0.0 if name.endswith("correction") else 1.0)
 
 
+SIPELORN_SIDE = 256     # columns of a token's input per layer
+SIPELORN_WINDOW = 8192  # positions
+
+
+def sipelorn_config(size: str, n_layers: int, window: int = SIPELORN_WINDOW) -> dict:
+    """attention within a window (heads of 128, kv heads of the size, three taps) with latent attention (heads of 128 + 64 rotated / 128, latent 512) in every
+    fourth layer, the sixth layer on the fifth one's keys; a dense feed-forward of the size in every fourth layer, in the others 64 experts in 8 groups, of which
+    a token takes 8 from 4 groups, and a shared one of the size of two."""
+    s, ff = STACK_SIZES[size], LUREPEL_FF[size]
+    attention = {"heads": s["heads"], "kv_heads": s["n_kv"], "dim": 128, "vdim": 128, "scale": 0.0884, "conv": 3, "mask": {"size": window}}
+    latent = {"heads": s["heads"], "dim": 128, "rot_dim": 64, "vdim": 128, "kv_rank": 512, "scale": 0.0722,
+              "rot": {"base": 500000.0, "dims": 64, "scaling": {"factor": 8.0, "original": 4096, "fast": 32.0, "slow": 1.0}}}
+    expert = ff // 640 * 64  # (ten of them at work: about the active feed-forward of the size)
+    moe = {"kind": "moe", "expert": {"ff": expert}, "router": {"experts": 64, "top": 8, "groups": {"count": 8, "keep": 4}}, "shared": {"ff": 2 * expert}}
+    layers = [{"type": "latent_attention", "mixer": latent, "mlp": moe} if i % 4 == 1 else
+              {"type": "attention", "mixer": dict(attention, kv_from=4) if i == 6 else attention, "mlp": moe if i % 4 else {"kind": "dense", "ff": s["ff"]}}
+              for i in range(n_layers)]
+    return {"architecture": "Sipelorn", "vocab": s["vocab"], "width": s["width"], "norm": {"eps": 1e-6},
+            "embedding": {"scale": 1.0, "bigram": {"buckets": 65521, "mul_prev": 8191, "mul_cur": 127}}, "token_side": {"dim": SIPELORN_SIDE}, "layers": layers}
+
+
+def write_sipelorn(folder: str, config: dict, seed: int = 42) -> str:
+    W, V, side, n = config["width"], config["vocab"], config["token_side"]["dim"], len(config["layers"])
+    shapes = {"embed": (V, W), "bigram": (config["embedding"]["bigram"]["buckets"] + 1, W), "side.embed": (V, n * side), "head": (V, W), "final.norm": (W,), "final.norm.b": (W,)}
+    for i, layer in enumerate(config["layers"]):
+        p, m, f = f"l{i}.", layer["mixer"], layer["mlp"]
+        q, H, D, VD = p + "mix.", m["heads"], m["dim"], m["vdim"]
+        for k in "12":
+            shapes.update({p + "norm" + k: (W,), p + f"norm{k}.b": (W,), p + "rg" + k: (W, W), p + f"rg{k}.b": (W,)})
+        shapes.update({p + "side.gate": (side, W), p + "side.proj": (W, side), p + "side.norm": (W,), q + "o": (W, H * VD)})
+        if layer["type"] == "attention":
+            G = m["kv_heads"]
+            for name, rows in (("q", H * D),) + (() if "kv_from" in m else (("k", G * D), ("v", G * VD))):
+                shapes.update({q + name: (rows, W), q + name + ".b": (rows,), q + name + ".conv": (rows, m["conv"])})
+            shapes.update({q + "g": (H * VD, W), q + "r1": (H,), q + "r2": (H,)})
+        else:
+            R, C = m["rot_dim"], m["kv_rank"]
+            shapes.update({q + "q": (H * (D + R), W), q + "dkv": (C + R, W), q + "dkv.norm": (C,), q + "uk": (H * D, C), q + "uv": (H * VD, C)})
+        if f["kind"] == "dense":
+            shapes.update({p + "mlp.up": (f["ff"], W), p + "mlp.down": (W, f["ff"]), p + "mlp.act": (2,)})
+        else:
+            parts = {f"e{e}": f["expert"]["ff"] for e in range(f["router"]["experts"])}
+            for e, ff in {**parts, "shared": f["shared"]["ff"]}.items():
+                shapes.update({f"{p}mlp.{e}.gate": (ff, W), f"{p}mlp.{e}.up": (ff, W), f"{p}mlp.{e}.down": (W, ff)})
+            shapes.update({p + "mlp.router": (f["router"]["experts"], W), p + "mlp.correction": (f["router"]["experts"],), p + "mlp.shared.sg": (1, W)})
+    ones = ("norm", "norm1", "norm2", "r1", "r2")
+    return write_random(folder, config, shapes, seed, lambda name: 1.0 if name.endswith(ones) else 0.0)
+
+
 def write_lasapel(folder: str, config: dict, seed: int = 42) -> str:
     shapes = {"embed": (config["vocab"], config["width"]), "head": (config["vocab"], config["width"]), "final.norm": (config["width"],)}
     W = config["width"]

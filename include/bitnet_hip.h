@@ -573,6 +573,7 @@ int bitnet_hip_hbm_read_ceiling(size_t bytes, int iters, double *best_gbs, doubl
 #define BITNET_HIP_ACT_SIGMOID 2
 #define BITNET_HIP_ACT_RELU2 3 /* square of relu */
 #define BITNET_HIP_ACT_GELU_TANH 4 /* v / 2 (1 + tanh(sqrt(2 / pi) (v + 0.044715 v^3))) */
+#define BITNET_HIP_ACT_XIELU 5 /* v > 0: a v^2 + v / 2, else b (exp(v) - 1 - v) + v / 2; a, b: bitnet_hip_epilogue.act_a, .act_b */
 /* added to an activation: rows 2 i and 2 i + 1 of W make ONE column, act(row 2 i) * (row 2 i + 1): the number of columns of the output is half
  * the number of rows given (which is even) */
 #define BITNET_HIP_ACT_GATED 0x100
@@ -583,6 +584,11 @@ int bitnet_hip_embed_bf16_dev(const uint16_t *table_dev, size_t ld, const int32_
 /* the same, every row divided by sqrt(mean(v^2) + eps) and multiplied by norm_weight */
 int bitnet_hip_embed_norm_bf16_dev(const uint16_t *table_dev, size_t ld, const int32_t *tokens_dev, const int32_t *offset_dev, size_t n,
                                    size_t width, size_t vocab, float scale, const float *norm_weight_dev, float eps, float *out_dev, void *stream);
+/* scale * table[token] + pairs[(previous token * mul_prev + token * mul_cur) mod buckets], the first token of the sequence (index 0 of tokens): row
+ * `buckets` of pairs, which has buckets + 1 of them */
+int bitnet_hip_embed_pairs_bf16_dev(const uint16_t *table_dev, size_t ld, const uint16_t *pairs_dev, size_t ld_pairs, size_t buckets, uint64_t mul_prev,
+                                    uint64_t mul_cur, const int32_t *tokens_dev, const int32_t *offset_dev, size_t n, size_t width, size_t vocab, float scale,
+                                    float *out_dev, void *stream);
 /* x[i] += scale * norm(y[i]; post_weight) (y NULL: skipped), then h[i] = norm(x[i]; next_weight) (next_weight NULL: x[i] itself; h NULL:
  * skipped), padding columns of h zero; norm(v; w) = v / sqrt(mean(v^2) + eps) * (weight_offset + w). */
 int bitnet_hip_residual_norm_rows_dev(float *x_dev, const float *y_dev, size_t ldy, const float *post_weight_dev, const float *scale_dev,
@@ -592,7 +598,8 @@ int bitnet_hip_residual_norm_rows_dev(float *x_dev, const float *y_dev, size_t l
  * experts' rows alone; top 0: no experts; neither: nothing is added; with `identity` a negative slot stands for the row input[i], or -- input
  * NULL -- for x[i] as it was), x[i] += mult * t or -- post_weight given -- scale * t / sqrt(mean(t^2) + eps) * (weight_offset + post_weight).  Then h[i] (NULL:
  * skipped) = norm(x[i]; weight) (weight NULL: x[i] itself), padding columns zero, or -- x2 given -- the unnormed [x[i]; x2[i]].  center: norm
- * is a layer norm, (v - mean) / sqrt(variance + eps) * weight + bias. */
+ * is a layer norm, (v - mean) / sqrt(variance + eps) * weight + bias.  y_scale: y[i] is multiplied by the number y_scale[i * ld_y_scale] first.  gate:
+ * what is added to x[i] is multiplied by gate[i], column by column. */
 typedef struct bitnet_hip_sum_rows {
     float *x;
     size_t m, width;
@@ -612,6 +619,10 @@ typedef struct bitnet_hip_sum_rows {
     const void *input;                /* of the expert rows' type; may be h */
     size_t ld_input;
     int32_t identity;
+    const float *y_scale;
+    size_t ld_y_scale;
+    const void *gate;                 /* of the expert rows' type */
+    size_t ld_gate;
 } bitnet_hip_sum_rows;
 int bitnet_hip_sum_norm_rows_dev(const bitnet_hip_sum_rows *rows, void *stream);
 /* h[i] = norm(o[i]; weight) * gate[i] over n columns; the mean divides by mean_n (padded heads hold zeros). */
@@ -620,11 +631,30 @@ int bitnet_hip_gated_norm_rows_dev(const float *o_dev, size_t ldo, const float *
                                    void *stream);
 /* out[i] = x[rows[i]] */
 int bitnet_hip_gather_rows_dev(const float *x_dev, const int32_t *rows_dev, size_t n, size_t width, float *out_dev, void *stream);
+/* What else a product does with its rows (all of it optional). */
+typedef struct bitnet_hip_epilogue {
+    float act_a, act_b; /* constants of BITNET_HIP_ACT_XIELU */
+    /* matrix-vector product: with BITNET_HIP_ACT_GATED in act0 only the first `pairs` rows come in pairs (0: all of them); the rows behind them take act1
+     * from act_split on (act_split >= pairs), act2 from act2_from on (0: none) */
+    size_t pairs, act2_from;
+    int32_t act2;
+    /* matrix-vector product: rows conv_from .. conv_from + channels - 1 pass, behind the bias, a causal convolution over time per row: tap j of conv [taps]
+     * [channels] meets the value of taps - 1 - j positions ago (none ahead of position 0).  ring f32 [taps][channels] holds position p's value at row
+     * p % taps; the launch puts its own there. */
+    size_t conv_from, channels, taps;
+    const float *conv;
+    float *ring;
+    const int32_t *pos;
+    /* row i of the output is multiplied, behind the activation, by row mul_tokens[*mul_at + i] of the table mul (a vector product: i = 0) */
+    const uint16_t *mul;
+    size_t ld_mul, mul_rows;
+    const int32_t *mul_tokens, *mul_at;
+} bitnet_hip_epilogue;
 /* C[m][n] = act(A[m][k] . W[n][k]^T + bias), k a multiple of 64 (<= lda, ldw); columns below act_split take act0, the others act1
  * (act_split 0: all act0).  batch > 1: that many products, the operands *_batch elements apart. */
 int bitnet_hip_dense_matmul_dev(const void *a_dev, size_t lda, int a_f32, const uint16_t *w_dev, size_t ldw, const float *bias_dev,
                                 size_t m, size_t n, size_t k, int act0, int act1, size_t act_split, void *c_dev, size_t ldc, int c_f32,
-                                size_t batch, size_t a_batch, size_t w_batch, size_t c_batch, void *stream);
+                                size_t batch, size_t a_batch, size_t w_batch, size_t c_batch, const bitnet_hip_epilogue *more, void *stream);
 
 /* How a matrix-vector product forms its input (every workgroup does so: no launch of its own). */
 #define BITNET_HIP_IN_PLAIN 0
@@ -644,6 +674,7 @@ typedef struct bitnet_hip_vector_input {
     int32_t center;
     const float *bias, *x2;
     float *h_out;
+    const float *y_gate; /* nullable: what is added to x is multiplied by it, element by element */
 } bitnet_hip_vector_input;
 /* The latent rows of a down-projection output z [m][ldz] = [q_rank | kv_rank | rot_dim]: cq[i] = norm(first q_rank; q_weight) (cq NULL:
  * skipped), and at position p = *pos + i of the caches the latent norm(next kv_rank; kv_weight) and the last rot_dim rotated by the
@@ -663,10 +694,10 @@ typedef struct bitnet_hip_latent_rows {
 } bitnet_hip_latent_rows;
 int bitnet_hip_latent_rows_dev(const bitnet_hip_latent_rows *rows, size_t m, int f32, void *stream);
 /* y[rows] = act(W . input + bias), f32 throughout; cols a multiple of 8, <= ld, <= 38400.  batch > 1: member b uses W + b w_batch,
- * x + b x_batch, y + b y_batch (PLAIN input only).  latent (nullable): one more workgroup writes that latent row (m = 1). */
+ * x + b x_batch, y + b y_batch (PLAIN input, and no `more` beyond its activation's constants).  latent (nullable): one more workgroup writes that latent row (m = 1). */
 int bitnet_hip_dense_gemv_dev(const bitnet_hip_vector_input *input, const uint16_t *w_dev, size_t rows, size_t cols, size_t ld,
                               const float *bias_dev, int act0, int act1, size_t act_split, float *y_dev, size_t batch, size_t w_batch,
-                              size_t x_batch, size_t y_batch, const bitnet_hip_latent_rows *latent, int latent_f32, void *stream);
+                              size_t x_batch, size_t y_batch, const bitnet_hip_latent_rows *latent, int latent_f32, const bitnet_hip_epilogue *more, void *stream);
 /* the same product as bitnet_hip_logits_f16_dev's tail: logits, greedy token, history and position (scratch >= 8 KiB; the token's and
  * the position's pointers as there) */
 int bitnet_hip_dense_logits_dev(const bitnet_hip_vector_input *input, const uint16_t *w_dev, size_t vocab, size_t cols, size_t ld,
@@ -674,7 +705,8 @@ int bitnet_hip_dense_logits_dev(const bitnet_hip_vector_input *input, const uint
                                 const int32_t *n_forced_dev, void *stream);
 
 /* Attention over the latent cache.  Head h's query [qd = dimp + ldr]: dimp unrotated (zero-padded to a multiple of 32), then the part to
- * rotate (rot_dim of ldr).  score = (unrotated . W_uk c + rotated . r) * scale; the softmax's denominator also holds exp(sink[h]). */
+ * rotate (rot_dim of ldr).  score = (unrotated . W_uk c + rotated . r) * scale; the softmax's denominator also holds exp(sink[h]) (sink
+ * NULL: nothing more). */
 typedef struct bitnet_hip_latent_attention {
     size_t heads, dimp, qd, vdimp, kv_rank, rot_dim; /* vdimp % 16 == 0 */
     float scale;
@@ -682,6 +714,7 @@ typedef struct bitnet_hip_latent_attention {
     const void *ccache, *rcache;
     size_t ldc, ldr, capacity;
     const float *rope_cos, *rope_sin;
+    size_t ldq; /* leading dimension of the queries, 0: heads * qd */
 } bitnet_hip_latent_attention;
 size_t bitnet_hip_latent_scratch_bytes(size_t heads, size_t ldc, size_t nq);
 /* nq queries at positions *pos + q0 + i, each over the keys up to its own.  q f32 [nq][heads * qd] (rotated part raw), qabs f32
@@ -722,7 +755,11 @@ int bitnet_hip_linear_chunked_dev(const uint16_t *qkv_dev, size_t ld, size_t n, 
  * turned by the tables' row of their position, (u, v) -> (u c - v s, v c + u s), behind the norm and its weight (without a weight the order
  * makes no difference).  chunk > 0: a query at position p sees the keys from floor(p / chunk) chunk on.  sink: the softmax's denominator also holds
  * exp(sink[head]) (one map).  values_are_keys: a row of projections has no values, they are the keys as projected (vdimp = dimp).  gate: every head's
- * output is multiplied by sigmoid(gate[query][head]), the queries counted from the call's first one. */
+ * output is multiplied by sigmoid(gate[query][head]), the queries counted from the call's first one; gate_columns: every column of it by
+ * sigmoid(gate[query][head * vdimp + column]).  window > 0: a query at position p sees itself and the window - 1 keys ahead of it.  far_weight, far_rate:
+ * far_weight[head] ln(1 + far_rate[head] (p - j)) is taken off the score of the key at j (one map).  queries_only: keys and values are another layer's, in the caches
+ * already; a row of projections is [heads * dimp] (one map).  taps > 0: a portion's queries, keys and values pass a causal convolution as described with
+ * bitnet_hip_epilogue (channels: the row of projections), ahead of everything else (gqa_rows; the decode step takes them convolved). */
 typedef struct bitnet_hip_gqa {
     size_t heads, kv_heads, maps, dim, dimp, vdim, vdimp, capacity; /* capacity % 128 == 0 */
     float eps, lambda, out_scale;
@@ -735,12 +772,19 @@ typedef struct bitnet_hip_gqa {
     const float *sink;                /* [heads] */
     const void *gate;                 /* [queries][ldgate], f32 or bf16 */
     size_t ldgate;
-    int32_t gate_f32;
+    int32_t gate_f32, gate_columns, queries_only;
+    size_t window, taps;
+    const float *far_weight, *far_rate; /* [heads] */
+    const float *conv, *ring;           /* [taps][a row of projections] */
 } bitnet_hip_gqa;
 size_t bitnet_hip_gqa_scratch_bytes(size_t heads, size_t maps, size_t vdimp, size_t nq);
-/* n rows of projections from position *pos on: queries in place, keys and values into the caches. */
+/* n rows of projections from position *pos on: queries into q [n][ldq] (NULL: in place; with taps they need a place of their own), keys and values into the
+ * caches. */
 int bitnet_hip_gqa_rows_dev(const bitnet_hip_gqa *attn, void *rows_dev, size_t ld, int rows_f32, int cache_f32, const int32_t *pos_dev, size_t n,
-                            void *stream);
+                            void *q_dev, size_t ldq, void *stream);
+/* the first `channels` columns of a portion's last rows into a convolution's ring, behind whatever reads the ring */
+int bitnet_hip_conv_keep_dev(const void *rows_dev, size_t ld, int rows_f32, size_t channels, size_t taps, float *ring_dev, const int32_t *pos_dev, size_t n,
+                             void *stream);
 /* The decode step on a bf16 cache: one raw f32 row of projections at *pos, appended by the same launch; leaves records in scratch.
  * dimp <= 256, vdimp <= 256 (bitnet_hip_gqa_supported). */
 int bitnet_hip_gqa_supported(size_t dimp, size_t vdimp);
@@ -788,13 +832,17 @@ int bitnet_hip_delta_chunked_dev(const bitnet_hip_delta *d, const float *qk_dev,
                                  size_t ld, size_t n, uint16_t *out_dev, size_t ldo, void *workspace_dev, size_t workspace_bytes, void *stream);
 
 /* Mixture of experts.  A router has one logit per expert and, behind them, one per identity expert, whose output is its input.  scores =
- * softmax(logits); chosen are the `top` largest of score + correction (correction NULL: of the scores; lower index first among equals), their
- * weights are score / (the chosen scores' sum + 1e-20) * scale, or -- raw -- score * scale.  experts + identity <= 1024, top <= 32. */
+ * softmax(logits), or -- sigmoid -- of every logit by itself; chosen are the `top` largest of score + correction (correction NULL: of the scores; lower index first among equals), their
+ * weights are score / (the chosen scores' sum + 1e-20) * scale, or -- raw -- score * scale.  experts + identity <= 1024, top <= 32.
+ * groups > 0: the experts form that many equal groups of neighbours (no identities), a group is worth the sum of its two largest score + correction, and only
+ * experts of the `keep` groups that are worth most can be chosen (lower index first among equals). */
 typedef struct bitnet_hip_router {
     size_t experts, identity, top;
     float scale;
     int32_t raw;
     const float *correction; /* [experts + identity] */
+    int32_t sigmoid;
+    size_t groups, keep;
 } bitnet_hip_router;
 typedef struct bitnet_hip_experts_plan { /* where m tokens' choices lie in a workspace */
     int32_t *counts, *offsets, *n_tiles, *tiles; /* tiles: (expert, first slot, slots, 0) */
@@ -813,11 +861,11 @@ int bitnet_hip_experts_matmul_dev(const bitnet_hip_experts_plan *plan, int gathe
  * experts are left out of y and ids (-1 behind the last one that is none); the sum of their weights goes to *identity (needed where the router has any). */
 int bitnet_hip_experts_up_dev(const float *logits_dev, const bitnet_hip_router *router, const float *x_dev, const uint16_t *w_dev, size_t rows, size_t cols,
                               size_t ld, int act, float *y_dev, size_t ldy, int32_t *ids_dev, float *identity_dev, void *stream);
-/* y = W0 . x0 + bias + sum over k of W1[ids[k]] . x1[k] + *identity * input; W1 bf16 [experts][rows][ld1]; x0 NULL: no first product; identity NULL:
- * no last term */
+/* y = W0 . (*x0_scale x0) + bias + sum over k of W1[ids[k]] . x1[k] + *identity * input; W1 bf16 [experts][rows][ld1]; x0 NULL: no first product;
+ * x0_scale NULL: 1; identity NULL: no last term */
 int bitnet_hip_experts_out_dev(const float *x0_dev, const uint16_t *w0_dev, size_t cols0, size_t ld0, const float *bias_dev, const float *x1_dev,
                                size_t ldx1, const uint16_t *w1_dev, size_t cols1, size_t ld1, const int32_t *ids_dev, size_t top, size_t rows,
-                               const float *identity_dev, const float *input_dev, float *y_dev, void *stream);
+                               const float *identity_dev, const float *input_dev, const float *x0_scale_dev, float *y_dev, void *stream);
 
 #ifdef __cplusplus
 }

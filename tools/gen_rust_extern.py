@@ -11,7 +11,7 @@ BASE = {"size_t": "usize", "int": "c_int", "float": "c_float", "double": "f64", 
         "uint16_t": "u16", "uint32_t": "u32", "int32_t": "i32", "uint64_t": "u64", "int64_t": "i64", "unsigned long long": "u64", "unsigned": "u32",
         "bitnet_hip_weights_t": "Weights", "bitnet_hip_device_info": "DeviceInfo", "bitnet_hip_gemv_item": "GemvItem", "bitnet_hip_vector_input": "VectorInput",
         "bitnet_hip_latent_rows": "LatentRows", "bitnet_hip_latent_attention": "LatentAttention", "bitnet_hip_sum_rows": "SumRows",
-        "bitnet_hip_gqa": "Gqa", "bitnet_hip_delta": "Delta", "bitnet_hip_experts_plan": "ExpertsPlan", "bitnet_hip_router": "Router", "_Float16": "u16"}
+        "bitnet_hip_gqa": "Gqa", "bitnet_hip_delta": "Delta", "bitnet_hip_experts_plan": "ExpertsPlan", "bitnet_hip_router": "Router", "bitnet_hip_epilogue": "Epilogue", "_Float16": "u16"}
 
 
 def rust_type(c: str) -> str:
