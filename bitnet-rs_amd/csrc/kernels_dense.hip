@@ -17,9 +17,19 @@ __global__ void k_embed_bf16(const uint16_t *__restrict__ table, size_t ld, cons
     auto token = [&](int i) { return min(max(tokens[i], 0), vocab - 1); };
     const int tok = token(at);
     if (pairs.table) {
-        const uint64_t pair = at == 0 ? pairs.buckets : ((uint64_t)token(max(at - 1, 0)) * pairs.mul_prev + (uint64_t)tok * pairs.mul_cur) % pairs.buckets;
+        const uint64_t sum = (uint64_t)token(max(at - 1, 0)) * pairs.mul_prev + (uint64_t)tok * pairs.mul_cur;
+        const uint64_t pair = at == 0 ? pairs.buckets : (sum | pairs.buckets) >> 32 ? sum % pairs.buckets : (uint32_t)sum % (uint32_t)pairs.buckets;
         const uint16_t *a = table + (size_t)tok * ld, *b = pairs.table + (size_t)pair * pairs.ld;
-        for (int i = threadIdx.x; i < width; i += blockDim.x) out[(size_t)blockIdx.x * width + i] = scale * bf2f(a[i]) + bf2f(b[i]);
+        float *o = out + (size_t)blockIdx.x * width;
+        if (width % 4 == 0) {
+            for (int i = 4 * (threadIdx.x + 256 * blockIdx.y); i < width; i += 1024 * gridDim.y) {
+                const u32x2 x = *reinterpret_cast<const u32x2 *>(a + i), y = *reinterpret_cast<const u32x2 *>(b + i);
+                *reinterpret_cast<f32x4 *>(o + i) = scale * f32x4{bf2f(x.x & 0xffffu), bf2f(x.x >> 16), bf2f(x.y & 0xffffu), bf2f(x.y >> 16)} +
+                                                    f32x4{bf2f(y.x & 0xffffu), bf2f(y.x >> 16), bf2f(y.y & 0xffffu), bf2f(y.y >> 16)};
+            }
+        } else {
+            for (int i = threadIdx.x + 256 * blockIdx.y; i < width; i += 256 * gridDim.y) o[i] = scale * bf2f(a[i]) + bf2f(b[i]);
+        }
         return;
     }
     if (norm_w) {
@@ -48,7 +58,8 @@ __global__ void k_embed_bf16(const uint16_t *__restrict__ table, size_t ld, cons
 
 hipError_t launch_embed_bf16(const uint16_t *table, size_t ld, const int *tokens, const int *offset, int n, int width, int vocab, float scale,
                              const float *norm_w, float eps, const TokenPairs &pairs, float *out, hipStream_t s) {
-    hipLaunchKernelGGL(k_embed_bf16, dim3(n), dim3(256), 0, s, table, ld, tokens, offset, width, vocab, scale, norm_w, eps, pairs, out);
+    const int parts = pairs.table && n == 1 ? (width + 1023) / 1024 : 1;  // (one token: its row at once)
+    hipLaunchKernelGGL(k_embed_bf16, dim3(n, parts), dim3(256), 0, s, table, ld, tokens, offset, width, vocab, scale, norm_w, eps, pairs, out);
     return hipGetLastError();
 }
 

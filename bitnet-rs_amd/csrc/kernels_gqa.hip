@@ -87,10 +87,12 @@ bool gqa_supported(int dimp, int vdimp) { return dimp <= 256 && vdimp <= 256; }
 // tokens, every fourth workgroup).
 constexpr int kRowTokens = 16, kRowCols = 32;
 
-// four tokens of a query or key head of up to 256 columns: a lane holds neighbouring elements, so that a pair turns within it
-template <class TR, class TC, bool CONV>
+// Four tokens of a query or key head of up to 128 NJ columns: a lane holds neighbouring elements, so that a pair turns within it.  TAPS: those of the convolution
+// (0: none, -1: any number).
+template <class TR, class TC, int NJ, int TAPS>
 __device__ __forceinline__ void head_rows(const Gqa &p, const TR *rows, size_t ld, int pos0, int t0, int n, int y, bool key, TC *cache, TR *queries, size_t ldq) {
-    constexpr int U = kRowTokens / 4, NJ = 2;
+    constexpr int U = kRowTokens / 4;
+    constexpr bool CONV = TAPS != 0;
     const int lane = threadIdx.x & 63, dim = (int)p.dim, dimp = (int)p.dimp, turned = (int)p.rot_dims, half = turned >> 1;
     const float *w = key ? p.k_weight : p.q_weight;
     float v[U][NJ][2], cs[U][NJ], sn[U][NJ], factor[U];
@@ -113,9 +115,36 @@ __device__ __forceinline__ void head_rows(const Gqa &p, const TR *rows, size_t l
             }
         }
     }
-    if (CONV) {
+    if (TAPS > 0) {  // the tokens and those ahead of them once, in registers
+        constexpr int T = TAPS > 0 ? TAPS : 1;
+        const int channels = gqa_channels(p);
+#pragma unroll
+        for (int j = 0; j < NJ; ++j) {
+            const int c = y * dimp + min(2 * lane + 128 * j, dimp - 2);
+            float f[T][2], raw[U + T - 1][2];
+#pragma unroll
+            for (int k = 0; k < T; ++k) f[k][0] = p.conv[(size_t)k * channels + c], f[k][1] = p.conv[(size_t)k * channels + c + 1];
+            if (t0 >= T - 1) {
+#pragma unroll
+                for (int k = 0; k < U + T - 1; ++k) {
+                    const TR *row = rows + (size_t)min(t0 - (T - 1) + k, n - 1) * ld;
+                    raw[k][0] = ld_act(row, c), raw[k][1] = ld_act(row, c + 1);
+                }
+            } else {
+#pragma unroll
+                for (int k = 0; k < U + T - 1; ++k) {
+                    const int t = min(t0 - (T - 1) + k, n - 1);
+                    raw[k][0] = raw_value(p, rows, ld, pos0, t, c, channels), raw[k][1] = raw_value(p, rows, ld, pos0, t, c + 1, channels);
+                }
+            }
+#pragma unroll
+            for (int u = 0; u < U; ++u)
+#pragma unroll
+                for (int k = 0; k < T; ++k) v[u][j][0] += f[k][0] * raw[u + k][0], v[u][j][1] += f[k][1] * raw[u + k][1];
+        }
+    } else if (CONV) {
         const int taps = (int)p.taps, channels = gqa_channels(p);
-        auto add = [&](int k, auto value) {  // tap k of the four tokens
+        for (int k = 0; k < taps; ++k)
 #pragma unroll
             for (int j = 0; j < NJ; ++j) {
                 const int c = y * dimp + min(2 * lane + 128 * j, dimp - 2);
@@ -123,16 +152,9 @@ __device__ __forceinline__ void head_rows(const Gqa &p, const TR *rows, size_t l
 #pragma unroll
                 for (int u = 0; u < U; ++u) {
                     const int t = min(t0 + u, n - 1) - (taps - 1) + k;
-                    v[u][j][0] += f0 * value(t, c), v[u][j][1] += f1 * value(t, c + 1);
+                    v[u][j][0] += f0 * raw_value(p, rows, ld, pos0, t, c, channels), v[u][j][1] += f1 * raw_value(p, rows, ld, pos0, t, c + 1, channels);
                 }
             }
-        };
-        for (int k = 0; k < taps; ++k) {
-            if (t0 - (taps - 1) + k >= 0)
-                add(k, [&](int t, int c) { return ld_act(rows + (size_t)t * ld, c); });
-            else
-                add(k, [&](int t, int c) { return raw_value(p, rows, ld, pos0, t, c, channels); });
-        }
     }
     float wv[NJ][2];
 #pragma unroll
@@ -165,11 +187,12 @@ __device__ __forceinline__ void head_rows(const Gqa &p, const TR *rows, size_t l
     }
 }
 
-// CONV: every column passes a convolution over time first, and the queries go to a place of their own
-template <class TR, class TC, bool CONV>
+// TAPS (as head_rows): every column passes a convolution over time first, and the queries go to a place of their own
+template <class TR, class TC, int NJ, int TAPS>
 __global__ __launch_bounds__(256) void k_gqa_rows(Gqa p, const TR *rows, size_t ld, const int *pos_ptr, int n, TR *queries, size_t ldq) {
     constexpr int STRIDE = sizeof(TR) == 4 ? kRowCols + 1 : kRowCols + 2;
-    __shared__ __attribute__((aligned(16))) TR tile[(64 + (CONV ? kMaxTaps - 1 : 0)) * STRIDE];
+    constexpr bool CONV = TAPS != 0;
+    __shared__ __attribute__((aligned(16))) TR tile[(64 + (TAPS < 0 ? kMaxTaps - 1 : TAPS > 0 ? TAPS - 1 : 0)) * STRIDE];
     const int tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, pos0 = *pos_ptr;
     const int nq = (int)(p.heads * p.maps), nk = (int)(p.kv_heads * p.maps), dim = (int)p.dim, dimp = (int)p.dimp, vdimp = (int)p.vdimp;
     int y = blockIdx.y;
@@ -179,8 +202,8 @@ __global__ __launch_bounds__(256) void k_gqa_rows(Gqa p, const TR *rows, size_t 
         const int turned = (int)p.rot_dims, half = turned >> 1, t0 = blockIdx.x * kRowTokens + wave * (kRowTokens / 4);
         TC *cache = key ? (TC *)p.kcache + (size_t)(y - nq) * p.capacity * dimp : nullptr;
         if (t0 >= n) return;
-        if (dimp <= 256) {
-            head_rows<TR, TC, CONV>(p, rows, ld, pos0, t0, n, y, key, cache, queries, ldq);
+        if (dimp <= 128 * NJ) {
+            head_rows<TR, TC, NJ, TAPS>(p, rows, ld, pos0, t0, n, y, key, cache, queries, ldq);
             return;
         }
         const int channels = gqa_channels(p), taps = (int)p.taps;
@@ -218,7 +241,7 @@ __global__ __launch_bounds__(256) void k_gqa_rows(Gqa p, const TR *rows, size_t 
     const int column = (p.values_are_keys ? nq : nq + nk) * dimp + head * vdimp + c0;
     const TR *src = rows + column;
     constexpr int V = 16 / sizeof(TR), PER = kRowCols / V;
-    const int taps = CONV ? (int)p.taps : 1, channels = gqa_channels(p);
+    const int taps = TAPS > 0 ? TAPS : CONV ? (int)p.taps : 1, channels = gqa_channels(p);
     if (CONV) {  // the tokens ahead of the first one in the tile's last rows
         for (int i = tid; i < (taps - 1) * kRowCols; i += 256) {
             const int k = i / kRowCols, c = i % kRowCols;
@@ -243,6 +266,7 @@ __global__ __launch_bounds__(256) void k_gqa_rows(Gqa p, const TR *rows, size_t 
             float x;
             if (CONV) {
                 x = 0.f;
+#pragma unroll TAPS > 0 ? TAPS : 1
                 for (int k = 0; k < taps; ++k) {
                     const int t = lane - (taps - 1) + k;
                     x += p.conv[(size_t)k * channels + column + v] * ld_act(tile, (t >= 0 ? t : 64 + taps - 1 + t) * STRIDE + v);
@@ -258,7 +282,12 @@ template <class TR, class TC>
 static hipError_t rows_go(const Gqa &g, const void *rows, size_t ld, const int *pos, int n, void *q, size_t ldq, hipStream_t s) {
     const int keys = g.queries_only ? 0 : (int)(g.kv_heads * g.maps + g.kv_heads * (g.vdimp / kRowCols));
     const dim3 grid((n + kRowTokens - 1) / kRowTokens, (int)(g.heads * g.maps) + keys);
-    auto fn = g.taps > 0 ? k_gqa_rows<TR, TC, true> : k_gqa_rows<TR, TC, false>;
+    auto pick = [&](auto narrow, auto wide) { return g.dimp <= 128 ? narrow : wide; };
+    auto fn = g.taps == 0   ? pick(k_gqa_rows<TR, TC, 1, 0>, k_gqa_rows<TR, TC, 2, 0>)
+              : g.taps == 2 ? pick(k_gqa_rows<TR, TC, 1, 2>, k_gqa_rows<TR, TC, 2, 2>)
+              : g.taps == 3 ? pick(k_gqa_rows<TR, TC, 1, 3>, k_gqa_rows<TR, TC, 2, 3>)
+              : g.taps == 4 ? pick(k_gqa_rows<TR, TC, 1, 4>, k_gqa_rows<TR, TC, 2, 4>)
+                            : pick(k_gqa_rows<TR, TC, 1, -1>, k_gqa_rows<TR, TC, 2, -1>);
     hipLaunchKernelGGL(fn, grid, dim3(256), 0, s, g, (const TR *)rows, ld, pos, n, (TR *)q, ldq);
     return hipGetLastError();
 }

@@ -50,6 +50,15 @@ StackModel::StackModel(const StackSpec &spec, bool f32, int max_pos) : spec_(spe
         }
         if (own && plan_block(i, 0, true, S.parallel) != 0) return;
         if (!S.parallel && (S.experts.count > 0 || (spec_.residual_gate && S.ff > 0)) && plan_block(i, 1, false, true) != 0) return;
+        if (S.mixer == LayerSpec::Latent && (S.latent.rot_dim != S.latent.rot.dims || S.latent.rot_dim % 2 || S.latent.rot_dim > 256)) {
+            err_ = "stack: the rotated part must be even, at most 256 and rotated whole";
+            return;
+        }
+        if ((S.mixer == LayerSpec::Latent || S.mixer == LayerSpec::Attention) && !fits_source(i)) {
+            const int from = S.mixer == LayerSpec::Latent ? S.latent.kv_from : S.attention.kv_from;
+            err_ = "stack: layer " + std::to_string(i) + " reads the cache of layer " + std::to_string(from) + ", which has none that fits";
+            return;
+        }
     }
     if (init_sequence(spec.vocab, spec.width, max_pos) != 0) return;
     cap_ = up_to((size_t)max_pos + 1, 128);
@@ -60,14 +69,6 @@ StackModel::StackModel(const StackSpec &spec, bool f32, int max_pos) : spec_(spe
         const LayerSpec &S = spec_.layers[i];
         if (S.mixer == LayerSpec::Latent) {
             const LatentSpec &m = S.latent;
-            if (m.rot_dim != m.rot.dims || m.rot_dim % 2 || m.rot_dim > 256) {
-                err_ = "stack: the rotated part must be even, at most 256 and rotated whole";
-                return;
-            }
-            if (!fits_source(i)) {
-                err_ = "stack: layer " + std::to_string(i) + " reads the cache of layer " + std::to_string(m.kv_from) + ", which has none that fits";
-                return;
-            }
             L.dimp = (int)up_to(m.dim, 32), L.rotp = (int)up_to(std::max(m.rot_dim, 1), 32), L.vdimp = (int)up_to(m.vdim, 32), L.ldc = (int)up_to(m.kv_rank, 64);
             if (L.ldc > 1024) {
                 err_ = "stack: kv_rank above 1024";
@@ -88,10 +89,6 @@ StackModel::StackModel(const StackSpec &spec, bool f32, int max_pos) : spec_(spe
             lin = std::max(lin, (size_t)m.heads * 2 * (L.dimp + L.vdimp));
             lino = std::max(lino, (size_t)m.heads * L.vdimp);
         } else if (S.mixer == LayerSpec::Attention) {
-            if (!fits_source(i)) {
-                err_ = "stack: layer " + std::to_string(i) + " reads the cache of layer " + std::to_string(S.attention.kv_from) + ", which has none that fits";
-                return;
-            }
             scratch = std::max(scratch, bitnet_hip_gqa_scratch_bytes(S.attention.heads, S.attention.maps, L.vdimp, 1) / 4);
         }
         for (const Block &B : L.block)

@@ -248,8 +248,158 @@ def random_lurepel(config: dict, seed: int) -> dict:
     return t
 
 
+YARN = {"factor": 5.0, "original": 60, "fast": 9.0, "slow": 1.5}
+
+
+def window_layer(heads=6, kv_heads=3, dim=20, vdim=28, scale=0.24, window=37, taps=3, kv_from=None, mlp=None) -> dict:
+    m = {"heads": heads, "kv_heads": kv_heads, "dim": dim, "vdim": vdim, "scale": scale, "conv": taps}
+    if window:
+        m["mask"] = {"size": window}
+    if kv_from is not None:
+        m["kv_from"] = kv_from
+    return {"type": "attention", "mixer": m, "mlp": mlp}
+
+
+def direct_latent_layer(heads=3, dim=24, rot_dim=12, vdim=40, kv_rank=72, scale=0.19, base=700.0, scaling=None, mlp=None) -> dict:
+    rot = {"base": base, "dims": rot_dim}
+    if scaling:
+        rot["scaling"] = scaling
+    return {"type": "latent_attention", "mixer": {"heads": heads, "dim": dim, "rot_dim": rot_dim, "vdim": vdim, "kv_rank": kv_rank, "scale": scale, "rot": rot}, "mlp": mlp}
+
+
+def xielu_mlp(ff=44) -> dict:
+    return {"kind": "dense", "ff": ff}
+
+
+def grouped_mlp(experts=8, groups=(4, 2), top=3, ff=24, shared=40) -> dict:
+    f = {"kind": "moe", "expert": {"ff": ff}, "router": {"experts": experts, "top": top}}
+    if groups:
+        f["router"]["groups"] = dict(zip(("count", "keep"), groups))
+    if shared:
+        f["shared"] = {"ff": shared}
+    return f
+
+
+def sipelorn(layers, width=120, vocab=150, eps=1e-5, embed=2.5, pairs=(61, 13, 5), side=20) -> dict:
+    return {"architecture": "Sipelorn", "vocab": vocab, "width": width, "norm": {"eps": eps},
+            "embedding": {"scale": embed, "bigram": dict(zip(("buckets", "mul_prev", "mul_cur"), pairs))}, "token_side": {"dim": side}, "layers": layers}
+
+
+def group_margins(choice, top, groups):
+    """how far the choice among these scores is from another one"""
+    margins = []
+    if groups:
+        part = choice.reshape(groups["count"], -1)
+        worth = np.sort(part, axis=1)[:, -2:].sum(axis=1)
+        order = np.argsort(-worth, kind="stable")
+        if groups["keep"] < groups["count"]:
+            margins.append(worth[order[groups["keep"] - 1]] - worth[order[groups["keep"]]])
+        choice = part[order[:groups["keep"]]].reshape(-1)
+    ranked = np.sort(choice)[::-1]
+    if top < len(ranked):
+        margins.append(ranked[top - 1] - ranked[top])
+    return min(margins, default=1.0)
+
+
+def random_sipelorn(config: dict, seed: int) -> dict:
+    """bf16-representable weights, everything away from its neutral value.  No choice of experts may hang on the last bit of the router's input: its first
+    columns are large, come from the token's embedding alone (nothing is added to them, and they make up most of the stream's variance), and embedding rows are
+    drawn until what is chosen and what is not lie apart in every layer, whatever the other columns' variance."""
+    g = np.random.default_rng(seed)
+    W, V, side = config["width"], config["vocab"], config["token_side"]["dim"]
+    routers = {i: layer["mlp"]["router"] for i, layer in enumerate(config["layers"]) if layer["mlp"] and layer["mlp"]["kind"] == "moe"}
+    codes = max([r["experts"] for r in routers.values()], default=0)
+    t = {}
+
+    def mat(name, rows, cols, gain=1.0):
+        t[name] = rounded(g.standard_normal((rows, cols)) * gain / np.sqrt(cols))
+
+    def back(name, cols):  # a matrix back to the residual stream
+        mat(name, W, cols)
+        t[name][:codes] = 0.0
+
+    def around(name, n, centre, spread):
+        t[name] = rounded(centre + spread * g.standard_normal(n))
+
+    def norm(name):
+        around(name, W, 1.0, 0.2)
+        around(name + ".b", W, 0.0, 0.2)
+        t[name][:codes], t[name + ".b"][:codes] = 1.0, 0.0
+
+    for i, r in routers.items():
+        n = r["experts"]
+        t[f"l{i}.mlp.router"] = rounded(np.concatenate([1.5 * np.eye(n)[g.permutation(n)], np.zeros((n, codes - n)), 0.0003 * g.standard_normal((n, W - codes))], axis=1))
+        t[f"l{i}.mlp.correction"] = rounded(g.uniform(-0.2, 0.2, n))
+
+    def apart(code):
+        for i, r in routers.items():
+            w, c = t[f"l{i}.mlp.router"][:, :codes].astype(np.float64), t[f"l{i}.mlp.correction"].astype(np.float64)
+            for rest in (0.3, 0.7, 1.2, 2.0, 3.5, 6.0):  # variance of the columns that are added to
+                for shift in (-0.15, 0.0, 0.15):
+                    mean = code.sum() / W + shift
+                    h = (code - mean) / np.sqrt(((code - mean) ** 2).sum() / W + rest * (W - codes) / W)
+                    if group_margins(1.0 / (1.0 + np.exp(-(w @ h))) + c, r["top"], r.get("groups")) < 0.012:
+                        return False
+        return True
+
+    scale = config["embedding"]["scale"]
+    t["embed"] = np.zeros((V, W), np.float32)
+    for k in range(V):
+        while True:
+            row = rounded(np.concatenate([g.uniform(-4.0, 4.0, codes), 0.8 * g.standard_normal(W - codes)]) / scale)
+            if apart(row[:codes].astype(np.float64) * scale):
+                break
+        t["embed"][k] = row
+    t["bigram"] = rounded(0.7 * g.standard_normal((config["embedding"]["bigram"]["buckets"] + 1, W)))
+    t["bigram"][:, :codes] = 0.0
+    t["side.embed"] = rounded(g.standard_normal((V, side * len(config["layers"]))))
+    for i, layer in enumerate(config["layers"]):
+        p, q, m, f = f"l{i}.", f"l{i}.mix.", layer["mixer"], layer["mlp"]
+        H, D, VD = m["heads"], m["dim"], m["vdim"]
+        for k in "12" if f else "1":
+            norm(p + "norm" + k)
+            mat(p + "rg" + k, W, W)
+            around(p + f"rg{k}.b", W, 0.0, 0.5)
+        if layer["type"] == "attention":
+            G = m["kv_heads"]
+            for name, rows in (("q", H * D),) + (() if "kv_from" in m else (("k", G * D), ("v", G * VD))):
+                mat(q + name, rows, W)
+                around(q + name + ".b", rows, 0.0, 0.4)
+                t[q + name + ".conv"] = rounded(0.2 + 0.6 * g.standard_normal((rows, m["conv"])))
+            t[q + "r1"], t[q + "r2"] = rounded(g.uniform(0.1, 0.9, H)), rounded(g.uniform(0.02, 1.5, H))
+            mat(q + "g", H * VD, W, 1.5)
+        else:
+            R, C = m["rot_dim"], m["kv_rank"]
+            mat(q + "q", H * (D + R), W, 1.5)
+            mat(q + "dkv", C + R, W)
+            around(q + "dkv.norm", C, 1.0, 0.3)
+            mat(q + "uk", H * D, C, 1.5)
+            mat(q + "uv", H * VD, C)
+        back(q + "o", H * VD)
+        if f and f["kind"] == "dense":
+            mat(p + "mlp.up", f["ff"], W)
+            back(p + "mlp.down", f["ff"])
+            around(p + "mlp.act", 2, 0.3, 0.5)
+        elif f:
+            parts = {f"e{e}.": f["expert"]["ff"] for e in range(f["router"]["experts"])}
+            if f.get("shared"):
+                parts["shared."] = f["shared"]["ff"]
+                mat(p + "mlp.shared.sg", 1, W, 1.5)
+            for e, ff in parts.items():
+                mat(p + f"mlp.{e}gate", ff, W)
+                mat(p + f"mlp.{e}up", ff, W)
+                back(p + f"mlp.{e}down", ff)
+        mat(p + "side.gate", side, W)
+        back(p + "side.proj", side)
+        around(p + "side.norm", W, 0.6, 0.2)
+        t[p + "side.norm"][:codes] = 0.0
+    norm("final.norm")
+    mat("head", V, W)
+    return t
+
+
 def random_tensors(config: dict, seed: int) -> dict:
-    return {"Lasapel": random_lasapel, "Mimolix": random_mimolix, "Lurepel": random_lurepel}[config["architecture"]](config, seed)
+    return {"Lasapel": random_lasapel, "Mimolix": random_mimolix, "Lurepel": random_lurepel, "Sipelorn": random_sipelorn}[config["architecture"]](config, seed)
 
 
 def random_lasapel(config: dict, seed: int) -> dict:

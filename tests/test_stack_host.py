@@ -23,7 +23,7 @@ BASE = u.lasapel([u.latent_layer(ff=24), u.lightning_layer()], width=40, vocab=2
 
 def test_registry_names(built):
     names = built.registered_models()
-    assert {"Lasapel", "Mimolix", "Lurepel"} <= set(names) and ".gguf" in names
+    assert {"Lasapel", "Mimolix", "Lurepel", "Sipelorn"} <= set(names) and ".gguf" in names
 
 
 PARALLEL = u.mimolix([u.delta_layer(mlp=u.expert_mlp()), u.attention_layer()], width=40, vocab=20, loop=(0, 1, 2))
@@ -73,6 +73,38 @@ def test_bad_chunked_configurations_say_why(built, tmp_path, change, message):
     c = copy.deepcopy(CHUNKED)
     change(c)
     path = u.save_model(str(tmp_path), c, u.random_tensors(CHUNKED, 1))
+    with pytest.raises(built.BitNetHipError, match=message):
+        built.open_model(path)
+
+
+WINDOWED = u.sipelorn([u.window_layer(mlp=u.xielu_mlp()), u.direct_latent_layer(scaling=u.YARN, mlp=u.grouped_mlp()), u.window_layer(kv_from=0)], width=40, vocab=20)
+
+
+@pytest.mark.parametrize("change,message", [
+    (lambda c: c["norm"].pop("eps"), "norm.eps: missing"),
+    (lambda c: c["embedding"].pop("scale"), "embedding.scale: missing"),
+    (lambda c: c["embedding"]["bigram"].update(buckets=0), "embedding.bigram.buckets: not an integer"),
+    (lambda c: c["embedding"]["bigram"].pop("mul_prev"), "embedding.bigram.mul_prev: missing"),
+    (lambda c: c["token_side"].update(dim=0), "token_side.dim: not an integer"),
+    (lambda c: c["layers"][0].update(type="delta"), r"layers\[0\].type: unknown mixer"),
+    (lambda c: c["layers"][0]["mixer"].pop("conv"), r"layers\[0\].mixer.conv: missing"),
+    (lambda c: c["layers"][0]["mixer"].update(conv=65), "layer 0: attention: at most 64 taps"),
+    (lambda c: c["layers"][0]["mixer"].update(kv_heads=4), "layer 0: attention: query heads in whole groups"),
+    (lambda c: c["layers"][0]["mixer"]["mask"].update(size=0), r"layers\[0\].mixer.mask.size: not an integer"),
+    (lambda c: c["layers"][2]["mixer"].update(kv_from=1), "layer 2 reads the cache of layer 1"),
+    (lambda c: c["layers"][2]["mixer"].update(kv_from=2), "layer 2 reads the cache of layer 2"),
+    (lambda c: c["layers"][2]["mixer"].update(dim=24), "layer 2 reads the cache of layer 0"),
+    (lambda c: c["layers"][1]["mixer"]["rot"].update(dims=10), "rotated part must be even"),
+    (lambda c: c["layers"][1]["mixer"]["rot"]["scaling"].pop("fast"), r"layers\[1\].mixer.rot.scaling.fast: missing"),
+    (lambda c: c["layers"][0]["mlp"].update(kind="sparse"), r"layers\[0\].mlp.kind: unknown"),
+    (lambda c: c["layers"][1]["mlp"]["router"].update(top=5), "layer 1: experts: equal groups"),
+    (lambda c: c["layers"][1]["mlp"]["router"]["groups"].update(count=3), "layer 1: experts: equal groups"),
+    (lambda c: c["layers"][1]["mlp"]["router"]["groups"].update(keep=5), "layer 1: experts: equal groups"),
+])
+def test_bad_windowed_configurations_say_why(built, tmp_path, change, message):
+    c = copy.deepcopy(WINDOWED)
+    change(c)
+    path = u.save_model(str(tmp_path), c, u.random_tensors(WINDOWED, 1))
     with pytest.raises(built.BitNetHipError, match=message):
         built.open_model(path)
 
@@ -150,6 +182,20 @@ def test_entry_points_check_shapes_before_any_launch(built):
         (lambda: hip.experts_up_dev(8, built.Router(8, 0, 2, 1.0), 8, 8, 16, 12, 64, 0, 8, 16, 8), "experts_up"),
         (lambda: hip.experts_out_dev(8, 8, 64, 64, None, 8, 8, 8, 16, 64, 8, 2, 16, 8), "experts_out"),
         (lambda: hip.sum_norm_rows_dev(built.SumRows(x=8, m=1, width=8, h=8, ldh=7)), "sum_norm_rows"),
+        (lambda: hip.sum_norm_rows_dev(built.SumRows(x=8, m=1, width=8, h=8, ldh=8, gate=8, ld_gate=7)), "sum_norm_rows: bad gate"),
+        (lambda: hip.gqa_step_dev(built.Gqa(4, 2, 2, 16, 32, 16, 32, 128, 1e-5, 0.1, 0.9, 8, 8, 8, 8, 8, far_weight=8, far_rate=8), 8, 8, 8), "gqa: bad window"),
+        (lambda: hip.gqa_step_dev(built.Gqa(4, 2, 1, 16, 32, 16, 32, 128, 1e-5, 0.1, 0.9, 8, 8, 8, 8, 8, far_weight=8), 8, 8, 8), "gqa: bad window"),
+        (lambda: hip.gqa_step_dev(built.Gqa(4, 2, 1, 16, 32, 16, 32, 128, 1e-5, 0.1, 0.9, 8, 8, 8, 8, 8, gate=8, ldgate=127, gate_columns=1), 8, 8, 8), "gqa: bad chunk"),
+        (lambda: hip.gqa_rows_dev(built.Gqa(4, 2, 1, 16, 32, 16, 32, 128, 1e-5, 0.1, 0.9, 8, 8, 8, 8, 8, taps=3, conv=8, ring=8), 16, 256, True, True, 8, 2), "place of the queries"),
+        (lambda: hip.gqa_rows_dev(built.Gqa(4, 2, 1, 16, 32, 16, 32, 128, 1e-5, 0.1, 0.9, 8, 8, 8, 8, 8, taps=3), 16, 256, True, True, 8, 2, 8, 128), "gqa: bad window"),
+        (lambda: hip.conv_keep_dev(8, 64, True, 65, 3, 8, 8, 2), "conv_keep"),
+        (lambda: hip.experts_up_dev(8, built.Router(8, 0, 4, 1.0, groups=4, keep=1), 8, 8, 16, 8, 64, 0, 8, 16, 8), "bad groups"),
+        (lambda: hip.experts_up_dev(8, built.Router(8, 0, 2, 1.0, groups=3, keep=1), 8, 8, 16, 8, 64, 0, 8, 16, 8), "bad groups"),
+        (lambda: hip.dense_gemv_dev(8, 8, 16, 64, 64, 8, act0=built.ACT_GATED, more=built.Epilogue(pairs=8)), "gated rows come in pairs"),
+        (lambda: hip.dense_gemv_dev(8, 8, 16, 64, 64, 8, more=built.Epilogue(conv=8, ring=8, pos=8, taps=3, channels=9, conv_from=8)), "bad convolution"),
+        (lambda: hip.dense_gemv_dev(8, 8, 16, 64, 64, 8, more=built.Epilogue(mul=8, mul_tokens=8, mul_at=8, mul_rows=4, ld_mul=15)), "bad table"),
+        (lambda: hip.dense_matmul_dev(8, 64, False, 8, 64, 4, 16, 64, 8, 16, True, more=built.Epilogue(mul=8, mul_tokens=8, mul_at=8, mul_rows=4, ld_mul=16)), "dense_matmul: what"),
+        (lambda: hip.embed_pairs_bf16_dev(8, 64, 8, 32, 5, 1, 1, 8, 8, 1, 64, 9), "embed_pairs"),
         (lambda: hip.latent_decode_dev(built.LatentAttention(1, 20, 52, 16, 64, 16, 1.0, 8, 8, 8, 64, 32, 64, 8, 8), 8, 8, 8, 0, 1, True, 8), "bad shape"),
     ]
     for call, message in bad:
@@ -242,6 +288,50 @@ def test_oracle_corrected_choice():
     ids, w = so.route_corrected(np.ones((1, 1)), z.T, np.array([0.35, 0.0, 0.0, -0.15]), 2)
     assert ids.tolist() == [[0, 2]] and np.allclose(w, [[0.1, 0.3]])
     assert np.allclose(so.gelu_tanh(np.array([-50.0, 0.0, 50.0])), [0.0, 0.0, 50.0]) and np.isclose(so.gelu_tanh(1.0), 0.841192, atol=1e-6)
+
+
+def test_oracle_window_and_penalty():
+    """scores of zero: the mean over the window; a penalty of r1 ln(1 + r2 d) leaves (1 + r2 d)^-r1 of a weight"""
+    v = np.arange(1.0, 6.0).reshape(5, 1, 1)
+    o = so.window_softmax(np.ones((5, 2, 3)), np.zeros((5, 1, 3)), v, 1.0, 3, np.zeros(2), np.ones(2))
+    assert np.allclose(o[:, :, 0].T, [1.0, 1.5, 2.0, 3.0, 4.0])
+    o = so.window_softmax(np.ones((3, 1, 3)), np.zeros((3, 1, 3)), v[:3], 1.0, 9, np.full(1, 2.0), np.full(1, 3.0))
+    w = np.array([7.0, 4.0, 1.0]) ** -2.0
+    assert np.isclose(o[2, 0, 0], (w @ [1.0, 2.0, 3.0]) / w.sum())
+
+
+def test_oracle_groups():
+    score = np.array([[0.9, 0.1, 0.1, 0.6, 0.6, 0.2, 0.8, 0.1, 0.05]])
+    z = np.log(score / (1 - score))
+    ids, w = so.route_in_groups(np.ones((1, 1)), z.T, np.zeros(9), 2, {"count": 3, "keep": 1})
+    assert ids.tolist() == [[3, 4]] and np.allclose(w, 0.6)  # the group of the two best together, not of the best one
+    ids, w = so.route_in_groups(np.ones((1, 1)), z.T, np.array([0.0] * 5 + [0.0, 0.0, 0.45, 0.0]), 2, {"count": 3, "keep": 1})
+    assert ids.tolist() == [[6, 7]] and np.allclose(w, [[0.8, 0.1]])
+    ids, _ = so.route_in_groups(np.ones((1, 1)), z.T, np.full(9, -2.0), 3, {"count": 3, "keep": 2})
+    assert ids.tolist() == [[0, 3, 4]]  # corrected scores below zero are still above what cannot be chosen
+
+
+def test_oracle_pairs_xielu_and_neighbours():
+    assert so.bigram_rows([4, 2, 7], {"buckets": 10, "mul_prev": 3, "mul_cur": 5}) == [10, (12 + 10) % 10, (6 + 35) % 10]
+    z = np.array([-30.0, -1e-4, 0.0, 1e-4, 3.0])
+    p, q = 0.4, -0.7
+    a, b = math.log(1 + math.exp(p)), 0.5 + math.log(1 + math.exp(q))
+    assert np.allclose(so.xielu(z, p, q), [b * 29.0 - 15.0, -0.5e-4 + b * 0.5e-8, 0.0, 0.5e-4 + a * 1e-8, 9 * a + 1.5], rtol=1e-5)
+    rot = {"dims": 6, "base": 30.0, "scaling": {"factor": 4.0, "original": 64, "fast": 16.0, "slow": 1.0}}
+    f, mult = so.rotary_frequencies(rot)
+    v = np.random.default_rng(1).standard_normal((1, 2, 6))
+    turned = so.rotate_pairs(v, [5], rot)
+    for i in range(3):
+        for h in range(2):
+            assert np.isclose(complex(*turned[0, h, 2 * i:2 * i + 2]), complex(*v[0, h, 2 * i:2 * i + 2]) * np.exp(5j * f[i]) * mult)
+    halves = so.rotate(np.concatenate([v[..., 0::2], v[..., 1::2]], axis=-1), [5], rot)
+    assert np.allclose(halves, np.concatenate([turned[..., 0::2], turned[..., 1::2]], axis=-1))
+
+
+def test_oracle_token_side_input():
+    x, t = np.array([[1.0, 2.0]]), {"gate": np.array([[1.0, -1.0]]), "proj": np.array([[3.0], [4.0]]), "norm": np.array([1.0, 2.0])}
+    y = so.token_side_input(x, np.array([[-2.0]]), t, "", 0.0)
+    assert np.allclose(y, np.array([[3.0, 8.0]]) / math.sqrt(12.5))  # (gelu(-1) < 0, times -2: positive)
 
 
 def test_oracle_convolution_and_routing():

@@ -44,9 +44,26 @@ MODELS = {
                               width=200, vocab=77),
     "lurepel_huge": u.lurepel([u.chunk_layer(heads=4, kv_heads=2, dim=300, dims=210, chunk=33, scale=0.05, scaling=u.BANDS, mlp=u.corrected_mlp(experts=4, identity=0, top=4, ff=100))],
                               width=64, vocab=50),
+    # windows of several sizes and none, convolutions of one to five taps, another layer's keys under another window, every kind of feed-forward and none
+    "sipelorn": u.sipelorn([u.window_layer(mlp=u.xielu_mlp()), u.direct_latent_layer(scaling=u.YARN, mlp=u.grouped_mlp()),
+                            u.window_layer(kv_from=0, window=100, taps=2, scale=0.4, mlp=u.grouped_mlp(experts=6, groups=(2, 1), top=2, ff=72, shared=24)),
+                            u.window_layer(heads=5, kv_heads=1, dim=36, vdim=16, window=0, taps=4), u.direct_latent_layer(heads=2, rot_dim=2, kv_rank=24),
+                            u.window_layer(heads=10, kv_heads=1, dim=36, vdim=16, window=64, taps=5, kv_from=3, mlp=u.xielu_mlp(9))], vocab=170),
+    "sipelorn_narrow": u.sipelorn([u.window_layer(heads=1, kv_heads=1, dim=8, vdim=8, window=1, taps=1, mlp=u.grouped_mlp(experts=9, groups=(3, 3), top=9, ff=16, shared=0)),
+                                   u.direct_latent_layer(heads=1, dim=8, rot_dim=2, vdim=8, kv_rank=8, base=50.0, mlp=u.grouped_mlp(experts=4, groups=None, top=1, ff=130, shared=8))],
+                                  width=77, vocab=60, eps=1e-3, embed=1.0, pairs=(1, 0, 1), side=1),
+    "sipelorn_attention": u.sipelorn([u.window_layer(heads=2, kv_heads=2, dim=128, vdim=64, window=128, taps=2, scale=0.1, mlp=u.xielu_mlp(71)),
+                                      u.window_layer(heads=4, kv_heads=4, dim=64, vdim=128, window=65, mlp=u.grouped_mlp(experts=20, groups=(5, 4), top=4, ff=8, shared=16))],
+                                     width=90, vocab=64, embed=0.7, pairs=(97, 3, 1), side=70),
+    "sipelorn_wide": u.sipelorn([u.window_layer(heads=20, kv_heads=1, dim=150, vdim=200, window=50, taps=3, scale=0.08),
+                                 u.direct_latent_layer(heads=2, dim=100, rot_dim=60, vdim=140, kv_rank=200, scaling=dict(u.YARN, factor=1.5), mlp=u.xielu_mlp(100))],
+                                width=136, vocab=77, side=8),
+    "sipelorn_huge": u.sipelorn([u.window_layer(heads=4, kv_heads=2, dim=300, vdim=270, window=33, taps=4, scale=0.05, mlp=u.xielu_mlp(33)),
+                                 u.direct_latent_layer(heads=2, dim=230, rot_dim=40, vdim=270, kv_rank=600, scale=0.07), u.window_layer(heads=6, kv_heads=2, dim=300, vdim=270, window=0,
+                                                                                                                                        taps=20, scale=0.05, kv_from=0)], width=64, vocab=50),
     "many_heads": u.lasapel([u.latent_layer(heads=19, dim=16, rot_dim=8, vdim=16, q_rank=40, kv_rank=136, ff=16)], width=64, vocab=500),
 }
-SEQUENCES = ["mixed", "mimolix", "lurepel"]  # the models of the tests about sequences
+SEQUENCES = ["mixed", "mimolix", "lurepel", "sipelorn"]  # the models of the tests about sequences
 LIMIT = {"float32": 2e-5, "bfloat16": 6e-2}
 
 
@@ -147,12 +164,14 @@ def test_residual_stream_after_each_layer(cases, pkg, tmp_path, dtype, name):
     c = cases(name)
     t = tokens_of(c.config, 21)
     for k in range(1, len(c.config["layers"]) + 1):
-        config = dict(c.config, layers=c.config["layers"][:k])
+        config, tensors = dict(c.config, layers=c.config["layers"][:k]), c.tensors
+        if config.get("token_side"):
+            tensors = dict(tensors, **{"side.embed": tensors["side.embed"][:, :k * config["token_side"]["dim"]]})
         loop = config.pop("loop", None)
         if loop and loop["start"] < k:
             config["loop"] = dict(loop, stop=min(loop["stop"], k))
-        after = so.forward(config, c.tensors, t)[1]
-        m = pkg.open_model(u.save_model(str(tmp_path / str(k)), config, c.tensors), dtype, 64)
+        after = so.forward(config, tensors, t)[1]
+        m = pkg.open_model(u.save_model(str(tmp_path / str(k)), config, tensors), dtype, 64)
         m.feed(t)
         m.prefill(20, with_logits=False)
         assert u.rms_error(m.last_hidden(), after[-1, 19]) < LIMIT[dtype]
@@ -209,7 +228,7 @@ def test_graph_replays_match_eager_steps(cases, dtype, name):
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-@pytest.mark.parametrize("name", ["mixed", "lightning_only", "many_heads", "mimolix", "mimolix_delta", "lurepel", "lurepel_identities"])
+@pytest.mark.parametrize("name", ["mixed", "lightning_only", "many_heads", "mimolix", "mimolix_delta", "lurepel", "lurepel_identities", "sipelorn", "sipelorn_narrow"])
 def test_greedy_generation(cases, name, dtype):
     """generate(): each token is the argmax of the oracle's logits over what was generated so far (or as good as it)"""
     c = cases(name)
@@ -370,6 +389,130 @@ def test_keys_at_the_edge_of_a_chunk(pkg, hip, tmp_path, dtype, chunk):
             assert np.array_equal(got, plain)
         else:
             assert u.rms_error(truth - truth.mean(), want - want.mean()) > 0.2
+    m.close()
+
+
+def one_key_windowed(root, windows, sharpen):
+    """Attention layers in which a marked token's query scores one other marked token far above all others, in the first or only in the last of them (which
+    reads the first one's keys); the convolutions pass the current token on unchanged.  sharpen: what the marked score is multiplied by."""
+    W, V, D = 32, 40, 8
+    layers = [u.window_layer(heads=2, kv_heads=1, dim=D, vdim=24, scale=1.0, window=windows[0], taps=3)]
+    if len(windows) > 1:
+        layers.append(u.window_layer(heads=2, kv_heads=1, dim=D, vdim=24, scale=1.0, window=windows[1], taps=2, kv_from=0))
+    config = u.sipelorn(layers, width=W, vocab=V, eps=1e-6, embed=1.0, side=4)
+    t = u.random_tensors(config, 14)
+    t["embed"] = u.rounded(np.random.default_rng(11).standard_normal((V, W)) * 0.3)
+    t["bigram"] *= 0.1
+    t["embed"][:, :2] = 0.0
+    t["embed"][1, 0] = 8.0   # the token looked for
+    t["embed"][2, 1] = 8.0   # the token that looks
+    looks = len(windows) - 1
+    for i in range(len(windows)):
+        for name in ("l%d.norm1" % i,):
+            t[name][:], t[name + ".b"][:] = 1.0, 0.0
+        for k in ("q", "k") if i == 0 else ("q",):
+            t[f"l{i}.mix.{k}"] *= 0.02
+            t[f"l{i}.mix.{k}.b"] *= 0.02
+            t[f"l{i}.mix.{k}.conv"][:, :-1] *= 0.05
+            t[f"l{i}.mix.{k}.conv"][:, -1] = 1.0
+    t["l0.mix.o"] *= 1.0 if looks == 0 else 0.02
+    t["l0.side.norm"] *= 1.0 if looks == 0 else 0.02
+    for head in range(2):
+        t[f"l{looks}.mix.q"][head * D + 4, 1] = sharpen
+    t["l0.mix.k"][4, 0] = 1.0
+    t = {k: u.rounded(v) for k, v in t.items()}
+    return config, t, u.save_model(str(root), config, t)
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+@pytest.mark.parametrize("windows", [(1,), (2,), (31,), (64,), (100,), (128,), (130,), (257,), (399,), (400,), (5000,), (0,), (9, 150), (200, 64), (3, 0)])
+def test_keys_at_the_edge_of_a_window(pkg, hip, tmp_path, dtype, windows):
+    """a marked key just inside the window, beside it and near its query shows; just outside it and far outside it changes nothing of what the query sees -- in
+    whole prompts, at the end of portions and decoded, also where the keys are another layer's that has a window of its own"""
+    config, t, path = one_key_windowed(tmp_path, windows, 6.0)
+    n, p = 400, 399
+    first = max(0, p - windows[-1] + 1) if windows[-1] else 0
+    base = np.random.default_rng(windows[-1]).integers(3, 40, n).astype(np.int32)
+    base[-1] = 2
+    m = pkg.open_model(path, dtype, n + 8)
+
+    def last(tokens):
+        rows = []
+        for cut in (0, n - 1, n - 2, max(first - 1, 1), min(first + 1, n - 1)):
+            m.reset()
+            if cut:
+                m.forward(tokens[:cut], [])
+            rows.append(m.forward(tokens[cut:], [n - cut - 1])[0])
+        return np.stack(rows)
+
+    plain = last(base)
+    want = so.forward(config, t, base)[0][-1]
+    assert error(plain, np.broadcast_to(want, plain.shape)) < LIMIT[dtype]
+    for far in {0, first - 5, first - 4, first - 1, first, first + 1, p - 4}:
+        if not 0 <= far < p - 3:  # (the convolution's taps and the pair table bring the neighbours of a token along)
+            continue
+        marked = base.copy()
+        marked[far] = 1
+        got, truth = last(marked), so.forward(config, t, marked)[0][-1]
+        assert error(got, np.broadcast_to(truth, got.shape)) < LIMIT[dtype]
+        shift = u.rms_error(truth - truth.mean(), want - want.mean())
+        if far >= first:
+            assert shift > 0.1, far
+        elif far + 3 < first and len(windows) == 1:
+            assert (got == plain).all() and shift < 1e-12
+    m.close()
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_penalty_of_the_distance(pkg, hip, tmp_path, dtype):
+    """two marked keys of equal scores, one near and one far: the far one's share is what the penalty leaves of it"""
+    config, t, path = one_key_windowed(tmp_path, (0,), 3.0)
+    t["l0.mix.r1"], t["l0.mix.r2"] = u.rounded(np.array([1.5, 0.4])), u.rounded(np.array([0.05, 2.0]))
+    path = u.save_model(str(tmp_path / "p"), config, t)
+    n = 400
+    m = pkg.open_model(path, dtype, n + 8)
+    base = np.random.default_rng(5).integers(3, 40, n).astype(np.int32)
+    base[-1] = 2
+    for far in (390, 300, 128, 63, 0):
+        tokens = base.copy()
+        tokens[far] = tokens[395] = 1
+        want = so.forward(config, t, tokens)[0][-1:]
+        m.reset()
+        assert error(m.forward(tokens, [n - 1]), want) < LIMIT[dtype]
+        m.reset()
+        m.forward(tokens[:-1], [])
+        assert error(m.forward(tokens[-1:], [0]), want) < LIMIT[dtype]
+    m.close()
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_decoding_across_windows(pkg, hip, tmp_path, dtype):
+    """single tokens until the windows have passed over prompt and decoded tokens; portions that end at, ahead of and behind their size; the taps of every
+    convolution across each cut"""
+    config = u.sipelorn([u.window_layer(window=48, taps=4), u.window_layer(window=65, heads=3, taps=2, kv_from=0, mlp=u.xielu_mlp()), u.direct_latent_layer(scaling=u.YARN)],
+                        width=72, vocab=60)
+    t = u.random_tensors(config, 42)
+    m = pkg.open_model(u.save_model(str(tmp_path), config, t), dtype, 260)
+    tokens = tokens_of(config, 250, 12)
+    want = so.forward(config, t, tokens)[0]
+    for sizes in ([1], [2], [3, 1], [47, 1, 1], [48], [49, 2], [65, 63, 2], [130, 1, 119], [200, 50]):
+        m.reset()
+        assert error(in_portions(m, tokens, sizes), want) < LIMIT[dtype], sizes
+    m.close()
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_pairs_of_tokens(pkg, hip, tmp_path, dtype):
+    """a pair table that outweighs the embedding, factors whose products leave 32 bits: the previous token across every cut, the first token's own row"""
+    config = u.sipelorn([u.window_layer(window=1, taps=1)], width=40, vocab=90, embed=0.25, pairs=(83, 99999989, 87654321))
+    t = u.random_tensors(config, 43)
+    t["bigram"] = u.rounded(4.0 * t["bigram"])
+    m = pkg.open_model(u.save_model(str(tmp_path), config, t), dtype, 80)
+    tokens = tokens_of(config, 60, 13)
+    want = so.forward(config, t, tokens)[0]
+    for sizes in ([60], [1], [2], [3, 1, 5]):
+        m.reset()
+        assert error(in_portions(m, tokens, sizes), want) < LIMIT[dtype], sizes
     m.close()
 
 
