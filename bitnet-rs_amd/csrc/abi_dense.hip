@@ -160,7 +160,7 @@ int bitnet_hip_dense_matmul_dev(const void *a, size_t lda, int a_f32, const uint
     BH_REQUIRE(k % 64 == 0 && lda >= k && ldw >= k && lda % 8 == 0 && ldw % 8 == 0 && ldc >= (gated ? n / 2 : n), "dense_matmul: k %zu must be a multiple of 64 inside lda %zu, ldw %zu; ldc %zu >= n %zu",
                k, lda, ldw, ldc, n);
     BH_REQUIRE(act_ok(act0) && act_ok(act1) && a_batch % 8 == 0 && w_batch % 8 == 0, "dense_matmul: bad activation or batch stride");
-    BH_REQUIRE(!gated || (n % 2 == 0 && act_split == 0 && (a_f32 || !c_f32)), "dense_matmul: gated columns come in pairs, with one activation, in the activations' type");
+    BH_REQUIRE(!gated || (n % 2 == 0 && act0 != BITNET_HIP_ACT_XIELU && act_split == 0 && (a_f32 || !c_f32)), "dense_matmul: gated columns come in pairs, with one activation, in the activations' type");
     BH_CHECK_DIMS(m, lda);
     BH_CHECK_DIMS(n, ldw);
     BH_CHECK_DIMS(m, ldc);
@@ -205,6 +205,7 @@ int bitnet_hip_dense_gemv_dev(const bitnet_hip_vector_input *input, const uint16
     act0 &= ~BITNET_HIP_ACT_GATED;
     BH_REQUIRE(act_ok(act0) && act_ok(act1), "dense_gemv: unknown activation");
     if (int rc = to_epilogue(more, rows, g.more)) return rc;
+    BH_REQUIRE(!gated || act0 != BITNET_HIP_ACT_XIELU, "dense_gemv: an activation with constants does not go with pairs");
     const size_t pairs = gated ? (more && more->pairs ? more->pairs : rows) : 0;
     BH_REQUIRE(!gated ? !more || more->pairs == 0 : pairs % 2 == 0 && (pairs < rows ? act_split >= pairs : act_split == 0), "dense_gemv: gated rows come in pairs, with one activation");
     BH_REQUIRE(batch > 0 && batch < 65536 && (batch == 1 || (g.in.kind == BITNET_HIP_IN_PLAIN && !g.more.conv && !g.more.mul && pairs == 0)) && w_batch % 8 == 0, "dense_gemv: bad batch");

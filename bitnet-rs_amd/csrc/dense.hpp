@@ -307,8 +307,8 @@ __device__ __forceinline__ float group_sum(float v, float *slot) {
 }
 
 __device__ __forceinline__ float gelu_argument(float v) { return 0.7978845608028654f * (v + 0.044715f * v * v * v); }  // sqrt(2 / pi)
-// BITNET_HIP_ACT_*
-__device__ __forceinline__ float activate(float v, int act, float a = 0.f, float b = 0.f) {
+// BITNET_HIP_ACT_* without constants
+__device__ __forceinline__ float activate(float v, int act) {
     switch (act) {
         case BITNET_HIP_ACT_SILU: return v / (1.0f + expf(-v));
         case BITNET_HIP_ACT_SIGMOID: return 1.0f / (1.0f + expf(-v));
@@ -317,9 +317,12 @@ __device__ __forceinline__ float activate(float v, int act, float a = 0.f, float
             return r * r;
         }
         case BITNET_HIP_ACT_GELU_TANH: return v / (1.0f + expf(-2.0f * gelu_argument(v)));  // (1 + tanh z) / 2 = 1 / (1 + exp(-2 z))
-        case BITNET_HIP_ACT_XIELU: return 0.5f * v + (v > 0.f ? a * v * v : b * (expm1f(v) - v));
         default: return v;
     }
+}
+// all of them
+__device__ __forceinline__ float activate(float v, int act, float a, float b) {
+    return act == BITNET_HIP_ACT_XIELU ? 0.5f * v + (v > 0.f ? a * v * v : b * (expm1f(v) - v)) : activate(v, act);
 }
 
 // a pair of floats as (high, low) bf16 pairs: high + low carries 16 of the 24 bits

@@ -189,8 +189,8 @@ __device__ __forceinline__ void st4(uint16_t *p, size_t i, f32x4 v) {
 }
 constexpr int kSumRegs = 4;
 
-// IDENTITY: slots may be negative.
-template <class T, bool VEC, bool IDENTITY>
+// IDENTITY: slots may be negative.  GATED: with a number per row on y, a gate per column on what is added, or both.
+template <class T, bool VEC, bool IDENTITY, bool GATED>
 __global__ __launch_bounds__(256) void k_sum_norm_rows(SumRows p) {
     __shared__ float slot[4];
     const int tid = threadIdx.x, width = (int)p.width;
@@ -201,8 +201,8 @@ __global__ __launch_bounds__(256) void k_sum_norm_rows(SumRows p) {
     const int *slots = p.slots + (size_t)blockIdx.x * p.top;
     const float *sw = p.slot_weights + (size_t)blockIdx.x * p.top;
     const float *x2 = p.x2 ? p.x2 + (size_t)blockIdx.x * width : nullptr;
-    const T *gate = p.gate ? (const T *)p.gate + (size_t)blockIdx.x * p.ld_gate : nullptr;
-    const float ys = p.y_scale ? p.y_scale[(size_t)blockIdx.x * p.ld_y_scale] : 1.0f;
+    const T *gate = GATED && p.gate ? (const T *)p.gate + (size_t)blockIdx.x * p.ld_gate : nullptr;
+    const float ys = GATED && p.y_scale ? p.y_scale[(size_t)blockIdx.x * p.ld_y_scale] : 1.0f;
     const T *input = p.input ? (const T *)p.input + (size_t)blockIdx.x * p.ld_input : nullptr;  // (may be h: a thread reads its columns ahead of writing them)
     const int top = (int)p.top;
     if (VEC) {
@@ -220,7 +220,8 @@ __global__ __launch_bounds__(256) void k_sum_norm_rows(SumRows p) {
             for (int j = 0; j < kSumRegs; ++j) {
                 const int i = tid + 256 * j;
                 a[j] = f32x4{0.f, 0.f, 0.f, 0.f};
-                if (y && i < n4) a[j] = ys * ld4(y, 4 * i);
+                if (y && i < n4) a[j] = ld4(y, 4 * i);
+                if (GATED) a[j] *= ys;
             }
             float through = 0.f;
 #pragma unroll 4
@@ -265,15 +266,14 @@ __global__ __launch_bounds__(256) void k_sum_norm_rows(SumRows p) {
             for (int j = 0; j < kSumRegs; ++j) {
                 const int i = tid + 256 * j;
                 if (i < n4) {
-                    f32x4 r;
+                    if (GATED && gate) a[j] *= ld4(gate, 4 * i);
                     if (p.post_weight) {
-                        r = a[j] * post * (p.weight_offset + ld4(p.post_weight, 4 * i));
+                        f32x4 r = a[j] * post * (p.weight_offset + ld4(p.post_weight, 4 * i));
                         if (p.scale) r *= ld4(p.scale, 4 * i);
+                        v[j] += r;
                     } else {
-                        r = p.mult * a[j];
+                        v[j] += p.mult * a[j];
                     }
-                    if (gate) r *= ld4(gate, 4 * i);
-                    v[j] += r;
                     st4(x, 4 * i, v[j]);
                 }
             }
@@ -362,12 +362,19 @@ __global__ __launch_bounds__(256) void k_sum_norm_rows(SumRows p) {
 hipError_t launch_sum_norm_rows(const SumRows &a, hipStream_t s) {
     // (four columns at a time: every row of every operand starts on its own alignment)
     const bool vec = a.width % 4 == 0 && a.width <= 1024 * kSumRegs && a.ldy % 4 == 0 && a.ld_expert % 4 == 0 && a.ldh % 4 == 0 && a.ld_input % 4 == 0 && a.ld_gate % 4 == 0;
-    auto pick = [&](auto all, auto some) { return a.identity ? some : all; };
-    auto fn = a.h_f32 ? (vec ? pick(k_sum_norm_rows<float, true, false>, k_sum_norm_rows<float, true, true>) : pick(k_sum_norm_rows<float, false, false>, k_sum_norm_rows<float, false, true>))
-                      : (vec ? pick(k_sum_norm_rows<uint16_t, true, false>, k_sum_norm_rows<uint16_t, true, true>)
-                             : pick(k_sum_norm_rows<uint16_t, false, false>, k_sum_norm_rows<uint16_t, false, true>));
-    hipLaunchKernelGGL(fn, dim3(a.m), dim3(256), 0, s, a);
-    return hipGetLastError();
+    auto go = [&](auto plain, auto identity, auto gated, auto both) {
+        const bool g = a.gate || a.y_scale;
+        hipLaunchKernelGGL(a.identity ? (g ? both : identity) : g ? gated : plain, dim3(a.m), dim3(256), 0, s, a);
+        return hipGetLastError();
+    };
+    if (a.h_f32)
+        return vec ? go(k_sum_norm_rows<float, true, false, false>, k_sum_norm_rows<float, true, true, false>, k_sum_norm_rows<float, true, false, true>, k_sum_norm_rows<float, true, true, true>)
+                   : go(k_sum_norm_rows<float, false, false, false>, k_sum_norm_rows<float, false, true, false>, k_sum_norm_rows<float, false, false, true>,
+                        k_sum_norm_rows<float, false, true, true>);
+    return vec ? go(k_sum_norm_rows<uint16_t, true, false, false>, k_sum_norm_rows<uint16_t, true, true, false>, k_sum_norm_rows<uint16_t, true, false, true>,
+                    k_sum_norm_rows<uint16_t, true, true, true>)
+               : go(k_sum_norm_rows<uint16_t, false, false, false>, k_sum_norm_rows<uint16_t, false, true, false>, k_sum_norm_rows<uint16_t, false, false, true>,
+                    k_sum_norm_rows<uint16_t, false, true, true>);
 }
 
 // h = norm(o; w) * gate (gate: already through its sigmoid); the mean runs over mean_n elements, padding columns of o are zero
@@ -456,6 +463,7 @@ struct GemvK {
     int lat_wg;    // workgroup index that writes the latent row, or -1
 };
 
+template <bool MORE>
 __device__ void form_input(const VecIn &in, const float *x, int cols, int kp, float *xs, float *slot, bool writer) {
     const int tid = threadIdx.x;
     const int n = in.n;
@@ -494,7 +502,7 @@ __device__ void form_input(const VecIn &in, const float *x, int cols, int kp, fl
 #pragma unroll
             for (int j = 0; j < NR; ++j) {
                 yv[j] = reinterpret_cast<const f32x4 *>(in.y)[min(tid + 256 * j, n4 - 1)];
-                yg[j] = in.y_gate ? reinterpret_cast<const f32x4 *>(in.y_gate)[min(tid + 256 * j, n4 - 1)] : f32x4{1.f, 1.f, 1.f, 1.f};
+                yg[j] = MORE && in.y_gate ? reinterpret_cast<const f32x4 *>(in.y_gate)[min(tid + 256 * j, n4 - 1)] : f32x4{1.f, 1.f, 1.f, 1.f};
             }
 #pragma unroll
             for (int j = 0; j < NR; ++j) {
@@ -521,7 +529,7 @@ __device__ void form_input(const VecIn &in, const float *x, int cols, int kp, fl
 #pragma unroll
                 for (int j = 0; j < NR; ++j) sc[j] = f32x4{1.f, 1.f, 1.f, 1.f};
             }
-            if (in.y_gate)
+            if (MORE && in.y_gate)
 #pragma unroll
                 for (int j = 0; j < NR; ++j) sc[j] *= reinterpret_cast<const f32x4 *>(in.y_gate)[min(tid + 256 * j, n4 - 1)];
 #pragma unroll
@@ -589,7 +597,7 @@ __device__ void form_input(const VecIn &in, const float *x, int cols, int kp, fl
         float ss = 0.f;
         if (in.kind >= BITNET_HIP_IN_RESIDUAL_NORM && in.y && !in.post_weight) {
             for (int i = tid; i < n; i += 256) {
-                const float v = x[i] + in.mult * in.y[i] * (in.y_gate ? in.y_gate[i] : 1.0f);
+                const float v = x[i] + in.mult * in.y[i] * (MORE && in.y_gate ? in.y_gate[i] : 1.0f);
                 xs[i] = v;
                 if (writer && in.x_out) in.x_out[i] = v;
                 ss += v * v;
@@ -599,7 +607,7 @@ __device__ void form_input(const VecIn &in, const float *x, int cols, int kp, fl
             const float inv = 1.0f / sqrtf(group_sum<4>(ss, slot) / (float)in.mean_n + in.eps);
             ss = 0.f;
             for (int i = tid; i < n; i += 256) {
-                const float v = x[i] + (in.scale ? in.scale[i] : 1.0f) * (in.y_gate ? in.y_gate[i] : 1.0f) * (in.y[i] * inv * (in.offset + in.post_weight[i]));
+                const float v = x[i] + (in.scale ? in.scale[i] : 1.0f) * (MORE && in.y_gate ? in.y_gate[i] : 1.0f) * (in.y[i] * inv * (in.offset + in.post_weight[i]));
                 xs[i] = v;
                 if (writer && in.x_out) in.x_out[i] = v;
                 ss += v * v;
@@ -648,7 +656,8 @@ __device__ __forceinline__ float lanes_total(float v) {
     return LPR == 64 ? rows_sum(v) : v;
 }
 
-template <int LPR, int R, int U>
+// MORE: whatever bitnet_hip_epilogue and a gate on the residual ask for
+template <int LPR, int R, int U, bool MORE>
 __global__ __launch_bounds__(256) void k_dense_gemv(GemvK p) {
     extern __shared__ __attribute__((aligned(16))) float xs[];
     __shared__ float slot[4];
@@ -688,7 +697,8 @@ __global__ __launch_bounds__(256) void k_dense_gemv(GemvK p) {
     };
     // the earlier positions of a convolution's rows, a tap per lane; summed behind the product
     const Epilogue &e = a.more;
-    const int pos = e.conv ? *e.pos : 0, mul_at = e.mul ? *e.mul_at : 0;
+    const bool conv = MORE && e.conv, mul = MORE && e.mul;
+    const int pos = conv ? *e.pos : 0, mul_at = mul ? *e.mul_at : 0;
     float past[R];
     auto fetch_past = [&](int grp) {
 #pragma unroll
@@ -703,8 +713,8 @@ __global__ __launch_bounds__(256) void k_dense_gemv(GemvK p) {
         }
     };
     if (g < p.groups) fetch(g, 0);
-    if (e.conv && g < p.groups) fetch_past(g);
-    form_input(a.in, a.in.x + (size_t)b * a.x_batch, a.cols, p.kp, xs, slot, blockIdx.x == 0 && b == 0);
+    if (conv && g < p.groups) fetch_past(g);
+    form_input<MORE>(a.in, a.in.x + (size_t)b * a.x_batch, a.cols, p.kp, xs, slot, blockIdx.x == 0 && b == 0);
     float bv = -INFINITY;
     int bi = 0x7fffffff;
     for (; g < p.groups; g += n_wg * 4) {
@@ -742,7 +752,7 @@ __global__ __launch_bounds__(256) void k_dense_gemv(GemvK p) {
         const int row0 = (g * G + sub) * R;
 #pragma unroll
         for (int r = 0; r < R; ++r) acc[r] = lanes_total<LPR>(acc[r]);
-        if (e.conv) {
+        if (conv) {
             float f[R];
 #pragma unroll
             for (int r = 0; r < R; ++r) f[r] = lanes_total<LPR>(past[r]);
@@ -756,14 +766,14 @@ __global__ __launch_bounds__(256) void k_dense_gemv(GemvK p) {
             }
             if (g + n_wg * 4 < p.groups) fetch_past(g + n_wg * 4);
         }
-        if (R > 1 && row0 < a.gated) {
+        if (R > 1 && (MORE ? row0 < a.gated : a.gated)) {
             if (l == 0)
 #pragma unroll
                 for (int r = 0; r + 1 < R; r += 2) {
                     const int row = row0 + r;  // (even, and so is the number of rows in pairs, in whole groups)
                     if (row >= a.rows) continue;
                     const float b0 = a.bias ? a.bias[row] : 0.f, b1 = a.bias ? a.bias[row + 1] : 0.f;
-                    a.y[(size_t)b * a.y_batch + (row >> 1)] = activate(acc[r] + b0, a.act0, e.act_a, e.act_b) * (acc[r + 1] + b1);
+                    a.y[(size_t)b * a.y_batch + (row >> 1)] = activate(acc[r] + b0, a.act0) * (acc[r + 1] + b1);
                 }
         } else if (l == 0) {
 #pragma unroll
@@ -771,10 +781,11 @@ __global__ __launch_bounds__(256) void k_dense_gemv(GemvK p) {
                 const int row = row0 + r, ch = row - e.conv_from;
                 if (row >= a.rows) continue;
                 float v = acc[r];
-                if (a.bias && (!e.conv || ch < 0 || ch >= e.channels)) v += a.bias[row];
-                v = activate(v, row >= e.act2_from ? e.act2 : row < a.act_split ? a.act0 : a.act1, e.act_a, e.act_b);
-                if (e.mul) v *= bf2f(e.mul[(size_t)min(max(e.mul_tokens[mul_at], 0), e.mul_rows - 1) * e.ld_mul + row]);
-                a.y[(size_t)b * a.y_batch + row - (a.gated >> 1)] = v;
+                if (a.bias && (!conv || ch < 0 || ch >= e.channels)) v += a.bias[row];
+                const int act = MORE && row >= e.act2_from ? e.act2 : row < a.act_split ? a.act0 : a.act1;
+                v = MORE ? activate(v, act, e.act_a, e.act_b) : activate(v, act);
+                if (mul) v *= bf2f(e.mul[(size_t)min(max(e.mul_tokens[mul_at], 0), e.mul_rows - 1) * e.ld_mul + row]);
+                a.y[(size_t)b * a.y_batch + row - (MORE ? a.gated >> 1 : 0)] = v;
                 if (a.best_val) {
                     const float t = v != v ? -INFINITY : v;
                     if (t > bv || (t == bv && row < bi)) {
@@ -813,13 +824,23 @@ __global__ __launch_bounds__(256) void k_dense_gemv(GemvK p) {
     }
 }
 
-template <int LPR, int R>
-static void gemv_pick_u(int u, const GemvK &k, dim3 grid, hipStream_t s) {
+template <int LPR, int R, bool MORE>
+static void gemv_go(int u, const GemvK &k, dim3 grid, hipStream_t s) {
     const size_t lds = (size_t)k.kp * 4;
-    void (*fn)(GemvK) = u == 1 ? k_dense_gemv<LPR, R, 1> : u == 2 ? k_dense_gemv<LPR, R, 2> : u == 3 ? k_dense_gemv<LPR, R, 3>
-                      : u == 4 ? k_dense_gemv<LPR, R, 4> : k_dense_gemv<LPR, R, 5>;
+    void (*fn)(GemvK) = u == 1 ? k_dense_gemv<LPR, R, 1, MORE> : u == 2 ? k_dense_gemv<LPR, R, 2, MORE> : u == 3 ? k_dense_gemv<LPR, R, 3, MORE>
+                      : u == 4 ? k_dense_gemv<LPR, R, 4, MORE> : k_dense_gemv<LPR, R, 5, MORE>;
     if (lds > 65536) (void)hipFuncSetAttribute(reinterpret_cast<const void *>(fn), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
     hipLaunchKernelGGL(fn, grid, dim3(256), lds, s, k);
+}
+
+template <int LPR, int R>
+static void gemv_pick_u(int u, const GemvK &k, dim3 grid, hipStream_t s) {
+    const GemvArgs &a = k.a;
+    const bool pairs = a.gated && a.gated < a.rows;
+    if (a.in.y_gate || pairs || a.more.conv || a.more.mul || a.more.act2_from < a.rows || a.act0 == BITNET_HIP_ACT_XIELU || a.act1 == BITNET_HIP_ACT_XIELU)
+        gemv_go<LPR, R, true>(u, k, grid, s);
+    else
+        gemv_go<LPR, R, false>(u, k, grid, s);
 }
 
 hipError_t launch_dense_gemv(const GemvArgs &a, int *n_wg_out, hipStream_t s) {
@@ -1045,11 +1066,13 @@ __global__ __launch_bounds__(64 * WN * WM, 2) void k_dense_gemm(GemmArgsD p, int
 #pragma unroll
                 for (int e = 0; e < 4; ++e) acc[i][j][e] = f(acc[i][j][e], nl + i * FS + e);
         };
+        // (exp(v) - 1 loses what a bf16 output does not keep)
+        auto xielu = [&](float v) { return 0.5f * v + (v > 0.f ? p.more.act_a * v * v : p.more.act_b * (__expf(v) - 1.0f - v)); };
         if (act < 0)
             apply([&](float v, int n) {
                 const int f = n < p.act_split ? p.act0 : p.act1;
                 const float sg = __builtin_amdgcn_rcpf(1.0f + __expf(-v)), r = fmaxf(v, 0.0f);
-                return f == BITNET_HIP_ACT_SILU ? v * sg : f == BITNET_HIP_ACT_SIGMOID ? sg : f == BITNET_HIP_ACT_RELU2 ? r * r : activate(v, f, p.more.act_a, p.more.act_b);
+                return f == BITNET_HIP_ACT_SILU ? v * sg : f == BITNET_HIP_ACT_SIGMOID ? sg : f == BITNET_HIP_ACT_RELU2 ? r * r : f == BITNET_HIP_ACT_XIELU ? xielu(v) : activate(v, f);
             });
         else if (act == BITNET_HIP_ACT_SILU)
             apply([](float v, int) { return v * __builtin_amdgcn_rcpf(1.0f + __expf(-v)); });
@@ -1059,8 +1082,8 @@ __global__ __launch_bounds__(64 * WN * WM, 2) void k_dense_gemm(GemmArgsD p, int
             apply([](float v, int) { return activate(v, BITNET_HIP_ACT_RELU2); });
         else if (act == BITNET_HIP_ACT_GELU_TANH)
             apply([](float v, int) { return v * __builtin_amdgcn_rcpf(1.0f + __expf(-2.0f * gelu_argument(v))); });
-        else if (act == BITNET_HIP_ACT_XIELU)  // (exp(v) - 1 loses what a bf16 output does not keep)
-            apply([&](float v, int) { return 0.5f * v + (v > 0.f ? p.more.act_a * v * v : p.more.act_b * (__expf(v) - 1.0f - v)); });
+        else if (act == BITNET_HIP_ACT_XIELU)
+            apply([&](float v, int) { return xielu(v); });
         if (MUL) {
             const int token = min(max(p.more.mul_tokens[*p.more.mul_at + m], 0), p.more.mul_rows - 1);
             const uint16_t *mul = p.more.mul + (size_t)token * p.more.ld_mul;

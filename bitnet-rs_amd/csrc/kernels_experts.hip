@@ -91,7 +91,7 @@ __device__ __forceinline__ void keep_groups(float (&s)[PL], const Router &r) {
     for (int j = 0; j < PL; ++j) s[j] = ahead[j] < keep ? s[j] : -INFINITY;
 }
 
-template <int LT, int PL>
+template <int LT, int PL, bool GROUPED>
 __device__ __forceinline__ void choose(float (&s)[PL], const Router &r, int &id, float &weight) {
     const int experts = (int)(r.experts + r.identity), top = (int)r.top;
     const int lane = threadIdx.x & 63, l = lane & (LT - 1), base = lane & ~(LT - 1);
@@ -118,7 +118,7 @@ __device__ __forceinline__ void choose(float (&s)[PL], const Router &r, int &id,
         score[j] = s[j];
         if (r.correction) s[j] += r.correction[min(l * PL + j, experts - 1)];
     }
-    if (r.groups) keep_groups<LT, PL>(s, r);
+    if (GROUPED) keep_groups<LT, PL>(s, r);
     id = 0, weight = 0.f;
     float chosen = 0.f;
     for (int k = 0; k < top; ++k) {
@@ -156,7 +156,7 @@ __device__ __forceinline__ void choose(float (&s)[PL], const Router &r, int &id,
 // ---- a prompt's choices -----------------------------------------------------------------------------------------------
 constexpr int kRouteTokens = 32;  // per workgroup; its choices are counted in LDS first
 
-template <int LT, int PL>
+template <int LT, int PL, bool GROUPED>
 __global__ __launch_bounds__(256) void k_route(const float *__restrict__ z, size_t ldz, Router r, ExpertsPlan p) {
     __shared__ int hist[kMaxExperts];
     const int tid = threadIdx.x, grp = tid / LT, l = tid & (LT - 1), experts = (int)p.experts, outputs = (int)(r.experts + r.identity), top = (int)p.top, m = (int)p.m;
@@ -171,7 +171,7 @@ __global__ __launch_bounds__(256) void k_route(const float *__restrict__ z, size
 #pragma unroll
     for (int i = 0; i < PER; ++i) {
         float w;
-        choose<LT, PL>(s[i], r, id[i], w);
+        choose<LT, PL, GROUPED>(s[i], r, id[i], w);
         rank[i] = 0;
         if (t0 + i < m && l < top) {
             if (id[i] < experts) rank[i] = atomicAdd(&hist[id[i]], 1);
@@ -225,7 +225,12 @@ __global__ __launch_bounds__(256) void k_route_slots(ExpertsPlan p) {
 hipError_t launch_experts_route(const float *logits, size_t ldz, const Router &r, const ExpertsPlan &p, hipStream_t s) {
     const bool row = p.top <= 16;  // sixteen lanes per token
     const int e = (int)(r.experts + r.identity);
-    auto fn = row && e <= 16 ? k_route<16, 1> : row && e <= 64 ? k_route<16, 4> : row && e <= 128 ? k_route<16, 8> : e <= 256 ? k_route<64, 4> : k_route<64, 16>;
+    auto pick = [&](auto any, auto grouped) { return r.groups ? grouped : any; };
+    auto fn = row && e <= 16    ? pick(k_route<16, 1, false>, k_route<16, 1, true>)
+              : row && e <= 64  ? pick(k_route<16, 4, false>, k_route<16, 4, true>)
+              : row && e <= 128 ? pick(k_route<16, 8, false>, k_route<16, 8, true>)
+              : e <= 256        ? pick(k_route<64, 4, false>, k_route<64, 4, true>)
+                                : pick(k_route<64, 16, false>, k_route<64, 16, true>);
     hipLaunchKernelGGL(fn, dim3((p.m + kRouteTokens - 1) / kRouteTokens), dim3(256), 0, s, logits, ldz, r, p);
     hipLaunchKernelGGL(k_route_tiles, dim3(1), dim3(1024), 0, s, p);
     hipLaunchKernelGGL(k_route_slots, dim3((p.m * p.top + 255) / 256), dim3(256), 0, s, p);
@@ -269,7 +274,7 @@ struct UpK {
     int kp, groups;
 };
 
-template <int LPR, int R, int U, int PL>
+template <int LPR, int R, int U, int PL, bool GROUPED>
 __global__ __launch_bounds__(256) void k_experts_up(UpK p) {
     extern __shared__ __attribute__((aligned(16))) float xs[];
     const ExpertsUp &a = p.a;
@@ -292,7 +297,7 @@ __global__ __launch_bounds__(256) void k_experts_up(UpK p) {
     load(tid);
     int mine;
     float weight;
-    choose<64, PL>(z, a.r, mine, weight);
+    choose<64, PL, GROUPED>(z, a.r, mine, weight);
     // member b of the launch takes the b-th chosen expert that is no identity
     const unsigned long long real = __ballot(lane < (int)a.r.top && mine < (int)a.r.experts);
     const int n_real = __popcll(real);
@@ -460,7 +465,7 @@ static int gemv_grid(int groups, int share) {
     return n;
 }
 
-template <int LPR, int R>
+template <int LPR, int R, bool GROUPED>
 static hipError_t up_go(const ExpertsUp &a, int chunks, hipStream_t s) {
     UpK k;
     k.a = a;
@@ -470,10 +475,10 @@ static hipError_t up_go(const ExpertsUp &a, int chunks, hipStream_t s) {
     if ((size_t)k.kp * 4 > 150 * 1024) return hipErrorInvalidValue;
     const int outputs = (int)(a.r.experts + a.r.identity), top = (int)a.r.top;
     auto pick = [&](auto f64, auto f256, auto f1024) { return outputs <= 64 ? f64 : outputs <= 256 ? f256 : f1024; };
-    auto fn = u == 1   ? pick(k_experts_up<LPR, R, 1, 1>, k_experts_up<LPR, R, 1, 4>, k_experts_up<LPR, R, 1, 16>)
-              : u == 2 ? pick(k_experts_up<LPR, R, 2, 1>, k_experts_up<LPR, R, 2, 4>, k_experts_up<LPR, R, 2, 16>)
-              : u == 3 ? pick(k_experts_up<LPR, R, 3, 1>, k_experts_up<LPR, R, 3, 4>, k_experts_up<LPR, R, 3, 16>)
-                       : pick(k_experts_up<LPR, R, 5, 1>, k_experts_up<LPR, R, 5, 4>, k_experts_up<LPR, R, 5, 16>);
+    auto fn = u == 1   ? pick(k_experts_up<LPR, R, 1, 1, GROUPED>, k_experts_up<LPR, R, 1, 4, GROUPED>, k_experts_up<LPR, R, 1, 16, GROUPED>)
+              : u == 2 ? pick(k_experts_up<LPR, R, 2, 1, GROUPED>, k_experts_up<LPR, R, 2, 4, GROUPED>, k_experts_up<LPR, R, 2, 16, GROUPED>)
+              : u == 3 ? pick(k_experts_up<LPR, R, 3, 1, GROUPED>, k_experts_up<LPR, R, 3, 4, GROUPED>, k_experts_up<LPR, R, 3, 16, GROUPED>)
+                       : pick(k_experts_up<LPR, R, 5, 1, GROUPED>, k_experts_up<LPR, R, 5, 4, GROUPED>, k_experts_up<LPR, R, 5, 16, GROUPED>);
     const size_t lds = (size_t)k.kp * 4;
     if (lds > 65536) {
         const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(fn), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
@@ -483,11 +488,14 @@ static hipError_t up_go(const ExpertsUp &a, int chunks, hipStream_t s) {
     return hipGetLastError();
 }
 
-hipError_t launch_experts_up(const ExpertsUp &a, hipStream_t s) {
-    if (a.cols <= 256) return a.gated ? up_go<16, 2>(a, (a.cols + 127) / 128, s) : up_go<16, 1>(a, (a.cols + 127) / 128, s);
+template <bool GROUPED>
+static hipError_t up_pick(const ExpertsUp &a, hipStream_t s) {
+    if (a.cols <= 256) return a.gated ? up_go<16, 2, GROUPED>(a, (a.cols + 127) / 128, s) : up_go<16, 1, GROUPED>(a, (a.cols + 127) / 128, s);
     const int chunks = (a.cols + 511) / 512;
-    return a.gated || (long)a.rows * (long)a.r.top >= 4096 ? up_go<64, 2>(a, chunks, s) : up_go<64, 1>(a, chunks, s);
+    return a.gated || (long)a.rows * (long)a.r.top >= 4096 ? up_go<64, 2, GROUPED>(a, chunks, s) : up_go<64, 1, GROUPED>(a, chunks, s);
 }
+
+hipError_t launch_experts_up(const ExpertsUp &a, hipStream_t s) { return a.r.groups ? up_pick<true>(a, s) : up_pick<false>(a, s); }
 
 template <int LPR, int R>
 static hipError_t out_go(const ExpertsOut &a, hipStream_t s) {

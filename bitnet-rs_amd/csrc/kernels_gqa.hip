@@ -688,7 +688,8 @@ hipError_t launch_gqa_merge(const Gqa &g, const int *pos, int q0, int nq, const 
 // ---- prompt -----------------------------------------------------------------------------------------------------------
 // One workgroup: one head, four waves; a wave holds two slots of 16 queries: both maps of one query tile, or two tiles of the only map.  Key tiles
 // of 64 (every map's) and the values of the tile staged through registers into LDS one step ahead.
-template <int NK, int NV, int MAPS>
+// FAR: with a distance penalty, gates per column, or both.
+template <int NK, int NV, int MAPS, bool FAR>
 __global__ __launch_bounds__(256, NV > 8 || NK > 4 ? 1 : 2) void k_gqa_prefill(Gqa p, const uint16_t *Q, size_t ldq, int n_ctx, int nq, uint16_t *out, size_t ldo, int n_qb) {
     extern __shared__ __attribute__((aligned(16))) uint8_t lds[];
     constexpr int SLOTS = 2, QW = 16 * SLOTS / MAPS, KS = NK * 64 + 16, VS = 64 * 2 + 16, NVL = NV / 2;
@@ -774,7 +775,7 @@ __global__ __launch_bounds__(256, NV > 8 || NK > 4 ? 1 : 2) void k_gqa_prefill(G
                     s[kt][t] = mfma_bf16(a, qf[t][kk], s[kt][t]);
                 }
         }
-        if (MAPS == 1 && p.far_weight)
+        if (FAR && p.far_weight)
 #pragma unroll
             for (int t = 0; t < SLOTS; ++t)
 #pragma unroll
@@ -848,7 +849,7 @@ __global__ __launch_bounds__(256, NV > 8 || NK > 4 ? 1 : 2) void k_gqa_prefill(G
     for (int t = 0; t < SLOTS / MAPS; ++t) gate[t] = 1.0f;
 #pragma unroll
     for (int t = 0; t < SLOTS; ++t) inv[t] = 1.0f / rows_sum(l[t]);
-    if (p.gate && !p.gate_columns)
+    if (p.gate && !(FAR && p.gate_columns))
 #pragma unroll
         for (int t = 0; t < SLOTS / MAPS; ++t) gate[t] = activate(gate_logit(p, min(qw + t * 16 + r16, nq - 1), h, 0), BITNET_HIP_ACT_SIGMOID);
     if (MAPS == 2) {
@@ -869,7 +870,7 @@ __global__ __launch_bounds__(256, NV > 8 || NK > 4 ? 1 : 2) void k_gqa_prefill(G
         for (int v = 0; v < NV; ++v)
             if (v * 16 < vdimp) {
                 f32x4 q = o[v][t] * (inv[t] * gate[t]);
-                if (p.gate_columns) {
+                if (FAR && p.gate_columns) {
                     float z[4];
 #pragma unroll
                     for (int i = 0; i < 4; ++i) z[i] = gate_logit(p, qi, h, v * 16 + g * 4 + i);
@@ -885,7 +886,7 @@ template <int NK, int NV>
 static hipError_t gqa_prefill_go(const Gqa &g, const uint16_t *q, size_t ldq, int n_ctx, int nq, uint16_t *out, size_t ldo, hipStream_t s) {
     const int rows = g.maps == 2 ? 64 : 128, n_qb = (nq + rows - 1) / rows;
     const size_t lds = (size_t)g.maps * 64 * (NK * 64 + 16) + (size_t)NV * 16 * (64 * 2 + 16);
-    auto fn = g.maps == 2 ? k_gqa_prefill<NK, NV, 2> : k_gqa_prefill<NK, NV, 1>;
+    auto fn = g.maps == 2 ? k_gqa_prefill<NK, NV, 2, false> : g.far_weight || g.gate_columns ? k_gqa_prefill<NK, NV, 1, true> : k_gqa_prefill<NK, NV, 1, false>;
     if (lds > 65536) {
         const hipError_t e = hipFuncSetAttribute(reinterpret_cast<const void *>(fn), hipFuncAttributeMaxDynamicSharedMemorySize, (int)lds);
         if (e != hipSuccess) return e;
